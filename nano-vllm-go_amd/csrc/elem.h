@@ -378,6 +378,10 @@ __global__ void rope_kv_kernel(const float* __restrict__ qkv, int qkv_stride,
 // ---------------------------------------------------------------------------------------
 // un-fused activations for the fp32 parity mode and the op-level entry points
 // ---------------------------------------------------------------------------------------
+__global__ void fill_i32_kernel(int32_t* __restrict__ p, int32_t v, int n) {
+    const int i = blockIdx.x * blockDim.x + threadIdx.x;
+    if (i < n) p[i] = v;
+}
 // h [rows][2F] = [gate | up] -> y [rows][F] = silu(gate)*up   (transformer.go:50-66)
 template <typename ActT>
 __global__ void swiglu_kernel(const float* __restrict__ h, ActT* __restrict__ y, int64_t rows, int F) {

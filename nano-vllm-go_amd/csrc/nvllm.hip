@@ -86,6 +86,25 @@ void clear_graphs(nvl_model* m) {
     if (m->stream) (void)hipStreamSynchronize(m->stream);
     reap_graphs(m);
 }
+// Uncached device memory is never freed before the process ends (allocations made after such a free have held wrong values on
+// these machines): the comm buffers of closed models are kept here for the next model that needs one of the same size.
+std::mutex g_p2p_spare_mu;
+std::multimap<std::pair<int, size_t>, char*> g_p2p_spare;      // (device, bytes)
+void p2p_give_back(char* p, size_t bytes) {
+    if (!p) return;
+    int dev = 0;
+    (void)hipGetDevice(&dev);
+    std::lock_guard<std::mutex> lk(g_p2p_spare_mu);
+    g_p2p_spare.emplace(std::make_pair(dev, bytes), p);
+}
+char* p2p_take_spare(int dev, size_t bytes) {
+    std::lock_guard<std::mutex> lk(g_p2p_spare_mu);
+    auto it = g_p2p_spare.find(std::make_pair(dev, bytes));
+    if (it == g_p2p_spare.end()) return nullptr;
+    char* p = it->second;
+    g_p2p_spare.erase(it);
+    return p;
+}
 void free_sample_bufs(SampleBufs& b) {
     dfree(b.work); dfree(b.cnt); dfree(b.hist); dfree(b.off); dfree(b.out); dfree(b.u); dfree(b.probs);
     b = SampleBufs{};
@@ -331,7 +350,7 @@ extern "C" void nvl_destroy(nvl_model* m) {
     dfree(m->expert_w); dfree(m->seg_start); dfree(m->moe_counts); dfree(m->moe_cursor); dfree(m->moe_tile_map); dfree(m->moe_n_mtiles); dfree(m->perm_token); dfree(m->slot_of); dfree(m->moe_eo); dfree(m->moe_xg);
     dfree(m->meta_dev); dfree(m->hidden); dfree(m->sk_part); dfree(m->tp_part); dfree(m->ring); dfree(m->rs_part);
     for (int r = 0; r < 8; r++) if (m->p2p_peer[r] && m->p2p_peer[r] != m->p2p_buf) (void)hipIpcCloseMemHandle(m->p2p_peer[r]);
-    dfree(m->p2p_buf);
+    p2p_give_back(m->p2p_buf, m->p2p_bytes);
     dfree(m->moe_gate); dfree(m->moe_hall); dfree(m->moe_part);
     clear_graphs(m);
     if (m->am_host) (void)hipHostFree(m->am_host);
@@ -882,8 +901,8 @@ void p2p_alloc(nvl_model* m) {
     m->p2p_off_in2 = round_up(m->p2p_off_in1 + 2 * T * m->p2p_in1_stride * esz, 256);
     m->p2p_off_res = round_up(m->p2p_off_in2 + 2 * T * m->p2p_in2_stride * esz, 256);
     m->p2p_bytes = (size_t)round_up(m->p2p_off_res + 2 * m->p2p_res_stride * esz, 256);
-    void* p = nullptr;
-    NVL_HIP(hipExtMallocWithFlags(&p, m->p2p_bytes, hipDeviceMallocUncached));     // coherent across GPUs: peers write it, we poll it
+    void* p = p2p_take_spare(m->device, m->p2p_bytes);
+    if (!p) NVL_HIP(hipExtMallocWithFlags(&p, m->p2p_bytes, hipDeviceMallocUncached));     // coherent across GPUs: peers write it, we poll it
     m->p2p_buf = (char*)p;
     NVL_HIP(hipMemset(m->p2p_buf, 0, m->p2p_bytes));
 }
@@ -1484,7 +1503,7 @@ bool moe(nvl_model* m, const LayerW& l, int M, bool deferred_norm = false, const
         NVL_HIP(hipGetLastError());
     } else {
         KScope ks(m, KC_OTHER, 0, KS_MOE_PLAN);
-        NVL_HIP(hipMemsetAsync(m->moe_counts, 0, (size_t)E * 4, m->stream));
+        hipLaunchKernelGGL(fill_i32_kernel, dim3(cdiv(E, 256)), dim3(256), 0, m->stream, m->moe_counts, 0, E);     // (a captured pass must hold no memset node)
         hipLaunchKernelGGL(moe_route_kernel, dim3(cdiv(M, 4)), dim3(256), 0, m->stream, m->router_logits, 128, M, E, k,
                            m->expert_ids, m->expert_w);
         hipLaunchKernelGGL(moe_hist_kernel, dim3(cdiv(pairs, MOE_PAIRS_PER_WG)), dim3(256), 0, m->stream, m->expert_ids, pairs, m->moe_counts);

@@ -1,5 +1,5 @@
 #!/bin/bash
-cd scripts/micro && /opt/rocm/bin/hipcc -O3 --offload-arch=gfx950 launch_floor.hip -o /tmp/launch_floor && cd ../..
+cd scripts/micro && /opt/rocm/bin/hipcc -O3 --offload-arch=gfx950 -Xclang -target-feature -Xclang -packed-fp32-ops launch_floor.hip -o /tmp/launch_floor && cd ../..
 echo "== default"; /tmp/launch_floor
 echo "== HIP_FORCE_DEV_KERNARG=1"; HIP_FORCE_DEV_KERNARG=1 /tmp/launch_floor
 for E in 0 1; do for B in 32 1; do
