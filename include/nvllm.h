@@ -27,8 +27,9 @@
 extern "C" {
 #endif
 
-#define NVL_ABI_VERSION 3      /* 2: Mamba2 / hybrid layers (config fields, tensor kinds), nvl_stats.evictions, kernel stats;
-                                  3: nvl_get_weight, nvl_get_stamps, nvl_tp_p2p_rearm, debug modes 2 / 4 (additions only) */
+#define NVL_ABI_VERSION 4      /* 2: Mamba2 / hybrid layers (config fields, tensor kinds), nvl_stats.evictions, kernel stats;
+                                  3: nvl_get_weight, nvl_get_stamps, nvl_tp_p2p_rearm, debug modes 2 / 4 (additions only);
+                                  4: models described by a list of layers, library-owned block pool, nvl_forward_rows (additions only) */
 
 typedef enum nvl_status {
     NVL_OK = 0,
@@ -46,8 +47,11 @@ typedef enum nvl_status {
 enum { NVL_ATTN_MHA = 0, NVL_ATTN_MQA = 1, NVL_ATTN_GQA = 2 };        /* config.go:18-22 */
 enum { NVL_NORM_LAYER = 0, NVL_NORM_RMS = 1 };                        /* config.go:27-30 */
 enum { NVL_POS_LEARNED = 0, NVL_POS_ROPE = 1, NVL_POS_NONE = 2 };     /* config.go:35-40 */
-enum { NVL_ACT_GELU = 0, NVL_ACT_SWIGLU = 1 };                        /* config.go:45-48 */
-enum { NVL_BLOCK_SEQUENTIAL = 0, NVL_BLOCK_PARALLEL = 1 };            /* config.go:53-56 */
+enum { NVL_ACT_GELU = 0, NVL_ACT_SWIGLU = 1,                          /* config.go:45-48 */
+       NVL_ACT_GEGLU = 2 };                                           /* gelu_tanh(gate) * up */
+enum { NVL_BLOCK_SEQUENTIAL = 0, NVL_BLOCK_PARALLEL = 1,              /* config.go:53-56 */
+       NVL_BLOCK_SANDWICH = 2 };   /* a norm before AND after each sublayer, x += norm_b(f(norm_a(x))); the model is described
+                                      by a list of layers (nvl_layer_config, nvl_create_layers)  */
 
 typedef struct nvl_model_config {
     int32_t vocab_size, hidden, num_layers, num_heads, num_kv_heads, head_dim;
@@ -64,6 +68,25 @@ typedef struct nvl_model_config {
     int32_t  mamba_expand, mamba_state_size, mamba_num_heads, mamba_head_dim, mamba_n_groups, mamba_conv_kernel;
     uint64_t mamba_layer_mask[2];
 } nvl_model_config;
+
+/* ---- models described by a list of layers: every layer names its mixer, the mixer's sizes and its feed-forward ---- */
+enum {
+    NVL_MIXER_LATENT_ATTENTION = 0, /* queries and keys/values through low-rank latents, no positions; the cache holds the latent */
+    NVL_MIXER_MAMBA2 = 1,           /* causal convolution + selective state space, gate before a grouped norm                     */
+    NVL_MIXER_GLA = 2               /* gated linear attention: a decay per key channel                                            */
+};
+typedef struct nvl_layer_config {
+    int32_t mixer;                  /* NVL_MIXER_*                                                                         */
+    int32_t weights_of;             /* the layer whose tensors this one uses (its cache / state is its own); -1: its own   */
+    int32_t heads, dim, vdim;       /* dim: query/key channels per head (not Mamba-2), vdim: value channels per head       */
+    int32_t q_rank, kv_rank;        /* latent attention: latent sizes                                                      */
+    int32_t window;                 /* latent attention: keys a query sees, itself included (0: all earlier tokens)        */
+    float   scale;                  /* latent attention: score multiplier                                                  */
+    int32_t state, groups, norm_groups, conv_taps;      /* Mamba-2                                                         */
+    float   tau;                    /* GLA: alpha = sigmoid(z)^(1/tau)                                                     */
+    int32_t decay_rank;             /* GLA: rank of the decay projection; 0: as the uploaded tensor says                   */
+    int32_t ffn_dim;                /* 0: no feed-forward                                                                  */
+} nvl_layer_config;
 
 /* Arithmetic the device path computes in. */
 enum {
@@ -89,7 +112,11 @@ typedef struct nvl_runtime_opts {
                                   0: one contiguous slab per sequence slot                              */
     int32_t kv_block_size;     /* tokens per block in paged mode: 0 = 256 (Sequence.BlockSize, sequence.go:51);
                                   a multiple of 64                                                     */
-    int32_t reserved;
+    int32_t kv_pool;           /* 1 with kv_num_blocks > 0: the LIBRARY allocates the pool's blocks to the sequences of the
+                                  slot calls as they grow (nvl_seq_*, nvl_forward, nvl_runner_run work; no block tables from
+                                  the host).  Always so for models described by a list of layers, whose recurrent layers
+                                  keep per-slot state; kv_num_blocks 0 then sizes the pool from max_seqs, the largest window
+                                  and max_batch_tokens                                                                     */
 } nvl_runtime_opts;
 
 typedef struct nvl_model nvl_model;
@@ -128,6 +155,22 @@ typedef enum nvl_tensor_kind {
     NVL_T_MAMBA_DT_BIAS,   /* [heads]                                                                */
     NVL_T_MAMBA_NORM,      /* [EH]                                                                   */
     NVL_T_MAMBA_OUT_PROJ,  /* OUT_IN: [H, EH]  OutProj, MatMul(y, Transpose(OutProj))           mamba2.go:175 */
+    /* models described by a list of layers: all matrices OUT_IN ([out, in], applied as W x).  Shared kinds: ATTN_NORM_W and
+     * FFN_NORM_W (the norms before the sublayers), WQ / WK / WV / WO, W1 (gate rows, then up rows), W2, the MAMBA_* kinds */
+    NVL_T_MIX_POST_NORM,   /* [H] norm after the mixer                                                */
+    NVL_T_FFN_POST_NORM,   /* [H] norm after the feed-forward                                         */
+    NVL_T_MIX_GATE,        /* [heads*vdim, H] output gate (latent attention, GLA)                     */
+    NVL_T_LAT_DQ,          /* [q_rank, H]         NVL_T_LAT_DQ_NORM  [q_rank]                         */
+    NVL_T_LAT_DQ_NORM,
+    NVL_T_LAT_UQ,          /* [heads*dim, q_rank]                                                     */
+    NVL_T_LAT_DKV,         /* [kv_rank, H]        NVL_T_LAT_DKV_NORM [kv_rank]                        */
+    NVL_T_LAT_DKV_NORM,
+    NVL_T_LAT_UK,          /* [heads*dim, kv_rank]                                                    */
+    NVL_T_LAT_UV,          /* [heads*vdim, kv_rank]                                                   */
+    NVL_T_GLA_NORM,        /* [vdim]                                                                  */
+    NVL_T_GLA_A1,          /* [rank, H]           decay projection, low-rank: z = A2 (A1 h) + b       */
+    NVL_T_GLA_A2,          /* [heads*dim, rank]                                                       */
+    NVL_T_GLA_A2_B,        /* [heads*dim]                                                             */
     NVL_T_COUNT
 } nvl_tensor_kind;
 
@@ -142,6 +185,10 @@ enum {
 /* Replaces tensor.NewTransformerModel (generic_model.go:41-61) + the runner's model ownership
  * (tensor_model_runner.go:21-33).  Fails with NVL_ERR_NO_DEVICE when no GPU is present. */
 int nvl_create(const nvl_model_config* cfg, const nvl_runtime_opts* opts, nvl_model** out);
+/* nvl_create for a model described by a list of layers (cfg->block_style == NVL_BLOCK_SANDWICH): `layers` has cfg->num_layers
+ * entries; of cfg only vocab_size, hidden, num_layers, max_seq_len, norm_eps, activation_type (NVL_ACT_GEGLU),
+ * embedding_multiplier, logits_scaling and tied_embedding are read. */
+int nvl_create_layers(const nvl_model_config* cfg, const nvl_layer_config* layers, const nvl_runtime_opts* opts, nvl_model** out);
 
 /* Replaces loadTensorFromData + the per-kind placement in loadAttention/loadFFN/loadMoE/loadNorm
  * (generic_loader.go:353-604,619-671).  `data` may be a host or a device pointer.  2-D kinds
@@ -161,6 +208,10 @@ int nvl_load_safetensors(nvl_model* m, const char* path);
  * the reference's model_info.json) -> nvl_model_config.  Reference quirks kept: max_position_embeddings and
  * rope_scaling are not read.  Errors are reported through nvl_last_error(NULL). */
 int nvl_load_config_json(const char* path, nvl_model_config* cfg);
+/* The layer list of a config.json whose architecture is described by one ("Potuzen"): writes up to `cap` entries, returns
+ * how many the file has; 0 for every other architecture.  Such a file names no longest sequence: nvl_load_config_json sets
+ * max_seq_len to 4096, the caller may change it before nvl_create_layers. */
+int nvl_load_layers_json(const char* path, nvl_layer_config* layers, int cap);
 
 /* Helpers for checkpoints that keep fused projections (generic_loader.go:674-765):
  * GPT-2 c_attn [H, 3H] split by columns; Falcon query_key_value given in the reference's
@@ -223,7 +274,12 @@ int nvl_forward(nvl_model* m, int n_seqs, const int64_t* seq_ids, const int32_t*
                 const int32_t* seq_lens, const int32_t* pos_offsets, uint32_t flags,
                 float* logits_out, int32_t* argmax_out);
 
-/* ---- paged KV (SURVEY §8 f-1): the host's block manager owns the cache ---- */
+/* nvl_forward with the logits rows named by the caller: rows[0 .. n_rows) are indices into the concatenated `tokens`
+ * (strictly increasing; n_rows may be 0: the tokens only enter the cache).  logits_out receives [n_rows, V], argmax_out one id per row. */
+int nvl_forward_rows(nvl_model* m, int n_seqs, const int64_t* seq_ids, const int32_t* tokens, const int32_t* seq_lens,
+                     const int32_t* pos_offsets, int n_rows, const int32_t* rows, float* logits_out, int32_t* argmax_out);
+
+/* ---- paged KV: the host's block manager owns the cache ---- */
 /* One forward pass like nvl_forward, for a model created with kv_num_blocks > 0.  The KV cache of sequence i is the
  * block list block_tables[table_offsets[i] .. table_offsets[i+1]) (Sequence.BlockTable, sequence.go:23): position p
  * lives in its block p / block_size at row p % block_size.  pos_offsets[i] tokens are already cached — after a
@@ -366,7 +422,7 @@ int nvl_reset_stats(nvl_model* m);
 const char* nvl_last_error(const nvl_model* m);   /* m may be NULL: last error of nvl_create */
 int nvl_abi_version(void);
 int nvl_device_count(void);                        /* number of visible HIP devices, 0 if none */
-int nvl_sizeof(int which);                         /* 0 nvl_model_config, 1 nvl_runtime_opts, 2 nvl_stats: lets a
+int nvl_sizeof(int which);                         /* 0 nvl_model_config, 1 nvl_runtime_opts, 2 nvl_stats, 3 nvl_sampling_params, 4 nvl_layer_config: lets a
                                                       binding (cgo/ctypes) verify its struct mirrors */
 
 /* ---- op-level entry points (host fp32 in / host fp32 out; used by the parity tests) ----

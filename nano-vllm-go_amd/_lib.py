@@ -19,18 +19,22 @@ SLOTS = [
     "wq", "wk", "wv", "wkv", "wo", "bq", "bk", "bv", "bo",
     "w1", "b1", "w2", "b2", "router", "moe_in", "moe_out",
     "mamba_in_proj", "mamba_conv_w", "mamba_conv_b", "mamba_a_log", "mamba_d", "mamba_dt_bias", "mamba_norm", "mamba_out_proj",
+    "mix_post_norm", "ffn_post_norm", "mix_gate", "lat_dq", "lat_dq_norm", "lat_uq", "lat_dkv", "lat_dkv_norm", "lat_uk", "lat_uv",
+    "gla_norm", "gla_a1", "gla_a2", "gla_a2_b",
 ]
 SLOT_ID = {n: i for i, n in enumerate(SLOTS)}
 ONE_D = {"final_norm_w", "final_norm_b", "attn_norm_w", "attn_norm_b", "ffn_norm_w", "ffn_norm_b",
          "bq", "bk", "bv", "bo", "b1", "b2",
-         "mamba_conv_w", "mamba_conv_b", "mamba_a_log", "mamba_d", "mamba_dt_bias", "mamba_norm"}
+         "mamba_conv_w", "mamba_conv_b", "mamba_a_log", "mamba_d", "mamba_dt_bias", "mamba_norm",
+         "mix_post_norm", "ffn_post_norm", "lat_dq_norm", "lat_dkv_norm", "gla_norm", "gla_a2_b"}
 OUT_IN_SLOTS = {"mamba_in_proj", "mamba_out_proj"}      # kept in the checkpoint's [out, in] layout by the reference's loader
 
 ATTN = {"mha": 0, "mqa": 1, "gqa": 2}
 NORM = {"layernorm": 0, "rmsnorm": 1}
 POS = {"learned": 0, "rope": 1, "nope": 2}
-ACT = {"gelu": 0, "swiglu": 1}
-BLOCK = {"sequential": 0, "parallel": 1}
+ACT = {"gelu": 0, "swiglu": 1, "geglu": 2}
+BLOCK = {"sequential": 0, "parallel": 1, "sandwich": 2}
+MIXER = {"latent_attention": 0, "mamba2": 1, "gla": 2}
 PRECISION = {"bf16": 0, "f32": 1}
 DTYPE_F32, DTYPE_BF16, DTYPE_F16 = 0, 1, 2
 LAYOUT_IN_OUT, LAYOUT_OUT_IN = 0, 1
@@ -64,11 +68,18 @@ class ModelConfigC(C.Structure):
     ]
 
 
+class LayerConfigC(C.Structure):        # nvl_layer_config
+    _fields_ = [("mixer", C.c_int32), ("weights_of", C.c_int32), ("heads", C.c_int32), ("dim", C.c_int32), ("vdim", C.c_int32),
+                ("q_rank", C.c_int32), ("kv_rank", C.c_int32), ("window", C.c_int32), ("scale", C.c_float),
+                ("state", C.c_int32), ("groups", C.c_int32), ("norm_groups", C.c_int32), ("conv_taps", C.c_int32),
+                ("tau", C.c_float), ("decay_rank", C.c_int32), ("ffn_dim", C.c_int32)]
+
+
 class RuntimeOptsC(C.Structure):
     _fields_ = [("device", C.c_int32), ("precision", C.c_int32), ("max_seqs", C.c_int32),
                 ("max_batch_tokens", C.c_int32), ("tp_rank", C.c_int32), ("tp_size", C.c_int32),
                 ("tp_force_single", C.c_int32), ("kv_num_blocks", C.c_int32), ("kv_block_size", C.c_int32),
-                ("reserved", C.c_int32)]
+                ("kv_pool", C.c_int32)]
 
 
 class StatsC(C.Structure):
@@ -124,6 +135,8 @@ def lib():
             pass
     L = C.CDLL(str(LIB_PATH))
     L.nvl_create.argtypes = [C.POINTER(ModelConfigC), C.POINTER(RuntimeOptsC), C.POINTER(vp)]
+    L.nvl_create_layers.argtypes = [C.POINTER(ModelConfigC), C.POINTER(LayerConfigC), C.POINTER(RuntimeOptsC), C.POINTER(vp)]
+    L.nvl_load_layers_json.argtypes = [C.c_char_p, C.POINTER(LayerConfigC), C.c_int]
     L.nvl_upload_tensor.argtypes = [vp, C.c_int, C.c_int, vp, C.c_int, i64, i64, C.c_int]
     L.nvl_upload_gpt2_qkv.argtypes = [vp, C.c_int, vp, vp]
     L.nvl_upload_falcon_qkv.argtypes = [vp, C.c_int, vp]
@@ -136,6 +149,7 @@ def lib():
         getattr(L, fn).argtypes = [vp, i64]
     L.nvl_seq_close_all.argtypes = [vp]
     L.nvl_forward.argtypes = [vp, C.c_int, vp, vp, vp, vp, C.c_uint32, vp, vp]
+    L.nvl_forward_rows.argtypes = [vp, C.c_int, vp, vp, vp, vp, C.c_int, vp, vp, vp]
     L.nvl_decode_greedy.argtypes = [vp, C.c_int, vp, vp, C.c_int, vp]
     L.nvl_forward_paged.argtypes = [vp, C.c_int, vp, vp, vp, vp, vp, C.c_uint32, vp, vp]
     L.nvl_runner_run_paged.argtypes = [vp, C.c_int, vp, vp, vp, vp, vp, C.c_int, vp, vp]

@@ -45,6 +45,7 @@ class ModelConfig:
     mamba_head_dim: int = 0
     mamba_n_groups: int = 0
     mamba_conv_kernel: int = 0
+    layers: list = field(default_factory=list)            # models described by a list of layers: one dict per layer (LAYER_FIELDS)
 
     @property
     def mamba_layer_mask(self):
@@ -133,6 +134,40 @@ def new_granite_config(size: str = "350m") -> ModelConfig:   # config.go:241-330
     return c
 
 
+LAYER_FIELDS = dict(mixer="", weights_of=-1, heads=0, dim=0, vdim=0, q_rank=0, kv_rank=0, window=0, scale=0.0, state=0, groups=0,
+                    norm_groups=0, conv_taps=0, tau=0.0, decay_rank=0, ffn_dim=0)      # nvl_layer_config
+
+
+def _potuzen_layer(e: dict) -> dict:
+    """One entry of a Potuzen config.json's layer list -> the fields of nvl_layer_config."""
+    mx, mlp, ty = e["mixer"], e.get("mlp"), e["type"]
+    out = dict(LAYER_FIELDS, mixer=ty, heads=mx["heads"], vdim=mx["vdim"])
+    if e.get("weights_of") is not None:
+        out["weights_of"] = e["weights_of"]
+    if ty == "latent_attention":
+        out.update(dim=mx["dim"], q_rank=mx["q_rank"], kv_rank=mx["kv_rank"], scale=float(mx["scale"]), window=(mx.get("mask") or {}).get("size", 0))
+    elif ty == "mamba2":
+        out.update(state=mx["state"], groups=mx["groups"], norm_groups=mx["norm_groups"], conv_taps=mx["conv"])
+    elif ty == "gla":
+        out.update(dim=mx["dim"], tau=float(mx["tau"]))
+    else:
+        raise ValueError(f"unknown mixer {ty!r}")
+    if mlp is not None:
+        if mlp.get("kind", "dense") != "dense":
+            raise ValueError(f"unknown feed-forward kind {mlp['kind']!r}")
+        out["ffn_dim"] = mlp["ff"]
+    return out
+
+
+def potuzen_config(raw: dict) -> ModelConfig:
+    """The Potuzen design: a list of layers (latent attention / Mamba-2 / gated linear attention), sandwich norms, GEGLU.  The
+    file names no longest sequence: 4096, as the library's own reader sets it; override max_seq_len as needed."""
+    return ModelConfig(architecture="Potuzen", model_name="potuzen", vocab_size=raw["vocab"], hidden=raw["width"],
+                       num_layers=len(raw["layers"]), max_seq_len=4096, attention_type="gqa", norm_type="rmsnorm", position_type="nope",
+                       activation_type="geglu", block_style="sandwich", rope_base=0.0, norm_eps=float(raw["norm"]["eps"]),
+                       layers=[_potuzen_layer(e) for e in raw["layers"]])
+
+
 def load_model_config(raw: dict | str) -> ModelConfig:
     """LoadModelConfig (generic_loader.go:808-972) on an already-parsed HF config.json (or its text).
     Reference quirks kept: max_position_embeddings and rope_scaling are never read, so max_seq_len
@@ -140,6 +175,8 @@ def load_model_config(raw: dict | str) -> ModelConfig:
     if isinstance(raw, str):
         raw = json.loads(raw)
     arch = raw.get("architecture")
+    if arch == "Potuzen":
+        return potuzen_config(raw)
     if arch == "gpt2":
         c = new_gpt2_config()
     elif arch == "falcon":

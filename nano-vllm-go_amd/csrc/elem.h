@@ -216,13 +216,13 @@ __global__ __launch_bounds__(1024) void norm_tile16_kernel(float* __restrict__ x
 template <typename ActT>
 __device__ __forceinline__ void norm_row_finish(f32x4 (&v)[NORM_ROW_MAXCH], f32x4 (&ww)[NORM_ROW_MAXCH],
                                                 f32x4 (&bb)[NORM_ROW_MAXCH], const float* b, float eps, ActT* y, int r,
-                                                int H, float* red) {
+                                                int H, float* red, int width = 0) {     // width: columns of the mean when the row is padded (0: H)
     const int H4 = H >> 2;
     if (b == nullptr) {
         float ss = 0.f;
 #pragma unroll
         for (int c = 0; c < NORM_ROW_MAXCH; c++) ss += v[c][0] * v[c][0] + v[c][1] * v[c][1] + v[c][2] * v[c][2] + v[c][3] * v[c][3];
-        const float rms = sqrtf(block256_sum(ss, red) / (float)H + eps);
+        const float rms = sqrtf(block256_sum(ss, red) / (float)(width ? width : H) + eps);
 #pragma unroll
         for (int c = 0; c < NORM_ROW_MAXCH; c++) {
             const int j = threadIdx.x + c * 256;
@@ -298,6 +298,139 @@ __global__ __launch_bounds__(256) void norm_row_kernel(float* __restrict__ x,
         }
     }
     norm_row_finish<ActT>(v, ww, bb, b, eps, y, r, H, red);
+}
+
+// ---------------------------------------------------------------------------------------
+// Sandwich norms: x += rms(y) * w_post completes a sublayer whose output y is normed before it joins the residual stream, and
+// the norm that opens the next sublayer follows at once: xn = rms(x) * w_next.  One launch does both (y == NULL: only the
+// second; w_next == NULL: only the first).  Rows are H floats apart, the mean runs over `width` <= H columns (the padding
+// columns of x, y and the weights are zero).  y may be split over `slices` partial sums (a K split of the projection).
+//   sandwich_row_kernel    : one 256-thread workgroup per row, the row in registers (decode, short batches, wide rows)
+//   sandwich_tile16_kernel : one wave per row, 16 rows per workgroup, operand blocks written whole (prefill, bf16)
+// ---------------------------------------------------------------------------------------
+struct SandwichArgs {
+    float* x;                 // residual stream [rows][H]
+    const float* y;           // [slices][.][H] or NULL
+    int slices; int64_t slice_stride;
+    const float* w_post;      // [H]
+    const float* w_next;      // [H] or NULL
+    const int32_t* rows_idx;  // y == NULL only: which row of x feeds output row r
+    int rows, H, width;
+    float eps;
+};
+template <typename ActT, int MAXCH>
+__global__ __launch_bounds__(256) void sandwich_row_kernel(SandwichArgs p, ActT* __restrict__ xn) {
+    __shared__ float red[4];
+    const int r = blockIdx.x, H4 = p.H >> 2;
+    const int src = p.rows_idx ? p.rows_idx[r] : r;
+    float* xr = p.x + (int64_t)src * p.H;
+    f32x4 x[MAXCH], y[MAXCH];
+    float ss = 0.f;
+#pragma unroll
+    for (int c = 0; c < MAXCH; c++) {
+        const int j = threadIdx.x + c * 256;
+        x[c] = f32x4{0.f, 0.f, 0.f, 0.f};
+        y[c] = x[c];
+        if (j < H4) {
+            x[c] = *(const f32x4*)(xr + j * 4);
+            if (p.y) {
+                const float* yr = p.y + (int64_t)r * p.H + j * 4;
+                y[c] = *(const f32x4*)yr;
+                for (int k = 1; k < p.slices; k++) y[c] += *(const f32x4*)(yr + k * p.slice_stride);
+            }
+        }
+        ss += y[c][0] * y[c][0] + y[c][1] * y[c][1] + y[c][2] * y[c][2] + y[c][3] * y[c][3];
+    }
+    if (p.y) {
+        const float rms = sqrtf(block256_sum(ss, red) / (float)p.width + p.eps);
+#pragma unroll
+        for (int c = 0; c < MAXCH; c++) {
+            const int j = threadIdx.x + c * 256;
+            if (j < H4) {
+                const f32x4 w = *(const f32x4*)(p.w_post + j * 4);
+#pragma unroll
+                for (int k = 0; k < 4; k++) x[c][k] += (y[c][k] / rms) * w[k];
+                *(f32x4*)(xr + j * 4) = x[c];
+            }
+        }
+    }
+    if (!p.w_next) return;
+    ss = 0.f;
+#pragma unroll
+    for (int c = 0; c < MAXCH; c++) ss += x[c][0] * x[c][0] + x[c][1] * x[c][1] + x[c][2] * x[c][2] + x[c][3] * x[c][3];
+    const float rms = sqrtf(block256_sum(ss, red) / (float)p.width + p.eps);
+#pragma unroll
+    for (int c = 0; c < MAXCH; c++) {
+        const int j = threadIdx.x + c * 256;
+        if (j < H4) {
+            const f32x4 w = *(const f32x4*)(p.w_next + j * 4);
+            f32x4 o;
+#pragma unroll
+            for (int k = 0; k < 4; k++) o[k] = (x[c][k] / rms) * w[k];
+            act_store4<ActT>(xn, r, j * 4, p.H, o);
+        }
+    }
+}
+template <int MAXCH>
+__global__ __launch_bounds__(1024) void sandwich_tile16_kernel(SandwichArgs p, bf16_t* __restrict__ xn) {
+    extern __shared__ __attribute__((aligned(16))) char smem_n[];
+    bf16_t* tile = (bf16_t*)smem_n;                       // [16][H]
+    const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
+    const int r = blockIdx.x * 16 + wave, H4 = p.H >> 2;
+    if (r < p.rows) {
+        const int src = p.rows_idx ? p.rows_idx[r] : r;
+        float* xr = p.x + (int64_t)src * p.H;
+        f32x4 x[MAXCH];
+#pragma unroll
+        for (int c = 0; c < MAXCH; c++) {
+            const int j = lane + c * 64;
+            x[c] = j < H4 ? *(const f32x4*)(xr + j * 4) : f32x4{0.f, 0.f, 0.f, 0.f};
+        }
+        if (p.y) {
+            f32x4 y[MAXCH];
+            float ss = 0.f;
+#pragma unroll
+            for (int c = 0; c < MAXCH; c++) {
+                const int j = lane + c * 64;
+                y[c] = j < H4 ? *(const f32x4*)(p.y + (int64_t)r * p.H + j * 4) : f32x4{0.f, 0.f, 0.f, 0.f};
+                ss += y[c][0] * y[c][0] + y[c][1] * y[c][1] + y[c][2] * y[c][2] + y[c][3] * y[c][3];
+            }
+            const float rms = sqrtf(wave_sum(ss) / (float)p.width + p.eps);
+#pragma unroll
+            for (int c = 0; c < MAXCH; c++) {
+                const int j = lane + c * 64;
+                if (j < H4) {
+                    const f32x4 w = *(const f32x4*)(p.w_post + j * 4);
+#pragma unroll
+                    for (int k = 0; k < 4; k++) x[c][k] += (y[c][k] / rms) * w[k];
+                    *(f32x4*)(xr + j * 4) = x[c];
+                }
+            }
+        }
+        if (p.w_next) {
+            float ss = 0.f;
+#pragma unroll
+            for (int c = 0; c < MAXCH; c++) ss += x[c][0] * x[c][0] + x[c][1] * x[c][1] + x[c][2] * x[c][2] + x[c][3] * x[c][3];
+            const float rms = sqrtf(wave_sum(ss) / (float)p.width + p.eps);
+#pragma unroll
+            for (int c = 0; c < MAXCH; c++) {
+                const int j = lane + c * 64;
+                if (j < H4) {
+                    const f32x4 w = *(const f32x4*)(p.w_next + j * 4);
+                    bf16x4 o;
+#pragma unroll
+                    for (int k = 0; k < 4; k++) o[k] = (bf16_t)((x[c][k] / rms) * w[k]);
+                    *(bf16x4*)(tile + wave * p.H + j * 4) = o;
+                }
+            }
+        }
+    }
+    if (!p.w_next) return;
+    __syncthreads();
+    const int nkb = p.H >> 5, lr = lane & 15, lc = lane >> 4;
+    if (blockIdx.x * 16 + lr < p.rows)
+        for (int kb = wave; kb < nkb; kb += 16)
+            *(bf16x8*)(xn + (((int64_t)blockIdx.x * nkb + kb) * 64 + lane) * 8) = *(const bf16x8*)(tile + lr * p.H + kb * 32 + lc * 8);
 }
 
 // Debug tap (nvl_set_debug mode 2): the residual stream after a layer as the NEXT kernel will see it — x plus whatever a
@@ -383,13 +516,13 @@ __global__ void fill_i32_kernel(int32_t* __restrict__ p, int32_t v, int n) {
     if (i < n) p[i] = v;
 }
 // h [rows][2F] = [gate | up] -> y [rows][F] = silu(gate)*up   (transformer.go:50-66)
-template <typename ActT>
+template <typename ActT, bool GELU = false>       // GELU: gelu_tanh(gate)*up
 __global__ void swiglu_kernel(const float* __restrict__ h, ActT* __restrict__ y, int64_t rows, int F) {
     const int64_t i = (int64_t)blockIdx.x * blockDim.x + threadIdx.x;
     if (i >= rows * F) return;
     const int64_t r = i / F; const int f = (int)(i - r * F);
     const float g = h[r * 2 * F + f], u = h[r * 2 * F + F + f];
-    ActIO<ActT>::st(y + i, (g / (1.0f + expf(-g))) * u);
+    ActIO<ActT>::st(y + i, (GELU ? gelu_tanh_f(g) : g / (1.0f + expf(-g))) * u);
 }
 __global__ void gelu_kernel(const float* __restrict__ x, float* __restrict__ y, int64_t n) {
     const int64_t i = (int64_t)blockIdx.x * blockDim.x + threadIdx.x;
@@ -496,7 +629,7 @@ __global__ __launch_bounds__(256) void decode_seam_kernel(const float* __restric
                                                           const bf16_t* __restrict__ emb, const bf16_t* __restrict__ pos_emb,
                                                           int max_seq, float mult, float* __restrict__ x,
                                                           const float* __restrict__ w, const float* __restrict__ b,
-                                                          float eps, bf16_t* __restrict__ y, int H) {
+                                                          float eps, bf16_t* __restrict__ y, int H, int width) {
     __shared__ float red[4];
     __shared__ int tok_s, pos_s;
     const int r = blockIdx.x;
@@ -549,7 +682,7 @@ __global__ __launch_bounds__(256) void decode_seam_kernel(const float* __restric
             if (b) bb[c] = *(const f32x4*)(b + j * 4);
         }
     }
-    norm_row_finish<bf16_t>(v, ww, bb, b, eps, y, r, H, red);
+    norm_row_finish<bf16_t>(v, ww, bb, b, eps, y, r, H, red, width);
 }
 
 // ---------------------------------------------------------------------------------------
@@ -848,6 +981,22 @@ __global__ void convert_1d_kernel(const void* __restrict__ src, int dtype, float
                                   int64_t src_off) {
     const int64_t i = (int64_t)blockIdx.x * blockDim.x + threadIdx.x;
     if (i < n) dst[i] = ld_as_f32(src, dtype, src_off + i);
+}
+
+// Placement of a [N][K] source into a larger, zero-filled destination [.][Kd]: source row n lands in row
+// row0 + (n / rg) * rgp + n % rg, source column k in column (k / cg) * cgp + k % cg (groups padded from rg to rgp rows, cg to cgp
+// columns: per-head padding, the 16-row interleave of gate and up).  TRANS: the destination's rows are the source's columns.
+struct Place2D { int64_t N, K, Kd, row0; int rg, rgp, cg, cgp; };
+template <typename DT, bool FM, bool TRANS>
+__global__ __launch_bounds__(256) void place_2d_kernel(const void* __restrict__ src, int dtype, int64_t src0, DT* __restrict__ dst, Place2D pl) {
+    const int64_t n = blockIdx.y;
+    for (int64_t k = (int64_t)blockIdx.x * 256 + threadIdx.x; k < pl.K; k += (int64_t)gridDim.x * 256) {
+        const float v = ld_as_f32(src, dtype, src0 + n * pl.K + k);
+        int64_t a = (n / pl.rg) * pl.rgp + n % pl.rg, b = (k / pl.cg) * pl.cgp + k % pl.cg;
+        if (TRANS) { const int64_t t = a; a = b; b = t; }
+        a += pl.row0;
+        dst[FM ? fm_index(a, b, pl.Kd) : a * pl.Kd + b] = (DT)v;
+    }
 }
 
 // tensor parallel: x[m][:] += alpha * (part[m][:] (+ bias))  after the all-reduce of a row-parallel projection

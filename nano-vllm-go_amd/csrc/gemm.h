@@ -39,7 +39,10 @@ enum GemmEpi {
     EPI_QKV = 4,     // fused QKV projection epilogue (head_dim 64 / 128): bias, RoPE on Q and K (rope.go:153-205),
                      // Q -> q buffer, K and V -> their KV slabs [pos][hd]  (replaces the fp32 qkv
                      // round trip + rope_kv_kernel in prefill; Concatenate tensor.go:283-321)
+    EPI_GEGLU = 5,   // C[m, f] = gelu_tanh(gate) * up   W rows interleaved as for EPI_SWIGLU
 };
+
+constexpr bool epi_glu(int epi) { return epi == 2 || epi == 5; }      // gate | up pairs in, one column out
 
 struct QkvEpi {             // EPI_QKV only
     const int32_t* tok_pos;
@@ -188,14 +191,14 @@ __device__ __forceinline__ float deferred_rstd(const GemmArgs& p, int m) {
     return 1.0f / sqrtf(s * p.rs_inv_h + p.rs_eps);
 }
 
-template <typename OutT, bool MOE = false>
-__device__ __forceinline__ void epilogue_swiglu4(const GemmArgs& p, int m, int f, f32x4 g, f32x4 u, float rstd = 1.0f) {
+template <int EPI, typename OutT, bool MOE = false>
+__device__ __forceinline__ void epilogue_glu4(const GemmArgs& p, int m, int f, f32x4 g, f32x4 u, float rstd = 1.0f) {
     // p.N counts fused rows (2F); the output has F = N/2 columns, ldc = F
     if (m >= p.M || f >= (p.N >> 1)) return;
     g *= rstd; u *= rstd;
     f32x4 v;
 #pragma unroll
-    for (int r = 0; r < 4; r++) v[r] = silu_f(g[r]) * u[r];
+    for (int r = 0; r < 4; r++) v[r] = (EPI == EPI_GEGLU ? gelu_tanh_f(g[r]) : silu_f(g[r])) * u[r];
     if constexpr (MOE) v *= p.moe_gate[m * p.moe_E + f / p.moe_I];      // routing weight of (token, expert); 0 = not routed
     act_store4<OutT>((OutT*)p.C, (int64_t)p.c_row0 + m, f, p.ldc, v);
 }
@@ -412,12 +415,12 @@ void gemm_bf16_kernel(GemmArgs p) {
             // the wave's column tile is exactly one head: TN = 4 <-> head_dim 64, TN = 8 <-> head_dim 128
             const int head = (n0 + wn * (TN * 16)) / (TN * 16);
             if (head * (TN * 16) < p.N) epilogue_qkv_head<TN>(p, m, head, fg, acc[i]);
-        } else if (EPI == EPI_SWIGLU) {
+        } else if (epi_glu(EPI)) {
 #pragma unroll
             for (int j = 0; j < TN; j += 2) {
                 const int ntile = (n0 + wn * (TN * 16) + j * 16) >> 4;   // even: gate block, +1: up block
                 const int f = (ntile >> 1) * 16 + 4 * fg;
-                epilogue_swiglu4<OutT>(p, m, f, acc[i][j], acc[i][j + 1]);
+                epilogue_glu4<EPI, OutT>(p, m, f, acc[i][j], acc[i][j + 1]);
             }
         } else if (EPI == EPI_RESID && p.sk_part) {
             GemmArgs q = p;                                   // this slice's partial tile: plain fp32 store, bias with slice 0
@@ -575,11 +578,11 @@ __global__ __launch_bounds__(512, 1) void gemm_bf16_pp_kernel(GemmArgs p) {
         if (EPI == EPI_QKV) {
             const int head = (n0 + wn * (TN * 16)) / (TN * 16);      // the wave's column block is exactly one head
             if (head * (TN * 16) < p.N) epilogue_qkv_head<TN>(p, m, head, fg, acc[i]);
-        } else if (EPI == EPI_SWIGLU) {
+        } else if (epi_glu(EPI)) {
 #pragma unroll
             for (int j = 0; j < TN; j += 2) {
                 const int ntile = (n0 + wn * (TN * 16) + j * 16) >> 4;
-                epilogue_swiglu4<OutT>(p, m, (ntile >> 1) * 16 + 4 * fg, acc[i][j], acc[i][j + 1]);
+                epilogue_glu4<EPI, OutT>(p, m, (ntile >> 1) * 16 + 4 * fg, acc[i][j], acc[i][j + 1]);
             }
         } else {
 #pragma unroll
@@ -662,7 +665,7 @@ __global__ __launch_bounds__(1024) void gemm_skinny_bf16_kernel(GemmArgs p) {
     // (MT = 4 — batches above 32 and the 64-row groups of larger ones — has no registers to hold it across the stream:
     // 34-54 spilled there, QKV at 128 rows 7.2 -> 10.8 us; those launches are long enough to fetch it in the epilogue)
     constexpr bool RSTD_PRE = MT <= 2;
-    const float rstd_pre = (RSTD_PRE && (EPI == EPI_STORE || EPI == EPI_SWIGLU) && wave < NTW * MT) ? deferred_rstd(p, 16 * i_pre + fr) : 1.0f;   // (only the waves that run an epilogue element)
+    const float rstd_pre = (RSTD_PRE && (EPI == EPI_STORE || epi_glu(EPI)) && wave < NTW * MT) ? deferred_rstd(p, 16 * i_pre + fr) : 1.0f;   // (only the waves that run an epilogue element)
     // (grid_y: gridDim.y as an explicit argument — the built-in lives in the hidden part of the kernarg block and costs a
     // dependent scalar round trip of its own before the first weight load)
     const int nslices = p.m_split ? 1 : p.grid_y, slice = p.m_split ? 0 : blockIdx.y;
@@ -792,10 +795,10 @@ __global__ __launch_bounds__(1024) void gemm_skinny_bf16_kernel(GemmArgs p) {
         for (int w = 1; w < ksplit; w++) s += red[((t * ksplit + w) * MT + i) * 64 + lane];
         return s;
     };
-    if (EPI == EPI_SWIGLU) {
+    if (epi_glu(EPI)) {
         for (int i = wave; i < MT; i += NTW * ksplit) {
             const int f = (nt0 >> 1) * 16 + 4 * fg;    // NTW == 2: tiles [gate 16 | up 16] of features 8*nt0..
-            epilogue_swiglu4<OutT, MOE>(p, 16 * i + fr, f, ksum(0, i), ksum(NTW - 1, i),
+            epilogue_glu4<EPI, OutT, MOE>(p, 16 * i + fr, f, ksum(0, i), ksum(NTW - 1, i),
                                         RSTD_PRE && i == i_pre ? rstd_pre : deferred_rstd(p, 16 * i + fr));
         }
     } else if (EPI == EPI_RESID && nslices > 1) {
@@ -927,7 +930,7 @@ __global__ __launch_bounds__(1024) void moe_router_gate_kernel(GemmArgs p, int t
 
 // ------------------------------------------------------------------------------------------
 // fp32 kernel (parity mode): 64x64 tile, BK=16, 256 threads, 4x4 outputs per thread, k ascending.
-// EPI_SWIGLU is not instantiated: the f32 path keeps W1 un-interleaved and applies the
+// EPI_SWIGLU / EPI_GEGLU are not instantiated: the f32 path keeps W1 un-interleaved and applies the
 // activation with swiglu_kernel.
 // ------------------------------------------------------------------------------------------
 template <int EPI, typename OutT>
@@ -1025,7 +1028,7 @@ __global__ __launch_bounds__(512) void gemm_skinny_wide_bf16_kernel(GemmArgs p) 
     // deferred RMSNorm: the scale of the rows this wave's epilogue elements belong to, fetched under the weight stream
     // (ahead of the first weight block: see the narrow kernel)
     const int i_pre = kw % MT;
-    const float rstd_pre = (EPI == EPI_SWIGLU || EPI == EPI_STORE) ? deferred_rstd(p, 16 * i_pre + fr) : 1.0f;
+    const float rstd_pre = (epi_glu(EPI) || EPI == EPI_STORE) ? deferred_rstd(p, 16 * i_pre + fr) : 1.0f;
     const bf16_t* wp = (const bf16_t*)p.W + (((int64_t)nt0 * nks + ks0) * 64 + lane) * 8;
     const bf16_t* xp = (const bf16_t*)p.A + ((int64_t)ks0 * 64 + lane) * 8;
     f32x4 acc[NTB][MT];
@@ -1092,12 +1095,12 @@ __global__ __launch_bounds__(512) void gemm_skinny_wide_bf16_kernel(GemmArgs p) 
         for (int w = 1; w < ksplit; w++) s += red[((w * NTB + t) * MT + i) * 64 + lane];
         return s;
     };
-    if (EPI == EPI_SWIGLU) {
+    if (epi_glu(EPI)) {
         // tiles come as [gate16 | up16] pairs of the same 16 features
         for (int e = kw; e < (NTB / 2) * MT; e += ksplit) {
             const int j = e / MT, i = e - j * MT;
             const int f = ((nt0 >> 1) + j) * 16 + 4 * fg;
-            epilogue_swiglu4<OutT, MOE>(p, 16 * i + fr, f, ksum(2 * j, i), ksum(2 * j + 1, i),
+            epilogue_glu4<EPI, OutT, MOE>(p, 16 * i + fr, f, ksum(2 * j, i), ksum(2 * j + 1, i),
                                         i == i_pre ? rstd_pre : deferred_rstd(p, 16 * i + fr));
         }
     } else {
@@ -1280,12 +1283,12 @@ static inline bool launch_gemm_skinny_bf16(hipStream_t st, const GemmArgs& a0) {
     if (skinny_rows(a0) > 64 || a0.a_rows || a0.seg || a0.tile_map) return false;
     GemmArgs a = a0;
     a.x_mask = (g_x_mask && a0.M % 16 != 0) ? 1 : 0;     // padded rows of the last 16-row activation tile are not fetched
-    if constexpr (EPI == EPI_SWIGLU || EPI == EPI_STORE || EPI == EPI_GELU) {
+    if constexpr (epi_glu(EPI) || EPI == EPI_STORE || EPI == EPI_GELU) {
         // wide-N form once its 64-row groups fill the chip (g_force_ntw: 8 forces it, 1/2/4 force the narrow form)
         const bool wide_ok = skinny_rows(a) > 16 && cdiv(a.N, 64) >= 256 && !a.sk_part;   // M <= 16: the narrow form streams as fast
         if (g_force_ntw == 8 || (g_force_ntw == 0 && wide_ok)) { if (launch_gemm_skinny_wide<EPI, OutT>(st, a)) return true; }
     }
-    if (EPI == EPI_SWIGLU) return launch_gemm_skinny_ntw<2, EPI, OutT>(st, a);
+    if (epi_glu(EPI)) return launch_gemm_skinny_ntw<2, EPI, OutT>(st, a);
     if (g_force_ntw == 2) return launch_gemm_skinny_ntw<2, EPI, OutT>(st, a);
     if (g_force_ntw == 4) return launch_gemm_skinny_ntw<4, EPI, OutT>(st, a);
     return launch_gemm_skinny_ntw<1, EPI, OutT>(st, a);

@@ -1,0 +1,803 @@
+// layered.h — models described by a list of layers (nvl_layer_config): every layer names a mixer (latent attention, Mamba-2, gated
+// linear attention), its sizes and its feed-forward, with a norm before and after each sublayer.  Host side: creation, tensor
+// staging, freezing into the kernels' layouts, the layer stack of one forward pass.  Included by nvllm.hip.
+//
+// What differs from the fixed-shape models around it:
+//   * widths need not be multiples of 64: rows, heads and latents are padded with zeros when the tensors are frozen (m->H is the
+//     padded row, m->Hn the real one), so the GEMM and norm kernels run unchanged;
+//   * the cache of a sequence is a slot (recurrent states, convolution rows) plus blocks of the library's pool (latents); blocks
+//     that no window reaches any more go back to the pool while the sequence runs (pool_trim);
+//   * a batch may mix prompt portions and single tokens: attention takes the absorbed form for sequences with up to
+//     LAT_ABSORB_MAX new tokens and the expanded form for the rest; recurrences go token by token up to REC_STEP_MAX.
+#pragma once
+
+namespace {
+
+constexpr int LAT_ABSORB_MAX = 16, LAT_ABSORB_MAX_RP = 512, LAT_SPLIT_MAX = 16, REC_STEP_MAX = 4;
+
+int pad_head(int d, int unit) {       // head sizes the attention instances exist for; larger ones take the plain kernel
+    for (int p : {32, 64, 128, 256}) if (d <= p) return p;
+    return (int)round_up(d, unit);
+}
+
+// ------------------------------------------------------------------------------------------
+// creation
+// ------------------------------------------------------------------------------------------
+int layered_create(const nvl_model_config& c, const nvl_layer_config* layers, const nvl_runtime_opts& opts, nvl_model** out) {
+    auto bad = [&](const std::string& why) { return fail(nullptr, NVL_ERR_INVALID, "nvl_create_layers: " + why); };
+    if (c.block_style != NVL_BLOCK_SANDWICH || c.activation_type != NVL_ACT_GEGLU) return bad("block_style NVL_BLOCK_SANDWICH and activation_type NVL_ACT_GEGLU expected");
+    if (c.hidden <= 0 || c.num_layers <= 0 || c.vocab_size <= 0 || c.max_seq_len <= 0) return bad("non-positive model dimension");
+    if (c.hidden > 20480) return bad("hidden larger than 20480");
+    if (opts.max_seqs <= 0) return bad("max_seqs must be >= 1");
+    if (opts.max_batch_tokens < 0 || opts.kv_num_blocks < 0 || opts.kv_block_size < 0 || opts.kv_block_size % 64) return bad("bad max_batch_tokens / kv_num_blocks / kv_block_size");
+    if (opts.tp_size > 1 || opts.tp_force_single) return bad("tensor parallelism does not cover models described by a list of layers");
+    const int L = c.num_layers;
+    for (int i = 0; i < L; i++) {
+        const nvl_layer_config& l = layers[i];
+        const std::string at = "layer " + std::to_string(i) + ": ";
+        if (l.heads <= 0 || l.vdim <= 0 || l.vdim > 2048 || l.ffn_dim < 0) return bad(at + "bad heads / vdim / ffn_dim");
+        switch (l.mixer) {
+            case NVL_MIXER_LATENT_ATTENTION:
+                if (l.dim <= 0 || l.q_rank <= 0 || l.kv_rank <= 0 || l.window < 0 || l.dim > 2048) return bad(at + "bad latent attention sizes");
+                break;
+            case NVL_MIXER_MAMBA2:
+                if (l.state <= 0 || l.state > 2048 || l.groups <= 0 || l.heads % l.groups || l.conv_taps <= 0 || l.norm_groups <= 0 ||
+                    (l.heads * l.vdim) % l.norm_groups) return bad(at + "bad Mamba-2 sizes");
+                break;
+            case NVL_MIXER_GLA:
+                if (l.dim <= 0 || l.dim > 2048 || !(l.tau > 0.f) || l.decay_rank < 0) return bad(at + "bad gated linear attention sizes");
+                break;
+            default: return bad(at + "unknown mixer");
+        }
+        if (l.weights_of >= L || l.weights_of == i) return bad(at + "weights_of names no other layer");
+    }
+    std::vector<int> owner((size_t)L);
+    for (int i = 0; i < L; i++) {
+        int o = i, hops = 0;
+        while (layers[o].weights_of >= 0) { o = layers[o].weights_of; if (++hops > L) return bad("weights_of goes round in a circle"); }
+        owner[(size_t)i] = o;
+        const nvl_layer_config &a = layers[i], &b = layers[o];
+        if (a.mixer != b.mixer || a.heads != b.heads || a.dim != b.dim || a.vdim != b.vdim || a.q_rank != b.q_rank || a.kv_rank != b.kv_rank ||
+            a.state != b.state || a.groups != b.groups || a.conv_taps != b.conv_taps || a.ffn_dim != b.ffn_dim)
+            return bad("layer " + std::to_string(i) + " does not have the shape of the layer whose tensors it uses");
+    }
+    if (opts.device < 0 || nvl_device_count() <= opts.device) return fail(nullptr, NVL_ERR_NO_DEVICE, "nvl_create_layers: no HIP device (this library has no CPU fallback)");
+    nvl_model* m = new (std::nothrow) nvl_model();
+    if (!m) return fail(nullptr, NVL_ERR_OOM, "nvl_create_layers: out of host memory");
+    try {
+        m->cfg = c; m->opts = opts; m->layered = true;
+        m->cfg.attention_type = NVL_ATTN_GQA; m->cfg.norm_type = NVL_NORM_RMS; m->cfg.position_type = NVL_POS_NONE; m->cfg.use_moe = 0;
+        m->f32 = opts.precision == NVL_PRECISION_F32;
+        m->wsize = m->f32 ? 4 : 2;
+        m->device = opts.device;
+        NVL_HIP(hipSetDevice(m->device));
+        NVL_HIP(hipStreamCreateWithFlags(&m->stream, hipStreamNonBlocking));
+        NVL_HIP(hipEventCreate(&m->ev0));
+        NVL_HIP(hipEventCreate(&m->ev1));
+        m->Hn = c.hidden; m->H = (int)round_up(c.hidden, 64); m->V = c.vocab_size; m->Vpad = (int)round_up(m->V, 128); m->L = L;
+        m->nH = m->nKV = 1; m->hd = 64; m->nH_full = m->nKV_full = 1;      // (unused by the layer stack)
+        m->layers.resize((size_t)L);
+        m->runs.resize((size_t)L); m->mixers.resize((size_t)L);
+        if (m->opts.max_batch_tokens <= 0) m->opts.max_batch_tokens = std::min(c.max_seq_len, 4096);
+        int64_t state = 0, cache = 0;
+        const int bs = opts.kv_block_size > 0 ? opts.kv_block_size : (opts.kv_num_blocks > 0 ? 256 : 64);
+        for (int i = 0; i < L; i++) {
+            LayerRun& r = m->runs[(size_t)i];
+            r.c = layers[i]; r.owner = owner[(size_t)i];
+            r.Fp = (int)round_up(r.c.ffn_dim, 64);
+            const int H = r.c.heads;
+            if (r.c.mixer == NVL_MIXER_LATENT_ATTENTION) {
+                r.dp = pad_head(r.c.dim, 64); r.vp = pad_head(r.c.vdim, 64);
+                r.qrp = (int)round_up(r.c.q_rank, 64); r.rp = (int)round_up(r.c.kv_rank, 64);
+                if (r.rp > 256 && r.rp < 512) r.rp = r.rp <= 384 ? 384 : 512;       // (instances of the absorbed form)
+                r.n_in = r.qrp + r.rp + H * r.vp; r.ko = (int)round_up((int64_t)H * r.vp, 64);
+                size_t w = 0;
+                while (w < m->windows.size() && m->windows[w] != r.c.window) w++;
+                if (w == m->windows.size()) m->windows.push_back(r.c.window);
+                r.win = (int)w;
+                r.cache_off = cache; cache += (int64_t)bs * r.rp;
+            } else {
+                const int DVp = (int)round_up(r.c.vdim, 4), DK = r.c.mixer == NVL_MIXER_MAMBA2 ? r.c.state : r.c.dim;
+                r.ko = (int)round_up((int64_t)H * r.c.vdim, 64);
+                r.state_off = state; state += round_up((int64_t)H * DK * DVp, 64);
+                if (r.c.mixer == NVL_MIXER_MAMBA2) {
+                    r.conv_dim = H * r.c.vdim + 2 * r.c.groups * r.c.state;
+                    r.n_in = H * r.c.vdim + r.conv_dim + H;
+                    r.ring_off = state; state += round_up((int64_t)r.c.conv_taps * r.conv_dim, 64);
+                }       // (GLA: n_in follows from the decay rank, layered_finalize)
+            }
+        }
+        m->lat_block_stride = cache; m->rec_slot_stride = state;
+        m->pool = 1; m->Tmax = bs; m->blocks_per_seq = cdiv(c.max_seq_len, bs);
+        if (opts.kv_num_blocks > 0) m->num_blocks = opts.kv_num_blocks;
+        else {      // what every slot can hold at once: its window and the tokens of the call that is running
+            int64_t span = c.max_seq_len;
+            int w = 0;
+            bool windowed = true;
+            for (int x : m->windows) { w = std::max(w, x); windowed &= x > 0; }
+            if (windowed) span = std::min<int64_t>(span, (int64_t)w + m->opts.max_batch_tokens + 2 * bs);
+            m->num_blocks = opts.max_seqs * cdiv(span, bs);
+        }
+        m->table_cap = opts.max_seqs * m->blocks_per_seq;
+        *out = m;
+        return NVL_OK;
+    } catch (const HipError& e) {
+        const std::string s = std::string("nvl_create_layers: HIP error: ") + hipGetErrorString(e.code);
+        delete m;
+        return fail(nullptr, NVL_ERR_HIP, s);
+    } catch (const std::exception& e) {
+        const std::string s = e.what();
+        delete m;
+        return fail(nullptr, NVL_ERR_INVALID, s);
+    }
+}
+
+// ------------------------------------------------------------------------------------------
+// tensors: staged on the device in the checkpoint's dtype, placed into the kernels' layouts by layered_finalize
+// ------------------------------------------------------------------------------------------
+void layered_shape(const nvl_model* m, int kind, int layer, int64_t& N, int64_t& K) {     // N = 0: the model has no such tensor; K = 1: a vector
+    const int64_t W = m->Hn;
+    N = 0; K = 1;
+    switch (kind) {
+        case NVL_T_TOK_EMB: case NVL_T_LM_HEAD: N = m->V; K = W; return;
+        case NVL_T_FINAL_NORM_W: N = W; return;
+        default: if (is_global(kind)) return;
+    }
+    const LayerRun& r = m->runs[(size_t)layer];
+    const nvl_layer_config& c = r.c;
+    if (r.owner != layer) return;
+    const bool lat = c.mixer == NVL_MIXER_LATENT_ATTENTION, mam = c.mixer == NVL_MIXER_MAMBA2, gla = c.mixer == NVL_MIXER_GLA;
+    const int64_t hv = (int64_t)c.heads * c.vdim, hd = (int64_t)c.heads * c.dim;
+    switch (kind) {
+        case NVL_T_ATTN_NORM_W: case NVL_T_MIX_POST_NORM: N = W; return;
+        case NVL_T_FFN_NORM_W: case NVL_T_FFN_POST_NORM: N = W; return;
+        case NVL_T_W1: N = 2 * (int64_t)c.ffn_dim; K = W; return;
+        case NVL_T_W2: if (c.ffn_dim) { N = W; K = c.ffn_dim; } return;
+        case NVL_T_WO: if (!mam) { N = W; K = hv; } return;
+        case NVL_T_MIX_GATE: if (!mam) { N = hv; K = W; } return;
+        case NVL_T_LAT_DQ: if (lat) { N = c.q_rank; K = W; } return;
+        case NVL_T_LAT_DQ_NORM: if (lat) N = c.q_rank; return;
+        case NVL_T_LAT_UQ: if (lat) { N = hd; K = c.q_rank; } return;
+        case NVL_T_LAT_DKV: if (lat) { N = c.kv_rank; K = W; } return;
+        case NVL_T_LAT_DKV_NORM: if (lat) N = c.kv_rank; return;
+        case NVL_T_LAT_UK: if (lat) { N = hd; K = c.kv_rank; } return;
+        case NVL_T_LAT_UV: if (lat) { N = hv; K = c.kv_rank; } return;
+        case NVL_T_WQ: case NVL_T_WK: if (gla) { N = hd; K = W; } return;
+        case NVL_T_WV: if (gla) { N = hv; K = W; } return;
+        case NVL_T_GLA_NORM: if (gla) N = c.vdim; return;
+        case NVL_T_GLA_A1: if (gla) { N = c.decay_rank ? c.decay_rank : -1; K = W; } return;       // -1: any
+        case NVL_T_GLA_A2: if (gla) { N = hd; K = c.decay_rank ? c.decay_rank : -1; } return;
+        case NVL_T_GLA_A2_B: if (gla) N = hd; return;
+        case NVL_T_MAMBA_IN_PROJ: if (mam) { N = r.n_in; K = W; } return;
+        case NVL_T_MAMBA_CONV_W: if (mam) N = (int64_t)r.conv_dim * c.conv_taps; return;
+        case NVL_T_MAMBA_CONV_B: if (mam) N = r.conv_dim; return;
+        case NVL_T_MAMBA_A_LOG: case NVL_T_MAMBA_D: case NVL_T_MAMBA_DT_BIAS: if (mam) N = c.heads; return;
+        case NVL_T_MAMBA_NORM: if (mam) N = hv; return;
+        case NVL_T_MAMBA_OUT_PROJ: if (mam) { N = W; K = hv; } return;
+        default: return;
+    }
+}
+bool layered_1d(int kind) {
+    if (is_1d(kind)) return true;
+    return kind == NVL_T_MIX_POST_NORM || kind == NVL_T_FFN_POST_NORM || kind == NVL_T_LAT_DQ_NORM || kind == NVL_T_LAT_DKV_NORM ||
+           kind == NVL_T_GLA_NORM || kind == NVL_T_GLA_A2_B;
+}
+int layered_upload(nvl_model* m, int kind, int layer, const void* data, int dtype, int64_t rows, int64_t cols, int layout) {
+    int64_t N, K;
+    layered_shape(m, kind, layer, N, K);
+    char buf[256];
+    if (N == 0) {
+        snprintf(buf, sizeof buf, "nvl_upload_tensor: layer %d has no tensor of kind %d", layer, kind);
+        return fail(m, NVL_ERR_INVALID, buf);
+    }
+    const bool vec = layered_1d(kind);
+    if (vec) { rows *= cols > 0 ? cols : 1; cols = 1; }
+    else if (layout != NVL_LAYOUT_OUT_IN && kind != NVL_T_TOK_EMB) return fail(m, NVL_ERR_INVALID, "nvl_upload_tensor: matrices of this model are given [out, in]");
+    if (rows <= 0 || cols <= 0 || (N > 0 && rows != N) || (K > 0 && cols != K)) {
+        snprintf(buf, sizeof buf, "tensor kind %d of layer %d: got [%lld,%lld], the model needs [%lld,%lld]", kind, layer, (long long)rows, (long long)cols, (long long)N, (long long)K);
+        return fail(m, NVL_ERR_INVALID, buf);
+    }
+    DevTensor* t = tensor_slot(m, kind, layer);
+    const size_t bytes = (size_t)(rows * cols) * (dtype == NVL_DTYPE_F32 ? 4 : 2);
+    dfree(t->p);
+    t->p = dmalloc_bytes((int64_t)bytes);
+    NVL_HIP(hipMemcpyAsync(t->p, data, bytes, hipMemcpyDefault, m->stream));
+    NVL_HIP(hipStreamSynchronize(m->stream));
+    t->rows = rows; t->cols = cols; t->rows_pad = rows; t->raw_dtype = dtype;
+    return NVL_OK;
+}
+
+void* lay_alloc(nvl_model* m, int64_t bytes, bool zero = true) {
+    void* p = dmalloc_bytes(bytes);
+    m->layered_allocs.push_back(p);
+    if (zero) NVL_HIP(hipMemsetAsync(p, 0, (size_t)std::max<int64_t>(bytes, 16), m->stream));
+    return p;
+}
+void* lay_matrix(nvl_model* m, int64_t N, int64_t Kd) {       // zero matrix of the weight dtype; rows padded to whole GEMM tiles
+    const int64_t bytes = round_up(N, W_ROW_PAD) * Kd * (int64_t)m->wsize;
+    m->stats.weight_bytes += (double)bytes;
+    return lay_alloc(m, bytes);
+}
+float* lay_vector(nvl_model* m, const DevTensor& t, int64_t padded) {
+    float* p = (float*)lay_alloc(m, padded * 4);
+    const int64_t n = t.rows * t.cols;
+    hipLaunchKernelGGL(convert_1d_kernel, dim3(cdiv(n, 256)), dim3(256), 0, m->stream, t.p, t.raw_dtype, p, n, (int64_t)0);
+    NVL_HIP(hipGetLastError());
+    m->stats.weight_bytes += (double)padded * 4;
+    return p;
+}
+// rows [n0, n0 + N) of a staged matrix into dst: grouped row / column padding as place_2d_kernel
+void lay_place(nvl_model* m, const DevTensor& t, void* dst, int64_t Kd, int64_t row0 = 0, int rg = 0, int rgp = 0, int cg = 0, int cgp = 0,
+               int64_t n0 = 0, int64_t N = -1, bool trans = false) {
+    if (N < 0) N = t.rows;
+    Place2D pl{N, t.cols, Kd, row0, rg ? rg : 1, rg ? rgp : 1, cg ? cg : 1, cg ? cgp : 1};
+    const dim3 grid((unsigned)std::min<int64_t>(cdiv(t.cols, 256), 64), (unsigned)N);
+    const int64_t src0 = n0 * t.cols;
+    if (m->f32) {
+        if (trans) hipLaunchKernelGGL((place_2d_kernel<float, false, true>), grid, dim3(256), 0, m->stream, t.p, t.raw_dtype, src0, (float*)dst, pl);
+        else hipLaunchKernelGGL((place_2d_kernel<float, false, false>), grid, dim3(256), 0, m->stream, t.p, t.raw_dtype, src0, (float*)dst, pl);
+    } else {
+        if (trans) hipLaunchKernelGGL((place_2d_kernel<bf16_t, true, true>), grid, dim3(256), 0, m->stream, t.p, t.raw_dtype, src0, (bf16_t*)dst, pl);
+        else hipLaunchKernelGGL((place_2d_kernel<bf16_t, true, false>), grid, dim3(256), 0, m->stream, t.p, t.raw_dtype, src0, (bf16_t*)dst, pl);
+    }
+    NVL_HIP(hipGetLastError());
+}
+
+// absorbed latent attention: available to a layer?
+bool lat_absorb_ok(const nvl_model* m, const LayerRun& r) { return !m->f32 && r.rp <= LAT_ABSORB_MAX_RP; }
+
+void layered_finalize(nvl_model* m) {
+    auto need = [&](const DevTensor& t, const std::string& what) -> const DevTensor& {
+        if (!t.present()) throw std::runtime_error("nvl_finalize: missing tensor: " + what);
+        return t;
+    };
+    const int64_t H = m->H;
+    need(m->g[NVL_T_TOK_EMB], "token embedding"); need(m->g[NVL_T_FINAL_NORM_W], "final norm");
+    m->final_norm = lay_vector(m, m->g[NVL_T_FINAL_NORM_W], H);
+    auto big = [&](int kind, const char* what) {      // [V][H]: the embedding table / LM head
+        void* p = lay_matrix(m, m->V, H);
+        lay_place(m, need(m->g[kind], what), p, H);
+        return p;
+    };
+    void* emb = big(NVL_T_TOK_EMB, "token embedding");
+    m->lm_head = m->g[NVL_T_LM_HEAD].present() && !m->cfg.tied_embedding ? big(NVL_T_LM_HEAD, "LM head") : emb;
+    NVL_HIP(hipStreamSynchronize(m->stream));
+    for (int k = 0; k < NVL_T_ATTN_NORM_W; k++) { dfree(m->g[k].p); m->g[k].p = nullptr; }
+    m->g[NVL_T_TOK_EMB].p = emb; m->g[NVL_T_TOK_EMB].raw_dtype = -1;      // (the embedding kernels' view of it)
+
+    int64_t ld_in = 0, q_cols = 0, cq_cols = 0, ko = 0, conv = 0, ocols = 0, Fmax = 0, abs_cols = 0;
+    for (int i = 0; i < m->L; i++) {
+        LayerRun& r = m->runs[(size_t)i];
+        const nvl_layer_config& c = r.c;
+        MixerW& w = m->mixers[(size_t)i];
+        LayerW& l = m->layers[(size_t)i];
+        const std::string at = "layer " + std::to_string(i) + " ";
+        if (r.owner == i) {
+            auto T = [&](int kind, const char* what) -> const DevTensor& { return need(l.t[kind], at + what); };
+            w.norm1 = lay_vector(m, T(NVL_T_ATTN_NORM_W, "norm before the mixer"), H);
+            w.norm1b = lay_vector(m, T(NVL_T_MIX_POST_NORM, "norm after the mixer"), H);
+            if (c.ffn_dim) {
+                w.norm2 = lay_vector(m, T(NVL_T_FFN_NORM_W, "norm before the feed-forward"), H);
+                w.norm2b = lay_vector(m, T(NVL_T_FFN_POST_NORM, "norm after the feed-forward"), H);
+                const DevTensor& w1 = T(NVL_T_W1, "feed-forward gate / up");
+                w.w1 = lay_matrix(m, 2 * r.Fp, H);
+                if (m->f32) { lay_place(m, w1, w.w1, H, 0, 0, 0, 0, 0, 0, c.ffn_dim); lay_place(m, w1, w.w1, H, r.Fp, 0, 0, 0, 0, c.ffn_dim, c.ffn_dim); }
+                else { lay_place(m, w1, w.w1, H, 0, 16, 32, 0, 0, 0, c.ffn_dim); lay_place(m, w1, w.w1, H, 16, 16, 32, 0, 0, c.ffn_dim, c.ffn_dim); }
+                w.w2 = lay_matrix(m, H, r.Fp);
+                lay_place(m, T(NVL_T_W2, "feed-forward down"), w.w2, r.Fp);
+            }
+            if (c.mixer == NVL_MIXER_LATENT_ATTENTION) {
+                w.in = lay_matrix(m, r.n_in, H);
+                lay_place(m, T(NVL_T_LAT_DQ, "query down projection"), w.in, H);
+                lay_place(m, T(NVL_T_LAT_DKV, "key/value down projection"), w.in, H, r.qrp);
+                lay_place(m, T(NVL_T_MIX_GATE, "output gate"), w.in, H, r.qrp + r.rp, c.vdim, r.vp);
+                w.dq_norm = lay_vector(m, T(NVL_T_LAT_DQ_NORM, "query latent norm"), r.qrp);
+                w.dkv_norm = lay_vector(m, T(NVL_T_LAT_DKV_NORM, "key/value latent norm"), r.rp);
+                w.uq = lay_matrix(m, (int64_t)c.heads * r.dp, r.qrp);
+                lay_place(m, T(NVL_T_LAT_UQ, "query up projection"), w.uq, r.qrp, 0, c.dim, r.dp);
+                const DevTensor& uk = T(NVL_T_LAT_UK, "key up projection");
+                w.uk = lay_matrix(m, (int64_t)c.heads * r.dp, r.rp);
+                lay_place(m, uk, w.uk, r.rp, 0, c.dim, r.dp);
+                if (lat_absorb_ok(m, r)) {
+                    w.ukt = lay_matrix(m, (int64_t)c.heads * r.rp, r.dp);
+                    for (int h = 0; h < c.heads; h++)
+                        lay_place(m, uk, (char*)w.ukt + (int64_t)h * r.rp * r.dp * (int64_t)m->wsize, r.dp, 0, 0, 0, 0, 0, (int64_t)h * c.dim, c.dim, true);
+                }
+                w.uv = lay_matrix(m, (int64_t)c.heads * r.vp, r.rp);
+                lay_place(m, T(NVL_T_LAT_UV, "value up projection"), w.uv, r.rp, 0, c.vdim, r.vp);
+                w.o = lay_matrix(m, H, r.ko);
+                lay_place(m, T(NVL_T_WO, "output projection"), w.o, r.ko, 0, 0, 0, c.vdim, r.vp);
+            } else if (c.mixer == NVL_MIXER_MAMBA2) {
+                w.in = lay_matrix(m, r.n_in, H);
+                lay_place(m, T(NVL_T_MAMBA_IN_PROJ, "input projection"), w.in, H);
+                w.conv_w = lay_vector(m, T(NVL_T_MAMBA_CONV_W, "convolution"), (int64_t)r.conv_dim * c.conv_taps);
+                w.conv_b = lay_vector(m, T(NVL_T_MAMBA_CONV_B, "convolution bias"), r.conv_dim);
+                w.a_log = lay_vector(m, T(NVL_T_MAMBA_A_LOG, "A_log"), c.heads);
+                w.dskip = lay_vector(m, T(NVL_T_MAMBA_D, "D"), c.heads);
+                w.dt_bias = lay_vector(m, T(NVL_T_MAMBA_DT_BIAS, "dt_bias"), c.heads);
+                w.mix_norm = lay_vector(m, T(NVL_T_MAMBA_NORM, "inner norm"), (int64_t)c.heads * c.vdim);
+                w.o = lay_matrix(m, H, r.ko);
+                lay_place(m, T(NVL_T_MAMBA_OUT_PROJ, "output projection"), w.o, r.ko);
+            } else {
+                const DevTensor& a1 = T(NVL_T_GLA_A1, "decay projection (a1)");
+                const DevTensor& a2 = T(NVL_T_GLA_A2, "decay projection (a2)");
+                if (a1.rows != a2.cols || a1.rows > 512) throw std::runtime_error("nvl_finalize: " + at + "the two decay projections do not fit (or their rank exceeds 512)");
+                w.rank = (int)a1.rows;
+                const int64_t hd = (int64_t)c.heads * c.dim, hv = (int64_t)c.heads * c.vdim;
+                w.in = lay_matrix(m, 2 * hd + 2 * hv + w.rank, H);
+                lay_place(m, T(NVL_T_WQ, "query projection"), w.in, H);
+                lay_place(m, T(NVL_T_WK, "key projection"), w.in, H, hd);
+                lay_place(m, T(NVL_T_WV, "value projection"), w.in, H, 2 * hd);
+                lay_place(m, T(NVL_T_MIX_GATE, "output gate"), w.in, H, 2 * hd + hv);
+                lay_place(m, a1, w.in, H, 2 * hd + 2 * hv);
+                w.a2 = lay_vector(m, a2, a2.rows * a2.cols);
+                w.a2_b = lay_vector(m, T(NVL_T_GLA_A2_B, "decay bias"), hd);
+                w.mix_norm = lay_vector(m, T(NVL_T_GLA_NORM, "head norm"), c.vdim);
+                w.o = lay_matrix(m, H, r.ko);
+                lay_place(m, T(NVL_T_WO, "output projection"), w.o, r.ko);
+            }
+            NVL_HIP(hipStreamSynchronize(m->stream));
+            for (auto& t : l.t) { dfree(t.p); t.p = nullptr; }
+        }
+    }
+    for (int i = 0; i < m->L; i++) {
+        LayerRun& r = m->runs[(size_t)i];
+        const nvl_layer_config& c = r.c;
+        if (c.mixer == NVL_MIXER_GLA) r.n_in = 2 * c.heads * (c.dim + c.vdim) + m->mixers[(size_t)r.owner].rank;
+        ld_in = std::max(ld_in, round_up(r.n_in, 4));
+        ko = std::max<int64_t>(ko, r.ko);
+        Fmax = std::max<int64_t>(Fmax, r.Fp);
+        if (c.mixer == NVL_MIXER_LATENT_ATTENTION) {
+            q_cols = std::max<int64_t>(q_cols, (int64_t)c.heads * r.dp);
+            cq_cols = std::max<int64_t>(cq_cols, r.qrp);
+            if (lat_absorb_ok(m, r)) abs_cols = std::max(abs_cols, round_up(c.heads, 16) * r.rp);
+        } else {
+            ocols = std::max<int64_t>(ocols, (int64_t)c.heads * c.vdim);
+            conv = std::max<int64_t>(conv, r.conv_dim);
+        }
+    }
+    m->F = (int)std::max<int64_t>(Fmax, 64);
+    const int64_t Mmax = m->opts.max_batch_tokens, S = m->opts.max_seqs, Mp = round_up(Mmax, 64), ws = (int64_t)m->wsize;
+    auto f32buf = [&](int64_t n) { return (float*)lay_alloc(m, n * 4); };
+    m->lproj_ld = ld_in; m->lq_ld = q_cols; m->lo_ld = round_up(ocols, 4); m->lconv_ld = round_up(conv, 4);
+    m->x = dmalloc<float>(Mmax * H);
+    m->xn = dmalloc_bytes(Mp * H * ws);
+    m->hbuf = dmalloc_bytes(Mp * m->F * ws);
+    m->xn_last = dmalloc_bytes(round_up(S, 64) * H * ws);
+    NVL_HIP(hipMemsetAsync(m->xn, 0, (size_t)(Mp * H * ws), m->stream));
+    NVL_HIP(hipMemsetAsync(m->hbuf, 0, (size_t)(Mp * m->F * ws), m->stream));
+    NVL_HIP(hipMemsetAsync(m->xn_last, 0, (size_t)(round_up(S, 64) * H * ws), m->stream));
+    if (m->f32) m->h2 = dmalloc<float>(Mmax * 2 * m->F);
+    m->lproj = f32buf(Mmax * ld_in);
+    m->ly = f32buf(Mmax * H);
+    if (q_cols) { m->lq = f32buf(Mmax * q_cols); m->lcq = lay_alloc(m, Mp * cq_cols * ws); }
+    m->lmix = lay_alloc(m, Mp * ko * ws);
+    if (ocols) m->lo = f32buf(Mmax * m->lo_ld);
+    if (conv) m->lconv = f32buf(Mmax * m->lconv_ld);
+    if (m->lat_block_stride) m->lat_cache = lay_alloc(m, m->lat_block_stride * m->num_blocks * ws);
+    if (m->rec_slot_stride) m->rec_state = f32buf(m->rec_slot_stride * S);
+    if (abs_cols) {     // tokens on the absorbed form, and their partial results: splits x tokens <= max(tokens, LAT_PART)
+        m->lat_abs_cap = (int)std::max<int64_t>(std::min(Mmax, S * LAT_ABSORB_MAX), 512);
+        m->lat_qa = (bf16_t*)lay_alloc(m, (int64_t)m->lat_abs_cap * abs_cols * 2);
+        m->lat_part_o = f32buf((int64_t)m->lat_abs_cap * abs_cols);
+        m->lat_part_ml = f32buf((int64_t)m->lat_abs_cap * abs_cols);
+    }
+    m->logit_rows = S;
+    m->logits = dmalloc<float>(S * (int64_t)m->Vpad);
+    m->argmax_dev = dmalloc<int32_t>(std::max<int64_t>(S, Mmax));
+    m->argmax_pval = dmalloc<float>(std::max<int64_t>(S, Mmax) * cdiv(m->V, ARGMAX_CHUNK));
+    m->argmax_pidx = dmalloc<int32_t>(std::max<int64_t>(S, Mmax) * cdiv(m->V, ARGMAX_CHUNK));
+    m->sk_rows = (int)std::min<int64_t>(std::max<int64_t>(Mmax, 64), SK_TILE_MAX_M);
+    if (!m->f32) m->sk_part = dmalloc<float>((int64_t)std::max(m->sk_max_slices, SK_TILE_MAX_SLICES) * m->sk_rows * H);
+    m->key_rows.assign(m->windows.size(), 0); m->key_max.assign(m->windows.size(), 0);
+    init_slots(m);
+    init_meta(m);
+    NVL_HIP(hipStreamSynchronize(m->stream));
+}
+
+void layered_free(nvl_model* m) {
+    if (!m->layered) return;
+    for (void* p : m->layered_allocs) dfree(p);
+    dfree(m->key_c); dfree(m->key_k); dfree(m->key_v); dfree(m->rec_z); dfree(m->rec_decay);
+    if (m->finalized) m->g[NVL_T_TOK_EMB].p = nullptr;
+    m->lm_head = nullptr;
+}
+
+// ------------------------------------------------------------------------------------------
+// the batch being enqueued
+// ------------------------------------------------------------------------------------------
+// Which tokens take the absorbed attention, and where every other sequence's keys sit in the key workspace.  hm: host metadata with
+// the sequences filled in; `steps` one-token passes will run on it (the positions advance on the device).
+void layered_meta(nvl_model* m, const Meta& hm, int n_seqs, int steps) {
+    bool absorb = !m->windows.empty();
+    for (const LayerRun& r : m->runs) if (r.c.mixer == NVL_MIXER_LATENT_ATTENTION) absorb &= lat_absorb_ok(m, r);
+    m->n_abs = 0; m->meta_dynamic = false;
+    m->min_len = hm.seq_len[0];
+    for (size_t w = 0; w < m->windows.size(); w++) { m->key_rows[w] = 0; m->key_max[w] = 0; }
+    const int64_t S = m->opts.max_seqs;
+    for (int i = 0; i < n_seqs; i++) {
+        const int n = hm.seq_len[i], pos = hm.seq_pos[i];
+        m->min_len = std::min(m->min_len, n);
+        const bool abs = absorb && n <= LAT_ABSORB_MAX;
+        if (abs) for (int j = 0; j < n; j++) { hm.abs_tok[m->n_abs] = hm.seq_tok_start[i] + j; hm.abs_seq[m->n_abs] = i; m->n_abs++; }
+        for (size_t w = 0; w < m->windows.size(); w++) {
+            if (abs) { hm.kbase[(int64_t)w * S + i] = -1; continue; }
+            int64_t nk = (int64_t)pos + n - latent_key0(pos, m->windows[w]);
+            if (steps > 1) {
+                nk = (int64_t)pos + n + steps;
+                if (m->windows[w] > 0) nk = std::min<int64_t>(nk, m->windows[w] + n + 31);
+            }
+            hm.kbase[(int64_t)w * S + i] = (int32_t)m->key_rows[w];
+            m->key_rows[w] += round_up(nk, 32);
+            m->key_max[w] = std::max<int>(m->key_max[w], (int)nk);
+            m->meta_dynamic = true;
+        }
+    }
+}
+
+// keys a launch has to cover in the absorbed form, as a power of two of 64-key tiles (a captured pass serves every context up to it)
+int layered_kt_log2(const nvl_model* m) {
+    int64_t ctx = m->ctx_hint > 0 ? m->ctx_hint : m->cfg.max_seq_len;
+    bool windowed = true;
+    int w = 0;
+    for (int x : m->windows) { windowed &= x > 0; w = std::max(w, x); }
+    if (windowed && !m->windows.empty()) ctx = std::min<int64_t>(ctx, w);
+    int b = 0;
+    while ((64ll << b) < ctx) b++;
+    return b;
+}
+int layered_decode_key(const nvl_model* m) { return layered_kt_log2(m); }
+
+// x += rms(y) * w_post and / or xn = rms(x) * w_next (elem.h SandwichArgs)
+void sandwich(nvl_model* m, const float* y, int slices, int64_t slice_stride, const float* w_post, const float* w_next, const int32_t* rows_idx,
+              void* xn, int rows) {
+    KScope ks(m, KC_OTHER, 0, KS_SANDWICH, (double)rows * m->Hn * ((y ? 8.0 + 4.0 * std::max(slices, 1) : 4.0) + (w_next ? (double)m->wsize : 0.0)));
+    SandwichArgs a{};
+    a.x = m->x; a.y = y; a.slices = slices; a.slice_stride = slice_stride; a.w_post = w_post; a.w_next = w_next; a.rows_idx = rows_idx;
+    a.rows = rows; a.H = m->H; a.width = m->Hn; a.eps = m->cfg.norm_eps;
+    if (!m->f32 && rows > 512 && m->H <= 4096 && slices <= 1) {
+        const size_t lds = (size_t)16 * m->H * 2;
+#define NVL_SW16(CH)                                                                                                        \
+        do {                                                                                                                \
+            NVL_LDS_ATTR((sandwich_tile16_kernel<CH>), 160 * 1024);                                                         \
+            hipLaunchKernelGGL((sandwich_tile16_kernel<CH>), dim3(cdiv(rows, 16)), dim3(1024), lds, m->stream, a, (bf16_t*)xn); \
+        } while (0)
+        if (m->H <= 1024) NVL_SW16(4); else if (m->H <= 2048) NVL_SW16(8); else NVL_SW16(16);
+#undef NVL_SW16
+    } else {
+#define NVL_SWR(CH)                                                                                                          \
+        do {                                                                                                                \
+            if (m->f32) hipLaunchKernelGGL((sandwich_row_kernel<float, CH>), dim3(rows), dim3(256), 0, m->stream, a, (float*)xn); \
+            else hipLaunchKernelGGL((sandwich_row_kernel<bf16_t, CH>), dim3(rows), dim3(256), 0, m->stream, a, (bf16_t*)xn);      \
+        } while (0)
+        if (m->H <= 1024) NVL_SWR(1); else if (m->H <= 2048) NVL_SWR(2); else if (m->H <= 4096) NVL_SWR(4); else NVL_SWR(20);
+#undef NVL_SWR
+    }
+    NVL_HIP(hipGetLastError());
+}
+
+// a sublayer's last projection: fp32 [M][H] in m->ly, or K-split partial sums in m->sk_part (the sandwich norm adds them up)
+struct SubOut { const float* y; int slices; int64_t stride; };
+SubOut sub_out(nvl_model* m, int site, const void* A, const void* W, int M, int K) {
+    const int N = m->H;
+    int slices = 1;
+    if (!m->f32 && M <= 64) {
+        const int nblocks = N / 16;
+        while (slices < m->sk_max_slices && nblocks * slices < 256 && (K >> 5) / (slices * 2) >= 8) slices *= 2;
+    } else if (!m->f32 && M <= 512 && M <= m->sk_rows && N % 128 == 0 && g_force_tile == 0) {
+        const int tiles = cdiv(M, 128) * (N / 128);
+        while (slices < SK_TILE_MAX_SLICES && tiles * slices < 512 && K / (slices * 2) >= 512) slices *= 2;
+        if (tiles * slices < 64) slices = 1;
+    }
+    m->site = site;
+    GemmArgs a = mk(A, K, W, m->ly, N, nullptr, 1.f, M, N, K);
+    if (slices > 1) {
+        a.C = m->x; a.sk_part = m->sk_part; a.sk_slices = slices;      // (EPI_RESID with slices: plain stores into sk_part, x is not touched)
+        gemm(m, EPI_RESID, true, a);
+        return {m->sk_part, slices, (int64_t)M * N};
+    }
+    gemm(m, EPI_STORE, true, a);
+    return {m->ly, 1, 0};
+}
+
+void grow(nvl_model* m, float*& p, int64_t& have, int64_t want) {
+    if (want <= have) return;
+    clear_graphs(m);
+    dfree(p);
+    p = dmalloc<float>(want);
+    have = want;
+}
+
+// ------------------------------------------------------------------------------------------
+// mixers: read the normed operand m->xn, leave the mixer's output before its last projection in m->lmix
+// ------------------------------------------------------------------------------------------
+void in_proj(nvl_model* m, const LayerRun& r, const MixerW& w, int M) {
+    m->site = KS_MIX_IN;
+    gemm(m, EPI_STORE, true, mk(m->xn, m->H, w.in, m->lproj, (int)m->lproj_ld, nullptr, 1.f, M, r.n_in, m->H));
+}
+
+void mix_latent(nvl_model* m, const LayerRun& r, const MixerW& w, const Meta& md, int n_seqs, int M, int max_len) {
+    const nvl_layer_config& c = r.c;
+    const int H = c.heads;
+    const double ws = (double)m->wsize;
+    in_proj(m, r, w, M);
+    LatentArgs a{};
+    a.H = H; a.dim = c.dim; a.dp = r.dp; a.vp = r.vp; a.qrank = c.q_rank; a.qrp = r.qrp; a.kvrank = c.kv_rank; a.rp = r.rp;
+    a.window = c.window; a.scale = c.scale; a.eps = m->cfg.norm_eps;
+    a.proj = m->lproj; a.proj_ld = m->lproj_ld; a.cq_norm = w.dq_norm; a.c_norm = w.dkv_norm; a.cq = m->lcq;
+    a.cache = (char*)m->lat_cache + r.cache_off * (int64_t)m->wsize; a.block_stride = m->lat_block_stride; a.bs = m->Tmax;
+    a.blk_table = md.blk_table; a.tok_pos = md.tok_pos; a.tok_tbl = md.tok_tbl; a.seq_tok_start = md.seq_tok_start; a.seq_len = md.seq_len;
+    a.seq_pos = md.seq_pos; a.tbl_stride = m->blocks_per_seq;
+    a.q = m->lq; a.q_ld = (int64_t)H * r.dp;
+    a.kbase = md.kbase + (int64_t)r.win * m->opts.max_seqs;
+    a.out = m->lmix; a.out_ld = r.ko;
+    {
+        KScope ks(m, KC_OTHER, 0, KS_LAT_NORM, (double)M * (c.q_rank + c.kv_rank) * (4.0 + ws));
+        if (m->f32) hipLaunchKernelGGL((latent_norm_kernel<float>), dim3(M), dim3(256), 0, m->stream, a);
+        else hipLaunchKernelGGL((latent_norm_kernel<bf16_t>), dim3(M), dim3(256), 0, m->stream, a);
+        NVL_HIP(hipGetLastError());
+    }
+    m->site = KS_LAT_UQ;
+    gemm(m, EPI_STORE, true, mk(m->lcq, r.qrp, w.uq, m->lq, H * r.dp, nullptr, 1.f, M, H * r.dp, r.qrp));
+    const int64_t rows = m->key_rows[(size_t)r.win];
+    if (rows > 0) {                       // sequences on the expanded form
+        if (rows > m->key_rows_cap) {
+            int64_t kc = 0, kk = 0, kv = 0;
+            for (const LayerRun& q : m->runs) if (q.c.mixer == NVL_MIXER_LATENT_ATTENTION) {
+                kc = std::max<int64_t>(kc, q.rp); kk = std::max<int64_t>(kk, (int64_t)q.c.heads * q.dp); kv = std::max<int64_t>(kv, (int64_t)q.c.heads * q.vp);
+            }
+            clear_graphs(m);
+            dfree(m->key_c); dfree(m->key_k); dfree(m->key_v);
+            m->key_c = m->key_k = m->key_v = nullptr; m->key_rows_cap = 0;
+            const int64_t cap = round_up(rows + rows / 4, 256) + 256, wsz = (int64_t)m->wsize;     // (+ whole GEMM tiles beyond the last row)
+            m->key_c = dmalloc_bytes(cap * kc * wsz); m->key_k = dmalloc_bytes(cap * kk * wsz); m->key_v = dmalloc_bytes(cap * kv * wsz);
+            NVL_HIP(hipMemsetAsync(m->key_c, 0, (size_t)(cap * kc * wsz), m->stream));
+            NVL_HIP(hipMemsetAsync(m->key_k, 0, (size_t)(cap * kk * wsz), m->stream));
+            NVL_HIP(hipMemsetAsync(m->key_v, 0, (size_t)(cap * kv * wsz), m->stream));
+            m->key_rows_cap = cap - 256;
+        }
+        a.cg = m->key_c; a.kx = m->key_k; a.vx = m->key_v; a.rows_pad = rows;
+        {
+            KScope ks(m, KC_OTHER, 0, KS_LAT_GATHER, 2.0 * (double)rows * c.kv_rank * ws);
+            const dim3 grid(cdiv(m->key_max[(size_t)r.win], 32), n_seqs);
+            if (m->f32) hipLaunchKernelGGL((latent_gather_kernel<float>), grid, dim3(256), 0, m->stream, a);
+            else hipLaunchKernelGGL((latent_gather_kernel<bf16_t>), grid, dim3(256), 0, m->stream, a);
+            NVL_HIP(hipGetLastError());
+        }
+        m->site = KS_LAT_KV;
+        gemm(m, EPI_STORE, m->f32, mk(m->key_c, r.rp, w.uk, m->key_k, H * r.dp, nullptr, 1.f, (int)rows, H * r.dp, r.rp));
+        m->site = KS_LAT_KV;
+        if (m->f32) gemm(m, EPI_STORE, true, mk(m->key_c, r.rp, w.uv, m->key_v, H * r.vp, nullptr, 1.f, (int)rows, H * r.vp, r.rp));
+        else gemm(m, EPI_STORE, false, mk(w.uv, r.rp, m->key_c, m->key_v, (int)rows, nullptr, 1.f, H * r.vp, (int)rows, r.rp));     // V^T = W_uv c^T
+        {
+            // visible (query, key) pairs are at most tokens x min(window, keys)
+            const double pairs = (double)(M - m->n_abs) * (c.window > 0 ? std::min<double>(c.window, m->key_max[(size_t)r.win]) : 0.5 * m->key_max[(size_t)r.win]);
+            KScope ks(m, KC_ATTN, 2.0 * pairs * H * (c.dim + c.vdim), KS_ATTN, ((double)rows * H * (c.dim + c.vdim)) * ws + (double)M * H * (4.0 * c.dim + 4.0 * c.vdim + ws * c.vdim));
+            if (m->f32 || r.dp > 256 || r.vp > 256) {
+                const dim3 grid(max_len, H, n_seqs);
+                const size_t lds = (size_t)(r.dp + r.vp) * 4;
+                if (m->f32) hipLaunchKernelGGL((latent_plain_kernel<float>), grid, dim3(256), lds, m->stream, a);
+                else hipLaunchKernelGGL((latent_plain_kernel<bf16_t>), grid, dim3(256), lds, m->stream, a);
+            } else {
+                const dim3 grid(cdiv(max_len, 128), H, n_seqs);
+#define NVL_LP(KSv, DTv) hipLaunchKernelGGL((latent_prefill_kernel<KSv, DTv>), grid, dim3(256), 0, m->stream, a)
+#define NVL_LPK(KSv)                                                                                        \
+                do {                                                                                         \
+                    if (r.vp == 32) NVL_LP(KSv, 2); else if (r.vp == 64) NVL_LP(KSv, 4);                      \
+                    else if (r.vp == 128) NVL_LP(KSv, 8); else NVL_LP(KSv, 16);                               \
+                } while (0)
+                if (r.dp == 32) NVL_LPK(1); else if (r.dp == 64) NVL_LPK(2); else if (r.dp == 128) NVL_LPK(4); else NVL_LPK(8);
+#undef NVL_LPK
+#undef NVL_LP
+            }
+            NVL_HIP(hipGetLastError());
+        }
+    }
+    if (m->n_abs > 0) {
+        const int n = m->n_abs, ht = cdiv(H, 16);
+        a.abs_tok = md.abs_tok; a.abs_seq = md.abs_seq; a.n_abs = n; a.ukt = (const bf16_t*)w.ukt; a.uv = (const bf16_t*)w.uv;
+        a.qa = m->lat_qa; a.Hp = ht * 16; a.part_o = m->lat_part_o; a.part_ml = m->lat_part_ml;
+        const int tiles = 1 << layered_kt_log2(m);
+        int split = 1;
+        while (split < LAT_SPLIT_MAX && ht * n * split < 256 && split * 2 <= tiles && (split * 2) * n <= m->lat_abs_cap) split *= 2;
+        a.n_split = split;
+        {
+            KScope ks(m, KC_OTHER, 2.0 * n * H * (double)c.dim * c.kv_rank, KS_LAT_ABSORB, (double)H * c.dim * c.kv_rank * 2.0 + (double)n * H * (4.0 * c.dim + 2.0 * c.kv_rank));
+            hipLaunchKernelGGL(latent_absorb_q_kernel, dim3(H, r.rp / 64, cdiv(n, 16)), dim3(256), 0, m->stream, a);
+            NVL_HIP(hipGetLastError());
+        }
+        {
+            const double keys = m->kv_tok > 0 && c.window > 0 ? std::min(m->kv_tok, (double)n * c.window) : (m->kv_tok > 0 ? m->kv_tok : (double)n * std::max(1, c.window));
+            KScope ks(m, KC_ATTN, 4.0 * keys * H * c.kv_rank, KS_ATTN, keys * c.kv_rank * 2.0 + (double)n * H * c.kv_rank * (2.0 + 4.0 * split));
+            const dim3 grid(ht, n, split);
+#define NVL_LD(NRv)                                                                                                        \
+            do {                                                                                                            \
+                constexpr int lds_ = latent_decode_lds_bytes<NRv>();                                                        \
+                NVL_LDS_ATTR((latent_decode_kernel<NRv>), lds_);                                                            \
+                hipLaunchKernelGGL((latent_decode_kernel<NRv>), grid, dim3(256), lds_, m->stream, a);                       \
+            } while (0)
+            switch (r.rp / 64) {
+                case 1: NVL_LD(1); break; case 2: NVL_LD(2); break; case 3: NVL_LD(3); break; case 4: NVL_LD(4); break;
+                case 6: NVL_LD(6); break; case 8: NVL_LD(8); break;
+                default: throw std::runtime_error("latent attention: no absorbed instance for this latent size");
+            }
+#undef NVL_LD
+            NVL_HIP(hipGetLastError());
+        }
+        {
+            KScope ks(m, KC_OTHER, 2.0 * n * H * (double)c.vdim * c.kv_rank, KS_LAT_UV, (double)H * c.vdim * c.kv_rank * 2.0 + (double)n * H * (4.0 * split * c.kv_rank + 6.0 * c.vdim));
+            hipLaunchKernelGGL(latent_uv_kernel, dim3(H, r.vp / 16, cdiv(n, 16)), dim3(256), 0, m->stream, a);
+            NVL_HIP(hipGetLastError());
+        }
+    }
+}
+
+// the recurrence of a layer over the batch; fused: one token (or a few) per sequence, everything between the projections in one launch
+template <bool CH>
+void linrec(nvl_model* m, LinRecArgs a, int n_seqs, int M, int max_len, bool fused, int site) {
+    const double elems = (double)a.H * a.DK * a.DVp;
+    const double bytes = (double)M * a.H * (2.0 * a.DK / a.kdiv + 2.0 * a.DV) * 4.0 + 2.0 * n_seqs * elems * 4.0;
+    KScope ks(m, KC_OTHER, 4.0 * (double)M * a.H * a.DK * a.DV, site, bytes);
+    const int lds = linrec_step_lds_bytes(a.DK, a.DVp);
+    const dim3 sgrid(a.H, n_seqs);
+    a.len_lo = 1; a.len_hi = 1 << 30;
+    if (fused) {
+        if (m->f32) hipLaunchKernelGGL((linrec_step_kernel<(CH ? 1 : 0) + 2, float>), sgrid, dim3(LR_STEP_THREADS), lds, m->stream, a);
+        else hipLaunchKernelGGL((linrec_step_kernel<(CH ? 1 : 0) + 2, bf16_t>), sgrid, dim3(LR_STEP_THREADS), lds, m->stream, a);
+        NVL_HIP(hipGetLastError());
+        return;
+    }
+    const int nk = a.DK <= 32 ? 2 : (a.DK <= 64 ? 4 : (a.DK <= 128 ? 8 : 16)), nw = a.DV <= 64 ? 4 : 8;
+    const bool chunks = a.DK <= 256 && (!CH || linrec_chunk_lds_bytes<16, 8, true>(a.rank) <= 160 * 1024 || nk < 16);
+    const bool steps = !chunks || m->min_len <= REC_STEP_MAX;
+    if (steps) {
+        a.len_hi = chunks ? REC_STEP_MAX : 1 << 30;
+        hipLaunchKernelGGL((linrec_step_kernel<(CH ? 1 : 0), float>), sgrid, dim3(LR_STEP_THREADS), lds, m->stream, a);
+        NVL_HIP(hipGetLastError());
+    }
+    if (!chunks || max_len <= REC_STEP_MAX) return;
+    a.len_lo = REC_STEP_MAX + 1; a.len_hi = 1 << 30;
+    a.n_slices = cdiv(a.DV, nw * 16);
+    // few (head, sequence, slice) workgroups and a long prompt: pieces of the prompt in parallel (MODE 1, prefix, MODE 2)
+    const int wgs = a.H * n_seqs * a.n_slices;
+    a.super = 0; a.n_super = 1;
+    if (wgs < 256 && max_len >= 512) {
+        const int want = std::max(2, 512 / wgs);
+        a.super = (int)round_up(std::max(128, cdiv(max_len, want)), 32);
+        a.n_super = cdiv(max_len, a.super);
+    }
+    const bool par = a.n_super > 1;
+    if (par) {
+        grow(m, m->rec_z, m->rec_z_floats, (int64_t)n_seqs * a.n_super * a.H * a.DK * a.DVp);
+        grow(m, m->rec_decay, m->rec_decay_floats, (int64_t)n_seqs * a.n_super * a.H * (CH ? a.DK : 1));
+        a.z = m->rec_z; a.zdecay = m->rec_decay;
+    }
+#define NVL_LC(NKv, NWv, MODEv)                                                                                              \
+    do {                                                                                                                     \
+        NVL_LDS_ATTR((linrec_chunk_kernel<NKv, NWv, CH, MODEv>), 160 * 1024);                                                \
+        hipLaunchKernelGGL((linrec_chunk_kernel<NKv, NWv, CH, MODEv>), dim3(a.H, n_seqs, a.n_slices * (MODEv ? a.n_super : 1)), dim3(NWv * 64), \
+                           (linrec_chunk_lds_bytes<NKv, NWv, CH>(a.rank)), m->stream, a);                                    \
+    } while (0)
+#define NVL_LCM(NKv, NWv)                                                                                                    \
+    do {                                                                                                                     \
+        if (par) {                                                                                                           \
+            NVL_LC(NKv, NWv, 1);                                                                                             \
+            hipLaunchKernelGGL((linrec_prefix_kernel<CH>), dim3(a.H, n_seqs, cdiv((int64_t)a.DK * a.DVp, 1024)), dim3(256), 0, m->stream, a); \
+            NVL_LC(NKv, NWv, 2);                                                                                             \
+        } else NVL_LC(NKv, NWv, 0);                                                                                          \
+    } while (0)
+#define NVL_LCN(NKv) do { if (nw == 4) NVL_LCM(NKv, 4); else NVL_LCM(NKv, 8); } while (0)
+    if (nk == 2) NVL_LCN(2); else if (nk == 4) NVL_LCN(4); else if (nk == 8) NVL_LCN(8); else NVL_LCN(16);
+#undef NVL_LCN
+#undef NVL_LCM
+#undef NVL_LC
+    NVL_HIP(hipGetLastError());
+}
+
+template <bool GATE_FIRST>
+void gated_norm(nvl_model* m, const GatedNormArgs& a, int site) {
+    KScope ks(m, KC_OTHER, 0, site, (double)a.rows * a.parts * a.part * (8.0 + (double)m->wsize));
+    const bool wide = a.part > 512;
+    const dim3 grid(wide ? a.rows * a.parts : cdiv((int64_t)a.rows * a.parts, 4));
+    if (m->f32) {
+        if (wide) hipLaunchKernelGGL((gated_norm_kernel<float, GATE_FIRST, true>), grid, dim3(256), 0, m->stream, a, (float*)m->lmix);
+        else hipLaunchKernelGGL((gated_norm_kernel<float, GATE_FIRST, false>), grid, dim3(256), 0, m->stream, a, (float*)m->lmix);
+    } else {
+        if (wide) hipLaunchKernelGGL((gated_norm_kernel<bf16_t, GATE_FIRST, true>), grid, dim3(256), 0, m->stream, a, (bf16_t*)m->lmix);
+        else hipLaunchKernelGGL((gated_norm_kernel<bf16_t, GATE_FIRST, false>), grid, dim3(256), 0, m->stream, a, (bf16_t*)m->lmix);
+    }
+    NVL_HIP(hipGetLastError());
+}
+
+LinRecArgs linrec_args(nvl_model* m, const LayerRun& r, const Meta& md) {
+    LinRecArgs a{};
+    a.H = r.c.heads; a.DV = r.c.vdim; a.DVp = (int)round_up(r.c.vdim, 4);
+    a.o = m->lo; a.o_ld = m->lo_ld;
+    a.state = m->rec_state + r.state_off; a.slot_stride = m->rec_slot_stride;
+    a.seq_tok_start = md.seq_tok_start; a.seq_len = md.seq_len; a.seq_pos = md.seq_pos; a.seq_slot = md.seq_slot;
+    a.eps = m->cfg.norm_eps; a.out = m->lmix; a.out_ld = r.ko;
+    return a;
+}
+
+void mix_mamba2(nvl_model* m, const LayerRun& r, const MixerW& w, const Meta& md, int n_seqs, int M, int max_len) {
+    const nvl_layer_config& c = r.c;
+    const int inner = c.heads * c.vdim, GN = c.groups * c.state;
+    in_proj(m, r, w, M);
+    LinRecArgs a = linrec_args(m, r, md);
+    a.DK = c.state; a.kdiv = c.heads / c.groups; a.q_scale = 1.f;
+    a.dt = m->lproj + inner + r.conv_dim; a.dt_ld = m->lproj_ld; a.dt_bias = w.dt_bias; a.a_log = w.a_log; a.Dskip = w.dskip;
+    float* ring = m->rec_state + r.ring_off;
+    const bool fused = max_len == 1;
+    if (fused) {
+        a.raw = m->lproj + inner; a.raw_ld = m->lproj_ld; a.conv_w = w.conv_w; a.conv_b = w.conv_b; a.taps = c.conv_taps; a.conv_dim = r.conv_dim;
+        a.ring = ring; a.ring_slot_stride = m->rec_slot_stride;
+    } else {
+        KScope ks(m, KC_OTHER, 0, KS_MAMBA_CONV, (double)M * r.conv_dim * 8.0);
+        ConvArgs v{};
+        v.raw = m->lproj + inner; v.raw_ld = m->lproj_ld; v.w = w.conv_w; v.b = w.conv_b; v.taps = c.conv_taps; v.channels = r.conv_dim;
+        v.out = m->lconv; v.out_ld = m->lconv_ld; v.ring = ring; v.ring_slot_stride = m->rec_slot_stride;
+        v.tok_seq = md.tok_seq; v.tok_pos = md.tok_pos; v.seq_tok_start = md.seq_tok_start; v.seq_len = md.seq_len; v.seq_pos = md.seq_pos; v.seq_slot = md.seq_slot;
+        hipLaunchKernelGGL(conv_silu_kernel, dim3(M), dim3(256), 0, m->stream, v);
+        hipLaunchKernelGGL(conv_ring_kernel, dim3(n_seqs, cdiv(r.conv_dim, 256)), dim3(256), 0, m->stream, v);
+        NVL_HIP(hipGetLastError());
+        a.v = m->lconv; a.k = m->lconv + inner; a.q = m->lconv + inner + GN; a.ld = m->lconv_ld;
+    }
+    linrec<false>(m, a, n_seqs, M, max_len, fused, KS_MAMBA_SCAN);
+    GatedNormArgs g{m->lo, m->lo_ld, m->lproj, m->lproj_ld, w.mix_norm, M, c.norm_groups, inner / c.norm_groups, m->cfg.norm_eps, r.ko};
+    gated_norm<true>(m, g, KS_MAMBA_GATE);
+}
+
+void mix_gla(nvl_model* m, const LayerRun& r, const MixerW& w, const Meta& md, int n_seqs, int M, int max_len) {
+    const nvl_layer_config& c = r.c;
+    const int64_t hd = (int64_t)c.heads * c.dim, hv = (int64_t)c.heads * c.vdim;
+    in_proj(m, r, w, M);
+    LinRecArgs a = linrec_args(m, r, md);
+    a.DK = c.dim; a.kdiv = 1; a.q_scale = 1.0f / sqrtf((float)c.dim);
+    a.q = m->lproj; a.k = m->lproj + hd; a.v = m->lproj + 2 * hd; a.ld = m->lproj_ld;
+    a.gate = m->lproj + 2 * hd + hv; a.gate_ld = m->lproj_ld; a.norm_w = w.mix_norm;
+    a.a1 = m->lproj + 2 * hd + 2 * hv; a.a1_ld = m->lproj_ld; a.rank = w.rank; a.a2 = w.a2; a.a2_b = w.a2_b; a.inv_tau = 1.0f / c.tau;
+    const bool fused = max_len <= REC_STEP_MAX;
+    linrec<true>(m, a, n_seqs, M, max_len, fused, KS_GLA_SCAN);
+    if (fused) return;
+    GatedNormArgs g{m->lo, m->lo_ld, a.gate, m->lproj_ld, w.mix_norm, M, c.heads, c.vdim, m->cfg.norm_eps, r.ko};
+    gated_norm<false>(m, g, KS_GLA_GATE);
+}
+
+void tap_layer(nvl_model* m, int li, int M);
+
+// The layers of one pass.  have_xn: m->xn already holds the first norm (decode seam).  all_rows: the logits of every row are wanted,
+// in order: the last sandwich norm then leaves the final norm of every row in m->xn; returns whether it did.
+bool layered_stack(nvl_model* m, const Meta& md, int n_seqs, int M, int max_len, bool have_xn, bool all_rows) {
+    auto W = [&](int li) -> const MixerW& { return m->mixers[(size_t)m->runs[(size_t)li].owner]; };
+    if (!have_xn) sandwich(m, nullptr, 0, 0, nullptr, W(0).norm1, nullptr, m->xn, M);
+    for (int li = 0; li < m->L; li++) {
+        const LayerRun& r = m->runs[(size_t)li];
+        const MixerW& w = W(li);
+        const float* after = li + 1 < m->L ? W(li + 1).norm1 : (all_rows ? m->final_norm : nullptr);      // the norm that follows this layer
+        switch (r.c.mixer) {
+            case NVL_MIXER_LATENT_ATTENTION: mix_latent(m, r, w, md, n_seqs, M, max_len); break;
+            case NVL_MIXER_MAMBA2: mix_mamba2(m, r, w, md, n_seqs, M, max_len); break;
+            default: mix_gla(m, r, w, md, n_seqs, M, max_len);
+        }
+        SubOut y = sub_out(m, KS_OPROJ, m->lmix, w.o, M, r.ko);
+        sandwich(m, y.y, y.slices, y.stride, w.norm1b, r.c.ffn_dim ? w.norm2 : after, nullptr, m->xn, M);
+        if (r.c.ffn_dim) {
+            m->site = KS_FFN_UP;
+            if (m->f32) {
+                gemm(m, EPI_STORE, true, mk(m->xn, m->H, w.w1, m->h2, 2 * r.Fp, nullptr, 1.f, M, 2 * r.Fp, m->H));
+                const int64_t n = (int64_t)M * r.Fp;
+                KScope ks(m, KC_OTHER);
+                hipLaunchKernelGGL((swiglu_kernel<float, true>), dim3(cdiv(n, 256)), dim3(256), 0, m->stream, m->h2, (float*)m->hbuf, (int64_t)M, r.Fp);
+                NVL_HIP(hipGetLastError());
+            } else {
+                gemm(m, EPI_GEGLU, false, mk(m->xn, m->H, w.w1, m->hbuf, r.Fp, nullptr, 1.f, M, 2 * r.Fp, m->H));
+            }
+            y = sub_out(m, KS_FFN_DOWN, m->hbuf, w.w2, M, r.Fp);
+            sandwich(m, y.y, y.slices, y.stride, w.norm2b, after, nullptr, m->xn, M);
+        }
+        tap_layer(m, li, M);
+    }
+    return all_rows;
+}
+
+}  // namespace

@@ -281,7 +281,115 @@ std::vector<float> to_f32(const StTensor& t) {
     for (int64_t i = 0; i < t.numel; i++) v[(size_t)i] = nvl_loader::f32_of(t, i);
     return v;
 }
+
+// ---- models described by a list of layers ("Potuzen") ----
+const char* const LAYERED_ARCH = "Potuzen";
+double need_num(const JVal* o, const char* key, const std::string& where) {
+    const JVal* v = o ? o->get(key) : nullptr;
+    if (!v || v->kind != JVal::NUM) throw std::runtime_error(where + "number '" + key + "' expected");
+    return v->num;
+}
+int need_int(const JVal* o, const char* key, const std::string& where) {
+    const double v = need_num(o, key, where);
+    if (v != std::floor(v) || v < -2147483648.0 || v > 2147483647.0) throw std::runtime_error(where + "'" + key + "' is not an integer");
+    return (int)v;
+}
+std::vector<nvl_layer_config> parse_layers(const JVal& raw) {
+    const JVal* ls = raw.get("layers");
+    if (!ls || ls->kind != JVal::ARR || ls->arr.empty()) throw std::runtime_error("config: list 'layers' expected");
+    std::vector<nvl_layer_config> out;
+    for (size_t i = 0; i < ls->arr.size(); i++) {
+        const JVal& e = ls->arr[i];
+        const std::string at = "config: layer " + std::to_string(i) + ": ";
+        nvl_layer_config c;
+        memset(&c, 0, sizeof c);
+        const JVal *ty = e.get("type"), *mx = e.get("mixer"), *mlp = e.get("mlp"), *wo = e.get("weights_of");
+        if (!ty || ty->kind != JVal::STR || !mx || mx->kind != JVal::OBJ) throw std::runtime_error(at + "'type' and 'mixer' expected");
+        c.weights_of = wo && wo->kind == JVal::NUM ? need_int(&e, "weights_of", at) : -1;
+        c.heads = need_int(mx, "heads", at); c.vdim = need_int(mx, "vdim", at);
+        if (ty->str == "latent_attention") {
+            c.mixer = NVL_MIXER_LATENT_ATTENTION;
+            c.dim = need_int(mx, "dim", at); c.q_rank = need_int(mx, "q_rank", at); c.kv_rank = need_int(mx, "kv_rank", at);
+            c.scale = (float)need_num(mx, "scale", at);
+            const JVal* mask = mx->get("mask");
+            if (mask && mask->kind == JVal::OBJ) {
+                c.window = need_int(mask, "size", at);
+                if (c.window <= 0) throw std::runtime_error(at + "the window is not positive");
+            }
+        } else if (ty->str == "mamba2") {
+            c.mixer = NVL_MIXER_MAMBA2;
+            c.state = need_int(mx, "state", at); c.groups = need_int(mx, "groups", at); c.norm_groups = need_int(mx, "norm_groups", at);
+            c.conv_taps = need_int(mx, "conv", at);
+        } else if (ty->str == "gla") {
+            c.mixer = NVL_MIXER_GLA;
+            c.dim = need_int(mx, "dim", at); c.tau = (float)need_num(mx, "tau", at);
+        } else throw std::runtime_error(at + "unknown mixer '" + ty->str + "'");
+        if (mlp && mlp->kind == JVal::OBJ) {
+            const JVal* kind = mlp->get("kind");
+            if (kind && !(kind->kind == JVal::STR && kind->str == "dense")) throw std::runtime_error(at + "unknown feed-forward kind");
+            c.ffn_dim = need_int(mlp, "ff", at);
+            if (c.ffn_dim <= 0) throw std::runtime_error(at + "the feed-forward size is not positive");
+        }
+        out.push_back(c);
+    }
+    return out;
+}
+void load_layered(nvl_model* m, const StSet& st) {
+    const int OI = NVL_LAYOUT_OUT_IN;
+    auto mat = [&](int kind, int layer, const std::string& name) { up2d(m, kind, layer, st.need(name), OI); };
+    auto vec = [&](int kind, int layer, const std::string& name) { up1d(m, kind, layer, st.need(name)); };
+    mat(NVL_T_TOK_EMB, 0, "embed");
+    mat(NVL_T_LM_HEAD, 0, "head");
+    vec(NVL_T_FINAL_NORM_W, 0, "final.norm");
+    for (int i = 0; i < m->L; i++) {
+        const LayerRun& r = m->runs[(size_t)i];
+        if (r.owner != i) continue;
+        const std::string l = "l" + std::to_string(i) + ".", x = l + "mix.";
+        vec(NVL_T_ATTN_NORM_W, i, l + "norm1"); vec(NVL_T_MIX_POST_NORM, i, l + "norm1b");
+        if (r.c.ffn_dim) {
+            vec(NVL_T_FFN_NORM_W, i, l + "norm2"); vec(NVL_T_FFN_POST_NORM, i, l + "norm2b");
+            const StTensor &g = st.need(l + "mlp.gate"), &u = st.need(l + "mlp.up");
+            if (u.dtype != g.dtype || u.shape != g.shape || g.shape.size() != 2) throw std::runtime_error("loader: " + l + "mlp.gate and .up do not match");
+            std::vector<uint8_t> cat(g.bytes + u.bytes);
+            memcpy(cat.data(), g.data, g.bytes);
+            memcpy(cat.data() + g.bytes, u.data, u.bytes);
+            if (nvl_upload_tensor(m, NVL_T_W1, i, cat.data(), g.dtype, 2 * g.shape[0], g.shape[1], OI)) throw std::runtime_error(nvl_last_error(m));
+            mat(NVL_T_W2, i, l + "mlp.down");
+        }
+        switch (r.c.mixer) {
+            case NVL_MIXER_LATENT_ATTENTION:
+                mat(NVL_T_LAT_DQ, i, x + "dq"); vec(NVL_T_LAT_DQ_NORM, i, x + "dq.norm"); mat(NVL_T_LAT_UQ, i, x + "uq");
+                mat(NVL_T_LAT_DKV, i, x + "dkv"); vec(NVL_T_LAT_DKV_NORM, i, x + "dkv.norm"); mat(NVL_T_LAT_UK, i, x + "uk"); mat(NVL_T_LAT_UV, i, x + "uv");
+                mat(NVL_T_MIX_GATE, i, x + "g"); mat(NVL_T_WO, i, x + "o");
+                break;
+            case NVL_MIXER_MAMBA2:
+                mat(NVL_T_MAMBA_IN_PROJ, i, x + "in"); vec(NVL_T_MAMBA_CONV_W, i, x + "conv"); vec(NVL_T_MAMBA_CONV_B, i, x + "conv.b");
+                vec(NVL_T_MAMBA_DT_BIAS, i, x + "dt_bias"); vec(NVL_T_MAMBA_A_LOG, i, x + "A_log"); vec(NVL_T_MAMBA_D, i, x + "D");
+                vec(NVL_T_MAMBA_NORM, i, x + "norm"); mat(NVL_T_MAMBA_OUT_PROJ, i, x + "o");
+                break;
+            default:
+                mat(NVL_T_WQ, i, x + "q"); mat(NVL_T_WK, i, x + "k"); mat(NVL_T_WV, i, x + "v"); mat(NVL_T_MIX_GATE, i, x + "g"); mat(NVL_T_WO, i, x + "o");
+                vec(NVL_T_GLA_NORM, i, x + "norm"); mat(NVL_T_GLA_A1, i, x + "a1"); mat(NVL_T_GLA_A2, i, x + "a2"); vec(NVL_T_GLA_A2_B, i, x + "a2.b");
+        }
+    }
+}
 }  // namespace
+
+extern "C" int nvl_load_layers_json(const char* path, nvl_layer_config* layers, int cap) {
+    if (!path || (cap > 0 && !layers)) return NVL_ERR_INVALID;
+    try {
+        const std::string txt = nvl_loader::read_text(path);
+        const JVal raw = nvl_loader::JParser(txt.c_str(), txt.size()).parse();
+        const JVal* a = raw.get("architecture");
+        if (!a || a->kind != JVal::STR || a->str != LAYERED_ARCH) return 0;
+        const auto ls = parse_layers(raw);
+        for (size_t i = 0; i < ls.size() && (int)i < cap; i++) layers[i] = ls[i];
+        return (int)ls.size();
+    } catch (const std::exception& e) {
+        g_create_err = std::string("nvl_load_layers_json: ") + e.what();
+        return NVL_ERR_INVALID;
+    }
+}
 
 extern "C" int nvl_load_safetensors(nvl_model* m, const char* path) {
     if (!m || !path) return NVL_ERR_INVALID;
@@ -290,6 +398,11 @@ extern "C" int nvl_load_safetensors(nvl_model* m, const char* path) {
     StSet st;
     st.open_path(path);
     const nvl_model_config& c = m->cfg;
+    if (m->layered) {
+        load_layered(m, st);
+        NVL_HIP(hipStreamSynchronize(m->stream));
+        return NVL_OK;
+    }
     // which WeightMapping (:60-181) — told from the checkpoint's own names
     const bool gpt2 = st.find("wte.weight") != nullptr;
     const bool falcon = st.find("transformer.word_embeddings.weight") != nullptr || st.find("word_embeddings.weight") != nullptr;
@@ -416,6 +529,16 @@ extern "C" int nvl_load_config_json(const char* path, nvl_model_config* out) {
         memset(&c, 0, sizeof c);
         // ---- templates (config.go:125-376); `architecture` first, then model_type (:822-836, :975-1007), default GPT-2
         std::string arch = str("architecture");
+        if (arch == LAYERED_ARCH) {       // sizes and constants come from the file; it names no longest sequence
+            c.vocab_size = need_int(&raw, "vocab", "config: "); c.hidden = need_int(&raw, "width", "config: ");
+            c.num_layers = (int)parse_layers(raw).size();
+            c.norm_eps = (float)need_num(raw.get("norm"), "eps", "config: norm: ");
+            c.max_seq_len = 4096;
+            c.attention_type = NVL_ATTN_GQA; c.norm_type = NVL_NORM_RMS; c.position_type = NVL_POS_NONE;
+            c.activation_type = NVL_ACT_GEGLU; c.block_style = NVL_BLOCK_SANDWICH;
+            *out = c;
+            return NVL_OK;
+        }
         const std::string mt = str("model_type");
         if (arch != "gpt2" && arch != "falcon" && arch != "llama") {
             if (mt == "gpt2") arch = "gpt2";

@@ -15,6 +15,8 @@
 #include "elem.h"
 #include "sample.h"
 #include "gemm.h"
+#include "latent.h"
+#include "linrec.h"
 #include "mamba.h"
 #include "tp_p2p.h"
 
@@ -23,6 +25,7 @@ namespace nvl {
 struct DevTensor {
     void* p = nullptr;      // canonical device copy: 2-D [rows_pad][cols] in weight dtype, 1-D fp32
     int64_t rows = 0, cols = 0, rows_pad = 0;
+    int raw_dtype = -1;     // >= 0: a staged copy in the checkpoint's dtype, row-major (models described by a list of layers, before finalize)
     bool present() const { return p != nullptr; }
 };
 
@@ -41,7 +44,31 @@ enum KClass { KC_GEMM = 0, KC_ATTN = 1, KC_OTHER = 2 };
 // where in the layer a launch sits (per-kernel roofline entries of nvl_get_kernel_stats; names in nvllm.hip)
 enum KSite { KS_OTHER = 0, KS_QKV, KS_ATTN, KS_OPROJ, KS_FFN_UP, KS_FFN_DOWN, KS_LM_HEAD, KS_NORM, KS_MOE_ROUTER, KS_MOE_PLAN,
              KS_MOE_UP, KS_MOE_DOWN, KS_MOE_COMBINE, KS_EMBED, KS_ARGMAX, KS_ROPE, KS_MAMBA_IN, KS_MAMBA_CONV, KS_MAMBA_SCAN,
-             KS_MAMBA_GATE, KS_MAMBA_OUT, KS_ALLREDUCE, KS_COUNT };
+             KS_MAMBA_GATE, KS_MAMBA_OUT, KS_ALLREDUCE, KS_MIX_IN, KS_LAT_NORM, KS_LAT_UQ, KS_LAT_GATHER, KS_LAT_KV, KS_LAT_ABSORB,
+             KS_LAT_UV, KS_GLA_SCAN, KS_GLA_GATE, KS_SANDWICH, KS_COUNT };
+
+// one layer of a model described by a list of layers: its configuration, padded sizes, where its tensors and its memory are
+struct LayerRun {
+    nvl_layer_config c{};
+    int owner = -1;              // the layer whose tensors it uses
+    int dp = 0, vp = 0, rp = 0, qrp = 0;     // padded head / latent sizes (latent attention)
+    int n_in = 0;                // columns of the fused input projection
+    int ko = 0;                  // K of the output projection (padded)
+    int Fp = 0;                  // feed-forward columns (padded), 0: none
+    int conv_dim = 0;
+    int win = -1;                // index into nvl_model::windows
+    int64_t cache_off = 0;       // latent attention: element offset inside a cache block
+    int64_t state_off = 0, ring_off = 0;     // recurrent layers: float offsets inside a slot
+};
+// its frozen tensors (owners only)
+struct MixerW {
+    void *in = nullptr, *o = nullptr, *w1 = nullptr, *w2 = nullptr;
+    void *uq = nullptr, *uk = nullptr, *ukt = nullptr, *uv = nullptr;
+    float *norm1 = nullptr, *norm1b = nullptr, *norm2 = nullptr, *norm2b = nullptr, *dq_norm = nullptr, *dkv_norm = nullptr;
+    float *conv_w = nullptr, *conv_b = nullptr, *a_log = nullptr, *dskip = nullptr, *dt_bias = nullptr, *mix_norm = nullptr;
+    float *a2 = nullptr, *a2_b = nullptr;
+    int rank = 0;
+};
 
 struct ProfRec { hipEvent_t a, b; int cls; double flops; int site, phase; double bytes; };
 struct SiteStat { double ms = 0, flops = 0, bytes = 0; uint64_t launches = 0; };
@@ -107,6 +134,33 @@ struct nvl_model {
     std::vector<char> slot_pin;        // 1 while the slot's sequence is part of the forward call being assembled
     uint64_t tick = 0;
 
+    // block pool (opts.kv_pool): the library names the blocks; per slot its block list (a block whose tokens no window can
+    // reach any more goes back to the pool and leaves -1 behind)
+    int pool = 0;
+    std::vector<std::vector<int32_t>> slot_blocks;
+    std::vector<int32_t> free_blocks;
+
+    // models described by a list of layers (layered.h)
+    bool layered = false;
+    int Hn = 0;                  // columns of the residual stream that carry data (H: padded to 64)
+    std::vector<nvl::LayerRun> runs;
+    std::vector<nvl::MixerW> mixers;
+    std::vector<void*> layered_allocs;
+    float *final_norm = nullptr;
+    std::vector<int> windows;    // distinct windows of the latent attention layers (0: none)
+    void* lat_cache = nullptr; int64_t lat_block_stride = 0;
+    float* rec_state = nullptr; int64_t rec_slot_stride = 0;
+    float *lproj = nullptr, *lq = nullptr, *ly = nullptr, *lconv = nullptr, *lo = nullptr;
+    void *lcq = nullptr, *lmix = nullptr;
+    int64_t lproj_ld = 0, lq_ld = 0, lo_ld = 0, lconv_ld = 0;
+    void *key_c = nullptr, *key_k = nullptr, *key_v = nullptr; int64_t key_rows_cap = 0;     // expanded latent attention, grown on demand
+    float *lat_part_o = nullptr, *lat_part_ml = nullptr; nvl::bf16_t* lat_qa = nullptr; int lat_abs_cap = 0;
+    float *rec_z = nullptr, *rec_decay = nullptr; int64_t rec_z_floats = 0, rec_decay_floats = 0;
+    // the batch being enqueued (layered_meta)
+    std::vector<int64_t> key_rows; std::vector<int> key_max;       // per window: rows of the key workspace, longest key list
+    int n_abs = 0; bool meta_dynamic = false;                      // tokens on the absorbed form; launch shapes depend on positions
+    int min_len = 1;
+
     // workspaces
     float* x = nullptr;          // residual stream fp32 [Mmax][H]
     void* xn = nullptr;          // normed activations (ActT)
@@ -149,6 +203,7 @@ struct nvl_model {
     SampleBufs samp;             // nvl_sample scratch
     int32_t* samp_hist = nullptr; int32_t* samp_hist_len = nullptr; int64_t samp_hist_cap = 0;   // nvl_decode_sampled: device-kept histories
     float* samp_u_steps = nullptr; int64_t samp_u_cap = 0;
+    int rows_named = -1;         // >= 0: the rows whose logits this pass computes (md.last_rows), set by forward_impl
     int last_rows = 0;           // logits rows the last forward left in `logits`
     int32_t* ring = nullptr; int64_t ring_ints = 0;   // nvl_decode_greedy: [steps][seqs] tokens on the device
     int32_t* ring_pos0 = nullptr;                     // position of every sequence when the fused loop started (ring row index)

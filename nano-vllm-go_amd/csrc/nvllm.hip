@@ -192,6 +192,7 @@ void gemm(nvl_model* m, int epi, bool out_f32, GemmArgs a, double flops = -1.0) 
             case EPI_RESID:  launch_gemm_bf16<EPI_RESID, float>(st, a); break;
             case EPI_SWIGLU: launch_gemm_bf16<EPI_SWIGLU, bf16_t>(st, a); break;
             case EPI_GELU:   launch_gemm_bf16<EPI_GELU, bf16_t>(st, a); break;
+            case EPI_GEGLU:  launch_gemm_bf16<EPI_GEGLU, bf16_t>(st, a); break;
             case EPI_QKV:    launch_gemm_bf16<EPI_QKV, bf16_t>(st, a); break;
             default: throw std::runtime_error("gemm: bad epilogue");
         }
@@ -212,6 +213,7 @@ extern "C" int nvl_sizeof(int which) {
         case 1: return (int)sizeof(nvl_runtime_opts);
         case 2: return (int)sizeof(nvl_stats);
         case 3: return (int)sizeof(nvl_sampling_params);
+        case 4: return (int)sizeof(nvl_layer_config);
         default: return -1;
     }
 }
@@ -224,10 +226,23 @@ extern "C" int nvl_device_count(void) {
 
 extern "C" const char* nvl_last_error(const nvl_model* m) { return m ? m->err.c_str() : g_create_err.c_str(); }
 
+namespace {
+// models described by a list of layers (layered.h)
+int layered_create(const nvl_model_config& c, const nvl_layer_config* layers, const nvl_runtime_opts& opts, nvl_model** out);
+int layered_upload(nvl_model* m, int kind, int layer, const void* data, int dtype, int64_t rows, int64_t cols, int layout);
+void layered_finalize(nvl_model* m);
+void layered_free(nvl_model* m);
+}  // namespace
+extern "C" int nvl_create_layers(const nvl_model_config* cfg, const nvl_layer_config* layers, const nvl_runtime_opts* opts, nvl_model** out) {
+    if (!cfg || !layers || !opts || !out) return fail(nullptr, NVL_ERR_INVALID, "nvl_create_layers: null argument");
+    *out = nullptr;
+    return layered_create(*cfg, layers, *opts, out);
+}
 extern "C" int nvl_create(const nvl_model_config* cfg, const nvl_runtime_opts* opts, nvl_model** out) {
     if (!cfg || !opts || !out) return fail(nullptr, NVL_ERR_INVALID, "nvl_create: null argument");
     *out = nullptr;
     const nvl_model_config& c = *cfg;
+    if (c.block_style == NVL_BLOCK_SANDWICH) return fail(nullptr, NVL_ERR_INVALID, "nvl_create: this model is described by a list of layers (nvl_create_layers)");
     if (c.hidden <= 0 || c.num_layers <= 0 || c.num_heads <= 0 || c.head_dim <= 0 || c.vocab_size <= 0 ||
         c.max_seq_len <= 0)
         return fail(nullptr, NVL_ERR_INVALID, "nvl_create: non-positive model dimension");
@@ -241,6 +256,7 @@ extern "C" int nvl_create(const nvl_model_config* cfg, const nvl_runtime_opts* o
     // a 0-block KV cache): max_seqs >= 1 is required, max_batch_tokens 0 selects max_seq_len
     if (opts->max_seqs <= 0)
         return fail(nullptr, NVL_ERR_INVALID, "nvl_create: max_seqs must be >= 1 (KV slots / sequences per call)");
+    if (c.activation_type == NVL_ACT_GEGLU) return fail(nullptr, NVL_ERR_INVALID, "nvl_create: GEGLU is available to models described by a list of layers");
     if (opts->max_batch_tokens < 0 || opts->kv_num_blocks < 0 || opts->kv_block_size < 0)
         return fail(nullptr, NVL_ERR_INVALID, "nvl_create: negative max_batch_tokens / kv_num_blocks / kv_block_size");
     const int tp = opts->tp_size > 1 ? opts->tp_size : 1;
@@ -268,7 +284,7 @@ extern "C" int nvl_create(const nvl_model_config* cfg, const nvl_runtime_opts* o
             (c.mamba_state_size / (256 / mhd)) % 4 != 0 || eh % 64 != 0 || c.mamba_num_heads % c.mamba_n_groups != 0)
             return fail(nullptr, NVL_ERR_INVALID, "nvl_create: Mamba2 head_dim / state_size not supported by the scan kernel");
         if (tp > 1) return fail(nullptr, NVL_ERR_INVALID, "nvl_create: tensor parallelism does not cover Mamba2 layers");
-        if (opts->kv_num_blocks > 0)
+        if (opts->kv_num_blocks > 0 && !opts->kv_pool)
             return fail(nullptr, NVL_ERR_INVALID, "nvl_create: Mamba2 layers keep per-sequence state in KV slots: not available in paged-KV mode");
         if (c.use_moe || c.block_style != NVL_BLOCK_SEQUENTIAL)
             return fail(nullptr, NVL_ERR_INVALID, "nvl_create: hybrid (Mamba2) models are sequential blocks with a dense MLP");
@@ -284,7 +300,7 @@ extern "C" int nvl_create(const nvl_model_config* cfg, const nvl_runtime_opts* o
     NVL_HIP(hipStreamCreateWithFlags(&m->stream, hipStreamNonBlocking));
     NVL_HIP(hipEventCreate(&m->ev0));
     NVL_HIP(hipEventCreate(&m->ev1));
-    m->H = c.hidden; m->nH = c.num_heads; m->hd = c.head_dim; m->F = c.ffn_dim; m->V = c.vocab_size;
+    m->H = m->Hn = c.hidden; m->nH = c.num_heads; m->hd = c.head_dim; m->F = c.ffn_dim; m->V = c.vocab_size;
     m->L = c.num_layers;
     m->nKV = c.attention_type == NVL_ATTN_MHA ? c.num_heads : (c.attention_type == NVL_ATTN_MQA ? 1 : c.num_kv_heads);
     if (m->nKV <= 0 || m->nH % m->nKV != 0) throw std::runtime_error("num_heads must be a multiple of num_kv_heads");
@@ -302,7 +318,8 @@ extern "C" int nvl_create(const nvl_model_config* cfg, const nvl_runtime_opts* o
     if (opts->kv_num_blocks > 0) {            // paged KV: the host's block manager names the blocks
         const int bs = opts->kv_block_size > 0 ? opts->kv_block_size : 256;
         if (bs % 64 != 0) throw std::runtime_error("kv_block_size must be a multiple of 64");
-        m->paged = 1; m->Tmax = bs; m->num_blocks = opts->kv_num_blocks;
+        m->pool = opts->kv_pool ? 1 : 0; m->paged = m->pool ? 0 : 1;
+        m->Tmax = bs; m->num_blocks = opts->kv_num_blocks;
         m->blocks_per_seq = cdiv(c.max_seq_len, bs);
     } else {
         m->num_blocks = opts->max_seqs;
@@ -338,6 +355,7 @@ extern "C" void nvl_destroy(nvl_model* m) {
     if (!m) return;
     (void)hipSetDevice(m->device);
     if (m->stream) (void)hipStreamSynchronize(m->stream);
+    layered_free(m);
     for (int k = 0; k < NVL_T_COUNT; k++) dfree(m->g[k].p);
     for (auto& l : m->layers) {
         for (int k = 0; k < NVL_T_COUNT; k++) dfree(l.t[k].p);
@@ -455,7 +473,9 @@ extern "C" int nvl_upload_tensor(nvl_model* m, int kind, int layer, const void* 
     if (dtype < 0 || dtype > 2) return fail(m, NVL_ERR_INVALID, "nvl_upload_tensor: unsupported dtype");
     DevTensor* t = tensor_slot(m, kind, layer);
     if (!t) return fail(m, NVL_ERR_INVALID, "nvl_upload_tensor: bad kind or layer");
+    if (!m->layered && kind >= NVL_T_MIX_POST_NORM) return fail(m, NVL_ERR_INVALID, "nvl_upload_tensor: the kind belongs to models described by a list of layers");
     NVL_TRY(m)
+    if (m->layered) return layered_upload(m, kind, layer, data, dtype, rows, cols, layout);
     NVL_HIP(hipSetDevice(m->device));
     char buf[256];
     const int r = m->tp_rank;
@@ -634,6 +654,26 @@ std::vector<int32_t> swiglu_interleave(int64_t F, int64_t src_base) {
     return idx;
 }
 
+void init_slots(nvl_model* m) {
+    m->slot_len.assign((size_t)m->opts.max_seqs, 0);
+    m->slot_tick.assign((size_t)m->opts.max_seqs, 0);
+    m->slot_pin.assign((size_t)m->opts.max_seqs, 0);
+    m->free_slots.clear();
+    for (int s = m->opts.max_seqs - 1; s >= 0; s--) m->free_slots.push_back(s);
+    m->slot_blocks.assign((size_t)m->opts.max_seqs, {});
+    m->free_blocks.clear();
+    if (m->pool) for (int b = m->num_blocks - 1; b >= 0; b--) m->free_blocks.push_back(b);
+}
+// per-call metadata: see bind_meta
+void init_meta(nvl_model* m) {
+    const int64_t Mmax = m->opts.max_batch_tokens, S = m->opts.max_seqs;
+    m->meta_ints = 5 * Mmax + (5 + (int64_t)m->windows.size()) * S + m->table_cap + 2 * (m->layered ? Mmax : 0) + 16;
+    NVL_HIP(hipHostMalloc((void**)&m->meta_host, (size_t)m->meta_ints * 4, hipHostMallocDefault));
+    m->meta_dev = dmalloc<int32_t>(m->meta_ints);
+    NVL_HIP(hipHostMalloc((void**)&m->am_host, (size_t)std::max<int64_t>(S, Mmax) * 4, hipHostMallocDefault));
+    m->ring_pos0 = dmalloc<int32_t>(S);
+}
+
 }  // namespace
 
 extern "C" int nvl_finalize(nvl_model* m) {
@@ -641,6 +681,7 @@ extern "C" int nvl_finalize(nvl_model* m) {
     if (m->finalized) return fail(m, NVL_ERR_STATE, "nvl_finalize: already finalized");
     NVL_TRY(m)
     NVL_HIP(hipSetDevice(m->device));
+    if (m->layered) { layered_finalize(m); m->finalized = true; return NVL_OK; }
     const nvl_model_config& c = m->cfg;
     const int64_t H = m->H, hd = m->hd;
     auto need = [&](bool ok, const char* what) { if (!ok) throw std::runtime_error(std::string("nvl_finalize: missing tensor: ") + what); };
@@ -776,11 +817,7 @@ extern "C" int nvl_finalize(nvl_model* m) {
     m->vcache = dmalloc_bytes(kv_elems * (int64_t)m->wsize);
     NVL_HIP(hipMemsetAsync(m->kcache, 0, (size_t)kv_elems * m->wsize, m->stream));
     NVL_HIP(hipMemsetAsync(m->vcache, 0, (size_t)kv_elems * m->wsize, m->stream));
-    m->slot_len.assign((size_t)m->opts.max_seqs, 0);
-    m->slot_tick.assign((size_t)m->opts.max_seqs, 0);
-    m->slot_pin.assign((size_t)m->opts.max_seqs, 0);
-    m->free_slots.clear();
-    for (int s = m->opts.max_seqs - 1; s >= 0; s--) m->free_slots.push_back(s);
+    init_slots(m);
 
     // ---- workspaces
     const int64_t Mmax = m->opts.max_batch_tokens, S = m->opts.max_seqs;
@@ -852,11 +889,7 @@ extern "C" int nvl_finalize(nvl_model* m) {
     if (!m->f32) m->sk_part = dmalloc<float>((int64_t)std::max(m->sk_max_slices, SK_TILE_MAX_SLICES) * m->sk_rows * H);
     if (!m->f32) m->rs_part = dmalloc<float>((int64_t)cdiv(H, 8) * DEFER_MAX_M);      // x^2 partials per 16 (half tiles: 8) columns
     if (m->tp > 1 || m->tp_force) m->tp_part = dmalloc<float>(Mmax * H);
-    m->meta_ints = 3 * Mmax + 5 * S + m->table_cap + 16;
-    NVL_HIP(hipHostMalloc((void**)&m->meta_host, (size_t)m->meta_ints * 4, hipHostMallocDefault));
-    m->meta_dev = dmalloc<int32_t>(m->meta_ints);
-    NVL_HIP(hipHostMalloc((void**)&m->am_host, (size_t)std::max<int64_t>(S, Mmax) * 4, hipHostMallocDefault));
-    m->ring_pos0 = dmalloc<int32_t>(S);
+    init_meta(m);
     NVL_HIP(hipStreamSynchronize(m->stream));   // every memset/copy above ran on the model's own (non-blocking) stream
     m->finalized = true;
     return NVL_OK;
@@ -988,6 +1021,47 @@ namespace {
 // forever and the engine never calls ClearCache (tensor_model_runner.go:11-18,59-68; llm_engine.go:35-37), so the runner
 // entry points evict; a later decode of an evicted sequence finds no slot and is re-prefilled from its full TokenIDs
 // (runner_impl), which is what makes eviction safe.  The explicit nvl_seq_open keeps its NVL_ERR_NO_SLOT contract.
+void pool_release(nvl_model* m, int slot) {
+    auto& b = m->slot_blocks[(size_t)slot];
+    for (int32_t x : b) if (x >= 0) m->free_blocks.push_back(x);
+    b.clear();
+}
+// Blocks for positions 0 .. end - 1 of a slot's sequence (pool mode).  evict: when the pool is empty, close the
+// least-recently-forwarded sequence that is not pinned and take its blocks.
+bool pool_reserve(nvl_model* m, int slot, int64_t end, bool evict) {
+    if (!m->pool) return true;
+    auto& b = m->slot_blocks[(size_t)slot];
+    while ((int64_t)b.size() * m->Tmax < end) {
+        if (m->free_blocks.empty()) {
+            if (!evict) return false;
+            auto victim = m->seq_slot.end();
+            for (auto jt = m->seq_slot.begin(); jt != m->seq_slot.end(); ++jt) {
+                if (jt->second == slot || m->slot_pin[(size_t)jt->second] || m->slot_blocks[(size_t)jt->second].empty()) continue;
+                if (victim == m->seq_slot.end() || m->slot_tick[(size_t)jt->second] < m->slot_tick[(size_t)victim->second]) victim = jt;
+            }
+            if (victim == m->seq_slot.end()) return false;
+            pool_release(m, victim->second);
+            m->free_slots.push_back(victim->second);
+            m->seq_slot.erase(victim);
+            m->stats.evictions++;
+            continue;
+        }
+        b.push_back(m->free_blocks.back());
+        m->free_blocks.pop_back();
+    }
+    return true;
+}
+// after a slot's sequence has grown to slot_len tokens: when every attention layer has a window, the blocks that lie before the
+// earliest key the next token can see go back to the pool
+void pool_trim(nvl_model* m, int slot) {
+    if (!m->pool || m->windows.empty()) return;
+    int w = 0;
+    for (int x : m->windows) { if (x == 0) return; w = std::max(w, x); }
+    auto& b = m->slot_blocks[(size_t)slot];
+    const int64_t first = (int64_t)m->slot_len[(size_t)slot] - w + 1;
+    for (int64_t i = 0; i < (int64_t)b.size() && (i + 1) * m->Tmax <= first; i++)
+        if (b[(size_t)i] >= 0) { m->free_blocks.push_back(b[(size_t)i]); b[(size_t)i] = -1; }
+}
 int seq_open_impl(nvl_model* m, int64_t seq_id, bool evict) {
     if (!m || !m->finalized) return fail(m, NVL_ERR_STATE, "nvl_seq_open: model not finalized");
     if (m->paged) return fail(m, NVL_ERR_STATE, "nvl_seq_open: the model is in paged-KV mode (the host's block manager owns the cache)");
@@ -1002,6 +1076,7 @@ int seq_open_impl(nvl_model* m, int64_t seq_id, bool evict) {
         }
         if (victim == m->seq_slot.end()) return fail(m, NVL_ERR_NO_SLOT, "nvl_runner_run: every KV slot belongs to the batch being assembled");
         m->free_slots.push_back(victim->second);
+        pool_release(m, victim->second);
         m->seq_slot.erase(victim);
         m->stats.evictions++;
     }
@@ -1019,6 +1094,7 @@ extern "C" int nvl_seq_reset(nvl_model* m, int64_t seq_id) {
     const int rc = nvl_seq_open(m, seq_id);
     if (rc) return rc;
     m->slot_len[(size_t)m->seq_slot[seq_id]] = 0;
+    pool_release(m, m->seq_slot[seq_id]);
     return NVL_OK;
 }
 extern "C" int nvl_seq_close(nvl_model* m, int64_t seq_id) {
@@ -1026,12 +1102,13 @@ extern "C" int nvl_seq_close(nvl_model* m, int64_t seq_id) {
     auto it = m->seq_slot.find(seq_id);
     if (it == m->seq_slot.end()) return NVL_OK;   // delete() of a missing key is a no-op in Go
     m->free_slots.push_back(it->second);
+    pool_release(m, it->second);
     m->seq_slot.erase(it);
     return NVL_OK;
 }
 extern "C" int nvl_seq_close_all(nvl_model* m) {
     if (!m) return NVL_ERR_INVALID;
-    for (auto& kv : m->seq_slot) m->free_slots.push_back(kv.second);
+    for (auto& kv : m->seq_slot) { m->free_slots.push_back(kv.second); pool_release(m, kv.second); }
     m->seq_slot.clear();
     return NVL_OK;
 }
@@ -1048,19 +1125,35 @@ extern "C" int nvl_seq_len(nvl_model* m, int64_t seq_id) {
 namespace {
 
 struct Meta {   // device pointers into meta_dev
-    int32_t *tokens, *tok_pos, *tok_tbl, *seq_tok_start, *seq_len, *seq_pos, *seq_tbl, *last_rows, *blk_table;
+    int32_t *tokens, *tok_pos, *tok_tbl, *tok_seq, *seq_tok_start, *seq_len, *seq_pos, *seq_tbl, *seq_slot, *last_rows, *blk_table, *kbase, *abs_tok, *abs_seq;
 };
 // layout of meta_host / meta_dev for a call carrying M tokens:
-//   [seq_tok_start S | seq_len S | seq_pos S | seq_tbl S | last_rows S | blk_table table_cap | tokens M | tok_pos M | tok_tbl M]
+//   [seq_tok_start S | seq_len S | seq_pos S | seq_tbl S | seq_slot S | kbase windows x S | blk_table table_cap |
+//    tokens M | tok_pos M | tok_tbl M | tok_seq M | last_rows M (the rows whose logits are wanted) | (layered) abs_tok M | abs_seq M]
+// (blk_table: sequence i's blocks start at i * blocks_per_seq; slab mode: one entry, its slot)
 Meta bind_meta(const nvl_model* m, int32_t* base, int M) {
     const int64_t S = m->opts.max_seqs;
     Meta md;
-    md.seq_tok_start = base; md.seq_len = base + S; md.seq_pos = base + 2 * S; md.seq_tbl = base + 3 * S;
-    md.last_rows = base + 4 * S; md.blk_table = base + 5 * S;
-    md.tokens = md.blk_table + m->table_cap; md.tok_pos = md.tokens + M; md.tok_tbl = md.tok_pos + M;
+    md.seq_tok_start = base; md.seq_len = base + S; md.seq_pos = base + 2 * S; md.seq_tbl = base + 3 * S; md.seq_slot = base + 4 * S;
+    md.kbase = base + 5 * S; md.blk_table = md.kbase + (int64_t)m->windows.size() * S;
+    md.tokens = md.blk_table + m->table_cap; md.tok_pos = md.tokens + M; md.tok_tbl = md.tok_pos + M; md.tok_seq = md.tok_tbl + M;
+    md.last_rows = md.tok_seq + M; md.abs_tok = md.last_rows + M; md.abs_seq = md.abs_tok + M;
     return md;
 }
-size_t meta_bytes(const nvl_model* m, int M) { return (size_t)(5 * (int64_t)m->opts.max_seqs + m->table_cap + 3 * (int64_t)M) * 4; }
+size_t meta_bytes(const nvl_model* m, int M) {
+    return (size_t)((5 + (int64_t)m->windows.size()) * (int64_t)m->opts.max_seqs + m->table_cap + (m->layered ? 7 : 5) * (int64_t)M) * 4;
+}
+// sequence i of the batch being assembled lives in `slot`: its table row, table start and slot
+void bind_slot(const nvl_model* m, const Meta& hm, int i, int slot) {
+    const int tb = i * m->blocks_per_seq;
+    hm.seq_tbl[i] = tb; hm.seq_slot[i] = slot;
+    if (m->pool) {
+        const auto& b = m->slot_blocks[(size_t)slot];
+        for (size_t j = 0; j < b.size(); j++) hm.blk_table[tb + (int64_t)j] = b[j] < 0 ? 0 : b[j];     // (released blocks are never read)
+    } else {
+        hm.blk_table[tb] = slot;
+    }
+}
 
 static int g_norm_t16 = 1;     // nvl_set_tuning key 9: norm_tile16_kernel for prefill-sized bf16 norms (0 = norm_kernel)
 template <typename ActT>
@@ -1129,7 +1222,8 @@ int decode_attn_cfg(const nvl_model* m, int n_seqs) {
     const int nw = n_kt <= 2 * per_wave ? 2 : (n_kt <= 4 * per_wave ? 4 : 8);
     return (g_attn_nw ? g_attn_nw : std::min(nw, cap)) | (1 << 8);
 }
-int decode_attn_waves(const nvl_model* m, int n_seqs) { return decode_attn_cfg(m, n_seqs); }   // (graph keys: the whole shape)
+int layered_decode_key(const nvl_model* m);
+int decode_attn_waves(const nvl_model* m, int n_seqs) { return m->layered ? layered_decode_key(m) : decode_attn_cfg(m, n_seqs); }   // (graph keys: the whole shape)
 void attention(nvl_model* m, int li, const Meta& md, int n_seqs, int max_len, double flops, bool fused_qkv = false) {
     AttnArgs a{};
     a.q = m->q; a.q_stride = m->nH * m->hd;
@@ -1570,6 +1664,8 @@ bool moe(nvl_model* m, const LayerW& l, int M, bool deferred_norm = false, const
 
 }  // namespace
 
+#include "layered.h"
+
 namespace {
 // ---- hipGraph replay of decode passes ----------------------------------------------------------------------------------
 // A decode pass is ~85 dependent launches of a few microseconds each.  A pass whose launch configuration (the key) has been
@@ -1651,6 +1747,8 @@ int enqueue_forward(nvl_model* m, const Meta& md, int n_seqs, int M, int max_len
         NVL_HIP(hipGetLastError());
     }
 
+    bool xn_final = false;          // m->xn already holds the final norm of every row (layered models)
+    if (m->layered) xn_final = layered_stack(m, md, n_seqs, M, max_len, (seam & 1) != 0, (flags & NVL_FWD_ALL_LOGITS) || (m->rows_named < 0 && M == n_seqs));
     const int qw = m->nH * m->hd;
     const bool parallel = c.block_style == NVL_BLOCK_PARALLEL;
 
@@ -1669,7 +1767,7 @@ int enqueue_forward(nvl_model* m, const Meta& md, int n_seqs, int M, int max_len
                               c.norm_type == NVL_NORM_RMS && H % 256 == 0 && m->rs_part && m->n_mamba == 0;
     const bool all_rows = (flags & NVL_FWD_ALL_LOGITS) != 0;
     bool xn_deferred = false;       // m->xn holds xn_raw of the upcoming norm, m->rs_part its x^2 partials
-    for (int li = 0; li < m->L; li++) {
+    for (int li = 0; li < m->L && !m->layered; li++) {
         const LayerW& l = m->layers[li];
         if (l.mamba) {
             // forwardMamba2 (generic_model.go:160-202): norm, Mamba2Layer.Forward (mamba2.go:74-181), residual; norm, shared MLP, residual
@@ -1684,8 +1782,8 @@ int enqueue_forward(nvl_model* m, const Meta& md, int n_seqs, int M, int max_len
             a.dt_bias = (const float*)l.t[NVL_T_MAMBA_DT_BIAS].p; a.norm_w = (const float*)l.t[NVL_T_MAMBA_NORM].p;
             a.xbc = m->mxbc; a.delta = m->mdelta; a.y = m->my;
             a.state = m->ssm_state + (int64_t)l.mamba_idx * m->ssm_layer_stride; a.state_slot_stride = m->ssm_slot_stride;
-            a.tok_pos = md.tok_pos; a.tok_seq = md.tok_tbl; a.seq_tok_start = md.seq_tok_start; a.seq_len = md.seq_len;
-            a.seq_pos = md.seq_pos; a.seq_slot = md.blk_table;     // slab mode: token -> sequence index i, blk_table[i] = slot
+            a.tok_pos = md.tok_pos; a.tok_seq = md.tok_seq; a.seq_tok_start = md.seq_tok_start; a.seq_len = md.seq_len;
+            a.seq_pos = md.seq_pos; a.seq_slot = md.seq_slot;
             a.chain = m->conv_tail ? m->conv_chain : 0;
             a.tail = m->conv_tail ? m->conv_tail + (int64_t)l.mamba_idx * m->conv_tail_layer_stride : nullptr;
             a.tail_slot_stride = m->conv_tail_slot_stride;
@@ -1836,7 +1934,9 @@ int enqueue_forward(nvl_model* m, const Meta& md, int n_seqs, int M, int max_len
 
     // ---- final norm + LM head on the rows the caller keeps (generic_model.go:464-477, :595-604) ----
     const bool all = (flags & NVL_FWD_ALL_LOGITS) != 0;
-    const int rows = all ? M : n_seqs;
+    const int rows = all ? M : (m->rows_named >= 0 ? m->rows_named : n_seqs);
+    m->last_rows = rows;
+    if (rows == 0) { m->ctx_hint = 0; return 0; }
     if (rows > m->logit_rows) {
         clear_graphs(m);               // (captured passes hold the old addresses)
         dfree(m->logits); dfree(m->xn_last);
@@ -1850,6 +1950,10 @@ int enqueue_forward(nvl_model* m, const Meta& md, int n_seqs, int M, int max_len
         set_deferred_in(m, al);
         m->site = KS_LM_HEAD;
         gemm(m, EPI_STORE, true, al);
+    } else if (m->layered) {
+        if (!xn_final) sandwich(m, nullptr, 0, 0, nullptr, m->final_norm, all ? nullptr : md.last_rows, m->xn_last, rows);
+        m->site = KS_LM_HEAD;
+        gemm(m, EPI_STORE, true, mk(xn_final ? m->xn : m->xn_last, H, m->lm_head, m->logits, m->Vpad, nullptr, 1.f, rows, m->V, H));
     } else {
         norm(m, m->x, all ? nullptr : md.last_rows, m->g[NVL_T_FINAL_NORM_W], m->g[NVL_T_FINAL_NORM_B], m->xn_last, rows);
         if (m->pending_slices != 0) throw std::runtime_error("forward: a split-K residual was left unconsumed");
@@ -1869,7 +1973,6 @@ int enqueue_forward(nvl_model* m, const Meta& md, int n_seqs, int M, int max_len
                       (seam & 2) ? nullptr : m->argmax_dev);
         NVL_HIP(hipGetLastError());
     }
-    m->last_rows = rows;
     m->ctx_hint = 0;
     return rows;
 }
@@ -1889,9 +1992,11 @@ __global__ void advance_decode_kernel(const int32_t* __restrict__ argmax, int32_
 }
 }  // namespace
 
-extern "C" int nvl_forward(nvl_model* m, int n_seqs, const int64_t* seq_ids, const int32_t* tokens,
-                           const int32_t* seq_lens, const int32_t* pos_offsets, uint32_t flags,
-                           float* logits_out, int32_t* argmax_out) {
+namespace {
+// n_rows < 0: the rows `flags` asks for (the last of each sequence, or all); else the rows named by `rows`.
+// evict: a pool without a free block may close the least-recently-forwarded sequences outside this batch (the runner's calls)
+int forward_impl(nvl_model* m, int n_seqs, const int64_t* seq_ids, const int32_t* tokens, const int32_t* seq_lens,
+                 const int32_t* pos_offsets, uint32_t flags, int n_rows, const int32_t* row_list, bool evict, float* logits_out, int32_t* argmax_out) {
     if (!m) return NVL_ERR_INVALID;
     if (!m->finalized) return fail(m, NVL_ERR_STATE, "nvl_forward: model not finalized");
     if (n_seqs <= 0 || !seq_ids || !tokens || !seq_lens || !pos_offsets)
@@ -1912,7 +2017,7 @@ extern "C" int nvl_forward(nvl_model* m, int n_seqs, const int64_t* seq_ids, con
     const int M = (int)M64;
     if (m->paged) return fail(m, NVL_ERR_STATE, "nvl_forward: the model is in paged-KV mode (use nvl_forward_paged)");
     const Meta hm = bind_meta(m, m->meta_host, M);
-    int32_t *h_sts = hm.seq_tok_start, *h_len = hm.seq_len, *h_pos = hm.seq_pos, *h_tbl = hm.seq_tbl, *h_last = hm.last_rows,
+    int32_t *h_sts = hm.seq_tok_start, *h_len = hm.seq_len, *h_pos = hm.seq_pos, *h_last = hm.last_rows,
             *h_tokens = hm.tokens, *h_tok_pos = hm.tok_pos, *h_tok_tbl = hm.tok_tbl;
     std::vector<int> h_slot((size_t)n_seqs);
     int t = 0;
@@ -1924,14 +2029,33 @@ extern "C" int nvl_forward(nvl_model* m, int n_seqs, const int64_t* seq_ids, con
         if (pos_offsets[i] != m->slot_len[(size_t)slot]) return fail(m, NVL_ERR_INVALID, "nvl_forward: pos_offset does not equal the cached length");
         if (pos_offsets[i] > c.max_seq_len - seq_lens[i])   // rope.go:84-86 / :176-178 panic
             return fail(m, NVL_ERR_POSITION, "nvl_forward: position exceeds max_seq_len");
-        // slab mode: the sequence's block table is the one entry blk_table[i] = its slot
-        h_sts[i] = t; h_len[i] = seq_lens[i]; h_pos[i] = pos_offsets[i]; h_slot[(size_t)i] = slot; h_tbl[i] = i; hm.blk_table[i] = slot;     // (blocks_per_seq == 1 here)
+        h_sts[i] = t; h_len[i] = seq_lens[i]; h_pos[i] = pos_offsets[i]; h_slot[(size_t)i] = slot;
         for (int j = 0; j < seq_lens[i]; j++, t++) {
             const int tok = tokens[t];
             if (tok < 0 || tok >= m->V) return fail(m, NVL_ERR_INVALID, "nvl_forward: token id out of range");
-            h_tokens[t] = tok; h_tok_pos[t] = pos_offsets[i] + j; h_tok_tbl[t] = i;
+            h_tokens[t] = tok; h_tok_pos[t] = pos_offsets[i] + j; h_tok_tbl[t] = i * m->blocks_per_seq; hm.tok_seq[t] = i;
         }
         h_last[i] = t - 1;
+    }
+    {   // cache blocks for the new tokens (pool mode), then every sequence's table row
+        std::vector<int> pinned;
+        for (int slot : h_slot) if (!m->slot_pin[(size_t)slot]) { m->slot_pin[(size_t)slot] = 1; pinned.push_back(slot); }
+        bool ok = true;
+        for (int i = 0; i < n_seqs && ok; i++) ok = pool_reserve(m, h_slot[(size_t)i], (int64_t)pos_offsets[i] + seq_lens[i], evict);
+        for (int slot : pinned) m->slot_pin[(size_t)slot] = 0;
+        if (!ok) return fail(m, NVL_ERR_NO_SLOT, "nvl_forward: the cache pool has no free block");
+        for (int i = 0; i < n_seqs; i++) bind_slot(m, hm, i, h_slot[(size_t)i]);
+    }
+    if (m->layered) layered_meta(m, hm, n_seqs, 1);
+    bool custom = false;
+    if (n_rows >= 0) {
+        if ((flags & NVL_FWD_ALL_LOGITS) || n_rows > M || (n_rows > 0 && !row_list)) return fail(m, NVL_ERR_INVALID, "nvl_forward_rows: bad row list");
+        custom = n_rows != n_seqs;
+        for (int i = 0; i < n_rows; i++) {
+            if (row_list[i] < 0 || row_list[i] >= M || (i > 0 && row_list[i] <= row_list[i - 1])) return fail(m, NVL_ERR_INVALID, "nvl_forward_rows: row indices must be increasing and inside the batch");
+            if (!custom && row_list[i] != h_last[i]) custom = true;
+        }
+        if (custom) for (int i = 0; i < n_rows; i++) h_last[i] = row_list[i];
     }
     const Meta md = bind_meta(m, m->meta_dev, M);
     NVL_HIP(hipEventRecord(m->ev0, m->stream));
@@ -1945,11 +2069,13 @@ extern "C" int nvl_forward(nvl_model* m, int n_seqs, const int64_t* seq_ids, con
     }
     m->kv_tok = kv_tok;
     const bool all = (flags & NVL_FWD_ALL_LOGITS) != 0;
-    int rows = all ? M : n_seqs;
+    int rows = all ? M : (custom ? n_rows : n_seqs);
+    struct Named { nvl_model* m; ~Named() { m->rows_named = -1; } } named{m};
+    m->rows_named = custom ? n_rows : -1;
     std::vector<int32_t> am;
     const int32_t* am_p = nullptr;
     bool replayed = false;
-    if (!prefill && rows <= m->logit_rows) {
+    if (!prefill && rows <= m->logit_rows && !custom && !m->meta_dynamic) {
         // a decode pass (what TensorModelRunner.Run issues every step): metadata upload + all launches + the argmax
         // download as ONE graph launch once this configuration has been seen
         const std::array<int, 5> key{0, n_seqs, decode_attn_waves(m, n_seqs), (int)flags, g_tune_epoch};
@@ -1964,11 +2090,11 @@ extern "C" int nvl_forward(nvl_model* m, int n_seqs, const int64_t* seq_ids, con
         NVL_HIP(hipMemcpyAsync(m->meta_dev, m->meta_host, meta_bytes(m, M), hipMemcpyHostToDevice, m->stream));
         rows = enqueue_forward(m, md, n_seqs, M, max_len, attn_flops, flags);
         am.resize((size_t)rows);
-        NVL_HIP(hipMemcpyAsync(am.data(), m->argmax_dev, (size_t)rows * 4, hipMemcpyDeviceToHost, m->stream));
+        if (rows) NVL_HIP(hipMemcpyAsync(am.data(), m->argmax_dev, (size_t)rows * 4, hipMemcpyDeviceToHost, m->stream));
         am_p = am.data();
     }
     NVL_HIP(hipEventRecord(m->ev1, m->stream));
-    if (logits_out)
+    if (logits_out && rows)
         NVL_HIP(hipMemcpy2DAsync(logits_out, (size_t)m->V * 4, m->logits, (size_t)m->Vpad * 4, (size_t)m->V * 4,
                                  (size_t)rows, hipMemcpyDeviceToHost, m->stream));
     NVL_HIP(hipStreamSynchronize(m->stream));
@@ -1977,9 +2103,13 @@ extern "C" int nvl_forward(nvl_model* m, int n_seqs, const int64_t* seq_ids, con
     m->last_rows = rows;
     if (argmax_out) {
         if (all) for (int i = 0; i < n_seqs; i++) argmax_out[i] = am_p[(size_t)h_last[i]];
-        else for (int i = 0; i < n_seqs; i++) argmax_out[i] = am_p[(size_t)i];
+        else for (int i = 0; i < rows; i++) argmax_out[i] = am_p[(size_t)i];
     }
-    for (int i = 0; i < n_seqs; i++) { m->slot_len[(size_t)h_slot[(size_t)i]] += seq_lens[i]; m->slot_tick[(size_t)h_slot[(size_t)i]] = ++m->tick; }
+    for (int i = 0; i < n_seqs; i++) {
+        const int slot = h_slot[(size_t)i];
+        m->slot_len[(size_t)slot] += seq_lens[i]; m->slot_tick[(size_t)slot] = ++m->tick;
+        pool_trim(m, slot);
+    }
     float ms = 0.f;
     (void)hipEventElapsedTime(&ms, m->ev0, m->ev1);
     m->stats.forward_calls++;
@@ -1988,6 +2118,17 @@ extern "C" int nvl_forward(nvl_model* m, int n_seqs, const int64_t* seq_ids, con
     if (m->profile) drain_profile(m);
     return NVL_OK;
     NVL_CATCH(m)
+}
+}  // namespace
+extern "C" int nvl_forward(nvl_model* m, int n_seqs, const int64_t* seq_ids, const int32_t* tokens,
+                           const int32_t* seq_lens, const int32_t* pos_offsets, uint32_t flags,
+                           float* logits_out, int32_t* argmax_out) {
+    return forward_impl(m, n_seqs, seq_ids, tokens, seq_lens, pos_offsets, flags, -1, nullptr, false, logits_out, argmax_out);
+}
+extern "C" int nvl_forward_rows(nvl_model* m, int n_seqs, const int64_t* seq_ids, const int32_t* tokens, const int32_t* seq_lens,
+                                const int32_t* pos_offsets, int n_rows, const int32_t* rows, float* logits_out, int32_t* argmax_out) {
+    if (n_rows < 0) return fail(m, NVL_ERR_INVALID, "nvl_forward_rows: negative row count");
+    return forward_impl(m, n_seqs, seq_ids, tokens, seq_lens, pos_offsets, 0, n_rows, rows, false, logits_out, argmax_out);
 }
 
 // nvl_forward for a model whose KV cache is the host block manager's pool (block_manager.go:128-263,
@@ -2035,7 +2176,7 @@ extern "C" int nvl_forward_paged(nvl_model* m, int n_seqs, const int32_t* tokens
         for (int j = 0; j < seq_lens[i]; j++, t++) {
             const int tok = tokens[t];
             if (tok < 0 || tok >= m->V) return fail(m, NVL_ERR_INVALID, "nvl_forward_paged: token id out of range");
-            hm.tokens[t] = tok; hm.tok_pos[t] = pos_offsets[i] + j; hm.tok_tbl[t] = tb;
+            hm.tokens[t] = tok; hm.tok_pos[t] = pos_offsets[i] + j; hm.tok_tbl[t] = tb; hm.tok_seq[t] = i;
         }
         hm.last_rows[i] = t - 1;
     }
@@ -2129,6 +2270,17 @@ extern "C" int nvl_runner_run_paged(nvl_model* m, int n_seqs, const int32_t* con
 }
 
 namespace {
+// blocks, table rows and (layered) metadata of n_steps one-token passes
+bool decode_reserve(nvl_model* m, const Meta& hm, const std::vector<int>& slots, int n_steps) {
+    for (size_t i = 0; i < slots.size(); i++)
+        if (!pool_reserve(m, slots[i], (int64_t)m->slot_len[(size_t)slots[i]] + n_steps, false)) return false;
+    for (size_t i = 0; i < slots.size(); i++) bind_slot(m, hm, (int)i, slots[i]);
+    if (m->layered) layered_meta(m, hm, (int)slots.size(), n_steps);
+    return true;
+}
+void decode_advance(nvl_model* m, const std::vector<int>& slots, int n_steps) {
+    for (int slot : slots) { m->slot_len[(size_t)slot] += n_steps; m->slot_tick[(size_t)slot] = ++m->tick; pool_trim(m, slot); }
+}
 // the n_steps decode passes of nvl_decode_greedy[_paged]: metadata for step 0 is in meta_host (one token per sequence),
 // every later step's tokens / positions are produced on the device
 // `sp` != NULL: every step samples (tensor.SampleWithHistory, sample.h) instead of taking the argmax; the histories live
@@ -2176,14 +2328,14 @@ void decode_loop(nvl_model* m, const Meta& hm, int n_seqs, int n_steps, int32_t*
         if (seam_ok) {
             const void* pe = (m->cfg.position_type == NVL_POS_LEARNED) ? m->g[NVL_T_POS_EMB].p : nullptr;
             const int pe_rows = pe ? (int)std::min<int64_t>(m->g[NVL_T_POS_EMB].rows, m->cfg.max_seq_len) : 0;
-            const LayerW& l0 = m->layers[0];
+            const float* norm0 = m->layered ? m->mixers[(size_t)m->runs[0].owner].norm1 : (const float*)m->layers[0].t[NVL_T_ATTN_NORM_W].p;
+            const float* bias0 = m->layered ? nullptr : (const float*)m->layers[0].t[NVL_T_ATTN_NORM_B].p;
             hipLaunchKernelGGL(decode_seam_kernel, dim3(n_seqs), dim3(256), 0, m->stream, m->argmax_pval, m->argmax_pidx,
                                cdiv(m->V, ARGMAX_CHUNK), sp ? (const int32_t*)m->samp.out : (const int32_t*)nullptr, m->samp_hist,
                                (int64_t)m->cfg.max_seq_len, m->samp_hist_len, m->argmax_dev, m->ring, (const int32_t*)m->ring_pos0, n_seqs,
                                md.tokens, md.tok_pos,
                                md.seq_pos, (const bf16_t*)m->g[NVL_T_TOK_EMB].p, (const bf16_t*)pe, pe_rows,
-                               m->cfg.embedding_multiplier, m->x, (const float*)l0.t[NVL_T_ATTN_NORM_W].p,
-                               (const float*)l0.t[NVL_T_ATTN_NORM_B].p, m->cfg.norm_eps, (bf16_t*)m->xn, m->H);
+                               m->cfg.embedding_multiplier, m->x, norm0, bias0, m->cfg.norm_eps, (bf16_t*)m->xn, m->H, m->Hn);
         } else {
             hipLaunchKernelGGL(advance_decode_kernel, dim3(cdiv(n_seqs, 256)), dim3(256), 0, m->stream, m->argmax_dev, md.tokens,
                                md.tok_pos, md.seq_pos, m->ring + (int64_t)s * n_seqs, n_seqs);
@@ -2193,7 +2345,7 @@ void decode_loop(nvl_model* m, const Meta& hm, int n_seqs, int n_steps, int32_t*
         // steps 1.. of the greedy seam loop launch the SAME kernels with the SAME arguments (the ring row comes from the
         // positions): one captured graph per (batch, attention wave count), replayed
         bool replayed = false;
-        if (s > 0 && seam_ok && !sp) {
+        if (s > 0 && seam_ok && !sp && !m->meta_dynamic) {
             const std::array<int, 5> key{1, n_seqs, decode_attn_waves(m, n_seqs), 0, g_tune_epoch};
             replayed = replay_or_capture(m, key, one_step);
             if (replayed) m->ctx_hint = 0;
@@ -2230,7 +2382,7 @@ extern "C" int nvl_decode_greedy(nvl_model* m, int n_seqs, const int64_t* seq_id
     if (m->paged) return fail(m, NVL_ERR_STATE, "nvl_decode_greedy: not available in paged-KV mode");
     const int M = n_seqs;
     const Meta hm = bind_meta(m, m->meta_host, M);
-    int32_t *h_sts = hm.seq_tok_start, *h_len = hm.seq_len, *h_pos = hm.seq_pos, *h_tbl = hm.seq_tbl, *h_last = hm.last_rows,
+    int32_t *h_sts = hm.seq_tok_start, *h_len = hm.seq_len, *h_pos = hm.seq_pos, *h_last = hm.last_rows,
             *h_tokens = hm.tokens, *h_tok_pos = hm.tok_pos, *h_tok_tbl = hm.tok_tbl;
     std::vector<int> h_slot((size_t)n_seqs);
     for (int i = 0; i < n_seqs; i++) {
@@ -2240,11 +2392,12 @@ extern "C" int nvl_decode_greedy(nvl_model* m, int n_seqs, const int64_t* seq_id
         const int slot = it->second, pos = m->slot_len[(size_t)slot];
         if (pos + n_steps > m->cfg.max_seq_len) return fail(m, NVL_ERR_POSITION, "nvl_decode_greedy: position exceeds max_seq_len");
         if (first_tokens[i] < 0 || first_tokens[i] >= m->V) return fail(m, NVL_ERR_INVALID, "nvl_decode_greedy: token id out of range");
-        h_sts[i] = i; h_len[i] = 1; h_pos[i] = pos; h_slot[(size_t)i] = slot; h_last[i] = i; h_tbl[i] = i; hm.blk_table[i] = slot;
-        h_tokens[i] = first_tokens[i]; h_tok_pos[i] = pos; h_tok_tbl[i] = i;
+        h_sts[i] = i; h_len[i] = 1; h_pos[i] = pos; h_slot[(size_t)i] = slot; h_last[i] = i;
+        h_tokens[i] = first_tokens[i]; h_tok_pos[i] = pos; h_tok_tbl[i] = i * m->blocks_per_seq; hm.tok_seq[i] = i;
     }
+    if (!decode_reserve(m, hm, h_slot, n_steps)) return fail(m, NVL_ERR_NO_SLOT, "nvl_decode_greedy: the cache pool has no free block");
     decode_loop(m, hm, n_seqs, n_steps, out_tokens);
-    for (int i = 0; i < n_seqs; i++) { m->slot_len[(size_t)h_slot[(size_t)i]] += n_steps; m->slot_tick[(size_t)h_slot[(size_t)i]] = ++m->tick; }
+    decode_advance(m, h_slot, n_steps);
     return NVL_OK;
     NVL_CATCH(m)
 }
@@ -2283,7 +2436,7 @@ extern "C" int nvl_decode_greedy_paged(nvl_model* m, int n_seqs, const int32_t* 
             hm.blk_table[tb + j] = b;
         }
         hm.seq_tok_start[i] = i; hm.seq_len[i] = 1; hm.seq_pos[i] = pos; hm.seq_tbl[i] = tb; hm.last_rows[i] = i;
-        hm.tokens[i] = first_tokens[i]; hm.tok_pos[i] = pos; hm.tok_tbl[i] = tb;
+        hm.tokens[i] = first_tokens[i]; hm.tok_pos[i] = pos; hm.tok_tbl[i] = tb; hm.tok_seq[i] = i;
     }
     decode_loop(m, hm, n_seqs, n_steps, out_tokens);
     return NVL_OK;
@@ -2330,8 +2483,7 @@ extern "C" int nvl_decode_sampled(nvl_model* m, int n_seqs, const int64_t* seq_i
         }
         hlen[(size_t)i] = hn;
         hm.seq_tok_start[i] = i; hm.seq_len[i] = 1; hm.seq_pos[i] = pos; h_slot[(size_t)i] = slot; hm.last_rows[i] = i;
-        hm.seq_tbl[i] = i; hm.blk_table[i] = slot;
-        hm.tokens[i] = first_tokens[i]; hm.tok_pos[i] = pos; hm.tok_tbl[i] = i;
+        hm.tokens[i] = first_tokens[i]; hm.tok_pos[i] = pos; hm.tok_tbl[i] = i * m->blocks_per_seq; hm.tok_seq[i] = i;
     }
     for (int64_t i = 0; i < (int64_t)n_steps * n_seqs; i++)
         if (!(uniforms[i] >= 0.f && uniforms[i] <= 1.f)) return fail(m, NVL_ERR_INVALID, "nvl_decode_sampled: uniform draw outside [0, 1]");
@@ -2361,8 +2513,9 @@ extern "C" int nvl_decode_sampled(nvl_model* m, int n_seqs, const int64_t* seq_i
     NVL_HIP(hipMemcpyAsync(m->samp_hist, hist.data(), hist.size() * 4, hipMemcpyHostToDevice, m->stream));
     NVL_HIP(hipMemcpyAsync(m->samp_hist_len, hlen.data(), hlen.size() * 4, hipMemcpyHostToDevice, m->stream));
     NVL_HIP(hipMemcpyAsync(m->samp_u_steps, uniforms, (size_t)n_steps * n_seqs * 4, hipMemcpyHostToDevice, m->stream));
+    if (!decode_reserve(m, hm, h_slot, n_steps)) return fail(m, NVL_ERR_NO_SLOT, "nvl_decode_sampled: the cache pool has no free block");
     decode_loop(m, hm, n_seqs, n_steps, out_tokens, params, m->samp_u_steps);   // (synchronises: the host vectors stay alive)
-    for (int i = 0; i < n_seqs; i++) { m->slot_len[(size_t)h_slot[(size_t)i]] += n_steps; m->slot_tick[(size_t)h_slot[(size_t)i]] = ++m->tick; }
+    decode_advance(m, h_slot, n_steps);
     return NVL_OK;
     NVL_CATCH(m)
 }
@@ -2417,6 +2570,11 @@ extern "C" int nvl_get_hidden(nvl_model* m, int layer, float* out, int64_t n_flo
     if (!m->hidden || layer < 0 || layer >= m->L) return fail(m, NVL_ERR_STATE, "nvl_get_hidden: nothing recorded");
     NVL_TRY(m)
     const int64_t per = (int64_t)m->hidden_last_M * m->H;   // [L][M][H] of the recording call
+    if (m->Hn != m->H) {                                     // padded rows: the data columns only
+        const int64_t rows = std::min<int64_t>(n_floats / m->Hn, m->hidden_last_M);
+        NVL_HIP(hipMemcpy2D(out, (size_t)m->Hn * 4, m->hidden + (int64_t)layer * per, (size_t)m->H * 4, (size_t)m->Hn * 4, (size_t)rows, hipMemcpyDeviceToHost));
+        return NVL_OK;
+    }
     if (n_floats > per) n_floats = per;
     NVL_HIP(hipMemcpy(out, m->hidden + (int64_t)layer * per, (size_t)n_floats * 4, hipMemcpyDeviceToHost));
     return NVL_OK;
@@ -2460,7 +2618,9 @@ extern "C" int nvl_get_kv(nvl_model* m, int64_t seq_id, int layer, float* k_out,
     NVL_HIP(hipSetDevice(m->device));
     const int32_t slot = it->second;
     const int T = m->slot_len[(size_t)slot];
-    read_kv(m, &slot, 1, T, layer, k_out, v_out);
+    if (m->layered) return fail(m, NVL_ERR_STATE, "nvl_get_kv: the model caches latents and states, not keys and values");
+    if (m->pool) read_kv(m, m->slot_blocks[(size_t)slot].data(), (int)m->slot_blocks[(size_t)slot].size(), T, layer, k_out, v_out);
+    else read_kv(m, &slot, 1, T, layer, k_out, v_out);
     return T;
     NVL_CATCH(m)
 }
@@ -2469,7 +2629,7 @@ extern "C" int nvl_get_mamba_state(nvl_model* m, int64_t seq_id, int layer, floa
     if (!m || !out) return NVL_ERR_INVALID;
     auto it = m->seq_slot.find(seq_id);
     if (it == m->seq_slot.end()) return fail(m, NVL_ERR_UNKNOWN_SEQ, "nvl_get_mamba_state: unknown sequence");
-    if (layer < 0 || layer >= m->L || !m->layers[(size_t)layer].mamba) return fail(m, NVL_ERR_INVALID, "nvl_get_mamba_state: not a Mamba2 layer");
+    if (layer < 0 || layer >= m->L || m->layered || !m->layers[(size_t)layer].mamba) return fail(m, NVL_ERR_INVALID, "nvl_get_mamba_state: not a Mamba2 layer");
     NVL_TRY(m)
     NVL_HIP(hipSetDevice(m->device));
     NVL_HIP(hipStreamSynchronize(m->stream));
@@ -2482,7 +2642,7 @@ extern "C" int nvl_get_mamba_state(nvl_model* m, int64_t seq_id, int layer, floa
 extern "C" int nvl_get_weight(nvl_model* m, int kind, int layer, float* out, int64_t in_features, int64_t out_features) {
     if (!m || !out) return NVL_ERR_INVALID;
     DevTensor* t = tensor_slot(m, kind, layer);
-    if (!t || is_1d(kind)) return fail(m, NVL_ERR_INVALID, "nvl_get_weight: not a 2-D weight kind");
+    if (!t || is_1d(kind) || m->layered) return fail(m, NVL_ERR_INVALID, "nvl_get_weight: not a 2-D weight kind this model keeps");
     if (!t->present()) return fail(m, NVL_ERR_STATE, "nvl_get_weight: the tensor is not on the device (never uploaded, or fused away by nvl_finalize)");
     if (t->rows != out_features || t->cols != in_features) return fail(m, NVL_ERR_INVALID, "nvl_get_weight: shape mismatch");
     NVL_TRY(m)
@@ -2538,7 +2698,8 @@ extern "C" int nvl_reset_stats(nvl_model* m) {
 static const char* const k_site_names[KS_COUNT] = {
     "other", "qkv_proj", "attention", "o_proj", "ffn_up", "ffn_down", "lm_head", "norm", "moe_router", "moe_plan", "moe_up",
     "moe_down", "moe_combine", "embed", "argmax", "rope_kv", "mamba_in_proj", "mamba_conv", "mamba_scan", "mamba_gate_norm",
-    "mamba_out_proj", "tp_allreduce"};
+    "mamba_out_proj", "tp_allreduce", "mix_in_proj", "latent_norm", "latent_uq", "latent_gather", "latent_kv", "latent_absorb_q",
+    "latent_uv", "gla_scan", "gla_gate_norm", "sandwich_norm"};
 extern "C" const char* nvl_kernel_site_name(int site) { return site >= 0 && site < KS_COUNT ? k_site_names[site] : ""; }
 extern "C" int nvl_get_kernel_stats(nvl_model* m, nvl_kernel_stat* out, int cap) {
     if (!m || (cap > 0 && !out)) return NVL_ERR_INVALID;
@@ -2698,8 +2859,8 @@ int runner_impl(nvl_model* m, int n_seqs, const int64_t* seq_ids, const int32_t*
             ids[j] = seq_ids[i]; toks[j] = token_ptrs[i][token_lens[i] - 1]; pos[j] = token_lens[i] - 1;
         }
         std::vector<float> lg(logits_out ? n * (size_t)V : 0);
-        const int rc = nvl_forward(m, (int)n, ids.data(), toks.data(), lens.data(), pos.data(), 0,
-                                   logits_out ? lg.data() : nullptr, out.data());
+        const int rc = forward_impl(m, (int)n, ids.data(), toks.data(), lens.data(), pos.data(), 0, -1, nullptr, true,
+                                    logits_out ? lg.data() : nullptr, out.data());
         if (rc) return rc;
         for (size_t j = 0; j < n; j++) {
             next_tokens[dec[base + j]] = out[j];
@@ -2719,6 +2880,7 @@ int runner_impl(nvl_model* m, int n_seqs, const int64_t* seq_ids, const int32_t*
         const int rc = seq_open_impl(m, id, true);
         if (rc) return rc;
         m->slot_len[(size_t)m->seq_slot[id]] = 0;
+        pool_release(m, m->seq_slot[id]);
         return NVL_OK;
     };
     for (int i : pre) {      // this call's own sequences are the most recently used: victims come from outside the batch first
@@ -2753,7 +2915,7 @@ int runner_impl(nvl_model* m, int n_seqs, const int64_t* seq_ids, const int32_t*
                 // hybrid models: the reference prefills the history in ONE Forward, whose Mamba2 convolution window spans
                 // the chunk seams (mamba2.go:183-254): chunks after the first take the previous chunk's tail (mamba.h)
                 m->conv_chain = done == 0 ? 1 : 2;
-                rc = nvl_forward(m, 1, &seq_ids[i], token_ptrs[i] + done, &n, &p0, 0, logits_out ? lg.data() : nullptr, &out);
+                rc = forward_impl(m, 1, &seq_ids[i], token_ptrs[i] + done, &n, &p0, 0, -1, nullptr, true, logits_out ? lg.data() : nullptr, &out);
                 m->conv_chain = 0;
                 if (rc) return rc;
                 done += n;
@@ -2769,8 +2931,8 @@ int runner_impl(nvl_model* m, int n_seqs, const int64_t* seq_ids, const int32_t*
         }
         std::vector<int32_t> out(ids.size());
         std::vector<float> lg(logits_out ? ids.size() * (size_t)V : 0);
-        const int rc = nvl_forward(m, (int)ids.size(), ids.data(), toks.data(), lens.data(), pos.data(), 0,
-                                   logits_out ? lg.data() : nullptr, out.data());
+        const int rc = forward_impl(m, (int)ids.size(), ids.data(), toks.data(), lens.data(), pos.data(), 0, -1, nullptr, true,
+                                    logits_out ? lg.data() : nullptr, out.data());
         if (rc) return rc;
         for (size_t j = 0; j < who.size(); j++) {
             next_tokens[who[j]] = out[j];

@@ -34,6 +34,15 @@ def _cfg_struct(cfg: dict) -> L.ModelConfigC:
     return c
 
 
+def _layer_structs(layers: list):
+    """config.LAYER_FIELDS dicts -> nvl_layer_config array."""
+    arr = (L.LayerConfigC * len(layers))()
+    for c, ly in zip(arr, layers):
+        for k, v in ly.items():
+            setattr(c, k, L.MIXER[v] if k == "mixer" else v)
+    return arr
+
+
 def _ptr(a):
     return None if a is None else a.ctypes.data_as(C.c_void_p)
 
@@ -45,7 +54,7 @@ class HipTransformerModel:
 
     def __init__(self, cfg: dict, tensors: dict | None, *, device: int = 0, precision: str = "bf16",
                  max_seqs: int = 8, max_batch_tokens: int | None = None, tp_rank: int = 0, tp_size: int = 1,
-                 tp_force_single: bool = False, kv_num_blocks: int = 0, kv_block_size: int = 0):
+                 tp_force_single: bool = False, kv_num_blocks: int = 0, kv_block_size: int = 0, kv_pool: bool = False):
         """tensors=None defers finalize(): upload() each tensor, then call finalize().
         tp_size > 1 makes this the tp_rank-th tensor-parallel shard: pass the FULL tensors, the library keeps
         its slice; join the shards with tp_init (RCCL, one process per GPU) or attach_local_group (tests)."""
@@ -57,10 +66,14 @@ class HipTransformerModel:
         if tp_force_single:
             opts.tp_force_single = 1
         # kv_num_blocks > 0: paged KV — the host's block manager (nanovllm/block_manager.go) owns the cache
-        opts.kv_num_blocks, opts.kv_block_size = int(kv_num_blocks), int(kv_block_size)
+        # (kv_pool: the library's own block allocator instead, under the slot calls; always so for a list of layers)
+        opts.kv_num_blocks, opts.kv_block_size, opts.kv_pool = int(kv_num_blocks), int(kv_block_size), int(bool(kv_pool))
         self.kv_block_size = (kv_block_size or 256) if kv_num_blocks else 0
         self._c = _cfg_struct(cfg)
-        L.check(self.lib.nvl_create(C.byref(self._c), C.byref(opts), C.byref(self.h)))
+        if cfg.get("layers"):
+            L.check(self.lib.nvl_create_layers(C.byref(self._c), _layer_structs(cfg["layers"]), C.byref(opts), C.byref(self.h)))
+        else:
+            L.check(self.lib.nvl_create(C.byref(self._c), C.byref(opts), C.byref(self.h)))
         self.V = cfg["vocab_size"]
         self.H = cfg["hidden"]
         if tensors is not None:
@@ -69,7 +82,7 @@ class HipTransformerModel:
             self.finalize()
 
     @classmethod
-    def from_pretrained(cls, path: str, **kw):
+    def from_pretrained(cls, path: str, *, max_seq_len: int | None = None, **kw):
         """tensor.LoadModelFromDirectory (generic_loader.go:1016-1040) without the fp32 host model: config.json (or
         model_info.json) through nvl_load_config_json, weights through nvl_load_safetensors (mmap -> device)."""
         import os
@@ -92,6 +105,14 @@ class HipTransformerModel:
                     cfg["hybrid_layers"] = ["mamba" if (v[i >> 6] >> (i & 63)) & 1 else "attention" for i in range(c.num_layers)]
                 continue
             cfg[name] = inv[name][v] if name in inv else (bool(v) if name in ("tied_embedding", "use_moe") else v)
+        n = L.check(L.lib().nvl_load_layers_json(cp.encode(), None, 0))
+        if n:
+            arr = (L.LayerConfigC * n)()
+            L.check(L.lib().nvl_load_layers_json(cp.encode(), arr, n))
+            names = {v: k for k, v in L.MIXER.items()}
+            cfg["layers"] = [{k: names[getattr(a, k)] if k == "mixer" else getattr(a, k) for k, _ in a._fields_} for a in arr]
+        if max_seq_len is not None:
+            cfg["max_seq_len"] = int(max_seq_len)
         m = cls(cfg, None, **kw)
         L.check(m.lib.nvl_load_safetensors(m.h, path.encode()), m.h)
         m.finalize()
@@ -133,7 +154,7 @@ class HipTransformerModel:
     # -- weights -----------------------------------------------------------------------------
     def upload(self, slot: str, layer: int, arr, layout: int | None = None):
         if layout is None:
-            layout = L.LAYOUT_OUT_IN if slot in L.OUT_IN_SLOTS else L.LAYOUT_IN_OUT
+            layout = L.LAYOUT_OUT_IN if slot in L.OUT_IN_SLOTS or self.cfg.get("layers") else L.LAYOUT_IN_OUT
         ptr, dtype, shape, keep = _as_pointer(arr)
         if slot in L.ONE_D:
             rows, cols = int(np.prod(shape)), 1
@@ -171,6 +192,22 @@ class HipTransformerModel:
         L.check(self.lib.nvl_forward(self.h, n, _ptr(ids), _ptr(toks), _ptr(lens), _ptr(pos),
                                      L.FWD_ALL_LOGITS if all_logits else 0, _ptr(logits), _ptr(am)), self.h)
         return logits, am
+
+    def forward_rows(self, seq_ids, token_lists, pos_offsets, rows, *, want_logits=True):
+        """nvl_forward_rows: logits [len(rows), V] (or None) and argmax of the named rows of the concatenated tokens."""
+        n = len(seq_ids)
+        ids = np.asarray(seq_ids, np.int64)
+        lens = np.asarray([len(t) for t in token_lists], np.int32)
+        toks = np.concatenate([np.asarray(t, np.int32) for t in token_lists]).astype(np.int32)
+        pos = np.asarray(pos_offsets, np.int32)
+        rw = np.asarray(rows, np.int32)
+        logits = np.empty((rw.size, self.V), np.float32) if want_logits else None
+        am = np.empty(max(rw.size, 1), np.int32)
+        L.check(self.lib.nvl_forward_rows(self.h, n, _ptr(ids), _ptr(toks), _ptr(lens), _ptr(pos), rw.size, _ptr(rw), _ptr(logits), _ptr(am)), self.h)
+        return logits, am[:rw.size]
+
+    def seq_open(self, seq_id: int):
+        L.check(self.lib.nvl_seq_open(self.h, seq_id), self.h)
 
     def forward_with_cache(self, token_ids, seq_id: int, pos_offset: int, *, all_logits=True):
         """TransformerModel.ForwardWithCache (generic_model.go:276): logits [S, V] for one sequence.

@@ -95,8 +95,8 @@ def test_native_config_loader_matches_python_mirror(pkg, tmp_path):
         dict(model_type="granitemoehybrid", hidden_size=1536),       # the "1b" template, no layer_types: all Mamba2
     ]
     enum = dict(attention_type=["mha", "mqa", "gqa"], norm_type=["layernorm", "rmsnorm"],
-                position_type=["learned", "rope", "nope"], activation_type=["gelu", "swiglu"],
-                block_style=["sequential", "parallel"])
+                position_type=["learned", "rope", "nope"], activation_type=["gelu", "swiglu", "geglu"],
+                block_style=["sequential", "parallel", "sandwich"])
     for i, raw in enumerate(cases):
         p = tmp_path / f"c{i}.json"
         p.write_text(json.dumps(raw) + "\n")
