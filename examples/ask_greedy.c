@@ -46,7 +46,17 @@ int main(int argc, char** argv) {
     opts.max_batch_tokens = n_prompt > 64 ? n_prompt : 64;
     opts.tp_size = 1;
     nvl_model* m = NULL;
-    if (nvl_create(&cfg, &opts, &m) != NVL_OK) return die(NULL, "nvl_create");
+    const int n_layers = nvl_load_layers_json(path, NULL, 0);         /* > 0: the model is described by a list of layers */
+    if (n_layers < 0) return die(NULL, "config");
+    if (n_layers > 0) {
+        nvl_layer_config* layers = (nvl_layer_config*)malloc(sizeof(nvl_layer_config) * (size_t)n_layers);
+        if (nvl_load_layers_json(path, layers, n_layers) != n_layers) return die(NULL, "config");
+        const int rc = nvl_create_layers(&cfg, layers, &opts, &m);
+        free(layers);
+        if (rc != NVL_OK) return die(NULL, "nvl_create_layers");
+    } else if (nvl_create(&cfg, &opts, &m) != NVL_OK) {
+        return die(NULL, "nvl_create");
+    }
     if (nvl_load_safetensors(m, dir) != NVL_OK) return die(m, "nvl_load_safetensors");
     if (nvl_finalize(m) != NVL_OK) return die(m, "nvl_finalize");
 

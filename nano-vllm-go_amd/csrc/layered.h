@@ -207,10 +207,11 @@ int layered_upload(nvl_model* m, int kind, int layer, const void* data, int dtyp
     return NVL_OK;
 }
 
-void* lay_alloc(nvl_model* m, int64_t bytes, bool zero = true) {
+void* lay_alloc(nvl_model* m, int64_t bytes) {      // zero-filled
+    bytes = round_up(std::max<int64_t>(bytes, 16), 16);
     void* p = dmalloc_bytes(bytes);
     m->layered_allocs.push_back(p);
-    if (zero) NVL_HIP(hipMemsetAsync(p, 0, (size_t)std::max<int64_t>(bytes, 16), m->stream));
+    NVL_HIP(hipMemsetAsync(p, 0, (size_t)bytes, m->stream));
     return p;
 }
 void* lay_matrix(nvl_model* m, int64_t N, int64_t Kd) {       // zero matrix of the weight dtype; rows padded to whole GEMM tiles

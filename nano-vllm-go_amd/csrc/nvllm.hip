@@ -1026,6 +1026,10 @@ void pool_release(nvl_model* m, int slot) {
     for (int32_t x : b) if (x >= 0) m->free_blocks.push_back(x);
     b.clear();
 }
+void pool_shrink(nvl_model* m, int slot, size_t blocks) {       // give back what a reservation that failed halfway had taken
+    auto& b = m->slot_blocks[(size_t)slot];
+    while (b.size() > blocks) { if (b.back() >= 0) m->free_blocks.push_back(b.back()); b.pop_back(); }
+}
 // Blocks for positions 0 .. end - 1 of a slot's sequence (pool mode).  evict: when the pool is empty, close the
 // least-recently-forwarded sequence that is not pinned and take its blocks.
 bool pool_reserve(nvl_model* m, int slot, int64_t end, bool evict) {
@@ -2041,7 +2045,10 @@ int forward_impl(nvl_model* m, int n_seqs, const int64_t* seq_ids, const int32_t
         std::vector<int> pinned;
         for (int slot : h_slot) if (!m->slot_pin[(size_t)slot]) { m->slot_pin[(size_t)slot] = 1; pinned.push_back(slot); }
         bool ok = true;
+        std::vector<size_t> before((size_t)n_seqs);
+        for (int i = 0; i < n_seqs; i++) before[(size_t)i] = m->slot_blocks[(size_t)h_slot[(size_t)i]].size();
         for (int i = 0; i < n_seqs && ok; i++) ok = pool_reserve(m, h_slot[(size_t)i], (int64_t)pos_offsets[i] + seq_lens[i], evict);
+        if (!ok) for (int i = 0; i < n_seqs; i++) pool_shrink(m, h_slot[(size_t)i], before[(size_t)i]);
         for (int slot : pinned) m->slot_pin[(size_t)slot] = 0;
         if (!ok) return fail(m, NVL_ERR_NO_SLOT, "nvl_forward: the cache pool has no free block");
         for (int i = 0; i < n_seqs; i++) bind_slot(m, hm, i, h_slot[(size_t)i]);
@@ -2272,8 +2279,13 @@ extern "C" int nvl_runner_run_paged(nvl_model* m, int n_seqs, const int32_t* con
 namespace {
 // blocks, table rows and (layered) metadata of n_steps one-token passes
 bool decode_reserve(nvl_model* m, const Meta& hm, const std::vector<int>& slots, int n_steps) {
+    std::vector<size_t> before;
+    for (int slot : slots) before.push_back(m->slot_blocks[(size_t)slot].size());
     for (size_t i = 0; i < slots.size(); i++)
-        if (!pool_reserve(m, slots[i], (int64_t)m->slot_len[(size_t)slots[i]] + n_steps, false)) return false;
+        if (!pool_reserve(m, slots[i], (int64_t)m->slot_len[(size_t)slots[i]] + n_steps, false)) {
+            for (size_t j = 0; j <= i; j++) pool_shrink(m, slots[j], before[j]);
+            return false;
+        }
     for (size_t i = 0; i < slots.size(); i++) bind_slot(m, hm, (int)i, slots[i]);
     if (m->layered) layered_meta(m, hm, (int)slots.size(), n_steps);
     return true;
