@@ -38,7 +38,8 @@ def parse():
     ap.add_argument("--gpus", type=int, default=1)
     ap.add_argument("--steps", type=int, default=3)
     ap.add_argument("--warmup", type=int, default=1)
-    ap.add_argument("--model", default="llama-3.2-1b")
+    ap.add_argument("--model", default="llama-3.2-1b", help="a synth.FULL_CONFIGS key; potuzen-2k / potuzen-4k are the Potuzen design at a real "
+                    "model's layer sizes, hybrid-2k / hybrid-4k the attention + Mamba-2 family at the same sizes")
     ap.add_argument("--batch", type=int, default=32, help="sequences per GPU")
     ap.add_argument("--prompt", type=int, default=512, help="prompt tokens per sequence")
     ap.add_argument("--gen", type=int, default=128, help="decode steps per sequence")
@@ -78,6 +79,15 @@ def gen_weights_on_device(pkg, cfg, model, torch, device, keep_host: bool):
     ln = cfg["norm_type"] == "layernorm"
     host = {}
     g = torch.Generator(device=device)
+    if cfg.get("layers"):                    # a model described by a list of layers: matrices N(0, 1 / inputs), decays of a trained model's range
+        for n, (slot, layer, shape, kind) in enumerate(pkg.synth.layered_shapes(cfg)):
+            g.manual_seed(42 + n)
+            t = torch.randn(*shape, device=device, generator=g)
+            u = torch.rand(*shape, device=device, generator=g)
+            t = {"matrix": lambda: t * shape[-1] ** -0.5, "norm": lambda: 1 + 0.02 * t, "conv": lambda: 0.3 * t, "bias": lambda: 0.5 * t,
+                 "dt_bias": lambda: 3.5 * u - 3, "a_log": lambda: torch.log(1 + 7 * u)}[kind]()
+            model.upload(slot, layer, t.to(torch.bfloat16))
+        return host
 
     def put(slot, layer, out_dim, in_dim=None, std=0.02, mean=0.0, seed=0):
         g.manual_seed(42 + layer * 1000 + seed)
@@ -115,6 +125,20 @@ def gen_weights_on_device(pkg, cfg, model, torch, device, keep_host: bool):
             put("ffn_norm_w", li, H, mean=1.0, seed=12)
             if ln:
                 put("ffn_norm_b", li, H, seed=13)
+        if (cfg.get("hybrid_layers") or [""] * Lyr)[li].startswith("mamba"):
+            EH, nh = cfg["mamba_expand"] * H, cfg["mamba_num_heads"]
+            conv = EH + 2 * cfg["mamba_n_groups"] * cfg["mamba_state_size"]
+            put("mamba_in_proj", li, EH + conv + nh, H, seed=60)
+            put("mamba_conv_w", li, conv * cfg["mamba_conv_kernel"], std=0.3, seed=61)
+            put("mamba_conv_b", li, conv, seed=62)
+            put("mamba_a_log", li, nh, mean=1.0, std=0.5, seed=63)
+            put("mamba_d", li, nh, mean=1.0, seed=64)
+            put("mamba_dt_bias", li, nh, mean=-1.5, std=0.8, seed=65)
+            put("mamba_norm", li, EH, mean=1.0, seed=66)
+            put("mamba_out_proj", li, H, EH, seed=67)
+            put("w1", li, 2 * F, H, seed=50)
+            put("w2", li, H, F, seed=51)
+            continue
         put("wq", li, nH * hd, H, seed=20)
         if at == "mqa":
             put("wkv", li, 2 * hd, H, seed=21)
@@ -142,6 +166,16 @@ def flops_per_token(cfg):
     nH, hd, F = cfg["num_heads"], cfg["head_dim"], cfg["ffn_dim"]
     at = cfg["attention_type"]
     nKV = nH if at == "mha" else (1 if at == "mqa" else cfg["num_kv_heads"])
+    if cfg.get("layers"):
+        from importlib import import_module
+        shapes = import_module("nano-vllm-go_amd").synth.layered_shapes(cfg)
+        return 2.0 * sum(s[0] * s[1] for slot, _, s, _ in shapes if len(s) == 2 and slot not in ("tok_emb", "lm_head")), 2.0 * H * V
+    if cfg.get("hybrid_layers"):
+        EH = cfg["mamba_expand"] * H
+        n_m = sum(t.startswith("mamba") for t in cfg["hybrid_layers"])
+        mam = H * (2 * EH + 2 * cfg["mamba_n_groups"] * cfg["mamba_state_size"] + cfg["mamba_num_heads"]) + EH * H
+        att = 2 * H * nH * hd + 2 * H * nKV * hd
+        return 2.0 * (n_m * mam + (L - n_m) * att + L * 3 * H * F), 2.0 * H * V
     if cfg.get("use_moe"):
         ffn = cfg["num_experts_per_tok"] * 3 * H * F + H * cfg["num_experts"]
     else:
@@ -195,7 +229,7 @@ def main():
     model = pkg.HipTransformerModel(cfg, None, device=local_rank, precision=args.precision, max_seqs=B,
                                     max_batch_tokens=max_batch_tokens, tp_rank=rank if tp else 0,
                                     tp_size=world if tp else 1, tp_force_single=tp and world == 1)
-    want_cpu = (rank == 0 and world == 1 and not args.no_cpu_baseline)
+    want_cpu = (rank == 0 and world == 1 and not args.no_cpu_baseline and not cfg.get("layers") and not cfg.get("hybrid_layers"))
     t0 = time.time()
     host_w = gen_weights_on_device(pkg, cfg, model, torch, device, keep_host=want_cpu)
     model.finalize()
@@ -304,6 +338,13 @@ def main():
     at = cfg["attention_type"]
     nKV = cfg["num_heads"] if at == "mha" else (1 if at == "mqa" else cfg["num_kv_heads"])
     kv_bytes = 2 * cfg["num_layers"] * nKV * cfg["head_dim"] * (S + G / 2) * 2 * B
+    if cfg.get("hybrid_layers"):      # attention layers' K/V once, the Mamba-2 layers' fp32 states read and written
+        n_m = sum(t.startswith("mamba") for t in cfg["hybrid_layers"])
+        kv_bytes *= 1 - n_m / cfg["num_layers"]
+        kv_bytes += n_m * B * 8.0 * cfg["mamba_expand"] * cfg["hidden"] * cfg["mamba_state_size"]
+    if cfg.get("layers"):             # cached latents once, fp32 states read and written
+        kv_bytes = sum(B * (2.0 * c["kv_rank"] * min(c["window"] or 1 << 30, S + G / 2) if c["mixer"] == "latent_attention" else
+                            8.0 * c["heads"] * c["vdim"] * (c["state"] or c["dim"])) for c in cfg["layers"])
     dec_gbs = (wbytes + kv_bytes) * G * args.steps / dec_s / 1e9
 
     # HBM-side traffic of the dominant kernel class comes from separate rocprofv3 --pmc passes (FETCH_SIZE x2 on

@@ -19,6 +19,7 @@
 
 namespace nvl {
 
+constexpr int LAT_SPLITS = 16;          // most workgroups the keys of a token are split over (absorbed form)
 __device__ __forceinline__ float lat_sigmoid(float x) { return 1.0f / (1.0f + __expf(-x)); }
 
 struct LatentArgs {
@@ -57,19 +58,16 @@ __host__ __device__ __forceinline__ int latent_key0(int pos0, int window) {
 // ---- norms of the two latents; c goes to its cache row.  grid (tokens), 256 threads ----
 template <typename ActT>
 __global__ __launch_bounds__(256) void latent_norm_kernel(LatentArgs p) {
-    __shared__ float red[4];
+    __shared__ float red[8];
     const int t = blockIdx.x;
     const float* pr = p.proj + (int64_t)t * p.proj_ld;
-    auto rms_of = [&](const float* v, int n) {
-        float ss = 0.f;
-        for (int i = threadIdx.x; i < n; i += 256) ss = fmaf(v[i], v[i], ss);
-        ss = wave_sum(ss);
-        __syncthreads();
-        if ((threadIdx.x & 63) == 0) red[threadIdx.x >> 6] = ss;
-        __syncthreads();
-        return sqrtf((red[0] + red[1] + red[2] + red[3]) / (float)n + p.eps);
-    };
-    const float rq = rms_of(pr, p.qrank), rc = rms_of(pr + p.qrp, p.kvrank);
+    float sq = 0.f, sc = 0.f;
+    for (int i = threadIdx.x; i < p.qrank; i += 256) sq = fmaf(pr[i], pr[i], sq);
+    for (int i = threadIdx.x; i < p.kvrank; i += 256) sc = fmaf(pr[p.qrp + i], pr[p.qrp + i], sc);
+    sq = wave_sum(sq); sc = wave_sum(sc);
+    if ((threadIdx.x & 63) == 0) { red[threadIdx.x >> 6] = sq; red[4 + (threadIdx.x >> 6)] = sc; }
+    __syncthreads();
+    const float rq = sqrtf((red[0] + red[1] + red[2] + red[3]) / (float)p.qrank + p.eps), rc = sqrtf((red[4] + red[5] + red[6] + red[7]) / (float)p.kvrank + p.eps);
     for (int i = threadIdx.x; i < p.qrp; i += 256)
         ActIO<ActT>::st((ActT*)p.cq + act_index<ActT>(t, i, p.qrp), (pr[i] / rq) * p.cq_norm[i]);
     int blk, row;
@@ -95,150 +93,254 @@ __global__ __launch_bounds__(256) void latent_gather_kernel(LatentArgs p) {
 }
 
 // ------------------------------------------------------------------------------------------
-// expanded form, bf16.  grid (ceil(longest portion / 128), H, sequences), 4 waves of 32 query rows.  S^T = K Q^T and
-// O^T += V^T P^T as in attn.h, but K and V^T come fragment-major from memory, so no operand passes through LDS: the K rows of a
-// 32-key unit are taken in the order that makes the score accumulators (keys 8 fg + r, 8 fg + 4 + r) the B operand against
-// V^T's natural key order.
+// expanded form, bf16.  S^T = K Q^T and O^T += V^T P^T as in attn.h; 32 query rows of one head per wave.  K and V^T come
+// fragment-major from memory; the K rows of a 32-key unit are taken in the order that makes the score accumulators
+// (keys 8 fg + r, 8 fg + 4 + r) the B operand against V^T's natural key order.
+//   latent_prefill_kernel      : 8 waves (256 query rows) share 64-key tiles of K and V^T through a 3-slot LDS ring filled by LDS-DMA two
+//                                tiles ahead, one barrier per tile; a tile is a set of 1-KiB operand blocks, so the image is
+//                                lane-linear and every fragment read conflict-free (the K row order is chosen by the DMA's source)
+//   latent_prefill_wide_kernel : 4 waves, operands straight from memory (heads of 256 x 256: three slots would not fit LDS)
+// A negative scale is moved onto the queries, so that the row maximum can be taken before scaling; zero: latent_plain_kernel.
 // ------------------------------------------------------------------------------------------
+struct LatentRows {            // the query rows of one wave
+    int tok0, pos0, n, k0, row0, first, last;
+    __device__ __forceinline__ LatentRows(const LatentArgs& p, int seq, int row0_) {
+        n = p.seq_len[seq]; tok0 = p.seq_tok_start[seq]; pos0 = p.seq_pos[seq]; k0 = latent_key0(pos0, p.window); row0 = row0_;
+        first = pos0 + row0; last = pos0 + min(row0 + 31, n - 1);
+    }
+    __device__ __forceinline__ int row(int i, int fq, bool& ok) const { const int r = row0 + 16 * i + fq; ok = r < n; return ok ? r : n - 1; }
+    __device__ __forceinline__ int key_lo(const LatentArgs& p) const { const int lo = p.window > 0 ? first - p.window + 1 : 0; return lo > k0 ? lo - k0 : 0; }
+};
+template <int KS>
+__device__ __forceinline__ void latent_load_q(const LatentArgs& p, int64_t tok, int h, int fg, bf16x8 (&qf)[KS]) {
+    const float* qp = p.q + tok * p.q_ld + h * p.dp;
+    const float sg = p.scale < 0.f ? -1.f : 1.f;
+#pragma unroll
+    for (int ks = 0; ks < KS; ks++) {
+        const f32x4 a = *(const f32x4*)(qp + ks * 32 + fg * 8), b = *(const f32x4*)(qp + ks * 32 + fg * 8 + 4);
+#pragma unroll
+        for (int e = 0; e < 4; e++) { qf[ks][e] = (bf16_t)(a[e] * sg); qf[ks][4 + e] = (bf16_t)(b[e] * sg); }
+    }
+}
+// this lane's K row inside a 32-key unit for score tile t
+__device__ __forceinline__ int latent_k_row(int t, int fq) { return 8 * (fq >> 2) + (fq & 3) + 4 * (t & 1); }
+// scores of one 64-key tile (tile-relative key 32 (t / 2) + 8 fg + 4 (t & 1) + r) -> weights, running maximum and rescale
+template <int DT>
+__device__ __forceinline__ void latent_softmax(f32x4 (&s)[4], bool whole, int back, int window, int fg, float sl2, float& m_run, f32x4& lacc, f32x4 (&o)[DT]) {
+    if (!whole) {
+        const int from = window > 0 ? back - window + 1 : 0;
+#pragma unroll
+        for (int t = 0; t < 4; t++)
+#pragma unroll
+            for (int r = 0; r < 4; r++) {
+                const int k = 32 * (t >> 1) + 8 * fg + 4 * (t & 1) + r;
+                if (k > back || k < from) s[t][r] = -INFINITY;
+            }
+    }
+    const float m_new = vmax2(m_run, rows_max(vmax16(s[0], s[1], s[2], s[3])) * sl2);
+    if (__any(m_new != m_run)) {
+        const float alpha = __builtin_amdgcn_exp2f(m_run - m_new);
+        lacc *= alpha;
+#pragma unroll
+        for (int d = 0; d < DT; d++) o[d] *= alpha;
+        m_run = m_new;
+    }
+#pragma unroll
+    for (int t = 0; t < 4; t++)
+#pragma unroll
+        for (int r = 0; r < 4; r++) s[t][r] = __builtin_amdgcn_exp2f(fmaf(s[t][r], sl2, -m_run));
+}
+__device__ __forceinline__ bf16x8 latent_pack_p(const f32x4& a, const f32x4& b) {
+    bf16x8 p;
+#pragma unroll
+    for (int r = 0; r < 4; r++) { p[r] = (bf16_t)a[r]; p[4 + r] = (bf16_t)b[r]; }
+    return p;
+}
+template <int DT>
+__device__ __forceinline__ void latent_store_o(const LatentArgs& p, int64_t tok, int h, int fg, float inv, const f32x4 (&o)[DT]) {
+    const float* gt = p.proj + tok * p.proj_ld + p.qrp + p.rp + h * p.vp;
+#pragma unroll
+    for (int d = 0; d < DT; d++) {
+        const f32x4 g = *(const f32x4*)(gt + 16 * d + 4 * fg);
+        f32x4 v = o[d] * inv;
+#pragma unroll
+        for (int r = 0; r < 4; r++) v[r] *= lat_sigmoid(g[r]);
+        act_store4<bf16_t>((bf16_t*)p.out, tok, h * p.vp + 16 * d + 4 * fg, p.out_ld, v);
+    }
+}
+
+template <int KS, int DT> constexpr int latent_prefill_pieces() { return 4 * KS + 2 * DT; }       // 1-KiB blocks of a tile
+template <int KS, int DT> constexpr int latent_prefill_lds_bytes() { return 3 * ((latent_prefill_pieces<KS, DT>() + 7) / 8 * 8) * 1024; }
+template <int N> __device__ __forceinline__ void wait_vm() { asm volatile("s_waitcnt vmcnt(%0)" ::"n"(N) : "memory"); }
+
 template <int KS, int DT>
-__global__ __launch_bounds__(256) void latent_prefill_kernel(LatentArgs p) {
-    constexpr int TQ = 2;
-    const int seq = blockIdx.z, h = blockIdx.y, qt = gridDim.x - 1 - blockIdx.x;
-    const int n = p.seq_len[seq];
-    if (qt * 128 >= n || p.kbase[seq] < 0) return;
+__global__ __launch_bounds__(512, (KS <= 2 && DT <= 4) ? 4 : 2) void latent_prefill_kernel(LatentArgs p) {
+    constexpr int TQ = 2, PIECES = latent_prefill_pieces<KS, DT>(), PW = (PIECES + 7) / 8, TILE = PW * 8 * 1024, NBUF = 3;
+    extern __shared__ __attribute__((aligned(16))) char lat_smc[];
+    // head fastest, query tile slowest and last first: the longest workgroups are dispatched first
+    const int h = blockIdx.x, seq = blockIdx.y, qt = gridDim.z - 1 - blockIdx.z;
+    if (qt * 256 >= p.seq_len[seq] || p.kbase[seq] < 0) return;
     const int lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
     const int fq = lane & 15, fg = lane >> 4;
-    const int tok0 = p.seq_tok_start[seq], pos0 = p.seq_pos[seq];
-    const int k0 = latent_key0(pos0, p.window), kb = p.kbase[seq];
-    const int row0 = qt * 128 + wave * 32;
-    if (row0 >= n) return;                                   // (no barrier in this kernel)
+    const LatentRows w(p, seq, qt * 256 + wave * 32);
+    const bool w_live = w.row0 < w.n;
     bf16x8 qf[TQ][KS];
-    int qpos[TQ], qtok[TQ];
-    bool qok[TQ];
+    int qpos[TQ];
 #pragma unroll
     for (int i = 0; i < TQ; i++) {
-        int r = row0 + 16 * i + fq;
-        qok[i] = r < n;
-        if (!qok[i]) r = n - 1;
-        qtok[i] = tok0 + r; qpos[i] = pos0 + r;
-        const float* qp = p.q + (int64_t)qtok[i] * p.q_ld + h * p.dp;
+        bool ok;
+        const int r = w.row(i, fq, ok);
+        qpos[i] = w.pos0 + r;
+        latent_load_q<KS>(p, w.tok0 + r, h, fg, qf[i]);
+    }
 #pragma unroll
-        for (int ks = 0; ks < KS; ks++) {
-            const f32x4 a = *(const f32x4*)(qp + ks * 32 + fg * 8), b = *(const f32x4*)(qp + ks * 32 + fg * 8 + 4);
+    for (int i = 0; i < TQ; i++)
 #pragma unroll
-            for (int e = 0; e < 4; e++) { qf[i][ks][e] = (bf16_t)a[e]; qf[i][ks][4 + e] = (bf16_t)b[e]; }
+        for (int ks = 0; ks < KS; ks++) asm volatile("" : "+v"(qf[i][ks]));      // complete before the first DMA is issued (attn.h)
+    // workspace-relative keys: the workgroup's tiles, and the part of them this wave's rows can see
+    const LatentRows wg(p, seq, qt * 256);
+    const int kb = p.kbase[seq];
+    const int wg_last = wg.pos0 + min(qt * 256 + 255, wg.n - 1) - wg.k0;
+    const int t0 = wg.key_lo(p) >> 6, n_kt = (wg_last >> 6) + 1;
+    const int wt0 = w_live ? w.key_lo(p) >> 6 : n_kt, wt1 = w_live ? ((w.last - w.k0) >> 6) + 1 : 0;
+    const int full_lo = (p.window > 0 ? w.last - p.window + 1 : 0) - w.k0, full_hi = w.first - w.k0;
+    // LDS-DMA: wave w moves pieces w * PW .. of [K: tile t, k-step | V^T: d, 32-key unit]; surplus pieces repeat the last one
+    const int64_t k_ld = (int64_t)(p.H * p.dp >> 5), v_ld = p.rows_pad >> 5;
+    const bf16_t* src[PW];
+    int64_t step[PW];
+#pragma unroll
+    for (int i = 0; i < PW; i++) {
+        int pc = wave * PW + i;
+        if (pc >= PIECES) pc = PIECES - 1;
+        if (pc < 4 * KS) {
+            const int t = pc / KS, ks = pc - t * KS, key = kb + 32 * (t >> 1) + latent_k_row(t, fq);
+            src[i] = (const bf16_t*)p.kx + (((int64_t)(key >> 4) * k_ld + h * KS + ks) * 64 + (key & 15) + 16 * fg) * 8;
+            step[i] = 4 * k_ld * 512;
+        } else {
+            const int v = pc - 4 * KS, d = v >> 1, u = v & 1;
+            src[i] = (const bf16_t*)p.vx + (((int64_t)(h * DT + d) * v_ld + (kb >> 5) + u) * 64 + lane) * 8;
+            step[i] = 2 * 512;
         }
     }
-    const int first = pos0 + row0, last = pos0 + min(row0 + 31, n - 1);       // positions of this wave's rows
-    int lo = p.window > 0 ? first - p.window + 1 : 0;
-    if (lo < k0) lo = k0;
-    const int j0 = (lo - k0) & ~63, j1 = last - k0;                            // workspace-relative keys
-    const int full_lo = p.window > 0 ? last - p.window + 1 : 0, full_hi = first;   // a tile inside [full_lo, full_hi] needs no mask
-    const int kt_ld = p.H * p.dp >> 5;                                          // 1-KiB blocks per 16 key rows of K
-    const bf16_t* kx = (const bf16_t*)p.kx;
-    const bf16_t* vx = (const bf16_t*)p.vx;
-    const int64_t vt_ld = p.rows_pad >> 5;
-    f32x4 o[TQ][DT];
-    float m_run[TQ], l_run[TQ];
+    const uint32_t smem_lds = (uint32_t)(size_t)(__attribute__((address_space(3))) char*)lat_smc;
+    auto issue = [&](int kt, int buf) {
+        const uint32_t dst = smem_lds + buf * TILE + wave * (PW * 1024);
+#pragma unroll
+        for (int i = 0; i < PW; i++) {
+            const uint64_t a = (uint64_t)(src[i] + (int64_t)kt * step[i]);
+            asm volatile("s_mov_b32 m0, %0\n\ts_nop 4\n\tglobal_load_lds_dwordx4 %1, off" ::"s"(dst + i * 1024), "v"(a) : "memory");
+        }
+    };
+    f32x4 o[TQ][DT], lacc[TQ];
+    float m_run[TQ];
 #pragma unroll
     for (int i = 0; i < TQ; i++) {
-        m_run[i] = -1e30f; l_run[i] = 0.f;
+        m_run[i] = -1e30f; lacc[i] = f32x4{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
         for (int d = 0; d < DT; d++) o[i][d] = f32x4{0.f, 0.f, 0.f, 0.f};
     }
-    const float sl2 = p.scale * 1.4426950408889634f;
-    for (int j = j0; j <= j1; j += 64) {
-        const int nu = j + 32 <= j1 ? 2 : 1;                                   // 32-key units of this step that hold keys
+    bf16x8 ones;
+#pragma unroll
+    for (int e = 0; e < 8; e++) ones[e] = (bf16_t)1.0f;
+    const float sl2 = fabsf(p.scale) * 1.4426950408889634f;
+    issue(t0, 0);
+    if (t0 + 1 < n_kt) issue(t0 + 1, 1);
+    int buf = 0;
+    for (int kt = t0; kt < n_kt; kt++) {
+        if (kt + 1 < n_kt) wait_vm<PW>(); else wait_vm<0>();      // my pieces of tile kt have landed
+        __builtin_amdgcn_s_barrier();
+        if (kt + 2 < n_kt) { int nb = buf + 2; if (nb >= NBUF) nb -= NBUF; issue(kt + 2, nb); }
+        const char* kimg = lat_smc + buf * TILE + lane * 16;
+        const char* vimg = kimg + 4 * KS * 1024;
+        buf = buf + 1 == NBUF ? 0 : buf + 1;
+        if (kt < wt0 || kt >= wt1) continue;                      // (wave-uniform)
         f32x4 s[TQ][4];
 #pragma unroll
         for (int i = 0; i < TQ; i++)
 #pragma unroll
             for (int t = 0; t < 4; t++) s[i][t] = f32x4{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
-        for (int t = 0; t < 4; t++) {
-            if ((t >> 1) >= nu) continue;
-            const int key = kb + j + 32 * (t >> 1) + 8 * (fq >> 2) + (fq & 3) + 4 * (t & 1);     // this lane's K row
-            const bf16_t* kr = kx + (((int64_t)(key >> 4) * kt_ld + h * KS) * 64 + (key & 15) + 16 * fg) * 8;
+        for (int t = 0; t < 4; t++)
 #pragma unroll
             for (int ks = 0; ks < KS; ks++) {
-                const bf16x8 kf = *(const bf16x8*)(kr + ks * 512);
+                const bf16x8 kf = *(const bf16x8*)(kimg + (t * KS + ks) * 1024);
 #pragma unroll
                 for (int i = 0; i < TQ; i++) s[i][t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf, qf[i][ks], s[i][t], 0, 0, 0);
             }
-        }
-        // lane: S^T[key = 32 (t / 2) + 8 fg + 4 (t & 1) + r][query fq]
-        const bool whole = k0 + j >= full_lo && k0 + j + 63 <= full_hi;
+        const bool whole = kt * 64 >= full_lo && kt * 64 + 63 <= full_hi;
 #pragma unroll
-        for (int i = 0; i < TQ; i++) {
-#pragma unroll
-            for (int t = 0; t < 4; t++)
-#pragma unroll
-                for (int r = 0; r < 4; r++) s[i][t][r] *= sl2;
-            if (!whole) {
-                const int back = qpos[i] - (k0 + j);                            // tile-relative: keys back - window + 1 .. back
-                const int from = p.window > 0 ? back - p.window + 1 : 0;
-#pragma unroll
-                for (int t = 0; t < 4; t++)
-#pragma unroll
-                    for (int r = 0; r < 4; r++) {
-                        const int k = 32 * (t >> 1) + 8 * fg + 4 * (t & 1) + r;
-                        if (k > back || k < from || (t >> 1) >= nu) s[i][t][r] = -INFINITY;
-                    }
-            }
-            float mx = s[i][0][0];
-#pragma unroll
-            for (int t = 0; t < 4; t++)
-#pragma unroll
-                for (int r = 0; r < 4; r++) mx = fmaxf(mx, s[i][t][r]);
-            mx = rows_max(mx);
-            const float m_new = fmaxf(m_run[i], mx);
-            const float alpha = __builtin_amdgcn_exp2f(m_run[i] - m_new);
-            m_run[i] = m_new;
-            float ls = 0.f;
-#pragma unroll
-            for (int t = 0; t < 4; t++)
-#pragma unroll
-                for (int r = 0; r < 4; r++) { s[i][t][r] = __builtin_amdgcn_exp2f(s[i][t][r] - m_new); ls += s[i][t][r]; }
-            l_run[i] = l_run[i] * alpha + ls;
-            if (__any(alpha != 1.0f)) {
-#pragma unroll
-                for (int d = 0; d < DT; d++) o[i][d] *= alpha;
-            }
-        }
+        for (int i = 0; i < TQ; i++) latent_softmax<DT>(s[i], whole, qpos[i] - w.k0 - kt * 64, p.window, fg, sl2, m_run[i], lacc[i], o[i]);
 #pragma unroll
         for (int u = 0; u < 2; u++) {
-            if (u >= nu) continue;
             bf16x8 pf[TQ];
 #pragma unroll
-            for (int i = 0; i < TQ; i++)
-#pragma unroll
-                for (int r = 0; r < 4; r++) { pf[i][r] = (bf16_t)s[i][2 * u][r]; pf[i][4 + r] = (bf16_t)s[i][2 * u + 1][r]; }
-            const bf16_t* vr = vx + (((int64_t)(h * DT) * vt_ld + ((kb + j) >> 5) + u) * 64 + lane) * 8;
+            for (int i = 0; i < TQ; i++) {
+                pf[i] = latent_pack_p(s[i][2 * u], s[i][2 * u + 1]);
+                lacc[i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(ones, pf[i], lacc[i], 0, 0, 0);      // denominators out of the same rounded weights
+            }
 #pragma unroll
             for (int d = 0; d < DT; d++) {
-                const bf16x8 vf = *(const bf16x8*)(vr + (int64_t)d * vt_ld * 512);
+                const bf16x8 vf = *(const bf16x8*)(vimg + (2 * d + u) * 1024);
 #pragma unroll
                 for (int i = 0; i < TQ; i++) o[i][d] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf, pf[i], o[i][d], 0, 0, 0);
             }
         }
     }
+    if (!w_live) return;
 #pragma unroll
     for (int i = 0; i < TQ; i++) {
-        float l = l_run[i];
-        l += __shfl_xor(l, 16, 64);
-        l += __shfl_xor(l, 32, 64);
-        if (!qok[i]) continue;
-        const float inv = 1.0f / l;
-        const float* gt = p.proj + (int64_t)qtok[i] * p.proj_ld + p.qrp + p.rp + h * p.vp;
+        bool ok;
+        const int r = w.row(i, fq, ok);
+        if (ok) latent_store_o<DT>(p, w.tok0 + r, h, fg, 1.0f / lacc[i][0], o[i]);
+    }
+}
+
+template <int KS, int DT>
+__global__ __launch_bounds__(256) void latent_prefill_wide_kernel(LatentArgs p) {
+    constexpr int TQ = 1;
+    const int h = blockIdx.x, seq = blockIdx.y, qt = gridDim.z - 1 - blockIdx.z;
+    const int lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
+    const int fq = lane & 15, fg = lane >> 4;
+    const int row0 = qt * 64 + wave * 16;
+    if (row0 >= p.seq_len[seq] || p.kbase[seq] < 0) return;      // (no barrier in this kernel)
+    const LatentRows w(p, seq, row0);
+    const int last = w.pos0 + min(row0 + 15, w.n - 1);
+    bool ok;
+    const int r0 = w.row(0, fq, ok), qpos = w.pos0 + r0;
+    bf16x8 qf[KS];
+    latent_load_q<KS>(p, w.tok0 + r0, h, fg, qf);
+    const int kb = p.kbase[seq], j1 = last - w.k0;
+    const int full_lo = (p.window > 0 ? last - p.window + 1 : 0) - w.k0, full_hi = w.first - w.k0;
+    const int64_t k_ld = (int64_t)(p.H * p.dp >> 5), v_ld = p.rows_pad >> 5;
+    f32x4 o[DT], lacc = f32x4{0.f, 0.f, 0.f, 0.f};
+    float m_run = -1e30f;
 #pragma unroll
-        for (int d = 0; d < DT; d++) {
-            const f32x4 g = *(const f32x4*)(gt + 16 * d + 4 * fg);
-            f32x4 v = o[i][d] * inv;
+    for (int d = 0; d < DT; d++) o[d] = f32x4{0.f, 0.f, 0.f, 0.f};
+    bf16x8 ones;
 #pragma unroll
-            for (int r = 0; r < 4; r++) v[r] *= lat_sigmoid(g[r]);
-            act_store4<bf16_t>((bf16_t*)p.out, qtok[i], h * p.vp + 16 * d + 4 * fg, p.out_ld, v);
+    for (int e = 0; e < 8; e++) ones[e] = (bf16_t)1.0f;
+    const float sl2 = fabsf(p.scale) * 1.4426950408889634f;
+    for (int j = w.key_lo(p) & ~63; j <= j1; j += 64) {
+        f32x4 s[4];
+#pragma unroll
+        for (int t = 0; t < 4; t++) {
+            s[t] = f32x4{0.f, 0.f, 0.f, 0.f};
+            const int key = kb + j + 32 * (t >> 1) + latent_k_row(t, fq);
+            const bf16_t* kr = (const bf16_t*)p.kx + (((int64_t)(key >> 4) * k_ld + h * KS) * 64 + (key & 15) + 16 * fg) * 8;
+#pragma unroll
+            for (int ks = 0; ks < KS; ks++) s[t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(*(const bf16x8*)(kr + ks * 512), qf[ks], s[t], 0, 0, 0);
+        }
+        latent_softmax<DT>(s, j >= full_lo && j + 63 <= full_hi, qpos - w.k0 - j, p.window, fg, sl2, m_run, lacc, o);
+#pragma unroll
+        for (int u = 0; u < 2; u++) {
+            const bf16x8 pf = latent_pack_p(s[2 * u], s[2 * u + 1]);
+            lacc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(ones, pf, lacc, 0, 0, 0);
+            const bf16_t* vr = (const bf16_t*)p.vx + (((int64_t)(h * DT) * v_ld + ((kb + j) >> 5) + u) * 64 + lane) * 8;
+#pragma unroll
+            for (int d = 0; d < DT; d++) o[d] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(*(const bf16x8*)(vr + (int64_t)d * v_ld * 512), pf, o[d], 0, 0, 0);
         }
     }
+    if (ok) latent_store_o<DT>(p, w.tok0 + r0, h, fg, 1.0f / lacc[0], o);
 }
 
 // ---- expanded form, any size: one 256-thread workgroup per (token, head), online softmax over 256 keys at a time, plain fp32
@@ -434,45 +536,54 @@ __global__ __launch_bounds__(256) void latent_decode_kernel(LatentArgs p) {
     for (int i = 0; i < NR; i++) *(f32x4*)(p.part_o + at * p.rp + (wave * NR + i) * 16 + 4 * fg) = o[i];
 }
 
-// combines the key splits, projects by W_uv and gates: grid (H, vp / 16, ceil(n_abs / 16)), 4 waves share K = rp
+// combines the key splits, projects by W_uv and gates: grid (H, ceil(vp / 64), ceil(n_abs / 16)), 4 waves, one 16-column tile of V each.
+// The combined latents of the 16 tokens are made once per workgroup (fragment-major bf16 in LDS) while the weight fragments are in flight.
 static __global__ __launch_bounds__(256) void latent_uv_kernel(LatentArgs p) {
-    __shared__ f32x4 red[4][64];
-    const int h = blockIdx.x, vt = blockIdx.y, mt = blockIdx.z, lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
-    const int fr = lane & 15, fg = lane >> 4, nks = p.rp >> 5;
-    const int i = mt * 16 + fr;
-    const bool ok = i < p.n_abs;
-    float M = -1e30f, L = 0.f;
-    if (ok) {
-        for (int z = 0; z < p.n_split; z++) M = fmaxf(M, p.part_ml[2 * (((int64_t)z * p.n_abs + i) * p.H + h)]);
-        for (int z = 0; z < p.n_split; z++) {
-            const float* ml = p.part_ml + 2 * (((int64_t)z * p.n_abs + i) * p.H + h);
-            L += ml[1] * __builtin_amdgcn_exp2f(ml[0] - M);
-        }
-    }
-    const float invL = ok ? 1.0f / L : 0.f;
+    extern __shared__ __attribute__((aligned(16))) char lat_smc[];       // [rp / 32][64 lanes][16 B]
+    __shared__ float sw[16][LAT_SPLITS];                                  // weight of a split's partial, 1 / L folded in
+    const int h = blockIdx.x, vt = blockIdx.y * 4 + (threadIdx.x >> 6), mt = blockIdx.z, lane = threadIdx.x & 63;
+    const int fr = lane & 15, fg = lane >> 4, nks = p.rp >> 5, tid = threadIdx.x;
+    constexpr int MAXKS = 16;
+    const bool v_live = vt * 16 < p.vp;
+    bf16x8 wf[MAXKS];
     const bf16_t* w = p.uv + ((int64_t)(h * (p.vp >> 4) + vt) * nks * 64 + lane) * 8;
-    f32x4 acc = f32x4{0.f, 0.f, 0.f, 0.f};
-    for (int ks = wave; ks < nks; ks += 4) {
-        const bf16x8 wf = *(const bf16x8*)(w + ks * 512);
-        bf16x8 af = {};
-        if (ok) {
-            f32x4 a = f32x4{0.f, 0.f, 0.f, 0.f}, b = a;
-            for (int z = 0; z < p.n_split; z++) {
-                const int64_t at = ((int64_t)z * p.n_abs + i) * p.H + h;
-                const float e = __builtin_amdgcn_exp2f(p.part_ml[2 * at] - M);
-                const float* po = p.part_o + at * p.rp + ks * 32 + fg * 8;
-                a += e * *(const f32x4*)po;
-                b += e * *(const f32x4*)(po + 4);
-            }
 #pragma unroll
-            for (int e = 0; e < 4; e++) { af[e] = (bf16_t)(a[e] * invL); af[4 + e] = (bf16_t)(b[e] * invL); }
+    for (int ks = 0; ks < MAXKS; ks++) { wf[ks] = bf16x8{}; if (v_live && ks < nks) wf[ks] = *(const bf16x8*)(w + ks * 512); }
+    {
+        const int i = mt * 16 + (tid >> 4), z = tid & 15;                 // 16 tokens x 16 splits
+        float m = -1e30f, l = 0.f;
+        if (i < p.n_abs && z < p.n_split) {
+            const float* ml = p.part_ml + 2 * (((int64_t)z * p.n_abs + i) * p.H + h);
+            m = ml[0]; l = ml[1];
         }
-        acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(wf, af, acc, 0, 0, 0);
+        float M = m;
+#pragma unroll
+        for (int o = 8; o > 0; o >>= 1) M = fmaxf(M, __shfl_xor(M, o, 16));
+        const float e = __builtin_amdgcn_exp2f(m - M);
+        float L = l * e;
+#pragma unroll
+        for (int o = 8; o > 0; o >>= 1) L += __shfl_xor(L, o, 16);
+        sw[tid >> 4][z] = L > 0.f ? e / L : 0.f;
     }
-    red[wave][lane] = acc;
     __syncthreads();
-    if (wave || !ok) return;
-    acc = (red[0][lane] + red[1][lane]) + (red[2][lane] + red[3][lane]);
+    for (int c = tid; c < 16 * (p.rp >> 2); c += 256) {                   // 4 latent columns of one token
+        const int r = c / (p.rp >> 2), col = (c - r * (p.rp >> 2)) * 4, i = mt * 16 + r;
+        f32x4 a = f32x4{0.f, 0.f, 0.f, 0.f};
+        if (i < p.n_abs)
+            for (int z = 0; z < p.n_split; z++) a += sw[r][z] * *(const f32x4*)(p.part_o + (((int64_t)z * p.n_abs + i) * p.H + h) * p.rp + col);
+        bf16x4 b;
+#pragma unroll
+        for (int e = 0; e < 4; e++) b[e] = (bf16_t)a[e];
+        *(bf16x4*)(lat_smc + (((col >> 5) * 64 + r + 16 * ((col & 31) >> 3)) * 16 + 2 * (col & 7))) = b;
+    }
+    __syncthreads();
+    const int i = mt * 16 + fr;
+    if (!v_live) return;
+    f32x4 acc = f32x4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+    for (int ks = 0; ks < MAXKS; ks++)
+        if (ks < nks) acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(wf[ks], *(const bf16x8*)(lat_smc + (ks * 64 + lane) * 16), acc, 0, 0, 0);
+    if (i >= p.n_abs) return;
     const int64_t t = p.abs_tok[i];
     const int col = h * p.vp + vt * 16 + 4 * fg;
     const f32x4 g = *(const f32x4*)(p.proj + t * p.proj_ld + p.qrp + p.rp + col);

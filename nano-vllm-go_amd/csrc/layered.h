@@ -13,7 +13,7 @@
 
 namespace {
 
-constexpr int LAT_ABSORB_MAX = 16, LAT_ABSORB_MAX_RP = 512, LAT_SPLIT_MAX = 16, REC_STEP_MAX = 4;
+constexpr int LAT_ABSORB_MAX = 16, LAT_ABSORB_MAX_RP = 512, REC_STEP_MAX = 4;
 
 int pad_head(int d, int unit) {       // head sizes the attention instances exist for; larger ones take the plain kernel
     for (int p : {32, 64, 128, 256}) if (d <= p) return p;
@@ -574,20 +574,29 @@ void mix_latent(nvl_model* m, const LayerRun& r, const MixerW& w, const Meta& md
             // visible (query, key) pairs are at most tokens x min(window, keys)
             const double pairs = (double)(M - m->n_abs) * (c.window > 0 ? std::min<double>(c.window, m->key_max[(size_t)r.win]) : 0.5 * m->key_max[(size_t)r.win]);
             KScope ks(m, KC_ATTN, 2.0 * pairs * H * (c.dim + c.vdim), KS_ATTN, ((double)rows * H * (c.dim + c.vdim)) * ws + (double)M * H * (4.0 * c.dim + 4.0 * c.vdim + ws * c.vdim));
-            if (m->f32 || r.dp > 256 || r.vp > 256) {
+            if (m->f32 || r.dp > 256 || r.vp > 256 || c.scale == 0.f) {
                 const dim3 grid(max_len, H, n_seqs);
                 const size_t lds = (size_t)(r.dp + r.vp) * 4;
                 if (m->f32) hipLaunchKernelGGL((latent_plain_kernel<float>), grid, dim3(256), lds, m->stream, a);
                 else hipLaunchKernelGGL((latent_plain_kernel<bf16_t>), grid, dim3(256), lds, m->stream, a);
             } else {
-                const dim3 grid(cdiv(max_len, 128), H, n_seqs);
-#define NVL_LP(KSv, DTv) hipLaunchKernelGGL((latent_prefill_kernel<KSv, DTv>), grid, dim3(256), 0, m->stream, a)
+                const dim3 grid(H, n_seqs, cdiv(max_len, 256));
+#define NVL_LP(KSv, DTv)                                                                                                      \
+                do {                                                                                                         \
+                    constexpr int lds_ = latent_prefill_lds_bytes<KSv, DTv>();                                               \
+                    NVL_LDS_ATTR((latent_prefill_kernel<KSv, DTv>), lds_);                                                   \
+                    hipLaunchKernelGGL((latent_prefill_kernel<KSv, DTv>), grid, dim3(512), lds_, m->stream, a);              \
+                } while (0)
 #define NVL_LPK(KSv)                                                                                        \
                 do {                                                                                         \
                     if (r.vp == 32) NVL_LP(KSv, 2); else if (r.vp == 64) NVL_LP(KSv, 4);                      \
                     else if (r.vp == 128) NVL_LP(KSv, 8); else NVL_LP(KSv, 16);                               \
                 } while (0)
-                if (r.dp == 32) NVL_LPK(1); else if (r.dp == 64) NVL_LPK(2); else if (r.dp == 128) NVL_LPK(4); else NVL_LPK(8);
+                if (r.dp == 256 && r.vp == 256) hipLaunchKernelGGL((latent_prefill_wide_kernel<8, 16>), dim3(H, n_seqs, cdiv(max_len, 64)), dim3(256), 0, m->stream, a);
+                else if (r.dp == 32) NVL_LPK(1);
+                else if (r.dp == 64) NVL_LPK(2);
+                else if (r.dp == 128) NVL_LPK(4);
+                else if (r.vp == 32) NVL_LP(8, 2); else if (r.vp == 64) NVL_LP(8, 4); else NVL_LP(8, 8);
 #undef NVL_LPK
 #undef NVL_LP
             }
@@ -600,7 +609,7 @@ void mix_latent(nvl_model* m, const LayerRun& r, const MixerW& w, const Meta& md
         a.qa = m->lat_qa; a.Hp = ht * 16; a.part_o = m->lat_part_o; a.part_ml = m->lat_part_ml;
         const int tiles = 1 << layered_kt_log2(m);
         int split = 1;
-        while (split < LAT_SPLIT_MAX && ht * n * split < 256 && split * 2 <= tiles && (split * 2) * n <= m->lat_abs_cap) split *= 2;
+        while (split < LAT_SPLITS && ht * n * split < 256 && split * 2 <= tiles && (split * 2) * n <= m->lat_abs_cap) split *= 2;
         a.n_split = split;
         {
             KScope ks(m, KC_OTHER, 2.0 * n * H * (double)c.dim * c.kv_rank, KS_LAT_ABSORB, (double)H * c.dim * c.kv_rank * 2.0 + (double)n * H * (4.0 * c.dim + 2.0 * c.kv_rank));
@@ -627,7 +636,7 @@ void mix_latent(nvl_model* m, const LayerRun& r, const MixerW& w, const Meta& md
         }
         {
             KScope ks(m, KC_OTHER, 2.0 * n * H * (double)c.vdim * c.kv_rank, KS_LAT_UV, (double)H * c.vdim * c.kv_rank * 2.0 + (double)n * H * (4.0 * split * c.kv_rank + 6.0 * c.vdim));
-            hipLaunchKernelGGL(latent_uv_kernel, dim3(H, r.vp / 16, cdiv(n, 16)), dim3(256), 0, m->stream, a);
+            hipLaunchKernelGGL(latent_uv_kernel, dim3(H, cdiv(r.vp, 64), cdiv(n, 16)), dim3(256), (size_t)16 * r.rp * 2, m->stream, a);
             NVL_HIP(hipGetLastError());
         }
     }
@@ -642,10 +651,20 @@ void linrec(nvl_model* m, LinRecArgs a, int n_seqs, int M, int max_len, bool fus
     const int lds = linrec_step_lds_bytes(a.DK, a.DVp);
     const dim3 sgrid(a.H, n_seqs);
     a.len_lo = 1; a.len_hi = 1 << 30;
-    if (fused) {
-        if (m->f32) hipLaunchKernelGGL((linrec_step_kernel<(CH ? 1 : 0) + 2, float>), sgrid, dim3(LR_STEP_THREADS), lds, m->stream, a);
-        else hipLaunchKernelGGL((linrec_step_kernel<(CH ? 1 : 0) + 2, bf16_t>), sgrid, dim3(LR_STEP_THREADS), lds, m->stream, a);
+    auto step = [&](auto kind, auto act) {
+        constexpr int KIND = decltype(kind)::value;
+        using ActT = decltype(act);
+        int tv = 1;
+        while (tv < a.DVp / 4) tv <<= 1;
+        const int rows = cdiv(a.DK, LR_STEP_THREADS / tv);        // state rows per thread
+        if (rows <= 4) hipLaunchKernelGGL((linrec_step_kernel<KIND, 4, ActT>), sgrid, dim3(LR_STEP_THREADS), lds, m->stream, a);
+        else if (rows <= 8) hipLaunchKernelGGL((linrec_step_kernel<KIND, 8, ActT>), sgrid, dim3(LR_STEP_THREADS), lds, m->stream, a);
+        else hipLaunchKernelGGL((linrec_step_kernel<KIND, 16, ActT>), sgrid, dim3(LR_STEP_THREADS), lds, m->stream, a);
         NVL_HIP(hipGetLastError());
+    };
+    if (fused) {
+        if (m->f32) step(std::integral_constant<int, (CH ? 1 : 0) + 2>{}, float{});
+        else step(std::integral_constant<int, (CH ? 1 : 0) + 2>{}, bf16_t{});
         return;
     }
     const int nk = a.DK <= 32 ? 2 : (a.DK <= 64 ? 4 : (a.DK <= 128 ? 8 : 16)), nw = a.DV <= 64 ? 4 : 8;
@@ -653,11 +672,11 @@ void linrec(nvl_model* m, LinRecArgs a, int n_seqs, int M, int max_len, bool fus
     const bool steps = !chunks || m->min_len <= REC_STEP_MAX;
     if (steps) {
         a.len_hi = chunks ? REC_STEP_MAX : 1 << 30;
-        hipLaunchKernelGGL((linrec_step_kernel<(CH ? 1 : 0), float>), sgrid, dim3(LR_STEP_THREADS), lds, m->stream, a);
-        NVL_HIP(hipGetLastError());
+        step(std::integral_constant<int, CH ? 1 : 0>{}, float{});
     }
     if (!chunks || max_len <= REC_STEP_MAX) return;
     a.len_lo = REC_STEP_MAX + 1; a.len_hi = 1 << 30;
+    a.vec4 = a.DK % 4 == 0 && a.DV % 4 == 0 && a.ld % 4 == 0 && (((uintptr_t)a.q | (uintptr_t)a.k | (uintptr_t)a.v) & 15) == 0;
     a.n_slices = cdiv(a.DV, nw * 16);
     // few (head, sequence, slice) workgroups and a long prompt: pieces of the prompt in parallel (MODE 1, prefix, MODE 2)
     const int wgs = a.H * n_seqs * a.n_slices;
@@ -738,7 +757,7 @@ void mix_mamba2(nvl_model* m, const LayerRun& r, const MixerW& w, const Meta& md
         v.raw = m->lproj + inner; v.raw_ld = m->lproj_ld; v.w = w.conv_w; v.b = w.conv_b; v.taps = c.conv_taps; v.channels = r.conv_dim;
         v.out = m->lconv; v.out_ld = m->lconv_ld; v.ring = ring; v.ring_slot_stride = m->rec_slot_stride;
         v.tok_seq = md.tok_seq; v.tok_pos = md.tok_pos; v.seq_tok_start = md.seq_tok_start; v.seq_len = md.seq_len; v.seq_pos = md.seq_pos; v.seq_slot = md.seq_slot;
-        hipLaunchKernelGGL(conv_silu_kernel, dim3(M), dim3(256), 0, m->stream, v);
+        hipLaunchKernelGGL(conv_silu_kernel, dim3(cdiv(M, CONV_TOKENS), cdiv(r.conv_dim, 256)), dim3(256), 0, m->stream, v, M);
         hipLaunchKernelGGL(conv_ring_kernel, dim3(n_seqs, cdiv(r.conv_dim, 256)), dim3(256), 0, m->stream, v);
         NVL_HIP(hipGetLastError());
         a.v = m->lconv; a.k = m->lconv + inner; a.q = m->lconv + inner + GN; a.ld = m->lconv_ld;

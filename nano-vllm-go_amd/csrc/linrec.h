@@ -40,6 +40,7 @@ struct LinRecArgs {
     float* o; int64_t o_ld;            // [token][H * DV]
     float* state; int64_t slot_stride; // slot s: state + s * slot_stride, [H][DK][DVp]
     const int32_t *seq_tok_start, *seq_len, *seq_pos, *seq_slot;
+    int vec4;                          // q, k and v rows may be read 16 bytes at a time
     int len_lo, len_hi;                // sequences with len_lo <= tokens of this call <= len_hi are served, the others skipped
     // chunk-parallel prefill: `super` tokens per workgroup, scratch [seq][n_super][H][DK * DVp] and decays [..][H][DK or 1]
     float *z, *zdecay; int super, n_super, n_slices;
@@ -59,13 +60,13 @@ __device__ __forceinline__ float lr_softplus(float x) { return fmaxf(x, 0.f) + l
 // token by token.  grid (H, sequences), 512 threads: tv threads side by side on a state row (4 columns each), 512 / tv rows at
 // a time.  KIND bit 0: per-channel decay; bit 1: fused (conv in front of / norm + gate behind the recurrence).
 // ------------------------------------------------------------------------------------------
-constexpr int LR_STEP_THREADS = 512, LR_STEP_ROWS = 16;
+constexpr int LR_STEP_THREADS = 512;
 static inline int linrec_step_lds_bytes(int DK, int DVp) {
     int tv = 1;
     while (tv < DVp / 4) tv <<= 1;
     return 4 * (3 * ((DK + 3) & ~3) + DVp + LR_STEP_THREADS / tv * DVp);
 }
-template <int KIND, typename ActT>
+template <int KIND, int LR_STEP_ROWS, typename ActT>      // LR_STEP_ROWS: state rows a thread keeps in registers
 __global__ __launch_bounds__(LR_STEP_THREADS) void linrec_step_kernel(LinRecArgs p) {
     constexpr bool CH = KIND & 1, FUSED = KIND & 2;
     constexpr int NT = LR_STEP_THREADS;
@@ -78,12 +79,13 @@ __global__ __launch_bounds__(LR_STEP_THREADS) void linrec_step_kernel(LinRecArgs
     float* sk = sq + DK4;                // [DK]
     float* sa = sk + DK4;                // [DK]   decay (CH)
     float* sv = sa + DK4;                // [DVp]
-    float* red = sv + p.DVp;             // [groups of rows][DVp]
+    float* red = sv + p.DVp;             // [waves or groups of rows][DVp]
     __shared__ float s_red[NT / 64], s_sc[2];
     const int nv4 = p.DVp >> 2;
     int tv = 1;
     while (tv < nv4) tv <<= 1;           // host: nv4 <= NT
     const int rg = tid / tv, tc = tid - rg * tv, RG = NT / tv;
+    const int NRED = tv >= 64 ? RG : NT / 64;
     const bool live = tc < nv4;
     const int t0 = p.seq_tok_start[seq], pos0 = p.seq_pos[seq], slot = p.seq_slot[seq];
     float* st = p.state + (int64_t)slot * p.slot_stride + (int64_t)h * p.DK * p.DVp + 4 * tc;
@@ -161,8 +163,12 @@ __global__ __launch_bounds__(LR_STEP_THREADS) void linrec_step_kernel(LinRecArgs
                 for (int r = 0; r < 4; r++) { w[r] = fmaf(al, w[r], kk * v[r]); acc[r] = fmaf(qq, w[r], acc[r]); }
                 *(f32x4*)(st + (int64_t)row * p.DVp) = w;
             }
-            *(f32x4*)(red + (int64_t)rg * p.DVp + 4 * tc) = acc;
         }
+        // row groups of one wave first (tv < 64: 64 / tv of them side by side), then over the waves through LDS
+        for (int o = tv; o < 64; o <<= 1)
+#pragma unroll
+            for (int r = 0; r < 4; r++) acc[r] += __shfl_xor(acc[r], o, 64);
+        if (live && (tv >= 64 || (tid & 63) < tv)) *(f32x4*)(red + (int64_t)(tv >= 64 ? rg : tid >> 6) * p.DVp + 4 * tc) = acc;
         __syncthreads();
         // sum over the row groups; one column per thread (DV <= 4 * NT: up to four columns)
         float ov[4], ss = 0.f;
@@ -172,7 +178,7 @@ __global__ __launch_bounds__(LR_STEP_THREADS) void linrec_step_kernel(LinRecArgs
             ov[c] = 0.f;
             if (i < p.DV) {
                 float a = 0.f;
-                for (int r = 0; r < RG && r < p.DK; r++) a += red[(int64_t)r * p.DVp + i];
+                for (int r = 0; r < NRED; r++) a += red[(int64_t)r * p.DVp + i];
                 if (!CH) a = fmaf(p.Dskip[h], sv[i], a);
                 ov[c] = a;
                 ss = fmaf(a, a, ss);
@@ -210,13 +216,13 @@ __global__ __launch_bounds__(LR_STEP_THREADS) void linrec_step_kernel(LinRecArgs
 // ------------------------------------------------------------------------------------------
 template <int NK, int NW, bool CH>
 constexpr int linrec_chunk_lds_bytes(int rank) {
-    return 4 * (32 * (NK * 16 + 4) * (CH ? 3 : 2) + 32 * (NW * 16 + 4) + 32 * 36 + (CH ? 16 * NK * 16 : 96) + (CH ? 32 * rank : 0));
+    return 4 * (32 * (NK * 16 + 4) * (CH ? 3 : 2) + 32 * (NW * 16 + 4) + 32 * 36 + (CH ? (NW * 64 / (NK * 16) < 16 ? NW * 64 / (NK * 16) : 16) * NK * 16 : 96) + (CH ? 32 * rank : 0));
 }
 __device__ __forceinline__ f32x4 mfma_f32(float a, float b, f32x4 c) { return __builtin_amdgcn_mfma_f32_16x16x4f32(a, b, c, 0, 0, 0); }
 __device__ __forceinline__ float ex2(float x) { return __builtin_amdgcn_exp2f(x); }
 
 template <int NK, int NW, bool CH, int MODE>
-__global__ __launch_bounds__(NW * 64) void linrec_chunk_kernel(LinRecArgs p) {
+__global__ __launch_bounds__(NW * 64, NK > 8 ? 1 : (NW == 8 ? 4 : 3)) void linrec_chunk_kernel(LinRecArgs p) {
     constexpr int C = 32, DKP = NK * 16, LQ = DKP + 4, DVS = NW * 16, LV = DVS + 4, LA = C + 4, NT = NW * 64;
     constexpr float LOG2E = 1.4426950408889634f;
     const int h = blockIdx.x, seq = blockIdx.y;
@@ -232,7 +238,8 @@ __global__ __launch_bounds__(NW * 64) void linrec_chunk_kernel(LinRecArgs p) {
     float* vs = bs + (CH ? C * LQ : 0);                          // [C][LV]
     float* As = vs + C * LV;                                     // [C][LA]
     float* aux = As + C * LA;                                    // CH: [groups][DKP] partial sums; else b[32] | dt[32] | w[32]
-    float* a1s = aux + (CH ? 16 * DKP : 96);                     // CH: [C][rank]
+    constexpr int NG = NT / DKP < 16 ? NT / DKP : 16, TPG = C / NG;      // CH: groups of threads that share the tokens of a channel
+    float* a1s = aux + (CH ? NG * DKP : 96);                     // CH: [C][rank]
     const int tid = threadIdx.x, lane = tid & 63;
     const int wave = __builtin_amdgcn_readfirstlane(tid >> 6);
     const int fr = lane & 15, fg = lane >> 4;
@@ -242,6 +249,7 @@ __global__ __launch_bounds__(NW * 64) void linrec_chunk_kernel(LinRecArgs p) {
     float* st = p.state + (int64_t)p.seq_slot[seq] * p.slot_stride + (int64_t)h * p.DK * p.DVp;
     float* zs = MODE != 0 ? p.z + (((int64_t)seq * p.n_super + sup) * p.H + h) * ((int64_t)p.DK * p.DVp) : nullptr;
     const bool vlive = vcol < p.DVp;
+    const int so = 4 * fg * p.DVp + vcol;                        // this lane's place in a 16-row block of the state
     f32x4 S[NK];
 #pragma unroll
     for (int i = 0; i < NK; i++)
@@ -249,33 +257,74 @@ __global__ __launch_bounds__(NW * 64) void linrec_chunk_kernel(LinRecArgs p) {
         for (int r = 0; r < 4; r++) {
             const int row = 16 * i + 4 * fg + r;
             S[i][r] = 0.f;
-            if (MODE != 1 && row < p.DK && vlive && (MODE == 2 || !fresh)) S[i][r] = (MODE == 2 ? zs : st)[(int64_t)row * p.DVp + vcol];
+            if (MODE != 1 && row < p.DK && vlive && (MODE == 2 || !fresh)) S[i][r] = ((MODE == 2 ? zs : st) + (16 * i + r) * p.DVp)[so];
         }
     for (int i = tid; i < C * LA; i += NT) As[i] = 0.f;          // (the blocks above the diagonal stay zero)
     float btot = 0.f;                                            // MODE 1: log2 of the decay over all chunks (one channel per thread)
     const float A = CH ? 0.f : -expf(p.a_log[h]), Dh = CH ? 0.f : p.Dskip[h];
+    // the next chunk's rows are fetched into registers while the current one is worked on
+    constexpr int RQ = NT / (DKP / 4), RV = NT / (DVS / 4), NQ = (C + RQ - 1) / RQ, NV = (C + RV - 1) / RV, NA1 = 2;      // rows per pass, passes
+    const int tq = tid / (DKP / 4), dq = tid % (DKP / 4) * 4, tv_ = tid / (DVS / 4), dv_ = tid % (DVS / 4) * 4;
+    f32x4 rq[NQ], rk[NQ], rv[NV];
+    float ra[NA1], rdt = 0.f;
+    const int ld = (int)p.ld;
+    auto ld4 = [&](const float* src, int off, int d, int lim) {
+        f32x4 x = f32x4{0.f, 0.f, 0.f, 0.f};
+        if (p.vec4) { if (d < lim) x = *(const f32x4*)(src + off); }
+        else {
+#pragma unroll
+            for (int r = 0; r < 4; r++) if (d + r < lim) x[r] = src[off + r];
+        }
+        return x;
+    };
+    auto fetch = [&](int c0) {
+        const int nv = min(C, c_end - c0);
+        const int64_t tb = (int64_t)t0 + c0;
+        const float *qb = p.q + tb * ld + (int64_t)g * p.DK, *kb = p.k + tb * ld + (int64_t)g * p.DK, *vb = p.v + tb * ld + (int64_t)h * p.DV + v0;
+#pragma unroll
+        for (int i = 0; i < NQ; i++) {
+            const bool ok = tq + i * RQ < nv;
+            const int off = (tq + i * RQ) * ld + dq;
+            if (MODE != 1) rq[i] = ok ? ld4(qb, off, dq, p.DK) : f32x4{0.f, 0.f, 0.f, 0.f};
+            rk[i] = ok ? ld4(kb, off, dq, p.DK) : f32x4{0.f, 0.f, 0.f, 0.f};
+        }
+#pragma unroll
+        for (int i = 0; i < NV; i++)
+            rv[i] = tv_ + i * RV < nv ? ld4(vb, (tv_ + i * RV) * ld + dv_, v0 + dv_, p.DV) : f32x4{0.f, 0.f, 0.f, 0.f};
+        if constexpr (CH) {
+#pragma unroll
+            for (int i = 0; i < NA1; i++) {
+                const int e = tid + i * NT, t = e / p.rank;
+                ra[i] = t < nv ? p.a1[(tb + t) * p.a1_ld + (e - t * p.rank)] : 0.f;      // (t < nv <= 32: inside the chunk)
+            }
+        } else if (tid < nv) rdt = p.dt[(tb + tid) * p.dt_ld + h];
+    };
+    fetch(c_first);
 
     for (int c0 = c_first; c0 < c_end; c0 += C) {
         const int nv = min(C, c_end - c0);
         const int64_t tb = (int64_t)t0 + c0;
         __syncthreads();                                         // the previous chunk's readers are done
-        for (int i = tid; i < C * DKP; i += NT) {
-            const int t = i / DKP, d = i % DKP;
-            const bool ok = t < nv && d < p.DK;
-            if (MODE != 1) qs[t * LQ + d] = ok ? p.q[(tb + t) * p.ld + (int64_t)g * p.DK + d] * p.q_scale : 0.f;
-            ks[t * LQ + d] = ok ? p.k[(tb + t) * p.ld + (int64_t)g * p.DK + d] : 0.f;
-        }
-        for (int i = tid; i < C * DVS; i += NT) {
-            const int t = i / DVS, d = i % DVS;
-            vs[t * LV + d] = (t < nv && v0 + d < p.DV) ? p.v[(tb + t) * p.ld + (int64_t)h * p.DV + v0 + d] : 0.f;
-        }
-        if constexpr (CH) {
-            for (int i = tid; i < C * p.rank; i += NT) {
-                const int t = i / p.rank;
-                a1s[i] = t < nv ? p.a1[(tb + t) * p.a1_ld + (i - t * p.rank)] : 0.f;
+#pragma unroll
+        for (int i = 0; i < NQ; i++)
+            if (tq + i * RQ < C) {
+                if (MODE != 1) *(f32x4*)(qs + (tq + i * RQ) * LQ + dq) = rq[i] * p.q_scale;
+                *(f32x4*)(ks + (tq + i * RQ) * LQ + dq) = rk[i];
             }
+#pragma unroll
+        for (int i = 0; i < NV; i++) if (tv_ + i * RV < C) *(f32x4*)(vs + (tv_ + i * RV) * LV + dv_) = rv[i];
+        const float dt_raw = rdt;
+        if constexpr (CH) {
+#pragma unroll
+            for (int i = 0; i < NA1; i++) { const int e = tid + i * NT; if (e < C * p.rank) a1s[e] = ra[i]; }
+            for (int e = tid + NA1 * NT; e < C * p.rank; e += NT) {
+                const int t = e / p.rank;
+                a1s[e] = t < nv ? p.a1[(tb + t) * p.a1_ld + (e - t * p.rank)] : 0.f;
+            }
+        }
+        if (c0 + C < c_end) fetch(c0 + C);
+        if constexpr (CH) {
             __syncthreads();
-            constexpr int NG = NT / DKP < 16 ? NT / DKP : 16, TPG = C / NG;
             const int d = tid % DKP, grp = tid / DKP;
             float pre[TPG];
             if (grp < NG) {
@@ -286,6 +335,7 @@ __global__ __launch_bounds__(NW * 64) void linrec_chunk_kernel(LinRecArgs p) {
                     const float* w = p.a2 + (int64_t)(h * p.DK + d) * p.rank;
 #pragma unroll
                     for (int j = 0; j < TPG; j++) pre[j] = bias;
+#pragma unroll 2
                     for (int e = 0; e < p.rank; e++) {
                         const float we = w[e];
 #pragma unroll
@@ -306,7 +356,7 @@ __global__ __launch_bounds__(NW * 64) void linrec_chunk_kernel(LinRecArgs p) {
                 for (int j = 0; j < TPG; j++) bs[(grp * TPG + j) * LQ + d] = off + pre[j];
             }
         } else if (wave == 0 && lane < 32) {
-            const float dt = lane < nv ? lr_softplus(p.dt[(tb + lane) * p.dt_ld + h] + p.dt_bias[h]) : 0.f;
+            const float dt = lane < nv ? lr_softplus(dt_raw + p.dt_bias[h]) : 0.f;
             float s = A * dt * LOG2E;
 #pragma unroll
             for (int o = 1; o < 32; o <<= 1) { const float v = __shfl_up(s, o, 32); if (lane >= o) s += v; }
@@ -325,6 +375,7 @@ __global__ __launch_bounds__(NW * 64) void linrec_chunk_kernel(LinRecArgs p) {
                     const int s = x - t * (t + 1) / 2;
                     const int tr = (16 * half + t) * LQ, sr = (16 * half + s) * LQ;
                     f32x4 acc = f32x4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll 2
                     for (int d = 0; d < DKP; d += 4) {
                         const f32x4 q4 = *(const f32x4*)(qs + tr + d), k4 = *(const f32x4*)(ks + sr + d);
                         const f32x4 bt = *(const f32x4*)(bs + tr + d), b2 = *(const f32x4*)(bs + sr + d);
@@ -335,7 +386,7 @@ __global__ __launch_bounds__(NW * 64) void linrec_chunk_kernel(LinRecArgs p) {
                 }
                 if (wave == NW - 1) {                            // tokens 16..31 against 0..15, token 15's sums as the reference
                     f32x4 acc = f32x4{0.f, 0.f, 0.f, 0.f};
-#pragma unroll
+#pragma unroll 2
                     for (int i = 0; i < NK; i++) {
                         const int c = 16 * i + 4 * fg;
                         const f32x4 ref = *(const f32x4*)(bs + 15 * LQ + c);
@@ -350,7 +401,7 @@ __global__ __launch_bounds__(NW * 64) void linrec_chunk_kernel(LinRecArgs p) {
             } else if (wave < 3) {
                 const int tt = wave > 0, sb = wave == 2;
                 f32x4 acc = f32x4{0.f, 0.f, 0.f, 0.f};
-#pragma unroll
+#pragma unroll 2
                 for (int i = 0; i < NK; i++) {
                     const f32x4 a = *(const f32x4*)(qs + (16 * tt + fr) * LQ + 16 * i + 4 * fg), b = *(const f32x4*)(ks + (16 * sb + fr) * LQ + 16 * i + 4 * fg);
 #pragma unroll
@@ -366,6 +417,7 @@ __global__ __launch_bounds__(NW * 64) void linrec_chunk_kernel(LinRecArgs p) {
             __syncthreads();
         }
         if constexpr (CH) {                                      // q e^{b}, k e^{b_end - b} in place
+#pragma unroll 4
             for (int i = tid; i < C * DKP; i += NT) {
                 const int t = i / DKP, d = i % DKP;
                 const float b = bs[t * LQ + d];
@@ -380,6 +432,8 @@ __global__ __launch_bounds__(NW * 64) void linrec_chunk_kernel(LinRecArgs p) {
 #pragma unroll
             for (int r = 0; r < 4; r++) vf[sb][r] = vs[(16 * sb + 4 * fg + r) * LV + 16 * wave + fr];
         if constexpr (MODE != 1) {
+            float* ob = p.o + tb * p.o_ld + (int64_t)h * p.DV;
+            const int old = (int)p.o_ld;
 #pragma unroll
             for (int tt = 0; tt < 2; tt++) {
                 f32x4 y = f32x4{0.f, 0.f, 0.f, 0.f};
@@ -402,7 +456,7 @@ __global__ __launch_bounds__(NW * 64) void linrec_chunk_kernel(LinRecArgs p) {
 #pragma unroll
                 for (int r = 0; r < 4; r++) {
                     const int t = 16 * tt + 4 * fg + r;
-                    if (t < nv && vcol < p.DV) p.o[(tb + t) * p.o_ld + (int64_t)h * p.DV + vcol] = CH ? y[r] : fmaf(Dh, vf[tt][r], y[r]);
+                    if (t < nv && vcol < p.DV) ob[t * old + vcol] = CH ? y[r] : fmaf(Dh, vf[tt][r], y[r]);
                 }
             }
         }
@@ -433,12 +487,14 @@ __global__ __launch_bounds__(NW * 64) void linrec_chunk_kernel(LinRecArgs p) {
     }
     if (MODE == 2) return;
     float* dst = MODE == 1 ? zs : st;
+    int so_end = so;
+    asm volatile("" : "+v"(so_end));                          // (or the addresses of the first loads are kept in registers all along)
 #pragma unroll
     for (int i = 0; i < NK; i++)
 #pragma unroll
         for (int r = 0; r < 4; r++) {
             const int row = 16 * i + 4 * fg + r;
-            if (row < p.DK && vlive) dst[(int64_t)row * p.DVp + vcol] = S[i][r];
+            if (row < p.DK && vlive) (dst + (16 * i + r) * p.DVp)[so_end] = S[i][r];
         }
     if (MODE == 1 && slice == 0) {
         if (CH) { if (tid < p.DK) p.zdecay[(((int64_t)seq * p.n_super + sup) * p.H + h) * p.DK + tid] = ex2(btot); }
@@ -470,7 +526,7 @@ __global__ __launch_bounds__(256) void linrec_prefix_kernel(LinRecArgs p) {
 
 // ------------------------------------------------------------------------------------------
 // Causal convolution per channel + bias + silu over a batch whose raw rows [x | B | C] sit in `raw`; positions before this call come
-// from the slot's ring (row = position mod taps).  grid (tokens).  conv_ring_kernel then records the newest rows (its own
+// from the slot's ring (row = position mod taps).  conv_ring_kernel then records the newest rows (its own
 // launch: a ring row may still be read by a token of the same call).
 // ------------------------------------------------------------------------------------------
 struct ConvArgs {
@@ -480,15 +536,20 @@ struct ConvArgs {
     float* ring; int64_t ring_slot_stride;
     const int32_t *tok_seq, *tok_pos, *seq_tok_start, *seq_len, *seq_pos, *seq_slot;
 };
-__global__ __launch_bounds__(256) void conv_silu_kernel(ConvArgs p) {
-    const int t = blockIdx.x, seq = p.tok_seq[t], pos = p.tok_pos[t], first = p.seq_pos[seq];
-    const float* ring = p.ring + (int64_t)p.seq_slot[seq] * p.ring_slot_stride;
-    for (int c = threadIdx.x; c < p.channels; c += 256) {
-        float acc = p.b[c];
+constexpr int CONV_TOKENS = 8;       // tokens per workgroup: the rows they share are fetched once
+__global__ __launch_bounds__(256) void conv_silu_kernel(ConvArgs p, int n_tok) {      // grid (ceil(tokens / 8), ceil(channels / 256))
+    const int c = blockIdx.y * 256 + threadIdx.x;
+    if (c >= p.channels) return;
+    const float bias = p.b[c];
+    const float* w = p.w + (int64_t)c * p.taps + p.taps - 1;
+    for (int t = blockIdx.x * CONV_TOKENS; t < min(n_tok, ((int)blockIdx.x + 1) * CONV_TOKENS); t++) {
+        const int seq = p.tok_seq[t], pos = p.tok_pos[t], first = p.seq_pos[seq];
+        const float* ring = p.ring + (int64_t)p.seq_slot[seq] * p.ring_slot_stride;
+        float acc = bias;
         for (int b = p.taps - 1; b >= 0; b--) {
             if (pos - b < 0) continue;
             const float v = pos - b >= first ? p.raw[(int64_t)(t - b) * p.raw_ld + c] : ring[(int64_t)((pos - b) % p.taps) * p.channels + c];
-            acc = fmaf(v, p.w[(int64_t)c * p.taps + p.taps - 1 - b], acc);
+            acc = fmaf(v, w[-b], acc);
         }
         p.out[(int64_t)t * p.out_ld + c] = lr_silu(acc);
     }
@@ -525,7 +586,7 @@ __global__ __launch_bounds__(256) void gated_norm_kernel(GatedNormArgs p, ActT* 
     const int c0 = (id % p.parts) * p.part;
     const float* y = p.y + t * p.y_ld + c0;
     const float* g = p.gate + t * p.gate_ld + c0;
-    constexpr int KEEP = 8;
+    constexpr int KEEP = 16;
     float u[KEEP];
     float ss = 0.f;
 #pragma unroll

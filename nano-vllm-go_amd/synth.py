@@ -135,8 +135,59 @@ def tiny_config(family: str, **over) -> dict:
     return base
 
 
+def layered_shapes(cfg: dict, decay_rank: int = 16) -> list:
+    """[(slot, layer, shape, kind)] of every tensor of a model described by a list of layers (cfg["layers"]: config.LAYER_FIELDS
+    dicts); kind: matrix | norm | conv | bias | dt_bias | a_log — how a synthetic checkpoint should draw it."""
+    H, V = cfg["hidden"], cfg["vocab_size"]
+    out = [("tok_emb", 0, (V, H), "matrix"), ("lm_head", 0, (V, H), "matrix"), ("final_norm_w", 0, (H,), "norm")]
+    for i, c in enumerate(cfg["layers"]):
+        if c["weights_of"] >= 0:
+            continue
+        h, d, dv = c["heads"], c["dim"], c["vdim"]
+        t = [("attn_norm_w", (H,), "norm"), ("mix_post_norm", (H,), "norm")]
+        if c["mixer"] == "latent_attention":
+            qr, kr = c["q_rank"], c["kv_rank"]
+            t += [("lat_dq", (qr, H), "matrix"), ("lat_dq_norm", (qr,), "norm"), ("lat_uq", (h * d, qr), "matrix"), ("lat_dkv", (kr, H), "matrix"),
+                  ("lat_dkv_norm", (kr,), "norm"), ("lat_uk", (h * d, kr), "matrix"), ("lat_uv", (h * dv, kr), "matrix"),
+                  ("mix_gate", (h * dv, H), "matrix"), ("wo", (H, h * dv), "matrix")]
+        elif c["mixer"] == "mamba2":
+            inner, conv = h * dv, h * dv + 2 * c["groups"] * c["state"]
+            t += [("mamba_in_proj", (inner + conv + h, H), "matrix"), ("mamba_conv_w", (conv * c["conv_taps"],), "conv"), ("mamba_conv_b", (conv,), "bias"),
+                  ("mamba_dt_bias", (h,), "dt_bias"), ("mamba_a_log", (h,), "a_log"), ("mamba_d", (h,), "norm"), ("mamba_norm", (inner,), "norm"),
+                  ("mamba_out_proj", (H, inner), "matrix")]
+        else:
+            t += [("wq", (h * d, H), "matrix"), ("wk", (h * d, H), "matrix"), ("wv", (h * dv, H), "matrix"), ("mix_gate", (h * dv, H), "matrix"),
+                  ("wo", (H, h * dv), "matrix"), ("gla_norm", (dv,), "norm"), ("gla_a1", (decay_rank, H), "matrix"),
+                  ("gla_a2", (h * d, decay_rank), "matrix"), ("gla_a2_b", (h * d,), "bias")]
+        if c["ffn_dim"]:
+            F = c["ffn_dim"]
+            t += [("ffn_norm_w", (H,), "norm"), ("ffn_post_norm", (H,), "norm"), ("w1", (2 * F, H), "matrix"), ("w2", (H, F), "matrix")]
+        out += [(slot, i, shape, kind) for slot, shape, kind in t]
+    return out
+
+
+def _potuzen(width: int, layers: int, heads: int, q_rank: int, ff: int, window: int = 1024) -> dict:
+    """A Potuzen model at a real model's layer sizes: latent attention, Mamba-2 and gated linear attention in turn."""
+    from .config import LAYER_FIELDS
+    kinds = [dict(mixer="latent_attention", heads=heads, dim=128, vdim=128, q_rank=q_rank, kv_rank=512, window=window, scale=128 ** -0.5),
+             dict(mixer="mamba2", heads=width // 32, vdim=64, state=128, groups=1, norm_groups=1, conv_taps=4),
+             dict(mixer="gla", heads=heads, dim=128, vdim=128, tau=16.0)]
+    return dict(vocab_size=32000, hidden=width, num_layers=layers, num_heads=0, num_kv_heads=0, head_dim=0, ffn_dim=0, max_seq_len=4096,
+                attention_type="gqa", norm_type="rmsnorm", position_type="nope", activation_type="geglu", block_style="sandwich",
+                rope_base=0.0, norm_eps=1e-6, tied_embedding=False, layers=[dict(LAYER_FIELDS, ffn_dim=ff, **kinds[i % 3]) for i in range(layers)])
+
+
+def _hybrid(hidden: int, layers: int, heads: int, ff: int) -> dict:
+    """The attention + Mamba-2 hybrid family at the same sizes (its attention where _potuzen has latent attention, Mamba-2 elsewhere)."""
+    return dict(vocab_size=32000, hidden=hidden, num_layers=layers, num_heads=heads, num_kv_heads=heads // 4, head_dim=128, ffn_dim=ff,
+                max_seq_len=4096, attention_type="gqa", norm_type="rmsnorm", position_type="nope", activation_type="swiglu",
+                block_style="sequential", norm_eps=1e-5, tied_embedding=False, mamba_expand=2, mamba_state_size=128,
+                mamba_num_heads=hidden // 32, mamba_head_dim=64, mamba_n_groups=1, mamba_conv_kernel=4,
+                hybrid_layers=["attention" if i % 3 == 0 else "mamba" for i in range(layers)])
+
+
 FULL_CONFIGS = {
-    # SURVEY.md §8 config shapes C1-C5
+    # the reference families' headline shapes
     "gpt2": dict(vocab_size=50257, hidden=768, num_layers=12, num_heads=12, num_kv_heads=12, head_dim=64,
                  ffn_dim=3072, max_seq_len=1024, attention_type="mha", norm_type="layernorm",
                  position_type="learned", activation_type="gelu", block_style="sequential", norm_eps=1e-5,
@@ -159,6 +210,9 @@ FULL_CONFIGS = {
                        ffn_dim=14336, max_seq_len=4096, attention_type="gqa", norm_type="rmsnorm",
                        position_type="rope", activation_type="swiglu", block_style="sequential",
                        rope_base=500000.0, norm_eps=1e-5, tied_embedding=False),
+    # the Potuzen design at a real model's layer sizes, and the closest other family at the same sizes
+    "potuzen-2k": _potuzen(2048, 12, 16, 768, 6144), "hybrid-2k": _hybrid(2048, 12, 16, 6144),
+    "potuzen-4k": _potuzen(4096, 6, 32, 1536, 12288), "hybrid-4k": _hybrid(4096, 6, 32, 12288),
 }
 for _c in FULL_CONFIGS.values():
     for _k, _v in dict(use_moe=False, num_experts=0, num_experts_per_tok=0, embedding_multiplier=0.0,
