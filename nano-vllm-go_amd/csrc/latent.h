@@ -61,20 +61,18 @@ __global__ __launch_bounds__(256) void latent_norm_kernel(LatentArgs p) {
     __shared__ float red[8];
     const int t = blockIdx.x;
     const float* pr = p.proj + (int64_t)t * p.proj_ld;
-    float sq = 0.f, sc = 0.f;
-    for (int i = threadIdx.x; i < p.qrank; i += 256) sq = fmaf(pr[i], pr[i], sq);
-    for (int i = threadIdx.x; i < p.kvrank; i += 256) sc = fmaf(pr[p.qrp + i], pr[p.qrp + i], sc);
+    float sq = 0.f, sc = 0.f;          // (the padding columns of c_q and c are zero)
+    for (int i = threadIdx.x * 4; i < p.qrp; i += 1024) { const f32x4 v = *(const f32x4*)(pr + i); sq += (v[0] * v[0] + v[1] * v[1]) + (v[2] * v[2] + v[3] * v[3]); }
+    for (int i = threadIdx.x * 4; i < p.rp; i += 1024) { const f32x4 v = *(const f32x4*)(pr + p.qrp + i); sc += (v[0] * v[0] + v[1] * v[1]) + (v[2] * v[2] + v[3] * v[3]); }
     sq = wave_sum(sq); sc = wave_sum(sc);
     if ((threadIdx.x & 63) == 0) { red[threadIdx.x >> 6] = sq; red[4 + (threadIdx.x >> 6)] = sc; }
     __syncthreads();
     const float rq = sqrtf((red[0] + red[1] + red[2] + red[3]) / (float)p.qrank + p.eps), rc = sqrtf((red[4] + red[5] + red[6] + red[7]) / (float)p.kvrank + p.eps);
-    for (int i = threadIdx.x; i < p.qrp; i += 256)
-        ActIO<ActT>::st((ActT*)p.cq + act_index<ActT>(t, i, p.qrp), (pr[i] / rq) * p.cq_norm[i]);
+    for (int i = threadIdx.x * 4; i < p.qrp; i += 1024) act_store4<ActT>((ActT*)p.cq, t, i, p.qrp, *(const f32x4*)(pr + i) / rq * *(const f32x4*)(p.cq_norm + i));
     int blk, row;
     kv_locate(p.blk_table, p.tok_tbl[t], p.tok_pos[t], p.bs, blk, row);
     ActT* c = (ActT*)p.cache + (int64_t)blk * p.block_stride;
-    for (int i = threadIdx.x; i < p.rp; i += 256)
-        ActIO<ActT>::st(c + act_index<ActT>(row, i, p.rp), (pr[p.qrp + i] / rc) * p.c_norm[i]);
+    for (int i = threadIdx.x * 4; i < p.rp; i += 1024) act_store4<ActT>(c, row, i, p.rp, *(const f32x4*)(pr + p.qrp + i) / rc * *(const f32x4*)(p.c_norm + i));
 }
 
 // ---- gather the latents a portion's keys need into contiguous rows: 32 rows (one unit of either layout) per workgroup ----
@@ -536,12 +534,12 @@ __global__ __launch_bounds__(256) void latent_decode_kernel(LatentArgs p) {
     for (int i = 0; i < NR; i++) *(f32x4*)(p.part_o + at * p.rp + (wave * NR + i) * 16 + 4 * fg) = o[i];
 }
 
-// combines the key splits, projects by W_uv and gates: grid (H, ceil(vp / 64), ceil(n_abs / 16)), 4 waves, one 16-column tile of V each.
+// combines the key splits, projects by W_uv and gates: grid (H, ceil(vp / 256), ceil(n_abs / 16)), 16 waves, one 16-column tile of V each.
 // The combined latents of the 16 tokens are made once per workgroup (fragment-major bf16 in LDS) while the weight fragments are in flight.
-static __global__ __launch_bounds__(256) void latent_uv_kernel(LatentArgs p) {
+static __global__ __launch_bounds__(1024) void latent_uv_kernel(LatentArgs p) {
     extern __shared__ __attribute__((aligned(16))) char lat_smc[];       // [rp / 32][64 lanes][16 B]
     __shared__ float sw[16][LAT_SPLITS];                                  // weight of a split's partial, 1 / L folded in
-    const int h = blockIdx.x, vt = blockIdx.y * 4 + (threadIdx.x >> 6), mt = blockIdx.z, lane = threadIdx.x & 63;
+    const int h = blockIdx.x, vt = blockIdx.y * 16 + (threadIdx.x >> 6), mt = blockIdx.z, lane = threadIdx.x & 63;
     const int fr = lane & 15, fg = lane >> 4, nks = p.rp >> 5, tid = threadIdx.x;
     constexpr int MAXKS = 16;
     const bool v_live = vt * 16 < p.vp;
@@ -549,7 +547,7 @@ static __global__ __launch_bounds__(256) void latent_uv_kernel(LatentArgs p) {
     const bf16_t* w = p.uv + ((int64_t)(h * (p.vp >> 4) + vt) * nks * 64 + lane) * 8;
 #pragma unroll
     for (int ks = 0; ks < MAXKS; ks++) { wf[ks] = bf16x8{}; if (v_live && ks < nks) wf[ks] = *(const bf16x8*)(w + ks * 512); }
-    {
+    if (tid < 256) {
         const int i = mt * 16 + (tid >> 4), z = tid & 15;                 // 16 tokens x 16 splits
         float m = -1e30f, l = 0.f;
         if (i < p.n_abs && z < p.n_split) {
@@ -566,10 +564,11 @@ static __global__ __launch_bounds__(256) void latent_uv_kernel(LatentArgs p) {
         sw[tid >> 4][z] = L > 0.f ? e / L : 0.f;
     }
     __syncthreads();
-    for (int c = tid; c < 16 * (p.rp >> 2); c += 256) {                   // 4 latent columns of one token
+    for (int c = tid; c < 16 * (p.rp >> 2); c += 1024) {                   // 4 latent columns of one token
         const int r = c / (p.rp >> 2), col = (c - r * (p.rp >> 2)) * 4, i = mt * 16 + r;
         f32x4 a = f32x4{0.f, 0.f, 0.f, 0.f};
         if (i < p.n_abs)
+#pragma unroll 8
             for (int z = 0; z < p.n_split; z++) a += sw[r][z] * *(const f32x4*)(p.part_o + (((int64_t)z * p.n_abs + i) * p.H + h) * p.rp + col);
         bf16x4 b;
 #pragma unroll

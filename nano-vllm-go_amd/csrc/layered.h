@@ -636,7 +636,7 @@ void mix_latent(nvl_model* m, const LayerRun& r, const MixerW& w, const Meta& md
         }
         {
             KScope ks(m, KC_OTHER, 2.0 * n * H * (double)c.vdim * c.kv_rank, KS_LAT_UV, (double)H * c.vdim * c.kv_rank * 2.0 + (double)n * H * (4.0 * split * c.kv_rank + 6.0 * c.vdim));
-            hipLaunchKernelGGL(latent_uv_kernel, dim3(H, cdiv(r.vp, 64), cdiv(n, 16)), dim3(256), (size_t)16 * r.rp * 2, m->stream, a);
+            hipLaunchKernelGGL(latent_uv_kernel, dim3(H, cdiv(r.vp, 256), cdiv(n, 16)), dim3(1024), (size_t)16 * r.rp * 2, m->stream, a);
             NVL_HIP(hipGetLastError());
         }
     }
@@ -714,18 +714,24 @@ void linrec(nvl_model* m, LinRecArgs a, int n_seqs, int M, int max_len, bool fus
     NVL_HIP(hipGetLastError());
 }
 
+template <typename ActT, bool GATE_FIRST>
+void gated_norm_launch(nvl_model* m, GatedNormArgs a) {
+    const bool v4 = a.part % 4 == 0 && a.y_ld % 4 == 0 && a.gate_ld % 4 == 0 && (((uintptr_t)a.y | (uintptr_t)a.gate) & 15) == 0;
+    const bool wide = a.part > 1024;
+    a.lanes = 4;
+    while (a.lanes < 64 && a.lanes * (v4 ? 4 : 1) < a.part) a.lanes *= 2;
+    const dim3 grid(wide ? a.rows * a.parts : cdiv((int64_t)a.rows * a.parts, 256 / a.lanes));
+    ActT* out = (ActT*)m->lmix;
+    if (wide && v4) hipLaunchKernelGGL((gated_norm_kernel<ActT, GATE_FIRST, true, true>), grid, dim3(256), 0, m->stream, a, out);
+    else if (wide) hipLaunchKernelGGL((gated_norm_kernel<ActT, GATE_FIRST, true, false>), grid, dim3(256), 0, m->stream, a, out);
+    else if (v4) hipLaunchKernelGGL((gated_norm_kernel<ActT, GATE_FIRST, false, true>), grid, dim3(256), 0, m->stream, a, out);
+    else hipLaunchKernelGGL((gated_norm_kernel<ActT, GATE_FIRST, false, false>), grid, dim3(256), 0, m->stream, a, out);
+}
 template <bool GATE_FIRST>
 void gated_norm(nvl_model* m, const GatedNormArgs& a, int site) {
     KScope ks(m, KC_OTHER, 0, site, (double)a.rows * a.parts * a.part * (8.0 + (double)m->wsize));
-    const bool wide = a.part > 512;
-    const dim3 grid(wide ? a.rows * a.parts : cdiv((int64_t)a.rows * a.parts, 4));
-    if (m->f32) {
-        if (wide) hipLaunchKernelGGL((gated_norm_kernel<float, GATE_FIRST, true>), grid, dim3(256), 0, m->stream, a, (float*)m->lmix);
-        else hipLaunchKernelGGL((gated_norm_kernel<float, GATE_FIRST, false>), grid, dim3(256), 0, m->stream, a, (float*)m->lmix);
-    } else {
-        if (wide) hipLaunchKernelGGL((gated_norm_kernel<bf16_t, GATE_FIRST, true>), grid, dim3(256), 0, m->stream, a, (bf16_t*)m->lmix);
-        else hipLaunchKernelGGL((gated_norm_kernel<bf16_t, GATE_FIRST, false>), grid, dim3(256), 0, m->stream, a, (bf16_t*)m->lmix);
-    }
+    if (m->f32) gated_norm_launch<float, GATE_FIRST>(m, a);
+    else gated_norm_launch<bf16_t, GATE_FIRST>(m, a);
     NVL_HIP(hipGetLastError());
 }
 
@@ -757,13 +763,18 @@ void mix_mamba2(nvl_model* m, const LayerRun& r, const MixerW& w, const Meta& md
         v.raw = m->lproj + inner; v.raw_ld = m->lproj_ld; v.w = w.conv_w; v.b = w.conv_b; v.taps = c.conv_taps; v.channels = r.conv_dim;
         v.out = m->lconv; v.out_ld = m->lconv_ld; v.ring = ring; v.ring_slot_stride = m->rec_slot_stride;
         v.tok_seq = md.tok_seq; v.tok_pos = md.tok_pos; v.seq_tok_start = md.seq_tok_start; v.seq_len = md.seq_len; v.seq_pos = md.seq_pos; v.seq_slot = md.seq_slot;
-        hipLaunchKernelGGL(conv_silu_kernel, dim3(cdiv(M, CONV_TOKENS), cdiv(r.conv_dim, 256)), dim3(256), 0, m->stream, v, M);
+        const bool v4 = r.conv_dim % 4 == 0 && v.raw_ld % 4 == 0 && ((uintptr_t)v.raw & 15) == 0;
+        const dim3 cgrid(cdiv(M, CONV_TOKENS), cdiv(r.conv_dim, 1024));
+        if (v4 && v.taps == 4) hipLaunchKernelGGL((conv_silu_kernel<4>), cgrid, dim3(256), 0, m->stream, v, M);
+        else if (v4 && v.taps == 3) hipLaunchKernelGGL((conv_silu_kernel<3>), cgrid, dim3(256), 0, m->stream, v, M);
+        else if (v4 && v.taps == 2) hipLaunchKernelGGL((conv_silu_kernel<2>), cgrid, dim3(256), 0, m->stream, v, M);
+        else hipLaunchKernelGGL((conv_silu_kernel<0>), cgrid, dim3(256), 0, m->stream, v, M);
         hipLaunchKernelGGL(conv_ring_kernel, dim3(n_seqs, cdiv(r.conv_dim, 256)), dim3(256), 0, m->stream, v);
         NVL_HIP(hipGetLastError());
         a.v = m->lconv; a.k = m->lconv + inner; a.q = m->lconv + inner + GN; a.ld = m->lconv_ld;
     }
     linrec<false>(m, a, n_seqs, M, max_len, fused, KS_MAMBA_SCAN);
-    GatedNormArgs g{m->lo, m->lo_ld, m->lproj, m->lproj_ld, w.mix_norm, M, c.norm_groups, inner / c.norm_groups, m->cfg.norm_eps, r.ko};
+    GatedNormArgs g{m->lo, m->lo_ld, m->lproj, m->lproj_ld, w.mix_norm, M, c.norm_groups, inner / c.norm_groups, m->cfg.norm_eps, r.ko, 0};
     gated_norm<true>(m, g, KS_MAMBA_GATE);
 }
 
@@ -779,7 +790,7 @@ void mix_gla(nvl_model* m, const LayerRun& r, const MixerW& w, const Meta& md, i
     const bool fused = max_len <= REC_STEP_MAX;
     linrec<true>(m, a, n_seqs, M, max_len, fused, KS_GLA_SCAN);
     if (fused) return;
-    GatedNormArgs g{m->lo, m->lo_ld, a.gate, m->lproj_ld, w.mix_norm, M, c.heads, c.vdim, m->cfg.norm_eps, r.ko};
+    GatedNormArgs g{m->lo, m->lo_ld, a.gate, m->lproj_ld, w.mix_norm, M, c.heads, c.vdim, m->cfg.norm_eps, r.ko, 0};
     gated_norm<false>(m, g, KS_GLA_GATE);
 }
 

@@ -67,7 +67,7 @@ static inline int linrec_step_lds_bytes(int DK, int DVp) {
     return 4 * (3 * ((DK + 3) & ~3) + DVp + LR_STEP_THREADS / tv * DVp);
 }
 template <int KIND, int LR_STEP_ROWS, typename ActT>      // LR_STEP_ROWS: state rows a thread keeps in registers
-__global__ __launch_bounds__(LR_STEP_THREADS) void linrec_step_kernel(LinRecArgs p) {
+__global__ __launch_bounds__(LR_STEP_THREADS, LR_STEP_ROWS <= 8 ? 4 : 2) void linrec_step_kernel(LinRecArgs p) {
     constexpr bool CH = KIND & 1, FUSED = KIND & 2;
     constexpr int NT = LR_STEP_THREADS;
     const int h = blockIdx.x, seq = blockIdx.y, tid = threadIdx.x;
@@ -88,15 +88,20 @@ __global__ __launch_bounds__(LR_STEP_THREADS) void linrec_step_kernel(LinRecArgs
     const int NRED = tv >= 64 ? RG : NT / 64;
     const bool live = tc < nv4;
     const int t0 = p.seq_tok_start[seq], pos0 = p.seq_pos[seq], slot = p.seq_slot[seq];
-    float* st = p.state + (int64_t)slot * p.slot_stride + (int64_t)h * p.DK * p.DVp + 4 * tc;
+    float* st = p.state + (int64_t)slot * p.slot_stride + (int64_t)h * p.DK * p.DVp;
+    int so = rg * p.DVp + 4 * tc;        // this thread's place in a pass of RG rows
+    const int pass = RG * p.DVp;
     const int g = h / p.kdiv;
     f32x4 s[LR_STEP_ROWS];               // the first LR_STEP_ROWS rows of this thread, fetched before anything else is known
 #pragma unroll
     for (int i = 0; i < LR_STEP_ROWS; i++) {
         const int row = rg + i * RG;
-        s[i] = f32x4{0.f, 0.f, 0.f, 0.f};
-        if (live && row < p.DK && pos0 > 0) s[i] = *(const f32x4*)(st + (int64_t)row * p.DVp);
+        const bool ok = live && row < p.DK;                     // (no branches around s: it stays in registers)
+        const f32x4 x = *(const f32x4*)(st + (ok ? i * pass + so : 0));
+#pragma unroll
+        for (int r = 0; r < 4; r++) s[i][r] = ok && pos0 > 0 ? x[r] : 0.f;
     }
+    asm volatile("" : "+v"(so));            // (or the addresses of these loads are kept in registers for the stores)
     for (int i = tid; i < p.DVp; i += NT) sv[i] = 0.f;
     __syncthreads();
     for (int it = 0; it < n; it++) {
@@ -142,26 +147,27 @@ __global__ __launch_bounds__(LR_STEP_THREADS) void linrec_step_kernel(LinRecArgs
         }
         __syncthreads();
         f32x4 acc = f32x4{0.f, 0.f, 0.f, 0.f};
-        if (live) {
-            const f32x4 v = *(const f32x4*)(sv + 4 * tc);
+        {
+            const f32x4 v = *(const f32x4*)(sv + (live ? 4 * tc : 0));
             const float ksc = CH ? 1.f : s_sc[0], al0 = CH ? 1.f : s_sc[1];
 #pragma unroll
             for (int i = 0; i < LR_STEP_ROWS; i++) {
                 const int row = rg + i * RG;
-                if (row < p.DK) {
-                    const float al = CH ? sa[row] : al0, kk = sk[row] * ksc, qq = sq[row];
+                const bool ok = live && row < p.DK;
+                const int rr = ok ? row : 0;
+                const float al = CH ? sa[rr] : al0, kk = ok ? sk[rr] * ksc : 0.f, qq = ok ? sq[rr] : 0.f;
 #pragma unroll
-                    for (int r = 0; r < 4; r++) { s[i][r] = fmaf(al, s[i][r], kk * v[r]); acc[r] = fmaf(qq, s[i][r], acc[r]); }
-                    if (it == n - 1) *(f32x4*)(st + (int64_t)row * p.DVp) = s[i];
-                }
+                for (int r = 0; r < 4; r++) { s[i][r] = fmaf(al, s[i][r], kk * v[r]); acc[r] = fmaf(qq, s[i][r], acc[r]); }
+                if (ok && it == n - 1) *(f32x4*)(st + i * pass + so) = s[i];
             }
-            for (int row = rg + LR_STEP_ROWS * RG; row < p.DK; row += RG) {     // (a state larger than the registers: streamed)
+#pragma unroll 1
+            for (int row = rg + LR_STEP_ROWS * RG; live && row < p.DK; row += RG) {     // (a state larger than the registers: streamed)
                 f32x4 w = f32x4{0.f, 0.f, 0.f, 0.f};
-                if (pos0 + it > 0) w = *(const f32x4*)(st + (int64_t)row * p.DVp);
+                if (pos0 + it > 0) w = *(const f32x4*)(st + (int64_t)row * p.DVp + 4 * tc);
                 const float al = CH ? sa[row] : al0, kk = sk[row] * ksc, qq = sq[row];
 #pragma unroll
                 for (int r = 0; r < 4; r++) { w[r] = fmaf(al, w[r], kk * v[r]); acc[r] = fmaf(qq, w[r], acc[r]); }
-                *(f32x4*)(st + (int64_t)row * p.DVp) = w;
+                *(f32x4*)(st + (int64_t)row * p.DVp + 4 * tc) = w;
             }
         }
         // row groups of one wave first (tv < 64: 64 / tv of them side by side), then over the waves through LDS
@@ -178,6 +184,7 @@ __global__ __launch_bounds__(LR_STEP_THREADS) void linrec_step_kernel(LinRecArgs
             ov[c] = 0.f;
             if (i < p.DV) {
                 float a = 0.f;
+#pragma unroll 4
                 for (int r = 0; r < NRED; r++) a += red[(int64_t)r * p.DVp + i];
                 if (!CH) a = fmaf(p.Dskip[h], sv[i], a);
                 ov[c] = a;
@@ -537,21 +544,62 @@ struct ConvArgs {
     const int32_t *tok_seq, *tok_pos, *seq_tok_start, *seq_len, *seq_pos, *seq_slot;
 };
 constexpr int CONV_TOKENS = 8;       // tokens per workgroup: the rows they share are fetched once
-__global__ __launch_bounds__(256) void conv_silu_kernel(ConvArgs p, int n_tok) {      // grid (ceil(tokens / 8), ceil(channels / 256))
-    const int c = blockIdx.y * 256 + threadIdx.x;
+__device__ __forceinline__ float conv_at(const ConvArgs& p, const float* ring, int t, int pos, int first, int c) {
+    float acc = p.b[c];
+    for (int b = p.taps - 1; b >= 0; b--) {
+        if (pos - b < 0) continue;
+        const float v = pos - b >= first ? p.raw[(int64_t)(t - b) * p.raw_ld + c] : ring[(int64_t)((pos - b) % p.taps) * p.channels + c];
+        acc = fmaf(v, p.w[(int64_t)c * p.taps + p.taps - 1 - b], acc);
+    }
+    return lr_silu(acc);
+}
+// grid (ceil(tokens / 8), ceil(channels / 1024)), 4 channels per thread.  TAPS > 0 (channel count, row pitch and base multiples of 4):
+// a tile that lies inside one sequence runs from registers.
+template <int TAPS>
+__global__ __launch_bounds__(256) void conv_silu_kernel(ConvArgs p, int n_tok) {
+    const int c = (blockIdx.y * 256 + threadIdx.x) * 4;
     if (c >= p.channels) return;
-    const float bias = p.b[c];
-    const float* w = p.w + (int64_t)c * p.taps + p.taps - 1;
-    for (int t = blockIdx.x * CONV_TOKENS; t < min(n_tok, ((int)blockIdx.x + 1) * CONV_TOKENS); t++) {
+    const int t0 = blockIdx.x * CONV_TOKENS, t1 = min(n_tok, t0 + CONV_TOKENS);
+    if constexpr (TAPS > 0) {
+        const int seq = p.tok_seq[t0], first = p.seq_pos[seq];
+        if (p.tok_seq[t1 - 1] == seq) {
+            const int pos0 = p.tok_pos[t0] - (TAPS - 1);             // position of r[0]
+            const float* x = p.raw + (int64_t)t0 * p.raw_ld + c;
+            const float* ring = p.ring + (int64_t)p.seq_slot[seq] * p.ring_slot_stride + c;
+            f32x4 r[CONV_TOKENS + TAPS - 1], w[TAPS];
+#pragma unroll
+            for (int i = 0; i < CONV_TOKENS + TAPS - 1; i++) {
+                r[i] = f32x4{0.f, 0.f, 0.f, 0.f};
+                if (i < TAPS - 1 && pos0 + i < first) {              // (uniform) before this call: zeros before the sequence, else the ring
+                    if (pos0 + i >= 0) r[i] = *(const f32x4*)(ring + (int64_t)((pos0 + i) % TAPS) * p.channels);
+                } else if (t0 + i - (TAPS - 1) < t1) {
+                    r[i] = *(const f32x4*)(x + (int64_t)(i - (TAPS - 1)) * p.raw_ld);
+                }
+            }
+#pragma unroll
+            for (int k = 0; k < TAPS; k++)
+#pragma unroll
+                for (int e = 0; e < 4; e++) w[k][e] = p.w[(int64_t)(c + e) * TAPS + k];
+            const f32x4 bias = *(const f32x4*)(p.b + c);
+#pragma unroll
+            for (int i = 0; i < CONV_TOKENS; i++) {
+                f32x4 a = bias;
+#pragma unroll
+                for (int k = 0; k < TAPS; k++)
+#pragma unroll
+                    for (int e = 0; e < 4; e++) a[e] = fmaf(r[i + k][e], w[k][e], a[e]);
+#pragma unroll
+                for (int e = 0; e < 4; e++) a[e] = lr_silu(a[e]);
+                if (t0 + i < t1) *(f32x4*)(p.out + (int64_t)(t0 + i) * p.out_ld + c) = a;
+            }
+            return;
+        }
+    }
+    for (int t = t0; t < t1; t++) {                                  // (tiles that span sequences)
         const int seq = p.tok_seq[t], pos = p.tok_pos[t], first = p.seq_pos[seq];
         const float* ring = p.ring + (int64_t)p.seq_slot[seq] * p.ring_slot_stride;
-        float acc = bias;
-        for (int b = p.taps - 1; b >= 0; b--) {
-            if (pos - b < 0) continue;
-            const float v = pos - b >= first ? p.raw[(int64_t)(t - b) * p.raw_ld + c] : ring[(int64_t)((pos - b) % p.taps) * p.channels + c];
-            acc = fmaf(v, w[-b], acc);
-        }
-        p.out[(int64_t)t * p.out_ld + c] = lr_silu(acc);
+#pragma unroll
+        for (int e = 0; e < 4; e++) if (c + e < p.channels) p.out[(int64_t)t * p.out_ld + c + e] = conv_at(p, ring, t, pos, first, c + e);
     }
 }
 __global__ __launch_bounds__(256) void conv_ring_kernel(ConvArgs p) {      // grid (sequences, ceil(channels / 256))
@@ -566,7 +614,8 @@ __global__ __launch_bounds__(256) void conv_ring_kernel(ConvArgs p) {      // gr
 // RMS norm over equal parts of a row with a silu gate, written as the next projection's operand.
 //   GATE_FIRST (Mamba-2):  u = y * silu(gate); out = rms(u) * w[column of the row]
 //   else (GLA)          :  out = rms(y) * w[column of the part] * silu(gate)
-// One wave per (token, part): grid ceil(tokens * parts / 4), or one 256-thread workgroup each when the parts are long (WIDE).
+// V4: parts, row pitches and bases are multiples of 4 columns.  `lanes` (a power of two <= 64) lanes share a part, or one 256-thread
+// workgroup each when the parts are long (WIDE): grid ceil(tokens * parts / (256 / lanes)).
 // ------------------------------------------------------------------------------------------
 struct GatedNormArgs {
     const float* y; int64_t y_ld;
@@ -575,43 +624,75 @@ struct GatedNormArgs {
     int rows, parts, part;     // part = columns per part
     float eps;
     int64_t out_ld;
+    int lanes;
 };
-template <typename ActT, bool GATE_FIRST, bool WIDE>
+template <typename ActT, bool GATE_FIRST, bool WIDE, bool V4>
 __global__ __launch_bounds__(256) void gated_norm_kernel(GatedNormArgs p, ActT* __restrict__ out) {
     __shared__ float red[4];
-    constexpr int NT = WIDE ? 256 : 64;
-    const int id = WIDE ? blockIdx.x : blockIdx.x * 4 + (threadIdx.x >> 6), l = threadIdx.x & (NT - 1);
-    if (!WIDE && id >= p.rows * p.parts) return;
-    const int64_t t = id / p.parts;
-    const int c0 = (id % p.parts) * p.part;
+    constexpr int E = V4 ? 4 : 1, KEEP = V4 ? 4 : 8;
+    const int nt = WIDE ? 256 : p.lanes, l = threadIdx.x & (nt - 1);
+    const int id = WIDE ? blockIdx.x : blockIdx.x * (256 / nt) + threadIdx.x / nt;
+    const bool ok = id < p.rows * p.parts;
+    const int64_t t = ok ? id / p.parts : 0;
+    const int c0 = ok ? (id % p.parts) * p.part : 0, part = ok ? p.part : 0;
     const float* y = p.y + t * p.y_ld + c0;
     const float* g = p.gate + t * p.gate_ld + c0;
-    constexpr int KEEP = 16;
-    float u[KEEP];
+    struct Vec { float v[E]; };
+    auto ld = [&](const float* a, int c) {
+        Vec r;
+        if constexpr (V4) { const f32x4 x = *(const f32x4*)(a + c); for (int e = 0; e < 4; e++) r.v[e] = x[e]; }
+        else r.v[0] = a[c];
+        return r;
+    };
+    auto load = [&](int c) {
+        Vec u = ld(y, c);
+        if (GATE_FIRST) {
+            const Vec s = ld(g, c);
+#pragma unroll
+            for (int e = 0; e < E; e++) u.v[e] *= lr_silu(s.v[e]);
+        }
+        return u;
+    };
+    Vec u[KEEP];
     float ss = 0.f;
 #pragma unroll
     for (int i = 0; i < KEEP; i++) {
-        const int c = l + i * NT;
-        u[i] = 0.f;
-        if (c < p.part) u[i] = GATE_FIRST ? y[c] * lr_silu(g[c]) : y[c];
-        ss = fmaf(u[i], u[i], ss);
+        const int c = (l + i * nt) * E;
+#pragma unroll
+        for (int e = 0; e < E; e++) u[i].v[e] = 0.f;
+        if (c < part) u[i] = load(c);
+#pragma unroll
+        for (int e = 0; e < E; e++) ss = fmaf(u[i].v[e], u[i].v[e], ss);
     }
-    for (int c = l + KEEP * NT; c < p.part; c += NT) { const float v = GATE_FIRST ? y[c] * lr_silu(g[c]) : y[c]; ss = fmaf(v, v, ss); }
-    ss = wave_sum(ss);
+    for (int c = (l + KEEP * nt) * E; c < part; c += nt * E) {
+        const Vec x = load(c);
+#pragma unroll
+        for (int e = 0; e < E; e++) ss = fmaf(x.v[e], x.v[e], ss);
+    }
     if (WIDE) {
+        ss = wave_sum(ss);
         if ((threadIdx.x & 63) == 0) red[threadIdx.x >> 6] = ss;
         __syncthreads();
         ss = red[0] + red[1] + red[2] + red[3];
+    } else {
+        for (int o = 1; o < nt; o <<= 1) ss += __shfl_xor(ss, o, 64);
     }
     const float inv = 1.0f / sqrtf(ss / (float)p.part + p.eps);
-    auto put = [&](int c, float v) {
-        v *= inv * p.w[GATE_FIRST ? c0 + c : c];
-        if (!GATE_FIRST) v *= lr_silu(g[c]);
-        ActIO<ActT>::st(out + act_index<ActT>(t, c0 + c, p.out_ld), v);
+    auto put = [&](int c, Vec x) {
+        const Vec w = ld(p.w, GATE_FIRST ? c0 + c : c);
+#pragma unroll
+        for (int e = 0; e < E; e++) x.v[e] *= inv * w.v[e];
+        if (!GATE_FIRST) {
+            const Vec s = ld(g, c);
+#pragma unroll
+            for (int e = 0; e < E; e++) x.v[e] *= lr_silu(s.v[e]);
+        }
+        if constexpr (V4) act_store4<ActT>(out, t, c0 + c, p.out_ld, f32x4{x.v[0], x.v[1], x.v[2], x.v[3]});
+        else ActIO<ActT>::st(out + act_index<ActT>(t, c0 + c, p.out_ld), x.v[0]);
     };
 #pragma unroll
-    for (int i = 0; i < KEEP; i++) { const int c = l + i * NT; if (c < p.part) put(c, u[i]); }
-    for (int c = l + KEEP * NT; c < p.part; c += NT) put(c, GATE_FIRST ? y[c] * lr_silu(g[c]) : y[c]);
+    for (int i = 0; i < KEEP; i++) { const int c = (l + i * nt) * E; if (c < part) put(c, u[i]); }
+    for (int c = (l + KEEP * nt) * E; c < part; c += nt * E) put(c, load(c));
 }
 
 }  // namespace nvl
