@@ -27,9 +27,10 @@
 extern "C" {
 #endif
 
-#define NVL_ABI_VERSION 4      /* 2: Mamba2 / hybrid layers (config fields, tensor kinds), nvl_stats.evictions, kernel stats;
+#define NVL_ABI_VERSION 5      /* 2: Mamba2 / hybrid layers (config fields, tensor kinds), nvl_stats.evictions, kernel stats;
                                   3: nvl_get_weight, nvl_get_stamps, nvl_tp_p2p_rearm, debug modes 2 / 4 (additions only);
-                                  4: models described by a list of layers, library-owned block pool, nvl_forward_rows (additions only) */
+                                  4: models described by a list of layers, library-owned block pool, nvl_forward_rows (additions only);
+                                  5: rotated latent attention, channel-wise gated delta rule, output-only norms (new config fields at the end) */
 
 typedef enum nvl_status {
     NVL_OK = 0,
@@ -48,10 +49,11 @@ enum { NVL_ATTN_MHA = 0, NVL_ATTN_MQA = 1, NVL_ATTN_GQA = 2 };        /* config.
 enum { NVL_NORM_LAYER = 0, NVL_NORM_RMS = 1 };                        /* config.go:27-30 */
 enum { NVL_POS_LEARNED = 0, NVL_POS_ROPE = 1, NVL_POS_NONE = 2 };     /* config.go:35-40 */
 enum { NVL_ACT_GELU = 0, NVL_ACT_SWIGLU = 1,                          /* config.go:45-48 */
-       NVL_ACT_GEGLU = 2 };                                           /* gelu_tanh(gate) * up */
+       NVL_ACT_GEGLU = 2,                                             /* gelu_tanh(gate) * up */
+       NVL_ACT_CLAMPED_GLU = 3 };   /* g sigmoid(1.702 g) (u + 1), g = min(gate, limit), u = clamp(up, -limit, limit): nvl_layer_config.ffn_limit */
 enum { NVL_BLOCK_SEQUENTIAL = 0, NVL_BLOCK_PARALLEL = 1,              /* config.go:53-56 */
-       NVL_BLOCK_SANDWICH = 2 };   /* a norm before AND after each sublayer, x += norm_b(f(norm_a(x))); the model is described
-                                      by a list of layers (nvl_layer_config, nvl_create_layers)  */
+       NVL_BLOCK_SANDWICH = 2,     /* a norm before AND after each sublayer, x += norm_b(f(norm_a(x)))  } the model is described by a list */
+       NVL_BLOCK_POST = 3 };       /* a norm after each sublayer only, x += scale * norm(f(x))           } of layers (nvl_create_layers)    */
 
 typedef struct nvl_model_config {
     int32_t vocab_size, hidden, num_layers, num_heads, num_kv_heads, head_dim;
@@ -67,13 +69,17 @@ typedef struct nvl_model_config {
      * mamba_head_dim 0 = expand * hidden / mamba_num_heads (mamba2.go:58-61).  All zero: no Mamba2 layers. */
     int32_t  mamba_expand, mamba_state_size, mamba_num_heads, mamba_head_dim, mamba_n_groups, mamba_conv_kernel;
     uint64_t mamba_layer_mask[2];
+    /* models described by a list of layers */
+    float   norm_weight_offset;     /* added to every stored weight of the model's norm (1: weights are kept as differences from one)     */
+    float   logit_softcap;          /* logits <- cap tanh(logits / cap); 0: none                                                          */
 } nvl_model_config;
 
 /* ---- models described by a list of layers: every layer names its mixer, the mixer's sizes and its feed-forward ---- */
 enum {
-    NVL_MIXER_LATENT_ATTENTION = 0, /* queries and keys/values through low-rank latents, no positions; the cache holds the latent */
+    NVL_MIXER_LATENT_ATTENTION = 0, /* queries and keys/values through low-rank latents; the cache holds the latent (and the rotated key part) */
     NVL_MIXER_MAMBA2 = 1,           /* causal convolution + selective state space, gate before a grouped norm                     */
-    NVL_MIXER_GLA = 2               /* gated linear attention: a decay per key channel                                            */
+    NVL_MIXER_GLA = 2,              /* gated linear attention: a decay per key channel                                            */
+    NVL_MIXER_CHANNEL_DELTA = 3     /* delta rule with a decay per key channel, short convolutions on q, k and v                  */
 };
 typedef struct nvl_layer_config {
     int32_t mixer;                  /* NVL_MIXER_*                                                                         */
@@ -86,6 +92,13 @@ typedef struct nvl_layer_config {
     float   tau;                    /* GLA: alpha = sigmoid(z)^(1/tau)                                                     */
     int32_t decay_rank;             /* GLA: rank of the decay projection; 0: as the uploaded tensor says                   */
     int32_t ffn_dim;                /* 0: no feed-forward                                                                  */
+    float   ffn_limit;              /* NVL_ACT_CLAMPED_GLU                                                                 */
+    int32_t kv_from;                /* latent attention: use this earlier layer's cached latents and rotated keys; -1: own */
+    int32_t rot_dim;                /* latent attention: rotated query/key dimensions per head beside `dim`; 0: none       */
+    int32_t gate_per_head;          /* latent attention: 1: one output gate per head; 0: one per channel                   */
+    int32_t kv_heads;               /* channel delta: heads of q and k (heads is a multiple)                               */
+    double  rot_base;               /* rotation: pair i turns by base^(-2 i / rot_dim) per position                        */
+    double  rot_factor, rot_original, rot_fast, rot_slow;       /* YaRN context extension; rot_factor 0: none              */
 } nvl_layer_config;
 
 /* Arithmetic the device path computes in. */
@@ -159,18 +172,24 @@ typedef enum nvl_tensor_kind {
      * FFN_NORM_W (the norms before the sublayers), WQ / WK / WV / WO, W1 (gate rows, then up rows), W2, the MAMBA_* kinds */
     NVL_T_MIX_POST_NORM,   /* [H] norm after the mixer                                                */
     NVL_T_FFN_POST_NORM,   /* [H] norm after the feed-forward                                         */
-    NVL_T_MIX_GATE,        /* [heads*vdim, H] output gate (latent attention, GLA)                     */
+    NVL_T_MIX_GATE,        /* [heads*vdim, H] output gate (latent attention, GLA); [heads, H] with gate_per_head */
     NVL_T_LAT_DQ,          /* [q_rank, H]         NVL_T_LAT_DQ_NORM  [q_rank]                         */
     NVL_T_LAT_DQ_NORM,
-    NVL_T_LAT_UQ,          /* [heads*dim, q_rank]                                                     */
-    NVL_T_LAT_DKV,         /* [kv_rank, H]        NVL_T_LAT_DKV_NORM [kv_rank]                        */
+    NVL_T_LAT_UQ,          /* [heads*(dim + rot_dim), q_rank]   per head: unrotated, then rotated     */
+    NVL_T_LAT_DKV,         /* [kv_rank + rot_dim, H]  NVL_T_LAT_DKV_NORM [kv_rank]  (not with kv_from) */
     NVL_T_LAT_DKV_NORM,
     NVL_T_LAT_UK,          /* [heads*dim, kv_rank]                                                    */
     NVL_T_LAT_UV,          /* [heads*vdim, kv_rank]                                                   */
-    NVL_T_GLA_NORM,        /* [vdim]                                                                  */
-    NVL_T_GLA_A1,          /* [rank, H]           decay projection, low-rank: z = A2 (A1 h) + b       */
+    NVL_T_GLA_NORM,        /* [vdim]              (channel delta too)                                 */
+    NVL_T_GLA_A1,          /* [rank, H]           decay projection, low-rank: z = A2 (A1 h) + b (channel delta too) */
     NVL_T_GLA_A2,          /* [heads*dim, rank]                                                       */
     NVL_T_GLA_A2_B,        /* [heads*dim]                                                             */
+    NVL_T_MIX_SCALE,       /* [H] layer scale of the mixer's result        (NVL_BLOCK_POST; optional) */
+    NVL_T_FFN_SCALE,       /* [H] layer scale of the feed-forward's result (NVL_BLOCK_POST; optional) */
+    NVL_T_DELTA_CONV,      /* [(2*kv_heads*dim + heads*vdim) * taps] q, k and v channels one after the other */
+    NVL_T_DELTA_BETA,      /* [heads, H]          step sizes of the delta rule                        */
+    NVL_T_DELTA_G1,        /* [rank, H]           output gate, low-rank: sigmoid(G2 (G1 h))           */
+    NVL_T_DELTA_G2,        /* [heads*vdim, rank]                                                      */
     NVL_T_COUNT
 } nvl_tensor_kind;
 
@@ -185,9 +204,9 @@ enum {
 /* Replaces tensor.NewTransformerModel (generic_model.go:41-61) + the runner's model ownership
  * (tensor_model_runner.go:21-33).  Fails with NVL_ERR_NO_DEVICE when no GPU is present. */
 int nvl_create(const nvl_model_config* cfg, const nvl_runtime_opts* opts, nvl_model** out);
-/* nvl_create for a model described by a list of layers (cfg->block_style == NVL_BLOCK_SANDWICH): `layers` has cfg->num_layers
- * entries; of cfg only vocab_size, hidden, num_layers, max_seq_len, norm_eps, activation_type (NVL_ACT_GEGLU),
- * embedding_multiplier, logits_scaling and tied_embedding are read. */
+/* nvl_create for a model described by a list of layers (cfg->block_style NVL_BLOCK_SANDWICH or NVL_BLOCK_POST): `layers` has
+ * cfg->num_layers entries; of cfg only vocab_size, hidden, num_layers, max_seq_len, norm_eps, norm_weight_offset, activation_type
+ * (NVL_ACT_GEGLU or NVL_ACT_CLAMPED_GLU), embedding_multiplier, logits_scaling, logit_softcap and tied_embedding are read. */
 int nvl_create_layers(const nvl_model_config* cfg, const nvl_layer_config* layers, const nvl_runtime_opts* opts, nvl_model** out);
 
 /* Replaces loadTensorFromData + the per-kind placement in loadAttention/loadFFN/loadMoE/loadNorm
@@ -208,7 +227,7 @@ int nvl_load_safetensors(nvl_model* m, const char* path);
  * the reference's model_info.json) -> nvl_model_config.  Reference quirks kept: max_position_embeddings and
  * rope_scaling are not read.  Errors are reported through nvl_last_error(NULL). */
 int nvl_load_config_json(const char* path, nvl_model_config* cfg);
-/* The layer list of a config.json whose architecture is described by one ("Potuzen"): writes up to `cap` entries, returns
+/* The layer list of a config.json whose architecture is described by one ("Potuzen", "Lufazen"): writes up to `cap` entries, returns
  * how many the file has; 0 for every other architecture.  Such a file names no longest sequence: nvl_load_config_json sets
  * max_seq_len to 4096, the caller may change it before nvl_create_layers. */
 int nvl_load_layers_json(const char* path, nvl_layer_config* layers, int cap);

@@ -46,6 +46,8 @@ class ModelConfig:
     mamba_n_groups: int = 0
     mamba_conv_kernel: int = 0
     layers: list = field(default_factory=list)            # models described by a list of layers: one dict per layer (LAYER_FIELDS)
+    norm_weight_offset: float = 0.0
+    logit_softcap: float = 0.0
 
     @property
     def mamba_layer_mask(self):
@@ -135,7 +137,8 @@ def new_granite_config(size: str = "350m") -> ModelConfig:   # config.go:241-330
 
 
 LAYER_FIELDS = dict(mixer="", weights_of=-1, heads=0, dim=0, vdim=0, q_rank=0, kv_rank=0, window=0, scale=0.0, state=0, groups=0,
-                    norm_groups=0, conv_taps=0, tau=0.0, decay_rank=0, ffn_dim=0)      # nvl_layer_config
+                    norm_groups=0, conv_taps=0, tau=0.0, decay_rank=0, ffn_dim=0, ffn_limit=0.0, kv_from=-1, rot_dim=0, gate_per_head=0, kv_heads=0,
+                    rot_base=0.0, rot_factor=0.0, rot_original=0.0, rot_fast=0.0, rot_slow=0.0)      # nvl_layer_config
 
 
 def _potuzen_layer(e: dict) -> dict:
@@ -168,6 +171,42 @@ def potuzen_config(raw: dict) -> ModelConfig:
                        layers=[_potuzen_layer(e) for e in raw["layers"]])
 
 
+def _lufazen_layer(e: dict) -> dict:
+    """One entry of a Lufazen config.json's layer list -> the fields of nvl_layer_config."""
+    mx, mlp, ty = e["mixer"], e.get("mlp"), e["type"]
+    out = dict(LAYER_FIELDS, mixer=ty, heads=mx["heads"], dim=mx["dim"], vdim=mx["vdim"])
+    if ty == "latent_attention":
+        rot = mx["rot"]
+        if rot["dims"] != mx["rot_dim"]:
+            raise ValueError("rot.dims differs from rot_dim")
+        out.update(q_rank=mx["q_rank"], kv_rank=mx["kv_rank"], scale=float(mx["scale"]), rot_dim=mx["rot_dim"], gate_per_head=1, rot_base=float(rot["base"]))
+        if mx.get("kv_from") is not None:
+            out["kv_from"] = mx["kv_from"]
+        if rot.get("scaling") is not None:
+            out.update({"rot_" + k: float(rot["scaling"][k]) for k in ("factor", "original", "fast", "slow")})
+    elif ty == "channel_delta":
+        out.update(kv_heads=mx["kv_heads"], conv_taps=mx["conv"])
+    else:
+        raise ValueError(f"unknown mixer {ty!r}")
+    if mlp is not None:
+        if mlp.get("kind", "dense") != "dense":
+            raise ValueError(f"unknown feed-forward kind {mlp['kind']!r}")
+        out.update(ffn_dim=mlp["ff"], ffn_limit=float(mlp["limit"]))
+    return out
+
+
+def lufazen_config(raw: dict) -> ModelConfig:
+    """The Lufazen design: a list of layers (rotated latent attention / channel-wise gated delta rule), norms on the sublayers' outputs
+    whose weights are kept as differences from one, layer scales, clamped gated feed-forwards, capped logits."""
+    return ModelConfig(architecture="Lufazen", model_name="lufazen", vocab_size=raw["vocab"], hidden=raw["width"],
+                       num_layers=len(raw["layers"]), max_seq_len=4096, attention_type="gqa", norm_type="rmsnorm", position_type="nope",
+                       activation_type="clamped_glu", block_style="post", rope_base=0.0, norm_eps=float(raw["norm"]["eps"]),
+                       norm_weight_offset=1.0, logit_softcap=float(raw.get("logit_softcap") or 0.0), layers=[_lufazen_layer(e) for e in raw["layers"]])
+
+
+LAYERED = {"Potuzen": potuzen_config, "Lufazen": lufazen_config}      # architectures described by a list of layers
+
+
 def load_model_config(raw: dict | str) -> ModelConfig:
     """LoadModelConfig (generic_loader.go:808-972) on an already-parsed HF config.json (or its text).
     Reference quirks kept: max_position_embeddings and rope_scaling are never read, so max_seq_len
@@ -175,8 +214,8 @@ def load_model_config(raw: dict | str) -> ModelConfig:
     if isinstance(raw, str):
         raw = json.loads(raw)
     arch = raw.get("architecture")
-    if arch == "Potuzen":
-        return potuzen_config(raw)
+    if arch in LAYERED:
+        return LAYERED[arch](raw)
     if arch == "gpt2":
         c = new_gpt2_config()
     elif arch == "falcon":

@@ -82,6 +82,13 @@ __device__ __forceinline__ float gelu_tanh_f(float x) {
     return 0.5f * x * (1.0f + th);
 }
 
+// gated unit with both inputs clamped: g sigmoid(slope g) (u + 1)
+__device__ __forceinline__ float clamp_glu_f(float g, float u, float limit, float slope) {
+    g = fminf(g, limit);
+    u = fminf(fmaxf(u, -limit), limit);
+    return g / (1.0f + __expf(-slope * g)) * (u + 1.0f);
+}
+
 // ---- wave reductions (64 lanes) ----------------------------------------------
 __device__ __forceinline__ float wave_sum(float v) {
 #pragma unroll

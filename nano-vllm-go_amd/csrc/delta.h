@@ -1,0 +1,603 @@
+// delta.h — gated delta rule with a decay per key channel, in fp32 throughout.  Per head, S [DK][DV]:
+//     S <- diag(a_t) S,  u_t = beta_t (v_t - S^T k_t),  S <- S + k_t u_t^T,  o_t = S^T q_t
+// q and k are unit vectors (q also times q_scale); a_t = exp(-exp(A_log) softplus(z_t + bias)), z_t a projection; a group of heads
+// shares q and k, decays and values are a head's own.
+//
+//   delta_step_kernel   token by token, the state streamed once per token (decode).  FUSED (one token per sequence): the short
+//                       convolutions, the low-rank decay and gate projections, the head norm and the output gate in the same launch.
+//   delta_prep_kernel   32 tokens of one head, independent of the state that enters them (prefill, all chunks at once).
+//   delta_scan_kernel   carries the state through the chunks of a sequence: three products per chunk.
+//
+// Chunk form.  With b_t = the inclusive sum of log a inside the chunk and S_in the state that enters it:
+//     u_t = beta_t (v_t - (k_t e^{b_t})^T S_in - sum_{s<t} M[t][s] u_s),      M[t][s] = sum_c k_t[c] k_s[c] e^{b_t[c] - b_s[c]}
+//     o_t = (q_t e^{b_t})^T S_in + sum_{s<=t} A[t][s] u_s,                    A[t][s] = sum_c q_t[c] k_s[c] e^{b_t[c] - b_s[c]}
+//     S_out = diag(e^{b_end}) S_in + sum_s (k_s e^{b_end - b_s}) u_s^T
+// With T = (I + diag(beta) M)^-1 diag(beta):  U = U0 - W S_in,  U0 = T V,  W = T (K e^b);  O = O0 + Q' S_in,  O0 = A U0,
+// Q' = Q e^b - A W.  prep leaves -W, Q', (K e^{b_end - b})^T and e^{b_end} in scratch, U0 in the place of v and O0 in the place of o.
+// Every exponent that is evaluated is <= 0: a decay per channel cannot be split into e^{b_t} e^{-b_s}, so the two 16 x 16 diagonal
+// blocks of A and M are summed pair by pair, and the block below the diagonal takes token 15's sums as its reference.  T comes from
+// forward substitution (16 x 16 blocks): the powers of M that a series would need can be far larger than T itself.
+// Products are v_mfma_f32_16x16x4_f32: operand element i of lane group g stands for k = 16 n + 4 g + i on both sides, so that an
+// accumulator (lane = column, rows 4 g + r) is the B operand of the next product as it stands.
+#pragma once
+#include "common.h"
+#include "linrec.h"
+
+namespace nvl {
+
+constexpr float DELTA_UNIT_EPS = 1e-6f;
+
+struct DeltaArgs {
+    int H, G, DK, DV, DVp;             // G: heads of q and k; DVp: row pitch of the state (DV padded to 4)
+    const float *q, *k; float* v;      // after convolution and silu; row pitch ld; v: prep leaves U0 there
+    int64_t ld;
+    float q_scale;
+    const float* z; int64_t z_ld;      // [token][H * DK] decay projections before the bias
+    const float *a_log, *dt_bias;      // [H], [H * DK]
+    const float* beta; int64_t beta_ld;        // raw step sizes (before sigmoid), one column per head
+    float* o; int64_t o_ld;            // [token][H * DV]
+    float* state; int64_t slot_stride; // slot s: state + s * slot_stride, [H][DK][DVp]
+    const int32_t *seq_tok_start, *seq_len, *seq_pos, *seq_slot;
+    int vec4;                          // q, k rows may be read 16 bytes at a time
+    int len_lo, len_hi;                // sequences with len_lo <= tokens of this call <= len_hi are served, the others skipped
+    float* ws;                         // chunk c of sequence i is (seq_tok_start / 32 + i + c); per chunk and head delta_ws_floats
+    // FUSED step: raw [q | k | v] columns before the convolution, a ring of the last `taps` raw rows per slot
+    const float* raw; int64_t raw_ld; const float* conv_w; int taps, channels; float* ring; int64_t ring_slot_stride;
+    const float *a1, *g1; int64_t lr_ld; int a_rank, g_rank, a_rkp, g_rkp;       // [token][rank]; ranks padded
+    const void *a2, *g2;               // [H * DK][a_rkp], [H * DV][g_rkp], row-major
+    const float* norm_w; float eps; void* out; int64_t out_ld;
+};
+
+constexpr int DELTA_C = 32;            // tokens per chunk
+static inline __host__ __device__ int64_t delta_ws_floats(int dkp) { return (int64_t)dkp * (3 * DELTA_C + 1); }     // -W | Q' | K^T | e^{b_end}
+__device__ __forceinline__ int64_t delta_chunk(const DeltaArgs& p, int seq, int c) { return p.seq_tok_start[seq] / DELTA_C + seq + c; }
+
+// ------------------------------------------------------------------------------------------
+// prep: grid (heads, sequences, chunks), 4 waves
+// ------------------------------------------------------------------------------------------
+template <int NK> constexpr int delta_prep_lds_bytes() { return 4 * (3 * DELTA_C * (NK * 16 + 4) + 2 * DELTA_C * 36 + DELTA_C + 256); }
+
+template <int NK>
+__global__ __launch_bounds__(256, NK > 8 ? 1 : 2) void delta_prep_kernel(DeltaArgs p) {
+    constexpr int C = DELTA_C, DKP = NK * 16, LQ = DKP + 4, LA = 36, NT = 256;
+    constexpr float LOG2E = 1.4426950408889634f;
+    const int h = blockIdx.x, seq = blockIdx.y, c0 = blockIdx.z * C;
+    const int n = p.seq_len[seq];
+    if (n < p.len_lo || n > p.len_hi || c0 >= n) return;         // (uniform: before any barrier)
+    extern __shared__ __attribute__((aligned(16))) float dl_sm[];
+    float* qs = dl_sm;                   // [C][LQ]  q, later q e^b
+    float* ks = qs + C * LQ;             // [C][LQ]  k, later k e^b
+    float* bs = ks + C * LQ;             // [C][LQ]  inclusive sums of log2 a
+    float* As = bs + C * LQ;             // [C][LA]
+    float* Ms = As + C * LA;             // [C][LA]  M, later T
+    float* be = Ms + C * LA;             // [C]
+    float* aux = be + C;                 // [256]
+    const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6);
+    const int fr = lane & 15, fg = lane >> 4;
+    const int nv = min(C, n - c0);
+    const int64_t tb = (int64_t)p.seq_tok_start[seq] + c0;
+    const int g = h / (p.H / p.G);
+    {   // q and k as unit vectors; DKP / 4 lanes hold a row
+        constexpr int LR = DKP / 4, R = NT / LR;
+        const int t0 = tid / LR, d = tid % LR * 4;
+        auto ld4 = [&](const float* src) {
+            f32x4 x = f32x4{0.f, 0.f, 0.f, 0.f};
+            if (p.vec4) { if (d < p.DK) x = *(const f32x4*)(src + d); }
+            else {
+#pragma unroll
+                for (int r = 0; r < 4; r++) if (d + r < p.DK) x[r] = src[d + r];
+            }
+            return x;
+        };
+#pragma unroll
+        for (int i = 0; i < C / R; i++) {
+            const int t = t0 + i * R;
+            f32x4 q = f32x4{0.f, 0.f, 0.f, 0.f}, k = q;
+            if (t < nv) { q = ld4(p.q + (tb + t) * p.ld + (int64_t)g * p.DK); k = ld4(p.k + (tb + t) * p.ld + (int64_t)g * p.DK); }
+            float sq = (q[0] * q[0] + q[1] * q[1]) + (q[2] * q[2] + q[3] * q[3]), sk = (k[0] * k[0] + k[1] * k[1]) + (k[2] * k[2] + k[3] * k[3]);
+#pragma unroll
+            for (int o = 1; o < LR; o <<= 1) { sq += __shfl_xor(sq, o, 64); sk += __shfl_xor(sk, o, 64); }
+            *(f32x4*)(qs + t * LQ + d) = q * (p.q_scale / sqrtf(sq + DELTA_UNIT_EPS));
+            *(f32x4*)(ks + t * LQ + d) = k * (1.0f / sqrtf(sk + DELTA_UNIT_EPS));
+        }
+    }
+    {   // decays: a channel per thread, NG groups share the tokens
+        constexpr int NG = NT / DKP, TPG = C / NG;
+        const int d = tid % DKP, grp = tid / DKP;
+        float pre[TPG];
+        const float A = -expf(p.a_log[h]) * LOG2E, bias = d < p.DK ? p.dt_bias[h * p.DK + d] : 0.f;
+#pragma unroll
+        for (int j = 0; j < TPG; j++) {
+            const int t = grp * TPG + j;
+            pre[j] = d < p.DK && t < nv ? p.z[(tb + t) * p.z_ld + (int64_t)h * p.DK + d] : 0.f;
+        }
+#pragma unroll
+        for (int j = 0; j < TPG; j++) pre[j] = d < p.DK && grp * TPG + j < nv ? A * lr_softplus(pre[j] + bias) : 0.f;
+#pragma unroll
+        for (int j = 1; j < TPG; j++) pre[j] += pre[j - 1];
+        aux[grp * DKP + d] = pre[TPG - 1];
+        if (tid < C) be[tid] = tid < nv ? lr_sigmoid(p.beta[(tb + tid) * p.beta_ld + h]) : 0.f;
+        __syncthreads();
+        float off = 0.f;
+        for (int j = 0; j < grp; j++) off += aux[j * DKP + d];
+#pragma unroll
+        for (int j = 0; j < TPG; j++) bs[(grp * TPG + j) * LQ + d] = off + pre[j];
+    }
+    for (int i = tid; i < 2 * C * LA; i += NT) As[i] = 0.f;      // (what lies above the diagonals stays zero)
+    __syncthreads();
+    // ---- A (s <= t) and M (s < t): 240 pairs of the two diagonal blocks, one per thread; the other 16 threads take A's diagonal ----
+    if (tid < 240) {
+        const int half = tid >= 120, x = tid - 120 * half;
+        int t = (int)((sqrtf(8.f * (float)x + 1.f) - 1.f) * 0.5f);
+        if ((t + 1) * (t + 2) / 2 <= x) t++;
+        if (t * (t + 1) / 2 > x) t--;
+        const int s = x - t * (t + 1) / 2, tr = (16 * half + t + 1) * LQ, sr = (16 * half + s) * LQ;
+        f32x4 aq = f32x4{0.f, 0.f, 0.f, 0.f}, ak = aq;
+#pragma unroll 2
+        for (int d = 0; d < DKP; d += 4) {
+            const f32x4 q4 = *(const f32x4*)(qs + tr + d), k4 = *(const f32x4*)(ks + tr + d), k2 = *(const f32x4*)(ks + sr + d);
+            const f32x4 bt = *(const f32x4*)(bs + tr + d), b2 = *(const f32x4*)(bs + sr + d);
+#pragma unroll
+            for (int r = 0; r < 4; r++) { const float e = ex2(bt[r] - b2[r]) * k2[r]; aq[r] = fmaf(q4[r], e, aq[r]); ak[r] = fmaf(k4[r], e, ak[r]); }
+        }
+        const int at = (16 * half + t + 1) * LA + 16 * half + s;
+        As[at] = (aq[0] + aq[1]) + (aq[2] + aq[3]);
+        Ms[at] = (ak[0] + ak[1]) + (ak[2] + ak[3]);
+    } else {
+#pragma unroll
+        for (int i = 0; i < 2; i++) {
+            const int t = tid - 240 + 16 * i;
+            f32x4 a = f32x4{0.f, 0.f, 0.f, 0.f};
+            for (int d = 0; d < DKP; d += 4) a += *(const f32x4*)(qs + t * LQ + d) * *(const f32x4*)(ks + t * LQ + d);
+            As[t * LA + t] = (a[0] + a[1]) + (a[2] + a[3]);
+        }
+    }
+    if (wave < 2) {                                              // tokens 16..31 against 0..15: wave 0 A, wave 1 M
+        const float* x = wave == 0 ? qs : ks;
+        f32x4 acc = f32x4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll 2
+        for (int i = 0; i < NK; i++) {
+            const int c = 16 * i + 4 * fg;
+            const f32x4 ref = *(const f32x4*)(bs + 15 * LQ + c);
+            const f32x4 a = *(const f32x4*)(x + (16 + fr) * LQ + c), b = *(const f32x4*)(ks + fr * LQ + c);
+            const f32x4 ba = *(const f32x4*)(bs + (16 + fr) * LQ + c), bb = *(const f32x4*)(bs + fr * LQ + c);
+#pragma unroll
+            for (int r = 0; r < 4; r++) acc = mfma_f32(a[r] * ex2(ba[r] - ref[r]), b[r] * ex2(ref[r] - bb[r]), acc);
+        }
+        float* dst = wave == 0 ? As : Ms;
+#pragma unroll
+        for (int r = 0; r < 4; r++) dst[(16 + 4 * fg + r) * LA + fr] = acc[r];
+    }
+    __syncthreads();
+    float* ws = p.ws + (delta_chunk(p, seq, blockIdx.z) * p.H + h) * delta_ws_floats(DKP);
+    if (wave == 0) {
+        // T: a column of a diagonal block's inverse per lane (lanes 0..31), then the block below
+        float x[16];
+        const int blk = (lane >> 4) & 1, col = lane & 15;
+        const float* mr = Ms + 16 * blk * LA + 16 * blk;
+#pragma unroll
+        for (int t = 0; t < 16; t++) {
+            float a = 0.f;
+#pragma unroll
+            for (int s = 0; s < t; s++) a = fmaf(mr[t * LA + s], x[s], a);
+            x[t] = t == col ? 1.0f : (t < col ? 0.f : -be[16 * blk + t] * a);
+        }
+        f32x4 a21 = *(const f32x4*)(Ms + (16 + fr) * LA + 4 * fg) * be[16 + fr];        // beta M, block below the diagonal, as an A operand
+        asm volatile("" : "+v"(a21));                                                  // (read before the block is written)
+        if (lane < 32)
+#pragma unroll
+            for (int t = 0; t < 16; t++) Ms[(16 * blk + t) * LA + 16 * blk + col] = x[t];
+        asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");
+        f32x4 y = f32x4{0.f, 0.f, 0.f, 0.f}, w = y;
+#pragma unroll
+        for (int r = 0; r < 4; r++) y = mfma_f32(a21[r], Ms[(4 * fg + r) * LA + fr], y);
+        const f32x4 a22 = *(const f32x4*)(Ms + (16 + fr) * LA + 16 + 4 * fg);
+#pragma unroll
+        for (int r = 0; r < 4; r++) w = mfma_f32(a22[r], y[r], w);
+#pragma unroll
+        for (int r = 0; r < 4; r++) Ms[(16 + 4 * fg + r) * LA + fr] = -w[r];
+    } else {
+        // (K e^{b_end - b})^T and e^{b_end}; 32 tokens of a channel side by side
+        float* kt = ws + 2 * C * DKP;
+#pragma unroll 2
+        for (int i = tid - 64; i < C * DKP; i += NT - 64) {
+            const int t = i & 31, d = i >> 5;
+            kt[d * C + t] = ks[t * LQ + d] * ex2(bs[31 * LQ + d] - bs[t * LQ + d]);
+        }
+        for (int d = tid - 64; d < DKP; d += NT - 64) ws[3 * C * DKP + d] = ex2(bs[31 * LQ + d]);
+    }
+    __syncthreads();
+#pragma unroll 4
+    for (int i = tid; i < C * DKP / 4; i += NT) {                // q e^b, k e^b in place
+        const int t = i / (DKP / 4), d = i % (DKP / 4) * 4;
+        const f32x4 b = *(const f32x4*)(bs + t * LQ + d);
+        f32x4 q = *(const f32x4*)(qs + t * LQ + d), k = *(const f32x4*)(ks + t * LQ + d);
+#pragma unroll
+        for (int r = 0; r < 4; r++) { const float e = ex2(b[r]); q[r] *= e; k[r] *= e; }
+        *(f32x4*)(qs + t * LQ + d) = q;
+        *(f32x4*)(ks + t * LQ + d) = k;
+    }
+    // A operands of T and A: blocks (0,0), (1,0), (1,1); the columns of T carry beta
+    f32x4 ta[3], aa[3];
+#pragma unroll
+    for (int x = 0; x < 3; x++) {
+        const int row = 16 * (x > 0) + fr, c = 16 * (x > 1) + 4 * fg;
+        ta[x] = *(const f32x4*)(Ms + row * LA + c) * *(const f32x4*)(be + c);
+        aa[x] = *(const f32x4*)(As + row * LA + c);
+    }
+    __syncthreads();
+    for (int i = wave; i < NK; i += 4) {                         // 16 key channels: -W and Q'
+        const int c = 16 * i + fr;
+        f32x4 w[2], q[2], k0, k1;
+#pragma unroll
+        for (int r = 0; r < 4; r++) {
+            k0[r] = -ks[(4 * fg + r) * LQ + c]; k1[r] = -ks[(16 + 4 * fg + r) * LQ + c];
+            q[0][r] = qs[(4 * fg + r) * LQ + c]; q[1][r] = qs[(16 + 4 * fg + r) * LQ + c];
+            w[0][r] = 0.f; w[1][r] = 0.f;
+        }
+#pragma unroll
+        for (int r = 0; r < 4; r++) { w[0] = mfma_f32(ta[0][r], k0[r], w[0]); w[1] = mfma_f32(ta[1][r], k0[r], w[1]); }
+#pragma unroll
+        for (int r = 0; r < 4; r++) w[1] = mfma_f32(ta[2][r], k1[r], w[1]);
+#pragma unroll
+        for (int r = 0; r < 4; r++) { q[0] = mfma_f32(aa[0][r], w[0][r], q[0]); q[1] = mfma_f32(aa[1][r], w[0][r], q[1]); }
+#pragma unroll
+        for (int r = 0; r < 4; r++) q[1] = mfma_f32(aa[2][r], w[1][r], q[1]);
+#pragma unroll
+        for (int tt = 0; tt < 2; tt++)
+#pragma unroll
+            for (int r = 0; r < 4; r++) {
+                const int t = 16 * tt + 4 * fg + r;
+                ws[t * DKP + c] = w[tt][r];
+                ws[(C + t) * DKP + c] = q[tt][r];
+            }
+    }
+    const int nvb = (p.DV + 15) >> 4;
+    for (int i = wave; i < nvb; i += 4) {                        // 16 value channels: U0 and O0
+        const int c = 16 * i + fr;
+        const bool live = c < p.DV;
+        float* vb = p.v + tb * p.ld + (int64_t)h * p.DV + c;
+        f32x4 v0, v1, u[2], o[2];
+#pragma unroll
+        for (int r = 0; r < 4; r++) {
+            v0[r] = live && 4 * fg + r < nv ? vb[(4 * fg + r) * p.ld] : 0.f;
+            v1[r] = live && 16 + 4 * fg + r < nv ? vb[(16 + 4 * fg + r) * p.ld] : 0.f;
+            u[0][r] = u[1][r] = o[0][r] = o[1][r] = 0.f;
+        }
+#pragma unroll
+        for (int r = 0; r < 4; r++) { u[0] = mfma_f32(ta[0][r], v0[r], u[0]); u[1] = mfma_f32(ta[1][r], v0[r], u[1]); }
+#pragma unroll
+        for (int r = 0; r < 4; r++) u[1] = mfma_f32(ta[2][r], v1[r], u[1]);
+#pragma unroll
+        for (int r = 0; r < 4; r++) { o[0] = mfma_f32(aa[0][r], u[0][r], o[0]); o[1] = mfma_f32(aa[1][r], u[0][r], o[1]); }
+#pragma unroll
+        for (int r = 0; r < 4; r++) o[1] = mfma_f32(aa[2][r], u[1][r], o[1]);
+        float* ob = p.o + tb * p.o_ld + (int64_t)h * p.DV + c;
+#pragma unroll
+        for (int tt = 0; tt < 2; tt++)
+#pragma unroll
+            for (int r = 0; r < 4; r++) {
+                const int t = 16 * tt + 4 * fg + r;
+                if (live && t < nv) { vb[t * p.ld] = u[tt][r]; ob[t * p.o_ld] = o[tt][r]; }
+            }
+    }
+}
+
+// ------------------------------------------------------------------------------------------
+// scan: grid (heads, sequences, slices of 16 NW value columns); wave w owns 16 columns and keeps their DK x 16 state in accumulators.
+// The next chunk's operands are on their way to registers while the current one's are used from LDS.
+// ------------------------------------------------------------------------------------------
+template <int NK> constexpr int delta_scan_lds_bytes() { return 4 * (2 * DELTA_C * (NK * 16 + 4) + NK * 16 * 36 + NK * 16); }
+
+template <int NK, int NW>
+__global__ __launch_bounds__(NW * 64, NK > 8 ? 1 : (NW == 8 ? 4 : 3)) void delta_scan_kernel(DeltaArgs p) {
+    constexpr int C = DELTA_C, DKP = NK * 16, LQ = DKP + 4, LK = 36, NT = NW * 64;
+    const int h = blockIdx.x, seq = blockIdx.y;
+    const int n = p.seq_len[seq];
+    if (n < p.len_lo || n > p.len_hi) return;
+    extern __shared__ __attribute__((aligned(16))) float dl_sm[];
+    float* wl = dl_sm;                   // [C][LQ]   -W
+    float* ql = wl + C * LQ;             // [C][LQ]   Q'
+    float* kl = ql + C * LQ;             // [DKP][LK] (K e^{b_end - b})^T
+    float* dl = kl + DKP * LK;           // [DKP]     e^{b_end}
+    const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6);
+    const int fr = lane & 15, fg = lane >> 4;
+    const int col = (blockIdx.z * NW + wave) * 16 + fr;
+    const bool live = col < p.DV, slive = col < p.DVp;
+    const int64_t tok0 = p.seq_tok_start[seq];
+    const bool fresh = p.seq_pos[seq] == 0;
+    float* st = p.state + (int64_t)p.seq_slot[seq] * p.slot_stride + (int64_t)h * p.DK * p.DVp;
+    const int so = 4 * fg * p.DVp + col;
+    f32x4 S[NK];
+#pragma unroll
+    for (int i = 0; i < NK; i++)
+#pragma unroll
+        for (int r = 0; r < 4; r++) S[i][r] = !fresh && slive && 16 * i + 4 * fg + r < p.DK ? (st + (16 * i + r) * p.DVp)[so] : 0.f;
+    constexpr int E = 3 * C * DKP / 4, NL = E / NT;              // 16-byte pieces of a chunk's operands, per thread
+    static_assert(E % NT == 0 && NT >= DKP, "whole pieces, one decay per thread");
+    const int64_t stride = p.H * delta_ws_floats(DKP);
+    const float* src = p.ws + (delta_chunk(p, seq, 0) * p.H + h) * delta_ws_floats(DKP);
+    f32x4 rg[NL], un[2], on[2];
+    float rd = 0.f;
+    const float* vb = p.v + tok0 * p.ld + (int64_t)h * p.DV + col;
+    float* ob = p.o + tok0 * p.o_ld + (int64_t)h * p.DV + col;
+    auto fetch = [&](int c0) {
+#pragma unroll
+        for (int i = 0; i < NL; i++) rg[i] = *(const f32x4*)(src + (tid + i * NT) * 4);
+        if (tid < DKP) rd = src[3 * C * DKP + tid];
+        src += stride;
+#pragma unroll
+        for (int tt = 0; tt < 2; tt++)
+#pragma unroll
+            for (int r = 0; r < 4; r++) {
+                const int t = c0 + 16 * tt + 4 * fg + r;
+                const bool ok = live && t < n;
+                un[tt][r] = ok ? vb[t * p.ld] : 0.f;
+                on[tt][r] = ok ? ob[t * p.o_ld] : 0.f;
+            }
+    };
+    fetch(0);
+    for (int c0 = 0; c0 < n; c0 += C) {
+        __syncthreads();                                         // the previous chunk's readers are done
+#pragma unroll
+        for (int i = 0; i < NL; i++) {
+            const int e = tid + i * NT;                          // 16-byte piece
+            if (e < 2 * C * DKP / 4) { const int row = e / (DKP / 4), d = e % (DKP / 4) * 4; *(f32x4*)(wl + row * LQ + d) = rg[i]; }
+            else { const int x = e - 2 * C * DKP / 4; *(f32x4*)(kl + (x >> 3) * LK + (x & 7) * 4) = rg[i]; }
+        }
+        if (tid < DKP) dl[tid] = rd;
+        f32x4 u[2] = {un[0], un[1]}, o[2] = {on[0], on[1]};
+        __syncthreads();
+        if (c0 + C < n) fetch(c0 + C);
+#pragma unroll
+        for (int i = 0; i < NK; i++) {
+            f32x4 a[4];
+#pragma unroll
+            for (int tt = 0; tt < 2; tt++) {
+                a[tt] = *(const f32x4*)(wl + (16 * tt + fr) * LQ + 16 * i + 4 * fg);
+                a[2 + tt] = *(const f32x4*)(ql + (16 * tt + fr) * LQ + 16 * i + 4 * fg);
+            }
+#pragma unroll
+            for (int r = 0; r < 4; r++) {
+                u[0] = mfma_f32(a[0][r], S[i][r], u[0]); u[1] = mfma_f32(a[1][r], S[i][r], u[1]);
+                o[0] = mfma_f32(a[2][r], S[i][r], o[0]); o[1] = mfma_f32(a[3][r], S[i][r], o[1]);
+            }
+        }
+#pragma unroll
+        for (int tt = 0; tt < 2; tt++)
+#pragma unroll
+            for (int r = 0; r < 4; r++) {
+                const int t = c0 + 16 * tt + 4 * fg + r;
+                if (live && t < n) ob[t * p.o_ld] = o[tt][r];
+            }
+#pragma unroll
+        for (int i = 0; i < NK; i++) S[i] *= *(const f32x4*)(dl + 16 * i + 4 * fg);
+#pragma unroll
+        for (int sb = 0; sb < 2; sb++)
+#pragma unroll
+            for (int i = 0; i < NK; i++) {
+                const f32x4 a = *(const f32x4*)(kl + (16 * i + fr) * LK + 16 * sb + 4 * fg);
+#pragma unroll
+                for (int r = 0; r < 4; r++) S[i] = mfma_f32(a[r], u[sb][r], S[i]);
+            }
+    }
+    int so_end = so;
+    asm volatile("" : "+v"(so_end));                             // (or the addresses of the first loads are kept in registers all along)
+#pragma unroll
+    for (int i = 0; i < NK; i++)
+#pragma unroll
+        for (int r = 0; r < 4; r++)
+            if (slive && 16 * i + 4 * fg + r < p.DK) (st + (16 * i + r) * p.DVp)[so_end] = S[i][r];
+}
+
+// ------------------------------------------------------------------------------------------
+// token by token.  grid (H, sequences), 512 threads: tv threads side by side on a state row (4 columns each), 512 / tv rows at a time.
+// With S' = diag(a) S both S'^T k and S'^T q come from one pass over the state: o = S'^T q + (k . q) u.
+// ------------------------------------------------------------------------------------------
+static inline int delta_step_lds_bytes(int DK, int DVp, int ranks) {
+    int tv = 1;
+    while (tv < DVp / 4) tv <<= 1;
+    const int nred = tv >= 64 ? LR_STEP_THREADS / tv : LR_STEP_THREADS / 64;
+    return 4 * (3 * ((DK + 3) & ~3) + 2 * DVp + 2 * nred * DVp + ranks);
+}
+template <typename WT> __device__ __forceinline__ float delta_dot16(const WT* w, const float* x);       // 16 bytes of weights
+template <> __device__ __forceinline__ float delta_dot16<float>(const float* w, const float* x) {
+    const f32x4 a = *(const f32x4*)w, b = *(const f32x4*)x;
+    return fmaf(a[3], b[3], fmaf(a[2], b[2], fmaf(a[1], b[1], a[0] * b[0])));
+}
+template <> __device__ __forceinline__ float delta_dot16<bf16_t>(const bf16_t* w, const float* x) {
+    const bf16x8 a = *(const bf16x8*)w;
+    float s = 0.f;
+#pragma unroll
+    for (int i = 0; i < 8; i++) s = fmaf((float)a[i], x[i], s);
+    return s;
+}
+
+template <bool FUSED, int ROWS, typename ActT>           // ROWS: state rows a thread keeps in registers; ActT: type of `out` and of a2 / g2
+__global__ __launch_bounds__(LR_STEP_THREADS, ROWS <= 8 ? 4 : 2) void delta_step_kernel(DeltaArgs p) {
+    constexpr int NT = LR_STEP_THREADS, NW = NT / 64;
+    const int h = blockIdx.x, seq = blockIdx.y, tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
+    const int n = p.seq_len[seq];
+    if (n < p.len_lo || n > p.len_hi) return;
+    extern __shared__ __attribute__((aligned(16))) float dl_sm[];
+    const int DK4 = (p.DK + 3) & ~3;
+    float* sq = dl_sm;                   // [DK]
+    float* sk = sq + DK4;                // [DK]
+    float* sa = sk + DK4;                // [DK]   decays
+    float* sv = sa + DK4;                // [DVp]
+    float* sg = sv + p.DVp;              // [DVp]  output gates (FUSED)
+    const int nv4 = p.DVp >> 2;
+    int tv = 1;
+    while (tv < nv4) tv <<= 1;           // host: nv4 <= NT
+    const int rg = tid / tv, tc = tid - rg * tv, RG = NT / tv, NRED = tv >= 64 ? RG : NW;
+    float* red = sg + p.DVp;             // [NRED][2][DVp]
+    float* lr = red + 2 * NRED * p.DVp;  // [a_rkp + g_rkp] (FUSED)
+    __shared__ float s_red[NW], s_sum[3];
+    const bool live = tc < nv4;
+    const int t0 = p.seq_tok_start[seq], pos0 = p.seq_pos[seq], slot = p.seq_slot[seq];
+    const int g = h / (p.H / p.G);
+    float* st = p.state + (int64_t)slot * p.slot_stride + (int64_t)h * p.DK * p.DVp;
+    int so = rg * p.DVp + 4 * tc;        // this thread's place in a pass of RG rows
+    const int pass = RG * p.DVp;
+    f32x4 s[ROWS];                       // the first ROWS rows of this thread, fetched before anything else is known
+#pragma unroll
+    for (int i = 0; i < ROWS; i++) {
+        const bool ok = live && rg + i * RG < p.DK;
+        const f32x4 x = *(const f32x4*)(st + (ok ? i * pass + so : 0));
+#pragma unroll
+        for (int r = 0; r < 4; r++) s[i][r] = ok && pos0 > 0 ? x[r] : 0.f;
+    }
+    asm volatile("" : "+v"(so));         // (or the addresses of these loads are kept in registers for the stores)
+    for (int i = tid; i < p.DVp; i += NT) { sv[i] = 0.f; sg[i] = 0.f; }
+    __syncthreads();
+    const float ea = expf(p.a_log[h]);
+    for (int it = 0; it < n; it++) {
+        const int64_t t = t0 + it;
+        if constexpr (FUSED) {
+            // causal convolution + silu of this head's channels (n == 1)
+            const float* rw = p.raw + t * p.raw_ld;
+            float* ring = p.ring + (int64_t)slot * p.ring_slot_stride;
+            const int KD = p.G * p.DK;
+            for (int i = tid; i < 2 * p.DK + p.DV; i += NT) {
+                const int c = i < p.DK ? g * p.DK + i : (i < 2 * p.DK ? KD + g * p.DK + i - p.DK : 2 * KD + h * p.DV + i - 2 * p.DK);
+                const float cur = rw[c];
+                float acc = 0.f;
+                for (int b = p.taps - 1; b >= 1; b--)
+                    if (pos0 - b >= 0) acc = fmaf(ring[(int64_t)((pos0 - b) % p.taps) * p.channels + c], p.conv_w[(int64_t)c * p.taps + p.taps - 1 - b], acc);
+                acc = fmaf(cur, p.conv_w[(int64_t)c * p.taps + p.taps - 1], acc);
+                ring[(int64_t)(pos0 % p.taps) * p.channels + c] = cur;      // (heads of a group write the same values; nobody reads this row now)
+                const float y = lr_silu(acc);
+                if (i < p.DK) sq[i] = y;
+                else if (i < 2 * p.DK) sk[i - p.DK] = y;
+                else sv[i - 2 * p.DK] = y;
+            }
+            for (int i = tid; i < p.a_rkp + p.g_rkp; i += NT) {
+                const int j = i - p.a_rkp;
+                lr[i] = j < 0 ? (i < p.a_rank ? p.a1[t * p.lr_ld + i] : 0.f) : (j < p.g_rank ? p.g1[t * p.lr_ld + j] : 0.f);
+            }
+            __syncthreads();
+            // decay and gate projections: four lanes per output
+            constexpr int CH = 16 / (int)sizeof(ActT);
+            for (int i = tid >> 2; i < p.DK + p.DV; i += NT / 4) {
+                const bool dec = i < p.DK;
+                const int rkp = dec ? p.a_rkp : p.g_rkp;
+                const ActT* w = dec ? (const ActT*)p.a2 + (int64_t)(h * p.DK + i) * rkp : (const ActT*)p.g2 + (int64_t)(h * p.DV + i - p.DK) * rkp;
+                const float* x = dec ? lr : lr + p.a_rkp;
+                float a = 0.f;
+                for (int e = (tid & 3) * CH; e < rkp; e += 4 * CH) a += delta_dot16<ActT>(w + e, x + e);
+                a += __shfl_xor(a, 1, 64);
+                a += __shfl_xor(a, 2, 64);
+                if ((tid & 3) == 0) {
+                    if (dec) sa[i] = expf(-ea * lr_softplus(a + p.dt_bias[h * p.DK + i]));
+                    else sg[i - p.DK] = lr_sigmoid(a);
+                }
+            }
+        } else {
+            for (int i = tid; i < p.DK; i += NT) {
+                sq[i] = p.q[t * p.ld + (int64_t)g * p.DK + i];
+                sk[i] = p.k[t * p.ld + (int64_t)g * p.DK + i];
+                sa[i] = expf(-ea * lr_softplus(p.z[t * p.z_ld + (int64_t)h * p.DK + i] + p.dt_bias[h * p.DK + i]));
+            }
+            for (int i = tid; i < p.DV; i += NT) sv[i] = p.v[t * p.ld + (int64_t)h * p.DV + i];
+        }
+        __syncthreads();
+        if (wave < 3) {                  // q . q, k . k, k . q
+            const float *x = wave == 1 ? sk : sq, *y = wave == 0 ? sq : sk;
+            float a = 0.f;
+            for (int i = lane; i < p.DK; i += 64) a = fmaf(x[i], y[i], a);
+            a = wave_sum(a);
+            if (lane == 0) s_sum[wave] = a;
+        }
+        __syncthreads();
+        const float iq = p.q_scale / sqrtf(s_sum[0] + DELTA_UNIT_EPS), ik = 1.0f / sqrtf(s_sum[1] + DELTA_UNIT_EPS), kq = s_sum[2] * iq * ik;
+        const float beta = lr_sigmoid(p.beta[t * p.beta_ld + h]);
+        f32x4 ra = f32x4{0.f, 0.f, 0.f, 0.f}, pa = ra;      // S'^T k, S'^T q
+#pragma unroll
+        for (int i = 0; i < ROWS; i++) {
+            const int row = rg + i * RG;
+            const bool ok = live && row < p.DK;
+            const int rr = ok ? row : 0;
+            const float al = sa[rr], kk = ok ? sk[rr] : 0.f, qq = ok ? sq[rr] : 0.f;
+#pragma unroll
+            for (int r = 0; r < 4; r++) { s[i][r] *= al; ra[r] = fmaf(kk, s[i][r], ra[r]); pa[r] = fmaf(qq, s[i][r], pa[r]); }
+        }
+#pragma unroll 1
+        for (int row = rg + ROWS * RG; live && row < p.DK; row += RG) {     // (a state larger than the registers: streamed)
+            f32x4 w = f32x4{0.f, 0.f, 0.f, 0.f};
+            if (pos0 + it > 0) w = *(const f32x4*)(st + (int64_t)row * p.DVp + 4 * tc);
+            w *= sa[row];
+            ra += sk[row] * w; pa += sq[row] * w;
+        }
+        for (int o = tv; o < 64; o <<= 1)
+#pragma unroll
+            for (int r = 0; r < 4; r++) { ra[r] += __shfl_xor(ra[r], o, 64); pa[r] += __shfl_xor(pa[r], o, 64); }
+        if (live && (tv >= 64 || lane < tv)) {
+            float* d = red + (int64_t)(tv >= 64 ? rg : wave) * 2 * p.DVp + 4 * tc;
+            *(f32x4*)d = ra;
+            *(f32x4*)(d + p.DVp) = pa;
+        }
+        __syncthreads();
+        f32x4 u = f32x4{0.f, 0.f, 0.f, 0.f}, ov = u;
+        if (live) {
+            ra = u; pa = u;
+#pragma unroll 4
+            for (int r = 0; r < NRED; r++) { ra += *(const f32x4*)(red + (int64_t)r * 2 * p.DVp + 4 * tc); pa += *(const f32x4*)(red + (int64_t)r * 2 * p.DVp + p.DVp + 4 * tc); }
+            u = beta * (*(const f32x4*)(sv + 4 * tc) - ra * ik);
+            ov = pa * iq + kq * u;
+        }
+#pragma unroll
+        for (int i = 0; i < ROWS; i++) {
+            const int row = rg + i * RG;
+            const bool ok = live && row < p.DK;
+            const float kk = ok ? sk[ok ? row : 0] * ik : 0.f;
+#pragma unroll
+            for (int r = 0; r < 4; r++) s[i][r] = fmaf(kk, u[r], s[i][r]);
+            if (ok && it == n - 1) *(f32x4*)(st + i * pass + so) = s[i];
+        }
+#pragma unroll 1
+        for (int row = rg + ROWS * RG; live && row < p.DK; row += RG) {
+            float* sr = st + (int64_t)row * p.DVp + 4 * tc;
+            f32x4 w = f32x4{0.f, 0.f, 0.f, 0.f};
+            if (pos0 + it > 0) w = *(const f32x4*)sr;
+            *(f32x4*)sr = w * sa[row] + sk[row] * ik * u;
+        }
+        if constexpr (FUSED) {
+            // (columns beyond DV: v, S and hence o are zero)
+            float ss = rg == 0 ? (ov[0] * ov[0] + ov[1] * ov[1]) + (ov[2] * ov[2] + ov[3] * ov[3]) : 0.f;
+            ss = wave_sum(ss);
+            if (lane == 0) s_red[wave] = ss;
+            __syncthreads();
+            float tot = 0.f;
+#pragma unroll
+            for (int i = 0; i < NW; i++) tot += s_red[i];
+            const float inv = 1.0f / sqrtf(tot / (float)p.DV + p.eps);
+            if (live && rg == 0)
+#pragma unroll
+                for (int r = 0; r < 4; r++)
+                    if (4 * tc + r < p.DV)
+                        ActIO<ActT>::st((ActT*)p.out + act_index<ActT>(t, (int64_t)h * p.DV + 4 * tc + r, p.out_ld), ov[r] * inv * p.norm_w[4 * tc + r] * sg[4 * tc + r]);
+        } else if (live && rg == 0) {
+#pragma unroll
+            for (int r = 0; r < 4; r++) if (4 * tc + r < p.DV) p.o[t * p.o_ld + (int64_t)h * p.DV + 4 * tc + r] = ov[r];
+        }
+        __syncthreads();
+    }
+}
+
+// ---- columns [0, n) and [off2, off2 + n2) of fp32 rows as the operands of two projections (padded with zeros): grid (tokens) ----
+struct PackArgs { const float* src; int64_t ld; int n1, np1, n2, np2, off2; void *d1, *d2; };
+template <typename ActT>
+__global__ __launch_bounds__(64) void pack_rows_kernel(PackArgs p) {
+    const int64_t t = blockIdx.x;
+    const float* x = p.src + t * p.ld;
+    for (int i = threadIdx.x * 4; i < p.np1 + p.np2; i += 256) {
+        const bool a = i < p.np1;
+        const int c = a ? i : i - p.np1, n = a ? p.n1 : p.n2;
+        f32x4 v;
+#pragma unroll
+        for (int r = 0; r < 4; r++) v[r] = c + r < n ? x[(a ? 0 : p.off2) + c + r] : 0.f;
+        act_store4<ActT>((ActT*)(a ? p.d1 : p.d2), t, c, a ? p.np1 : p.np2, v);
+    }
+}
+
+}  // namespace nvl

@@ -303,7 +303,7 @@ __global__ __launch_bounds__(256) void norm_row_kernel(float* __restrict__ x,
 // ---------------------------------------------------------------------------------------
 // Sandwich norms: x += rms(y) * w_post completes a sublayer whose output y is normed before it joins the residual stream, and
 // the norm that opens the next sublayer follows at once: xn = rms(x) * w_next.  One launch does both (y == NULL: only the
-// second; w_next == NULL: only the first).  Rows are H floats apart, the mean runs over `width` <= H columns (the padding
+// second; w_next == NULL: only the first, or with `raw_next` xn = x, for blocks without a norm in front).  Rows are H floats apart, the mean runs over `width` <= H columns (the padding
 // columns of x, y and the weights are zero).  y may be split over `slices` partial sums (a K split of the projection).
 //   sandwich_row_kernel    : one 256-thread workgroup per row, the row in registers (decode, short batches, wide rows)
 //   sandwich_tile16_kernel : one wave per row, 16 rows per workgroup, operand blocks written whole (prefill, bf16)
@@ -317,6 +317,7 @@ struct SandwichArgs {
     const int32_t* rows_idx;  // y == NULL only: which row of x feeds output row r
     int rows, H, width;
     float eps;
+    int raw_next;             // w_next == NULL: xn = x
 };
 template <typename ActT, int MAXCH>
 __global__ __launch_bounds__(256) void sandwich_row_kernel(SandwichArgs p, ActT* __restrict__ xn) {
@@ -354,7 +355,12 @@ __global__ __launch_bounds__(256) void sandwich_row_kernel(SandwichArgs p, ActT*
             }
         }
     }
-    if (!p.w_next) return;
+    if (!p.w_next) {
+        if (p.raw_next)
+#pragma unroll
+            for (int c = 0; c < MAXCH; c++) { const int j = threadIdx.x + c * 256; if (j < H4) act_store4<ActT>(xn, r, j * 4, p.H, x[c]); }
+        return;
+    }
     ss = 0.f;
 #pragma unroll
     for (int c = 0; c < MAXCH; c++) ss += x[c][0] * x[c][0] + x[c][1] * x[c][1] + x[c][2] * x[c][2] + x[c][3] * x[c][3];
@@ -407,6 +413,16 @@ __global__ __launch_bounds__(1024) void sandwich_tile16_kernel(SandwichArgs p, b
                 }
             }
         }
+        if (!p.w_next && p.raw_next) {
+#pragma unroll
+            for (int c = 0; c < MAXCH; c++) {
+                const int j = lane + c * 64;
+                bf16x4 o;
+#pragma unroll
+                for (int k = 0; k < 4; k++) o[k] = (bf16_t)x[c][k];
+                if (j < H4) *(bf16x4*)(tile + wave * p.H + j * 4) = o;
+            }
+        }
         if (p.w_next) {
             float ss = 0.f;
 #pragma unroll
@@ -425,7 +441,7 @@ __global__ __launch_bounds__(1024) void sandwich_tile16_kernel(SandwichArgs p, b
             }
         }
     }
-    if (!p.w_next) return;
+    if (!p.w_next && !p.raw_next) return;
     __syncthreads();
     const int nkb = p.H >> 5, lr = lane & 15, lc = lane >> 4;
     if (blockIdx.x * 16 + lr < p.rows)
@@ -524,6 +540,13 @@ __global__ void swiglu_kernel(const float* __restrict__ h, ActT* __restrict__ y,
     const float g = h[r * 2 * F + f], u = h[r * 2 * F + F + f];
     ActIO<ActT>::st(y + i, (GELU ? gelu_tanh_f(g) : g / (1.0f + expf(-g))) * u);
 }
+template <typename ActT>
+__global__ void clamp_glu_kernel(const float* __restrict__ h, ActT* __restrict__ y, int64_t rows, int F, float limit, float slope) {
+    const int64_t i = (int64_t)blockIdx.x * blockDim.x + threadIdx.x;
+    if (i >= rows * F) return;
+    const int64_t r = i / F; const int f = (int)(i - r * F);
+    ActIO<ActT>::st(y + i, clamp_glu_f(h[r * 2 * F + f], h[r * 2 * F + F + f], limit, slope));
+}
 __global__ void gelu_kernel(const float* __restrict__ x, float* __restrict__ y, int64_t n) {
     const int64_t i = (int64_t)blockIdx.x * blockDim.x + threadIdx.x;
     if (i >= n) return;
@@ -567,7 +590,7 @@ __device__ __forceinline__ void argmax_merge(float& best, int& bi, float ov, int
 }
 
 __global__ __launch_bounds__(256) void argmax_partial_kernel(float* __restrict__ logits, int ld, int V,
-                                                             float logits_scaling, float* __restrict__ pval,
+                                                             float logits_scaling, float softcap, float* __restrict__ pval,
                                                              int32_t* __restrict__ pidx) {
     __shared__ float sv[4];
     __shared__ int si[4];
@@ -580,6 +603,7 @@ __global__ __launch_bounds__(256) void argmax_partial_kernel(float* __restrict__
     for (int j = c0 + threadIdx.x; j < c1; j += 256) {
         float v = row[j];
         if (logits_scaling != 0.f) { v = v / logits_scaling; row[j] = v; }
+        if (softcap != 0.f) { v = softcap * tanhf(v / softcap); row[j] = v; }
         if (v > best) { best = v; bi = j; }      // strict >, ascending j => first max per thread
     }
 #pragma unroll
@@ -608,9 +632,14 @@ __global__ __launch_bounds__(64) void argmax_final_kernel(const float* __restric
 
 // logits /= LogitsScaling (generic_model.go:472-477) for the rows a sampler reads (the argmax path folds it into
 // argmax_partial_kernel)
-__global__ void scale_rows_kernel(float* __restrict__ x, int ld, int n, float div) {
+__global__ void scale_rows_kernel(float* __restrict__ x, int ld, int n, float div, float softcap) {
     const int j = blockIdx.x * blockDim.x + threadIdx.x;
-    if (j < n) { float* p = x + (int64_t)blockIdx.y * ld + j; *p = *p / div; }
+    if (j >= n) return;
+    float* p = x + (int64_t)blockIdx.y * ld + j;
+    float v = *p;
+    if (div != 0.f) v = v / div;
+    if (softcap != 0.f) v = softcap * tanhf(v / softcap);
+    *p = v;
 }
 
 // ---------------------------------------------------------------------------------------
@@ -678,10 +707,12 @@ __global__ __launch_bounds__(256) void decode_seam_kernel(const float* __restric
                 v[c][k] = f;
             }
             *(f32x4*)(xr + j * 4) = v[c];
-            ww[c] = *(const f32x4*)(w + j * 4);
+            if (w) ww[c] = *(const f32x4*)(w + j * 4);
+            else act_store4<bf16_t>(y, r, j * 4, H, v[c]);           // no norm in front of layer 0
             if (b) bb[c] = *(const f32x4*)(b + j * 4);
         }
     }
+    if (!w) return;
     norm_row_finish<bf16_t>(v, ww, bb, b, eps, y, r, H, red, width);
 }
 

@@ -39,10 +39,11 @@ enum GemmEpi {
     EPI_QKV = 4,     // fused QKV projection epilogue (head_dim 64 / 128): bias, RoPE on Q and K (rope.go:153-205),
                      // Q -> q buffer, K and V -> their KV slabs [pos][hd]  (replaces the fp32 qkv
                      // round trip + rope_kv_kernel in prefill; Concatenate tensor.go:283-321)
+    EPI_CLAMP_GLU = 6,   // C[m, f] = g sigmoid(slope g) (u + 1), g = min(gate, limit), u = clamp(up, -limit, limit); W as for EPI_SWIGLU
     EPI_GEGLU = 5,   // C[m, f] = gelu_tanh(gate) * up   W rows interleaved as for EPI_SWIGLU
 };
 
-constexpr bool epi_glu(int epi) { return epi == 2 || epi == 5; }      // gate | up pairs in, one column out
+constexpr bool epi_glu(int epi) { return epi == 2 || epi == 5 || epi == 6; }      // gate | up pairs in, one column out
 
 struct QkvEpi {             // EPI_QKV only
     const int32_t* tok_pos;
@@ -66,6 +67,7 @@ struct GemmArgs {
     int ldc;
     const float* bias;      // [N] or NULL
     float alpha;            // EPI_RESID multiplier
+    float glu_limit, glu_slope;     // EPI_CLAMP_GLU
     int M, N, K;            // logical sizes
     const int32_t* seg;     // optional device {start,end}: rows [start,end) of A (via a_rows if set)
                             // and of C; M is then only the grid bound (MoE expert segments)
@@ -198,7 +200,10 @@ __device__ __forceinline__ void epilogue_glu4(const GemmArgs& p, int m, int f, f
     g *= rstd; u *= rstd;
     f32x4 v;
 #pragma unroll
-    for (int r = 0; r < 4; r++) v[r] = (EPI == EPI_GEGLU ? gelu_tanh_f(g[r]) : silu_f(g[r])) * u[r];
+    for (int r = 0; r < 4; r++) {
+        if constexpr (EPI == EPI_CLAMP_GLU) v[r] = clamp_glu_f(g[r], u[r], p.glu_limit, p.glu_slope);
+        else v[r] = (EPI == EPI_GEGLU ? gelu_tanh_f(g[r]) : silu_f(g[r])) * u[r];
+    }
     if constexpr (MOE) v *= p.moe_gate[m * p.moe_E + f / p.moe_I];      // routing weight of (token, expert); 0 = not routed
     act_store4<OutT>((OutT*)p.C, (int64_t)p.c_row0 + m, f, p.ldc, v);
 }
@@ -930,7 +935,7 @@ __global__ __launch_bounds__(1024) void moe_router_gate_kernel(GemmArgs p, int t
 
 // ------------------------------------------------------------------------------------------
 // fp32 kernel (parity mode): 64x64 tile, BK=16, 256 threads, 4x4 outputs per thread, k ascending.
-// EPI_SWIGLU / EPI_GEGLU are not instantiated: the f32 path keeps W1 un-interleaved and applies the
+// EPI_SWIGLU / EPI_GEGLU / EPI_CLAMP_GLU are not instantiated: the f32 path keeps W1 un-interleaved and applies the
 // activation with swiglu_kernel.
 // ------------------------------------------------------------------------------------------
 template <int EPI, typename OutT>

@@ -1,6 +1,8 @@
-// latent.h — attention over a cached low-rank latent (multi-head latent attention without a rotated part), with an optional sliding
-// window.  Per token: c_q = rms(W_dq h) * w, q = W_uq c_q; c = rms(W_dkv h) * w; per head k = W_uk c, v = W_uv c; only c is
-// cached.  The concatenated heads are multiplied by sigmoid(W_g h) before the output projection.
+// latent.h — attention over a cached low-rank latent (multi-head latent attention), with an optional sliding window and an optional
+// rotated part.  Per token: c_q = rms(W_dq h) * w, q = W_uq c_q; c = rms(W_dkv h) * w; per head k = W_uk c, v = W_uv c; only c is
+// cached.  The concatenated heads are multiplied by sigmoid(W_g h) (per channel or per head) before the output projection.
+// Rotated part (rot > 0): every head of q has `rot` more dimensions, turned by the token's position; their key is ONE vector per
+// token, shared by the heads, turned before it is cached beside c; the two scores add up.
 //
 // Two forms of the same attention, chosen per token:
 //   expanded (prompt portions): the latents of the keys the portion can see are gathered from the cache, two projections make
@@ -11,7 +13,8 @@
 // Scores, softmax and their sums are fp32; the scale is applied to the fp32 scores.
 //
 // Cache: blocks of `bs` tokens (64 | bs) named by block tables, as for K/V; a layer's part of a block is [bs][rp] latents, rp =
-// kv_rank padded to 64 (the padding is zero).  bf16: fragment-major in units of 16 tokens x 32 columns (common.h fm_index on the
+// kv_rank padded to 64, and after them [bs][rotp] rotated keys, rotp = rot padded to 32 (the padding is zero).  A layer may read
+// another layer's part (it then has no W_dkv).  bf16: fragment-major in units of 16 tokens x 32 columns (common.h fm_index on the
 // block's rows), so that a score operand is one contiguous KiB; fp32 mode: row-major.
 #pragma once
 #include "attn.h"
@@ -23,29 +26,33 @@ constexpr int LAT_SPLITS = 16;          // most workgroups the keys of a token a
 __device__ __forceinline__ float lat_sigmoid(float x) { return 1.0f / (1.0f + __expf(-x)); }
 
 struct LatentArgs {
-    int H, dim, dp, vp, qrank, qrp, kvrank, rp;   // dp / vp / qrp / rp: padded sizes
+    int H, dim, dn, dp, vp, qrank, qrp, kvrank, rp;   // dn / vp / qrp / rp: padded sizes; dp = dn + rotp: a head's columns of q
+    int rot, rotp;                                // rotated dimensions per head (0: none), padded
+    const f32x2* turn;                            // [position][rot / 2] (cos, sin)
     int window;                                   // 0: every earlier token
     float scale, eps;
-    const float* proj; int64_t proj_ld;           // [token][c_q : qrp | c : rp | gate : H * vp] of the fused input projection
+    const float* proj; int64_t proj_ld;           // [token][c_q : qrp | c : rp | rotated key : rotp | gate] of the fused input projection
+    int own;                                      // the layer makes its own latents (else: no c and rotated key columns)
+    int gate_off, gate_head;                      // first gate column; one gate per head instead of one per channel
     const float *cq_norm, *c_norm;                // padded with zeros
     void* cq;                                     // operand of W_uq: [token][qrp]
     void* cache; int64_t block_stride;            // this layer's part of block 0; elements between blocks
     int bs;
     const int32_t *blk_table, *tok_pos, *tok_tbl, *seq_tok_start, *seq_len, *seq_pos;
     int tbl_stride;
-    const float* q; int64_t q_ld;                 // [token][H * dp]
+    const float* q; int64_t q_ld;                 // [token][H * dp], per head [unrotated : dn | to be rotated : rotp]
     // expanded form
     const int32_t* kbase;                         // per sequence: its first row in the key workspace (-1: the sequence takes the absorbed form)
-    void* cg;                                     // gathered latents [rows][rp]
-    const void *kx, *vx;                          // bf16: K [rows][H * dp] and V^T [H * vp][rows_pad], both fragment-major; fp32: K, V [rows][H * .]
+    void *cg, *kr;                                // gathered latents [rows][rp] and rotated keys [rows][rotp]
+    const void *kx, *vx;                          // bf16: K [rows][H * dn] and V^T [H * vp][rows_pad], both fragment-major; fp32: K, V [rows][H * .]
     int64_t rows_pad;
     void* out; int64_t out_ld;                    // operand of W_o: [token][out_ld], head h at column h * vp
     // absorbed form
     const int32_t* abs_tok;                       // the tokens that take it
     const int32_t* abs_seq;
     int n_abs, n_split;
-    const bf16_t *ukt, *uv;                       // per head [rp][dp]; [H * vp][rp]; fragment-major
-    bf16_t* qa; int Hp;                           // [n_abs][Hp][rp], Hp = H padded to 16
+    const bf16_t *ukt, *uv;                       // per head [rp][dn]; [H * vp][rp]; fragment-major
+    bf16_t* qa; int Hp;                           // [n_abs][Hp][rp + rotp], Hp = H padded to 16
     float *part_o, *part_ml;                      // [split][n_abs][H][rp], [split][n_abs][H][2]
 };
 
@@ -53,6 +60,24 @@ struct LatentArgs {
 __host__ __device__ __forceinline__ int latent_key0(int pos0, int window) {
     const int lo = window > 0 ? pos0 - window + 1 : 0;
     return lo > 0 ? (lo & ~31) : 0;
+}
+
+// dimension i of a vector of `rot` dimensions turned by position pos: pairs (i, i + rot / 2)
+__device__ __forceinline__ float lat_turn(const LatentArgs& p, const float* x, int i, int pos) {
+    const int half = p.rot >> 1;
+    if (i >= p.rot) return 0.f;
+    const int j = i < half ? i : i - half;
+    const f32x2 cs = p.turn[(int64_t)pos * half + j];
+    const float u = x[j], v = x[j + half];
+    return i < half ? u * cs[0] - v * cs[1] : v * cs[0] + u * cs[1];
+}
+__device__ __forceinline__ float lat_gate(const LatentArgs& p, int64_t tok, int h, int col) {      // col: column of W_o's operand inside head h
+    return p.proj[tok * p.proj_ld + p.gate_off + (p.gate_head ? h : h * p.vp + col)];
+}
+__device__ __forceinline__ f32x4 lat_gate4(const LatentArgs& p, int64_t tok, int h, int col) {
+    if (!p.gate_head) return *(const f32x4*)(p.proj + tok * p.proj_ld + p.gate_off + h * p.vp + col);
+    const float g = lat_gate(p, tok, h, col);
+    return f32x4{g, g, g, g};
 }
 
 // ---- norms of the two latents; c goes to its cache row.  grid (tokens), 256 threads ----
@@ -63,16 +88,20 @@ __global__ __launch_bounds__(256) void latent_norm_kernel(LatentArgs p) {
     const float* pr = p.proj + (int64_t)t * p.proj_ld;
     float sq = 0.f, sc = 0.f;          // (the padding columns of c_q and c are zero)
     for (int i = threadIdx.x * 4; i < p.qrp; i += 1024) { const f32x4 v = *(const f32x4*)(pr + i); sq += (v[0] * v[0] + v[1] * v[1]) + (v[2] * v[2] + v[3] * v[3]); }
-    for (int i = threadIdx.x * 4; i < p.rp; i += 1024) { const f32x4 v = *(const f32x4*)(pr + p.qrp + i); sc += (v[0] * v[0] + v[1] * v[1]) + (v[2] * v[2] + v[3] * v[3]); }
+    if (p.own) for (int i = threadIdx.x * 4; i < p.rp; i += 1024) { const f32x4 v = *(const f32x4*)(pr + p.qrp + i); sc += (v[0] * v[0] + v[1] * v[1]) + (v[2] * v[2] + v[3] * v[3]); }
     sq = wave_sum(sq); sc = wave_sum(sc);
     if ((threadIdx.x & 63) == 0) { red[threadIdx.x >> 6] = sq; red[4 + (threadIdx.x >> 6)] = sc; }
     __syncthreads();
     const float rq = sqrtf((red[0] + red[1] + red[2] + red[3]) / (float)p.qrank + p.eps), rc = sqrtf((red[4] + red[5] + red[6] + red[7]) / (float)p.kvrank + p.eps);
     for (int i = threadIdx.x * 4; i < p.qrp; i += 1024) act_store4<ActT>((ActT*)p.cq, t, i, p.qrp, *(const f32x4*)(pr + i) / rq * *(const f32x4*)(p.cq_norm + i));
+    if (!p.own) return;
     int blk, row;
-    kv_locate(p.blk_table, p.tok_tbl[t], p.tok_pos[t], p.bs, blk, row);
+    const int pos = p.tok_pos[t];
+    kv_locate(p.blk_table, p.tok_tbl[t], pos, p.bs, blk, row);
     ActT* c = (ActT*)p.cache + (int64_t)blk * p.block_stride;
     for (int i = threadIdx.x * 4; i < p.rp; i += 1024) act_store4<ActT>(c, row, i, p.rp, *(const f32x4*)(pr + p.qrp + i) / rc * *(const f32x4*)(p.c_norm + i));
+    ActT* kr = c + (int64_t)p.bs * p.rp;
+    for (int i = threadIdx.x; i < p.rotp; i += 256) ActIO<ActT>::st(kr + act_index<ActT>(row, i, p.rotp), lat_turn(p, pr + p.qrp + p.rp, i, pos));
 }
 
 // ---- gather the latents a portion's keys need into contiguous rows: 32 rows (one unit of either layout) per workgroup ----
@@ -88,6 +117,10 @@ __global__ __launch_bounds__(256) void latent_gather_kernel(LatentArgs p) {
     const char* src = (const char*)((const ActT*)p.cache + (int64_t)blk * p.block_stride + (int64_t)row * p.rp);
     char* dst = (char*)((ActT*)p.cg + (int64_t)(p.kbase[seq] + r0) * p.rp);
     for (int64_t i = threadIdx.x * 16; i < (int64_t)32 * p.rp * (int)sizeof(ActT); i += 256 * 16) *(f32x4*)(dst + i) = *(const f32x4*)(src + i);
+    if (!p.rot) return;
+    const char* rs = (const char*)((const ActT*)p.cache + (int64_t)blk * p.block_stride + (int64_t)p.bs * p.rp + (int64_t)row * p.rotp);
+    char* rd = (char*)((ActT*)p.kr + (int64_t)(p.kbase[seq] + r0) * p.rotp);
+    for (int i = threadIdx.x * 16; i < 32 * p.rotp * (int)sizeof(ActT); i += 256 * 16) *(f32x4*)(rd + i) = *(const f32x4*)(rs + i);
 }
 
 // ------------------------------------------------------------------------------------------
@@ -110,11 +143,16 @@ struct LatentRows {            // the query rows of one wave
     __device__ __forceinline__ int key_lo(const LatentArgs& p) const { const int lo = p.window > 0 ? first - p.window + 1 : 0; return lo > k0 ? lo - k0 : 0; }
 };
 template <int KS>
-__device__ __forceinline__ void latent_load_q(const LatentArgs& p, int64_t tok, int h, int fg, bf16x8 (&qf)[KS]) {
+__device__ __forceinline__ void latent_load_q(const LatentArgs& p, int64_t tok, int pos, int h, int fg, bf16x8 (&qf)[KS]) {
     const float* qp = p.q + tok * p.q_ld + h * p.dp;
     const float sg = p.scale < 0.f ? -1.f : 1.f;
 #pragma unroll
     for (int ks = 0; ks < KS; ks++) {
+        if (ks * 32 >= p.dn) {            // (uniform) the rotated part
+#pragma unroll
+            for (int e = 0; e < 8; e++) qf[ks][e] = (bf16_t)(lat_turn(p, qp + p.dn, ks * 32 - p.dn + fg * 8 + e, pos) * sg);
+            continue;
+        }
         const f32x4 a = *(const f32x4*)(qp + ks * 32 + fg * 8), b = *(const f32x4*)(qp + ks * 32 + fg * 8 + 4);
 #pragma unroll
         for (int e = 0; e < 4; e++) { qf[ks][e] = (bf16_t)(a[e] * sg); qf[ks][4 + e] = (bf16_t)(b[e] * sg); }
@@ -156,10 +194,9 @@ __device__ __forceinline__ bf16x8 latent_pack_p(const f32x4& a, const f32x4& b) 
 }
 template <int DT>
 __device__ __forceinline__ void latent_store_o(const LatentArgs& p, int64_t tok, int h, int fg, float inv, const f32x4 (&o)[DT]) {
-    const float* gt = p.proj + tok * p.proj_ld + p.qrp + p.rp + h * p.vp;
 #pragma unroll
     for (int d = 0; d < DT; d++) {
-        const f32x4 g = *(const f32x4*)(gt + 16 * d + 4 * fg);
+        const f32x4 g = lat_gate4(p, tok, h, 16 * d + 4 * fg);
         f32x4 v = o[d] * inv;
 #pragma unroll
         for (int r = 0; r < 4; r++) v[r] *= lat_sigmoid(g[r]);
@@ -189,7 +226,7 @@ __global__ __launch_bounds__(512, (KS <= 2 && DT <= 4) ? 4 : 2) void latent_pref
         bool ok;
         const int r = w.row(i, fq, ok);
         qpos[i] = w.pos0 + r;
-        latent_load_q<KS>(p, w.tok0 + r, h, fg, qf[i]);
+        latent_load_q<KS>(p, w.tok0 + r, qpos[i], h, fg, qf[i]);
     }
 #pragma unroll
     for (int i = 0; i < TQ; i++)
@@ -203,7 +240,8 @@ __global__ __launch_bounds__(512, (KS <= 2 && DT <= 4) ? 4 : 2) void latent_pref
     const int wt0 = w_live ? w.key_lo(p) >> 6 : n_kt, wt1 = w_live ? ((w.last - w.k0) >> 6) + 1 : 0;
     const int full_lo = (p.window > 0 ? w.last - p.window + 1 : 0) - w.k0, full_hi = w.first - w.k0;
     // LDS-DMA: wave w moves pieces w * PW .. of [K: tile t, k-step | V^T: d, 32-key unit]; surplus pieces repeat the last one
-    const int64_t k_ld = (int64_t)(p.H * p.dp >> 5), v_ld = p.rows_pad >> 5;
+    const int64_t k_ld = (int64_t)(p.H * p.dn >> 5), r_ld = p.rotp >> 5, v_ld = p.rows_pad >> 5;
+    const int ksn = p.dn >> 5;                                // k-steps of the heads' own keys; the shared rotated keys follow
     const bf16_t* src[PW];
     int64_t step[PW];
 #pragma unroll
@@ -212,8 +250,10 @@ __global__ __launch_bounds__(512, (KS <= 2 && DT <= 4) ? 4 : 2) void latent_pref
         if (pc >= PIECES) pc = PIECES - 1;
         if (pc < 4 * KS) {
             const int t = pc / KS, ks = pc - t * KS, key = kb + 32 * (t >> 1) + latent_k_row(t, fq);
-            src[i] = (const bf16_t*)p.kx + (((int64_t)(key >> 4) * k_ld + h * KS + ks) * 64 + (key & 15) + 16 * fg) * 8;
-            step[i] = 4 * k_ld * 512;
+            const bool rk = ks >= ksn;
+            const int64_t ld = rk ? r_ld : k_ld;
+            src[i] = (const bf16_t*)(rk ? p.kr : p.kx) + (((int64_t)(key >> 4) * ld + (rk ? ks - ksn : h * ksn + ks)) * 64 + (key & 15) + 16 * fg) * 8;
+            step[i] = 4 * ld * 512;
         } else {
             const int v = pc - 4 * KS, d = v >> 1, u = v & 1;
             src[i] = (const bf16_t*)p.vx + (((int64_t)(h * DT + d) * v_ld + (kb >> 5) + u) * 64 + lane) * 8;
@@ -306,10 +346,11 @@ __global__ __launch_bounds__(256) void latent_prefill_wide_kernel(LatentArgs p) 
     bool ok;
     const int r0 = w.row(0, fq, ok), qpos = w.pos0 + r0;
     bf16x8 qf[KS];
-    latent_load_q<KS>(p, w.tok0 + r0, h, fg, qf);
+    latent_load_q<KS>(p, w.tok0 + r0, qpos, h, fg, qf);
     const int kb = p.kbase[seq], j1 = last - w.k0;
     const int full_lo = (p.window > 0 ? last - p.window + 1 : 0) - w.k0, full_hi = w.first - w.k0;
-    const int64_t k_ld = (int64_t)(p.H * p.dp >> 5), v_ld = p.rows_pad >> 5;
+    const int64_t k_ld = (int64_t)(p.H * p.dn >> 5), r_ld = p.rotp >> 5, v_ld = p.rows_pad >> 5;
+    const int ksn = p.dn >> 5;
     f32x4 o[DT], lacc = f32x4{0.f, 0.f, 0.f, 0.f};
     float m_run = -1e30f;
 #pragma unroll
@@ -324,9 +365,11 @@ __global__ __launch_bounds__(256) void latent_prefill_wide_kernel(LatentArgs p) 
         for (int t = 0; t < 4; t++) {
             s[t] = f32x4{0.f, 0.f, 0.f, 0.f};
             const int key = kb + j + 32 * (t >> 1) + latent_k_row(t, fq);
-            const bf16_t* kr = (const bf16_t*)p.kx + (((int64_t)(key >> 4) * k_ld + h * KS) * 64 + (key & 15) + 16 * fg) * 8;
+            const int64_t lo = ((key & 15) + 16 * fg) * 8;
+            const bf16_t* kn = (const bf16_t*)p.kx + ((int64_t)(key >> 4) * k_ld + h * ksn) * 512 + lo;
+            const bf16_t* kr = (const bf16_t*)p.kr + ((int64_t)(key >> 4) * r_ld - ksn) * 512 + lo;
 #pragma unroll
-            for (int ks = 0; ks < KS; ks++) s[t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(*(const bf16x8*)(kr + ks * 512), qf[ks], s[t], 0, 0, 0);
+            for (int ks = 0; ks < KS; ks++) s[t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(*(const bf16x8*)((ks < ksn ? kn : kr) + ks * 512), qf[ks], s[t], 0, 0, 0);
         }
         latent_softmax<DT>(s, j >= full_lo && j + 63 <= full_hi, qpos - w.k0 - j, p.window, fg, sl2, m_run, lacc, o);
 #pragma unroll
@@ -344,7 +387,7 @@ __global__ __launch_bounds__(256) void latent_prefill_wide_kernel(LatentArgs p) 
 // ---- expanded form, any size: one 256-thread workgroup per (token, head), online softmax over 256 keys at a time, plain fp32
 // arithmetic.  The fp32 mode's kernel, and the bf16 mode's for heads wider than the instances above. ----
 template <typename T>
-__device__ __forceinline__ float lat_k(const LatentArgs& p, int64_t row, int64_t col) { return ((const T*)p.kx)[act_index<T>(row, col, (int64_t)p.H * p.dp)]; }
+__device__ __forceinline__ float lat_k(const LatentArgs& p, int64_t row, int64_t col) { return ((const T*)p.kx)[act_index<T>(row, col, (int64_t)p.H * p.dn)]; }
 template <typename T> __device__ __forceinline__ float lat_v(const LatentArgs& p, int64_t row, int64_t col);
 template <> __device__ __forceinline__ float lat_v<float>(const LatentArgs& p, int64_t row, int64_t col) { return ((const float*)p.vx)[row * (p.H * p.vp) + col]; }
 template <> __device__ __forceinline__ float lat_v<bf16_t>(const LatentArgs& p, int64_t row, int64_t col) { return (float)((const bf16_t*)p.vx)[fm_index(col, row, p.rows_pad)]; }
@@ -360,7 +403,7 @@ __global__ __launch_bounds__(256) void latent_plain_kernel(LatentArgs p) {
     if (lo < 0) lo = 0;
     float* sq = lat_sm;
     float* so = sq + p.dp;
-    for (int i = tid; i < p.dp; i += 256) sq[i] = p.q[t * p.q_ld + h * p.dp + i];
+    for (int i = tid; i < p.dp; i += 256) sq[i] = i < p.dn ? p.q[t * p.q_ld + h * p.dp + i] : lat_turn(p, p.q + t * p.q_ld + h * p.dp + p.dn, i - p.dn, pos);
     for (int i = tid; i < p.vp; i += 256) so[i] = 0.f;
     float m = -1e30f, l = 0.f;
     __syncthreads();
@@ -372,7 +415,8 @@ __global__ __launch_bounds__(256) void latent_plain_kernel(LatentArgs p) {
         if (key <= pos) {
             float a = 0.f;
             const int64_t row = p.kbase[seq] + key - k0;
-            for (int d = 0; d < p.dim; d++) a = fmaf(sq[d], lat_k<T>(p, row, h * p.dp + d), a);
+            for (int d = 0; d < p.dim; d++) a = fmaf(sq[d], lat_k<T>(p, row, h * p.dn + d), a);
+            for (int d = 0; d < p.rot; d++) a = fmaf(sq[p.dn + d], (float)((const T*)p.kr)[act_index<T>(row, d, p.rotp)], a);
             s = a * p.scale;
         }
         const float mn = fmaxf(m, bmax(s)), alpha = expf(m - mn);
@@ -390,7 +434,7 @@ __global__ __launch_bounds__(256) void latent_plain_kernel(LatentArgs p) {
         __syncthreads();
     }
     for (int i = tid; i < p.vp; i += 256) {
-        const float g = p.proj[t * p.proj_ld + p.qrp + p.rp + h * p.vp + i];
+        const float g = lat_gate(p, t, h, i);
         ActIO<T>::st((T*)p.out + act_index<T>(t, h * p.vp + i, p.out_ld), so[i] / l * (1.0f / (1.0f + expf(-g))));
     }
 }
@@ -398,14 +442,25 @@ __global__ __launch_bounds__(256) void latent_plain_kernel(LatentArgs p) {
 // ------------------------------------------------------------------------------------------
 // absorbed form (bf16)
 // ------------------------------------------------------------------------------------------
-// q'[token][head][:] = W_uk[head]^T q[token][head]: grid (H, rp / 64, ceil(n_abs / 16)), one 16-column tile per wave, K = dp
+// q'[token][head][:] = W_uk[head]^T q[token][head]: grid (H, rp / 64 (+ 1: the rotated part), ceil(n_abs / 16)), one 16-column tile per
+// wave, K = dn
 static __global__ __launch_bounds__(256) void latent_absorb_q_kernel(LatentArgs p) {
     const int h = blockIdx.x, nt = blockIdx.y * 4 + (threadIdx.x >> 6), mt = blockIdx.z, lane = threadIdx.x & 63;
-    const int fr = lane & 15, fg = lane >> 4, nks = p.dp >> 5;
+    const int fr = lane & 15, fg = lane >> 4, nks = p.dn >> 5;
+    const int64_t rt = p.rp + p.rotp;
+    if (nt * 16 >= p.rp) {                                    // (workgroup-uniform: 64 | rp)
+        for (int e = threadIdx.x; e < 16 * p.rotp; e += 256) {
+            const int j = mt * 16 + e / p.rotp, d = e % p.rotp;
+            if (j >= p.n_abs) break;
+            const int64_t t = p.abs_tok[j];
+            p.qa[((int64_t)j * p.Hp + h) * rt + p.rp + d] = (bf16_t)lat_turn(p, p.q + t * p.q_ld + h * p.dp + p.dn, d, p.tok_pos[t]);
+        }
+        return;
+    }
     const int i = mt * 16 + fr;
     const bool ok = i < p.n_abs;
     const float* qp = ok ? p.q + (int64_t)p.abs_tok[i] * p.q_ld + h * p.dp + fg * 8 : nullptr;
-    const bf16_t* w = p.ukt + (int64_t)h * p.rp * p.dp + ((int64_t)nt * nks * 64 + lane) * 8;
+    const bf16_t* w = p.ukt + (int64_t)h * p.rp * p.dn + ((int64_t)nt * nks * 64 + lane) * 8;
     f32x4 acc = f32x4{0.f, 0.f, 0.f, 0.f};
     for (int ks = 0; ks < nks; ks++) {
         const bf16x8 wf = *(const bf16x8*)(w + ks * 512);
@@ -421,15 +476,16 @@ static __global__ __launch_bounds__(256) void latent_absorb_q_kernel(LatentArgs 
     bf16x4 o;
 #pragma unroll
     for (int r = 0; r < 4; r++) o[r] = (bf16_t)acc[r];
-    *(bf16x4*)(p.qa + ((int64_t)i * p.Hp + h) * p.rp + nt * 16 + 4 * fg) = o;
+    *(bf16x4*)(p.qa + ((int64_t)i * p.Hp + h) * rt + nt * 16 + 4 * fg) = o;
 }
 
 // grid (ceil(H / 16), n_abs, n_split), 4 waves, 64 keys per step (inside one block: 64 | bs).  Wave w scores keys 16 w .. of the step
 // (operand blocks straight from the cache, copied to an LDS image on the way), the waves agree on the maximum, exchange the
 // weights through LDS, and wave w accumulates its rp / 4 latent columns over all 64 keys from the image by transposed reads.
+// KR: 32-column steps of the rotated keys, which only the scores take.
 template <int NR>                  // rp = 64 NR
 constexpr int latent_decode_lds_bytes() { return 2 * 64 * NR * 64 * 2 + 16 * 16 * 8 + 2 * 4 * 16 * 4; }
-template <int NR>
+template <int NR, int KR>
 __global__ __launch_bounds__(256) void latent_decode_kernel(LatentArgs p) {
     constexpr int IMG = 64 * NR * 64 * 2, KSN = 2 * NR;
     extern __shared__ __attribute__((aligned(16))) char lat_smc[];
@@ -446,26 +502,27 @@ __global__ __launch_bounds__(256) void latent_decode_kernel(LatentArgs p) {
     const int kt_first = lo >> 6, n_kt = (pos >> 6) - kt_first + 1, per = (n_kt + p.n_split - 1) / p.n_split;
     const int kt0 = kt_first + z * per, kt1 = min(kt0 + per, kt_first + n_kt);
     const int32_t* tbl = p.blk_table + (int64_t)seq * p.tbl_stride;
-    bf16x8 qf[KSN];
+    bf16x8 qf[KSN + KR];
 #pragma unroll
-    for (int ks = 0; ks < KSN; ks++) qf[ks] = *(const bf16x8*)(p.qa + ((int64_t)ia * p.Hp + ht * 16 + fq) * p.rp + ks * 32 + fg * 8);
+    for (int ks = 0; ks < KSN + KR; ks++) qf[ks] = *(const bf16x8*)(p.qa + ((int64_t)ia * p.Hp + ht * 16 + fq) * (NR * 64 + KR * 32) + ks * 32 + fg * 8);
     f32x4 o[NR];
 #pragma unroll
     for (int i = 0; i < NR; i++) o[i] = f32x4{0.f, 0.f, 0.f, 0.f};
     float m = -1e30f, l = 0.f;
     const float sl2 = p.scale * 1.4426950408889634f;
     const int tr_row = 4 * fg + (fq >> 2), tr_p = fq & 3;
-    auto src_of = [&](int kt) {
+    bf16x8 a[KSN + KR];
+    auto fetch = [&](int kt) {
         const int key = kt * 64, bi = key / p.bs, row = key - bi * p.bs;
         const int blk = __builtin_amdgcn_readfirstlane(tbl[bi]);
-        return (const bf16_t*)p.cache + (int64_t)blk * p.block_stride + (int64_t)(row + 16 * wave) * p.rp + lane * 8;
-    };
-    bf16x8 a[KSN];
-    if (kt0 < kt1) {
-        const bf16_t* s = src_of(kt0);
+        const bf16_t* b = (const bf16_t*)p.cache + (int64_t)blk * p.block_stride + lane * 8;
+        const int64_t r16 = row + 16 * wave;
 #pragma unroll
-        for (int ks = 0; ks < KSN; ks++) a[ks] = *(const bf16x8*)(s + ks * 512);
-    }
+        for (int ks = 0; ks < KSN; ks++) a[ks] = *(const bf16x8*)(b + r16 * p.rp + ks * 512);
+#pragma unroll
+        for (int ks = 0; ks < KR; ks++) a[KSN + ks] = *(const bf16x8*)(b + (int64_t)p.bs * p.rp + r16 * (KR * 32) + ks * 512);
+    };
+    if (kt0 < kt1) fetch(kt0);
     for (int kt = kt0; kt < kt1; kt++) {
         char* img = lat_smc + ((kt - kt0) & 1) * IMG;
         f32x4 s = f32x4{0.f, 0.f, 0.f, 0.f};
@@ -474,11 +531,9 @@ __global__ __launch_bounds__(256) void latent_decode_kernel(LatentArgs p) {
             s = __builtin_amdgcn_mfma_f32_16x16x32_bf16(a[ks], qf[ks], s, 0, 0, 0);
             *(bf16x8*)(img + ((wave * KSN + ks) * 64 + lane) * 16) = a[ks];
         }
-        if (kt + 1 < kt1) {
-            const bf16_t* sn = src_of(kt + 1);
 #pragma unroll
-            for (int ks = 0; ks < KSN; ks++) a[ks] = *(const bf16x8*)(sn + ks * 512);
-        }
+        for (int ks = KSN; ks < KSN + KR; ks++) s = __builtin_amdgcn_mfma_f32_16x16x32_bf16(a[ks], qf[ks], s, 0, 0, 0);
+        if (kt + 1 < kt1) fetch(kt + 1);
         const int key = kt * 64 + 16 * wave + 4 * fg;
         float mx = -INFINITY;
 #pragma unroll
@@ -585,7 +640,7 @@ static __global__ __launch_bounds__(1024) void latent_uv_kernel(LatentArgs p) {
     if (i >= p.n_abs) return;
     const int64_t t = p.abs_tok[i];
     const int col = h * p.vp + vt * 16 + 4 * fg;
-    const f32x4 g = *(const f32x4*)(p.proj + t * p.proj_ld + p.qrp + p.rp + col);
+    const f32x4 g = lat_gate4(p, t, h, vt * 16 + 4 * fg);
 #pragma unroll
     for (int r = 0; r < 4; r++) acc[r] *= lat_sigmoid(g[r]);
     act_store4<bf16_t>((bf16_t*)p.out, t, col, p.out_ld, acc);

@@ -1,5 +1,6 @@
 // layered.h — models described by a list of layers (nvl_layer_config): every layer names a mixer (latent attention, Mamba-2, gated
-// linear attention), its sizes and its feed-forward, with a norm before and after each sublayer.  Host side: creation, tensor
+// linear attention, channel-wise delta rule), its sizes and its feed-forward, with a norm before and after each sublayer
+// (NVL_BLOCK_SANDWICH) or after it only (NVL_BLOCK_POST: the sublayers read the residual stream itself).  Host side: creation, tensor
 // staging, freezing into the kernels' layouts, the layer stack of one forward pass.  Included by nvllm.hip.
 //
 // What differs from the fixed-shape models around it:
@@ -13,8 +14,18 @@
 
 namespace {
 
+constexpr float CLAMPED_GLU_SLOPE = 1.702f;
 constexpr int LAT_ABSORB_MAX = 16, LAT_ABSORB_MAX_RP = 512, REC_STEP_MAX = 4;
 
+bool same_rotation(const nvl_layer_config& a, const nvl_layer_config& b) {
+    return a.rot_dim == b.rot_dim && a.rot_base == b.rot_base && a.rot_factor == b.rot_factor && a.rot_original == b.rot_original &&
+           a.rot_fast == b.rot_fast && a.rot_slow == b.rot_slow;
+}
+// unrotated (padded to 32) + rotated part; d + rot = 192 with 256 value channels has no LDS left for its ring of tiles
+int pad_rotated(int d, int vp) {
+    for (int p : {32, 64, 96, 128, 192, 256}) if (d <= p && !(p == 192 && vp > 128)) return p;
+    return (int)round_up(d, 64);
+}
 int pad_head(int d, int unit) {       // head sizes the attention instances exist for; larger ones take the plain kernel
     for (int p : {32, 64, 128, 256}) if (d <= p) return p;
     return (int)round_up(d, unit);
@@ -25,7 +36,9 @@ int pad_head(int d, int unit) {       // head sizes the attention instances exis
 // ------------------------------------------------------------------------------------------
 int layered_create(const nvl_model_config& c, const nvl_layer_config* layers, const nvl_runtime_opts& opts, nvl_model** out) {
     auto bad = [&](const std::string& why) { return fail(nullptr, NVL_ERR_INVALID, "nvl_create_layers: " + why); };
-    if (c.block_style != NVL_BLOCK_SANDWICH || c.activation_type != NVL_ACT_GEGLU) return bad("block_style NVL_BLOCK_SANDWICH and activation_type NVL_ACT_GEGLU expected");
+    if (c.block_style != NVL_BLOCK_SANDWICH && c.block_style != NVL_BLOCK_POST) return bad("block_style NVL_BLOCK_SANDWICH or NVL_BLOCK_POST expected");
+    if (c.activation_type != NVL_ACT_GEGLU && c.activation_type != NVL_ACT_CLAMPED_GLU) return bad("activation_type NVL_ACT_GEGLU or NVL_ACT_CLAMPED_GLU expected");
+    if (!(c.logit_softcap >= 0.f)) return bad("logit_softcap is negative");
     if (c.hidden <= 0 || c.num_layers <= 0 || c.vocab_size <= 0 || c.max_seq_len <= 0) return bad("non-positive model dimension");
     if (c.hidden > 20480) return bad("hidden larger than 20480");
     if (opts.max_seqs <= 0) return bad("max_seqs must be >= 1");
@@ -36,8 +49,17 @@ int layered_create(const nvl_model_config& c, const nvl_layer_config* layers, co
         const nvl_layer_config& l = layers[i];
         const std::string at = "layer " + std::to_string(i) + ": ";
         if (l.heads <= 0 || l.vdim <= 0 || l.vdim > 2048 || l.ffn_dim < 0) return bad(at + "bad heads / vdim / ffn_dim");
+        if (l.ffn_dim && c.activation_type == NVL_ACT_CLAMPED_GLU && !(l.ffn_limit > 0.f)) return bad(at + "ffn_limit is not positive");
         switch (l.mixer) {
             case NVL_MIXER_LATENT_ATTENTION:
+                if (l.rot_dim < 0 || l.rot_dim % 2 || l.rot_dim > 1024 || (l.rot_dim && !(l.rot_base > 1.0)) ||
+                    (l.rot_factor != 0.0 && !(l.rot_factor > 0.0 && l.rot_original > 0.0 && l.rot_fast > 0.0 && l.rot_slow > 0.0))) return bad(at + "bad rotation");
+                if (l.kv_from >= 0) {
+                    if (l.kv_from >= i) return bad(at + "kv_from names no earlier layer");
+                    const nvl_layer_config& s = layers[l.kv_from];
+                    if (s.mixer != l.mixer || s.kv_from >= 0) return bad(at + "kv_from names a layer without latents of its own");
+                    if (s.kv_rank != l.kv_rank || !same_rotation(s, l)) return bad(at + "kv_from names a layer with another latent or rotation");
+                }
                 if (l.dim <= 0 || l.q_rank <= 0 || l.kv_rank <= 0 || l.window < 0 || l.dim > 2048) return bad(at + "bad latent attention sizes");
                 break;
             case NVL_MIXER_MAMBA2:
@@ -46,6 +68,9 @@ int layered_create(const nvl_model_config& c, const nvl_layer_config* layers, co
                 break;
             case NVL_MIXER_GLA:
                 if (l.dim <= 0 || l.dim > 2048 || !(l.tau > 0.f) || l.decay_rank < 0) return bad(at + "bad gated linear attention sizes");
+                break;
+            case NVL_MIXER_CHANNEL_DELTA:
+                if (l.dim <= 0 || l.dim > 2048 || l.kv_heads <= 0 || l.heads % l.kv_heads || l.conv_taps <= 0 || l.decay_rank < 0) return bad(at + "bad channel delta sizes");
                 break;
             default: return bad(at + "unknown mixer");
         }
@@ -58,7 +83,8 @@ int layered_create(const nvl_model_config& c, const nvl_layer_config* layers, co
         owner[(size_t)i] = o;
         const nvl_layer_config &a = layers[i], &b = layers[o];
         if (a.mixer != b.mixer || a.heads != b.heads || a.dim != b.dim || a.vdim != b.vdim || a.q_rank != b.q_rank || a.kv_rank != b.kv_rank ||
-            a.state != b.state || a.groups != b.groups || a.conv_taps != b.conv_taps || a.ffn_dim != b.ffn_dim)
+            a.state != b.state || a.groups != b.groups || a.conv_taps != b.conv_taps || a.ffn_dim != b.ffn_dim || a.rot_dim != b.rot_dim ||
+            a.kv_heads != b.kv_heads || a.gate_per_head != b.gate_per_head || (i != o && a.mixer == NVL_MIXER_LATENT_ATTENTION && (a.kv_from >= 0) != (b.kv_from >= 0)))
             return bad("layer " + std::to_string(i) + " does not have the shape of the layer whose tensors it uses");
     }
     if (opts.device < 0 || nvl_device_count() <= opts.device) return fail(nullptr, NVL_ERR_NO_DEVICE, "nvl_create_layers: no HIP device (this library has no CPU fallback)");
@@ -87,15 +113,21 @@ int layered_create(const nvl_model_config& c, const nvl_layer_config* layers, co
             r.Fp = (int)round_up(r.c.ffn_dim, 64);
             const int H = r.c.heads;
             if (r.c.mixer == NVL_MIXER_LATENT_ATTENTION) {
-                r.dp = pad_head(r.c.dim, 64); r.vp = pad_head(r.c.vdim, 64);
+                r.vp = pad_head(r.c.vdim, 64);
+                r.rotp = (int)round_up(r.c.rot_dim, 32);
+                r.dp = r.rotp ? pad_rotated((int)round_up(r.c.dim, 32) + r.rotp, r.vp) : pad_head(r.c.dim, 64);
+                r.dn = r.dp - r.rotp;
+                r.src = r.c.kv_from >= 0 ? r.c.kv_from : i;
                 r.qrp = (int)round_up(r.c.q_rank, 64); r.rp = (int)round_up(r.c.kv_rank, 64);
                 if (r.rp > 256 && r.rp < 512) r.rp = r.rp <= 384 ? 384 : 512;       // (instances of the absorbed form)
-                r.n_in = r.qrp + r.rp + H * r.vp; r.ko = (int)round_up((int64_t)H * r.vp, 64);
+                r.gate_off = r.qrp + (r.src == i ? r.rp + r.rotp : 0);
+                r.n_in = r.gate_off + (r.c.gate_per_head ? H : H * r.vp); r.ko = (int)round_up((int64_t)H * r.vp, 64);
                 size_t w = 0;
                 while (w < m->windows.size() && m->windows[w] != r.c.window) w++;
                 if (w == m->windows.size()) m->windows.push_back(r.c.window);
                 r.win = (int)w;
-                r.cache_off = cache; cache += (int64_t)bs * r.rp;
+                if (r.src == i) { r.cache_off = cache; cache += (int64_t)bs * (r.rp + r.rotp); }
+                else r.cache_off = m->runs[(size_t)r.src].cache_off;
             } else {
                 const int DVp = (int)round_up(r.c.vdim, 4), DK = r.c.mixer == NVL_MIXER_MAMBA2 ? r.c.state : r.c.dim;
                 r.ko = (int)round_up((int64_t)H * r.c.vdim, 64);
@@ -104,7 +136,10 @@ int layered_create(const nvl_model_config& c, const nvl_layer_config* layers, co
                     r.conv_dim = H * r.c.vdim + 2 * r.c.groups * r.c.state;
                     r.n_in = H * r.c.vdim + r.conv_dim + H;
                     r.ring_off = state; state += round_up((int64_t)r.c.conv_taps * r.conv_dim, 64);
-                }       // (GLA: n_in follows from the decay rank, layered_finalize)
+                } else if (r.c.mixer == NVL_MIXER_CHANNEL_DELTA) {
+                    r.conv_dim = 2 * r.c.kv_heads * r.c.dim + H * r.c.vdim;
+                    r.ring_off = state; state += round_up((int64_t)r.c.conv_taps * r.conv_dim, 64);
+                }       // (GLA, channel delta: n_in follows from the decay rank, layered_finalize)
             }
         }
         m->lat_block_stride = cache; m->rec_slot_stride = state;
@@ -146,32 +181,39 @@ void layered_shape(const nvl_model* m, int kind, int layer, int64_t& N, int64_t&
     const LayerRun& r = m->runs[(size_t)layer];
     const nvl_layer_config& c = r.c;
     if (r.owner != layer) return;
+    const bool post = m->cfg.block_style == NVL_BLOCK_POST, delta = c.mixer == NVL_MIXER_CHANNEL_DELTA;
     const bool lat = c.mixer == NVL_MIXER_LATENT_ATTENTION, mam = c.mixer == NVL_MIXER_MAMBA2, gla = c.mixer == NVL_MIXER_GLA;
     const int64_t hv = (int64_t)c.heads * c.vdim, hd = (int64_t)c.heads * c.dim;
     switch (kind) {
-        case NVL_T_ATTN_NORM_W: case NVL_T_MIX_POST_NORM: N = W; return;
-        case NVL_T_FFN_NORM_W: case NVL_T_FFN_POST_NORM: N = W; return;
+        case NVL_T_ATTN_NORM_W: case NVL_T_FFN_NORM_W: if (!post) N = W; return;
+        case NVL_T_MIX_POST_NORM: case NVL_T_FFN_POST_NORM: N = W; return;
+        case NVL_T_MIX_SCALE: case NVL_T_FFN_SCALE: if (post) N = W; return;
         case NVL_T_W1: N = 2 * (int64_t)c.ffn_dim; K = W; return;
         case NVL_T_W2: if (c.ffn_dim) { N = W; K = c.ffn_dim; } return;
         case NVL_T_WO: if (!mam) { N = W; K = hv; } return;
-        case NVL_T_MIX_GATE: if (!mam) { N = hv; K = W; } return;
+        case NVL_T_MIX_GATE: if (lat || gla) { N = c.gate_per_head && lat ? c.heads : hv; K = W; } return;
         case NVL_T_LAT_DQ: if (lat) { N = c.q_rank; K = W; } return;
         case NVL_T_LAT_DQ_NORM: if (lat) N = c.q_rank; return;
-        case NVL_T_LAT_UQ: if (lat) { N = hd; K = c.q_rank; } return;
-        case NVL_T_LAT_DKV: if (lat) { N = c.kv_rank; K = W; } return;
-        case NVL_T_LAT_DKV_NORM: if (lat) N = c.kv_rank; return;
+        case NVL_T_LAT_UQ: if (lat) { N = hd + (int64_t)c.heads * c.rot_dim; K = c.q_rank; } return;
+        case NVL_T_LAT_DKV: if (lat && r.src == layer) { N = c.kv_rank + c.rot_dim; K = W; } return;
+        case NVL_T_LAT_DKV_NORM: if (lat && r.src == layer) N = c.kv_rank; return;
         case NVL_T_LAT_UK: if (lat) { N = hd; K = c.kv_rank; } return;
         case NVL_T_LAT_UV: if (lat) { N = hv; K = c.kv_rank; } return;
-        case NVL_T_WQ: case NVL_T_WK: if (gla) { N = hd; K = W; } return;
-        case NVL_T_WV: if (gla) { N = hv; K = W; } return;
-        case NVL_T_GLA_NORM: if (gla) N = c.vdim; return;
-        case NVL_T_GLA_A1: if (gla) { N = c.decay_rank ? c.decay_rank : -1; K = W; } return;       // -1: any
-        case NVL_T_GLA_A2: if (gla) { N = hd; K = c.decay_rank ? c.decay_rank : -1; } return;
-        case NVL_T_GLA_A2_B: if (gla) N = hd; return;
+        case NVL_T_WQ: case NVL_T_WK: if (gla || delta) { N = delta ? (int64_t)c.kv_heads * c.dim : hd; K = W; } return;
+        case NVL_T_WV: if (gla || delta) { N = hv; K = W; } return;
+        case NVL_T_DELTA_CONV: if (delta) N = (int64_t)r.conv_dim * c.conv_taps; return;
+        case NVL_T_DELTA_BETA: if (delta) { N = c.heads; K = W; } return;
+        case NVL_T_DELTA_G1: if (delta) { N = -1; K = W; } return;
+        case NVL_T_DELTA_G2: if (delta) { N = hv; K = -1; } return;
+        case NVL_T_GLA_NORM: if (gla || delta) N = c.vdim; return;
+        case NVL_T_GLA_A1: if (gla || delta) { N = c.decay_rank ? c.decay_rank : -1; K = W; } return;       // -1: any
+        case NVL_T_GLA_A2: if (gla || delta) { N = hd; K = c.decay_rank ? c.decay_rank : -1; } return;
+        case NVL_T_GLA_A2_B: if (gla || delta) N = hd; return;
         case NVL_T_MAMBA_IN_PROJ: if (mam) { N = r.n_in; K = W; } return;
         case NVL_T_MAMBA_CONV_W: if (mam) N = (int64_t)r.conv_dim * c.conv_taps; return;
         case NVL_T_MAMBA_CONV_B: if (mam) N = r.conv_dim; return;
-        case NVL_T_MAMBA_A_LOG: case NVL_T_MAMBA_D: case NVL_T_MAMBA_DT_BIAS: if (mam) N = c.heads; return;
+        case NVL_T_MAMBA_A_LOG: if (mam || delta) N = c.heads; return;
+        case NVL_T_MAMBA_D: case NVL_T_MAMBA_DT_BIAS: if (mam) N = c.heads; return;
         case NVL_T_MAMBA_NORM: if (mam) N = hv; return;
         case NVL_T_MAMBA_OUT_PROJ: if (mam) { N = W; K = hv; } return;
         default: return;
@@ -180,7 +222,7 @@ void layered_shape(const nvl_model* m, int kind, int layer, int64_t& N, int64_t&
 bool layered_1d(int kind) {
     if (is_1d(kind)) return true;
     return kind == NVL_T_MIX_POST_NORM || kind == NVL_T_FFN_POST_NORM || kind == NVL_T_LAT_DQ_NORM || kind == NVL_T_LAT_DKV_NORM ||
-           kind == NVL_T_GLA_NORM || kind == NVL_T_GLA_A2_B;
+           kind == NVL_T_GLA_NORM || kind == NVL_T_GLA_A2_B || kind == NVL_T_MIX_SCALE || kind == NVL_T_FFN_SCALE || kind == NVL_T_DELTA_CONV;
 }
 int layered_upload(nvl_model* m, int kind, int layer, const void* data, int dtype, int64_t rows, int64_t cols, int layout) {
     int64_t N, K;
@@ -227,9 +269,51 @@ float* lay_vector(nvl_model* m, const DevTensor& t, int64_t padded) {
     m->stats.weight_bytes += (double)padded * 4;
     return p;
 }
+// (w + offset) * scale (scale: NULL or another staged vector), zero beyond the vector: what a norm multiplies by
+__global__ void norm_weight_kernel(float* w, const void* scale, int scale_dtype, float offset, int64_t n) {
+    const int64_t i = (int64_t)blockIdx.x * 256 + threadIdx.x;
+    if (i < n) w[i] = (w[i] + offset) * (scale ? ld_as_f32(scale, scale_dtype, i) : 1.0f);
+}
+float* lay_norm(nvl_model* m, const DevTensor& t, int64_t padded, const DevTensor* scale = nullptr) {
+    float* p = lay_vector(m, t, padded);
+    const bool sc = scale && scale->present();
+    if (m->cfg.norm_weight_offset != 0.f || sc) {
+        const int64_t n = t.rows * t.cols;
+        hipLaunchKernelGGL(norm_weight_kernel, dim3(cdiv(n, 256)), dim3(256), 0, m->stream, p, sc ? (const void*)scale->p : nullptr, sc ? scale->raw_dtype : 0, m->cfg.norm_weight_offset, n);
+        NVL_HIP(hipGetLastError());
+    }
+    return p;
+}
+// (cos, sin) of every position for a rotation; angles in double
+f32x2* lay_rotation(nvl_model* m, const nvl_layer_config& c) {
+    const int half = c.rot_dim / 2;
+    std::vector<double> f((size_t)half);
+    double mag = 1.0;
+    for (int i = 0; i < half; i++) f[(size_t)i] = std::pow(c.rot_base, -2.0 * i / c.rot_dim);
+    if (c.rot_factor > 0.0) {      // YaRN: pairs that turn often over the original length keep their frequency, the others are slowed down
+        auto place = [&](double turns) { return c.rot_dim * std::log(c.rot_original / (2.0 * M_PI * turns)) / (2.0 * std::log(c.rot_base)); };
+        const double lo = std::max(std::floor(place(c.rot_fast)), 0.0), hi = std::min(std::ceil(place(c.rot_slow)), c.rot_dim - 1.0);
+        for (int i = 0; i < half; i++) {
+            const double ramp = std::min(std::max((i - lo) / std::max(hi - lo, 0.001), 0.0), 1.0);
+            f[(size_t)i] = f[(size_t)i] / c.rot_factor * ramp + f[(size_t)i] * (1.0 - ramp);
+        }
+        mag = 0.1 * std::log(c.rot_factor) + 1.0;
+    }
+    std::vector<float> t((size_t)m->cfg.max_seq_len * half * 2);
+    for (int p = 0; p < m->cfg.max_seq_len; p++)
+        for (int i = 0; i < half; i++) {
+            const double a = p * f[(size_t)i];
+            t[((size_t)p * half + i) * 2] = (float)(std::cos(a) * mag);
+            t[((size_t)p * half + i) * 2 + 1] = (float)(std::sin(a) * mag);
+        }
+    f32x2* d = (f32x2*)lay_alloc(m, (int64_t)t.size() * 4);
+    NVL_HIP(hipMemcpyAsync(d, t.data(), t.size() * 4, hipMemcpyHostToDevice, m->stream));
+    NVL_HIP(hipStreamSynchronize(m->stream));
+    return d;
+}
 // rows [n0, n0 + N) of a staged matrix into dst: grouped row / column padding as place_2d_kernel
 void lay_place(nvl_model* m, const DevTensor& t, void* dst, int64_t Kd, int64_t row0 = 0, int rg = 0, int rgp = 0, int cg = 0, int cgp = 0,
-               int64_t n0 = 0, int64_t N = -1, bool trans = false) {
+               int64_t n0 = 0, int64_t N = -1, bool trans = false, bool row_major = false) {
     if (N < 0) N = t.rows;
     Place2D pl{N, t.cols, Kd, row0, rg ? rg : 1, rg ? rgp : 1, cg ? cg : 1, cg ? cgp : 1};
     const dim3 grid((unsigned)std::min<int64_t>(cdiv(t.cols, 256), 64), (unsigned)N);
@@ -238,14 +322,15 @@ void lay_place(nvl_model* m, const DevTensor& t, void* dst, int64_t Kd, int64_t 
         if (trans) hipLaunchKernelGGL((place_2d_kernel<float, false, true>), grid, dim3(256), 0, m->stream, t.p, t.raw_dtype, src0, (float*)dst, pl);
         else hipLaunchKernelGGL((place_2d_kernel<float, false, false>), grid, dim3(256), 0, m->stream, t.p, t.raw_dtype, src0, (float*)dst, pl);
     } else {
-        if (trans) hipLaunchKernelGGL((place_2d_kernel<bf16_t, true, true>), grid, dim3(256), 0, m->stream, t.p, t.raw_dtype, src0, (bf16_t*)dst, pl);
+        if (row_major) hipLaunchKernelGGL((place_2d_kernel<bf16_t, false, false>), grid, dim3(256), 0, m->stream, t.p, t.raw_dtype, src0, (bf16_t*)dst, pl);
+        else if (trans) hipLaunchKernelGGL((place_2d_kernel<bf16_t, true, true>), grid, dim3(256), 0, m->stream, t.p, t.raw_dtype, src0, (bf16_t*)dst, pl);
         else hipLaunchKernelGGL((place_2d_kernel<bf16_t, true, false>), grid, dim3(256), 0, m->stream, t.p, t.raw_dtype, src0, (bf16_t*)dst, pl);
     }
     NVL_HIP(hipGetLastError());
 }
 
 // absorbed latent attention: available to a layer?
-bool lat_absorb_ok(const nvl_model* m, const LayerRun& r) { return !m->f32 && r.rp <= LAT_ABSORB_MAX_RP; }
+bool lat_absorb_ok(const nvl_model* m, const LayerRun& r) { return !m->f32 && r.rp <= LAT_ABSORB_MAX_RP && (r.rotp <= 64 || r.rotp == 128); }
 
 void layered_finalize(nvl_model* m) {
     auto need = [&](const DevTensor& t, const std::string& what) -> const DevTensor& {
@@ -254,7 +339,8 @@ void layered_finalize(nvl_model* m) {
     };
     const int64_t H = m->H;
     need(m->g[NVL_T_TOK_EMB], "token embedding"); need(m->g[NVL_T_FINAL_NORM_W], "final norm");
-    m->final_norm = lay_vector(m, m->g[NVL_T_FINAL_NORM_W], H);
+    const bool post = m->cfg.block_style == NVL_BLOCK_POST;
+    m->final_norm = lay_norm(m, m->g[NVL_T_FINAL_NORM_W], H);
     auto big = [&](int kind, const char* what) {      // [V][H]: the embedding table / LM head
         void* p = lay_matrix(m, m->V, H);
         lay_place(m, need(m->g[kind], what), p, H);
@@ -266,7 +352,7 @@ void layered_finalize(nvl_model* m) {
     for (int k = 0; k < NVL_T_ATTN_NORM_W; k++) { dfree(m->g[k].p); m->g[k].p = nullptr; }
     m->g[NVL_T_TOK_EMB].p = emb; m->g[NVL_T_TOK_EMB].raw_dtype = -1;      // (the embedding kernels' view of it)
 
-    int64_t ld_in = 0, q_cols = 0, cq_cols = 0, ko = 0, conv = 0, ocols = 0, Fmax = 0, abs_cols = 0;
+    int64_t ld_in = 0, q_cols = 0, cq_cols = 0, ko = 0, conv = 0, ocols = 0, Fmax = 0, abs_cols = 0, z_cols = 0, g_cols = 0, pa_cols = 0, pg_cols = 0;
     for (int i = 0; i < m->L; i++) {
         LayerRun& r = m->runs[(size_t)i];
         const nvl_layer_config& c = r.c;
@@ -275,11 +361,11 @@ void layered_finalize(nvl_model* m) {
         const std::string at = "layer " + std::to_string(i) + " ";
         if (r.owner == i) {
             auto T = [&](int kind, const char* what) -> const DevTensor& { return need(l.t[kind], at + what); };
-            w.norm1 = lay_vector(m, T(NVL_T_ATTN_NORM_W, "norm before the mixer"), H);
-            w.norm1b = lay_vector(m, T(NVL_T_MIX_POST_NORM, "norm after the mixer"), H);
+            if (!post) w.norm1 = lay_norm(m, T(NVL_T_ATTN_NORM_W, "norm before the mixer"), H);
+            w.norm1b = lay_norm(m, T(NVL_T_MIX_POST_NORM, "norm after the mixer"), H, &l.t[NVL_T_MIX_SCALE]);
             if (c.ffn_dim) {
-                w.norm2 = lay_vector(m, T(NVL_T_FFN_NORM_W, "norm before the feed-forward"), H);
-                w.norm2b = lay_vector(m, T(NVL_T_FFN_POST_NORM, "norm after the feed-forward"), H);
+                if (!post) w.norm2 = lay_norm(m, T(NVL_T_FFN_NORM_W, "norm before the feed-forward"), H);
+                w.norm2b = lay_norm(m, T(NVL_T_FFN_POST_NORM, "norm after the feed-forward"), H, &l.t[NVL_T_FFN_SCALE]);
                 const DevTensor& w1 = T(NVL_T_W1, "feed-forward gate / up");
                 w.w1 = lay_matrix(m, 2 * r.Fp, H);
                 if (m->f32) { lay_place(m, w1, w.w1, H, 0, 0, 0, 0, 0, 0, c.ffn_dim); lay_place(m, w1, w.w1, H, r.Fp, 0, 0, 0, 0, c.ffn_dim, c.ffn_dim); }
@@ -290,19 +376,31 @@ void layered_finalize(nvl_model* m) {
             if (c.mixer == NVL_MIXER_LATENT_ATTENTION) {
                 w.in = lay_matrix(m, r.n_in, H);
                 lay_place(m, T(NVL_T_LAT_DQ, "query down projection"), w.in, H);
-                lay_place(m, T(NVL_T_LAT_DKV, "key/value down projection"), w.in, H, r.qrp);
-                lay_place(m, T(NVL_T_MIX_GATE, "output gate"), w.in, H, r.qrp + r.rp, c.vdim, r.vp);
+                if (r.src == i) {
+                    const DevTensor& dkv = T(NVL_T_LAT_DKV, "key/value down projection");
+                    lay_place(m, dkv, w.in, H, r.qrp, 0, 0, 0, 0, 0, c.kv_rank);
+                    if (c.rot_dim) lay_place(m, dkv, w.in, H, r.qrp + r.rp, 0, 0, 0, 0, c.kv_rank, c.rot_dim);
+                    w.dkv_norm = lay_vector(m, T(NVL_T_LAT_DKV_NORM, "key/value latent norm"), r.rp);
+                }
+                const DevTensor& gate = T(NVL_T_MIX_GATE, "output gate");
+                if (c.gate_per_head) lay_place(m, gate, w.in, H, r.gate_off);
+                else lay_place(m, gate, w.in, H, r.gate_off, c.vdim, r.vp);
                 w.dq_norm = lay_vector(m, T(NVL_T_LAT_DQ_NORM, "query latent norm"), r.qrp);
-                w.dkv_norm = lay_vector(m, T(NVL_T_LAT_DKV_NORM, "key/value latent norm"), r.rp);
                 w.uq = lay_matrix(m, (int64_t)c.heads * r.dp, r.qrp);
-                lay_place(m, T(NVL_T_LAT_UQ, "query up projection"), w.uq, r.qrp, 0, c.dim, r.dp);
+                const DevTensor& uq = T(NVL_T_LAT_UQ, "query up projection");
+                if (!c.rot_dim) lay_place(m, uq, w.uq, r.qrp, 0, c.dim, r.dp);
+                else for (int64_t h = 0; h < c.heads; h++) {
+                    const int64_t from = h * (c.dim + c.rot_dim);
+                    lay_place(m, uq, w.uq, r.qrp, h * r.dp, 0, 0, 0, 0, from, c.dim);
+                    lay_place(m, uq, w.uq, r.qrp, h * r.dp + r.dn, 0, 0, 0, 0, from + c.dim, c.rot_dim);
+                }
                 const DevTensor& uk = T(NVL_T_LAT_UK, "key up projection");
-                w.uk = lay_matrix(m, (int64_t)c.heads * r.dp, r.rp);
-                lay_place(m, uk, w.uk, r.rp, 0, c.dim, r.dp);
+                w.uk = lay_matrix(m, (int64_t)c.heads * r.dn, r.rp);
+                lay_place(m, uk, w.uk, r.rp, 0, c.dim, r.dn);
                 if (lat_absorb_ok(m, r)) {
-                    w.ukt = lay_matrix(m, (int64_t)c.heads * r.rp, r.dp);
+                    w.ukt = lay_matrix(m, (int64_t)c.heads * r.rp, r.dn);
                     for (int h = 0; h < c.heads; h++)
-                        lay_place(m, uk, (char*)w.ukt + (int64_t)h * r.rp * r.dp * (int64_t)m->wsize, r.dp, 0, 0, 0, 0, 0, (int64_t)h * c.dim, c.dim, true);
+                        lay_place(m, uk, (char*)w.ukt + (int64_t)h * r.rp * r.dn * (int64_t)m->wsize, r.dn, 0, 0, 0, 0, 0, (int64_t)h * c.dim, c.dim, true);
                 }
                 w.uv = lay_matrix(m, (int64_t)c.heads * r.vp, r.rp);
                 lay_place(m, T(NVL_T_LAT_UV, "value up projection"), w.uv, r.rp, 0, c.vdim, r.vp);
@@ -319,6 +417,37 @@ void layered_finalize(nvl_model* m) {
                 w.mix_norm = lay_vector(m, T(NVL_T_MAMBA_NORM, "inner norm"), (int64_t)c.heads * c.vdim);
                 w.o = lay_matrix(m, H, r.ko);
                 lay_place(m, T(NVL_T_MAMBA_OUT_PROJ, "output projection"), w.o, r.ko);
+            } else if (c.mixer == NVL_MIXER_CHANNEL_DELTA) {
+                const DevTensor &a1 = T(NVL_T_GLA_A1, "decay projection (a1)"), &a2 = T(NVL_T_GLA_A2, "decay projection (a2)");
+                const DevTensor &g1 = T(NVL_T_DELTA_G1, "output gate (g1)"), &g2 = T(NVL_T_DELTA_G2, "output gate (g2)");
+                if (a1.rows != a2.cols || g1.rows != g2.cols || a1.rows > 2048 || g1.rows > 2048)
+                    throw std::runtime_error("nvl_finalize: " + at + "the low-rank projections do not fit (or a rank exceeds 2048)");
+                w.rank = (int)a1.rows; w.grank = (int)g1.rows;
+                w.a_rkp = (int)round_up(w.rank, 64); w.g_rkp = (int)round_up(w.grank, 64);
+                const int64_t qk = (int64_t)c.kv_heads * c.dim, hd = (int64_t)c.heads * c.dim, hv = (int64_t)c.heads * c.vdim;
+                r.a1_off = (int)round_up(r.conv_dim, 4); r.g1_off = r.a1_off + (int)round_up(w.rank, 4); r.b_off = r.g1_off + (int)round_up(w.grank, 4);
+                r.n_in = r.b_off + c.heads;
+                w.in = lay_matrix(m, r.n_in, H);
+                lay_place(m, T(NVL_T_WQ, "query projection"), w.in, H);
+                lay_place(m, T(NVL_T_WK, "key projection"), w.in, H, qk);
+                lay_place(m, T(NVL_T_WV, "value projection"), w.in, H, 2 * qk);
+                lay_place(m, a1, w.in, H, r.a1_off);
+                lay_place(m, g1, w.in, H, r.g1_off);
+                lay_place(m, T(NVL_T_DELTA_BETA, "step size projection"), w.in, H, r.b_off);
+                w.conv_w = lay_vector(m, T(NVL_T_DELTA_CONV, "convolution"), (int64_t)r.conv_dim * c.conv_taps);
+                w.conv_b = (float*)lay_alloc(m, (int64_t)r.conv_dim * 4);
+                w.a_log = lay_vector(m, T(NVL_T_MAMBA_A_LOG, "A_log"), c.heads);
+                w.dt_bias = lay_vector(m, T(NVL_T_GLA_A2_B, "decay bias"), hd);
+                w.mix_norm = lay_vector(m, T(NVL_T_GLA_NORM, "head norm"), c.vdim);
+                w.a2m = lay_matrix(m, hd, w.a_rkp); lay_place(m, a2, w.a2m, w.a_rkp);
+                w.g2m = lay_matrix(m, hv, w.g_rkp); lay_place(m, g2, w.g2m, w.g_rkp);
+                w.a2r = w.a2m; w.g2r = w.g2m;
+                if (!m->f32) {
+                    w.a2r = lay_matrix(m, hd, w.a_rkp); lay_place(m, a2, w.a2r, w.a_rkp, 0, 0, 0, 0, 0, 0, -1, false, true);
+                    w.g2r = lay_matrix(m, hv, w.g_rkp); lay_place(m, g2, w.g2r, w.g_rkp, 0, 0, 0, 0, 0, 0, -1, false, true);
+                }
+                w.o = lay_matrix(m, H, r.ko);
+                lay_place(m, T(NVL_T_WO, "output projection"), w.o, r.ko);
             } else {
                 const DevTensor& a1 = T(NVL_T_GLA_A1, "decay projection (a1)");
                 const DevTensor& a2 = T(NVL_T_GLA_A2, "decay projection (a2)");
@@ -344,6 +473,18 @@ void layered_finalize(nvl_model* m) {
     for (int i = 0; i < m->L; i++) {
         LayerRun& r = m->runs[(size_t)i];
         const nvl_layer_config& c = r.c;
+        if (c.mixer == NVL_MIXER_LATENT_ATTENTION && c.rot_dim) {
+            for (int j = 0; j < i && !r.turn; j++)
+                if (m->runs[(size_t)j].turn && same_rotation(m->runs[(size_t)j].c, c)) r.turn = m->runs[(size_t)j].turn;
+            if (!r.turn) r.turn = lay_rotation(m, c);
+        }
+        if (c.mixer == NVL_MIXER_CHANNEL_DELTA) {      // (also the layers that use another layer's tensors)
+            const LayerRun& o = m->runs[(size_t)r.owner];
+            const MixerW& w = m->mixers[(size_t)r.owner];
+            r.a1_off = o.a1_off; r.g1_off = o.g1_off; r.b_off = o.b_off; r.n_in = o.n_in;
+            z_cols = std::max(z_cols, (int64_t)c.heads * c.dim); g_cols = std::max(g_cols, (int64_t)c.heads * c.vdim);
+            pa_cols = std::max<int64_t>(pa_cols, w.a_rkp); pg_cols = std::max<int64_t>(pg_cols, w.g_rkp);
+        }
         if (c.mixer == NVL_MIXER_GLA) r.n_in = 2 * c.heads * (c.dim + c.vdim) + m->mixers[(size_t)r.owner].rank;
         ld_in = std::max(ld_in, round_up(r.n_in, 4));
         ko = std::max<int64_t>(ko, r.ko);
@@ -351,7 +492,7 @@ void layered_finalize(nvl_model* m) {
         if (c.mixer == NVL_MIXER_LATENT_ATTENTION) {
             q_cols = std::max<int64_t>(q_cols, (int64_t)c.heads * r.dp);
             cq_cols = std::max<int64_t>(cq_cols, r.qrp);
-            if (lat_absorb_ok(m, r)) abs_cols = std::max(abs_cols, round_up(c.heads, 16) * r.rp);
+            if (lat_absorb_ok(m, r)) abs_cols = std::max(abs_cols, round_up(c.heads, 16) * (r.rp + r.rotp));
         } else {
             ocols = std::max<int64_t>(ocols, (int64_t)c.heads * c.vdim);
             conv = std::max<int64_t>(conv, r.conv_dim);
@@ -374,6 +515,11 @@ void layered_finalize(nvl_model* m) {
     if (q_cols) { m->lq = f32buf(Mmax * q_cols); m->lcq = lay_alloc(m, Mp * cq_cols * ws); }
     m->lmix = lay_alloc(m, Mp * ko * ws);
     if (ocols) m->lo = f32buf(Mmax * m->lo_ld);
+    if (z_cols) {
+        m->lz_ld = round_up(z_cols, 4); m->lg_ld = round_up(g_cols, 4);
+        m->lz = f32buf(Mmax * m->lz_ld); m->lg = f32buf(Mmax * m->lg_ld);
+        m->lpa = lay_alloc(m, Mp * pa_cols * ws); m->lpg = lay_alloc(m, Mp * pg_cols * ws);
+    }
     if (conv) m->lconv = f32buf(Mmax * m->lconv_ld);
     if (m->lat_block_stride) m->lat_cache = lay_alloc(m, m->lat_block_stride * m->num_blocks * ws);
     if (m->rec_slot_stride) m->rec_state = f32buf(m->rec_slot_stride * S);
@@ -399,7 +545,7 @@ void layered_finalize(nvl_model* m) {
 void layered_free(nvl_model* m) {
     if (!m->layered) return;
     for (void* p : m->layered_allocs) dfree(p);
-    dfree(m->key_c); dfree(m->key_k); dfree(m->key_v); dfree(m->rec_z); dfree(m->rec_decay);
+    dfree(m->key_c); dfree(m->key_r); dfree(m->key_k); dfree(m->key_v); dfree(m->rec_z); dfree(m->rec_decay); dfree(m->delta_ws);
     if (m->finalized) m->g[NVL_T_TOK_EMB].p = nullptr;
     m->lm_head = nullptr;
 }
@@ -451,11 +597,11 @@ int layered_decode_key(const nvl_model* m) { return layered_kt_log2(m); }
 
 // x += rms(y) * w_post and / or xn = rms(x) * w_next (elem.h SandwichArgs)
 void sandwich(nvl_model* m, const float* y, int slices, int64_t slice_stride, const float* w_post, const float* w_next, const int32_t* rows_idx,
-              void* xn, int rows) {
-    KScope ks(m, KC_OTHER, 0, KS_SANDWICH, (double)rows * m->Hn * ((y ? 8.0 + 4.0 * std::max(slices, 1) : 4.0) + (w_next ? (double)m->wsize : 0.0)));
+              void* xn, int rows, bool raw_next = false) {
+    KScope ks(m, KC_OTHER, 0, KS_SANDWICH, (double)rows * m->Hn * ((y ? 8.0 + 4.0 * std::max(slices, 1) : 4.0) + (w_next || raw_next ? (double)m->wsize : 0.0)));
     SandwichArgs a{};
     a.x = m->x; a.y = y; a.slices = slices; a.slice_stride = slice_stride; a.w_post = w_post; a.w_next = w_next; a.rows_idx = rows_idx;
-    a.rows = rows; a.H = m->H; a.width = m->Hn; a.eps = m->cfg.norm_eps;
+    a.rows = rows; a.H = m->H; a.width = m->Hn; a.eps = m->cfg.norm_eps; a.raw_next = raw_next;
     if (!m->f32 && rows > 512 && m->H <= 4096 && slices <= 1) {
         const size_t lds = (size_t)16 * m->H * 2;
 #define NVL_SW16(CH)                                                                                                        \
@@ -523,7 +669,8 @@ void mix_latent(nvl_model* m, const LayerRun& r, const MixerW& w, const Meta& md
     const double ws = (double)m->wsize;
     in_proj(m, r, w, M);
     LatentArgs a{};
-    a.H = H; a.dim = c.dim; a.dp = r.dp; a.vp = r.vp; a.qrank = c.q_rank; a.qrp = r.qrp; a.kvrank = c.kv_rank; a.rp = r.rp;
+    a.H = H; a.dim = c.dim; a.dn = r.dn; a.dp = r.dp; a.rot = c.rot_dim; a.rotp = r.rotp; a.turn = r.turn;
+    a.own = m->mixers[(size_t)r.owner].dkv_norm != nullptr; a.gate_off = r.gate_off; a.gate_head = c.gate_per_head; a.vp = r.vp; a.qrank = c.q_rank; a.qrp = r.qrp; a.kvrank = c.kv_rank; a.rp = r.rp;
     a.window = c.window; a.scale = c.scale; a.eps = m->cfg.norm_eps;
     a.proj = m->lproj; a.proj_ld = m->lproj_ld; a.cq_norm = w.dq_norm; a.c_norm = w.dkv_norm; a.cq = m->lcq;
     a.cache = (char*)m->lat_cache + r.cache_off * (int64_t)m->wsize; a.block_stride = m->lat_block_stride; a.bs = m->Tmax;
@@ -533,7 +680,7 @@ void mix_latent(nvl_model* m, const LayerRun& r, const MixerW& w, const Meta& md
     a.kbase = md.kbase + (int64_t)r.win * m->opts.max_seqs;
     a.out = m->lmix; a.out_ld = r.ko;
     {
-        KScope ks(m, KC_OTHER, 0, KS_LAT_NORM, (double)M * (c.q_rank + c.kv_rank) * (4.0 + ws));
+        KScope ks(m, KC_OTHER, 0, KS_LAT_NORM, (double)M * (c.q_rank + (a.own ? c.kv_rank + c.rot_dim : 0)) * (4.0 + ws));
         if (m->f32) hipLaunchKernelGGL((latent_norm_kernel<float>), dim3(M), dim3(256), 0, m->stream, a);
         else hipLaunchKernelGGL((latent_norm_kernel<bf16_t>), dim3(M), dim3(256), 0, m->stream, a);
         NVL_HIP(hipGetLastError());
@@ -543,37 +690,39 @@ void mix_latent(nvl_model* m, const LayerRun& r, const MixerW& w, const Meta& md
     const int64_t rows = m->key_rows[(size_t)r.win];
     if (rows > 0) {                       // sequences on the expanded form
         if (rows > m->key_rows_cap) {
-            int64_t kc = 0, kk = 0, kv = 0;
+            int64_t kc = 0, kr = 0, kk = 0, kv = 0;
             for (const LayerRun& q : m->runs) if (q.c.mixer == NVL_MIXER_LATENT_ATTENTION) {
-                kc = std::max<int64_t>(kc, q.rp); kk = std::max<int64_t>(kk, (int64_t)q.c.heads * q.dp); kv = std::max<int64_t>(kv, (int64_t)q.c.heads * q.vp);
+                kc = std::max<int64_t>(kc, q.rp); kr = std::max<int64_t>(kr, q.rotp); kk = std::max<int64_t>(kk, (int64_t)q.c.heads * q.dn); kv = std::max<int64_t>(kv, (int64_t)q.c.heads * q.vp);
             }
             clear_graphs(m);
-            dfree(m->key_c); dfree(m->key_k); dfree(m->key_v);
-            m->key_c = m->key_k = m->key_v = nullptr; m->key_rows_cap = 0;
+            dfree(m->key_c); dfree(m->key_r); dfree(m->key_k); dfree(m->key_v);
+            m->key_c = m->key_r = m->key_k = m->key_v = nullptr; m->key_rows_cap = 0; m->key_src = -1;
             const int64_t cap = round_up(rows + rows / 4, 256) + 256, wsz = (int64_t)m->wsize;     // (+ whole GEMM tiles beyond the last row)
-            m->key_c = dmalloc_bytes(cap * kc * wsz); m->key_k = dmalloc_bytes(cap * kk * wsz); m->key_v = dmalloc_bytes(cap * kv * wsz);
+            m->key_c = dmalloc_bytes(cap * kc * wsz); m->key_r = dmalloc_bytes(std::max<int64_t>(cap * kr * wsz, 16)); m->key_k = dmalloc_bytes(cap * kk * wsz); m->key_v = dmalloc_bytes(cap * kv * wsz);
             NVL_HIP(hipMemsetAsync(m->key_c, 0, (size_t)(cap * kc * wsz), m->stream));
             NVL_HIP(hipMemsetAsync(m->key_k, 0, (size_t)(cap * kk * wsz), m->stream));
             NVL_HIP(hipMemsetAsync(m->key_v, 0, (size_t)(cap * kv * wsz), m->stream));
             m->key_rows_cap = cap - 256;
         }
-        a.cg = m->key_c; a.kx = m->key_k; a.vx = m->key_v; a.rows_pad = rows;
-        {
-            KScope ks(m, KC_OTHER, 0, KS_LAT_GATHER, 2.0 * (double)rows * c.kv_rank * ws);
+        a.cg = m->key_c; a.kr = m->key_r; a.kx = m->key_k; a.vx = m->key_v; a.rows_pad = rows;
+        if (m->key_src != r.src || m->key_win != r.win) {       // (else: the layer before this one read the same latents)
+            m->key_src = r.src; m->key_win = r.win;
+            KScope ks(m, KC_OTHER, 0, KS_LAT_GATHER, 2.0 * (double)rows * (c.kv_rank + c.rot_dim) * ws);
             const dim3 grid(cdiv(m->key_max[(size_t)r.win], 32), n_seqs);
             if (m->f32) hipLaunchKernelGGL((latent_gather_kernel<float>), grid, dim3(256), 0, m->stream, a);
             else hipLaunchKernelGGL((latent_gather_kernel<bf16_t>), grid, dim3(256), 0, m->stream, a);
             NVL_HIP(hipGetLastError());
         }
         m->site = KS_LAT_KV;
-        gemm(m, EPI_STORE, m->f32, mk(m->key_c, r.rp, w.uk, m->key_k, H * r.dp, nullptr, 1.f, (int)rows, H * r.dp, r.rp));
+        gemm(m, EPI_STORE, m->f32, mk(m->key_c, r.rp, w.uk, m->key_k, H * r.dn, nullptr, 1.f, (int)rows, H * r.dn, r.rp));
         m->site = KS_LAT_KV;
         if (m->f32) gemm(m, EPI_STORE, true, mk(m->key_c, r.rp, w.uv, m->key_v, H * r.vp, nullptr, 1.f, (int)rows, H * r.vp, r.rp));
         else gemm(m, EPI_STORE, false, mk(w.uv, r.rp, m->key_c, m->key_v, (int)rows, nullptr, 1.f, H * r.vp, (int)rows, r.rp));     // V^T = W_uv c^T
         {
             // visible (query, key) pairs are at most tokens x min(window, keys)
             const double pairs = (double)(M - m->n_abs) * (c.window > 0 ? std::min<double>(c.window, m->key_max[(size_t)r.win]) : 0.5 * m->key_max[(size_t)r.win]);
-            KScope ks(m, KC_ATTN, 2.0 * pairs * H * (c.dim + c.vdim), KS_ATTN, ((double)rows * H * (c.dim + c.vdim)) * ws + (double)M * H * (4.0 * c.dim + 4.0 * c.vdim + ws * c.vdim));
+            KScope ks(m, KC_ATTN, 2.0 * pairs * H * (c.dim + c.rot_dim + c.vdim), KS_ATTN,
+                      ((double)rows * (H * (c.dim + c.vdim) + c.rot_dim)) * ws + (double)M * H * (4.0 * (c.dim + c.rot_dim) + (c.gate_per_head ? 4.0 : 4.0 * c.vdim) + ws * c.vdim));
             if (m->f32 || r.dp > 256 || r.vp > 256 || c.scale == 0.f) {
                 const dim3 grid(max_len, H, n_seqs);
                 const size_t lds = (size_t)(r.dp + r.vp) * 4;
@@ -595,7 +744,9 @@ void mix_latent(nvl_model* m, const LayerRun& r, const MixerW& w, const Meta& md
                 if (r.dp == 256 && r.vp == 256) hipLaunchKernelGGL((latent_prefill_wide_kernel<8, 16>), dim3(H, n_seqs, cdiv(max_len, 64)), dim3(256), 0, m->stream, a);
                 else if (r.dp == 32) NVL_LPK(1);
                 else if (r.dp == 64) NVL_LPK(2);
+                else if (r.dp == 96) NVL_LPK(3);
                 else if (r.dp == 128) NVL_LPK(4);
+                else if (r.dp == 192) { if (r.vp == 32) NVL_LP(6, 2); else if (r.vp == 64) NVL_LP(6, 4); else NVL_LP(6, 8); }
                 else if (r.vp == 32) NVL_LP(8, 2); else if (r.vp == 64) NVL_LP(8, 4); else NVL_LP(8, 8);
 #undef NVL_LPK
 #undef NVL_LP
@@ -612,26 +763,28 @@ void mix_latent(nvl_model* m, const LayerRun& r, const MixerW& w, const Meta& md
         while (split < LAT_SPLITS && ht * n * split < 256 && split * 2 <= tiles && (split * 2) * n <= m->lat_abs_cap) split *= 2;
         a.n_split = split;
         {
-            KScope ks(m, KC_OTHER, 2.0 * n * H * (double)c.dim * c.kv_rank, KS_LAT_ABSORB, (double)H * c.dim * c.kv_rank * 2.0 + (double)n * H * (4.0 * c.dim + 2.0 * c.kv_rank));
-            hipLaunchKernelGGL(latent_absorb_q_kernel, dim3(H, r.rp / 64, cdiv(n, 16)), dim3(256), 0, m->stream, a);
+            KScope ks(m, KC_OTHER, 2.0 * n * H * (double)c.dim * c.kv_rank, KS_LAT_ABSORB, (double)H * c.dim * c.kv_rank * 2.0 + (double)n * H * (4.0 * (c.dim + c.rot_dim) + 2.0 * (c.kv_rank + c.rot_dim)));
+            hipLaunchKernelGGL(latent_absorb_q_kernel, dim3(H, r.rp / 64 + (c.rot_dim > 0), cdiv(n, 16)), dim3(256), 0, m->stream, a);
             NVL_HIP(hipGetLastError());
         }
         {
             const double keys = m->kv_tok > 0 && c.window > 0 ? std::min(m->kv_tok, (double)n * c.window) : (m->kv_tok > 0 ? m->kv_tok : (double)n * std::max(1, c.window));
-            KScope ks(m, KC_ATTN, 4.0 * keys * H * c.kv_rank, KS_ATTN, keys * c.kv_rank * 2.0 + (double)n * H * c.kv_rank * (2.0 + 4.0 * split));
+            KScope ks(m, KC_ATTN, keys * H * (4.0 * c.kv_rank + 2.0 * c.rot_dim), KS_ATTN, keys * (c.kv_rank + c.rot_dim) * 2.0 + (double)n * H * c.kv_rank * (2.0 + 4.0 * split));
             const dim3 grid(ht, n, split);
-#define NVL_LD(NRv)                                                                                                        \
+#define NVL_LDR(NRv, KRv)                                                                                                  \
             do {                                                                                                            \
                 constexpr int lds_ = latent_decode_lds_bytes<NRv>();                                                        \
-                NVL_LDS_ATTR((latent_decode_kernel<NRv>), lds_);                                                            \
-                hipLaunchKernelGGL((latent_decode_kernel<NRv>), grid, dim3(256), lds_, m->stream, a);                       \
+                NVL_LDS_ATTR((latent_decode_kernel<NRv, KRv>), lds_);                                                       \
+                hipLaunchKernelGGL((latent_decode_kernel<NRv, KRv>), grid, dim3(256), lds_, m->stream, a);                  \
             } while (0)
+#define NVL_LD(NRv) do { if (r.rotp == 0) NVL_LDR(NRv, 0); else if (r.rotp == 32) NVL_LDR(NRv, 1); else if (r.rotp == 64) NVL_LDR(NRv, 2); else NVL_LDR(NRv, 4); } while (0)
             switch (r.rp / 64) {
                 case 1: NVL_LD(1); break; case 2: NVL_LD(2); break; case 3: NVL_LD(3); break; case 4: NVL_LD(4); break;
                 case 6: NVL_LD(6); break; case 8: NVL_LD(8); break;
                 default: throw std::runtime_error("latent attention: no absorbed instance for this latent size");
             }
 #undef NVL_LD
+#undef NVL_LDR
             NVL_HIP(hipGetLastError());
         }
         {
@@ -745,6 +898,22 @@ LinRecArgs linrec_args(nvl_model* m, const LayerRun& r, const Meta& md) {
     return a;
 }
 
+// causal convolution + silu of the batch's raw rows into m->lconv, then the newest rows into the slots' rings
+void conv_launch(nvl_model* m, const LayerRun& r, const MixerW& w, const Meta& md, float* ring, const float* raw, int n_seqs, int M) {
+    ConvArgs v{};
+    v.raw = raw; v.raw_ld = m->lproj_ld; v.w = w.conv_w; v.b = w.conv_b; v.taps = r.c.conv_taps; v.channels = r.conv_dim;
+    v.out = m->lconv; v.out_ld = m->lconv_ld; v.ring = ring; v.ring_slot_stride = m->rec_slot_stride;
+    v.tok_seq = md.tok_seq; v.tok_pos = md.tok_pos; v.seq_tok_start = md.seq_tok_start; v.seq_len = md.seq_len; v.seq_pos = md.seq_pos; v.seq_slot = md.seq_slot;
+    const bool v4 = r.conv_dim % 4 == 0 && v.raw_ld % 4 == 0 && ((uintptr_t)v.raw & 15) == 0;
+    const dim3 cgrid(cdiv(M, CONV_TOKENS), cdiv(r.conv_dim, 1024));
+    if (v4 && v.taps == 4) hipLaunchKernelGGL((conv_silu_kernel<4>), cgrid, dim3(256), 0, m->stream, v, M);
+    else if (v4 && v.taps == 3) hipLaunchKernelGGL((conv_silu_kernel<3>), cgrid, dim3(256), 0, m->stream, v, M);
+    else if (v4 && v.taps == 2) hipLaunchKernelGGL((conv_silu_kernel<2>), cgrid, dim3(256), 0, m->stream, v, M);
+    else hipLaunchKernelGGL((conv_silu_kernel<0>), cgrid, dim3(256), 0, m->stream, v, M);
+    hipLaunchKernelGGL(conv_ring_kernel, dim3(n_seqs, cdiv(r.conv_dim, 256)), dim3(256), 0, m->stream, v);
+    NVL_HIP(hipGetLastError());
+}
+
 void mix_mamba2(nvl_model* m, const LayerRun& r, const MixerW& w, const Meta& md, int n_seqs, int M, int max_len) {
     const nvl_layer_config& c = r.c;
     const int inner = c.heads * c.vdim, GN = c.groups * c.state;
@@ -759,22 +928,11 @@ void mix_mamba2(nvl_model* m, const LayerRun& r, const MixerW& w, const Meta& md
         a.ring = ring; a.ring_slot_stride = m->rec_slot_stride;
     } else {
         KScope ks(m, KC_OTHER, 0, KS_MAMBA_CONV, (double)M * r.conv_dim * 8.0);
-        ConvArgs v{};
-        v.raw = m->lproj + inner; v.raw_ld = m->lproj_ld; v.w = w.conv_w; v.b = w.conv_b; v.taps = c.conv_taps; v.channels = r.conv_dim;
-        v.out = m->lconv; v.out_ld = m->lconv_ld; v.ring = ring; v.ring_slot_stride = m->rec_slot_stride;
-        v.tok_seq = md.tok_seq; v.tok_pos = md.tok_pos; v.seq_tok_start = md.seq_tok_start; v.seq_len = md.seq_len; v.seq_pos = md.seq_pos; v.seq_slot = md.seq_slot;
-        const bool v4 = r.conv_dim % 4 == 0 && v.raw_ld % 4 == 0 && ((uintptr_t)v.raw & 15) == 0;
-        const dim3 cgrid(cdiv(M, CONV_TOKENS), cdiv(r.conv_dim, 1024));
-        if (v4 && v.taps == 4) hipLaunchKernelGGL((conv_silu_kernel<4>), cgrid, dim3(256), 0, m->stream, v, M);
-        else if (v4 && v.taps == 3) hipLaunchKernelGGL((conv_silu_kernel<3>), cgrid, dim3(256), 0, m->stream, v, M);
-        else if (v4 && v.taps == 2) hipLaunchKernelGGL((conv_silu_kernel<2>), cgrid, dim3(256), 0, m->stream, v, M);
-        else hipLaunchKernelGGL((conv_silu_kernel<0>), cgrid, dim3(256), 0, m->stream, v, M);
-        hipLaunchKernelGGL(conv_ring_kernel, dim3(n_seqs, cdiv(r.conv_dim, 256)), dim3(256), 0, m->stream, v);
-        NVL_HIP(hipGetLastError());
+        conv_launch(m, r, w, md, ring, m->lproj + inner, n_seqs, M);
         a.v = m->lconv; a.k = m->lconv + inner; a.q = m->lconv + inner + GN; a.ld = m->lconv_ld;
     }
     linrec<false>(m, a, n_seqs, M, max_len, fused, KS_MAMBA_SCAN);
-    GatedNormArgs g{m->lo, m->lo_ld, m->lproj, m->lproj_ld, w.mix_norm, M, c.norm_groups, inner / c.norm_groups, m->cfg.norm_eps, r.ko, 0};
+    GatedNormArgs g{m->lo, m->lo_ld, m->lproj, m->lproj_ld, w.mix_norm, M, c.norm_groups, inner / c.norm_groups, m->cfg.norm_eps, r.ko, 0, 0};
     gated_norm<true>(m, g, KS_MAMBA_GATE);
 }
 
@@ -790,8 +948,119 @@ void mix_gla(nvl_model* m, const LayerRun& r, const MixerW& w, const Meta& md, i
     const bool fused = max_len <= REC_STEP_MAX;
     linrec<true>(m, a, n_seqs, M, max_len, fused, KS_GLA_SCAN);
     if (fused) return;
-    GatedNormArgs g{m->lo, m->lo_ld, a.gate, m->lproj_ld, w.mix_norm, M, c.heads, c.vdim, m->cfg.norm_eps, r.ko, 0};
+    GatedNormArgs g{m->lo, m->lo_ld, a.gate, m->lproj_ld, w.mix_norm, M, c.heads, c.vdim, m->cfg.norm_eps, r.ko, 0, 0};
     gated_norm<false>(m, g, KS_GLA_GATE);
+}
+
+void delta_step(nvl_model* m, const DeltaArgs& a, int n_seqs, bool fused) {
+    const int lds = delta_step_lds_bytes(a.DK, a.DVp, fused ? a.a_rkp + a.g_rkp : 0);
+    const dim3 grid(a.H, n_seqs);
+    int tv = 1;
+    while (tv < a.DVp / 4) tv <<= 1;
+    const int rows = cdiv(a.DK, LR_STEP_THREADS / tv);        // state rows per thread
+#define NVL_DS(FU, RO, ACT)                                                                                                  \
+    do {                                                                                                                     \
+        NVL_LDS_ATTR((delta_step_kernel<FU, RO, ACT>), 128 * 1024);                                                          \
+        hipLaunchKernelGGL((delta_step_kernel<FU, RO, ACT>), grid, dim3(LR_STEP_THREADS), lds, m->stream, a);                \
+    } while (0)
+#define NVL_DSR(FU, ACT) do { if (rows <= 4) NVL_DS(FU, 4, ACT); else if (rows <= 8) NVL_DS(FU, 8, ACT); else NVL_DS(FU, 16, ACT); } while (0)
+    if (!fused) NVL_DSR(false, float);
+    else if (m->f32) NVL_DSR(true, float);
+    else NVL_DSR(true, bf16_t);
+#undef NVL_DSR
+#undef NVL_DS
+    NVL_HIP(hipGetLastError());
+}
+
+void mix_delta(nvl_model* m, const LayerRun& r, const MixerW& w, const Meta& md, int n_seqs, int M, int max_len) {
+    const nvl_layer_config& c = r.c;
+    const int64_t qk = (int64_t)c.kv_heads * c.dim, hd = (int64_t)c.heads * c.dim, hv = (int64_t)c.heads * c.vdim;
+    in_proj(m, r, w, M);
+    DeltaArgs a{};
+    a.H = c.heads; a.G = c.kv_heads; a.DK = c.dim; a.DV = c.vdim; a.DVp = (int)round_up(c.vdim, 4);
+    a.q_scale = 1.0f / sqrtf((float)c.dim);
+    a.a_log = w.a_log; a.dt_bias = w.dt_bias;
+    a.beta = m->lproj + r.b_off; a.beta_ld = m->lproj_ld;
+    a.o = m->lo; a.o_ld = m->lo_ld;
+    a.state = m->rec_state + r.state_off; a.slot_stride = m->rec_slot_stride;
+    a.seq_tok_start = md.seq_tok_start; a.seq_len = md.seq_len; a.seq_pos = md.seq_pos; a.seq_slot = md.seq_slot;
+    a.len_lo = 1; a.len_hi = 1 << 30;
+    float* ring = m->rec_state + r.ring_off;
+    const double elems = (double)a.H * a.DK * a.DVp;
+    if (max_len == 1) {       // everything between the projections in one launch
+        a.raw = m->lproj; a.raw_ld = m->lproj_ld; a.conv_w = w.conv_w; a.taps = c.conv_taps; a.channels = r.conv_dim;
+        a.ring = ring; a.ring_slot_stride = m->rec_slot_stride;
+        a.a1 = m->lproj + r.a1_off; a.g1 = m->lproj + r.g1_off; a.lr_ld = m->lproj_ld;
+        a.a_rank = w.rank; a.g_rank = w.grank; a.a_rkp = w.a_rkp; a.g_rkp = w.g_rkp; a.a2 = w.a2r; a.g2 = w.g2r;
+        a.norm_w = w.mix_norm; a.eps = m->cfg.norm_eps; a.out = m->lmix; a.out_ld = r.ko;
+        KScope ks(m, KC_OTHER, 6.0 * M * elems, KS_DELTA_SCAN, 2.0 * n_seqs * elems * 4.0 + (double)M * (r.conv_dim * 4.0 * (c.conv_taps + 1) + hv * (double)m->wsize) +
+                                                                   ((double)hd * w.rank + (double)hv * w.grank) * (double)m->wsize);
+        delta_step(m, a, n_seqs, true);
+        return;
+    }
+    {
+        KScope ks(m, KC_OTHER, 0, KS_DELTA_CONV, (double)M * r.conv_dim * 8.0);
+        conv_launch(m, r, w, md, ring, m->lproj, n_seqs, M);
+    }
+    {
+        KScope ks(m, KC_OTHER, 0, KS_DELTA_PACK, (double)M * (w.rank + w.grank) * (4.0 + (double)m->wsize));
+        const PackArgs p{m->lproj + r.a1_off, m->lproj_ld, w.rank, w.a_rkp, w.grank, w.g_rkp, r.g1_off - r.a1_off, m->lpa, m->lpg};
+        if (m->f32) hipLaunchKernelGGL((pack_rows_kernel<float>), dim3(M), dim3(64), 0, m->stream, p);
+        else hipLaunchKernelGGL((pack_rows_kernel<bf16_t>), dim3(M), dim3(64), 0, m->stream, p);
+        NVL_HIP(hipGetLastError());
+    }
+    m->site = KS_DELTA_RANK;
+    gemm(m, EPI_STORE, true, mk(m->lpa, w.a_rkp, w.a2m, m->lz, (int)m->lz_ld, nullptr, 1.f, M, (int)hd, w.a_rkp));
+    m->site = KS_DELTA_RANK;
+    gemm(m, EPI_STORE, true, mk(m->lpg, w.g_rkp, w.g2m, m->lg, (int)m->lg_ld, nullptr, 1.f, M, (int)hv, w.g_rkp));
+    a.q = m->lconv; a.k = m->lconv + qk; a.v = m->lconv + 2 * qk; a.ld = m->lconv_ld;
+    a.z = m->lz; a.z_ld = m->lz_ld;
+    const double io = (double)M * (2.0 * qk + hd + 2.0 * hv) * 4.0;
+    const bool chunks = c.dim <= 256;
+    if (!chunks || m->min_len <= REC_STEP_MAX) {
+        a.len_hi = chunks ? REC_STEP_MAX : 1 << 30;
+        KScope ks(m, KC_OTHER, chunks ? 0.0 : 6.0 * M * elems, KS_DELTA_SCAN, chunks ? 0.0 : io + 2.0 * n_seqs * elems * 4.0);
+        delta_step(m, a, n_seqs, false);
+    }
+    if (chunks && max_len > REC_STEP_MAX) {
+        a.len_lo = REC_STEP_MAX + 1; a.len_hi = 1 << 30;
+        a.vec4 = c.dim % 4 == 0 && qk % 4 == 0 && a.ld % 4 == 0;
+        const int nk = c.dim <= 32 ? 2 : (c.dim <= 64 ? 4 : (c.dim <= 128 ? 8 : 16));
+        grow(m, m->delta_ws, m->delta_ws_cap, (int64_t)(m->opts.max_batch_tokens / DELTA_C + m->opts.max_seqs + 1) * c.heads * delta_ws_floats(nk * 16));
+        a.ws = m->delta_ws;
+        const dim3 pgrid(c.heads, n_seqs, cdiv(max_len, DELTA_C));
+        const double scratch = (double)M * c.heads * (3.0 * nk * 16 + 2.0 * c.vdim) * 4.0;
+        {
+            KScope ks(m, KC_OTHER, 0, KS_DELTA_PREP, io + scratch);
+#define NVL_DP(NKv)                                                                                                           \
+            do {                                                                                                              \
+                constexpr int lds_ = delta_prep_lds_bytes<NKv>();                                                              \
+                NVL_LDS_ATTR((delta_prep_kernel<NKv>), lds_);                                                                  \
+                hipLaunchKernelGGL((delta_prep_kernel<NKv>), pgrid, dim3(256), lds_, m->stream, a);                            \
+            } while (0)
+            if (nk == 2) NVL_DP(2); else if (nk == 4) NVL_DP(4); else if (nk == 8) NVL_DP(8); else NVL_DP(16);
+#undef NVL_DP
+            NVL_HIP(hipGetLastError());
+        }
+        {
+            KScope ks(m, KC_OTHER, 6.0 * M * elems, KS_DELTA_SCAN, scratch + 2.0 * n_seqs * elems * 4.0);
+            const int nw = nk == 2 || c.vdim <= 64 || c.heads * n_seqs * cdiv(c.vdim, 128) < 256 ? 4 : 8;
+            const dim3 sgrid(c.heads, n_seqs, cdiv(c.vdim, 16 * nw));
+#define NVL_DC(NKv, NWv)                                                                                                      \
+            do {                                                                                                              \
+                constexpr int lds_ = delta_scan_lds_bytes<NKv>();                                                              \
+                NVL_LDS_ATTR((delta_scan_kernel<NKv, NWv>), lds_);                                                             \
+                hipLaunchKernelGGL((delta_scan_kernel<NKv, NWv>), sgrid, dim3(NWv * 64), lds_, m->stream, a);                  \
+            } while (0)
+#define NVL_DCK(NKv) do { if (nw == 4) NVL_DC(NKv, 4); else NVL_DC(NKv, 8); } while (0)
+            if (nk == 2) NVL_DC(2, 4); else if (nk == 4) NVL_DCK(4); else if (nk == 8) NVL_DCK(8); else NVL_DCK(16);
+#undef NVL_DCK
+#undef NVL_DC
+            NVL_HIP(hipGetLastError());
+        }
+    }
+    GatedNormArgs g{m->lo, m->lo_ld, m->lg, m->lg_ld, w.mix_norm, M, c.heads, c.vdim, m->cfg.norm_eps, r.ko, 0, 1};
+    gated_norm<false>(m, g, KS_DELTA_GATE);
 }
 
 void tap_layer(nvl_model* m, int li, int M);
@@ -800,7 +1069,9 @@ void tap_layer(nvl_model* m, int li, int M);
 // in order: the last sandwich norm then leaves the final norm of every row in m->xn; returns whether it did.
 bool layered_stack(nvl_model* m, const Meta& md, int n_seqs, int M, int max_len, bool have_xn, bool all_rows) {
     auto W = [&](int li) -> const MixerW& { return m->mixers[(size_t)m->runs[(size_t)li].owner]; };
-    if (!have_xn) sandwich(m, nullptr, 0, 0, nullptr, W(0).norm1, nullptr, m->xn, M);
+    const bool post = m->cfg.block_style == NVL_BLOCK_POST;        // sublayers read x itself
+    m->key_src = m->key_win = -1;
+    if (!have_xn) sandwich(m, nullptr, 0, 0, nullptr, W(0).norm1, nullptr, m->xn, M, post);
     for (int li = 0; li < m->L; li++) {
         const LayerRun& r = m->runs[(size_t)li];
         const MixerW& w = W(li);
@@ -808,23 +1079,28 @@ bool layered_stack(nvl_model* m, const Meta& md, int n_seqs, int M, int max_len,
         switch (r.c.mixer) {
             case NVL_MIXER_LATENT_ATTENTION: mix_latent(m, r, w, md, n_seqs, M, max_len); break;
             case NVL_MIXER_MAMBA2: mix_mamba2(m, r, w, md, n_seqs, M, max_len); break;
+            case NVL_MIXER_CHANNEL_DELTA: mix_delta(m, r, w, md, n_seqs, M, max_len); break;
             default: mix_gla(m, r, w, md, n_seqs, M, max_len);
         }
         SubOut y = sub_out(m, KS_OPROJ, m->lmix, w.o, M, r.ko);
-        sandwich(m, y.y, y.slices, y.stride, w.norm1b, r.c.ffn_dim ? w.norm2 : after, nullptr, m->xn, M);
+        sandwich(m, y.y, y.slices, y.stride, w.norm1b, r.c.ffn_dim ? w.norm2 : after, nullptr, m->xn, M, post);
         if (r.c.ffn_dim) {
             m->site = KS_FFN_UP;
+            const bool clamped = m->cfg.activation_type == NVL_ACT_CLAMPED_GLU;
             if (m->f32) {
                 gemm(m, EPI_STORE, true, mk(m->xn, m->H, w.w1, m->h2, 2 * r.Fp, nullptr, 1.f, M, 2 * r.Fp, m->H));
                 const int64_t n = (int64_t)M * r.Fp;
                 KScope ks(m, KC_OTHER);
-                hipLaunchKernelGGL((swiglu_kernel<float, true>), dim3(cdiv(n, 256)), dim3(256), 0, m->stream, m->h2, (float*)m->hbuf, (int64_t)M, r.Fp);
+                if (clamped) hipLaunchKernelGGL((clamp_glu_kernel<float>), dim3(cdiv(n, 256)), dim3(256), 0, m->stream, m->h2, (float*)m->hbuf, (int64_t)M, r.Fp, r.c.ffn_limit, CLAMPED_GLU_SLOPE);
+                else hipLaunchKernelGGL((swiglu_kernel<float, true>), dim3(cdiv(n, 256)), dim3(256), 0, m->stream, m->h2, (float*)m->hbuf, (int64_t)M, r.Fp);
                 NVL_HIP(hipGetLastError());
             } else {
-                gemm(m, EPI_GEGLU, false, mk(m->xn, m->H, w.w1, m->hbuf, r.Fp, nullptr, 1.f, M, 2 * r.Fp, m->H));
+                GemmArgs up = mk(m->xn, m->H, w.w1, m->hbuf, r.Fp, nullptr, 1.f, M, 2 * r.Fp, m->H);
+                up.glu_limit = r.c.ffn_limit; up.glu_slope = CLAMPED_GLU_SLOPE;
+                gemm(m, clamped ? EPI_CLAMP_GLU : EPI_GEGLU, false, up);
             }
             y = sub_out(m, KS_FFN_DOWN, m->hbuf, w.w2, M, r.Fp);
-            sandwich(m, y.y, y.slices, y.stride, w.norm2b, after, nullptr, m->xn, M);
+            sandwich(m, y.y, y.slices, y.stride, w.norm2b, after, nullptr, m->xn, M, post);
         }
         tap_layer(m, li, M);
     }

@@ -613,7 +613,7 @@ __global__ __launch_bounds__(256) void conv_ring_kernel(ConvArgs p) {      // gr
 // ------------------------------------------------------------------------------------------
 // RMS norm over equal parts of a row with a silu gate, written as the next projection's operand.
 //   GATE_FIRST (Mamba-2):  u = y * silu(gate); out = rms(u) * w[column of the row]
-//   else (GLA)          :  out = rms(y) * w[column of the part] * silu(gate)
+//   else                :  out = rms(y) * w[column of the part] * silu(gate) (GLA), or * sigmoid(gate) with `sig` (delta rule)
 // V4: parts, row pitches and bases are multiples of 4 columns.  `lanes` (a power of two <= 64) lanes share a part, or one 256-thread
 // workgroup each when the parts are long (WIDE): grid ceil(tokens * parts / (256 / lanes)).
 // ------------------------------------------------------------------------------------------
@@ -625,6 +625,7 @@ struct GatedNormArgs {
     float eps;
     int64_t out_ld;
     int lanes;
+    int sig;
 };
 template <typename ActT, bool GATE_FIRST, bool WIDE, bool V4>
 __global__ __launch_bounds__(256) void gated_norm_kernel(GatedNormArgs p, ActT* __restrict__ out) {
@@ -685,7 +686,7 @@ __global__ __launch_bounds__(256) void gated_norm_kernel(GatedNormArgs p, ActT* 
         if (!GATE_FIRST) {
             const Vec s = ld(g, c);
 #pragma unroll
-            for (int e = 0; e < E; e++) x.v[e] *= lr_silu(s.v[e]);
+            for (int e = 0; e < E; e++) x.v[e] *= p.sig ? lr_sigmoid(s.v[e]) : lr_silu(s.v[e]);
         }
         if constexpr (V4) act_store4<ActT>(out, t, c0 + c, p.out_ld, f32x4{x.v[0], x.v[1], x.v[2], x.v[3]});
         else ActIO<ActT>::st(out + act_index<ActT>(t, c0 + c, p.out_ld), x.v[0]);

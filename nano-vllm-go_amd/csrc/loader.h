@@ -282,8 +282,13 @@ std::vector<float> to_f32(const StTensor& t) {
     return v;
 }
 
-// ---- models described by a list of layers ("Potuzen") ----
-const char* const LAYERED_ARCH = "Potuzen";
+// ---- models described by a list of layers ----
+struct LayeredArch { const char* name; int block_style, activation; float norm_offset; };
+const LayeredArch LAYERED_ARCHS[] = {{"Potuzen", NVL_BLOCK_SANDWICH, NVL_ACT_GEGLU, 0.f}, {"Lufazen", NVL_BLOCK_POST, NVL_ACT_CLAMPED_GLU, 1.f}};
+const LayeredArch* layered_arch(const std::string& name) {
+    for (const LayeredArch& a : LAYERED_ARCHS) if (name == a.name) return &a;
+    return nullptr;
+}
 double need_num(const JVal* o, const char* key, const std::string& where) {
     const JVal* v = o ? o->get(key) : nullptr;
     if (!v || v->kind != JVal::NUM) throw std::runtime_error(where + "number '" + key + "' expected");
@@ -294,7 +299,20 @@ int need_int(const JVal* o, const char* key, const std::string& where) {
     if (v != std::floor(v) || v < -2147483648.0 || v > 2147483647.0) throw std::runtime_error(where + "'" + key + "' is not an integer");
     return (int)v;
 }
-std::vector<nvl_layer_config> parse_layers(const JVal& raw) {
+// the rotation of a latent attention layer: {dims, base, scaling: null | {factor, original, fast, slow}}
+void parse_rotation(const JVal* mx, nvl_layer_config& c, const std::string& at) {
+    c.rot_dim = need_int(mx, "rot_dim", at);
+    const JVal* rot = mx->get("rot");
+    if (need_int(rot, "dims", at) != c.rot_dim) throw std::runtime_error(at + "rot.dims differs from rot_dim");
+    c.rot_base = need_num(rot, "base", at);
+    const JVal* sc = rot->get("scaling");
+    if (sc && sc->kind == JVal::OBJ) {
+        c.rot_factor = need_num(sc, "factor", at); c.rot_original = need_num(sc, "original", at);
+        c.rot_fast = need_num(sc, "fast", at); c.rot_slow = need_num(sc, "slow", at);
+    }
+}
+std::vector<nvl_layer_config> parse_layers(const JVal& raw, const LayeredArch& arch) {
+    const bool post = arch.block_style == NVL_BLOCK_POST;
     const JVal* ls = raw.get("layers");
     if (!ls || ls->kind != JVal::ARR || ls->arr.empty()) throw std::runtime_error("config: list 'layers' expected");
     std::vector<nvl_layer_config> out;
@@ -303,6 +321,7 @@ std::vector<nvl_layer_config> parse_layers(const JVal& raw) {
         const std::string at = "config: layer " + std::to_string(i) + ": ";
         nvl_layer_config c;
         memset(&c, 0, sizeof c);
+        c.kv_from = -1;
         const JVal *ty = e.get("type"), *mx = e.get("mixer"), *mlp = e.get("mlp"), *wo = e.get("weights_of");
         if (!ty || ty->kind != JVal::STR || !mx || mx->kind != JVal::OBJ) throw std::runtime_error(at + "'type' and 'mixer' expected");
         c.weights_of = wo && wo->kind == JVal::NUM ? need_int(&e, "weights_of", at) : -1;
@@ -311,16 +330,25 @@ std::vector<nvl_layer_config> parse_layers(const JVal& raw) {
             c.mixer = NVL_MIXER_LATENT_ATTENTION;
             c.dim = need_int(mx, "dim", at); c.q_rank = need_int(mx, "q_rank", at); c.kv_rank = need_int(mx, "kv_rank", at);
             c.scale = (float)need_num(mx, "scale", at);
+            if (post) {
+                parse_rotation(mx, c, at);
+                c.gate_per_head = 1;
+                const JVal* kf = mx->get("kv_from");
+                if (kf && kf->kind == JVal::NUM) c.kv_from = need_int(mx, "kv_from", at);
+            }
             const JVal* mask = mx->get("mask");
             if (mask && mask->kind == JVal::OBJ) {
                 c.window = need_int(mask, "size", at);
                 if (c.window <= 0) throw std::runtime_error(at + "the window is not positive");
             }
-        } else if (ty->str == "mamba2") {
+        } else if (ty->str == "channel_delta" && post) {
+            c.mixer = NVL_MIXER_CHANNEL_DELTA;
+            c.dim = need_int(mx, "dim", at); c.kv_heads = need_int(mx, "kv_heads", at); c.conv_taps = need_int(mx, "conv", at);
+        } else if (ty->str == "mamba2" && !post) {
             c.mixer = NVL_MIXER_MAMBA2;
             c.state = need_int(mx, "state", at); c.groups = need_int(mx, "groups", at); c.norm_groups = need_int(mx, "norm_groups", at);
             c.conv_taps = need_int(mx, "conv", at);
-        } else if (ty->str == "gla") {
+        } else if (ty->str == "gla" && !post) {
             c.mixer = NVL_MIXER_GLA;
             c.dim = need_int(mx, "dim", at); c.tau = (float)need_num(mx, "tau", at);
         } else throw std::runtime_error(at + "unknown mixer '" + ty->str + "'");
@@ -329,6 +357,7 @@ std::vector<nvl_layer_config> parse_layers(const JVal& raw) {
             if (kind && !(kind->kind == JVal::STR && kind->str == "dense")) throw std::runtime_error(at + "unknown feed-forward kind");
             c.ffn_dim = need_int(mlp, "ff", at);
             if (c.ffn_dim <= 0) throw std::runtime_error(at + "the feed-forward size is not positive");
+            if (arch.activation == NVL_ACT_CLAMPED_GLU) c.ffn_limit = (float)need_num(mlp, "limit", at);
         }
         out.push_back(c);
     }
@@ -338,6 +367,19 @@ void load_layered(nvl_model* m, const StSet& st) {
     const int OI = NVL_LAYOUT_OUT_IN;
     auto mat = [&](int kind, int layer, const std::string& name) { up2d(m, kind, layer, st.need(name), OI); };
     auto vec = [&](int kind, int layer, const std::string& name) { up1d(m, kind, layer, st.need(name)); };
+    auto cat = [&](int kind, int layer, const std::vector<std::string>& names) {      // tensors one after the other (along their rows)
+        const StTensor& a = st.need(names[0]);
+        std::vector<uint8_t> all;
+        int64_t rows = 0;
+        for (const std::string& n : names) {
+            const StTensor& t = st.need(n);
+            if (t.dtype != a.dtype || t.shape.size() != 2 || a.shape.size() != 2 || t.shape[1] != a.shape[1]) throw std::runtime_error("loader: " + names[0] + " and " + n + " do not match");
+            all.insert(all.end(), (const uint8_t*)t.data, (const uint8_t*)t.data + t.bytes);
+            rows += t.shape[0];
+        }
+        if (nvl_upload_tensor(m, kind, layer, all.data(), a.dtype, rows, a.shape[1], OI)) throw std::runtime_error(nvl_last_error(m));
+    };
+    const bool post = m->cfg.block_style == NVL_BLOCK_POST;
     mat(NVL_T_TOK_EMB, 0, "embed");
     mat(NVL_T_LM_HEAD, 0, "head");
     vec(NVL_T_FINAL_NORM_W, 0, "final.norm");
@@ -345,27 +387,32 @@ void load_layered(nvl_model* m, const StSet& st) {
         const LayerRun& r = m->runs[(size_t)i];
         if (r.owner != i) continue;
         const std::string l = "l" + std::to_string(i) + ".", x = l + "mix.";
-        vec(NVL_T_ATTN_NORM_W, i, l + "norm1"); vec(NVL_T_MIX_POST_NORM, i, l + "norm1b");
-        if (r.c.ffn_dim) {
-            vec(NVL_T_FFN_NORM_W, i, l + "norm2"); vec(NVL_T_FFN_POST_NORM, i, l + "norm2b");
-            const StTensor &g = st.need(l + "mlp.gate"), &u = st.need(l + "mlp.up");
-            if (u.dtype != g.dtype || u.shape != g.shape || g.shape.size() != 2) throw std::runtime_error("loader: " + l + "mlp.gate and .up do not match");
-            std::vector<uint8_t> cat(g.bytes + u.bytes);
-            memcpy(cat.data(), g.data, g.bytes);
-            memcpy(cat.data() + g.bytes, u.data, u.bytes);
-            if (nvl_upload_tensor(m, NVL_T_W1, i, cat.data(), g.dtype, 2 * g.shape[0], g.shape[1], OI)) throw std::runtime_error(nvl_last_error(m));
-            mat(NVL_T_W2, i, l + "mlp.down");
+        if (post) {
+            vec(NVL_T_MIX_POST_NORM, i, l + "norm1"); vec(NVL_T_MIX_SCALE, i, l + "ls1");
+            if (r.c.ffn_dim) { vec(NVL_T_FFN_POST_NORM, i, l + "norm2"); vec(NVL_T_FFN_SCALE, i, l + "ls2"); }
+        } else {
+            vec(NVL_T_ATTN_NORM_W, i, l + "norm1"); vec(NVL_T_MIX_POST_NORM, i, l + "norm1b");
+            if (r.c.ffn_dim) { vec(NVL_T_FFN_NORM_W, i, l + "norm2"); vec(NVL_T_FFN_POST_NORM, i, l + "norm2b"); }
         }
+        if (r.c.ffn_dim) { cat(NVL_T_W1, i, {l + "mlp.gate", l + "mlp.up"}); mat(NVL_T_W2, i, l + "mlp.down"); }
         switch (r.c.mixer) {
             case NVL_MIXER_LATENT_ATTENTION:
                 mat(NVL_T_LAT_DQ, i, x + "dq"); vec(NVL_T_LAT_DQ_NORM, i, x + "dq.norm"); mat(NVL_T_LAT_UQ, i, x + "uq");
-                mat(NVL_T_LAT_DKV, i, x + "dkv"); vec(NVL_T_LAT_DKV_NORM, i, x + "dkv.norm"); mat(NVL_T_LAT_UK, i, x + "uk"); mat(NVL_T_LAT_UV, i, x + "uv");
+                if (r.c.kv_from < 0) { mat(NVL_T_LAT_DKV, i, x + "dkv"); vec(NVL_T_LAT_DKV_NORM, i, x + "dkv.norm"); }
+                mat(NVL_T_LAT_UK, i, x + "uk"); mat(NVL_T_LAT_UV, i, x + "uv");
                 mat(NVL_T_MIX_GATE, i, x + "g"); mat(NVL_T_WO, i, x + "o");
                 break;
             case NVL_MIXER_MAMBA2:
                 mat(NVL_T_MAMBA_IN_PROJ, i, x + "in"); vec(NVL_T_MAMBA_CONV_W, i, x + "conv"); vec(NVL_T_MAMBA_CONV_B, i, x + "conv.b");
                 vec(NVL_T_MAMBA_DT_BIAS, i, x + "dt_bias"); vec(NVL_T_MAMBA_A_LOG, i, x + "A_log"); vec(NVL_T_MAMBA_D, i, x + "D");
                 vec(NVL_T_MAMBA_NORM, i, x + "norm"); mat(NVL_T_MAMBA_OUT_PROJ, i, x + "o");
+                break;
+            case NVL_MIXER_CHANNEL_DELTA:
+                mat(NVL_T_WQ, i, x + "q"); mat(NVL_T_WK, i, x + "k"); mat(NVL_T_WV, i, x + "v"); mat(NVL_T_WO, i, x + "o");
+                cat(NVL_T_DELTA_CONV, i, {x + "q.conv", x + "k.conv", x + "v.conv"}); mat(NVL_T_DELTA_BETA, i, x + "b");
+                vec(NVL_T_MAMBA_A_LOG, i, x + "A_log"); vec(NVL_T_GLA_NORM, i, x + "norm");
+                mat(NVL_T_GLA_A1, i, x + "a1"); mat(NVL_T_GLA_A2, i, x + "a2"); vec(NVL_T_GLA_A2_B, i, x + "dt_bias");
+                mat(NVL_T_DELTA_G1, i, x + "g1"); mat(NVL_T_DELTA_G2, i, x + "g2");
                 break;
             default:
                 mat(NVL_T_WQ, i, x + "q"); mat(NVL_T_WK, i, x + "k"); mat(NVL_T_WV, i, x + "v"); mat(NVL_T_MIX_GATE, i, x + "g"); mat(NVL_T_WO, i, x + "o");
@@ -381,8 +428,9 @@ extern "C" int nvl_load_layers_json(const char* path, nvl_layer_config* layers, 
         const std::string txt = nvl_loader::read_text(path);
         const JVal raw = nvl_loader::JParser(txt.c_str(), txt.size()).parse();
         const JVal* a = raw.get("architecture");
-        if (!a || a->kind != JVal::STR || a->str != LAYERED_ARCH) return 0;
-        const auto ls = parse_layers(raw);
+        const LayeredArch* arch = a && a->kind == JVal::STR ? layered_arch(a->str) : nullptr;
+        if (!arch) return 0;
+        const auto ls = parse_layers(raw, *arch);
         for (size_t i = 0; i < ls.size() && (int)i < cap; i++) layers[i] = ls[i];
         return (int)ls.size();
     } catch (const std::exception& e) {
@@ -529,13 +577,15 @@ extern "C" int nvl_load_config_json(const char* path, nvl_model_config* out) {
         memset(&c, 0, sizeof c);
         // ---- templates (config.go:125-376); `architecture` first, then model_type (:822-836, :975-1007), default GPT-2
         std::string arch = str("architecture");
-        if (arch == LAYERED_ARCH) {       // sizes and constants come from the file; it names no longest sequence
+        if (const LayeredArch* la = layered_arch(arch)) {       // sizes and constants come from the file; it names no longest sequence
             c.vocab_size = need_int(&raw, "vocab", "config: "); c.hidden = need_int(&raw, "width", "config: ");
-            c.num_layers = (int)parse_layers(raw).size();
+            c.num_layers = (int)parse_layers(raw, *la).size();
             c.norm_eps = (float)need_num(raw.get("norm"), "eps", "config: norm: ");
             c.max_seq_len = 4096;
             c.attention_type = NVL_ATTN_GQA; c.norm_type = NVL_NORM_RMS; c.position_type = NVL_POS_NONE;
-            c.activation_type = NVL_ACT_GEGLU; c.block_style = NVL_BLOCK_SANDWICH;
+            c.activation_type = la->activation; c.block_style = la->block_style; c.norm_weight_offset = la->norm_offset;
+            double cap;
+            if (num("logit_softcap", cap)) c.logit_softcap = (float)cap;
             *out = c;
             return NVL_OK;
         }

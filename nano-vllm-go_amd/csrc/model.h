@@ -16,6 +16,7 @@
 #include "sample.h"
 #include "gemm.h"
 #include "latent.h"
+#include "delta.h"
 #include "linrec.h"
 #include "mamba.h"
 #include "tp_p2p.h"
@@ -45,13 +46,17 @@ enum KClass { KC_GEMM = 0, KC_ATTN = 1, KC_OTHER = 2 };
 enum KSite { KS_OTHER = 0, KS_QKV, KS_ATTN, KS_OPROJ, KS_FFN_UP, KS_FFN_DOWN, KS_LM_HEAD, KS_NORM, KS_MOE_ROUTER, KS_MOE_PLAN,
              KS_MOE_UP, KS_MOE_DOWN, KS_MOE_COMBINE, KS_EMBED, KS_ARGMAX, KS_ROPE, KS_MAMBA_IN, KS_MAMBA_CONV, KS_MAMBA_SCAN,
              KS_MAMBA_GATE, KS_MAMBA_OUT, KS_ALLREDUCE, KS_MIX_IN, KS_LAT_NORM, KS_LAT_UQ, KS_LAT_GATHER, KS_LAT_KV, KS_LAT_ABSORB,
-             KS_LAT_UV, KS_GLA_SCAN, KS_GLA_GATE, KS_SANDWICH, KS_COUNT };
+             KS_LAT_UV, KS_GLA_SCAN, KS_GLA_GATE, KS_SANDWICH, KS_DELTA_CONV, KS_DELTA_PACK, KS_DELTA_RANK, KS_DELTA_PREP, KS_DELTA_SCAN, KS_DELTA_GATE, KS_COUNT };
 
 // one layer of a model described by a list of layers: its configuration, padded sizes, where its tensors and its memory are
 struct LayerRun {
     nvl_layer_config c{};
     int owner = -1;              // the layer whose tensors it uses
-    int dp = 0, vp = 0, rp = 0, qrp = 0;     // padded head / latent sizes (latent attention)
+    int dn = 0, dp = 0, vp = 0, rp = 0, qrp = 0, rotp = 0;     // padded head / latent sizes (latent attention)
+    int gate_off = 0;            // latent attention: first gate column of the fused input projection
+    int src = -1;                // latent attention: the layer whose cached latents it reads (itself, or kv_from)
+    const f32x2* turn = nullptr; // rotated latent attention: [position][rot / 2] (cos, sin)
+    int a1_off = 0, g1_off = 0, b_off = 0;   // channel delta: columns of the fused input projection
     int n_in = 0;                // columns of the fused input projection
     int ko = 0;                  // K of the output projection (padded)
     int Fp = 0;                  // feed-forward columns (padded), 0: none
@@ -68,6 +73,9 @@ struct MixerW {
     float *conv_w = nullptr, *conv_b = nullptr, *a_log = nullptr, *dskip = nullptr, *dt_bias = nullptr, *mix_norm = nullptr;
     float *a2 = nullptr, *a2_b = nullptr;
     int rank = 0;
+    void *a2m = nullptr, *g2m = nullptr;     // channel delta: the second decay / gate projections as GEMM operands ...
+    void *a2r = nullptr, *g2r = nullptr;     // ... and row-major for the one-token step
+    int grank = 0, a_rkp = 0, g_rkp = 0;
 };
 
 struct ProfRec { hipEvent_t a, b; int cls; double flops; int site, phase; double bytes; };
@@ -153,7 +161,10 @@ struct nvl_model {
     float *lproj = nullptr, *lq = nullptr, *ly = nullptr, *lconv = nullptr, *lo = nullptr;
     void *lcq = nullptr, *lmix = nullptr;
     int64_t lproj_ld = 0, lq_ld = 0, lo_ld = 0, lconv_ld = 0;
-    void *key_c = nullptr, *key_k = nullptr, *key_v = nullptr; int64_t key_rows_cap = 0;     // expanded latent attention, grown on demand
+    void *key_c = nullptr, *key_r = nullptr, *key_k = nullptr, *key_v = nullptr; int64_t key_rows_cap = 0;     // expanded latent attention, grown on demand
+    int key_src = -1, key_win = -1;    // whose latents key_c / key_r hold in the pass being enqueued
+    float *lz = nullptr, *lg = nullptr; void *lpa = nullptr, *lpg = nullptr; int64_t lz_ld = 0, lg_ld = 0;     // channel delta: decay / gate projections, their operands
+    float* delta_ws = nullptr; int64_t delta_ws_cap = 0;
     float *lat_part_o = nullptr, *lat_part_ml = nullptr; nvl::bf16_t* lat_qa = nullptr; int lat_abs_cap = 0;
     float *rec_z = nullptr, *rec_decay = nullptr; int64_t rec_z_floats = 0, rec_decay_floats = 0;
     // the batch being enqueued (layered_meta)

@@ -193,6 +193,7 @@ void gemm(nvl_model* m, int epi, bool out_f32, GemmArgs a, double flops = -1.0) 
             case EPI_SWIGLU: launch_gemm_bf16<EPI_SWIGLU, bf16_t>(st, a); break;
             case EPI_GELU:   launch_gemm_bf16<EPI_GELU, bf16_t>(st, a); break;
             case EPI_GEGLU:  launch_gemm_bf16<EPI_GEGLU, bf16_t>(st, a); break;
+            case EPI_CLAMP_GLU: launch_gemm_bf16<EPI_CLAMP_GLU, bf16_t>(st, a); break;
             case EPI_QKV:    launch_gemm_bf16<EPI_QKV, bf16_t>(st, a); break;
             default: throw std::runtime_error("gemm: bad epilogue");
         }
@@ -242,7 +243,7 @@ extern "C" int nvl_create(const nvl_model_config* cfg, const nvl_runtime_opts* o
     if (!cfg || !opts || !out) return fail(nullptr, NVL_ERR_INVALID, "nvl_create: null argument");
     *out = nullptr;
     const nvl_model_config& c = *cfg;
-    if (c.block_style == NVL_BLOCK_SANDWICH) return fail(nullptr, NVL_ERR_INVALID, "nvl_create: this model is described by a list of layers (nvl_create_layers)");
+    if (c.block_style == NVL_BLOCK_SANDWICH || c.block_style == NVL_BLOCK_POST) return fail(nullptr, NVL_ERR_INVALID, "nvl_create: this model is described by a list of layers (nvl_create_layers)");
     if (c.hidden <= 0 || c.num_layers <= 0 || c.num_heads <= 0 || c.head_dim <= 0 || c.vocab_size <= 0 ||
         c.max_seq_len <= 0)
         return fail(nullptr, NVL_ERR_INVALID, "nvl_create: non-positive model dimension");
@@ -256,7 +257,8 @@ extern "C" int nvl_create(const nvl_model_config* cfg, const nvl_runtime_opts* o
     // a 0-block KV cache): max_seqs >= 1 is required, max_batch_tokens 0 selects max_seq_len
     if (opts->max_seqs <= 0)
         return fail(nullptr, NVL_ERR_INVALID, "nvl_create: max_seqs must be >= 1 (KV slots / sequences per call)");
-    if (c.activation_type == NVL_ACT_GEGLU) return fail(nullptr, NVL_ERR_INVALID, "nvl_create: GEGLU is available to models described by a list of layers");
+    if (c.activation_type == NVL_ACT_GEGLU || c.activation_type == NVL_ACT_CLAMPED_GLU) return fail(nullptr, NVL_ERR_INVALID, "nvl_create: this activation is available to models described by a list of layers");
+    if (c.norm_weight_offset != 0.f || c.logit_softcap != 0.f) return fail(nullptr, NVL_ERR_INVALID, "nvl_create: norm_weight_offset and logit_softcap are available to models described by a list of layers");
     if (opts->max_batch_tokens < 0 || opts->kv_num_blocks < 0 || opts->kv_block_size < 0)
         return fail(nullptr, NVL_ERR_INVALID, "nvl_create: negative max_batch_tokens / kv_num_blocks / kv_block_size");
     const int tp = opts->tp_size > 1 ? opts->tp_size : 1;
@@ -1316,10 +1318,10 @@ void rope_kv(nvl_model* m, int li, const Meta& md, int M) {
     NVL_HIP(hipGetLastError());
 }
 
-void launch_argmax(hipStream_t st, float* logits, int ld, int V, int rows, float scaling, float* pval, int32_t* pidx,
+void launch_argmax(hipStream_t st, float* logits, int ld, int V, int rows, float scaling, float softcap, float* pval, int32_t* pidx,
                    int32_t* out) {
     const int chunks = cdiv(V, ARGMAX_CHUNK);
-    hipLaunchKernelGGL(argmax_partial_kernel, dim3(chunks, rows), dim3(256), 0, st, logits, ld, V, scaling, pval, pidx);
+    hipLaunchKernelGGL(argmax_partial_kernel, dim3(chunks, rows), dim3(256), 0, st, logits, ld, V, scaling, softcap, pval, pidx);
     if (out) hipLaunchKernelGGL(argmax_final_kernel, dim3(rows), dim3(64), 0, st, pval, pidx, chunks, out);
 }
 
@@ -1965,15 +1967,15 @@ int enqueue_forward(nvl_model* m, const Meta& md, int n_seqs, int M, int max_len
         gemm(m, EPI_STORE, true, mk(m->xn_last, H, m->lm_head, m->logits, m->Vpad, nullptr, 1.f, rows, m->V, H));
     }
     if (seam & 4) {      // sampling reads the logits: apply LogitsScaling here (argmax_partial_kernel does it otherwise)
-        if (c.logits_scaling != 0.f) {
+        if (c.logits_scaling != 0.f || c.logit_softcap != 0.f) {
             KScope ks(m, KC_OTHER);
             hipLaunchKernelGGL(scale_rows_kernel, dim3(cdiv(m->V, 256), rows), dim3(256), 0, m->stream, m->logits, m->Vpad, m->V,
-                               c.logits_scaling);
+                               c.logits_scaling, c.logit_softcap);
             NVL_HIP(hipGetLastError());
         }
     } else {
         KScope ks(m, KC_OTHER, 0, KS_ARGMAX, (double)rows * m->V * 4.0);
-        launch_argmax(m->stream, m->logits, m->Vpad, m->V, rows, c.logits_scaling, m->argmax_pval, m->argmax_pidx,
+        launch_argmax(m->stream, m->logits, m->Vpad, m->V, rows, c.logits_scaling, c.logit_softcap, m->argmax_pval, m->argmax_pidx,
                       (seam & 2) ? nullptr : m->argmax_dev);
         NVL_HIP(hipGetLastError());
     }
@@ -2711,7 +2713,7 @@ static const char* const k_site_names[KS_COUNT] = {
     "other", "qkv_proj", "attention", "o_proj", "ffn_up", "ffn_down", "lm_head", "norm", "moe_router", "moe_plan", "moe_up",
     "moe_down", "moe_combine", "embed", "argmax", "rope_kv", "mamba_in_proj", "mamba_conv", "mamba_scan", "mamba_gate_norm",
     "mamba_out_proj", "tp_allreduce", "mix_in_proj", "latent_norm", "latent_uq", "latent_gather", "latent_kv", "latent_absorb_q",
-    "latent_uv", "gla_scan", "gla_gate_norm", "sandwich_norm"};
+    "latent_uv", "gla_scan", "gla_gate_norm", "sandwich_norm", "delta_conv", "delta_pack", "delta_rank_out", "delta_prep", "delta_scan", "delta_gate_norm"};
 extern "C" const char* nvl_kernel_site_name(int site) { return site >= 0 && site < KS_COUNT ? k_site_names[site] : ""; }
 extern "C" int nvl_get_kernel_stats(nvl_model* m, nvl_kernel_stat* out, int cap) {
     if (!m || (cap > 0 && !out)) return NVL_ERR_INVALID;

@@ -317,7 +317,7 @@ extern "C" int nvl_op_argmax(int device, const float* x, int rows, int cols, int
     const int chunks = cdiv(cols, ARGMAX_CHUNK);
     float* pv = (float*)cx.alloc((int64_t)rows * chunks * 4);
     int32_t* pi = (int32_t*)cx.alloc((int64_t)rows * chunks * 4);
-    launch_argmax(cx.m.stream, dx, cols, cols, rows, 0.f, pv, pi, d);
+    launch_argmax(cx.m.stream, dx, cols, cols, rows, 0.f, 0.f, pv, pi, d);
     NVL_HIP(hipGetLastError());
     NVL_HIP(hipMemcpyAsync(out, d, (size_t)rows * 4, hipMemcpyDeviceToHost, cx.m.stream));
     NVL_HIP(hipStreamSynchronize(cx.m.stream));

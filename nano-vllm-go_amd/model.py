@@ -24,7 +24,7 @@ def _cfg_struct(cfg: dict) -> L.ModelConfigC:
     c.norm_eps = float(cfg.get("norm_eps", 1e-5))
     c.tied_embedding = int(bool(cfg.get("tied_embedding", False)))
     c.use_moe = int(bool(cfg.get("use_moe", False)))
-    for k in ("embedding_multiplier", "attention_multiplier", "residual_multiplier", "logits_scaling"):
+    for k in ("embedding_multiplier", "attention_multiplier", "residual_multiplier", "logits_scaling", "norm_weight_offset", "logit_softcap"):
         setattr(c, k, float(cfg.get(k, 0.0)))
     for k in ("mamba_expand", "mamba_state_size", "mamba_num_heads", "mamba_head_dim", "mamba_n_groups", "mamba_conv_kernel"):
         setattr(c, k, int(cfg.get(k, 0)))
