@@ -38,7 +38,7 @@ def parse():
     ap.add_argument("--gpus", type=int, default=1)
     ap.add_argument("--steps", type=int, default=3)
     ap.add_argument("--warmup", type=int, default=1)
-    ap.add_argument("--model", default="llama-3.2-1b", help="a synth.FULL_CONFIGS key; potuzen-2k / potuzen-4k are the Potuzen design at a real "
+    ap.add_argument("--model", default="llama-3.2-1b", help="a synth.FULL_CONFIGS key; lufazen-2k / -4k and potuzen-2k / -4k are those designs at a real "
                     "model's layer sizes, hybrid-2k / hybrid-4k the attention + Mamba-2 family at the same sizes")
     ap.add_argument("--batch", type=int, default=32, help="sequences per GPU")
     ap.add_argument("--prompt", type=int, default=512, help="prompt tokens per sequence")
@@ -84,7 +84,7 @@ def gen_weights_on_device(pkg, cfg, model, torch, device, keep_host: bool):
             g.manual_seed(42 + n)
             t = torch.randn(*shape, device=device, generator=g)
             u = torch.rand(*shape, device=device, generator=g)
-            t = {"matrix": lambda: t * shape[-1] ** -0.5, "norm": lambda: 1 + 0.02 * t, "conv": lambda: 0.3 * t, "bias": lambda: 0.5 * t,
+            t = {"matrix": lambda: t * shape[-1] ** -0.5, "norm": lambda: 1 + 0.02 * t, "norm0": lambda: 0.02 * t, "conv": lambda: 0.3 * t, "bias": lambda: 0.5 * t,
                  "dt_bias": lambda: 3.5 * u - 3, "a_log": lambda: torch.log(1 + 7 * u)}[kind]()
             model.upload(slot, layer, t.to(torch.bfloat16))
         return host

@@ -86,7 +86,11 @@ __device__ __forceinline__ float gelu_tanh_f(float x) {
 __device__ __forceinline__ float clamp_glu_f(float g, float u, float limit, float slope) {
     g = fminf(g, limit);
     u = fminf(fmaxf(u, -limit), limit);
-    return g / (1.0f + __expf(-slope * g)) * (u + 1.0f);
+    return g * (u + 1.0f) * __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(-1.4426950408889634f * slope * g));      // (exp2 -> inf: rcp gives 0)
+}
+// cap tanh(v / cap); the absolute error of tanh is ~1e-7 (as in gelu_tanh_f)
+__device__ __forceinline__ float softcap_f(float v, float cap, float inv_cap) {
+    return cap * (1.0f - 2.0f * __builtin_amdgcn_rcpf(__builtin_amdgcn_exp2f(v * inv_cap * 2.8853900817779268f) + 1.0f));
 }
 
 // ---- wave reductions (64 lanes) ----------------------------------------------

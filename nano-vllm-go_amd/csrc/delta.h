@@ -284,14 +284,15 @@ __global__ __launch_bounds__(256, NK > 8 ? 1 : 2) void delta_prep_kernel(DeltaAr
 }
 
 // ------------------------------------------------------------------------------------------
-// scan: grid (heads, sequences, slices of 16 NW value columns); wave w owns 16 columns and keeps their DK x 16 state in accumulators.
-// The next chunk's operands are on their way to registers while the current one's are used from LDS.
+// scan: grid (heads, sequences, slices of 16 NW / KSP value columns).  A wave keeps DK / KSP x 16 of the state in accumulators: 16 columns,
+// and with KSP > 1 (few heads and sequences) a part of the key channels — the parts' sums of U and O meet in LDS.
+// The next chunk's operands are on their way to registers while the state is updated.
 // ------------------------------------------------------------------------------------------
-template <int NK> constexpr int delta_scan_lds_bytes() { return 4 * (2 * DELTA_C * (NK * 16 + 4) + NK * 16 * 36 + NK * 16); }
+template <int NK, int NW, int KSP> constexpr int delta_scan_lds_bytes() { return 4 * (2 * DELTA_C * (NK * 16 + 4) + NK * 16 * 36 + NK * 16 + (KSP > 1 ? NW * 1024 : 0)); }
 
-template <int NK, int NW>
-__global__ __launch_bounds__(NW * 64, NK > 8 ? 1 : (NW == 8 ? 4 : 3)) void delta_scan_kernel(DeltaArgs p) {
-    constexpr int C = DELTA_C, DKP = NK * 16, LQ = DKP + 4, LK = 36, NT = NW * 64;
+template <int NK, int NW, int KSP>
+__global__ __launch_bounds__(NW * 64, NK > 8 ? 1 : (NW == 8 ? (KSP > 1 ? 2 : 4) : 3)) void delta_scan_kernel(DeltaArgs p) {
+    constexpr int C = DELTA_C, DKP = NK * 16, LQ = DKP + 4, LK = 36, NT = NW * 64, NKW = NK / KSP, NCG = NW / KSP;
     const int h = blockIdx.x, seq = blockIdx.y;
     const int n = p.seq_len[seq];
     if (n < p.len_lo || n > p.len_hi) return;
@@ -300,94 +301,139 @@ __global__ __launch_bounds__(NW * 64, NK > 8 ? 1 : (NW == 8 ? 4 : 3)) void delta
     float* ql = wl + C * LQ;             // [C][LQ]   Q'
     float* kl = ql + C * LQ;             // [DKP][LK] (K e^{b_end - b})^T
     float* dl = kl + DKP * LK;           // [DKP]     e^{b_end}
+    f32x4* xb = (f32x4*)(dl + DKP);      // KSP > 1: [part][column group][U, U, O, O][lane]
     const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6);
     const int fr = lane & 15, fg = lane >> 4;
-    const int col = (blockIdx.z * NW + wave) * 16 + fr;
+    const int cg = wave % NCG, kq = wave / NCG, ch0 = kq * NKW * 16;       // this wave's column group, part and first key channel
+    const int col = (blockIdx.z * NCG + cg) * 16 + fr;
     const bool live = col < p.DV, slive = col < p.DVp;
     const int64_t tok0 = p.seq_tok_start[seq];
     const bool fresh = p.seq_pos[seq] == 0;
     float* st = p.state + (int64_t)p.seq_slot[seq] * p.slot_stride + (int64_t)h * p.DK * p.DVp;
-    const int so = 4 * fg * p.DVp + col;
-    f32x4 S[NK];
+    f32x4 S[NKW];
+    {   // (clamped addresses instead of branches)
+        const int sc = min(col, p.DVp - 1);
 #pragma unroll
-    for (int i = 0; i < NK; i++)
+        for (int i = 0; i < NKW; i++)
 #pragma unroll
-        for (int r = 0; r < 4; r++) S[i][r] = !fresh && slive && 16 * i + 4 * fg + r < p.DK ? (st + (16 * i + r) * p.DVp)[so] : 0.f;
+            for (int r = 0; r < 4; r++) {
+                const int row = ch0 + 16 * i + 4 * fg + r;
+                const float x = st[min(row, p.DK - 1) * p.DVp + sc];
+                S[i][r] = !fresh && slive && row < p.DK ? x : 0.f;
+            }
+    }
     constexpr int E = 3 * C * DKP / 4, NL = E / NT;              // 16-byte pieces of a chunk's operands, per thread
-    static_assert(E % NT == 0 && NT >= DKP, "whole pieces, one decay per thread");
+    static_assert(NKW % 2 == 0 && NW % KSP == 0, "pairs of 16 channels");
+    static_assert(E % (3 * NT) == 0 && NT >= DKP, "whole pieces, one decay per thread");
     const int64_t stride = p.H * delta_ws_floats(DKP);
     const float* src = p.ws + (delta_chunk(p, seq, 0) * p.H + h) * delta_ws_floats(DKP);
-    f32x4 rg[NL], un[2], on[2];
+    f32x4 rg[NL], u[2], o[2];
     float rd = 0.f;
-    const float* vb = p.v + tok0 * p.ld + (int64_t)h * p.DV + col;
-    float* ob = p.o + tok0 * p.o_ld + (int64_t)h * p.DV + col;
-    auto fetch = [&](int c0) {
+    const int ld = (int)p.ld, old = (int)p.o_ld;
+    const char* vb = (const char*)(p.v + tok0 * p.ld + (int64_t)h * p.DV);
+    char* ob = (char*)(p.o + tok0 * p.o_ld + (int64_t)h * p.DV);
+    const uint32_t cb = 4 * min(col, p.DV - 1);
+    constexpr bool EARLY = NW == 4 || KSP > 1;       // registers for a whole chunk of lead
+    auto fetch = [&]() {
 #pragma unroll
-        for (int i = 0; i < NL; i++) rg[i] = *(const f32x4*)(src + (tid + i * NT) * 4);
-        if (tid < DKP) rd = src[3 * C * DKP + tid];
-        src += stride;
+        for (int i = 0; i < NL; i++) rg[i] = ((const f32x4*)src + i * NT)[tid];
+        rd = src[3 * C * DKP + min(tid, DKP - 1)];
+    };
+    // U0 and O0 of 32 tokens.  Beyond the sequence's end the last token is read again: finite, against zero columns of K, never stored.
+    auto fetch_uo = [&](const char* v, const char* oc, int left) {
+        if (KSP > 1 && kq > 0) {         // (wave-uniform: the first part starts from U0 and O0)
+            u[0] = u[1] = o[0] = o[1] = f32x4{0.f, 0.f, 0.f, 0.f};
+            return;
+        }
 #pragma unroll
         for (int tt = 0; tt < 2; tt++)
 #pragma unroll
             for (int r = 0; r < 4; r++) {
-                const int t = c0 + 16 * tt + 4 * fg + r;
-                const bool ok = live && t < n;
-                un[tt][r] = ok ? vb[t * p.ld] : 0.f;
-                on[tt][r] = ok ? ob[t * p.o_ld] : 0.f;
+                const uint32_t t = min(16 * tt + 4 * fg + r, left - 1);
+                const float x = *(const float*)(v + (t * (uint32_t)ld * 4 + cb));
+                u[tt][r] = live ? x : 0.f;                       // (the state's padding columns stay zero)
+                o[tt][r] = *(const float*)(oc + (t * (uint32_t)old * 4 + cb));
             }
     };
-    fetch(0);
+    fetch();
+    fetch_uo(vb, ob, n);
     for (int c0 = 0; c0 < n; c0 += C) {
         __syncthreads();                                         // the previous chunk's readers are done
+        float *w0 = wl + tid / (DKP / 4) * LQ + tid % (DKP / 4) * 4, *k0 = kl + (tid >> 3) * LK + (tid & 7) * 4;
 #pragma unroll
-        for (int i = 0; i < NL; i++) {
-            const int e = tid + i * NT;                          // 16-byte piece
-            if (e < 2 * C * DKP / 4) { const int row = e / (DKP / 4), d = e % (DKP / 4) * 4; *(f32x4*)(wl + row * LQ + d) = rg[i]; }
-            else { const int x = e - 2 * C * DKP / 4; *(f32x4*)(kl + (x >> 3) * LK + (x & 7) * 4) = rg[i]; }
-        }
+        for (int i = 0; i < NL; i++)
+            if (i < NL / 3 * 2) *(f32x4*)(w0 + i * (NT / (DKP / 4)) * LQ) = rg[i];
+            else *(f32x4*)(k0 + (i - NL / 3 * 2) * (NT / 8) * LK) = rg[i];
         if (tid < DKP) dl[tid] = rd;
-        f32x4 u[2] = {un[0], un[1]}, o[2] = {on[0], on[1]};
         __syncthreads();
-        if (c0 + C < n) fetch(c0 + C);
+        const bool more = c0 + C < n;                            // (the last chunk is fetched once more instead of a branch)
+        src += more ? stride : 0;
+        if (EARLY) fetch();
 #pragma unroll
-        for (int i = 0; i < NK; i++) {
+        for (int i = 0; i < NKW; i++) {
             f32x4 a[4];
 #pragma unroll
             for (int tt = 0; tt < 2; tt++) {
-                a[tt] = *(const f32x4*)(wl + (16 * tt + fr) * LQ + 16 * i + 4 * fg);
-                a[2 + tt] = *(const f32x4*)(ql + (16 * tt + fr) * LQ + 16 * i + 4 * fg);
+                a[tt] = *(const f32x4*)(wl + (16 * tt + fr) * LQ + ch0 + 16 * i + 4 * fg);
+                a[2 + tt] = *(const f32x4*)(ql + (16 * tt + fr) * LQ + ch0 + 16 * i + 4 * fg);
             }
 #pragma unroll
             for (int r = 0; r < 4; r++) {
                 u[0] = mfma_f32(a[0][r], S[i][r], u[0]); u[1] = mfma_f32(a[1][r], S[i][r], u[1]);
                 o[0] = mfma_f32(a[2][r], S[i][r], o[0]); o[1] = mfma_f32(a[3][r], S[i][r], o[1]);
             }
+            if (i & 1) __builtin_amdgcn_sched_barrier(0);        // (or all reads are hoisted to the front, and registers spill)
+        }
+        if constexpr (KSP > 1) {
+            f32x4* x = xb + (kq * NCG + cg) * 256 + lane;
+            x[0] = u[0]; x[64] = u[1]; x[128] = o[0]; x[192] = o[1];
+            __syncthreads();
+            u[0] = u[1] = o[0] = o[1] = f32x4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+            for (int q = 0; q < KSP; q++) {
+                const f32x4* y = xb + (q * NCG + cg) * 256 + lane;
+                u[0] += y[0]; u[1] += y[64];
+                if (kq == 0) o[0] += y[128];                     // (the first two parts store 16 tokens each)
+                if (kq == 1) o[1] += y[192];
+            }
         }
 #pragma unroll
         for (int tt = 0; tt < 2; tt++)
 #pragma unroll
             for (int r = 0; r < 4; r++) {
-                const int t = c0 + 16 * tt + 4 * fg + r;
-                if (live && t < n) ob[t * p.o_ld] = o[tt][r];
+                const int t = 16 * tt + 4 * fg + r;
+                if (live && c0 + t < n && (KSP == 1 || kq == tt)) *(float*)(ob + ((uint32_t)t * (uint32_t)old * 4 + cb)) = o[tt][r];
             }
+        f32x4 ub[2] = {u[0], u[1]};
+        __builtin_amdgcn_sched_barrier(0);
+        vb += more ? (int64_t)C * ld * 4 : 0; ob += more ? (int64_t)C * old * 4 : 0;
+        if (!EARLY) fetch();
+        fetch_uo(vb, ob, more ? n - c0 - C : n - c0);
+        __builtin_amdgcn_sched_barrier(0);
 #pragma unroll
-        for (int i = 0; i < NK; i++) S[i] *= *(const f32x4*)(dl + 16 * i + 4 * fg);
+        for (int i = 0; i < NKW; i += 2) {
+            f32x4 a[2][2];
 #pragma unroll
-        for (int sb = 0; sb < 2; sb++)
+            for (int x = 0; x < 2; x++)
 #pragma unroll
-            for (int i = 0; i < NK; i++) {
-                const f32x4 a = *(const f32x4*)(kl + (16 * i + fr) * LK + 16 * sb + 4 * fg);
+                for (int sb = 0; sb < 2; sb++) a[x][sb] = *(const f32x4*)(kl + (ch0 + 16 * (i + x) + fr) * LK + 16 * sb + 4 * fg);
+            S[i] *= *(const f32x4*)(dl + ch0 + 16 * i + 4 * fg);
+            S[i + 1] *= *(const f32x4*)(dl + ch0 + 16 * (i + 1) + 4 * fg);
 #pragma unroll
-                for (int r = 0; r < 4; r++) S[i] = mfma_f32(a[r], u[sb][r], S[i]);
-            }
+            for (int sb = 0; sb < 2; sb++)
+#pragma unroll
+                for (int r = 0; r < 4; r++) { S[i] = mfma_f32(a[0][sb][r], ub[sb][r], S[i]); S[i + 1] = mfma_f32(a[1][sb][r], ub[sb][r], S[i + 1]); }
+            __builtin_amdgcn_sched_barrier(0);
+        }
     }
-    int so_end = so;
-    asm volatile("" : "+v"(so_end));                             // (or the addresses of the first loads are kept in registers all along)
+    int so = 4 * fg * p.DVp + col;
+    asm volatile("" : "+v"(so));                                 // (or addresses are kept in registers all along)
+    st += ch0 * p.DVp;
 #pragma unroll
-    for (int i = 0; i < NK; i++)
+    for (int i = 0; i < NKW; i++)
 #pragma unroll
         for (int r = 0; r < 4; r++)
-            if (slive && 16 * i + 4 * fg + r < p.DK) (st + (16 * i + r) * p.DVp)[so_end] = S[i][r];
+            if (slive && ch0 + 16 * i + 4 * fg + r < p.DK) (st + (16 * i + r) * p.DVp)[so] = S[i][r];
 }
 
 // ------------------------------------------------------------------------------------------
@@ -417,7 +463,7 @@ template <bool FUSED, int ROWS, typename ActT>           // ROWS: state rows a t
 __global__ __launch_bounds__(LR_STEP_THREADS, ROWS <= 8 ? 4 : 2) void delta_step_kernel(DeltaArgs p) {
     constexpr int NT = LR_STEP_THREADS, NW = NT / 64;
     const int h = blockIdx.x, seq = blockIdx.y, tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
-    const int n = p.seq_len[seq];
+    const int n = FUSED ? 1 : p.seq_len[seq];
     if (n < p.len_lo || n > p.len_hi) return;
     extern __shared__ __attribute__((aligned(16))) float dl_sm[];
     const int DK4 = (p.DK + 3) & ~3;
@@ -458,6 +504,7 @@ __global__ __launch_bounds__(LR_STEP_THREADS, ROWS <= 8 ? 4 : 2) void delta_step
             const float* rw = p.raw + t * p.raw_ld;
             float* ring = p.ring + (int64_t)slot * p.ring_slot_stride;
             const int KD = p.G * p.DK;
+#pragma unroll 1
             for (int i = tid; i < 2 * p.DK + p.DV; i += NT) {
                 const int c = i < p.DK ? g * p.DK + i : (i < 2 * p.DK ? KD + g * p.DK + i - p.DK : 2 * KD + h * p.DV + i - 2 * p.DK);
                 const float cur = rw[c];
@@ -478,6 +525,7 @@ __global__ __launch_bounds__(LR_STEP_THREADS, ROWS <= 8 ? 4 : 2) void delta_step
             __syncthreads();
             // decay and gate projections: four lanes per output
             constexpr int CH = 16 / (int)sizeof(ActT);
+#pragma unroll 1
             for (int i = tid >> 2; i < p.DK + p.DV; i += NT / 4) {
                 const bool dec = i < p.DK;
                 const int rkp = dec ? p.a_rkp : p.g_rkp;

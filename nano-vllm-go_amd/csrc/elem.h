@@ -599,11 +599,24 @@ __global__ __launch_bounds__(256) void argmax_partial_kernel(float* __restrict__
     const int c1 = min(V, c0 + ARGMAX_CHUNK);
     float best = -INFINITY;
     int bi = 0x7fffffff;
+    if (softcap != 0.f) {                        // (all loads before the first store)
+        float v[ARGMAX_CHUNK / 256];
+#pragma unroll
+        for (int i = 0; i < ARGMAX_CHUNK / 256; i++) v[i] = row[min(c0 + (int)threadIdx.x + i * 256, c1 - 1)];
+#pragma unroll
+        for (int i = 0; i < ARGMAX_CHUNK / 256; i++) {
+            const int j = c0 + threadIdx.x + i * 256;
+            if (j >= c1) break;
+            if (logits_scaling != 0.f) v[i] = v[i] / logits_scaling;
+            v[i] = softcap_f(v[i], softcap, 1.0f / softcap);
+            row[j] = v[i];
+            if (v[i] > best) { best = v[i]; bi = j; }
+        }
+    } else
 #pragma unroll 4
     for (int j = c0 + threadIdx.x; j < c1; j += 256) {
         float v = row[j];
         if (logits_scaling != 0.f) { v = v / logits_scaling; row[j] = v; }
-        if (softcap != 0.f) { v = softcap * tanhf(v / softcap); row[j] = v; }
         if (v > best) { best = v; bi = j; }      // strict >, ascending j => first max per thread
     }
 #pragma unroll
@@ -638,7 +651,7 @@ __global__ void scale_rows_kernel(float* __restrict__ x, int ld, int n, float di
     float* p = x + (int64_t)blockIdx.y * ld + j;
     float v = *p;
     if (div != 0.f) v = v / div;
-    if (softcap != 0.f) v = softcap * tanhf(v / softcap);
+    if (softcap != 0.f) v = softcap_f(v, softcap, 1.0f / softcap);
     *p = v;
 }
 

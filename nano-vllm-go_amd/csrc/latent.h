@@ -29,6 +29,7 @@ struct LatentArgs {
     int H, dim, dn, dp, vp, qrank, qrp, kvrank, rp;   // dn / vp / qrp / rp: padded sizes; dp = dn + rotp: a head's columns of q
     int rot, rotp;                                // rotated dimensions per head (0: none), padded
     const f32x2* turn;                            // [position][rot / 2] (cos, sin)
+    int turn_q;                                   // whoever reads q turns it (16 | rot); else latent_turn_q_kernel has done it
     int window;                                   // 0: every earlier token
     float scale, eps;
     const float* proj; int64_t proj_ld;           // [token][c_q : qrp | c : rp | rotated key : rotp | gate] of the fused input projection
@@ -104,6 +105,19 @@ __global__ __launch_bounds__(256) void latent_norm_kernel(LatentArgs p) {
     for (int i = threadIdx.x; i < p.rotp; i += 256) ActIO<ActT>::st(kr + act_index<ActT>(row, i, p.rotp), lat_turn(p, pr + p.qrp + p.rp, i, pos));
 }
 
+// ---- q's rotated part in place, for sizes its readers do not turn themselves: grid (tokens, heads) ----
+__global__ __launch_bounds__(64) void latent_turn_q_kernel(LatentArgs p) {
+    const int64_t t = blockIdx.x;
+    float* q = (float*)p.q + t * p.q_ld + (int64_t)blockIdx.y * p.dp + p.dn;
+    const int half = p.rot >> 1;
+    for (int i = threadIdx.x; i < half; i += 64) {
+        const f32x2 cs = p.turn[(int64_t)p.tok_pos[t] * half + i];
+        const float u = q[i], v = q[i + half];
+        q[i] = u * cs[0] - v * cs[1];
+        q[i + half] = v * cs[0] + u * cs[1];
+    }
+}
+
 // ---- gather the latents a portion's keys need into contiguous rows: 32 rows (one unit of either layout) per workgroup ----
 template <typename ActT>
 __global__ __launch_bounds__(256) void latent_gather_kernel(LatentArgs p) {
@@ -148,12 +162,21 @@ __device__ __forceinline__ void latent_load_q(const LatentArgs& p, int64_t tok, 
     const float sg = p.scale < 0.f ? -1.f : 1.f;
 #pragma unroll
     for (int ks = 0; ks < KS; ks++) {
-        if (ks * 32 >= p.dn) {            // (uniform) the rotated part
+        f32x4 a = *(const f32x4*)(qp + ks * 32 + fg * 8), b = *(const f32x4*)(qp + ks * 32 + fg * 8 + 4);
+        const int j = ks * 32 - p.dn + fg * 8, half = p.rot >> 1;
+        if (p.turn_q && j >= 0 && j < p.rot) {      // eight dimensions on one side of the pairs (16 | rot)
+            const bool lo = j < half;
+            const float* other = qp + p.dn + (lo ? j + half : j - half);
+            const float* cs = (const float*)(p.turn + (int64_t)pos * half + (lo ? j : j - half));
+            const float sn = lo ? -1.f : 1.f;
 #pragma unroll
-            for (int e = 0; e < 8; e++) qf[ks][e] = (bf16_t)(lat_turn(p, qp + p.dn, ks * 32 - p.dn + fg * 8 + e, pos) * sg);
-            continue;
+            for (int e = 0; e < 4; e += 2) {
+                const f32x4 c0 = *(const f32x4*)(cs + 2 * e), c1 = *(const f32x4*)(cs + 2 * e + 8);
+                const f32x2 o0 = *(const f32x2*)(other + e), o1 = *(const f32x2*)(other + e + 4);
+                a[e] = fmaf(o0[0] * sn, c0[1], a[e] * c0[0]); a[e + 1] = fmaf(o0[1] * sn, c0[3], a[e + 1] * c0[2]);
+                b[e] = fmaf(o1[0] * sn, c1[1], b[e] * c1[0]); b[e + 1] = fmaf(o1[1] * sn, c1[3], b[e + 1] * c1[2]);
+            }
         }
-        const f32x4 a = *(const f32x4*)(qp + ks * 32 + fg * 8), b = *(const f32x4*)(qp + ks * 32 + fg * 8 + 4);
 #pragma unroll
         for (int e = 0; e < 4; e++) { qf[ks][e] = (bf16_t)(a[e] * sg); qf[ks][4 + e] = (bf16_t)(b[e] * sg); }
     }
@@ -403,7 +426,10 @@ __global__ __launch_bounds__(256) void latent_plain_kernel(LatentArgs p) {
     if (lo < 0) lo = 0;
     float* sq = lat_sm;
     float* so = sq + p.dp;
-    for (int i = tid; i < p.dp; i += 256) sq[i] = i < p.dn ? p.q[t * p.q_ld + h * p.dp + i] : lat_turn(p, p.q + t * p.q_ld + h * p.dp + p.dn, i - p.dn, pos);
+    for (int i = tid; i < p.dp; i += 256) {
+        const float* qh = p.q + t * p.q_ld + h * p.dp;
+        sq[i] = i < p.dn || !p.turn_q ? qh[i] : lat_turn(p, qh + p.dn, i - p.dn, pos);
+    }
     for (int i = tid; i < p.vp; i += 256) so[i] = 0.f;
     float m = -1e30f, l = 0.f;
     __syncthreads();
@@ -453,7 +479,8 @@ static __global__ __launch_bounds__(256) void latent_absorb_q_kernel(LatentArgs 
             const int j = mt * 16 + e / p.rotp, d = e % p.rotp;
             if (j >= p.n_abs) break;
             const int64_t t = p.abs_tok[j];
-            p.qa[((int64_t)j * p.Hp + h) * rt + p.rp + d] = (bf16_t)lat_turn(p, p.q + t * p.q_ld + h * p.dp + p.dn, d, p.tok_pos[t]);
+            const float* qr = p.q + t * p.q_ld + h * p.dp + p.dn;
+            p.qa[((int64_t)j * p.Hp + h) * rt + p.rp + d] = (bf16_t)(p.turn_q ? lat_turn(p, qr, d, p.tok_pos[t]) : qr[d]);
         }
         return;
     }

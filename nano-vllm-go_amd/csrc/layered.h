@@ -687,6 +687,12 @@ void mix_latent(nvl_model* m, const LayerRun& r, const MixerW& w, const Meta& md
     }
     m->site = KS_LAT_UQ;
     gemm(m, EPI_STORE, true, mk(m->lcq, r.qrp, w.uq, m->lq, H * r.dp, nullptr, 1.f, M, H * r.dp, r.qrp));
+    a.turn_q = c.rot_dim && c.rot_dim % 16 == 0;
+    if (c.rot_dim && !a.turn_q) {
+        KScope ks(m, KC_OTHER, 0, KS_ROPE, 8.0 * M * H * c.rot_dim);
+        hipLaunchKernelGGL(latent_turn_q_kernel, dim3(M, H), dim3(64), 0, m->stream, a);
+        NVL_HIP(hipGetLastError());
+    }
     const int64_t rows = m->key_rows[(size_t)r.win];
     if (rows > 0) {                       // sequences on the expanded form
         if (rows > m->key_rows_cap) {
@@ -1044,16 +1050,22 @@ void mix_delta(nvl_model* m, const LayerRun& r, const MixerW& w, const Meta& md,
         }
         {
             KScope ks(m, KC_OTHER, 6.0 * M * elems, KS_DELTA_SCAN, scratch + 2.0 * n_seqs * elems * 4.0);
-            const int nw = nk == 2 || c.vdim <= 64 || c.heads * n_seqs * cdiv(c.vdim, 128) < 256 ? 4 : 8;
-            const dim3 sgrid(c.heads, n_seqs, cdiv(c.vdim, 16 * nw));
-#define NVL_DC(NKv, NWv)                                                                                                      \
+            // columns per workgroup, and with few of them the key channels split over the waves too
+            const int pairs = c.heads * n_seqs;
+#define NVL_DC(NKv, NWv, KSPv)                                                                                                \
             do {                                                                                                              \
-                constexpr int lds_ = delta_scan_lds_bytes<NKv>();                                                              \
-                NVL_LDS_ATTR((delta_scan_kernel<NKv, NWv>), lds_);                                                             \
-                hipLaunchKernelGGL((delta_scan_kernel<NKv, NWv>), sgrid, dim3(NWv * 64), lds_, m->stream, a);                  \
+                constexpr int lds_ = delta_scan_lds_bytes<NKv, NWv, KSPv>();                                                   \
+                NVL_LDS_ATTR((delta_scan_kernel<NKv, NWv, KSPv>), lds_);                                                       \
+                hipLaunchKernelGGL((delta_scan_kernel<NKv, NWv, KSPv>), dim3(c.heads, n_seqs, cdiv(c.vdim, 16 * NWv / KSPv)), dim3(NWv * 64), lds_, m->stream, a); \
             } while (0)
-#define NVL_DCK(NKv) do { if (nw == 4) NVL_DC(NKv, 4); else NVL_DC(NKv, 8); } while (0)
-            if (nk == 2) NVL_DC(2, 4); else if (nk == 4) NVL_DCK(4); else if (nk == 8) NVL_DCK(8); else NVL_DCK(16);
+#define NVL_DCK(NKv, LOW)                                                                                                     \
+            do {                                                                                                              \
+                if (pairs * cdiv(c.vdim, 64) < 128) NVL_DC(NKv, 4, LOW);                                                       \
+                else if (pairs * cdiv(c.vdim, 128) < 256) NVL_DC(NKv, 8, 2);                                                   \
+                else if (c.vdim <= 64) NVL_DC(NKv, 4, 1);                                                                      \
+                else NVL_DC(NKv, 8, 1);                                                                                        \
+            } while (0)
+            if (nk == 2) NVL_DC(2, 4, 1); else if (nk == 4) NVL_DCK(4, 2); else if (nk == 8) NVL_DCK(8, 4); else NVL_DCK(16, 4);
 #undef NVL_DCK
 #undef NVL_DC
             NVL_HIP(hipGetLastError());

@@ -137,19 +137,29 @@ def tiny_config(family: str, **over) -> dict:
 
 def layered_shapes(cfg: dict, decay_rank: int = 16) -> list:
     """[(slot, layer, shape, kind)] of every tensor of a model described by a list of layers (cfg["layers"]: config.LAYER_FIELDS
-    dicts); kind: matrix | norm | conv | bias | dt_bias | a_log — how a synthetic checkpoint should draw it."""
-    H, V = cfg["hidden"], cfg["vocab_size"]
-    out = [("tok_emb", 0, (V, H), "matrix"), ("lm_head", 0, (V, H), "matrix"), ("final_norm_w", 0, (H,), "norm")]
+    dicts); kind: matrix | norm | norm0 (kept as a difference from one) | conv | bias | dt_bias | a_log — how a synthetic checkpoint
+    should draw it.  decay_rank: of the low-rank decay (and gate) projections whose rank the configuration leaves open."""
+    H, V, post = cfg["hidden"], cfg["vocab_size"], cfg["block_style"] == "post"
+    norm = "norm0" if cfg.get("norm_weight_offset") else "norm"
+    out = [("tok_emb", 0, (V, H), "matrix"), ("lm_head", 0, (V, H), "matrix"), ("final_norm_w", 0, (H,), norm)]
     for i, c in enumerate(cfg["layers"]):
         if c["weights_of"] >= 0:
             continue
         h, d, dv = c["heads"], c["dim"], c["vdim"]
-        t = [("attn_norm_w", (H,), "norm"), ("mix_post_norm", (H,), "norm")]
+        t = [("mix_scale", (H,), "norm")] if post else [("attn_norm_w", (H,), norm)]
+        t += [("mix_post_norm", (H,), norm)]
         if c["mixer"] == "latent_attention":
-            qr, kr = c["q_rank"], c["kv_rank"]
-            t += [("lat_dq", (qr, H), "matrix"), ("lat_dq_norm", (qr,), "norm"), ("lat_uq", (h * d, qr), "matrix"), ("lat_dkv", (kr, H), "matrix"),
-                  ("lat_dkv_norm", (kr,), "norm"), ("lat_uk", (h * d, kr), "matrix"), ("lat_uv", (h * dv, kr), "matrix"),
-                  ("mix_gate", (h * dv, H), "matrix"), ("wo", (H, h * dv), "matrix")]
+            qr, kr, rot = c["q_rank"], c["kv_rank"], c["rot_dim"]
+            t += [("lat_dq", (qr, H), "matrix"), ("lat_dq_norm", (qr,), "norm"), ("lat_uq", (h * (d + rot), qr), "matrix"), ("lat_uk", (h * d, kr), "matrix"),
+                  ("lat_uv", (h * dv, kr), "matrix"), ("mix_gate", (h if c["gate_per_head"] else h * dv, H), "matrix"), ("wo", (H, h * dv), "matrix")]
+            if c["kv_from"] < 0:
+                t += [("lat_dkv", (kr + rot, H), "matrix"), ("lat_dkv_norm", (kr,), "norm")]
+        elif c["mixer"] == "channel_delta":
+            qk, r = c["kv_heads"] * d, c["decay_rank"] or decay_rank
+            t += [("wq", (qk, H), "matrix"), ("wk", (qk, H), "matrix"), ("wv", (h * dv, H), "matrix"), ("wo", (H, h * dv), "matrix"),
+                  ("delta_conv", ((2 * qk + h * dv) * c["conv_taps"],), "conv"), ("delta_beta", (h, H), "matrix"), ("mamba_a_log", (h,), "a_log"),
+                  ("gla_norm", (dv,), "norm"), ("gla_a1", (r, H), "matrix"), ("gla_a2", (h * d, r), "matrix"), ("gla_a2_b", (h * d,), "dt_bias"),
+                  ("delta_g1", (r, H), "matrix"), ("delta_g2", (h * dv, r), "matrix")]
         elif c["mixer"] == "mamba2":
             inner, conv = h * dv, h * dv + 2 * c["groups"] * c["state"]
             t += [("mamba_in_proj", (inner + conv + h, H), "matrix"), ("mamba_conv_w", (conv * c["conv_taps"],), "conv"), ("mamba_conv_b", (conv,), "bias"),
@@ -161,7 +171,8 @@ def layered_shapes(cfg: dict, decay_rank: int = 16) -> list:
                   ("gla_a2", (h * d, decay_rank), "matrix"), ("gla_a2_b", (h * d,), "bias")]
         if c["ffn_dim"]:
             F = c["ffn_dim"]
-            t += [("ffn_norm_w", (H,), "norm"), ("ffn_post_norm", (H,), "norm"), ("w1", (2 * F, H), "matrix"), ("w2", (H, F), "matrix")]
+            t += [("ffn_scale", (H,), "norm")] if post else [("ffn_norm_w", (H,), norm)]
+            t += [("ffn_post_norm", (H,), norm), ("w1", (2 * F, H), "matrix"), ("w2", (H, F), "matrix")]
         out += [(slot, i, shape, kind) for slot, shape, kind in t]
     return out
 
@@ -175,6 +186,22 @@ def _potuzen(width: int, layers: int, heads: int, q_rank: int, ff: int, window: 
     return dict(vocab_size=32000, hidden=width, num_layers=layers, num_heads=0, num_kv_heads=0, head_dim=0, ffn_dim=0, max_seq_len=4096,
                 attention_type="gqa", norm_type="rmsnorm", position_type="nope", activation_type="geglu", block_style="sandwich",
                 rope_base=0.0, norm_eps=1e-6, tied_embedding=False, layers=[dict(LAYER_FIELDS, ffn_dim=ff, **kinds[i % 3]) for i in range(layers)])
+
+
+def _lufazen(width: int, layers: int, heads: int, q_rank: int, ff: int) -> dict:
+    """A Lufazen model at a real model's layer sizes: rotated latent attention (every other one reads the latents of the one before it)
+    and two channel-wise delta rules in turn."""
+    from .config import LAYER_FIELDS
+    lat = dict(mixer="latent_attention", heads=heads, dim=128, vdim=128, q_rank=q_rank, kv_rank=512, scale=192 ** -0.5, rot_dim=64, gate_per_head=1,
+               rot_base=1e6, rot_factor=4.0, rot_original=4096.0, rot_fast=32.0, rot_slow=1.0)
+    delta = dict(mixer="channel_delta", heads=heads, kv_heads=heads, dim=128, vdim=128, conv_taps=4, decay_rank=128)
+    kinds = [lat, delta, delta]
+    ls = [dict(LAYER_FIELDS, ffn_dim=ff, ffn_limit=7.0, **kinds[i % 3]) for i in range(layers)]
+    for i in range(3, layers, 6):
+        ls[i]["kv_from"] = i - 3
+    return dict(vocab_size=32000, hidden=width, num_layers=layers, num_heads=0, num_kv_heads=0, head_dim=0, ffn_dim=0, max_seq_len=4096,
+                attention_type="gqa", norm_type="rmsnorm", position_type="nope", activation_type="clamped_glu", block_style="post",
+                rope_base=0.0, norm_eps=1e-5, tied_embedding=False, norm_weight_offset=1.0, logit_softcap=30.0, layers=ls)
 
 
 def _hybrid(hidden: int, layers: int, heads: int, ff: int) -> dict:
@@ -210,7 +237,8 @@ FULL_CONFIGS = {
                        ffn_dim=14336, max_seq_len=4096, attention_type="gqa", norm_type="rmsnorm",
                        position_type="rope", activation_type="swiglu", block_style="sequential",
                        rope_base=500000.0, norm_eps=1e-5, tied_embedding=False),
-    # the Potuzen design at a real model's layer sizes, and the closest other family at the same sizes
+    # designs described by a list of layers at a real model's layer sizes, and the closest other family at the same sizes
+    "lufazen-2k": _lufazen(2048, 12, 16, 768, 6144), "lufazen-4k": _lufazen(4096, 6, 32, 1536, 12288),
     "potuzen-2k": _potuzen(2048, 12, 16, 768, 6144), "hybrid-2k": _hybrid(2048, 12, 16, 6144),
     "potuzen-4k": _potuzen(4096, 6, 32, 1536, 12288), "hybrid-4k": _hybrid(4096, 6, 32, 12288),
 }

@@ -5,62 +5,20 @@ import json
 import os
 import subprocess
 import sys
+from functools import partial
 from pathlib import Path
 
 import numpy as np
 import pytest
 
+import layered_helpers as H
 import potuzen_models as PM
 import potuzen_oracle as O
+from layered_helpers import TOL, build, cut, err, feed
 
 pytestmark = pytest.mark.gpu
 ROOT = Path(__file__).resolve().parent.parent
-TOL = {"f32": 1e-4, "bf16": 0.12}       # at any position: rms over the vocabulary of the difference / rms of the logits
-
-
-def build(gpu, d, cfg, w, precision="f32", **kw):
-    PM.write(d, cfg, w)
-    kw = dict(dict(max_seq_len=1024, max_seqs=4, max_batch_tokens=1024, kv_num_blocks=64, kv_block_size=64, kv_pool=True), **kw)
-    return gpu.HipTransformerModel.from_pretrained(str(d), precision=precision, **kw)
-
-
-def err(got, want, precision="f32"):
-    """The worst position.  bf16: leaving out 3 in 100 — a norm over a nearly vanishing vector (a Mamba-2 head whose C . B dt is close to
-    -D, say) turns the rounding of its input into a flipped sign at single positions, in any implementation."""
-    d = np.asarray(got, np.float64) - want
-    e = np.sort((np.sqrt((d ** 2).mean(axis=-1)) / np.sqrt((want ** 2).mean())).reshape(-1))
-    return float(e[-1 - (e.size * 3 // 100 if precision == "bf16" else 0)])
-
-
-def steady(cfg, w, draw, limit=0.035):
-    """Tokens from draw() on which the model is well conditioned: a norm over a nearly vanishing vector can blow up rounding at single
-    positions, and tells nothing about the device.  Measured on the restatement, with the embeddings perturbed by a bf16 rounding."""
-    e = np.asarray(w["embed"], np.float64)
-    noisy = [dict(w, embed=e * (1 + np.random.default_rng(i).uniform(-1, 1, e.shape) * 2.0 ** -9)) for i in range(3)]
-    for _ in range(100):
-        tok = list(draw())
-        want = O.forward(cfg, w, tok)
-        if all(err(O.forward(cfg, n, tok), want) < limit for n in noisy):
-            return tok, want
-    raise AssertionError("no well-conditioned sequence found")
-
-
-def feed(m, seq, tokens, cuts):
-    """All logits of `tokens` fed in portions; the sequence stays open."""
-    if m.seq_len(seq) < 0:
-        m.seq_open(seq)
-    out, at = [], m.seq_len(seq)
-    for n in cuts:
-        part = tokens[at:at + n]
-        out.append(m.forward_rows([seq], [part], [at], range(len(part)))[0])
-        at += n
-    assert at == len(tokens)
-    return np.concatenate(out)
-
-
-def cut(total, n):
-    return [n] * (total // n) + ([total % n] if total % n else [])
-
+steady, greedy_oracle = partial(H.steady, O), partial(H.greedy_oracle, O)
 
 SINGLE = {
     "latent-odd": (PM.latent(), 96), "latent-64": (PM.latent(heads=6, dim=64, vdim=64, q_rank=96, kv_rank=64, window=64), 128),
@@ -168,37 +126,10 @@ def test_mixed_batches_and_reuse(gpu, tmp_path, stack, precision):
     """Portions of some sequences beside single tokens of others, sequences left out of steps, slots and blocks given back and used
     again: every logit as if the sequence were alone.  The pool is exactly as large as the live sequences need."""
     cfg, w, seqs, want = stack
-    g = np.random.default_rng(17)
     need = sum(-(-len(s) // 64) for s in seqs)
     m = build(gpu, tmp_path, cfg, w, precision, max_seqs=4, kv_num_blocks=need)
-    live, todo, done, sid = {}, [0, 1, 2, 3, 1, 3, 2, 0, 3, 1], 0, 100
-    used, seen = set(), []
-    while todo or live:
-        while todo and len(live) < 4 and todo[0] not in {v[0] for v in live.values()}:
-            live[sid] = [todo.pop(0), 0]
-            m.seq_open(sid)
-            sid += 1
-        ids = [s for s in live if g.random() < 0.8] or list(live)[:1]
-        toks, pos = [], []
-        for s in ids:
-            k, at = live[s]
-            n = int(g.choice([1, 1, 1, 2, 5, 16, 30, 64, 90]))
-            toks.append(seqs[k][at:at + n])
-            pos.append(at)
-        total = sum(map(len, toks))
-        rows = sorted(g.choice(total, min(total, 40), replace=False).tolist())
-        got, am = m.forward_rows(ids, toks, pos, rows)
-        ref = np.concatenate([want[live[s][0]][p:p + len(t)] for s, t, p in zip(ids, toks, pos)])[rows]
-        assert np.array_equal(am, got.argmax(axis=1))
-        seen.append((got, ref))
-        for s, t in zip(ids, toks):
-            live[s][1] += len(t)
-            if live[s][1] == len(seqs[live[s][0]]):
-                used.add(live.pop(s)[0])
-                m.seq_close(s)
-                done += 1
-    assert done == 10 and used == {0, 1, 2, 3}
-    assert err(np.concatenate([a for a, _ in seen]), np.concatenate([b for _, b in seen]), precision) < TOL[precision]
+    got, ref = H.mixed_run(m, seqs, want, [0, 1, 2, 3, 1, 3, 2, 0, 3, 1], 17)
+    assert err(got, ref, precision) < TOL[precision]
     m.close()
 
 
@@ -277,15 +208,6 @@ def test_far_key_among_hundreds(gpu, tmp_path, precision):
 
 
 # ---- the framework's own entry points ----
-def greedy_oracle(cfg, w, prompt, n):
-    tok, gaps = list(prompt), []
-    for _ in range(n):
-        lg = np.sort(O.forward(cfg, w, tok)[-1])
-        gaps.append(lg[-1] - lg[-2])
-        tok.append(int(O.forward(cfg, w, tok)[-1].argmax()))
-    return tok[len(prompt):], min(gaps)
-
-
 def test_greedy_generation(gpu, tmp_path, stack):
     """Stepwise, fused on the device, and through the runner give the restatement's tokens (fp32)."""
     cfg, w, seqs, _ = stack
