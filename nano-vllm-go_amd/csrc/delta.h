@@ -12,11 +12,11 @@
 //     u_t = beta_t (v_t - (k_t e^{b_t})^T S_in - sum_{s<t} M[t][s] u_s),      M[t][s] = sum_c k_t[c] k_s[c] e^{b_t[c] - b_s[c]}
 //     o_t = (q_t e^{b_t})^T S_in + sum_{s<=t} A[t][s] u_s,                    A[t][s] = sum_c q_t[c] k_s[c] e^{b_t[c] - b_s[c]}
 //     S_out = diag(e^{b_end}) S_in + sum_s (k_s e^{b_end - b_s}) u_s^T
-// With T = (I + diag(beta) M)^-1 diag(beta):  U = U0 - W S_in,  U0 = T V,  W = T (K e^b);  O = O0 + Q' S_in,  O0 = A U0,
-// Q' = Q e^b - A W.  prep leaves -W, Q', (K e^{b_end - b})^T and e^{b_end} in scratch, U0 in the place of v and O0 in the place of o.
+// With T = (I + diag(beta) M)^-1 diag(beta):  U = U0 - W S_in,  U0 = T V,  W = T (K e^b);  O = O0 + Q' S_in,  O0 = (A T) V,
+// Q' = Q e^b - (A T) (K e^b).  prep leaves -W, Q', (K e^{b_end - b})^T and e^{b_end} in scratch, U0 in the place of v and O0 in the place of o.
 // Every exponent that is evaluated is <= 0: a decay per channel cannot be split into e^{b_t} e^{-b_s}, so the two 16 x 16 diagonal
-// blocks of A and M are summed pair by pair, and the block below the diagonal takes token 15's sums as its reference.  T comes from
-// forward substitution (16 x 16 blocks): the powers of M that a series would need can be far larger than T itself.
+// blocks of A and M are summed pair by pair, and the block below the diagonal takes token 15's sums as its reference.  T is built
+// block by block from exact inverses: the powers of M that a series would need can be far larger than T itself.
 // Products are v_mfma_f32_16x16x4_f32: operand element i of lane group g stands for k = 16 n + 4 g + i on both sides, so that an
 // accumulator (lane = column, rows 4 g + r) is the B operand of the next product as it stands.
 #pragma once
@@ -38,7 +38,7 @@ struct DeltaArgs {
     float* o; int64_t o_ld;            // [token][H * DV]
     float* state; int64_t slot_stride; // slot s: state + s * slot_stride, [H][DK][DVp]
     const int32_t *seq_tok_start, *seq_len, *seq_pos, *seq_slot;
-    int vec4;                          // q, k rows may be read 16 bytes at a time
+    int vec4, vec4v;                   // q, k / v, o rows may be accessed 16 bytes at a time
     int len_lo, len_hi;                // sequences with len_lo <= tokens of this call <= len_hi are served, the others skipped
     float* ws;                         // chunk c of sequence i is (seq_tok_start / 32 + i + c); per chunk and head delta_ws_floats
     // FUSED step: raw [q | k | v] columns before the convolution, a ring of the last `taps` raw rows per slot
@@ -52,14 +52,20 @@ constexpr int DELTA_C = 32;            // tokens per chunk
 static inline __host__ __device__ int64_t delta_ws_floats(int dkp) { return (int64_t)dkp * (3 * DELTA_C + 1); }     // -W | Q' | K^T | e^{b_end}
 __device__ __forceinline__ int64_t delta_chunk(const DeltaArgs& p, int seq, int c) { return p.seq_tok_start[seq] / DELTA_C + seq + c; }
 
+// log(1 + e^x) from the hardware's base-2 exponential and logarithm; what 1 + y rounds away is added back
+__device__ __forceinline__ float delta_softplus(float x) {
+    const float y = ex2(-1.4426950408889634f * fabsf(x)), u = 1.0f + y;
+    return fmaxf(x, 0.f) + fmaf(0.6931471805599453f, __builtin_amdgcn_logf(u), (y - (u - 1.0f)) * __builtin_amdgcn_rcpf(u));
+}
+
 // ------------------------------------------------------------------------------------------
-// prep: grid (heads, sequences, chunks), 4 waves
+// prep: grid (heads, sequences, chunks), 8 waves
 // ------------------------------------------------------------------------------------------
-template <int NK> constexpr int delta_prep_lds_bytes() { return 4 * (3 * DELTA_C * (NK * 16 + 4) + 2 * DELTA_C * 36 + DELTA_C + 256); }
+template <int NK> constexpr int delta_prep_lds_bytes() { return 4 * (3 * DELTA_C * (NK * 16 + 4) + 2 * DELTA_C * 36 + DELTA_C + 512); }
 
 template <int NK>
-__global__ __launch_bounds__(256, NK > 8 ? 1 : 2) void delta_prep_kernel(DeltaArgs p) {
-    constexpr int C = DELTA_C, DKP = NK * 16, LQ = DKP + 4, LA = 36, NT = 256;
+__global__ __launch_bounds__(512, NK > 8 ? 2 : 4) void delta_prep_kernel(DeltaArgs p) {
+    constexpr int C = DELTA_C, DKP = NK * 16, LQ = DKP + 4, LA = 36, NT = 512, NW = NT / 64;
     constexpr float LOG2E = 1.4426950408889634f;
     const int h = blockIdx.x, seq = blockIdx.y, c0 = blockIdx.z * C;
     const int n = p.seq_len[seq];
@@ -68,89 +74,103 @@ __global__ __launch_bounds__(256, NK > 8 ? 1 : 2) void delta_prep_kernel(DeltaAr
     float* qs = dl_sm;                   // [C][LQ]  q, later q e^b
     float* ks = qs + C * LQ;             // [C][LQ]  k, later k e^b
     float* bs = ks + C * LQ;             // [C][LQ]  inclusive sums of log2 a
-    float* As = bs + C * LQ;             // [C][LA]
-    float* Ms = As + C * LA;             // [C][LA]  M, later T
+    float* As = bs + C * LQ;             // [C][LA]  A, later A T
+    float* Ms = As + C * LA;             // [C][LA]  M, later X = (I + diag(beta) M)^-1
     float* be = Ms + C * LA;             // [C]
-    float* aux = be + C;                 // [256]
+    float* aux = be + C;                 // [512]
     const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6);
     const int fr = lane & 15, fg = lane >> 4;
     const int nv = min(C, n - c0);
     const int64_t tb = (int64_t)p.seq_tok_start[seq] + c0;
     const int g = h / (p.H / p.G);
-    {   // q and k as unit vectors; DKP / 4 lanes hold a row
-        constexpr int LR = DKP / 4, R = NT / LR;
-        const int t0 = tid / LR, d = tid % LR * 4;
-        auto ld4 = [&](const float* src) {
-            f32x4 x = f32x4{0.f, 0.f, 0.f, 0.f};
-            if (p.vec4) { if (d < p.DK) x = *(const f32x4*)(src + d); }
-            else {
+    // every load of the chunk first: q and k (DKP / 4 lanes hold a row), z (a channel per thread, NG groups share the tokens) and the
+    // first value channels of this wave
+    constexpr int LR = DKP / 4, R = NT / LR, NQ = (C + R - 1) / R, NG = NT / DKP, TPG = C / NG;
+    const int qt = tid / LR, qd = tid % LR * 4, zd = tid % DKP, grp = tid / DKP, nvb = (p.DV + 15) >> 4;
+    f32x4 q4[NQ], k4[NQ], v4[2];
+    float pre[TPG];
+    auto ld4 = [&](const float* src) {
+        f32x4 x = f32x4{0.f, 0.f, 0.f, 0.f};
+        if (p.vec4) { if (qd < p.DK) x = *(const f32x4*)(src + qd); }
+        else {
 #pragma unroll
-                for (int r = 0; r < 4; r++) if (d + r < p.DK) x[r] = src[d + r];
+            for (int r = 0; r < 4; r++) if (qd + r < p.DK) x[r] = src[qd + r];
+        }
+        return x;
+    };
+    auto ldv = [&](int i, f32x4 (&v)[2]) {       // 16 value channels as the A operand of a transposed product
+        const int c = 16 * i + fr;
+        const float* vb = p.v + tb * p.ld + (int64_t)h * p.DV + min(c, p.DV - 1);
+#pragma unroll
+        for (int sb = 0; sb < 2; sb++)
+#pragma unroll
+            for (int r = 0; r < 4; r++) {
+                const int t = 16 * sb + 4 * fg + r;
+                const float x = vb[min(t, nv - 1) * p.ld];
+                v[sb][r] = c < p.DV && t < nv ? x : 0.f;
             }
-            return x;
-        };
+    };
 #pragma unroll
-        for (int i = 0; i < C / R; i++) {
-            const int t = t0 + i * R;
-            f32x4 q = f32x4{0.f, 0.f, 0.f, 0.f}, k = q;
-            if (t < nv) { q = ld4(p.q + (tb + t) * p.ld + (int64_t)g * p.DK); k = ld4(p.k + (tb + t) * p.ld + (int64_t)g * p.DK); }
-            float sq = (q[0] * q[0] + q[1] * q[1]) + (q[2] * q[2] + q[3] * q[3]), sk = (k[0] * k[0] + k[1] * k[1]) + (k[2] * k[2] + k[3] * k[3]);
-#pragma unroll
-            for (int o = 1; o < LR; o <<= 1) { sq += __shfl_xor(sq, o, 64); sk += __shfl_xor(sk, o, 64); }
-            *(f32x4*)(qs + t * LQ + d) = q * (p.q_scale / sqrtf(sq + DELTA_UNIT_EPS));
-            *(f32x4*)(ks + t * LQ + d) = k * (1.0f / sqrtf(sk + DELTA_UNIT_EPS));
-        }
+    for (int i = 0; i < NQ; i++) {
+        const int t = qt + i * R;
+        q4[i] = k4[i] = f32x4{0.f, 0.f, 0.f, 0.f};
+        if (t < nv) { q4[i] = ld4(p.q + (tb + t) * p.ld + (int64_t)g * p.DK); k4[i] = ld4(p.k + (tb + t) * p.ld + (int64_t)g * p.DK); }
     }
-    {   // decays: a channel per thread, NG groups share the tokens
-        constexpr int NG = NT / DKP, TPG = C / NG;
-        const int d = tid % DKP, grp = tid / DKP;
-        float pre[TPG];
-        const float A = -expf(p.a_log[h]) * LOG2E, bias = d < p.DK ? p.dt_bias[h * p.DK + d] : 0.f;
 #pragma unroll
-        for (int j = 0; j < TPG; j++) {
-            const int t = grp * TPG + j;
-            pre[j] = d < p.DK && t < nv ? p.z[(tb + t) * p.z_ld + (int64_t)h * p.DK + d] : 0.f;
-        }
+    for (int j = 0; j < TPG; j++) pre[j] = p.z[(tb + min(grp * TPG + j, nv - 1)) * p.z_ld + (int64_t)h * p.DK + min(zd, p.DK - 1)];
+    if (wave < nvb) ldv(wave, v4);
 #pragma unroll
-        for (int j = 0; j < TPG; j++) pre[j] = d < p.DK && grp * TPG + j < nv ? A * lr_softplus(pre[j] + bias) : 0.f;
+    for (int i = 0; i < NQ; i++) {               // unit vectors
+        const f32x4 q = q4[i], k = k4[i];
+        float sq = (q[0] * q[0] + q[1] * q[1]) + (q[2] * q[2] + q[3] * q[3]), sk = (k[0] * k[0] + k[1] * k[1]) + (k[2] * k[2] + k[3] * k[3]);
+#pragma unroll
+        for (int o = 1; o < LR; o <<= 1) { sq += __shfl_xor(sq, o, 64); sk += __shfl_xor(sk, o, 64); }
+        if (C % R && qt + i * R >= C) continue;
+        *(f32x4*)(qs + (qt + i * R) * LQ + qd) = q * (p.q_scale / sqrtf(sq + DELTA_UNIT_EPS));
+        *(f32x4*)(ks + (qt + i * R) * LQ + qd) = k * (1.0f / sqrtf(sk + DELTA_UNIT_EPS));
+    }
+    {   // decays
+        const float A = -expf(p.a_log[h]) * LOG2E, bias = zd < p.DK ? p.dt_bias[h * p.DK + zd] : 0.f;
+#pragma unroll
+        for (int j = 0; j < TPG; j++) pre[j] = zd < p.DK && grp * TPG + j < nv ? A * delta_softplus(pre[j] + bias) : 0.f;
 #pragma unroll
         for (int j = 1; j < TPG; j++) pre[j] += pre[j - 1];
-        aux[grp * DKP + d] = pre[TPG - 1];
+        aux[grp * DKP + zd] = pre[TPG - 1];
         if (tid < C) be[tid] = tid < nv ? lr_sigmoid(p.beta[(tb + tid) * p.beta_ld + h]) : 0.f;
         __syncthreads();
         float off = 0.f;
-        for (int j = 0; j < grp; j++) off += aux[j * DKP + d];
+        for (int j = 0; j < grp; j++) off += aux[j * DKP + zd];
 #pragma unroll
-        for (int j = 0; j < TPG; j++) bs[(grp * TPG + j) * LQ + d] = off + pre[j];
+        for (int j = 0; j < TPG; j++) bs[(grp * TPG + j) * LQ + zd] = off + pre[j];
     }
     for (int i = tid; i < 2 * C * LA; i += NT) As[i] = 0.f;      // (what lies above the diagonals stays zero)
     __syncthreads();
-    // ---- A (s <= t) and M (s < t): 240 pairs of the two diagonal blocks, one per thread; the other 16 threads take A's diagonal ----
-    if (tid < 240) {
-        const int half = tid >= 120, x = tid - 120 * half;
+    // ---- A (s <= t) and M (s < t): 240 pairs of the two diagonal blocks, two threads each; the other 32 threads take A's diagonal ----
+    if (tid < 480) {
+        const int pr = tid >> 1, half = pr >= 120, x = pr - 120 * half;
         int t = (int)((sqrtf(8.f * (float)x + 1.f) - 1.f) * 0.5f);
         if ((t + 1) * (t + 2) / 2 <= x) t++;
         if (t * (t + 1) / 2 > x) t--;
         const int s = x - t * (t + 1) / 2, tr = (16 * half + t + 1) * LQ, sr = (16 * half + s) * LQ;
         f32x4 aq = f32x4{0.f, 0.f, 0.f, 0.f}, ak = aq;
 #pragma unroll 2
-        for (int d = 0; d < DKP; d += 4) {
+        for (int d = 4 * (tid & 1); d < DKP; d += 8) {
             const f32x4 q4 = *(const f32x4*)(qs + tr + d), k4 = *(const f32x4*)(ks + tr + d), k2 = *(const f32x4*)(ks + sr + d);
             const f32x4 bt = *(const f32x4*)(bs + tr + d), b2 = *(const f32x4*)(bs + sr + d);
 #pragma unroll
             for (int r = 0; r < 4; r++) { const float e = ex2(bt[r] - b2[r]) * k2[r]; aq[r] = fmaf(q4[r], e, aq[r]); ak[r] = fmaf(k4[r], e, ak[r]); }
         }
         const int at = (16 * half + t + 1) * LA + 16 * half + s;
-        As[at] = (aq[0] + aq[1]) + (aq[2] + aq[3]);
-        Ms[at] = (ak[0] + ak[1]) + (ak[2] + ak[3]);
+        float sa = (aq[0] + aq[1]) + (aq[2] + aq[3]), sm = (ak[0] + ak[1]) + (ak[2] + ak[3]);
+        sa += __shfl_xor(sa, 1, 64);
+        sm += __shfl_xor(sm, 1, 64);
+        if (tid & 1) Ms[at] = sm; else As[at] = sa;
     } else {
-#pragma unroll
-        for (int i = 0; i < 2; i++) {
-            const int t = tid - 240 + 16 * i;
-            f32x4 a = f32x4{0.f, 0.f, 0.f, 0.f};
-            for (int d = 0; d < DKP; d += 4) a += *(const f32x4*)(qs + t * LQ + d) * *(const f32x4*)(ks + t * LQ + d);
-            As[t * LA + t] = (a[0] + a[1]) + (a[2] + a[3]);
-        }
+        const int t = tid - 480;
+        f32x4 a = f32x4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll 2
+        for (int d = 0; d < DKP; d += 4) a += *(const f32x4*)(qs + t * LQ + d) * *(const f32x4*)(ks + t * LQ + d);
+        As[t * LA + t] = (a[0] + a[1]) + (a[2] + a[3]);
     }
     if (wave < 2) {                                              // tokens 16..31 against 0..15: wave 0 A, wave 1 M
         const float* x = wave == 0 ? qs : ks;
@@ -170,116 +190,132 @@ __global__ __launch_bounds__(256, NK > 8 ? 1 : 2) void delta_prep_kernel(DeltaAr
     }
     __syncthreads();
     float* ws = p.ws + (delta_chunk(p, seq, blockIdx.z) * p.H + h) * delta_ws_floats(DKP);
-    if (wave == 0) {
-        // T: a column of a diagonal block's inverse per lane (lanes 0..31), then the block below
-        float x[16];
-        const int blk = (lane >> 4) & 1, col = lane & 15;
-        const float* mr = Ms + 16 * blk * LA + 16 * blk;
+    if (wave < 2) {
+        // inverses of the two diagonal blocks of I + N, N = diag(beta) M, from 1 x 1 blocks upwards: with X the inverse of the part inside
+        // b x b blocks and N_b the part that a 2b x 2b block adds, X - X N_b X is the inverse inside 2b x 2b blocks
+        const int o = 16 * wave;
+        float* xt = aux + 256 * wave;                            // X's turn from accumulator to A operand
+        const f32x4 na = *(const f32x4*)(Ms + (o + fr) * LA + o + 4 * fg) * be[o + fr];
+        f32x4 xa, xd;
 #pragma unroll
-        for (int t = 0; t < 16; t++) {
-            float a = 0.f;
-#pragma unroll
-            for (int s = 0; s < t; s++) a = fmaf(mr[t * LA + s], x[s], a);
-            x[t] = t == col ? 1.0f : (t < col ? 0.f : -be[16 * blk + t] * a);
+        for (int r = 0; r < 4; r++) {
+            const int c = 4 * fg + r;                            // (row fr, column c) as an A operand, (row c, column fr) as an accumulator
+            xa[r] = fr == c ? 1.f : ((fr ^ c) == 1 ? -na[r] : 0.f);
+            xd[r] = fr == c ? 1.f : ((fr ^ c) == 1 ? -Ms[(o + c) * LA + o + fr] * be[o + c] : 0.f);
         }
-        f32x4 a21 = *(const f32x4*)(Ms + (16 + fr) * LA + 4 * fg) * be[16 + fr];        // beta M, block below the diagonal, as an A operand
-        asm volatile("" : "+v"(a21));                                                  // (read before the block is written)
-        if (lane < 32)
 #pragma unroll
-            for (int t = 0; t < 16; t++) Ms[(16 * blk + t) * LA + 16 * blk + col] = x[t];
-        asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");
-        f32x4 y = f32x4{0.f, 0.f, 0.f, 0.f}, w = y;
+        for (int lb = 1; lb < 4; lb++) {                         // b = 2, 4, 8
+            f32x4 y = f32x4{0.f, 0.f, 0.f, 0.f}, z = y;
 #pragma unroll
-        for (int r = 0; r < 4; r++) y = mfma_f32(a21[r], Ms[(4 * fg + r) * LA + fr], y);
-        const f32x4 a22 = *(const f32x4*)(Ms + (16 + fr) * LA + 16 + 4 * fg);
+            for (int r = 0; r < 4; r++) y = mfma_f32(((fr ^ (4 * fg + r)) >> lb) == 1 ? na[r] : 0.f, xd[r], y);
 #pragma unroll
-        for (int r = 0; r < 4; r++) w = mfma_f32(a22[r], y[r], w);
+            for (int r = 0; r < 4; r++) z = mfma_f32(xa[r], y[r], z);
+            xd -= z;
+            if (lb == 3) break;
 #pragma unroll
-        for (int r = 0; r < 4; r++) Ms[(16 + 4 * fg + r) * LA + fr] = -w[r];
+            for (int r = 0; r < 4; r++) xt[(4 * fg + r) * 16 + fr] = xd[r];
+            asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");
+            xa = *(const f32x4*)(xt + fr * 16 + 4 * fg);
+        }
+#pragma unroll
+        for (int r = 0; r < 4; r++) Ms[(o + 4 * fg + r) * LA + o + fr] = xd[r];
     } else {
         // (K e^{b_end - b})^T and e^{b_end}; 32 tokens of a channel side by side
         float* kt = ws + 2 * C * DKP;
 #pragma unroll 2
-        for (int i = tid - 64; i < C * DKP; i += NT - 64) {
+        for (int i = tid - 128; i < C * DKP; i += NT - 128) {
             const int t = i & 31, d = i >> 5;
             kt[d * C + t] = ks[t * LQ + d] * ex2(bs[31 * LQ + d] - bs[t * LQ + d]);
         }
-        for (int d = tid - 64; d < DKP; d += NT - 64) ws[3 * C * DKP + d] = ex2(bs[31 * LQ + d]);
+        for (int d = tid - 128; d < DKP; d += NT - 128) ws[3 * C * DKP + d] = ex2(bs[31 * LQ + d]);
     }
     __syncthreads();
-#pragma unroll 4
-    for (int i = tid; i < C * DKP / 4; i += NT) {                // q e^b, k e^b in place
-        const int t = i / (DKP / 4), d = i % (DKP / 4) * 4;
-        const f32x4 b = *(const f32x4*)(bs + t * LQ + d);
-        f32x4 q = *(const f32x4*)(qs + t * LQ + d), k = *(const f32x4*)(ks + t * LQ + d);
+    if (wave == 0) {
+        // the block below the diagonal: -X22 N21 X11; then A T, T = X diag(beta), in A's place
+        const f32x4 n21 = *(const f32x4*)(Ms + (16 + fr) * LA + 4 * fg) * be[16 + fr], x22 = *(const f32x4*)(Ms + (16 + fr) * LA + 16 + 4 * fg);
+        f32x4 x11, y = f32x4{0.f, 0.f, 0.f, 0.f}, w = y, aa[3], at[3];
 #pragma unroll
-        for (int r = 0; r < 4; r++) { const float e = ex2(b[r]); q[r] *= e; k[r] *= e; }
-        *(f32x4*)(qs + t * LQ + d) = q;
-        *(f32x4*)(ks + t * LQ + d) = k;
+        for (int x = 0; x < 3; x++) {
+            aa[x] = *(const f32x4*)(As + (16 * (x > 0) + fr) * LA + 16 * (x > 1) + 4 * fg);
+            at[x] = w;
+        }
+#pragma unroll
+        for (int r = 0; r < 4; r++) { x11[r] = Ms[(4 * fg + r) * LA + fr]; y = mfma_f32(n21[r], x11[r], y); }
+#pragma unroll
+        for (int r = 0; r < 4; r++) w = mfma_f32(x22[r], y[r], w);
+#pragma unroll
+        for (int r = 0; r < 4; r++) {
+            const float t00 = x11[r] * be[fr], t10 = -w[r] * be[fr], t11 = Ms[(16 + 4 * fg + r) * LA + 16 + fr] * be[16 + fr];
+            at[0] = mfma_f32(aa[0][r], t00, at[0]); at[1] = mfma_f32(aa[1][r], t00, at[1]);
+            at[1] = mfma_f32(aa[2][r], t10, at[1]); at[2] = mfma_f32(aa[2][r], t11, at[2]);
+            Ms[(16 + 4 * fg + r) * LA + fr] = -w[r];
+        }
+#pragma unroll
+        for (int x = 0; x < 3; x++)
+#pragma unroll
+            for (int r = 0; r < 4; r++) As[(16 * (x > 0) + 4 * fg + r) * LA + 16 * (x > 1) + fr] = at[x][r];
+    } else {
+#pragma unroll 2
+        for (int i = tid - 64; i < C * DKP / 4; i += NT - 64) {  // q e^b, k e^b in place
+            const int t = i / (DKP / 4), d = i % (DKP / 4) * 4;
+            const f32x4 b = *(const f32x4*)(bs + t * LQ + d);
+            f32x4 q = *(const f32x4*)(qs + t * LQ + d), k = *(const f32x4*)(ks + t * LQ + d);
+#pragma unroll
+            for (int r = 0; r < 4; r++) { const float e = ex2(b[r]); q[r] *= e; k[r] *= e; }
+            *(f32x4*)(qs + t * LQ + d) = q;
+            *(f32x4*)(ks + t * LQ + d) = k;
+        }
     }
-    // A operands of T and A: blocks (0,0), (1,0), (1,1); the columns of T carry beta
-    f32x4 ta[3], aa[3];
+    __syncthreads();
+    // rows of T and of A T, blocks (0,0), (1,0), (1,1): B operands of the transposed products, whose accumulators hold four channels of a token
+    f32x4 ta[3], ba[3];
 #pragma unroll
     for (int x = 0; x < 3; x++) {
-        const int row = 16 * (x > 0) + fr, c = 16 * (x > 1) + 4 * fg;
-        ta[x] = *(const f32x4*)(Ms + row * LA + c) * *(const f32x4*)(be + c);
-        aa[x] = *(const f32x4*)(As + row * LA + c);
+        const int at = (16 * (x > 0) + fr) * LA + 16 * (x > 1) + 4 * fg;
+        ta[x] = *(const f32x4*)(Ms + at) * *(const f32x4*)(be + 16 * (x > 1) + 4 * fg);
+        ba[x] = *(const f32x4*)(As + at);
     }
-    __syncthreads();
-    for (int i = wave; i < NK; i += 4) {                         // 16 key channels: -W and Q'
-        const int c = 16 * i + fr;
-        f32x4 w[2], q[2], k0, k1;
+    auto times = [&](const f32x4 (&x)[2], const f32x4 (&m)[3], f32x4 (&d)[2]) {          // d += (m x)^T
 #pragma unroll
-        for (int r = 0; r < 4; r++) {
-            k0[r] = -ks[(4 * fg + r) * LQ + c]; k1[r] = -ks[(16 + 4 * fg + r) * LQ + c];
-            q[0][r] = qs[(4 * fg + r) * LQ + c]; q[1][r] = qs[(16 + 4 * fg + r) * LQ + c];
-            w[0][r] = 0.f; w[1][r] = 0.f;
+        for (int r = 0; r < 4; r++) { d[0] = mfma_f32(x[0][r], m[0][r], d[0]); d[1] = mfma_f32(x[0][r], m[1][r], d[1]); }
+#pragma unroll
+        for (int r = 0; r < 4; r++) d[1] = mfma_f32(x[1][r], m[2][r], d[1]);
+    };
+    for (int i = wave; i < NK; i += NW) {                         // 16 key channels: -W and Q'
+        f32x4 k[2], w[2], q[2];
+#pragma unroll
+        for (int sb = 0; sb < 2; sb++) {
+#pragma unroll
+            for (int r = 0; r < 4; r++) k[sb][r] = -ks[(16 * sb + 4 * fg + r) * LQ + 16 * i + fr];
+            w[sb] = f32x4{0.f, 0.f, 0.f, 0.f};
+            q[sb] = *(const f32x4*)(qs + (16 * sb + fr) * LQ + 16 * i + 4 * fg);
         }
+        times(k, ta, w);
+        times(k, ba, q);
 #pragma unroll
-        for (int r = 0; r < 4; r++) { w[0] = mfma_f32(ta[0][r], k0[r], w[0]); w[1] = mfma_f32(ta[1][r], k0[r], w[1]); }
-#pragma unroll
-        for (int r = 0; r < 4; r++) w[1] = mfma_f32(ta[2][r], k1[r], w[1]);
-#pragma unroll
-        for (int r = 0; r < 4; r++) { q[0] = mfma_f32(aa[0][r], w[0][r], q[0]); q[1] = mfma_f32(aa[1][r], w[0][r], q[1]); }
-#pragma unroll
-        for (int r = 0; r < 4; r++) q[1] = mfma_f32(aa[2][r], w[1][r], q[1]);
-#pragma unroll
-        for (int tt = 0; tt < 2; tt++)
-#pragma unroll
-            for (int r = 0; r < 4; r++) {
-                const int t = 16 * tt + 4 * fg + r;
-                ws[t * DKP + c] = w[tt][r];
-                ws[(C + t) * DKP + c] = q[tt][r];
-            }
+        for (int tt = 0; tt < 2; tt++) {
+            *(f32x4*)(ws + (16 * tt + fr) * DKP + 16 * i + 4 * fg) = w[tt];
+            *(f32x4*)(ws + (C + 16 * tt + fr) * DKP + 16 * i + 4 * fg) = q[tt];
+        }
     }
-    const int nvb = (p.DV + 15) >> 4;
-    for (int i = wave; i < nvb; i += 4) {                        // 16 value channels: U0 and O0
-        const int c = 16 * i + fr;
-        const bool live = c < p.DV;
-        float* vb = p.v + tb * p.ld + (int64_t)h * p.DV + c;
-        f32x4 v0, v1, u[2], o[2];
+    for (int i = wave; i < nvb; i += NW) {                       // 16 value channels: U0 and O0
+        f32x4 v[2] = {v4[0], v4[1]}, u[2], o[2];
+        if (i != wave) ldv(i, v);
+        u[0] = u[1] = o[0] = o[1] = f32x4{0.f, 0.f, 0.f, 0.f};
+        times(v, ta, u);
+        times(v, ba, o);
+        const int c = 16 * i + 4 * fg;
 #pragma unroll
-        for (int r = 0; r < 4; r++) {
-            v0[r] = live && 4 * fg + r < nv ? vb[(4 * fg + r) * p.ld] : 0.f;
-            v1[r] = live && 16 + 4 * fg + r < nv ? vb[(16 + 4 * fg + r) * p.ld] : 0.f;
-            u[0][r] = u[1][r] = o[0][r] = o[1][r] = 0.f;
+        for (int tt = 0; tt < 2; tt++) {
+            const int t = 16 * tt + fr;
+            float* ub = p.v + (tb + t) * p.ld + (int64_t)h * p.DV + c;
+            float* ob = p.o + (tb + t) * p.o_ld + (int64_t)h * p.DV + c;
+            if (t >= nv) continue;
+            if (p.vec4v) { if (c < p.DV) { *(f32x4*)ub = u[tt]; *(f32x4*)ob = o[tt]; } }
+            else
+#pragma unroll
+                for (int r = 0; r < 4; r++) if (c + r < p.DV) { ub[r] = u[tt][r]; ob[r] = o[tt][r]; }
         }
-#pragma unroll
-        for (int r = 0; r < 4; r++) { u[0] = mfma_f32(ta[0][r], v0[r], u[0]); u[1] = mfma_f32(ta[1][r], v0[r], u[1]); }
-#pragma unroll
-        for (int r = 0; r < 4; r++) u[1] = mfma_f32(ta[2][r], v1[r], u[1]);
-#pragma unroll
-        for (int r = 0; r < 4; r++) { o[0] = mfma_f32(aa[0][r], u[0][r], o[0]); o[1] = mfma_f32(aa[1][r], u[0][r], o[1]); }
-#pragma unroll
-        for (int r = 0; r < 4; r++) o[1] = mfma_f32(aa[2][r], u[1][r], o[1]);
-        float* ob = p.o + tb * p.o_ld + (int64_t)h * p.DV + c;
-#pragma unroll
-        for (int tt = 0; tt < 2; tt++)
-#pragma unroll
-            for (int r = 0; r < 4; r++) {
-                const int t = 16 * tt + 4 * fg + r;
-                if (live && t < nv) { vb[t * p.ld] = u[tt][r]; ob[t * p.o_ld] = o[tt][r]; }
-            }
     }
 }
 
@@ -333,7 +369,6 @@ __global__ __launch_bounds__(NW * 64, NK > 8 ? 1 : (NW == 8 ? (KSP > 1 ? 2 : 4) 
     const char* vb = (const char*)(p.v + tok0 * p.ld + (int64_t)h * p.DV);
     char* ob = (char*)(p.o + tok0 * p.o_ld + (int64_t)h * p.DV);
     const uint32_t cb = 4 * min(col, p.DV - 1);
-    constexpr bool EARLY = NW == 4 || KSP > 1;       // registers for a whole chunk of lead
     auto fetch = [&]() {
 #pragma unroll
         for (int i = 0; i < NL; i++) rg[i] = ((const f32x4*)src + i * NT)[tid];
@@ -366,9 +401,6 @@ __global__ __launch_bounds__(NW * 64, NK > 8 ? 1 : (NW == 8 ? (KSP > 1 ? 2 : 4) 
             else *(f32x4*)(k0 + (i - NL / 3 * 2) * (NT / 8) * LK) = rg[i];
         if (tid < DKP) dl[tid] = rd;
         __syncthreads();
-        const bool more = c0 + C < n;                            // (the last chunk is fetched once more instead of a branch)
-        src += more ? stride : 0;
-        if (EARLY) fetch();
 #pragma unroll
         for (int i = 0; i < NKW; i++) {
             f32x4 a[4];
@@ -406,8 +438,9 @@ __global__ __launch_bounds__(NW * 64, NK > 8 ? 1 : (NW == 8 ? (KSP > 1 ? 2 : 4) 
             }
         f32x4 ub[2] = {u[0], u[1]};
         __builtin_amdgcn_sched_barrier(0);
-        vb += more ? (int64_t)C * ld * 4 : 0; ob += more ? (int64_t)C * old * 4 : 0;
-        if (!EARLY) fetch();
+        const bool more = c0 + C < n;                            // (the last chunk is fetched once more instead of a branch)
+        src += more ? stride : 0; vb += more ? (int64_t)C * ld * 4 : 0; ob += more ? (int64_t)C * old * 4 : 0;
+        fetch();
         fetch_uo(vb, ob, more ? n - c0 - C : n - c0);
         __builtin_amdgcn_sched_barrier(0);
 #pragma unroll
@@ -536,7 +569,7 @@ __global__ __launch_bounds__(LR_STEP_THREADS, ROWS <= 8 ? 4 : 2) void delta_step
                 a += __shfl_xor(a, 1, 64);
                 a += __shfl_xor(a, 2, 64);
                 if ((tid & 3) == 0) {
-                    if (dec) sa[i] = expf(-ea * lr_softplus(a + p.dt_bias[h * p.DK + i]));
+                    if (dec) sa[i] = expf(-ea * delta_softplus(a + p.dt_bias[h * p.DK + i]));
                     else sg[i - p.DK] = lr_sigmoid(a);
                 }
             }
@@ -544,7 +577,7 @@ __global__ __launch_bounds__(LR_STEP_THREADS, ROWS <= 8 ? 4 : 2) void delta_step
             for (int i = tid; i < p.DK; i += NT) {
                 sq[i] = p.q[t * p.ld + (int64_t)g * p.DK + i];
                 sk[i] = p.k[t * p.ld + (int64_t)g * p.DK + i];
-                sa[i] = expf(-ea * lr_softplus(p.z[t * p.z_ld + (int64_t)h * p.DK + i] + p.dt_bias[h * p.DK + i]));
+                sa[i] = expf(-ea * delta_softplus(p.z[t * p.z_ld + (int64_t)h * p.DK + i] + p.dt_bias[h * p.DK + i]));
             }
             for (int i = tid; i < p.DV; i += NT) sv[i] = p.v[t * p.ld + (int64_t)h * p.DV + i];
         }

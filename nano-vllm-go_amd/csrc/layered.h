@@ -1031,6 +1031,7 @@ void mix_delta(nvl_model* m, const LayerRun& r, const MixerW& w, const Meta& md,
     if (chunks && max_len > REC_STEP_MAX) {
         a.len_lo = REC_STEP_MAX + 1; a.len_hi = 1 << 30;
         a.vec4 = c.dim % 4 == 0 && qk % 4 == 0 && a.ld % 4 == 0;
+        a.vec4v = c.vdim % 4 == 0 && 2 * qk % 4 == 0 && a.ld % 4 == 0 && a.o_ld % 4 == 0;
         const int nk = c.dim <= 32 ? 2 : (c.dim <= 64 ? 4 : (c.dim <= 128 ? 8 : 16));
         grow(m, m->delta_ws, m->delta_ws_cap, (int64_t)(m->opts.max_batch_tokens / DELTA_C + m->opts.max_seqs + 1) * c.heads * delta_ws_floats(nk * 16));
         a.ws = m->delta_ws;
@@ -1042,7 +1043,7 @@ void mix_delta(nvl_model* m, const LayerRun& r, const MixerW& w, const Meta& md,
             do {                                                                                                              \
                 constexpr int lds_ = delta_prep_lds_bytes<NKv>();                                                              \
                 NVL_LDS_ATTR((delta_prep_kernel<NKv>), lds_);                                                                  \
-                hipLaunchKernelGGL((delta_prep_kernel<NKv>), pgrid, dim3(256), lds_, m->stream, a);                            \
+                hipLaunchKernelGGL((delta_prep_kernel<NKv>), pgrid, dim3(512), lds_, m->stream, a);                            \
             } while (0)
             if (nk == 2) NVL_DP(2); else if (nk == 4) NVL_DP(4); else if (nk == 8) NVL_DP(8); else NVL_DP(16);
 #undef NVL_DP
@@ -1061,8 +1062,7 @@ void mix_delta(nvl_model* m, const LayerRun& r, const MixerW& w, const Meta& md,
 #define NVL_DCK(NKv, LOW)                                                                                                     \
             do {                                                                                                              \
                 if (pairs * cdiv(c.vdim, 64) < 128) NVL_DC(NKv, 4, LOW);                                                       \
-                else if (pairs * cdiv(c.vdim, 128) < 256) NVL_DC(NKv, 8, 2);                                                   \
-                else if (c.vdim <= 64) NVL_DC(NKv, 4, 1);                                                                      \
+                else if (c.vdim <= 64 || pairs * cdiv(c.vdim, 128) < 256) NVL_DC(NKv, 4, 1);                                                                      \
                 else NVL_DC(NKv, 8, 1);                                                                                        \
             } while (0)
             if (nk == 2) NVL_DC(2, 4, 1); else if (nk == 4) NVL_DCK(4, 2); else if (nk == 8) NVL_DCK(8, 4); else NVL_DCK(16, 4);
