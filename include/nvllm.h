@@ -27,10 +27,11 @@
 extern "C" {
 #endif
 
-#define NVL_ABI_VERSION 5      /* 2: Mamba2 / hybrid layers (config fields, tensor kinds), nvl_stats.evictions, kernel stats;
+#define NVL_ABI_VERSION 6      /* 2: Mamba2 / hybrid layers (config fields, tensor kinds), nvl_stats.evictions, kernel stats;
                                   3: nvl_get_weight, nvl_get_stamps, nvl_tp_p2p_rearm, debug modes 2 / 4 (additions only);
                                   4: models described by a list of layers, library-owned block pool, nvl_forward_rows (additions only);
-                                  5: rotated latent attention, channel-wise gated delta rule, output-only norms (new config fields at the end) */
+                                  5: rotated latent attention, channel-wise gated delta rule, output-only norms (new config fields at the end);
+                                  6: grouped-query attention, parallel blocks, experts and per-layer token inputs in lists of layers (new config fields at the end) */
 
 typedef enum nvl_status {
     NVL_OK = 0,
@@ -51,7 +52,8 @@ enum { NVL_POS_LEARNED = 0, NVL_POS_ROPE = 1, NVL_POS_NONE = 2 };     /* config.
 enum { NVL_ACT_GELU = 0, NVL_ACT_SWIGLU = 1,                          /* config.go:45-48 */
        NVL_ACT_GEGLU = 2,                                             /* gelu_tanh(gate) * up */
        NVL_ACT_CLAMPED_GLU = 3 };   /* g sigmoid(1.702 g) (u + 1), g = min(gate, limit), u = clamp(up, -limit, limit): nvl_layer_config.ffn_limit */
-enum { NVL_BLOCK_SEQUENTIAL = 0, NVL_BLOCK_PARALLEL = 1,              /* config.go:53-56 */
+enum { NVL_ACT_RELU2 = 4 };         /* max(z, 0)^2, no gate (lists of layers) */
+enum { NVL_BLOCK_SEQUENTIAL = 0, NVL_BLOCK_PARALLEL = 1,              /* config.go:53-56 (parallel: with a list of layers too) */
        NVL_BLOCK_SANDWICH = 2,     /* a norm before AND after each sublayer, x += norm_b(f(norm_a(x)))  } the model is described by a list */
        NVL_BLOCK_POST = 3 };       /* a norm after each sublayer only, x += scale * norm(f(x))           } of layers (nvl_create_layers)    */
 
@@ -72,6 +74,7 @@ typedef struct nvl_model_config {
     /* models described by a list of layers */
     float   norm_weight_offset;     /* added to every stored weight of the model's norm (1: weights are kept as differences from one)     */
     float   logit_softcap;          /* logits <- cap tanh(logits / cap); 0: none                                                          */
+    int32_t side_dim;               /* per-layer token inputs: columns of NVL_T_SIDE_EMB a layer takes; 0: none (NVL_BLOCK_PARALLEL)        */
 } nvl_model_config;
 
 /* ---- models described by a list of layers: every layer names its mixer, the mixer's sizes and its feed-forward ---- */
@@ -79,26 +82,32 @@ enum {
     NVL_MIXER_LATENT_ATTENTION = 0, /* queries and keys/values through low-rank latents; the cache holds the latent (and the rotated key part) */
     NVL_MIXER_MAMBA2 = 1,           /* causal convolution + selective state space, gate before a grouped norm                     */
     NVL_MIXER_GLA = 2,              /* gated linear attention: a decay per key channel                                            */
-    NVL_MIXER_CHANNEL_DELTA = 3     /* delta rule with a decay per key channel, short convolutions on q, k and v                  */
+    NVL_MIXER_CHANNEL_DELTA = 3,    /* delta rule with a decay per key channel, short convolutions on q, k and v                  */
+    NVL_MIXER_ATTENTION = 4         /* grouped-query attention: capped scores, logarithmic distance bias, value mixing, output gate */
 };
 typedef struct nvl_layer_config {
     int32_t mixer;                  /* NVL_MIXER_*                                                                         */
     int32_t weights_of;             /* the layer whose tensors this one uses (its cache / state is its own); -1: its own   */
     int32_t heads, dim, vdim;       /* dim: query/key channels per head (not Mamba-2), vdim: value channels per head       */
     int32_t q_rank, kv_rank;        /* latent attention: latent sizes                                                      */
-    int32_t window;                 /* latent attention: keys a query sees, itself included (0: all earlier tokens)        */
-    float   scale;                  /* latent attention: score multiplier                                                  */
+    int32_t window;                 /* attention: keys a query sees, itself included (0: all earlier tokens)               */
+    float   scale;                  /* attention: score multiplier                                                         */
     int32_t state, groups, norm_groups, conv_taps;      /* Mamba-2                                                         */
     float   tau;                    /* GLA: alpha = sigmoid(z)^(1/tau)                                                     */
     int32_t decay_rank;             /* GLA: rank of the decay projection; 0: as the uploaded tensor says                   */
-    int32_t ffn_dim;                /* 0: no feed-forward                                                                  */
+    int32_t ffn_dim;                /* 0: no feed-forward (with experts: the shared expert, 0: none)                       */
     float   ffn_limit;              /* NVL_ACT_CLAMPED_GLU                                                                 */
     int32_t kv_from;                /* latent attention: use this earlier layer's cached latents and rotated keys; -1: own */
     int32_t rot_dim;                /* latent attention: rotated query/key dimensions per head beside `dim`; 0: none       */
     int32_t gate_per_head;          /* latent attention: 1: one output gate per head; 0: one per channel                   */
-    int32_t kv_heads;               /* channel delta: heads of q and k (heads is a multiple)                               */
+    int32_t kv_heads;               /* channel delta: heads of q and k; attention: heads of k and v (heads is a multiple)  */
     double  rot_base;               /* rotation: pair i turns by base^(-2 i / rot_dim) per position                        */
     double  rot_factor, rot_original, rot_fast, rot_slow;       /* YaRN context extension; rot_factor 0: none              */
+    float   softcap;                /* attention: score <- cap tanh(score / cap); 0: none                                  */
+    int32_t v_mix;                  /* attention: 1: v <- (1 - lambda) v + lambda v_first, v_first the values of the first such layer */
+    int32_t ffn_act;                /* activation of ffn_dim's feed-forward: NVL_ACT_*; 0: the model's activation_type     */
+    int32_t experts, top_k, expert_dim;        /* mixture of experts (SwiGLU, sigmoid scores); experts 0: none             */
+    int32_t expert_groups, groups_kept;        /* only experts of the best groups_kept of expert_groups equal groups can be chosen */
 } nvl_layer_config;
 
 /* Arithmetic the device path computes in. */
@@ -169,7 +178,8 @@ typedef enum nvl_tensor_kind {
     NVL_T_MAMBA_NORM,      /* [EH]                                                                   */
     NVL_T_MAMBA_OUT_PROJ,  /* OUT_IN: [H, EH]  OutProj, MatMul(y, Transpose(OutProj))           mamba2.go:175 */
     /* models described by a list of layers: all matrices OUT_IN ([out, in], applied as W x).  Shared kinds: ATTN_NORM_W and
-     * FFN_NORM_W (the norms before the sublayers), WQ / WK / WV / WO, W1 (gate rows, then up rows), W2, the MAMBA_* kinds */
+     * FFN_NORM_W (the norms before the sublayers; ATTN_NORM_B / FINAL_NORM_B make them layer norms), POS_EMB, WQ / WK / WV / WO, W1 (gate
+     * rows, then up rows), W2, ROUTER [experts, H], MOE_IN, MOE_OUT, the MAMBA_* kinds */
     NVL_T_MIX_POST_NORM,   /* [H] norm after the mixer                                                */
     NVL_T_FFN_POST_NORM,   /* [H] norm after the feed-forward                                         */
     NVL_T_MIX_GATE,        /* [heads*vdim, H] output gate (latent attention, GLA); [heads, H] with gate_per_head */
@@ -190,6 +200,14 @@ typedef enum nvl_tensor_kind {
     NVL_T_DELTA_BETA,      /* [heads, H]          step sizes of the delta rule                        */
     NVL_T_DELTA_G1,        /* [rank, H]           output gate, low-rank: sigmoid(G2 (G1 h))           */
     NVL_T_DELTA_G2,        /* [heads*vdim, rank]                                                      */
+    NVL_T_BIAS_R1,         /* [heads] distance bias of the scores: - r1 ln(1 + r2 distance); optional  */
+    NVL_T_BIAS_R2,         /* [heads]                                                                 */
+    NVL_T_V_MIX,           /* [1] lambda of the value mixing                                          */
+    NVL_T_ROUTER_BIAS,     /* [experts] added to the scores the choice goes by; optional              */
+    NVL_T_SIDE_GATE,       /* [side_dim, H]       per-layer token input: x += rms(P (gelu(G x) * e)) * w */
+    NVL_T_SIDE_PROJ,       /* [H, side_dim]                                                           */
+    NVL_T_SIDE_NORM,       /* [H]                                                                     */
+    NVL_T_SIDE_EMB,        /* model: [V, layers*side_dim] e of every token and layer                  */
     NVL_T_COUNT
 } nvl_tensor_kind;
 
@@ -204,9 +222,11 @@ enum {
 /* Replaces tensor.NewTransformerModel (generic_model.go:41-61) + the runner's model ownership
  * (tensor_model_runner.go:21-33).  Fails with NVL_ERR_NO_DEVICE when no GPU is present. */
 int nvl_create(const nvl_model_config* cfg, const nvl_runtime_opts* opts, nvl_model** out);
-/* nvl_create for a model described by a list of layers (cfg->block_style NVL_BLOCK_SANDWICH or NVL_BLOCK_POST): `layers` has
- * cfg->num_layers entries; of cfg only vocab_size, hidden, num_layers, max_seq_len, norm_eps, norm_weight_offset, activation_type
- * (NVL_ACT_GEGLU or NVL_ACT_CLAMPED_GLU), embedding_multiplier, logits_scaling, logit_softcap and tied_embedding are read. */
+/* nvl_create for a model described by a list of layers (cfg->block_style NVL_BLOCK_SANDWICH, NVL_BLOCK_POST or NVL_BLOCK_PARALLEL): `layers`
+ * has cfg->num_layers entries; of cfg only vocab_size, hidden, num_layers, max_seq_len, norm_eps, norm_type, norm_weight_offset, position_type
+ * (learned or none), activation_type (NVL_ACT_GEGLU, NVL_ACT_CLAMPED_GLU; NVL_ACT_RELU2 or NVL_ACT_SWIGLU in parallel blocks),
+ * embedding_multiplier, logits_scaling, logit_softcap, side_dim and tied_embedding are read.  Layer norms, learned positions, NVL_MIXER_ATTENTION,
+ * experts and side_dim belong to NVL_BLOCK_PARALLEL: x += mixer(h) + ff(h), h = norm(x). */
 int nvl_create_layers(const nvl_model_config* cfg, const nvl_layer_config* layers, const nvl_runtime_opts* opts, nvl_model** out);
 
 /* Replaces loadTensorFromData + the per-kind placement in loadAttention/loadFFN/loadMoE/loadNorm
@@ -227,9 +247,9 @@ int nvl_load_safetensors(nvl_model* m, const char* path);
  * the reference's model_info.json) -> nvl_model_config.  Reference quirks kept: max_position_embeddings and
  * rope_scaling are not read.  Errors are reported through nvl_last_error(NULL). */
 int nvl_load_config_json(const char* path, nvl_model_config* cfg);
-/* The layer list of a config.json whose architecture is described by one ("Potuzen", "Lufazen"): writes up to `cap` entries, returns
- * how many the file has; 0 for every other architecture.  Such a file names no longest sequence: nvl_load_config_json sets
- * max_seq_len to 4096, the caller may change it before nvl_create_layers. */
+/* The layer list of a config.json whose architecture is described by one ("Potuzen", "Lufazen", "Bolinex"): writes up to `cap` entries, returns
+ * how many the file has; 0 for every other architecture.  A file that names no longest sequence (max_positions): nvl_load_config_json
+ * sets max_seq_len to 4096, the caller may change it before nvl_create_layers (a smaller one always). */
 int nvl_load_layers_json(const char* path, nvl_layer_config* layers, int cap);
 
 /* Helpers for checkpoints that keep fused projections (generic_loader.go:674-765):

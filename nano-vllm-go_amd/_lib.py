@@ -21,20 +21,22 @@ SLOTS = [
     "mamba_in_proj", "mamba_conv_w", "mamba_conv_b", "mamba_a_log", "mamba_d", "mamba_dt_bias", "mamba_norm", "mamba_out_proj",
     "mix_post_norm", "ffn_post_norm", "mix_gate", "lat_dq", "lat_dq_norm", "lat_uq", "lat_dkv", "lat_dkv_norm", "lat_uk", "lat_uv",
     "gla_norm", "gla_a1", "gla_a2", "gla_a2_b", "mix_scale", "ffn_scale", "delta_conv", "delta_beta", "delta_g1", "delta_g2",
+    "bias_r1", "bias_r2", "v_mix", "router_bias", "side_gate", "side_proj", "side_norm", "side_emb",
 ]
 SLOT_ID = {n: i for i, n in enumerate(SLOTS)}
 ONE_D = {"final_norm_w", "final_norm_b", "attn_norm_w", "attn_norm_b", "ffn_norm_w", "ffn_norm_b",
          "bq", "bk", "bv", "bo", "b1", "b2",
          "mamba_conv_w", "mamba_conv_b", "mamba_a_log", "mamba_d", "mamba_dt_bias", "mamba_norm",
-         "mix_post_norm", "ffn_post_norm", "lat_dq_norm", "lat_dkv_norm", "gla_norm", "gla_a2_b", "mix_scale", "ffn_scale", "delta_conv"}
+         "mix_post_norm", "ffn_post_norm", "lat_dq_norm", "lat_dkv_norm", "gla_norm", "gla_a2_b", "mix_scale", "ffn_scale", "delta_conv",
+         "bias_r1", "bias_r2", "v_mix", "router_bias", "side_norm"}
 OUT_IN_SLOTS = {"mamba_in_proj", "mamba_out_proj"}      # kept in the checkpoint's [out, in] layout by the reference's loader
 
 ATTN = {"mha": 0, "mqa": 1, "gqa": 2}
 NORM = {"layernorm": 0, "rmsnorm": 1}
 POS = {"learned": 0, "rope": 1, "nope": 2}
-ACT = {"gelu": 0, "swiglu": 1, "geglu": 2, "clamped_glu": 3}
+ACT = {"gelu": 0, "swiglu": 1, "geglu": 2, "clamped_glu": 3, "relu2": 4}
 BLOCK = {"sequential": 0, "parallel": 1, "sandwich": 2, "post": 3}
-MIXER = {"latent_attention": 0, "mamba2": 1, "gla": 2, "channel_delta": 3}
+MIXER = {"latent_attention": 0, "mamba2": 1, "gla": 2, "channel_delta": 3, "attention": 4}
 PRECISION = {"bf16": 0, "f32": 1}
 DTYPE_F32, DTYPE_BF16, DTYPE_F16 = 0, 1, 2
 LAYOUT_IN_OUT, LAYOUT_OUT_IN = 0, 1
@@ -65,7 +67,7 @@ class ModelConfigC(C.Structure):
         ("mamba_expand", C.c_int32), ("mamba_state_size", C.c_int32), ("mamba_num_heads", C.c_int32),
         ("mamba_head_dim", C.c_int32), ("mamba_n_groups", C.c_int32), ("mamba_conv_kernel", C.c_int32),
         ("mamba_layer_mask", C.c_uint64 * 2),
-        ("norm_weight_offset", C.c_float), ("logit_softcap", C.c_float),
+        ("norm_weight_offset", C.c_float), ("logit_softcap", C.c_float), ("side_dim", C.c_int32),
     ]
 
 
@@ -75,7 +77,9 @@ class LayerConfigC(C.Structure):        # nvl_layer_config
                 ("state", C.c_int32), ("groups", C.c_int32), ("norm_groups", C.c_int32), ("conv_taps", C.c_int32),
                 ("tau", C.c_float), ("decay_rank", C.c_int32), ("ffn_dim", C.c_int32),
                 ("ffn_limit", C.c_float), ("kv_from", C.c_int32), ("rot_dim", C.c_int32), ("gate_per_head", C.c_int32), ("kv_heads", C.c_int32),
-                ("rot_base", C.c_double), ("rot_factor", C.c_double), ("rot_original", C.c_double), ("rot_fast", C.c_double), ("rot_slow", C.c_double)]
+                ("rot_base", C.c_double), ("rot_factor", C.c_double), ("rot_original", C.c_double), ("rot_fast", C.c_double), ("rot_slow", C.c_double),
+                ("softcap", C.c_float), ("v_mix", C.c_int32), ("ffn_act", C.c_int32), ("experts", C.c_int32), ("top_k", C.c_int32),
+                ("expert_dim", C.c_int32), ("expert_groups", C.c_int32), ("groups_kept", C.c_int32)]
 
 
 class RuntimeOptsC(C.Structure):

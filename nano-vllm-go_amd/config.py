@@ -48,6 +48,7 @@ class ModelConfig:
     layers: list = field(default_factory=list)            # models described by a list of layers: one dict per layer (LAYER_FIELDS)
     norm_weight_offset: float = 0.0
     logit_softcap: float = 0.0
+    side_dim: int = 0                 # per-layer token inputs
 
     @property
     def mamba_layer_mask(self):
@@ -138,7 +139,9 @@ def new_granite_config(size: str = "350m") -> ModelConfig:   # config.go:241-330
 
 LAYER_FIELDS = dict(mixer="", weights_of=-1, heads=0, dim=0, vdim=0, q_rank=0, kv_rank=0, window=0, scale=0.0, state=0, groups=0,
                     norm_groups=0, conv_taps=0, tau=0.0, decay_rank=0, ffn_dim=0, ffn_limit=0.0, kv_from=-1, rot_dim=0, gate_per_head=0, kv_heads=0,
-                    rot_base=0.0, rot_factor=0.0, rot_original=0.0, rot_fast=0.0, rot_slow=0.0)      # nvl_layer_config
+                    rot_base=0.0, rot_factor=0.0, rot_original=0.0, rot_fast=0.0, rot_slow=0.0, softcap=0.0, v_mix=0, ffn_act=0, experts=0, top_k=0,
+                    expert_dim=0, expert_groups=0, groups_kept=0)      # nvl_layer_config
+ACT_SWIGLU = 1                                                         # NVL_ACT_SWIGLU (ffn_act)
 
 
 def _potuzen_layer(e: dict) -> dict:
@@ -204,7 +207,37 @@ def lufazen_config(raw: dict) -> ModelConfig:
                        norm_weight_offset=1.0, logit_softcap=float(raw.get("logit_softcap") or 0.0), layers=[_lufazen_layer(e) for e in raw["layers"]])
 
 
-LAYERED = {"Potuzen": potuzen_config, "Lufazen": lufazen_config}      # architectures described by a list of layers
+def _bolinex_layer(e: dict) -> dict:
+    """One entry of a Bolinex config.json's layer list -> the fields of nvl_layer_config."""
+    mx, mlp, ty = e["mixer"], e.get("mlp"), e["type"]
+    if ty != "attention":
+        raise ValueError(f"unknown mixer {ty!r}")
+    out = dict(LAYER_FIELDS, mixer=ty, heads=mx["heads"], kv_heads=mx["kv_heads"], dim=mx["dim"], vdim=mx["vdim"], scale=float(mx["scale"]),
+               softcap=float(mx.get("softcap") or 0.0), v_mix=int(bool(mx.get("v_mix"))), window=(mx.get("mask") or {}).get("size", 0))
+    if mlp is None:
+        return out
+    kind = mlp.get("kind", "dense")
+    if kind == "moe":
+        ro, groups = mlp["router"], mlp["router"].get("groups") or dict(count=1, keep=1)
+        out.update(expert_dim=mlp["expert"]["ff"], experts=ro["experts"], top_k=ro["top"], expert_groups=groups["count"], groups_kept=groups["keep"],
+                   ffn_dim=(mlp.get("shared") or {}).get("ff", 0), ffn_act=ACT_SWIGLU)
+    elif kind == "dense":
+        out["ffn_dim"] = mlp["ff"]
+    else:
+        raise ValueError(f"unknown feed-forward kind {kind!r}")
+    return out
+
+
+def bolinex_config(raw: dict) -> ModelConfig:
+    """The Bolinex design: parallel blocks behind one layer norm, grouped-query attention (capped scores, logarithmic distance bias,
+    windows, mixed values, output gate), squared-ReLU or expert feed-forwards, learned positions, per-layer token inputs."""
+    return ModelConfig(architecture="Bolinex", model_name="bolinex", vocab_size=raw["vocab"], hidden=raw["width"],
+                       num_layers=len(raw["layers"]), max_seq_len=raw["max_positions"], attention_type="gqa", norm_type="layernorm", position_type="learned",
+                       activation_type="relu2", block_style="parallel", rope_base=0.0, norm_eps=float(raw["norm"]["eps"]),
+                       side_dim=(raw.get("token_side") or {}).get("dim", 0), layers=[_bolinex_layer(e) for e in raw["layers"]])
+
+
+LAYERED = {"Potuzen": potuzen_config, "Lufazen": lufazen_config, "Bolinex": bolinex_config}      # architectures described by a list of layers
 
 
 def load_model_config(raw: dict | str) -> ModelConfig:

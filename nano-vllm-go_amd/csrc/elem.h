@@ -237,17 +237,18 @@ __device__ __forceinline__ void norm_row_finish(f32x4 (&v)[NORM_ROW_MAXCH], f32x
         float s = 0.f;
 #pragma unroll
         for (int c = 0; c < NORM_ROW_MAXCH; c++) s += v[c][0] + v[c][1] + v[c][2] + v[c][3];   // zero-filled beyond H
-        const float mean = block256_sum(s, red) / (float)H;
+        const int W = width ? width : H;
+        const float mean = block256_sum(s, red) / (float)W;
         float vs = 0.f;
 #pragma unroll
         for (int c = 0; c < NORM_ROW_MAXCH; c++) {
             const int j = threadIdx.x + c * 256;
             if (j < H4) {
 #pragma unroll
-                for (int k = 0; k < 4; k++) { const float d = v[c][k] - mean; vs += d * d; }
+                for (int k = 0; k < 4; k++) { const float d = v[c][k] - mean; vs += j * 4 + k < W ? d * d : 0.f; }
             }
         }
-        const float sd = sqrtf(block256_sum(vs, red) / (float)H + eps);
+        const float sd = sqrtf(block256_sum(vs, red) / (float)W + eps);
 #pragma unroll
         for (int c = 0; c < NORM_ROW_MAXCH; c++) {
             const int j = threadIdx.x + c * 256;
@@ -312,14 +313,39 @@ struct SandwichArgs {
     float* x;                 // residual stream [rows][H]
     const float* y;           // [slices][.][H] or NULL
     int slices; int64_t slice_stride;
-    const float* w_post;      // [H]
+    const float* w_post;      // [H]; EXT: NULL: y is added as it is
     const float* w_next;      // [H] or NULL
     const int32_t* rows_idx;  // y == NULL only: which row of x feeds output row r
     int rows, H, width;
     float eps;
     int raw_next;             // w_next == NULL: xn = x
+    // EXT instances
+    const float* b_next;      // not NULL: the norm that follows is a layer norm with this bias
+    const float* y2;          // a second source, added as it is: [slices2][.][H], or with slot_of the rows slot_of[r * slices2 + k], weighted by gate_w
+    int slices2; int64_t stride2;
+    const int32_t* slot_of; const float* gate_w;
 };
-template <typename ActT, int MAXCH>
+// four columns of everything that joins row r (EXT)
+__device__ __forceinline__ f32x4 sandwich_more(const SandwichArgs& p, int r, int col) {
+    f32x4 a = f32x4{0.f, 0.f, 0.f, 0.f};
+    if (p.slot_of) for (int k = 0; k < p.slices2; k++) a += p.gate_w[(int64_t)r * p.slices2 + k] * *(const f32x4*)(p.y2 + (int64_t)p.slot_of[(int64_t)r * p.slices2 + k] * p.H + col);
+    else for (int k = 0; k < p.slices2; k++) a += *(const f32x4*)(p.y2 + k * p.stride2 + (int64_t)r * p.H + col);
+    return a;
+}
+// sum over the row's data columns of (x - mean)^2 held by this thread: chunk c is columns (first + c * step) * 4 ..
+template <int MAXCH>
+__device__ __forceinline__ float sandwich_sq_dev(const f32x4 (&x)[MAXCH], float mean, int first, int step, int width) {
+    float vs = 0.f;
+#pragma unroll
+    for (int c = 0; c < MAXCH; c++) {
+        const int j = (first + c * step) * 4;
+#pragma unroll
+        for (int k = 0; k < 4; k++) { const float d = x[c][k] - mean; vs += j + k < width ? d * d : 0.f; }
+    }
+    return vs;
+}
+// EXT: layer norms, plain adds and a second source (layers whose sublayers join the stream together)
+template <typename ActT, int MAXCH, bool EXT = false>
 __global__ __launch_bounds__(256) void sandwich_row_kernel(SandwichArgs p, ActT* __restrict__ xn) {
     __shared__ float red[4];
     const int r = blockIdx.x, H4 = p.H >> 2;
@@ -339,10 +365,18 @@ __global__ __launch_bounds__(256) void sandwich_row_kernel(SandwichArgs p, ActT*
                 y[c] = *(const f32x4*)yr;
                 for (int k = 1; k < p.slices; k++) y[c] += *(const f32x4*)(yr + k * p.slice_stride);
             }
+            if constexpr (EXT) if (p.y2) y[c] += sandwich_more(p, r, j * 4);
         }
         ss += y[c][0] * y[c][0] + y[c][1] * y[c][1] + y[c][2] * y[c][2] + y[c][3] * y[c][3];
     }
-    if (p.y) {
+    if (EXT && p.y && !p.w_post) {
+#pragma unroll
+        for (int c = 0; c < MAXCH; c++) {
+            const int j = threadIdx.x + c * 256;
+            x[c] += y[c];
+            if (j < H4) *(f32x4*)(xr + j * 4) = x[c];
+        }
+    } else if (p.y) {
         const float rms = sqrtf(block256_sum(ss, red) / (float)p.width + p.eps);
 #pragma unroll
         for (int c = 0; c < MAXCH; c++) {
@@ -361,6 +395,25 @@ __global__ __launch_bounds__(256) void sandwich_row_kernel(SandwichArgs p, ActT*
             for (int c = 0; c < MAXCH; c++) { const int j = threadIdx.x + c * 256; if (j < H4) act_store4<ActT>(xn, r, j * 4, p.H, x[c]); }
         return;
     }
+    if constexpr (EXT) if (p.b_next) {
+        float sx = 0.f;
+#pragma unroll
+        for (int c = 0; c < MAXCH; c++) sx += (x[c][0] + x[c][1]) + (x[c][2] + x[c][3]);
+        const float mean = block256_sum(sx, red) / (float)p.width;
+        const float sd = sqrtf(block256_sum(sandwich_sq_dev<MAXCH>(x, mean, threadIdx.x, 256, p.width), red) / (float)p.width + p.eps);
+#pragma unroll
+        for (int c = 0; c < MAXCH; c++) {
+            const int j = threadIdx.x + c * 256;
+            if (j < H4) {
+                const f32x4 w = *(const f32x4*)(p.w_next + j * 4), b = *(const f32x4*)(p.b_next + j * 4);
+                f32x4 o;
+#pragma unroll
+                for (int k = 0; k < 4; k++) o[k] = ((x[c][k] - mean) / sd) * w[k] + b[k];
+                act_store4<ActT>(xn, r, j * 4, p.H, o);
+            }
+        }
+        return;
+    }
     ss = 0.f;
 #pragma unroll
     for (int c = 0; c < MAXCH; c++) ss += x[c][0] * x[c][0] + x[c][1] * x[c][1] + x[c][2] * x[c][2] + x[c][3] * x[c][3];
@@ -377,7 +430,7 @@ __global__ __launch_bounds__(256) void sandwich_row_kernel(SandwichArgs p, ActT*
         }
     }
 }
-template <int MAXCH>
+template <int MAXCH, bool EXT = false>
 __global__ __launch_bounds__(1024) void sandwich_tile16_kernel(SandwichArgs p, bf16_t* __restrict__ xn) {
     extern __shared__ __attribute__((aligned(16))) char smem_n[];
     bf16_t* tile = (bf16_t*)smem_n;                       // [16][H]
@@ -392,7 +445,17 @@ __global__ __launch_bounds__(1024) void sandwich_tile16_kernel(SandwichArgs p, b
             const int j = lane + c * 64;
             x[c] = j < H4 ? *(const f32x4*)(xr + j * 4) : f32x4{0.f, 0.f, 0.f, 0.f};
         }
-        if (p.y) {
+        if (EXT && p.y && !p.w_post) {
+#pragma unroll
+            for (int c = 0; c < MAXCH; c++) {
+                const int j = lane + c * 64;
+                if (j < H4) {
+                    x[c] += *(const f32x4*)(p.y + (int64_t)r * p.H + j * 4);
+                    if (p.y2) x[c] += sandwich_more(p, r, j * 4);
+                    *(f32x4*)(xr + j * 4) = x[c];
+                }
+            }
+        } else if (p.y) {
             f32x4 y[MAXCH];
             float ss = 0.f;
 #pragma unroll
@@ -423,7 +486,24 @@ __global__ __launch_bounds__(1024) void sandwich_tile16_kernel(SandwichArgs p, b
                 if (j < H4) *(bf16x4*)(tile + wave * p.H + j * 4) = o;
             }
         }
-        if (p.w_next) {
+        if (EXT && p.w_next && p.b_next) {
+            float sx = 0.f;
+#pragma unroll
+            for (int c = 0; c < MAXCH; c++) sx += (x[c][0] + x[c][1]) + (x[c][2] + x[c][3]);
+            const float mean = wave_sum(sx) / (float)p.width;
+            const float sd = sqrtf(wave_sum(sandwich_sq_dev<MAXCH>(x, mean, lane, 64, p.width)) / (float)p.width + p.eps);
+#pragma unroll
+            for (int c = 0; c < MAXCH; c++) {
+                const int j = lane + c * 64;
+                if (j < H4) {
+                    const f32x4 w = *(const f32x4*)(p.w_next + j * 4), b = *(const f32x4*)(p.b_next + j * 4);
+                    bf16x4 o;
+#pragma unroll
+                    for (int k = 0; k < 4; k++) o[k] = (bf16_t)(((x[c][k] - mean) / sd) * w[k] + b[k]);
+                    *(bf16x4*)(tile + wave * p.H + j * 4) = o;
+                }
+            }
+        } else if (p.w_next) {
             float ss = 0.f;
 #pragma unroll
             for (int c = 0; c < MAXCH; c++) ss += x[c][0] * x[c][0] + x[c][1] * x[c][1] + x[c][2] * x[c][2] + x[c][3] * x[c][3];
@@ -531,14 +611,14 @@ __global__ void fill_i32_kernel(int32_t* __restrict__ p, int32_t v, int n) {
     const int i = blockIdx.x * blockDim.x + threadIdx.x;
     if (i < n) p[i] = v;
 }
-// h [rows][2F] = [gate | up] -> y [rows][F] = silu(gate)*up   (transformer.go:50-66)
+// h [rows][2F] = [gate | up] -> y [rows][ld] at column col = silu(gate)*up   (transformer.go:50-66)
 template <typename ActT, bool GELU = false>       // GELU: gelu_tanh(gate)*up
-__global__ void swiglu_kernel(const float* __restrict__ h, ActT* __restrict__ y, int64_t rows, int F) {
+__global__ void swiglu_kernel(const float* __restrict__ h, ActT* __restrict__ y, int64_t rows, int F, int64_t ld, int col) {
     const int64_t i = (int64_t)blockIdx.x * blockDim.x + threadIdx.x;
     if (i >= rows * F) return;
     const int64_t r = i / F; const int f = (int)(i - r * F);
     const float g = h[r * 2 * F + f], u = h[r * 2 * F + F + f];
-    ActIO<ActT>::st(y + i, (GELU ? gelu_tanh_f(g) : g / (1.0f + expf(-g))) * u);
+    ActIO<ActT>::st(y + r * ld + col + f, (GELU ? gelu_tanh_f(g) : g / (1.0f + expf(-g))) * u);
 }
 template <typename ActT>
 __global__ void clamp_glu_kernel(const float* __restrict__ h, ActT* __restrict__ y, int64_t rows, int F, float limit, float slope) {
@@ -546,6 +626,23 @@ __global__ void clamp_glu_kernel(const float* __restrict__ h, ActT* __restrict__
     if (i >= rows * F) return;
     const int64_t r = i / F; const int f = (int)(i - r * F);
     ActIO<ActT>::st(y + i, clamp_glu_f(h[r * 2 * F + f], h[r * 2 * F + F + f], limit, slope));
+}
+// h [rows][F] -> y [rows][ld] at column col: max(h, 0)^2
+template <typename ActT>
+__global__ void relu2_kernel(const float* __restrict__ h, ActT* __restrict__ y, int64_t rows, int F, int64_t ld, int col) {
+    const int64_t i = (int64_t)blockIdx.x * blockDim.x + threadIdx.x;
+    if (i >= rows * F) return;
+    const int64_t r = i / F; const int f = (int)(i - r * F);
+    const float v = fmaxf(h[i], 0.f);
+    ActIO<ActT>::st(y + act_index<ActT>(r, col + f, ld), v * v);
+}
+// h [rows][n] -> y [rows][ld]: gelu_tanh(h) * (the token's row of a table)
+template <typename ActT, typename TabT>
+__global__ void gelu_token_kernel(const float* __restrict__ h, int64_t h_ld, const TabT* __restrict__ table, int64_t table_ld, const int32_t* __restrict__ ids,
+                                  ActT* __restrict__ y, int64_t ld, int n) {
+    const int64_t r = blockIdx.x;
+    for (int i = threadIdx.x; i < n; i += blockDim.x)
+        ActIO<ActT>::st(y + act_index<ActT>(r, i, ld), gelu_tanh_f(h[r * h_ld + i]) * (float)table[(int64_t)ids[r] * table_ld + i]);
 }
 __global__ void gelu_kernel(const float* __restrict__ x, float* __restrict__ y, int64_t n) {
     const int64_t i = (int64_t)blockIdx.x * blockDim.x + threadIdx.x;
@@ -874,6 +971,68 @@ __global__ __launch_bounds__(1024) void moe_plan_kernel(const float* __restrict_
     }
 }
 
+// Group-limited routing on sigmoid scores.  s = sigmoid(z); the choice goes by s + correction, the weights are the s of the chosen
+// experts as they are.  Experts form `groups` equal groups of neighbours; a group counts as much as its two largest choice scores
+// together, and only the experts of the best `keep` groups can be chosen.  Ties go to the lower index.  One wave per token, E <= 256;
+// writes (id, weight) in rank order, or with `gate` the dense [rows][gate_ld] matrix of weights (0: not chosen).
+constexpr int ROUTE_MAX_E = 256;
+struct GroupRouteArgs { const float* logits; int64_t ld; const float* correction; int rows, E, top, groups, keep; int32_t* ids; float* w; float* gate; int gate_ld; };
+__global__ __launch_bounds__(256) void moe_route_grouped_kernel(GroupRouteArgs p) {
+    __shared__ float choice_s[4][ROUTE_MAX_E], group_s[4][ROUTE_MAX_E];
+    const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, r = blockIdx.x * 4 + wave;
+    const int size = p.E / p.groups;
+    float *choice = choice_s[wave], *group = group_s[wave];
+    float s[ROUTE_MAX_E / 64];
+    if (r < p.rows)
+#pragma unroll
+        for (int i = 0; i < ROUTE_MAX_E / 64; i++) {
+            const int e = lane + 64 * i;
+            s[i] = 0.f;
+            if (e < p.E) {
+                s[i] = 1.0f / (1.0f + expf(-p.logits[r * p.ld + e]));
+                choice[e] = s[i] + (p.correction ? p.correction[e] : 0.f);
+            }
+        }
+    __syncthreads();
+    if (r < p.rows)
+        for (int g = lane; g < p.groups; g += 64) {
+            float a = -INFINITY, b = -INFINITY;           // the two largest
+            for (int j = 0; j < size; j++) {
+                const float c = choice[g * size + j];
+                if (c > a) { b = a; a = c; } else b = fmaxf(b, c);
+            }
+            group[g] = size > 1 ? a + b : a;
+        }
+    __syncthreads();
+    auto kept = [&](int g) {
+        int rank = 0;
+        const float v = group[g];
+        for (int j = 0; j < p.groups; j++) rank += group[j] > v || (group[j] == v && j < g);
+        return rank < p.keep;
+    };
+    bool in[ROUTE_MAX_E / 64];
+    float c[ROUTE_MAX_E / 64];
+#pragma unroll
+    for (int i = 0; i < ROUTE_MAX_E / 64; i++) {
+        const int e = lane + 64 * i;
+        in[i] = r < p.rows && e < p.E && kept(e / size);
+        c[i] = r < p.rows && e < p.E ? choice[e] : 0.f;
+        if (r < p.rows && e < p.E && !in[i]) choice[e] = -INFINITY;       // (read by nobody but this lane so far)
+    }
+    __syncthreads();
+#pragma unroll
+    for (int i = 0; i < ROUTE_MAX_E / 64; i++) {
+        const int e = lane + 64 * i;
+        if (r < p.rows && p.gate && e >= p.E && e < p.gate_ld) p.gate[(int64_t)r * p.gate_ld + e] = 0.f;       // padding experts
+        if (r >= p.rows || e >= p.E) continue;
+        int rank = 0;
+        if (in[i]) for (int j = 0; j < p.E; j++) { const float v = choice[j]; rank += v > c[i] || (v == c[i] && j < e); }
+        const bool chosen = in[i] && rank < p.top;
+        if (p.gate) p.gate[(int64_t)r * p.gate_ld + e] = chosen ? s[i] : 0.f;
+        else if (chosen) { p.ids[(int64_t)r * p.top + rank] = e; p.w[(int64_t)r * p.top + rank] = s[i]; }
+    }
+}
+
 // out[t] (+)= resid_mult * sum_rank w[t][rank] * eo[slot_of(t,rank)]   in rank order
 // (moe.go:117-119 accumulates in expert-rank order; generic_model.go:383-389 adds the residual)
 __global__ void moe_combine_kernel(const float* __restrict__ eo, const int32_t* __restrict__ slot_of,
@@ -899,12 +1058,12 @@ __global__ void moe_combine_kernel(const float* __restrict__ eo, const int32_t* 
 //   moe_scatter_kernel each pair takes the next row of its expert's segment (atomic cursor).  The row a pair
 //                      lands on can differ from run to run, the VALUES cannot: every pair is computed
 //                      independently and moe_combine_kernel reads them back through slot_of in rank order.
-// prefill-sized batches: per-workgroup counts in LDS first (E <= 64), so the global counters see one atomic per
+// prefill-sized batches: per-workgroup counts in LDS first (E <= MOE_MAX_E), so the global counters see one atomic per
 // (workgroup, expert) instead of one per pair (32768 pairs on 32 addresses: 57 -> ~10 us)
-constexpr int MOE_PAIRS_PER_WG = 1024;
+constexpr int MOE_PAIRS_PER_WG = 1024, MOE_MAX_E = 256;
 __global__ __launch_bounds__(256) void moe_hist_kernel(const int32_t* __restrict__ expert_ids, int n_pairs, int32_t* __restrict__ counts) {
-    __shared__ int lc[64];
-    if (threadIdx.x < 64) lc[threadIdx.x] = 0;
+    __shared__ int lc[MOE_MAX_E];
+    lc[threadIdx.x] = 0;
     __syncthreads();
 #pragma unroll
     for (int j = 0; j < MOE_PAIRS_PER_WG / 256; j++) {
@@ -912,7 +1071,7 @@ __global__ __launch_bounds__(256) void moe_hist_kernel(const int32_t* __restrict
         if (i < n_pairs) atomicAdd(&lc[expert_ids[i]], 1);
     }
     __syncthreads();
-    if (threadIdx.x < 64 && lc[threadIdx.x]) atomicAdd(&counts[threadIdx.x], lc[threadIdx.x]);
+    if (lc[threadIdx.x]) atomicAdd(&counts[threadIdx.x], lc[threadIdx.x]);
 }
 // prefill: rows of the fragment-major activation matrix copied into expert order (dst row i = src row perm[i]), one
 // workgroup per 16 destination rows; a wave moves whole 1-KiB operand blocks (coalesced stores, 16-byte gathers)
@@ -931,27 +1090,31 @@ __global__ __launch_bounds__(256) void moe_gather_fm_kernel(const bf16_t* __rest
 __global__ __launch_bounds__(64) void moe_scan_kernel(const int32_t* __restrict__ counts, int E, int BM,
                                                       int32_t* __restrict__ seg_start, int32_t* __restrict__ cursor,
                                                       int32_t* __restrict__ tile_map, int32_t* __restrict__ n_mtiles) {
-    // exclusive scans over the experts (E <= 64: one lane each): first row and first m-tile of every segment
+    // exclusive scans over the experts, 64 at a time (one lane each): first row and first m-tile of every segment
     const int lane = threadIdx.x;
-    const int c = lane < E ? counts[lane] : 0;
-    const int nt_e = (c + BM - 1) / BM;
-    int row = c, tile = nt_e;
+    int rows = 0, tiles = 0;                         // of the experts before this batch of 64
+    for (int e0 = 0; e0 < E; e0 += 64) {
+        const int e = e0 + lane, c = e < E ? counts[e] : 0;
+        const int nt_e = (c + BM - 1) / BM;
+        int row = c, tile = nt_e;
 #pragma unroll
-    for (int o = 1; o < 64; o <<= 1) {
-        const int yr = __shfl_up(row, o, 64), yt = __shfl_up(tile, o, 64);
-        if (lane >= o) { row += yr; tile += yt; }
-    }
-    const int row0 = row - c, tile0 = tile - nt_e;
-    if (lane < E) {
-        seg_start[lane] = row0;
-        cursor[lane] = row0;
-        for (int t = 0; t < nt_e; t++) {
-            const int r = t * BM;
-            tile_map[4 * (tile0 + t)] = lane; tile_map[4 * (tile0 + t) + 1] = row0 + r;
-            tile_map[4 * (tile0 + t) + 2] = (c - r < BM) ? (c - r) : BM; tile_map[4 * (tile0 + t) + 3] = 0;
+        for (int o = 1; o < 64; o <<= 1) {
+            const int yr = __shfl_up(row, o, 64), yt = __shfl_up(tile, o, 64);
+            if (lane >= o) { row += yr; tile += yt; }
         }
+        const int row0 = rows + row - c, tile0 = tiles + tile - nt_e;
+        if (e < E) {
+            seg_start[e] = row0;
+            cursor[e] = row0;
+            for (int t = 0; t < nt_e; t++) {
+                const int r = t * BM;
+                tile_map[4 * (tile0 + t)] = e; tile_map[4 * (tile0 + t) + 1] = row0 + r;
+                tile_map[4 * (tile0 + t) + 2] = (c - r < BM) ? (c - r) : BM; tile_map[4 * (tile0 + t) + 3] = 0;
+            }
+        }
+        rows += __shfl(row, 63, 64); tiles += __shfl(tile, 63, 64);
     }
-    if (lane == 63) { seg_start[E] = row; *n_mtiles = tile; }
+    if (lane == 0) { seg_start[E] = rows; *n_mtiles = tiles; }
 }
 __global__ __launch_bounds__(256) void moe_scatter_kernel(const int32_t* __restrict__ expert_ids, int n_pairs, int top_k,
                                    int32_t* __restrict__ cursor, int32_t* __restrict__ perm_token,
@@ -959,8 +1122,8 @@ __global__ __launch_bounds__(256) void moe_scatter_kernel(const int32_t* __restr
     // rank inside the workgroup from LDS atomics, one global reservation per (workgroup, expert).  The row order inside
     // an expert's segment varies from run to run; no output depends on it (rows are independent, the combine sums a
     // token's slots in rank order through slot_of).
-    __shared__ int lc[64], base[64];
-    if (threadIdx.x < 64) lc[threadIdx.x] = 0;
+    __shared__ int lc[MOE_MAX_E], base[MOE_MAX_E];
+    lc[threadIdx.x] = 0;
     __syncthreads();
     int e[MOE_PAIRS_PER_WG / 256], r[MOE_PAIRS_PER_WG / 256];
 #pragma unroll
@@ -970,7 +1133,7 @@ __global__ __launch_bounds__(256) void moe_scatter_kernel(const int32_t* __restr
         if (i < n_pairs) { e[j] = expert_ids[i]; r[j] = atomicAdd(&lc[e[j]], 1); }
     }
     __syncthreads();
-    if (threadIdx.x < 64 && lc[threadIdx.x]) base[threadIdx.x] = atomicAdd(&cursor[threadIdx.x], lc[threadIdx.x]);
+    if (lc[threadIdx.x]) base[threadIdx.x] = atomicAdd(&cursor[threadIdx.x], lc[threadIdx.x]);
     __syncthreads();
 #pragma unroll
     for (int j = 0; j < MOE_PAIRS_PER_WG / 256; j++) {
@@ -1029,16 +1192,17 @@ __global__ void convert_1d_kernel(const void* __restrict__ src, int dtype, float
 
 // Placement of a [N][K] source into a larger, zero-filled destination [.][Kd]: source row n lands in row
 // row0 + (n / rg) * rgp + n % rg, source column k in column (k / cg) * cgp + k % cg (groups padded from rg to rgp rows, cg to cgp
-// columns: per-head padding, the 16-row interleave of gate and up).  TRANS: the destination's rows are the source's columns.
-struct Place2D { int64_t N, K, Kd, row0; int rg, rgp, cg, cgp; };
+// columns: per-head padding, the 16-row interleave of gate and up), all shifted by col0 columns.  TRANS: the destination's rows are the source's columns.
+struct Place2D { int64_t N, K, Kd, row0; int rg, rgp, cg, cgp; int64_t col0; };
 template <typename DT, bool FM, bool TRANS>
 __global__ __launch_bounds__(256) void place_2d_kernel(const void* __restrict__ src, int dtype, int64_t src0, DT* __restrict__ dst, Place2D pl) {
-    const int64_t n = blockIdx.y;
+    const int64_t n = blockIdx.y + (int64_t)gridDim.y * blockIdx.z;
+    if (n >= pl.N) return;
     for (int64_t k = (int64_t)blockIdx.x * 256 + threadIdx.x; k < pl.K; k += (int64_t)gridDim.x * 256) {
         const float v = ld_as_f32(src, dtype, src0 + n * pl.K + k);
         int64_t a = (n / pl.rg) * pl.rgp + n % pl.rg, b = (k / pl.cg) * pl.cgp + k % pl.cg;
         if (TRANS) { const int64_t t = a; a = b; b = t; }
-        a += pl.row0;
+        a += pl.row0; b += pl.col0;
         dst[FM ? fm_index(a, b, pl.Kd) : a * pl.Kd + b] = (DT)v;
     }
 }

@@ -41,6 +41,8 @@ enum GemmEpi {
                      // round trip + rope_kv_kernel in prefill; Concatenate tensor.go:283-321)
     EPI_CLAMP_GLU = 6,   // C[m, f] = g sigmoid(slope g) (u + 1), g = min(gate, limit), u = clamp(up, -limit, limit); W as for EPI_SWIGLU
     EPI_GEGLU = 5,   // C[m, f] = gelu_tanh(gate) * up   W rows interleaved as for EPI_SWIGLU
+    EPI_RELU2 = 7,   // C = max(acc, 0)^2
+    EPI_GELU_TOK = 8,    // C[m, n] = gelu_tanh(acc) * tok_table[tok_ids[m]][n]   (an input of the token's own, GemmArgs::tok_*)
 };
 
 constexpr bool epi_glu(int epi) { return epi == 2 || epi == 5 || epi == 6; }      // gate | up pairs in, one column out
@@ -68,6 +70,7 @@ struct GemmArgs {
     const float* bias;      // [N] or NULL
     float alpha;            // EPI_RESID multiplier
     float glu_limit, glu_slope;     // EPI_CLAMP_GLU
+    const int32_t* tok_ids; const bf16_t* tok_table; int64_t tok_ld;      // EPI_GELU_TOK: row-major, rows of 4 k entries
     int M, N, K;            // logical sizes
     const int32_t* seg;     // optional device {start,end}: rows [start,end) of A (via a_rows if set)
                             // and of C; M is then only the grid bound (MoE expert segments)
@@ -144,7 +147,16 @@ __device__ __forceinline__ void epilogue4(const GemmArgs& p, int m, int n, f32x4
 #pragma unroll
         for (int r = 0; r < 4; r++) v[r] = gelu_tanh_f(v[r]);
     }
+    if (EPI == EPI_RELU2) {
+#pragma unroll
+        for (int r = 0; r < 4; r++) { const float t = fmaxf(v[r], 0.f); v[r] = t * t; }
+    }
     const int64_t row = (int64_t)p.c_row0 + m;
+    if (EPI == EPI_GELU_TOK) {
+        const bf16x4 e = *(const bf16x4*)(p.tok_table + (int64_t)p.tok_ids[row] * p.tok_ld + n);
+#pragma unroll
+        for (int r = 0; r < 4; r++) v[r] = gelu_tanh_f(v[r]) * (float)e[r];
+    }
     if (EPI == EPI_RESID) {
         float* x = (float*)p.C + row * p.ldc + n;
         if (full) {
@@ -1288,7 +1300,7 @@ static inline bool launch_gemm_skinny_bf16(hipStream_t st, const GemmArgs& a0) {
     if (skinny_rows(a0) > 64 || a0.a_rows || a0.seg || a0.tile_map) return false;
     GemmArgs a = a0;
     a.x_mask = (g_x_mask && a0.M % 16 != 0) ? 1 : 0;     // padded rows of the last 16-row activation tile are not fetched
-    if constexpr (epi_glu(EPI) || EPI == EPI_STORE || EPI == EPI_GELU) {
+    if constexpr (epi_glu(EPI) || EPI == EPI_STORE || EPI == EPI_GELU || EPI == EPI_RELU2) {
         // wide-N form once its 64-row groups fill the chip (g_force_ntw: 8 forces it, 1/2/4 force the narrow form)
         const bool wide_ok = skinny_rows(a) > 16 && cdiv(a.N, 64) >= 256 && !a.sk_part;   // M <= 16: the narrow form streams as fast
         if (g_force_ntw == 8 || (g_force_ntw == 0 && wide_ok)) { if (launch_gemm_skinny_wide<EPI, OutT>(st, a)) return true; }

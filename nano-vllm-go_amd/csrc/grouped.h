@@ -1,0 +1,501 @@
+// grouped.h — grouped-query attention of models described by a list of layers: H query heads share G key/value heads, query/key and
+// value sizes differ freely, and every score passes through
+//     s = q . k * scale;   s <- softcap tanh(s / softcap);   s <- s - r1 ln(1 + r2 (i - j))
+// (cap and bias are optional, r1 and r2 belong to the query head) before an ordinary softmax over an optional sliding window.  The
+// values may be mixed with those of an earlier layer before they are cached; the concatenated heads are multiplied by sigmoid(gate).
+// Scores, cap, bias, softmax and their sums are fp32.
+//
+// Cache: blocks of `bs` tokens (64 | bs) named by block tables.  A layer's part of a block is [G][bs][dp] keys, then [G][vp][bs] values,
+// dp / vp = padded head sizes (the padding is zero).  bf16: both are stored as the MFMA operand blocks they are read as (common.h
+// fm_index), so every operand of either kernel is one contiguous KiB of the cache: the keys of a 32-token unit in the order that
+// makes the score accumulators (keys 8 fg + r, 8 fg + 4 + r) the B operand against the values' natural order (grouped_k_row), the
+// values transposed.  fp32 mode: plain rows, values [G][bs][vp].
+//
+// A "query row" is a (token, head of the group) pair, token-major, so that all heads of a group use one pass over K and V:
+//   grouped_prefill_kernel : 8 waves x 32 rows, 64-key tiles of K and V^T through a 3-slot LDS ring filled by LDS-DMA (as latent.h)
+//   grouped_short_kernel   : sequences with few query rows (decoding, short portions): 16 rows, key tiles dealt over waves and workgroups
+//   grouped_plain_kernel   : fp32 mode, and heads wider than the instances above
+#pragma once
+#include "attn.h"
+#include "common.h"
+#include "latent.h"
+
+namespace nvl {
+
+struct GroupedArgs {
+    int H, G, group, dim, dp, vdim, vp;
+    int window;                                   // 0: every earlier token
+    float scale, softcap;                         // softcap 0: none
+    const float *r1, *r2;                         // [H] or NULL: no distance bias
+    const float* proj; int64_t proj_ld;           // [token][q : H dp | k : G dp | v : G vp | gate : H vp | ...] of the fused input projection
+    int k_off, v_off, gate_off;                   // gate_off < 0: no output gate
+    int mix;                                      // values: 0 as they are, 1 also the model's first (kept in vfirst), 2 mixed with vfirst
+    const float* lambda; float* vfirst; int64_t vfirst_ld;      // [token][G vp]
+    void* cache; int64_t block_stride; int bs;    // this layer's part of block 0; elements between blocks
+    const int32_t *blk_table, *seq_tok_start, *seq_len, *seq_pos;
+    int tbl_stride;
+    int short_rows;                               // sequences with up to this many query rows belong to grouped_short_kernel
+    void* out; int64_t out_ld;                    // operand of W_o: [token][out_ld], head h at column h * vp
+    float* part; int32_t* part_cnt;               // keys split over workgroups: partial results, arrival tickets (zero between launches)
+};
+
+// where token row `row` of a block's keys sits: tile row 16 t + 4 a + r holds token 8 a + 4 t + r of its 32-token unit
+__host__ __device__ __forceinline__ int grouped_k_row(int row) {
+    const int k = row & 31;
+    return (row & ~31) + 16 * ((k >> 2) & 1) + 4 * (k >> 3) + (k & 3);
+}
+
+// ---- keys and values of the batch's tokens into the cache: grid (32-token units of a sequence's new positions, sequences, G) ----
+template <typename ActT>
+__global__ __launch_bounds__(256) void grouped_place_kernel(GroupedArgs p) {
+    const int seq = blockIdx.y, g = blockIdx.z, n = p.seq_len[seq], pos0 = p.seq_pos[seq], tok0 = p.seq_tok_start[seq];
+    const int u0 = (pos0 & ~31) + blockIdx.x * 32;                     // first position of the unit
+    const int a = max(u0, pos0), b = min(u0 + 32, pos0 + n);           // positions [a, b) are written
+    if (a >= b) return;
+    const int bi = u0 / p.bs, row0 = u0 - bi * p.bs;
+    ActT* base = (ActT*)p.cache + (int64_t)p.blk_table[(int64_t)seq * p.tbl_stride + bi] * p.block_stride;
+    ActT* kc = base + (int64_t)g * p.bs * p.dp;
+    ActT* vc = base + (int64_t)p.G * p.bs * p.dp + (int64_t)g * p.bs * p.vp;
+    constexpr bool FM = sizeof(ActT) == 2;
+    const int q4 = p.dp >> 2;
+    for (int i = threadIdx.x; i < (b - a) * q4; i += 256) {
+        const int j = i / q4, c = (i - j * q4) * 4, row = row0 + a - u0 + j;
+        const f32x4 v = *(const f32x4*)(p.proj + (int64_t)(tok0 + a - pos0 + j) * p.proj_ld + p.k_off + g * p.dp + c);
+        act_store4<ActT>(kc, FM ? grouped_k_row(row) : row, c, p.dp, v);
+    }
+    const float lam = p.mix == 2 ? *p.lambda : 0.f;
+    for (int i = threadIdx.x; i < 4 * p.vp; i += 256) {                // (eight positions, value channel)
+        const int o = i / p.vp, c = i - o * p.vp, p0 = u0 + 8 * o;
+        if (p0 + 8 <= a || p0 >= b) continue;
+        float v[8];
+#pragma unroll
+        for (int e = 0; e < 8; e++) {
+            v[e] = 0.f;
+            const int pos = p0 + e;
+            if (pos < a || pos >= b) continue;
+            const int64_t t = tok0 + pos - pos0;
+            v[e] = p.proj[t * p.proj_ld + p.v_off + g * p.vp + c];
+            if (p.mix) {
+                float* f = p.vfirst + t * p.vfirst_ld + g * p.vp + c;
+                if (p.mix == 1) *f = v[e];
+                else v[e] = (1.0f - lam) * v[e] + lam * *f;
+            }
+        }
+        if constexpr (FM) {
+            ActT* d = vc + fm_index(c, row0 + 8 * o, p.bs);            // eight consecutive positions of a channel are contiguous
+            if (p0 >= a && p0 + 8 <= b) {
+                bf16x8 w;
+#pragma unroll
+                for (int e = 0; e < 8; e++) w[e] = (bf16_t)v[e];
+                *(bf16x8*)d = w;
+            } else {
+#pragma unroll
+                for (int e = 0; e < 8; e++) if (p0 + e >= a && p0 + e < b) d[e] = (ActT)v[e];
+            }
+        } else {
+#pragma unroll
+            for (int e = 0; e < 8; e++) if (p0 + e >= a && p0 + e < b) vc[(int64_t)(row0 + 8 * o + e) * p.vp + c] = (ActT)v[e];
+        }
+    }
+}
+
+// ---- scores in the exp2 domain ----
+struct GroupedScore {       // constants of one query row
+    float sc, c2, nr1, r2;
+    bool cap, bias;
+    __device__ __forceinline__ GroupedScore(const GroupedArgs& p, int head) {
+        constexpr float L2E = 1.4426950408889634f;
+        cap = p.softcap > 0.f; bias = p.r1 != nullptr;
+        sc = cap ? p.scale / p.softcap * (2.0f * L2E) : p.scale * L2E;      // cap: exp2(s sc) = exp(2 s scale / softcap)
+        c2 = -2.0f * p.softcap * L2E;                                       // softcap tanh(x) = softcap - 2 softcap / (exp(2 x) + 1); the softmax drops the first term
+        nr1 = bias ? -p.r1[head] : 0.f; r2 = bias ? p.r2[head] : 0.f;       // r1 ln(.) log2(e) = r1 log2(.)
+    }
+};
+// raw scores of one 64-key tile (tile-relative key 32 (t / 2) + 8 fg + 4 (t & 1) + r; `back`: the query's own place, tile-relative)
+__device__ __forceinline__ void grouped_scores(const GroupedScore& f, f32x4 (&s)[4], int back, int fg) {
+    if (f.cap) {
+#pragma unroll
+        for (int t = 0; t < 4; t++)
+#pragma unroll
+            for (int r = 0; r < 4; r++) s[t][r] = f.c2 * __builtin_amdgcn_rcpf(__builtin_amdgcn_exp2f(s[t][r] * f.sc) + 1.0f);
+    } else {
+#pragma unroll
+        for (int t = 0; t < 4; t++) s[t] *= f.sc;
+    }
+    if (f.bias) {
+        const float b = fmaf(f.r2, (float)(back - 8 * fg), 1.0f);
+#pragma unroll
+        for (int t = 0; t < 4; t++)
+#pragma unroll
+            for (int r = 0; r < 4; r++) s[t][r] = fmaf(f.nr1, __builtin_amdgcn_logf(fmaf(-f.r2, (float)(32 * (t >> 1) + 4 * (t & 1) + r), b)), s[t][r]);
+    }
+}
+__device__ __forceinline__ void grouped_mask(f32x4 (&s)[4], int back, int window, int fg) {
+    const int from = window > 0 ? back - window + 1 : 0;
+#pragma unroll
+    for (int t = 0; t < 4; t++)
+#pragma unroll
+        for (int r = 0; r < 4; r++) {
+            const int k = 32 * (t >> 1) + 8 * fg + 4 * (t & 1) + r;
+            if (k > back || k < from) s[t][r] = -INFINITY;
+        }
+}
+__device__ __forceinline__ void grouped_load_q(const float* q, int ks, int fg, bf16x8& f) {
+    const f32x4 a = *(const f32x4*)(q + ks * 32 + fg * 8), b = *(const f32x4*)(q + ks * 32 + fg * 8 + 4);
+#pragma unroll
+    for (int e = 0; e < 4; e++) { f[e] = (bf16_t)a[e]; f[4 + e] = (bf16_t)b[e]; }
+}
+// four channels of a finished row: gate, store
+__device__ __forceinline__ void grouped_store(const GroupedArgs& p, int64_t tok, int head, int c, f32x4 v) {
+    if (p.gate_off >= 0) {
+        const f32x4 g = *(const f32x4*)(p.proj + tok * p.proj_ld + p.gate_off + head * p.vp + c);
+#pragma unroll
+        for (int r = 0; r < 4; r++) v[r] *= lat_sigmoid(g[r]);
+    }
+    act_store4<bf16_t>((bf16_t*)p.out, tok, head * p.vp + c, p.out_ld, v);
+}
+
+template <int KS, int DT> constexpr int grouped_prefill_pieces() { return 4 * KS + 2 * DT; }       // 1-KiB operand blocks of a tile
+template <int KS, int DT> constexpr int grouped_prefill_ring_bytes() { return 3 * ((grouped_prefill_pieces<KS, DT>() + 7) / 8 * 8) * 1024; }
+
+// grid (G, sequences, 256-row tiles); dynamic LDS: the ring, then (block, row) of every key tile the workgroup walks
+template <int KS, int DT>
+__global__ __launch_bounds__(512, (KS <= 2 && DT <= 4) ? 4 : 2) void grouped_prefill_kernel(GroupedArgs p) {
+    constexpr int TQ = 2, PIECES = grouped_prefill_pieces<KS, DT>(), PW = (PIECES + 7) / 8, TILE = PW * 8 * 1024, NBUF = 3;
+    extern __shared__ __attribute__((aligned(16))) char grp_sm[];
+    int2* stile = (int2*)(grp_sm + NBUF * TILE);
+    // kv head fastest, query tile slowest and last first: the longest workgroups are dispatched first
+    const int kvh = blockIdx.x, seq = blockIdx.y, qt = gridDim.z - 1 - blockIdx.z;
+    const int R = p.seq_len[seq] * p.group;
+    if (R <= p.short_rows || qt * 256 >= R) return;
+    const int tok0 = p.seq_tok_start[seq], pos0 = p.seq_pos[seq];
+    const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6);
+    const int fq = lane & 15, fg = lane >> 4;
+    auto key_lo = [&](int pos) { const int lo = p.window > 0 ? pos - p.window + 1 : 0; return lo > 0 ? lo : 0; };
+    // key tiles of the workgroup, and of this wave (rows w_row0 .. + 31)
+    const int wg_first = pos0 + qt * 256 / p.group, wg_last = pos0 + (min(qt * 256 + 255, R - 1)) / p.group;
+    const int t0 = key_lo(wg_first) >> 6, n_kt = (wg_last >> 6) + 1;
+    const int w_row0 = qt * 256 + wave * 32;
+    const bool w_live = w_row0 < R;
+    const int first = pos0 + min(w_row0, R - 1) / p.group, last = pos0 + min(w_row0 + 31, R - 1) / p.group;
+    const int wt0 = w_live ? key_lo(first) >> 6 : n_kt, wt1 = w_live ? (last >> 6) + 1 : 0;
+    const int full_lo = p.window > 0 ? last - p.window + 1 : 0, full_hi = first;
+    for (int i = tid; i < n_kt - t0; i += 512) {
+        const int key = (t0 + i) * 64, bi = key / p.bs;
+        stile[i] = make_int2(p.blk_table[(int64_t)seq * p.tbl_stride + bi], key - bi * p.bs);
+    }
+    auto row_of = [&](int i, bool& ok) { const int r = w_row0 + 16 * i + fq; ok = r < R; return ok ? r : R - 1; };
+    bf16x8 qf[TQ][KS];
+    int qpos[TQ];
+    float r1v[TQ], r2v[TQ];
+#pragma unroll
+    for (int i = 0; i < TQ; i++) {
+        bool ok;
+        const int row = row_of(i, ok), si = row / p.group, head = kvh * p.group + row - si * p.group;
+        qpos[i] = pos0 + si;
+        const float* q = p.proj + (int64_t)(tok0 + si) * p.proj_ld + head * p.dp;
+#pragma unroll
+        for (int ks = 0; ks < KS; ks++) grouped_load_q(q, ks, fg, qf[i][ks]);
+        const GroupedScore f(p, head);
+        r1v[i] = f.nr1; r2v[i] = f.r2;
+    }
+    GroupedScore f(p, 0);
+#pragma unroll
+    for (int i = 0; i < TQ; i++) {
+#pragma unroll
+        for (int ks = 0; ks < KS; ks++) asm volatile("" : "+v"(qf[i][ks]));      // complete before the first DMA is issued (attn.h)
+        asm volatile("" : "+v"(r1v[i]), "+v"(r2v[i]));
+    }
+    asm volatile("" : "+v"(f.nr1), "+v"(f.r2));
+    __syncthreads();                      // stile is visible
+    // LDS-DMA: wave w moves pieces w * PW .. of [K: 16-key tile, k-step | V^T: d, 32-key unit]; surplus pieces repeat the last one
+    int64_t src[PW];
+#pragma unroll
+    for (int i = 0; i < PW; i++) {
+        int pc = wave * PW + i;
+        if (pc >= PIECES) pc = PIECES - 1;
+        if (pc < 4 * KS) src[i] = (int64_t)kvh * p.bs * p.dp + pc * 512 + lane * 8;
+        else {
+            const int v = pc - 4 * KS;
+            src[i] = (int64_t)p.G * p.bs * p.dp + (int64_t)kvh * p.bs * p.vp + ((int64_t)(v >> 1) * (p.bs >> 5) + (v & 1)) * 512 + lane * 8;
+        }
+    }
+    const uint32_t smem_lds = (uint32_t)(size_t)(__attribute__((address_space(3))) char*)grp_sm;
+    auto issue = [&](int kt, int buf) {
+        const int2 tl = stile[kt - t0];
+        const int blk = __builtin_amdgcn_readfirstlane(tl.x), row = __builtin_amdgcn_readfirstlane(tl.y);
+        const bf16_t* base = (const bf16_t*)p.cache + (int64_t)blk * p.block_stride;
+        const uint32_t dst = smem_lds + buf * TILE + wave * (PW * 1024);
+#pragma unroll
+        for (int i = 0; i < PW; i++) {
+            // a tile's 64 keys are 64 dp elements of the key blocks and two operand blocks of every value row
+            const bool is_k = wave * PW + i < 4 * KS;
+            const uint64_t a = (uint64_t)(base + src[i] + (int64_t)row * (is_k ? p.dp : 16));
+            asm volatile("s_mov_b32 m0, %0\n\ts_nop 4\n\tglobal_load_lds_dwordx4 %1, off" ::"s"(dst + i * 1024), "v"(a) : "memory");
+        }
+    };
+    f32x4 o[TQ][DT], lacc[TQ];
+    float m_run[TQ];
+#pragma unroll
+    for (int i = 0; i < TQ; i++) {
+        m_run[i] = -1e30f; lacc[i] = f32x4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+        for (int d = 0; d < DT; d++) o[i][d] = f32x4{0.f, 0.f, 0.f, 0.f};
+    }
+    bf16x8 ones;
+#pragma unroll
+    for (int e = 0; e < 8; e++) ones[e] = (bf16_t)1.0f;
+    issue(t0, 0);
+    if (t0 + 1 < n_kt) issue(t0 + 1, 1);
+    int buf = 0;
+    for (int kt = t0; kt < n_kt; kt++) {
+        if (kt + 1 < n_kt) wait_vm<PW>(); else wait_vm<0>();      // my pieces of tile kt have landed
+        __builtin_amdgcn_s_barrier();
+        if (kt + 2 < n_kt) { int nb = buf + 2; if (nb >= NBUF) nb -= NBUF; issue(kt + 2, nb); }
+        const char* kimg = grp_sm + buf * TILE + lane * 16;
+        const char* vimg = kimg + 4 * KS * 1024;
+        buf = buf + 1 == NBUF ? 0 : buf + 1;
+        if (kt < wt0 || kt >= wt1) continue;                      // (wave-uniform)
+        f32x4 s[TQ][4];
+#pragma unroll
+        for (int i = 0; i < TQ; i++)
+#pragma unroll
+            for (int t = 0; t < 4; t++) s[i][t] = f32x4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+        for (int t = 0; t < 4; t++)
+#pragma unroll
+            for (int ks = 0; ks < KS; ks++) {
+                const bf16x8 kf = *(const bf16x8*)(kimg + (t * KS + ks) * 1024);
+#pragma unroll
+                for (int i = 0; i < TQ; i++) s[i][t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf, qf[i][ks], s[i][t], 0, 0, 0);
+            }
+        const bool whole = kt * 64 >= full_lo && kt * 64 + 63 <= full_hi;
+#pragma unroll
+        for (int i = 0; i < TQ; i++) {
+            const int back = qpos[i] - kt * 64;
+            f.nr1 = r1v[i]; f.r2 = r2v[i];
+            grouped_scores(f, s[i], back, fg);
+            if (!whole) grouped_mask(s[i], back, p.window, fg);
+            const float m_new = vmax2(m_run[i], rows_max(vmax16(s[i][0], s[i][1], s[i][2], s[i][3])));
+            if (__any(m_new != m_run[i])) {
+                const float alpha = __builtin_amdgcn_exp2f(m_run[i] - m_new);
+                lacc[i] *= alpha;
+#pragma unroll
+                for (int d = 0; d < DT; d++) o[i][d] *= alpha;
+                m_run[i] = m_new;
+            }
+#pragma unroll
+            for (int t = 0; t < 4; t++)
+#pragma unroll
+                for (int r = 0; r < 4; r++) s[i][t][r] = __builtin_amdgcn_exp2f(s[i][t][r] - m_new);
+        }
+#pragma unroll
+        for (int u = 0; u < 2; u++) {
+            bf16x8 pf[TQ];
+#pragma unroll
+            for (int i = 0; i < TQ; i++) {
+                pf[i] = latent_pack_p(s[i][2 * u], s[i][2 * u + 1]);
+                lacc[i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(ones, pf[i], lacc[i], 0, 0, 0);      // denominators out of the same rounded weights
+            }
+#pragma unroll
+            for (int d = 0; d < DT; d++) {
+                const bf16x8 vf = *(const bf16x8*)(vimg + (2 * d + u) * 1024);
+#pragma unroll
+                for (int i = 0; i < TQ; i++) o[i][d] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf, pf[i], o[i][d], 0, 0, 0);
+            }
+        }
+    }
+    if (!w_live) return;
+#pragma unroll
+    for (int i = 0; i < TQ; i++) {
+        bool ok;
+        const int row = row_of(i, ok), si = row / p.group, head = kvh * p.group + row - si * p.group;
+        if (!ok) continue;
+        const float inv = 1.0f / lacc[i][0];
+#pragma unroll
+        for (int d = 0; d < DT; d++) grouped_store(p, tok0 + si, head, 16 * d + 4 * fg, o[i][d] * inv);
+    }
+}
+
+// grid (G x 16-row tiles, sequences, key splits).  Wave w of workgroup z takes the key tiles z NW + w, + NW gridDim.z, ...; operands
+// come straight from the cache.  The waves' results are combined through LDS; with gridDim.z > 1 every workgroup leaves a partial
+// record {O^T [DT][64 lanes] f32x4, m[16], l[16]} and the one that draws the last ticket combines them in z order.
+template <int DT> constexpr int grouped_part_floats() { return DT * 256 + 32; }
+template <int KS, int DT, int NW>
+__global__ __launch_bounds__(NW * 64) void grouped_short_kernel(GroupedArgs p) {
+    extern __shared__ __attribute__((aligned(16))) char grp_sm[];       // [NW][DT][64] f32x4
+    __shared__ float red_m[NW][16], red_l[NW][16];
+    __shared__ int ticket;
+    const int kvh = blockIdx.x % p.G, rt = blockIdx.x / p.G, seq = blockIdx.y;
+    const int R = p.seq_len[seq] * p.group;
+    if (R > p.short_rows || rt * 16 >= R) return;
+    const int tok0 = p.seq_tok_start[seq], pos0 = p.seq_pos[seq];
+    const int32_t* tbl = p.blk_table + (int64_t)seq * p.tbl_stride;
+    const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6);
+    const int fq = lane & 15, fg = lane >> 4;
+    const bool ok = rt * 16 + fq < R;
+    const int row = ok ? rt * 16 + fq : R - 1, si = row / p.group, head = kvh * p.group + row - si * p.group;
+    const int first = pos0 + rt * 16 / p.group, last = pos0 + min(rt * 16 + 15, R - 1) / p.group, qpos = pos0 + si;
+    const int lo = p.window > 0 && first - p.window + 1 > 0 ? first - p.window + 1 : 0;
+    const int t0 = lo >> 6, n_kt = (last >> 6) + 1;
+    const int full_lo = p.window > 0 ? last - p.window + 1 : 0, full_hi = first;
+    const int64_t tok = tok0 + si;
+    bf16x8 qf[KS], kf[4][KS], vf[DT][2];
+    const float* q = p.proj + tok * p.proj_ld + head * p.dp;
+#pragma unroll
+    for (int ks = 0; ks < KS; ks++) grouped_load_q(q, ks, fg, qf[ks]);
+    const GroupedScore f(p, head);
+    f32x4 o[DT];
+#pragma unroll
+    for (int d = 0; d < DT; d++) o[d] = f32x4{0.f, 0.f, 0.f, 0.f};
+    float m = -1e30f, l = 0.f;
+    const int64_t v_ld = p.bs >> 5;
+    for (int kt = t0 + blockIdx.z * NW + wave; kt < n_kt; kt += NW * gridDim.z) {
+        const int bi = kt * 64 / p.bs, r0 = kt * 64 - bi * p.bs;
+        const bf16_t* base = (const bf16_t*)p.cache + (int64_t)__builtin_amdgcn_readfirstlane(tbl[bi]) * p.block_stride + lane * 8;
+        const bf16_t* kp = base + ((int64_t)kvh * p.bs + r0) * p.dp;
+        const bf16_t* vp = base + (int64_t)p.G * p.bs * p.dp + (int64_t)kvh * p.bs * p.vp + (r0 >> 5) * 512;
+#pragma unroll
+        for (int t = 0; t < 4; t++)
+#pragma unroll
+            for (int ks = 0; ks < KS; ks++) kf[t][ks] = *(const bf16x8*)(kp + (t * KS + ks) * 512);
+#pragma unroll
+        for (int d = 0; d < DT; d++)
+#pragma unroll
+            for (int u = 0; u < 2; u++) vf[d][u] = *(const bf16x8*)(vp + (d * v_ld + u) * 512);
+        f32x4 s[4];
+#pragma unroll
+        for (int t = 0; t < 4; t++) {
+            s[t] = f32x4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+            for (int ks = 0; ks < KS; ks++) s[t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf[t][ks], qf[ks], s[t], 0, 0, 0);
+        }
+        const int back = qpos - kt * 64;
+        grouped_scores(f, s, back, fg);
+        if (!(kt * 64 >= full_lo && kt * 64 + 63 <= full_hi)) grouped_mask(s, back, p.window, fg);
+        float mx = -INFINITY;
+#pragma unroll
+        for (int t = 0; t < 4; t++)
+#pragma unroll
+            for (int r = 0; r < 4; r++) mx = fmaxf(mx, s[t][r]);
+        const float mn = fmaxf(m, rows_max(mx)), alpha = __builtin_amdgcn_exp2f(m - mn);
+        m = mn;
+        l *= alpha;
+#pragma unroll
+        for (int t = 0; t < 4; t++)
+#pragma unroll
+            for (int r = 0; r < 4; r++) { s[t][r] = __builtin_amdgcn_exp2f(s[t][r] - mn); l += s[t][r]; }
+        const bf16x8 p0 = latent_pack_p(s[0], s[1]), p1 = latent_pack_p(s[2], s[3]);
+#pragma unroll
+        for (int d = 0; d < DT; d++) {
+            o[d] *= alpha;
+            o[d] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf[d][0], p0, o[d], 0, 0, 0);
+            o[d] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf[d][1], p1, o[d], 0, 0, 0);
+        }
+    }
+    l += __shfl_xor(l, 16, 64);
+    l += __shfl_xor(l, 32, 64);
+    if (fg == 0) { red_m[wave][fq] = m; red_l[wave][fq] = l; }
+    f32x4* po = (f32x4*)grp_sm;
+#pragma unroll
+    for (int d = 0; d < DT; d++) po[(wave * DT + d) * 64 + lane] = o[d];
+    __syncthreads();
+    float ms = red_m[0][fq], L = 0.f, sc[NW];
+#pragma unroll
+    for (int w = 1; w < NW; w++) ms = fmaxf(ms, red_m[w][fq]);
+#pragma unroll
+    for (int w = 0; w < NW; w++) { sc[w] = __builtin_amdgcn_exp2f(red_m[w][fq] - ms); L += red_l[w][fq] * sc[w]; }      // (a wave without a tile: l = 0, O = 0)
+    const int nz = gridDim.z, pair = seq * gridDim.x + blockIdx.x;
+    float* rec = p.part + ((int64_t)pair * nz + blockIdx.z) * grouped_part_floats<DT>();
+    for (int d = wave; d < DT; d += NW) {
+        f32x4 a = f32x4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+        for (int w = 0; w < NW; w++) a += po[(w * DT + d) * 64 + lane] * sc[w];
+        if (nz > 1) ((f32x4*)rec)[d * 64 + lane] = a;
+        else if (ok) grouped_store(p, tok, head, 16 * d + 4 * fg, a * (1.0f / L));
+    }
+    if (nz == 1) return;
+    if (wave == 0 && fg == 0) { rec[DT * 256 + fq] = ms; rec[DT * 256 + 16 + fq] = L; }
+    __threadfence();                       // release: the other workgroups may sit on other XCDs
+    __syncthreads();
+    if (tid == 0) ticket = __hip_atomic_fetch_add(p.part_cnt + pair, 1, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
+    __syncthreads();
+    if (ticket != nz - 1) return;
+    __threadfence();                       // acquire
+    const float* rec0 = p.part + (int64_t)pair * nz * grouped_part_floats<DT>();
+    float M = -1e30f, LL = 0.f;
+    for (int z = 0; z < nz; z++) M = fmaxf(M, rec0[(int64_t)z * grouped_part_floats<DT>() + DT * 256 + fq]);
+    for (int z = 0; z < nz; z++) {
+        const float* rz = rec0 + (int64_t)z * grouped_part_floats<DT>() + DT * 256;
+        LL += rz[16 + fq] * __builtin_amdgcn_exp2f(rz[fq] - M);
+    }
+    for (int d = wave; d < DT; d += NW) {
+        f32x4 a = f32x4{0.f, 0.f, 0.f, 0.f};
+        for (int z = 0; z < nz; z++) {
+            const float* rz = rec0 + (int64_t)z * grouped_part_floats<DT>();
+            a += ((const f32x4*)rz)[d * 64 + lane] * __builtin_amdgcn_exp2f(rz[DT * 256 + fq] - M);
+        }
+        if (ok) grouped_store(p, tok, head, 16 * d + 4 * fg, a * (1.0f / LL));
+    }
+    if (tid == 0) __hip_atomic_store(p.part_cnt + pair, 0, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);      // for the next launch
+}
+
+// ---- any size: one 256-thread workgroup per (token, head), online softmax over 256 keys at a time, plain fp32 arithmetic ----
+template <typename T>
+__global__ __launch_bounds__(256) void grouped_plain_kernel(GroupedArgs p) {
+    __shared__ float red[4], sp[256];
+    extern __shared__ __attribute__((aligned(16))) float grp_f[];      // q [dp] | o [vp]
+    const int seq = blockIdx.z, h = blockIdx.y, r = blockIdx.x, tid = threadIdx.x, kvh = h / p.group;
+    if (r >= p.seq_len[seq]) return;
+    constexpr bool FM = sizeof(T) == 2;
+    const int64_t t = p.seq_tok_start[seq] + r;
+    const int pos = p.seq_pos[seq] + r, lo = p.window > 0 && pos - p.window + 1 > 0 ? pos - p.window + 1 : 0;
+    const int32_t* tbl = p.blk_table + (int64_t)seq * p.tbl_stride;
+    float *sq = grp_f, *so = grp_f + p.dp;
+    for (int i = tid; i < p.dp; i += 256) sq[i] = p.proj[t * p.proj_ld + h * p.dp + i];
+    for (int i = tid; i < p.vp; i += 256) so[i] = 0.f;
+    const float r1 = p.r1 ? p.r1[h] : 0.f, r2 = p.r1 ? p.r2[h] : 0.f;
+    float m = -1e30f, l = 0.f;
+    __syncthreads();
+    auto bmax = [&](float v) { v = wave_max(v); if ((tid & 63) == 0) red[tid >> 6] = v; __syncthreads(); v = fmaxf(fmaxf(red[0], red[1]), fmaxf(red[2], red[3])); __syncthreads(); return v; };
+    auto bsum = [&](float v) { v = wave_sum(v); if ((tid & 63) == 0) red[tid >> 6] = v; __syncthreads(); v = red[0] + red[1] + red[2] + red[3]; __syncthreads(); return v; };
+    auto part = [&](int key, int& row) { const int bi = key / p.bs; row = key - bi * p.bs; return (const T*)p.cache + (int64_t)tbl[bi] * p.block_stride; };
+    for (int base = lo; base <= pos; base += 256) {
+        const int key = base + tid;
+        float s = -INFINITY;
+        if (key <= pos) {
+            int row;
+            const T* k = part(key, row) + (int64_t)kvh * p.bs * p.dp;
+            if (FM) row = grouped_k_row(row);
+            float a = 0.f;
+            for (int d = 0; d < p.dim; d++) a = fmaf(sq[d], (float)k[act_index<T>(row, d, p.dp)], a);
+            s = a * p.scale;
+            if (p.softcap > 0.f) s = p.softcap * tanhf(s / p.softcap);
+            if (p.r1) s -= r1 * log1pf(r2 * (float)(pos - key));
+        }
+        const float mn = fmaxf(m, bmax(s)), alpha = expf(m - mn);
+        const float e = key <= pos ? expf(s - mn) : 0.f;
+        m = mn;
+        l = l * alpha + bsum(e);
+        sp[tid] = e;
+        __syncthreads();
+        const int nk = min(256, pos - base + 1);
+        for (int i = tid; i < p.vp; i += 256) {
+            float a = so[i] * alpha;
+            for (int j = 0; j < nk; j++) {
+                int row;
+                const T* v = part(base + j, row) + (int64_t)p.G * p.bs * p.dp + (int64_t)kvh * p.bs * p.vp;
+                a = fmaf(sp[j], (float)(FM ? v[fm_index(i, row, p.bs)] : v[(int64_t)row * p.vp + i]), a);
+            }
+            so[i] = a;
+        }
+        __syncthreads();
+    }
+    for (int i = tid; i < p.vp; i += 256) {
+        float o = so[i] / l;
+        if (p.gate_off >= 0) o *= 1.0f / (1.0f + expf(-p.proj[t * p.proj_ld + p.gate_off + h * p.vp + i]));
+        ActIO<T>::st((T*)p.out + act_index<T>(t, h * p.vp + i, p.out_ld), o);
+    }
+}
+
+}  // namespace nvl

@@ -1,21 +1,29 @@
 // layered.h — models described by a list of layers (nvl_layer_config): every layer names a mixer (latent attention, Mamba-2, gated
-// linear attention, channel-wise delta rule), its sizes and its feed-forward, with a norm before and after each sublayer
-// (NVL_BLOCK_SANDWICH) or after it only (NVL_BLOCK_POST: the sublayers read the residual stream itself).  Host side: creation, tensor
-// staging, freezing into the kernels' layouts, the layer stack of one forward pass.  Included by nvllm.hip.
+// linear attention, channel-wise delta rule, grouped-query attention), its sizes and its feed-forward, with a norm before and after each
+// sublayer (NVL_BLOCK_SANDWICH), after it only (NVL_BLOCK_POST: the sublayers read the residual stream itself), or one norm that both
+// sublayers read (NVL_BLOCK_PARALLEL).  Host side: creation, tensor staging, freezing into the kernels' layouts, the layer stack of one
+// forward pass.  Included by nvllm.hip.
+//
+// A parallel block's two sublayers end in ONE projection: their operands sit side by side in m->lmix (kd = ko + Fp columns) and W_o
+// and W_down side by side in one matrix.  The feed-forward is dense, or a mixture of experts whose shared expert takes the dense one's
+// place; the experts' sum joins in the launch that completes the residual.  A per-layer token input (side_dim) follows:
+// x += rms(P (gelu(G x) * e_token)) * w.
 //
 // What differs from the fixed-shape models around it:
 //   * widths need not be multiples of 64: rows, heads and latents are padded with zeros when the tensors are frozen (m->H is the
 //     padded row, m->Hn the real one), so the GEMM and norm kernels run unchanged;
 //   * the cache of a sequence is a slot (recurrent states, convolution rows) plus blocks of the library's pool (latents); blocks
 //     that no window reaches any more go back to the pool while the sequence runs (pool_trim);
-//   * a batch may mix prompt portions and single tokens: attention takes the absorbed form for sequences with up to
-//     LAT_ABSORB_MAX new tokens and the expanded form for the rest; recurrences go token by token up to REC_STEP_MAX.
+//   * a batch may mix prompt portions and single tokens: latent attention takes the absorbed form for sequences with up to
+//     LAT_ABSORB_MAX new tokens and the expanded form for the rest, grouped attention its short form up to GROUPED_SHORT_ROWS
+//     query rows; recurrences go token by token up to REC_STEP_MAX.
 #pragma once
 
 namespace {
 
 constexpr float CLAMPED_GLU_SLOPE = 1.702f;
 constexpr int LAT_ABSORB_MAX = 16, LAT_ABSORB_MAX_RP = 512, REC_STEP_MAX = 4;
+constexpr int GROUPED_SHORT_ROWS = 64, GROUPED_SPLITS = 16, GROUPED_SPLIT_WGS = 512;      // GROUPED_SPLIT_WGS: workgroups of a launch whose keys are split
 
 bool same_rotation(const nvl_layer_config& a, const nvl_layer_config& b) {
     return a.rot_dim == b.rot_dim && a.rot_base == b.rot_base && a.rot_factor == b.rot_factor && a.rot_original == b.rot_original &&
@@ -36,8 +44,14 @@ int pad_head(int d, int unit) {       // head sizes the attention instances exis
 // ------------------------------------------------------------------------------------------
 int layered_create(const nvl_model_config& c, const nvl_layer_config* layers, const nvl_runtime_opts& opts, nvl_model** out) {
     auto bad = [&](const std::string& why) { return fail(nullptr, NVL_ERR_INVALID, "nvl_create_layers: " + why); };
-    if (c.block_style != NVL_BLOCK_SANDWICH && c.block_style != NVL_BLOCK_POST) return bad("block_style NVL_BLOCK_SANDWICH or NVL_BLOCK_POST expected");
-    if (c.activation_type != NVL_ACT_GEGLU && c.activation_type != NVL_ACT_CLAMPED_GLU) return bad("activation_type NVL_ACT_GEGLU or NVL_ACT_CLAMPED_GLU expected");
+    const bool par = c.block_style == NVL_BLOCK_PARALLEL;
+    if (c.block_style != NVL_BLOCK_SANDWICH && c.block_style != NVL_BLOCK_POST && !par) return bad("block_style NVL_BLOCK_SANDWICH, NVL_BLOCK_POST or NVL_BLOCK_PARALLEL expected");
+    auto act_ok = [&](int a) { return par ? a == NVL_ACT_RELU2 || a == NVL_ACT_SWIGLU : a == NVL_ACT_GEGLU || a == NVL_ACT_CLAMPED_GLU; };
+    if (!act_ok(c.activation_type)) return bad("activation_type does not fit the block style (NVL_ACT_GEGLU, NVL_ACT_CLAMPED_GLU; parallel: NVL_ACT_RELU2, NVL_ACT_SWIGLU)");
+    if (!par && (c.norm_type != NVL_NORM_RMS || c.position_type != NVL_POS_NONE || c.side_dim)) return bad("layer norms, learned positions and side_dim need NVL_BLOCK_PARALLEL");
+    if ((c.norm_type != NVL_NORM_RMS && c.norm_type != NVL_NORM_LAYER) || (c.position_type != NVL_POS_NONE && c.position_type != NVL_POS_LEARNED)) return bad("bad norm_type / position_type");
+    if (c.norm_type == NVL_NORM_LAYER && c.norm_weight_offset != 0.f) return bad("layer norms take their weights as they are");
+    if (c.side_dim < 0 || c.side_dim > 8192) return bad("bad side_dim");
     if (!(c.logit_softcap >= 0.f)) return bad("logit_softcap is negative");
     if (c.hidden <= 0 || c.num_layers <= 0 || c.vocab_size <= 0 || c.max_seq_len <= 0) return bad("non-positive model dimension");
     if (c.hidden > 20480) return bad("hidden larger than 20480");
@@ -50,6 +64,12 @@ int layered_create(const nvl_model_config& c, const nvl_layer_config* layers, co
         const std::string at = "layer " + std::to_string(i) + ": ";
         if (l.heads <= 0 || l.vdim <= 0 || l.vdim > 2048 || l.ffn_dim < 0) return bad(at + "bad heads / vdim / ffn_dim");
         if (l.ffn_dim && c.activation_type == NVL_ACT_CLAMPED_GLU && !(l.ffn_limit > 0.f)) return bad(at + "ffn_limit is not positive");
+        if (l.ffn_act && !act_ok(l.ffn_act)) return bad(at + "ffn_act does not fit the block style");
+        if (l.experts) {
+            if (!par) return bad(at + "experts need NVL_BLOCK_PARALLEL");
+            if (l.experts < 0 || l.experts > std::min(MOE_MAX_E, ROUTE_MAX_E) || l.expert_dim <= 0 || l.expert_groups <= 0 || l.experts % l.expert_groups || l.groups_kept <= 0 ||
+                l.groups_kept > l.expert_groups || l.top_k <= 0 || l.top_k > l.groups_kept * (l.experts / l.expert_groups)) return bad(at + "bad expert sizes");
+        }
         switch (l.mixer) {
             case NVL_MIXER_LATENT_ATTENTION:
                 if (l.rot_dim < 0 || l.rot_dim % 2 || l.rot_dim > 1024 || (l.rot_dim && !(l.rot_base > 1.0)) ||
@@ -72,6 +92,12 @@ int layered_create(const nvl_model_config& c, const nvl_layer_config* layers, co
             case NVL_MIXER_CHANNEL_DELTA:
                 if (l.dim <= 0 || l.dim > 2048 || l.kv_heads <= 0 || l.heads % l.kv_heads || l.conv_taps <= 0 || l.decay_rank < 0) return bad(at + "bad channel delta sizes");
                 break;
+            case NVL_MIXER_ATTENTION: {
+                if (l.dim <= 0 || l.dim > 2048 || l.kv_heads <= 0 || l.heads % l.kv_heads || l.window < 0 || !(l.softcap >= 0.f)) return bad(at + "bad attention sizes");
+                for (int j = 0; j < i && l.v_mix; j++)
+                    if (layers[j].mixer == l.mixer && layers[j].v_mix && (layers[j].kv_heads != l.kv_heads || layers[j].vdim != l.vdim)) return bad(at + "mixes values of another shape");
+                break;
+            }
             default: return bad(at + "unknown mixer");
         }
         if (l.weights_of >= L || l.weights_of == i) return bad(at + "weights_of names no other layer");
@@ -84,7 +110,7 @@ int layered_create(const nvl_model_config& c, const nvl_layer_config* layers, co
         const nvl_layer_config &a = layers[i], &b = layers[o];
         if (a.mixer != b.mixer || a.heads != b.heads || a.dim != b.dim || a.vdim != b.vdim || a.q_rank != b.q_rank || a.kv_rank != b.kv_rank ||
             a.state != b.state || a.groups != b.groups || a.conv_taps != b.conv_taps || a.ffn_dim != b.ffn_dim || a.rot_dim != b.rot_dim ||
-            a.kv_heads != b.kv_heads || a.gate_per_head != b.gate_per_head || (i != o && a.mixer == NVL_MIXER_LATENT_ATTENTION && (a.kv_from >= 0) != (b.kv_from >= 0)))
+            a.kv_heads != b.kv_heads || a.gate_per_head != b.gate_per_head || a.experts != b.experts || a.expert_dim != b.expert_dim || a.v_mix != b.v_mix || a.ffn_act != b.ffn_act || (i != o && a.mixer == NVL_MIXER_LATENT_ATTENTION && (a.kv_from >= 0) != (b.kv_from >= 0)))
             return bad("layer " + std::to_string(i) + " does not have the shape of the layer whose tensors it uses");
     }
     if (opts.device < 0 || nvl_device_count() <= opts.device) return fail(nullptr, NVL_ERR_NO_DEVICE, "nvl_create_layers: no HIP device (this library has no CPU fallback)");
@@ -92,7 +118,7 @@ int layered_create(const nvl_model_config& c, const nvl_layer_config* layers, co
     if (!m) return fail(nullptr, NVL_ERR_OOM, "nvl_create_layers: out of host memory");
     try {
         m->cfg = c; m->opts = opts; m->layered = true;
-        m->cfg.attention_type = NVL_ATTN_GQA; m->cfg.norm_type = NVL_NORM_RMS; m->cfg.position_type = NVL_POS_NONE; m->cfg.use_moe = 0;
+        m->cfg.attention_type = NVL_ATTN_GQA; m->cfg.use_moe = 0;
         m->f32 = opts.precision == NVL_PRECISION_F32;
         m->wsize = m->f32 ? 4 : 2;
         m->device = opts.device;
@@ -111,6 +137,17 @@ int layered_create(const nvl_model_config& c, const nvl_layer_config* layers, co
             LayerRun& r = m->runs[(size_t)i];
             r.c = layers[i]; r.owner = owner[(size_t)i];
             r.Fp = (int)round_up(r.c.ffn_dim, 64);
+            r.act = r.c.ffn_act ? r.c.ffn_act : c.activation_type;
+            if (r.c.experts) {      // padded so that a wave of the decode down projection owns one expert, at most 16 of them a workgroup
+                r.Ep = (int)round_up(r.c.experts, r.c.experts <= 32 ? 2 : 16); r.moe_slices = r.Ep <= 32 ? 2 : r.Ep / 16;
+                r.Ip = (int)round_up(r.c.expert_dim, 64);
+            }
+            if (r.c.mixer == NVL_MIXER_LATENT_ATTENTION || r.c.mixer == NVL_MIXER_ATTENTION) {
+                size_t w = 0;
+                while (w < m->windows.size() && m->windows[w] != r.c.window) w++;
+                if (w == m->windows.size()) m->windows.push_back(r.c.window);
+                r.win = (int)w;
+            }
             const int H = r.c.heads;
             if (r.c.mixer == NVL_MIXER_LATENT_ATTENTION) {
                 r.vp = pad_head(r.c.vdim, 64);
@@ -122,12 +159,18 @@ int layered_create(const nvl_model_config& c, const nvl_layer_config* layers, co
                 if (r.rp > 256 && r.rp < 512) r.rp = r.rp <= 384 ? 384 : 512;       // (instances of the absorbed form)
                 r.gate_off = r.qrp + (r.src == i ? r.rp + r.rotp : 0);
                 r.n_in = r.gate_off + (r.c.gate_per_head ? H : H * r.vp); r.ko = (int)round_up((int64_t)H * r.vp, 64);
-                size_t w = 0;
-                while (w < m->windows.size() && m->windows[w] != r.c.window) w++;
-                if (w == m->windows.size()) m->windows.push_back(r.c.window);
-                r.win = (int)w;
                 if (r.src == i) { r.cache_off = cache; cache += (int64_t)bs * (r.rp + r.rotp); }
                 else r.cache_off = m->runs[(size_t)r.src].cache_off;
+            } else if (r.c.mixer == NVL_MIXER_ATTENTION) {
+                const int G = r.c.kv_heads;
+                r.dp = pad_head(r.c.dim, 64); r.vp = pad_head(r.c.vdim, 64);
+                r.k_off = H * r.dp; r.v_off = r.k_off + G * r.dp; r.gate_off = r.v_off + G * r.vp; r.route_off = r.gate_off + H * r.vp;
+                r.n_in = r.route_off + r.c.experts; r.ko = (int)round_up((int64_t)H * r.vp, 64);
+                r.cache_off = cache; cache += (int64_t)bs * G * (r.dp + r.vp);
+                if (r.c.v_mix) {
+                    r.mix = m->lvf_ld ? 2 : 1;
+                    m->lvf_ld = (int64_t)G * r.vp;
+                }
             } else {
                 const int DVp = (int)round_up(r.c.vdim, 4), DK = r.c.mixer == NVL_MIXER_MAMBA2 ? r.c.state : r.c.dim;
                 r.ko = (int)round_up((int64_t)H * r.c.vdim, 64);
@@ -141,6 +184,7 @@ int layered_create(const nvl_model_config& c, const nvl_layer_config* layers, co
                     r.ring_off = state; state += round_up((int64_t)r.c.conv_taps * r.conv_dim, 64);
                 }       // (GLA, channel delta: n_in follows from the decay rank, layered_finalize)
             }
+            r.kd = r.ko + (par ? r.Fp : 0);
         }
         m->lat_block_stride = cache; m->rec_slot_stride = state;
         m->pool = 1; m->Tmax = bs; m->blocks_per_seq = cdiv(c.max_seq_len, bs);
@@ -176,22 +220,36 @@ void layered_shape(const nvl_model* m, int kind, int layer, int64_t& N, int64_t&
     switch (kind) {
         case NVL_T_TOK_EMB: case NVL_T_LM_HEAD: N = m->V; K = W; return;
         case NVL_T_FINAL_NORM_W: N = W; return;
+        case NVL_T_FINAL_NORM_B: if (m->cfg.norm_type == NVL_NORM_LAYER) N = W; return;
+        case NVL_T_POS_EMB: if (m->cfg.position_type == NVL_POS_LEARNED) { N = -1; K = W; } return;
+        case NVL_T_SIDE_EMB: if (m->cfg.side_dim) { N = m->V; K = (int64_t)m->L * m->cfg.side_dim; } return;
         default: if (is_global(kind)) return;
     }
     const LayerRun& r = m->runs[(size_t)layer];
     const nvl_layer_config& c = r.c;
     if (r.owner != layer) return;
-    const bool post = m->cfg.block_style == NVL_BLOCK_POST, delta = c.mixer == NVL_MIXER_CHANNEL_DELTA;
-    const bool lat = c.mixer == NVL_MIXER_LATENT_ATTENTION, mam = c.mixer == NVL_MIXER_MAMBA2, gla = c.mixer == NVL_MIXER_GLA;
+    const bool post = m->cfg.block_style == NVL_BLOCK_POST, par = m->cfg.block_style == NVL_BLOCK_PARALLEL, delta = c.mixer == NVL_MIXER_CHANNEL_DELTA;
+    const bool att = c.mixer == NVL_MIXER_ATTENTION, lat = c.mixer == NVL_MIXER_LATENT_ATTENTION, mam = c.mixer == NVL_MIXER_MAMBA2, gla = c.mixer == NVL_MIXER_GLA;
     const int64_t hv = (int64_t)c.heads * c.vdim, hd = (int64_t)c.heads * c.dim;
     switch (kind) {
-        case NVL_T_ATTN_NORM_W: case NVL_T_FFN_NORM_W: if (!post) N = W; return;
-        case NVL_T_MIX_POST_NORM: case NVL_T_FFN_POST_NORM: N = W; return;
+        case NVL_T_ATTN_NORM_W: if (!post) N = W; return;
+        case NVL_T_FFN_NORM_W: if (!post && !par) N = W; return;
+        case NVL_T_ATTN_NORM_B: if (m->cfg.norm_type == NVL_NORM_LAYER) N = W; return;
+        case NVL_T_MIX_POST_NORM: case NVL_T_FFN_POST_NORM: if (!par) N = W; return;
+        case NVL_T_SIDE_GATE: if (m->cfg.side_dim) { N = m->cfg.side_dim; K = W; } return;
+        case NVL_T_SIDE_PROJ: if (m->cfg.side_dim) { N = W; K = m->cfg.side_dim; } return;
+        case NVL_T_SIDE_NORM: if (m->cfg.side_dim) N = W; return;
+        case NVL_T_ROUTER: if (c.experts) { N = c.experts; K = W; } return;
+        case NVL_T_ROUTER_BIAS: if (c.experts) N = c.experts; return;
+        case NVL_T_MOE_IN: if (c.experts) { N = (int64_t)c.experts * 2 * c.expert_dim; K = W; } return;
+        case NVL_T_MOE_OUT: if (c.experts) { N = c.experts * W; K = c.expert_dim; } return;
+        case NVL_T_BIAS_R1: case NVL_T_BIAS_R2: if (att) N = c.heads; return;
+        case NVL_T_V_MIX: if (att && c.v_mix) N = 1; return;
         case NVL_T_MIX_SCALE: case NVL_T_FFN_SCALE: if (post) N = W; return;
-        case NVL_T_W1: N = 2 * (int64_t)c.ffn_dim; K = W; return;
+        case NVL_T_W1: N = (r.act == NVL_ACT_RELU2 ? 1 : 2) * (int64_t)c.ffn_dim; K = W; return;
         case NVL_T_W2: if (c.ffn_dim) { N = W; K = c.ffn_dim; } return;
         case NVL_T_WO: if (!mam) { N = W; K = hv; } return;
-        case NVL_T_MIX_GATE: if (lat || gla) { N = c.gate_per_head && lat ? c.heads : hv; K = W; } return;
+        case NVL_T_MIX_GATE: if (lat || gla || att) { N = c.gate_per_head && lat ? c.heads : hv; K = W; } return;
         case NVL_T_LAT_DQ: if (lat) { N = c.q_rank; K = W; } return;
         case NVL_T_LAT_DQ_NORM: if (lat) N = c.q_rank; return;
         case NVL_T_LAT_UQ: if (lat) { N = hd + (int64_t)c.heads * c.rot_dim; K = c.q_rank; } return;
@@ -199,8 +257,9 @@ void layered_shape(const nvl_model* m, int kind, int layer, int64_t& N, int64_t&
         case NVL_T_LAT_DKV_NORM: if (lat && r.src == layer) N = c.kv_rank; return;
         case NVL_T_LAT_UK: if (lat) { N = hd; K = c.kv_rank; } return;
         case NVL_T_LAT_UV: if (lat) { N = hv; K = c.kv_rank; } return;
-        case NVL_T_WQ: case NVL_T_WK: if (gla || delta) { N = delta ? (int64_t)c.kv_heads * c.dim : hd; K = W; } return;
-        case NVL_T_WV: if (gla || delta) { N = hv; K = W; } return;
+        case NVL_T_WQ: if (att) { N = hd; K = W; return; } [[fallthrough]];
+        case NVL_T_WK: if (att) { N = (int64_t)c.kv_heads * c.dim; K = W; } else if (gla || delta) { N = delta ? (int64_t)c.kv_heads * c.dim : hd; K = W; } return;
+        case NVL_T_WV: if (att) { N = (int64_t)c.kv_heads * c.vdim; K = W; } else if (gla || delta) { N = hv; K = W; } return;
         case NVL_T_DELTA_CONV: if (delta) N = (int64_t)r.conv_dim * c.conv_taps; return;
         case NVL_T_DELTA_BETA: if (delta) { N = c.heads; K = W; } return;
         case NVL_T_DELTA_G1: if (delta) { N = -1; K = W; } return;
@@ -222,6 +281,7 @@ void layered_shape(const nvl_model* m, int kind, int layer, int64_t& N, int64_t&
 bool layered_1d(int kind) {
     if (is_1d(kind)) return true;
     return kind == NVL_T_MIX_POST_NORM || kind == NVL_T_FFN_POST_NORM || kind == NVL_T_LAT_DQ_NORM || kind == NVL_T_LAT_DKV_NORM ||
+           kind == NVL_T_BIAS_R1 || kind == NVL_T_BIAS_R2 || kind == NVL_T_V_MIX || kind == NVL_T_ROUTER_BIAS || kind == NVL_T_SIDE_NORM ||
            kind == NVL_T_GLA_NORM || kind == NVL_T_GLA_A2_B || kind == NVL_T_MIX_SCALE || kind == NVL_T_FFN_SCALE || kind == NVL_T_DELTA_CONV;
 }
 int layered_upload(nvl_model* m, int kind, int layer, const void* data, int dtype, int64_t rows, int64_t cols, int layout) {
@@ -234,7 +294,7 @@ int layered_upload(nvl_model* m, int kind, int layer, const void* data, int dtyp
     }
     const bool vec = layered_1d(kind);
     if (vec) { rows *= cols > 0 ? cols : 1; cols = 1; }
-    else if (layout != NVL_LAYOUT_OUT_IN && kind != NVL_T_TOK_EMB) return fail(m, NVL_ERR_INVALID, "nvl_upload_tensor: matrices of this model are given [out, in]");
+    else if (layout != NVL_LAYOUT_OUT_IN && kind != NVL_T_TOK_EMB && kind != NVL_T_POS_EMB) return fail(m, NVL_ERR_INVALID, "nvl_upload_tensor: matrices of this model are given [out, in]");
     if (rows <= 0 || cols <= 0 || (N > 0 && rows != N) || (K > 0 && cols != K)) {
         snprintf(buf, sizeof buf, "tensor kind %d of layer %d: got [%lld,%lld], the model needs [%lld,%lld]", kind, layer, (long long)rows, (long long)cols, (long long)N, (long long)K);
         return fail(m, NVL_ERR_INVALID, buf);
@@ -313,10 +373,10 @@ f32x2* lay_rotation(nvl_model* m, const nvl_layer_config& c) {
 }
 // rows [n0, n0 + N) of a staged matrix into dst: grouped row / column padding as place_2d_kernel
 void lay_place(nvl_model* m, const DevTensor& t, void* dst, int64_t Kd, int64_t row0 = 0, int rg = 0, int rgp = 0, int cg = 0, int cgp = 0,
-               int64_t n0 = 0, int64_t N = -1, bool trans = false, bool row_major = false) {
+               int64_t n0 = 0, int64_t N = -1, bool trans = false, bool row_major = false, int64_t col0 = 0) {
     if (N < 0) N = t.rows;
-    Place2D pl{N, t.cols, Kd, row0, rg ? rg : 1, rg ? rgp : 1, cg ? cg : 1, cg ? cgp : 1};
-    const dim3 grid((unsigned)std::min<int64_t>(cdiv(t.cols, 256), 64), (unsigned)N);
+    Place2D pl{N, t.cols, Kd, row0, rg ? rg : 1, rg ? rgp : 1, cg ? cg : 1, cg ? cgp : 1, col0};
+    const dim3 grid((unsigned)std::min<int64_t>(cdiv(t.cols, 256), 64), (unsigned)std::min<int64_t>(N, 32768), (unsigned)cdiv(N, 32768));
     const int64_t src0 = n0 * t.cols;
     if (m->f32) {
         if (trans) hipLaunchKernelGGL((place_2d_kernel<float, false, true>), grid, dim3(256), 0, m->stream, t.p, t.raw_dtype, src0, (float*)dst, pl);
@@ -340,7 +400,9 @@ void layered_finalize(nvl_model* m) {
     const int64_t H = m->H;
     need(m->g[NVL_T_TOK_EMB], "token embedding"); need(m->g[NVL_T_FINAL_NORM_W], "final norm");
     const bool post = m->cfg.block_style == NVL_BLOCK_POST;
+    const bool par = m->cfg.block_style == NVL_BLOCK_PARALLEL, ln = m->cfg.norm_type == NVL_NORM_LAYER, learned = m->cfg.position_type == NVL_POS_LEARNED;
     m->final_norm = lay_norm(m, m->g[NVL_T_FINAL_NORM_W], H);
+    if (ln) m->final_norm_b = lay_vector(m, need(m->g[NVL_T_FINAL_NORM_B], "final norm bias"), H);
     auto big = [&](int kind, const char* what) {      // [V][H]: the embedding table / LM head
         void* p = lay_matrix(m, m->V, H);
         lay_place(m, need(m->g[kind], what), p, H);
@@ -348,11 +410,27 @@ void layered_finalize(nvl_model* m) {
     };
     void* emb = big(NVL_T_TOK_EMB, "token embedding");
     m->lm_head = m->g[NVL_T_LM_HEAD].present() && !m->cfg.tied_embedding ? big(NVL_T_LM_HEAD, "LM head") : emb;
+    void* pos = nullptr;
+    if (learned) {
+        const DevTensor& t = need(m->g[NVL_T_POS_EMB], "position embedding");
+        if (t.rows < m->cfg.max_seq_len) throw std::runtime_error("nvl_finalize: max_seq_len exceeds the learned positions");
+        pos = lay_matrix(m, t.rows, H);
+        lay_place(m, t, pos, H);
+    }
+    const int sd = m->cfg.side_dim, sd4 = (int)round_up(sd, 4);
+    if (sd) {       // [V][layer][sd4], row-major
+        const DevTensor& t = need(m->g[NVL_T_SIDE_EMB], "per-layer token embedding");
+        m->side_ld = (int64_t)m->L * sd4; m->side_kp = (int)round_up(sd, 64);
+        m->side_emb = lay_alloc(m, (int64_t)m->V * m->side_ld * (int64_t)m->wsize);
+        lay_place(m, t, m->side_emb, m->side_ld, 0, 0, 0, sd, sd4, 0, -1, false, true);
+    }
     NVL_HIP(hipStreamSynchronize(m->stream));
-    for (int k = 0; k < NVL_T_ATTN_NORM_W; k++) { dfree(m->g[k].p); m->g[k].p = nullptr; }
+    for (int k = 0; k < NVL_T_COUNT; k++) if (is_global(k)) { dfree(m->g[k].p); m->g[k].p = nullptr; }
     m->g[NVL_T_TOK_EMB].p = emb; m->g[NVL_T_TOK_EMB].raw_dtype = -1;      // (the embedding kernels' view of it)
+    m->g[NVL_T_POS_EMB].p = pos;
 
     int64_t ld_in = 0, q_cols = 0, cq_cols = 0, ko = 0, conv = 0, ocols = 0, Fmax = 0, abs_cols = 0, z_cols = 0, g_cols = 0, pa_cols = 0, pg_cols = 0;
+    int64_t moe_k = 0, moe_e = 0, moe_kI = 0, moe_ep = 0, moe_all = 0, moe_sl = 0, grp_vp = 0;
     for (int i = 0; i < m->L; i++) {
         LayerRun& r = m->runs[(size_t)i];
         const nvl_layer_config& c = r.c;
@@ -362,16 +440,40 @@ void layered_finalize(nvl_model* m) {
         if (r.owner == i) {
             auto T = [&](int kind, const char* what) -> const DevTensor& { return need(l.t[kind], at + what); };
             if (!post) w.norm1 = lay_norm(m, T(NVL_T_ATTN_NORM_W, "norm before the mixer"), H);
-            w.norm1b = lay_norm(m, T(NVL_T_MIX_POST_NORM, "norm after the mixer"), H, &l.t[NVL_T_MIX_SCALE]);
+            if (ln) w.norm1_bias = lay_vector(m, T(NVL_T_ATTN_NORM_B, "bias of the norm before the mixer"), H);
+            if (!par) w.norm1b = lay_norm(m, T(NVL_T_MIX_POST_NORM, "norm after the mixer"), H, &l.t[NVL_T_MIX_SCALE]);
             if (c.ffn_dim) {
-                if (!post) w.norm2 = lay_norm(m, T(NVL_T_FFN_NORM_W, "norm before the feed-forward"), H);
-                w.norm2b = lay_norm(m, T(NVL_T_FFN_POST_NORM, "norm after the feed-forward"), H, &l.t[NVL_T_FFN_SCALE]);
+                if (!post && !par) w.norm2 = lay_norm(m, T(NVL_T_FFN_NORM_W, "norm before the feed-forward"), H);
+                if (!par) w.norm2b = lay_norm(m, T(NVL_T_FFN_POST_NORM, "norm after the feed-forward"), H, &l.t[NVL_T_FFN_SCALE]);
                 const DevTensor& w1 = T(NVL_T_W1, "feed-forward gate / up");
-                w.w1 = lay_matrix(m, 2 * r.Fp, H);
-                if (m->f32) { lay_place(m, w1, w.w1, H, 0, 0, 0, 0, 0, 0, c.ffn_dim); lay_place(m, w1, w.w1, H, r.Fp, 0, 0, 0, 0, c.ffn_dim, c.ffn_dim); }
+                w.w1 = lay_matrix(m, (r.act == NVL_ACT_RELU2 ? 1 : 2) * r.Fp, H);
+                if (r.act == NVL_ACT_RELU2) lay_place(m, w1, w.w1, H);
+                else if (m->f32) { lay_place(m, w1, w.w1, H, 0, 0, 0, 0, 0, 0, c.ffn_dim); lay_place(m, w1, w.w1, H, r.Fp, 0, 0, 0, 0, c.ffn_dim, c.ffn_dim); }
                 else { lay_place(m, w1, w.w1, H, 0, 16, 32, 0, 0, 0, c.ffn_dim); lay_place(m, w1, w.w1, H, 16, 16, 32, 0, 0, c.ffn_dim, c.ffn_dim); }
-                w.w2 = lay_matrix(m, H, r.Fp);
-                lay_place(m, T(NVL_T_W2, "feed-forward down"), w.w2, r.Fp);
+                if (!par) {
+                    w.w2 = lay_matrix(m, H, r.Fp);
+                    lay_place(m, T(NVL_T_W2, "feed-forward down"), w.w2, r.Fp);
+                }
+            }
+            if (c.experts) {
+                const int64_t E = c.experts, I = c.expert_dim, Ip = r.Ip;
+                const DevTensor &up = T(NVL_T_MOE_IN, "experts' gate / up"), &down = T(NVL_T_MOE_OUT, "experts' down");
+                w.moe_up = lay_matrix(m, E * 2 * Ip, H);
+                w.moe_down = lay_matrix(m, E * H, Ip);
+                if (!m->f32) w.moe_cat = lay_matrix(m, H, r.Ep * Ip);
+                for (int64_t e = 0; e < E; e++) {
+                    const int64_t row = e * 2 * Ip, from = e * 2 * I;
+                    if (m->f32) { lay_place(m, up, w.moe_up, H, row, 0, 0, 0, 0, from, I); lay_place(m, up, w.moe_up, H, row + Ip, 0, 0, 0, 0, from + I, I); }
+                    else { lay_place(m, up, w.moe_up, H, row, 16, 32, 0, 0, from, I); lay_place(m, up, w.moe_up, H, row + 16, 16, 32, 0, 0, from + I, I); }
+                    lay_place(m, down, w.moe_down, Ip, e * H, 0, 0, 0, 0, e * m->Hn, m->Hn);
+                    if (!m->f32) lay_place(m, down, w.moe_cat, r.Ep * Ip, 0, 0, 0, 0, 0, e * m->Hn, m->Hn, false, false, e * Ip);
+                }
+                if (l.t[NVL_T_ROUTER_BIAS].present()) w.route_bias = lay_vector(m, l.t[NVL_T_ROUTER_BIAS], E);
+            }
+            if (sd) {
+                w.side_gate = lay_matrix(m, sd, H); lay_place(m, T(NVL_T_SIDE_GATE, "token input gate"), w.side_gate, H);
+                w.side_proj = lay_matrix(m, H, m->side_kp); lay_place(m, T(NVL_T_SIDE_PROJ, "token input projection"), w.side_proj, m->side_kp);
+                w.side_norm = lay_vector(m, T(NVL_T_SIDE_NORM, "token input norm"), H);
             }
             if (c.mixer == NVL_MIXER_LATENT_ATTENTION) {
                 w.in = lay_matrix(m, r.n_in, H);
@@ -404,8 +506,21 @@ void layered_finalize(nvl_model* m) {
                 }
                 w.uv = lay_matrix(m, (int64_t)c.heads * r.vp, r.rp);
                 lay_place(m, T(NVL_T_LAT_UV, "value up projection"), w.uv, r.rp, 0, c.vdim, r.vp);
-                w.o = lay_matrix(m, H, r.ko);
-                lay_place(m, T(NVL_T_WO, "output projection"), w.o, r.ko, 0, 0, 0, c.vdim, r.vp);
+                w.o = lay_matrix(m, H, r.kd);
+                lay_place(m, T(NVL_T_WO, "output projection"), w.o, r.kd, 0, 0, 0, c.vdim, r.vp);
+            } else if (c.mixer == NVL_MIXER_ATTENTION) {
+                w.in = lay_matrix(m, r.n_in, H);
+                lay_place(m, T(NVL_T_WQ, "query projection"), w.in, H, 0, c.dim, r.dp);
+                lay_place(m, T(NVL_T_WK, "key projection"), w.in, H, r.k_off, c.dim, r.dp);
+                lay_place(m, T(NVL_T_WV, "value projection"), w.in, H, r.v_off, c.vdim, r.vp);
+                lay_place(m, T(NVL_T_MIX_GATE, "output gate"), w.in, H, r.gate_off, c.vdim, r.vp);
+                if (l.t[NVL_T_BIAS_R1].present()) {
+                    w.r1 = lay_vector(m, l.t[NVL_T_BIAS_R1], c.heads);
+                    w.r2 = lay_vector(m, T(NVL_T_BIAS_R2, "distance bias (r2)"), c.heads);
+                }
+                if (c.v_mix) w.v_lambda = lay_vector(m, T(NVL_T_V_MIX, "value mixing"), 1);
+                w.o = lay_matrix(m, H, r.kd);
+                lay_place(m, T(NVL_T_WO, "output projection"), w.o, r.kd, 0, 0, 0, c.vdim, r.vp);
             } else if (c.mixer == NVL_MIXER_MAMBA2) {
                 w.in = lay_matrix(m, r.n_in, H);
                 lay_place(m, T(NVL_T_MAMBA_IN_PROJ, "input projection"), w.in, H);
@@ -415,8 +530,8 @@ void layered_finalize(nvl_model* m) {
                 w.dskip = lay_vector(m, T(NVL_T_MAMBA_D, "D"), c.heads);
                 w.dt_bias = lay_vector(m, T(NVL_T_MAMBA_DT_BIAS, "dt_bias"), c.heads);
                 w.mix_norm = lay_vector(m, T(NVL_T_MAMBA_NORM, "inner norm"), (int64_t)c.heads * c.vdim);
-                w.o = lay_matrix(m, H, r.ko);
-                lay_place(m, T(NVL_T_MAMBA_OUT_PROJ, "output projection"), w.o, r.ko);
+                w.o = lay_matrix(m, H, r.kd);
+                lay_place(m, T(NVL_T_MAMBA_OUT_PROJ, "output projection"), w.o, r.kd);
             } else if (c.mixer == NVL_MIXER_CHANNEL_DELTA) {
                 const DevTensor &a1 = T(NVL_T_GLA_A1, "decay projection (a1)"), &a2 = T(NVL_T_GLA_A2, "decay projection (a2)");
                 const DevTensor &g1 = T(NVL_T_DELTA_G1, "output gate (g1)"), &g2 = T(NVL_T_DELTA_G2, "output gate (g2)");
@@ -446,8 +561,8 @@ void layered_finalize(nvl_model* m) {
                     w.a2r = lay_matrix(m, hd, w.a_rkp); lay_place(m, a2, w.a2r, w.a_rkp, 0, 0, 0, 0, 0, 0, -1, false, true);
                     w.g2r = lay_matrix(m, hv, w.g_rkp); lay_place(m, g2, w.g2r, w.g_rkp, 0, 0, 0, 0, 0, 0, -1, false, true);
                 }
-                w.o = lay_matrix(m, H, r.ko);
-                lay_place(m, T(NVL_T_WO, "output projection"), w.o, r.ko);
+                w.o = lay_matrix(m, H, r.kd);
+                lay_place(m, T(NVL_T_WO, "output projection"), w.o, r.kd);
             } else {
                 const DevTensor& a1 = T(NVL_T_GLA_A1, "decay projection (a1)");
                 const DevTensor& a2 = T(NVL_T_GLA_A2, "decay projection (a2)");
@@ -463,9 +578,11 @@ void layered_finalize(nvl_model* m) {
                 w.a2 = lay_vector(m, a2, a2.rows * a2.cols);
                 w.a2_b = lay_vector(m, T(NVL_T_GLA_A2_B, "decay bias"), hd);
                 w.mix_norm = lay_vector(m, T(NVL_T_GLA_NORM, "head norm"), c.vdim);
-                w.o = lay_matrix(m, H, r.ko);
-                lay_place(m, T(NVL_T_WO, "output projection"), w.o, r.ko);
+                w.o = lay_matrix(m, H, r.kd);
+                lay_place(m, T(NVL_T_WO, "output projection"), w.o, r.kd);
             }
+            if (c.experts) lay_place(m, T(NVL_T_ROUTER, "router"), w.in, H, r.route_off);
+            if (par && c.ffn_dim) lay_place(m, T(NVL_T_W2, "feed-forward down"), w.o, r.kd, 0, 0, 0, 0, 0, 0, -1, false, false, r.ko);
             NVL_HIP(hipStreamSynchronize(m->stream));
             for (auto& t : l.t) { dfree(t.p); t.p = nullptr; }
         }
@@ -487,12 +604,19 @@ void layered_finalize(nvl_model* m) {
         }
         if (c.mixer == NVL_MIXER_GLA) r.n_in = 2 * c.heads * (c.dim + c.vdim) + m->mixers[(size_t)r.owner].rank;
         ld_in = std::max(ld_in, round_up(r.n_in, 4));
-        ko = std::max<int64_t>(ko, r.ko);
+        ko = std::max<int64_t>(ko, r.kd);
         Fmax = std::max<int64_t>(Fmax, r.Fp);
+        if (c.experts) {
+            const int64_t k = c.top_k;
+            moe_k = std::max(moe_k, k); moe_e = std::max<int64_t>(moe_e, c.experts); moe_kI = std::max(moe_kI, k * r.Ip);
+            moe_ep = std::max<int64_t>(moe_ep, r.Ep); moe_all = std::max(moe_all, (int64_t)r.Ep * r.Ip); moe_sl = std::max<int64_t>(moe_sl, r.moe_slices);
+        }
         if (c.mixer == NVL_MIXER_LATENT_ATTENTION) {
             q_cols = std::max<int64_t>(q_cols, (int64_t)c.heads * r.dp);
             cq_cols = std::max<int64_t>(cq_cols, r.qrp);
             if (lat_absorb_ok(m, r)) abs_cols = std::max(abs_cols, round_up(c.heads, 16) * (r.rp + r.rotp));
+        } else if (c.mixer == NVL_MIXER_ATTENTION) {
+            grp_vp = std::max<int64_t>(grp_vp, r.vp);
         } else {
             ocols = std::max<int64_t>(ocols, (int64_t)c.heads * c.vdim);
             conv = std::max<int64_t>(conv, r.conv_dim);
@@ -504,12 +628,34 @@ void layered_finalize(nvl_model* m) {
     m->lproj_ld = ld_in; m->lq_ld = q_cols; m->lo_ld = round_up(ocols, 4); m->lconv_ld = round_up(conv, 4);
     m->x = dmalloc<float>(Mmax * H);
     m->xn = dmalloc_bytes(Mp * H * ws);
-    m->hbuf = dmalloc_bytes(Mp * m->F * ws);
+    const int64_t hbuf = std::max(Mp * m->F, round_up(Mmax * std::max<int64_t>(moe_k, 1), 64) * (moe_k ? moe_kI / moe_k : 0) + 64 * moe_kI);
+    m->hbuf = dmalloc_bytes(hbuf * ws);
     m->xn_last = dmalloc_bytes(round_up(S, 64) * H * ws);
     NVL_HIP(hipMemsetAsync(m->xn, 0, (size_t)(Mp * H * ws), m->stream));
-    NVL_HIP(hipMemsetAsync(m->hbuf, 0, (size_t)(Mp * m->F * ws), m->stream));
+    NVL_HIP(hipMemsetAsync(m->hbuf, 0, (size_t)(hbuf * ws), m->stream));
     NVL_HIP(hipMemsetAsync(m->xn_last, 0, (size_t)(round_up(S, 64) * H * ws), m->stream));
-    if (m->f32) m->h2 = dmalloc<float>(Mmax * 2 * m->F);
+    if (m->f32) m->h2 = dmalloc<float>(Mmax * std::max<int64_t>(2 * std::max<int64_t>(m->F, moe_kI), sd4));
+    if (moe_k) {
+        m->expert_ids = dmalloc<int32_t>(Mmax * moe_k); m->expert_w = dmalloc<float>(Mmax * moe_k);
+        m->seg_start = dmalloc<int32_t>(moe_e + 1); m->moe_counts = dmalloc<int32_t>(moe_e); m->moe_cursor = dmalloc<int32_t>(moe_e);
+        m->moe_tile_map = dmalloc<int32_t>(4 * (cdiv(Mmax * moe_k, 128) + moe_e)); m->moe_n_mtiles = dmalloc<int32_t>(4);
+        m->perm_token = dmalloc<int32_t>(Mmax * moe_k); m->slot_of = dmalloc<int32_t>(Mmax * moe_k);
+        m->moe_eo = dmalloc<float>(Mmax * moe_k * H);
+        if (!m->f32) {
+            m->moe_xg = dmalloc_bytes(round_up(Mmax * moe_k, 64) * H * 2);
+            m->moe_gate = dmalloc<float>(64 * moe_ep);
+            m->moe_hall = dmalloc_bytes(64 * moe_all * 2);
+            NVL_HIP(hipMemsetAsync(m->moe_hall, 0, (size_t)(64 * moe_all * 2), m->stream));
+            m->moe_part = dmalloc<float>(moe_sl * 64 * H);
+        }
+    }
+    if (sd) m->lside = lay_alloc(m, Mp * m->side_kp * ws);
+    if (m->lvf_ld) m->lvf = (float*)lay_alloc(m, Mmax * m->lvf_ld * 4);
+    if (grp_vp && !m->f32 && grp_vp <= 256) {
+        m->grp_cap = GROUPED_SPLIT_WGS;
+        m->grp_part = (float*)lay_alloc(m, m->grp_cap * (grp_vp * 16 + 32) * 4);
+        m->grp_cnt = (int32_t*)lay_alloc(m, m->grp_cap * 4);
+    }
     m->lproj = f32buf(Mmax * ld_in);
     m->ly = f32buf(Mmax * H);
     if (q_cols) { m->lq = f32buf(Mmax * q_cols); m->lcq = lay_alloc(m, Mp * cq_cols * ws); }
@@ -546,7 +692,7 @@ void layered_free(nvl_model* m) {
     if (!m->layered) return;
     for (void* p : m->layered_allocs) dfree(p);
     dfree(m->key_c); dfree(m->key_r); dfree(m->key_k); dfree(m->key_v); dfree(m->rec_z); dfree(m->rec_decay); dfree(m->delta_ws);
-    if (m->finalized) m->g[NVL_T_TOK_EMB].p = nullptr;
+    if (m->finalized) m->g[NVL_T_TOK_EMB].p = m->g[NVL_T_POS_EMB].p = nullptr;
     m->lm_head = nullptr;
 }
 
@@ -562,8 +708,15 @@ void layered_meta(nvl_model* m, const Meta& hm, int n_seqs, int steps) {
     m->min_len = hm.seq_len[0];
     for (size_t w = 0; w < m->windows.size(); w++) { m->key_rows[w] = 0; m->key_max[w] = 0; }
     const int64_t S = m->opts.max_seqs;
+    m->win_pairs.assign(m->windows.size(), {0.0, 0.0}); m->win_keys.assign(m->windows.size(), {0.0, 0.0});
     for (int i = 0; i < n_seqs; i++) {
         const int n = hm.seq_len[i], pos = hm.seq_pos[i];
+        for (size_t w = 0; w < m->windows.size(); w++) {       // visible (query, key) pairs, keys read: [several new tokens]
+            const double W = m->windows[w] > 0 ? m->windows[w] : 1e18, full = std::min<double>(n, std::max(0.0, pos + n - W));      // tokens whose window is full
+            const double part = n - full;                       // the others are the first ones: they see pos + 1 .. pos + part keys
+            m->win_pairs[w][n > 1] += full * std::min(W, 1e17) * (full > 0) + part * pos + part * (part + 1) / 2;
+            m->win_keys[w][n > 1] += std::min<double>(pos + n, W + n - 1);
+        }
         m->min_len = std::min(m->min_len, n);
         const bool abs = absorb && n <= LAT_ABSORB_MAX;
         if (abs) for (int j = 0; j < n; j++) { hm.abs_tok[m->n_abs] = hm.seq_tok_start[i] + j; hm.abs_seq[m->n_abs] = i; m->n_abs++; }
@@ -595,26 +748,38 @@ int layered_kt_log2(const nvl_model* m) {
 }
 int layered_decode_key(const nvl_model* m) { return layered_kt_log2(m); }
 
-// x += rms(y) * w_post and / or xn = rms(x) * w_next (elem.h SandwichArgs)
-void sandwich(nvl_model* m, const float* y, int slices, int64_t slice_stride, const float* w_post, const float* w_next, const int32_t* rows_idx,
-              void* xn, int rows, bool raw_next = false) {
-    KScope ks(m, KC_OTHER, 0, KS_SANDWICH, (double)rows * m->Hn * ((y ? 8.0 + 4.0 * std::max(slices, 1) : 4.0) + (w_next || raw_next ? (double)m->wsize : 0.0)));
+// a sublayer's last projection: fp32 [M][H] in m->ly, or K-split partial sums in m->sk_part (the sandwich norm adds them up)
+struct SubOut { const float* y; int slices; int64_t stride; };
+// the norm that follows: rms(x) * w, with b a layer norm, or (w NULL, raw) x as it is
+struct NextNorm { const float *w, *b; bool raw; };
+// experts' results that join the stream beside a sublayer's: K slices, or rows of pairs to be gathered and weighted
+struct ExpertOut { const float* y = nullptr; int slices = 0; int64_t stride = 0; const int32_t* slot_of = nullptr; const float* gate_w = nullptr; };
+
+// x += rms(y) * w_post (w_post NULL: x += y + experts) and / or xn = next(x) (elem.h SandwichArgs)
+void sandwich(nvl_model* m, SubOut y, const float* w_post, NextNorm next, void* xn, int rows, const int32_t* rows_idx = nullptr, ExpertOut ex = {}) {
+    KScope ks(m, KC_OTHER, 0, KS_SANDWICH, (double)rows * m->Hn * ((y.y ? 8.0 + 4.0 * (std::max(y.slices, 1) + ex.slices) : 4.0) + (next.w || next.raw ? (double)m->wsize : 0.0)));
     SandwichArgs a{};
-    a.x = m->x; a.y = y; a.slices = slices; a.slice_stride = slice_stride; a.w_post = w_post; a.w_next = w_next; a.rows_idx = rows_idx;
-    a.rows = rows; a.H = m->H; a.width = m->Hn; a.eps = m->cfg.norm_eps; a.raw_next = raw_next;
-    if (!m->f32 && rows > 512 && m->H <= 4096 && slices <= 1) {
+    a.x = m->x; a.y = y.y; a.slices = y.slices; a.slice_stride = y.stride; a.w_post = w_post; a.w_next = next.w; a.b_next = next.b; a.rows_idx = rows_idx;
+    a.rows = rows; a.H = m->H; a.width = m->Hn; a.eps = m->cfg.norm_eps; a.raw_next = next.raw;
+    a.y2 = ex.y; a.slices2 = ex.slices; a.stride2 = ex.stride; a.slot_of = ex.slot_of; a.gate_w = ex.gate_w;
+    const bool ext = (y.y && !w_post) || next.b;
+    if (!m->f32 && rows > 512 && m->H <= 4096 && y.slices <= 1) {
         const size_t lds = (size_t)16 * m->H * 2;
-#define NVL_SW16(CH)                                                                                                        \
+#define NVL_SW16E(CH, EXT)                                                                                                  \
         do {                                                                                                                \
-            NVL_LDS_ATTR((sandwich_tile16_kernel<CH>), 160 * 1024);                                                         \
-            hipLaunchKernelGGL((sandwich_tile16_kernel<CH>), dim3(cdiv(rows, 16)), dim3(1024), lds, m->stream, a, (bf16_t*)xn); \
+            NVL_LDS_ATTR((sandwich_tile16_kernel<CH, EXT>), 160 * 1024);                                                    \
+            hipLaunchKernelGGL((sandwich_tile16_kernel<CH, EXT>), dim3(cdiv(rows, 16)), dim3(1024), lds, m->stream, a, (bf16_t*)xn); \
         } while (0)
+#define NVL_SW16(CH) do { if (ext) NVL_SW16E(CH, true); else NVL_SW16E(CH, false); } while (0)
         if (m->H <= 1024) NVL_SW16(4); else if (m->H <= 2048) NVL_SW16(8); else NVL_SW16(16);
 #undef NVL_SW16
+#undef NVL_SW16E
     } else {
 #define NVL_SWR(CH)                                                                                                          \
         do {                                                                                                                \
-            if (m->f32) hipLaunchKernelGGL((sandwich_row_kernel<float, CH>), dim3(rows), dim3(256), 0, m->stream, a, (float*)xn); \
+            if (m->f32 && ext) hipLaunchKernelGGL((sandwich_row_kernel<float, CH, true>), dim3(rows), dim3(256), 0, m->stream, a, (float*)xn); \
+            else if (m->f32) hipLaunchKernelGGL((sandwich_row_kernel<float, CH>), dim3(rows), dim3(256), 0, m->stream, a, (float*)xn); \
+            else if (ext) hipLaunchKernelGGL((sandwich_row_kernel<bf16_t, CH, true>), dim3(rows), dim3(256), 0, m->stream, a, (bf16_t*)xn); \
             else hipLaunchKernelGGL((sandwich_row_kernel<bf16_t, CH>), dim3(rows), dim3(256), 0, m->stream, a, (bf16_t*)xn);      \
         } while (0)
         if (m->H <= 1024) NVL_SWR(1); else if (m->H <= 2048) NVL_SWR(2); else if (m->H <= 4096) NVL_SWR(4); else NVL_SWR(20);
@@ -623,8 +788,6 @@ void sandwich(nvl_model* m, const float* y, int slices, int64_t slice_stride, co
     NVL_HIP(hipGetLastError());
 }
 
-// a sublayer's last projection: fp32 [M][H] in m->ly, or K-split partial sums in m->sk_part (the sandwich norm adds them up)
-struct SubOut { const float* y; int slices; int64_t stride; };
 SubOut sub_out(nvl_model* m, int site, const void* A, const void* W, int M, int K) {
     const int N = m->H;
     int slices = 1;
@@ -678,7 +841,7 @@ void mix_latent(nvl_model* m, const LayerRun& r, const MixerW& w, const Meta& md
     a.seq_pos = md.seq_pos; a.tbl_stride = m->blocks_per_seq;
     a.q = m->lq; a.q_ld = (int64_t)H * r.dp;
     a.kbase = md.kbase + (int64_t)r.win * m->opts.max_seqs;
-    a.out = m->lmix; a.out_ld = r.ko;
+    a.out = m->lmix; a.out_ld = r.kd;
     {
         KScope ks(m, KC_OTHER, 0, KS_LAT_NORM, (double)M * (c.q_rank + (a.own ? c.kv_rank + c.rot_dim : 0)) * (4.0 + ws));
         if (m->f32) hipLaunchKernelGGL((latent_norm_kernel<float>), dim3(M), dim3(256), 0, m->stream, a);
@@ -900,7 +1063,7 @@ LinRecArgs linrec_args(nvl_model* m, const LayerRun& r, const Meta& md) {
     a.o = m->lo; a.o_ld = m->lo_ld;
     a.state = m->rec_state + r.state_off; a.slot_stride = m->rec_slot_stride;
     a.seq_tok_start = md.seq_tok_start; a.seq_len = md.seq_len; a.seq_pos = md.seq_pos; a.seq_slot = md.seq_slot;
-    a.eps = m->cfg.norm_eps; a.out = m->lmix; a.out_ld = r.ko;
+    a.eps = m->cfg.norm_eps; a.out = m->lmix; a.out_ld = r.kd;
     return a;
 }
 
@@ -938,7 +1101,7 @@ void mix_mamba2(nvl_model* m, const LayerRun& r, const MixerW& w, const Meta& md
         a.v = m->lconv; a.k = m->lconv + inner; a.q = m->lconv + inner + GN; a.ld = m->lconv_ld;
     }
     linrec<false>(m, a, n_seqs, M, max_len, fused, KS_MAMBA_SCAN);
-    GatedNormArgs g{m->lo, m->lo_ld, m->lproj, m->lproj_ld, w.mix_norm, M, c.norm_groups, inner / c.norm_groups, m->cfg.norm_eps, r.ko, 0, 0};
+    GatedNormArgs g{m->lo, m->lo_ld, m->lproj, m->lproj_ld, w.mix_norm, M, c.norm_groups, inner / c.norm_groups, m->cfg.norm_eps, r.kd, 0, 0};
     gated_norm<true>(m, g, KS_MAMBA_GATE);
 }
 
@@ -954,7 +1117,7 @@ void mix_gla(nvl_model* m, const LayerRun& r, const MixerW& w, const Meta& md, i
     const bool fused = max_len <= REC_STEP_MAX;
     linrec<true>(m, a, n_seqs, M, max_len, fused, KS_GLA_SCAN);
     if (fused) return;
-    GatedNormArgs g{m->lo, m->lo_ld, a.gate, m->lproj_ld, w.mix_norm, M, c.heads, c.vdim, m->cfg.norm_eps, r.ko, 0, 0};
+    GatedNormArgs g{m->lo, m->lo_ld, a.gate, m->lproj_ld, w.mix_norm, M, c.heads, c.vdim, m->cfg.norm_eps, r.kd, 0, 0};
     gated_norm<false>(m, g, KS_GLA_GATE);
 }
 
@@ -998,7 +1161,7 @@ void mix_delta(nvl_model* m, const LayerRun& r, const MixerW& w, const Meta& md,
         a.ring = ring; a.ring_slot_stride = m->rec_slot_stride;
         a.a1 = m->lproj + r.a1_off; a.g1 = m->lproj + r.g1_off; a.lr_ld = m->lproj_ld;
         a.a_rank = w.rank; a.g_rank = w.grank; a.a_rkp = w.a_rkp; a.g_rkp = w.g_rkp; a.a2 = w.a2r; a.g2 = w.g2r;
-        a.norm_w = w.mix_norm; a.eps = m->cfg.norm_eps; a.out = m->lmix; a.out_ld = r.ko;
+        a.norm_w = w.mix_norm; a.eps = m->cfg.norm_eps; a.out = m->lmix; a.out_ld = r.kd;
         KScope ks(m, KC_OTHER, 6.0 * M * elems, KS_DELTA_SCAN, 2.0 * n_seqs * elems * 4.0 + (double)M * (r.conv_dim * 4.0 * (c.conv_taps + 1) + hv * (double)m->wsize) +
                                                                    ((double)hd * w.rank + (double)hv * w.grank) * (double)m->wsize);
         delta_step(m, a, n_seqs, true);
@@ -1071,31 +1234,186 @@ void mix_delta(nvl_model* m, const LayerRun& r, const MixerW& w, const Meta& md,
             NVL_HIP(hipGetLastError());
         }
     }
-    GatedNormArgs g{m->lo, m->lo_ld, m->lg, m->lg_ld, w.mix_norm, M, c.heads, c.vdim, m->cfg.norm_eps, r.ko, 0, 1};
+    GatedNormArgs g{m->lo, m->lo_ld, m->lg, m->lg_ld, w.mix_norm, M, c.heads, c.vdim, m->cfg.norm_eps, r.kd, 0, 1};
     gated_norm<false>(m, g, KS_DELTA_GATE);
 }
 
 void tap_layer(nvl_model* m, int li, int M);
+
+// ---- grouped-query attention: m->xn -> m->lmix columns [0, ko) ----
+void mix_grouped(nvl_model* m, const LayerRun& r, const MixerW& w, const Meta& md, int n_seqs, int M, int max_len) {
+    const nvl_layer_config& c = r.c;
+    in_proj(m, r, w, M);
+    GroupedArgs a{};
+    a.H = c.heads; a.G = c.kv_heads; a.group = c.heads / c.kv_heads; a.dim = c.dim; a.dp = r.dp; a.vdim = c.vdim; a.vp = r.vp;
+    a.window = c.window; a.scale = c.scale; a.softcap = c.softcap; a.r1 = w.r1; a.r2 = w.r2;
+    a.proj = m->lproj; a.proj_ld = m->lproj_ld; a.k_off = r.k_off; a.v_off = r.v_off; a.gate_off = r.gate_off;
+    a.mix = r.mix; a.lambda = w.v_lambda; a.vfirst = m->lvf; a.vfirst_ld = m->lvf_ld;
+    a.cache = (char*)m->lat_cache + r.cache_off * (int64_t)m->wsize; a.block_stride = m->lat_block_stride; a.bs = m->Tmax;
+    a.blk_table = md.blk_table; a.seq_tok_start = md.seq_tok_start; a.seq_len = md.seq_len; a.seq_pos = md.seq_pos; a.tbl_stride = m->blocks_per_seq;
+    a.out = m->lmix; a.out_ld = r.kd;
+    const double ws = (double)m->wsize;
+    {
+        KScope ks(m, KC_OTHER, 0, KS_KV_PLACE, (double)M * a.G * (c.dim + c.vdim) * (4.0 + ws) + (r.mix ? (double)M * a.G * c.vdim * 4.0 : 0.0));
+        const dim3 grid(cdiv(max_len + 31, 32), n_seqs, a.G);
+        if (m->f32) hipLaunchKernelGGL((grouped_place_kernel<float>), grid, dim3(256), 0, m->stream, a);
+        else hipLaunchKernelGGL((grouped_place_kernel<bf16_t>), grid, dim3(256), 0, m->stream, a);
+        NVL_HIP(hipGetLastError());
+    }
+    const bool plain = m->f32 || r.dp > 256 || r.vp > 256;
+    const int ctx = m->ctx_hint > 0 ? m->ctx_hint : m->cfg.max_seq_len;
+    int tiles = cdiv(ctx, 64) + 1;                              // most key tiles a 256-row workgroup walks
+    if (c.window > 0) tiles = std::min(tiles, (c.window + cdiv(256, a.group) + 1) / 64 + 3);
+    const size_t ring = (size_t)3 * round_up(4 * (r.dp >> 5) + 2 * (r.vp >> 4), 8) * 1024, lds = ring + (size_t)tiles * 8;
+    a.short_rows = GROUPED_SHORT_ROWS;
+    if ((r.dp == 256 && r.vp == 256) || lds > 160 * 1024) a.short_rows = 1 << 30;      // (three slots would not fit LDS)
+    const bool any_short = m->min_len * a.group <= a.short_rows, any_long = max_len * a.group > a.short_rows;
+    auto scope = [&](int several) {
+        const double pairs = m->win_pairs[(size_t)r.win][(size_t)several], keys = m->win_keys[(size_t)r.win][(size_t)several];
+        return KScope(m, KC_ATTN, 2.0 * pairs * a.H * (c.dim + c.vdim), KS_ATTN, keys * a.G * (c.dim + c.vdim) * ws + (double)M * a.H * (4.0 * c.dim + (4.0 + ws) * c.vdim));
+    };
+    if (plain) {
+        KScope ks = scope(max_len > 1);
+        const dim3 grid(max_len, a.H, n_seqs);
+        const size_t sm = (size_t)(r.dp + r.vp) * 4;
+        if (m->f32) hipLaunchKernelGGL((grouped_plain_kernel<float>), grid, dim3(256), sm, m->stream, a);
+        else hipLaunchKernelGGL((grouped_plain_kernel<bf16_t>), grid, dim3(256), sm, m->stream, a);
+        NVL_HIP(hipGetLastError());
+        return;
+    }
+    const int ks = r.dp == 32 ? 1 : r.dp >> 5, dt = r.vp >> 4;
+    if (any_long) {
+        KScope scp = scope(1);
+        const dim3 grid(a.G, n_seqs, cdiv((int64_t)max_len * a.group, 256));
+#define NVL_GP(KSv, DTv)                                                                                                     \
+        do {                                                                                                                 \
+            NVL_LDS_ATTR((grouped_prefill_kernel<KSv, DTv>), 160 * 1024);                                                    \
+            hipLaunchKernelGGL((grouped_prefill_kernel<KSv, DTv>), grid, dim3(512), lds, m->stream, a);                      \
+        } while (0)
+#define NVL_GPK(KSv) do { if (dt == 2) NVL_GP(KSv, 2); else if (dt == 4) NVL_GP(KSv, 4); else if (dt == 8) NVL_GP(KSv, 8); else NVL_GP(KSv, 16); } while (0)
+        if (ks == 1) NVL_GPK(1); else if (ks == 2) NVL_GPK(2); else if (ks == 4) NVL_GPK(4);
+        else if (dt == 2) NVL_GP(8, 2); else if (dt == 4) NVL_GP(8, 4); else NVL_GP(8, 8);
+#undef NVL_GPK
+#undef NVL_GP
+        NVL_HIP(hipGetLastError());
+    }
+    if (any_short) {
+        KScope scp = scope(any_long ? 0 : max_len > 1);
+        const int64_t wgs = (int64_t)a.G * cdiv(std::min<int64_t>((int64_t)max_len * a.group, a.short_rows), 16);
+        int z = 1;
+        while (z < GROUPED_SPLITS && wgs * n_seqs * z * 2 <= m->grp_cap && z * 2 * 4 <= (1 << layered_kt_log2(m))) z *= 2;
+        a.part = m->grp_part; a.part_cnt = m->grp_cnt;
+        const dim3 grid((unsigned)wgs, n_seqs, z);
+#define NVL_GS(KSv, DTv)                                                                                                     \
+        do {                                                                                                                 \
+            NVL_LDS_ATTR((grouped_short_kernel<KSv, DTv, 4>), 4 * DTv * 1024);                                               \
+            hipLaunchKernelGGL((grouped_short_kernel<KSv, DTv, 4>), grid, dim3(256), 4 * DTv * 1024, m->stream, a);          \
+        } while (0)
+#define NVL_GSK(KSv) do { if (dt == 2) NVL_GS(KSv, 2); else if (dt == 4) NVL_GS(KSv, 4); else if (dt == 8) NVL_GS(KSv, 8); else NVL_GS(KSv, 16); } while (0)
+        if (ks == 1) NVL_GSK(1); else if (ks == 2) NVL_GSK(2); else if (ks == 4) NVL_GSK(4); else NVL_GSK(8);
+#undef NVL_GSK
+#undef NVL_GS
+        NVL_HIP(hipGetLastError());
+    }
+}
+
+// ---- feed-forward of a parallel block: m->xn -> m->lmix columns [ko, kd); the experts' results for the join ----
+ExpertOut parallel_ffn(nvl_model* m, const LayerRun& r, const MixerW& w, int M) {
+    const nvl_layer_config& c = r.c;
+    if (c.ffn_dim) {
+        m->site = KS_FFN_UP;
+        const bool relu2 = r.act == NVL_ACT_RELU2;
+        const int N = relu2 ? r.Fp : 2 * r.Fp;
+        if (m->f32) {
+            gemm(m, EPI_STORE, true, mk(m->xn, m->H, w.w1, m->h2, N, nullptr, 1.f, M, N, m->H));
+            const int64_t n = (int64_t)M * r.Fp;
+            KScope ks(m, KC_OTHER);
+            if (relu2) hipLaunchKernelGGL((relu2_kernel<float>), dim3(cdiv(n, 256)), dim3(256), 0, m->stream, m->h2, (float*)m->lmix, (int64_t)M, r.Fp, (int64_t)r.kd, r.ko);
+            else hipLaunchKernelGGL((swiglu_kernel<float>), dim3(cdiv(n, 256)), dim3(256), 0, m->stream, m->h2, (float*)m->lmix, (int64_t)M, r.Fp, (int64_t)r.kd, r.ko);
+            NVL_HIP(hipGetLastError());
+        } else      // (the operand's column blocks are 32 wide: a shift by ko columns is a shift of the base)
+            gemm(m, relu2 ? EPI_RELU2 : EPI_SWIGLU, false, mk(m->xn, m->H, w.w1, (bf16_t*)m->lmix + (r.ko >> 5) * 512, r.kd, nullptr, 1.f, M, N, m->H));
+    }
+    if (!c.experts) return {};
+    const int E = c.experts, k = c.top_k, pairs = M * k;
+    // decode: all experts as one projection each way with the routing weights as a mask (gemm.h GemmArgs::moe_gate)
+    const bool dense = !m->f32 && M <= 64 && r.Ip <= 2048;
+    GroupRouteArgs ra{m->lproj + r.route_off, m->lproj_ld, w.route_bias, M, E, k, c.expert_groups, c.groups_kept, m->expert_ids, m->expert_w, dense ? m->moe_gate : nullptr, r.Ep};
+    {
+        KScope ks(m, KC_OTHER, 0, KS_MOE_ROUTER, (double)M * (E + 2.0 * k) * 4.0);
+        hipLaunchKernelGGL(moe_route_grouped_kernel, dim3(cdiv(M, 4)), dim3(256), 0, m->stream, ra);
+        NVL_HIP(hipGetLastError());
+    }
+    const double touch = (double)std::min(E, pairs);
+    if (dense) {
+        GemmArgs u = mk(m->xn, m->H, w.moe_up, m->moe_hall, r.Ep * r.Ip, nullptr, 1.f, M, E * 2 * r.Ip, m->H);
+        u.moe_gate = m->moe_gate; u.moe_E = r.Ep; u.moe_I = r.Ip;
+        m->site = KS_MOE_UP; m->site_bytes = (touch * 2 * c.expert_dim * m->Hn + (double)M * m->Hn + (double)pairs * c.expert_dim) * (double)m->wsize;
+        gemm(m, EPI_SWIGLU, false, u, 4.0 * pairs * c.expert_dim * m->Hn);
+        GemmArgs d = mk(m->moe_hall, r.Ep * r.Ip, w.moe_cat, m->x, m->H, nullptr, 1.f, M, m->H, r.Ep * r.Ip);      // (K slices: plain stores into moe_part)
+        d.moe_gate = m->moe_gate; d.moe_E = r.Ep; d.moe_I = r.Ip; d.sk_part = m->moe_part; d.sk_slices = r.moe_slices;
+        m->site = KS_MOE_DOWN; m->site_bytes = (touch * m->Hn * c.expert_dim + (double)pairs * c.expert_dim) * (double)m->wsize + (double)r.moe_slices * M * m->Hn * 4.0;
+        gemm(m, EPI_RESID, true, d, 2.0 * pairs * m->Hn * c.expert_dim);
+        return {m->moe_part, r.moe_slices, (int64_t)M * m->H, nullptr, nullptr};
+    }
+    const bool pp = moe_pp_ok(m, r.Ip, false);
+    const int BM = pp ? 256 : ((!m->f32 && g_moe_bm == 256) ? 256 : 128);
+    moe_sort(m, E, k, M, BM);
+    moe_expert_gemms(m, MoeW{E, k, r.Ip, w.moe_up, w.moe_down}, M, BM, pp, false);
+    return {m->moe_eo, k, 0, m->slot_of, m->expert_w};
+}
+
+// ---- per-layer token input: x (as m->xn) -> m->ly or its K slices ----
+SubOut side_input(nvl_model* m, const MixerW& w, const Meta& md, int li, int M) {
+    const int sd = m->cfg.side_dim, kp = m->side_kp;
+    const int64_t col = (int64_t)li * round_up(sd, 4);
+    m->site = KS_SIDE_GATE;
+    if (m->f32) {
+        gemm(m, EPI_STORE, true, mk(m->xn, m->H, w.side_gate, m->h2, (int)round_up(sd, 4), nullptr, 1.f, M, sd, m->H));
+        KScope ks(m, KC_OTHER);
+        hipLaunchKernelGGL((gelu_token_kernel<float, float>), dim3(M), dim3(256), 0, m->stream, m->h2, round_up(sd, 4), (const float*)m->side_emb + col, m->side_ld, md.tokens, (float*)m->lside, (int64_t)kp, sd);
+        NVL_HIP(hipGetLastError());
+    } else {
+        GemmArgs a = mk(m->xn, m->H, w.side_gate, m->lside, kp, nullptr, 1.f, M, sd, m->H);
+        a.tok_ids = md.tokens; a.tok_table = (const bf16_t*)m->side_emb + col; a.tok_ld = m->side_ld;
+        gemm(m, EPI_GELU_TOK, false, a);
+    }
+    return sub_out(m, KS_SIDE_PROJ, m->lside, w.side_proj, M, kp);
+}
 
 // The layers of one pass.  have_xn: m->xn already holds the first norm (decode seam).  all_rows: the logits of every row are wanted,
 // in order: the last sandwich norm then leaves the final norm of every row in m->xn; returns whether it did.
 bool layered_stack(nvl_model* m, const Meta& md, int n_seqs, int M, int max_len, bool have_xn, bool all_rows) {
     auto W = [&](int li) -> const MixerW& { return m->mixers[(size_t)m->runs[(size_t)li].owner]; };
     const bool post = m->cfg.block_style == NVL_BLOCK_POST;        // sublayers read x itself
+    const bool par = m->cfg.block_style == NVL_BLOCK_PARALLEL;
     m->key_src = m->key_win = -1;
-    if (!have_xn) sandwich(m, nullptr, 0, 0, nullptr, W(0).norm1, nullptr, m->xn, M, post);
+    if (!have_xn) sandwich(m, SubOut{}, nullptr, {W(0).norm1, W(0).norm1_bias, post}, m->xn, M);
     for (int li = 0; li < m->L; li++) {
         const LayerRun& r = m->runs[(size_t)li];
         const MixerW& w = W(li);
-        const float* after = li + 1 < m->L ? W(li + 1).norm1 : (all_rows ? m->final_norm : nullptr);      // the norm that follows this layer
+        NextNorm after{nullptr, nullptr, post};                    // the norm that follows this layer
+        if (li + 1 < m->L) { after.w = W(li + 1).norm1; after.b = W(li + 1).norm1_bias; }
+        else if (all_rows) { after.w = m->final_norm; after.b = m->final_norm_b; }
         switch (r.c.mixer) {
             case NVL_MIXER_LATENT_ATTENTION: mix_latent(m, r, w, md, n_seqs, M, max_len); break;
             case NVL_MIXER_MAMBA2: mix_mamba2(m, r, w, md, n_seqs, M, max_len); break;
             case NVL_MIXER_CHANNEL_DELTA: mix_delta(m, r, w, md, n_seqs, M, max_len); break;
+            case NVL_MIXER_ATTENTION: mix_grouped(m, r, w, md, n_seqs, M, max_len); break;
             default: mix_gla(m, r, w, md, n_seqs, M, max_len);
         }
-        SubOut y = sub_out(m, KS_OPROJ, m->lmix, w.o, M, r.ko);
-        sandwich(m, y.y, y.slices, y.stride, w.norm1b, r.c.ffn_dim ? w.norm2 : after, nullptr, m->xn, M, post);
+        if (par) {
+            const ExpertOut ex = parallel_ffn(m, r, w, M);
+            const SubOut y = sub_out(m, KS_OPROJ, m->lmix, w.o, M, r.kd);
+            if (m->cfg.side_dim) {
+                sandwich(m, y, nullptr, {nullptr, nullptr, true}, m->xn, M, nullptr, ex);
+                sandwich(m, side_input(m, w, md, li, M), w.side_norm, after, m->xn, M);
+            } else sandwich(m, y, nullptr, after, m->xn, M, nullptr, ex);
+            tap_layer(m, li, M);
+            continue;
+        }
+        SubOut y = sub_out(m, KS_OPROJ, m->lmix, w.o, M, r.kd);
+        sandwich(m, y, w.norm1b, r.c.ffn_dim ? NextNorm{w.norm2, nullptr, post} : after, m->xn, M);
         if (r.c.ffn_dim) {
             m->site = KS_FFN_UP;
             const bool clamped = m->cfg.activation_type == NVL_ACT_CLAMPED_GLU;
@@ -1104,7 +1422,7 @@ bool layered_stack(nvl_model* m, const Meta& md, int n_seqs, int M, int max_len,
                 const int64_t n = (int64_t)M * r.Fp;
                 KScope ks(m, KC_OTHER);
                 if (clamped) hipLaunchKernelGGL((clamp_glu_kernel<float>), dim3(cdiv(n, 256)), dim3(256), 0, m->stream, m->h2, (float*)m->hbuf, (int64_t)M, r.Fp, r.c.ffn_limit, CLAMPED_GLU_SLOPE);
-                else hipLaunchKernelGGL((swiglu_kernel<float, true>), dim3(cdiv(n, 256)), dim3(256), 0, m->stream, m->h2, (float*)m->hbuf, (int64_t)M, r.Fp);
+                else hipLaunchKernelGGL((swiglu_kernel<float, true>), dim3(cdiv(n, 256)), dim3(256), 0, m->stream, m->h2, (float*)m->hbuf, (int64_t)M, r.Fp, (int64_t)r.Fp, 0);
                 NVL_HIP(hipGetLastError());
             } else {
                 GemmArgs up = mk(m->xn, m->H, w.w1, m->hbuf, r.Fp, nullptr, 1.f, M, 2 * r.Fp, m->H);
@@ -1112,7 +1430,7 @@ bool layered_stack(nvl_model* m, const Meta& md, int n_seqs, int M, int max_len,
                 gemm(m, clamped ? EPI_CLAMP_GLU : EPI_GEGLU, false, up);
             }
             y = sub_out(m, KS_FFN_DOWN, m->hbuf, w.w2, M, r.Fp);
-            sandwich(m, y.y, y.slices, y.stride, w.norm2b, after, nullptr, m->xn, M, post);
+            sandwich(m, y, w.norm2b, after, m->xn, M);
         }
         tap_layer(m, li, M);
     }

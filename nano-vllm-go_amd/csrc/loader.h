@@ -283,8 +283,10 @@ std::vector<float> to_f32(const StTensor& t) {
 }
 
 // ---- models described by a list of layers ----
-struct LayeredArch { const char* name; int block_style, activation; float norm_offset; };
-const LayeredArch LAYERED_ARCHS[] = {{"Potuzen", NVL_BLOCK_SANDWICH, NVL_ACT_GEGLU, 0.f}, {"Lufazen", NVL_BLOCK_POST, NVL_ACT_CLAMPED_GLU, 1.f}};
+struct LayeredArch { const char* name; int block_style, activation; float norm_offset; int norm_type, position_type; };
+const LayeredArch LAYERED_ARCHS[] = {{"Potuzen", NVL_BLOCK_SANDWICH, NVL_ACT_GEGLU, 0.f, NVL_NORM_RMS, NVL_POS_NONE},
+                                     {"Lufazen", NVL_BLOCK_POST, NVL_ACT_CLAMPED_GLU, 1.f, NVL_NORM_RMS, NVL_POS_NONE},
+                                     {"Bolinex", NVL_BLOCK_PARALLEL, NVL_ACT_RELU2, 0.f, NVL_NORM_LAYER, NVL_POS_LEARNED}};
 const LayeredArch* layered_arch(const std::string& name) {
     for (const LayeredArch& a : LAYERED_ARCHS) if (name == a.name) return &a;
     return nullptr;
@@ -311,8 +313,30 @@ void parse_rotation(const JVal* mx, nvl_layer_config& c, const std::string& at) 
         c.rot_fast = need_num(sc, "fast", at); c.rot_slow = need_num(sc, "slow", at);
     }
 }
+// grouped-query attention: kv_heads, softcap (a number or null), v_mix (true / false)
+void parse_attention(const JVal* mx, nvl_layer_config& c, const std::string& at) {
+    c.mixer = NVL_MIXER_ATTENTION;
+    c.dim = need_int(mx, "dim", at); c.kv_heads = need_int(mx, "kv_heads", at); c.scale = (float)need_num(mx, "scale", at);
+    const JVal *cap = mx->get("softcap"), *mix = mx->get("v_mix");
+    if (cap && cap->kind != JVal::NUL) {
+        c.softcap = (float)need_num(mx, "softcap", at);
+        if (!(c.softcap > 0.f)) throw std::runtime_error(at + "softcap is not positive");
+    }
+    c.v_mix = mix && ((mix->kind == JVal::BOOL && mix->b) || (mix->kind == JVal::NUM && mix->num != 0));
+}
+// a mixture of experts: {expert: {ff}, router: {experts, top, groups: null | {count, keep}}, shared: null | {ff}}
+void parse_experts(const JVal* mlp, nvl_layer_config& c, const std::string& at) {
+    const JVal *ex = mlp->get("expert"), *ro = mlp->get("router"), *sh = mlp->get("shared");
+    c.expert_dim = need_int(ex, "ff", at); c.experts = need_int(ro, "experts", at); c.top_k = need_int(ro, "top", at);
+    c.expert_groups = c.groups_kept = 1;
+    const JVal* gr = ro->get("groups");
+    if (gr && gr->kind == JVal::OBJ) { c.expert_groups = need_int(gr, "count", at); c.groups_kept = need_int(gr, "keep", at); }
+    c.ffn_act = NVL_ACT_SWIGLU;
+    if (sh && sh->kind == JVal::OBJ) c.ffn_dim = need_int(sh, "ff", at);
+    if (c.experts <= 0 || c.expert_dim <= 0 || c.ffn_dim < 0) throw std::runtime_error(at + "an expert size is not positive");
+}
 std::vector<nvl_layer_config> parse_layers(const JVal& raw, const LayeredArch& arch) {
-    const bool post = arch.block_style == NVL_BLOCK_POST;
+    const bool post = arch.block_style == NVL_BLOCK_POST, par = arch.block_style == NVL_BLOCK_PARALLEL;
     const JVal* ls = raw.get("layers");
     if (!ls || ls->kind != JVal::ARR || ls->arr.empty()) throw std::runtime_error("config: list 'layers' expected");
     std::vector<nvl_layer_config> out;
@@ -326,7 +350,8 @@ std::vector<nvl_layer_config> parse_layers(const JVal& raw, const LayeredArch& a
         if (!ty || ty->kind != JVal::STR || !mx || mx->kind != JVal::OBJ) throw std::runtime_error(at + "'type' and 'mixer' expected");
         c.weights_of = wo && wo->kind == JVal::NUM ? need_int(&e, "weights_of", at) : -1;
         c.heads = need_int(mx, "heads", at); c.vdim = need_int(mx, "vdim", at);
-        if (ty->str == "latent_attention") {
+        if (ty->str == "attention" && par) parse_attention(mx, c, at);
+        else if (ty->str == "latent_attention" && !par) {
             c.mixer = NVL_MIXER_LATENT_ATTENTION;
             c.dim = need_int(mx, "dim", at); c.q_rank = need_int(mx, "q_rank", at); c.kv_rank = need_int(mx, "kv_rank", at);
             c.scale = (float)need_num(mx, "scale", at);
@@ -336,24 +361,25 @@ std::vector<nvl_layer_config> parse_layers(const JVal& raw, const LayeredArch& a
                 const JVal* kf = mx->get("kv_from");
                 if (kf && kf->kind == JVal::NUM) c.kv_from = need_int(mx, "kv_from", at);
             }
-            const JVal* mask = mx->get("mask");
-            if (mask && mask->kind == JVal::OBJ) {
-                c.window = need_int(mask, "size", at);
-                if (c.window <= 0) throw std::runtime_error(at + "the window is not positive");
-            }
         } else if (ty->str == "channel_delta" && post) {
             c.mixer = NVL_MIXER_CHANNEL_DELTA;
             c.dim = need_int(mx, "dim", at); c.kv_heads = need_int(mx, "kv_heads", at); c.conv_taps = need_int(mx, "conv", at);
-        } else if (ty->str == "mamba2" && !post) {
+        } else if (ty->str == "mamba2" && !post && !par) {
             c.mixer = NVL_MIXER_MAMBA2;
             c.state = need_int(mx, "state", at); c.groups = need_int(mx, "groups", at); c.norm_groups = need_int(mx, "norm_groups", at);
             c.conv_taps = need_int(mx, "conv", at);
-        } else if (ty->str == "gla" && !post) {
+        } else if (ty->str == "gla" && !post && !par) {
             c.mixer = NVL_MIXER_GLA;
             c.dim = need_int(mx, "dim", at); c.tau = (float)need_num(mx, "tau", at);
         } else throw std::runtime_error(at + "unknown mixer '" + ty->str + "'");
+        const JVal* mask = mx->get("mask");
+        if (mask && mask->kind == JVal::OBJ && (c.mixer == NVL_MIXER_LATENT_ATTENTION || c.mixer == NVL_MIXER_ATTENTION)) {
+            c.window = need_int(mask, "size", at);
+            if (c.window <= 0) throw std::runtime_error(at + "the window is not positive");
+        }
         if (mlp && mlp->kind == JVal::OBJ) {
             const JVal* kind = mlp->get("kind");
+            if (par && kind && kind->kind == JVal::STR && kind->str == "moe") { parse_experts(mlp, c, at); out.push_back(c); continue; }
             if (kind && !(kind->kind == JVal::STR && kind->str == "dense")) throw std::runtime_error(at + "unknown feed-forward kind");
             c.ffn_dim = need_int(mlp, "ff", at);
             if (c.ffn_dim <= 0) throw std::runtime_error(at + "the feed-forward size is not positive");
@@ -379,7 +405,10 @@ void load_layered(nvl_model* m, const StSet& st) {
         }
         if (nvl_upload_tensor(m, kind, layer, all.data(), a.dtype, rows, a.shape[1], OI)) throw std::runtime_error(nvl_last_error(m));
     };
-    const bool post = m->cfg.block_style == NVL_BLOCK_POST;
+    const bool post = m->cfg.block_style == NVL_BLOCK_POST, par = m->cfg.block_style == NVL_BLOCK_PARALLEL;
+    if (m->cfg.norm_type == NVL_NORM_LAYER) vec(NVL_T_FINAL_NORM_B, 0, "final.norm.b");
+    if (m->cfg.position_type == NVL_POS_LEARNED) mat(NVL_T_POS_EMB, 0, "pos");
+    if (m->cfg.side_dim) mat(NVL_T_SIDE_EMB, 0, "side.embed");
     mat(NVL_T_TOK_EMB, 0, "embed");
     mat(NVL_T_LM_HEAD, 0, "head");
     vec(NVL_T_FINAL_NORM_W, 0, "final.norm");
@@ -387,20 +416,42 @@ void load_layered(nvl_model* m, const StSet& st) {
         const LayerRun& r = m->runs[(size_t)i];
         if (r.owner != i) continue;
         const std::string l = "l" + std::to_string(i) + ".", x = l + "mix.";
-        if (post) {
+        if (par) {
+            vec(NVL_T_ATTN_NORM_W, i, l + "norm1");
+            if (m->cfg.norm_type == NVL_NORM_LAYER) vec(NVL_T_ATTN_NORM_B, i, l + "norm1.b");
+            if (m->cfg.side_dim) { mat(NVL_T_SIDE_GATE, i, l + "side.gate"); mat(NVL_T_SIDE_PROJ, i, l + "side.proj"); vec(NVL_T_SIDE_NORM, i, l + "side.norm"); }
+        } else if (post) {
             vec(NVL_T_MIX_POST_NORM, i, l + "norm1"); vec(NVL_T_MIX_SCALE, i, l + "ls1");
             if (r.c.ffn_dim) { vec(NVL_T_FFN_POST_NORM, i, l + "norm2"); vec(NVL_T_FFN_SCALE, i, l + "ls2"); }
         } else {
             vec(NVL_T_ATTN_NORM_W, i, l + "norm1"); vec(NVL_T_MIX_POST_NORM, i, l + "norm1b");
             if (r.c.ffn_dim) { vec(NVL_T_FFN_NORM_W, i, l + "norm2"); vec(NVL_T_FFN_POST_NORM, i, l + "norm2b"); }
         }
-        if (r.c.ffn_dim) { cat(NVL_T_W1, i, {l + "mlp.gate", l + "mlp.up"}); mat(NVL_T_W2, i, l + "mlp.down"); }
+        if (r.c.ffn_dim) {
+            const std::string f = l + (r.c.experts ? "mlp.shared." : "mlp.");
+            if (r.act == NVL_ACT_RELU2) mat(NVL_T_W1, i, f + "up"); else cat(NVL_T_W1, i, {f + "gate", f + "up"});
+            mat(NVL_T_W2, i, f + "down");
+        }
+        if (r.c.experts) {
+            std::vector<std::string> up, down;
+            for (int e = 0; e < r.c.experts; e++) {
+                const std::string x = l + "mlp.e" + std::to_string(e) + ".";
+                up.push_back(x + "gate"); up.push_back(x + "up"); down.push_back(x + "down");
+            }
+            cat(NVL_T_MOE_IN, i, up); cat(NVL_T_MOE_OUT, i, down);
+            mat(NVL_T_ROUTER, i, l + "mlp.router"); vec(NVL_T_ROUTER_BIAS, i, l + "mlp.correction");
+        }
         switch (r.c.mixer) {
             case NVL_MIXER_LATENT_ATTENTION:
                 mat(NVL_T_LAT_DQ, i, x + "dq"); vec(NVL_T_LAT_DQ_NORM, i, x + "dq.norm"); mat(NVL_T_LAT_UQ, i, x + "uq");
                 if (r.c.kv_from < 0) { mat(NVL_T_LAT_DKV, i, x + "dkv"); vec(NVL_T_LAT_DKV_NORM, i, x + "dkv.norm"); }
                 mat(NVL_T_LAT_UK, i, x + "uk"); mat(NVL_T_LAT_UV, i, x + "uv");
                 mat(NVL_T_MIX_GATE, i, x + "g"); mat(NVL_T_WO, i, x + "o");
+                break;
+            case NVL_MIXER_ATTENTION:
+                mat(NVL_T_WQ, i, x + "q"); mat(NVL_T_WK, i, x + "k"); mat(NVL_T_WV, i, x + "v"); mat(NVL_T_MIX_GATE, i, x + "g"); mat(NVL_T_WO, i, x + "o");
+                vec(NVL_T_BIAS_R1, i, x + "r1"); vec(NVL_T_BIAS_R2, i, x + "r2");
+                if (r.c.v_mix) vec(NVL_T_V_MIX, i, x + "vmix");
                 break;
             case NVL_MIXER_MAMBA2:
                 mat(NVL_T_MAMBA_IN_PROJ, i, x + "in"); vec(NVL_T_MAMBA_CONV_W, i, x + "conv"); vec(NVL_T_MAMBA_CONV_B, i, x + "conv.b");
@@ -577,12 +628,14 @@ extern "C" int nvl_load_config_json(const char* path, nvl_model_config* out) {
         memset(&c, 0, sizeof c);
         // ---- templates (config.go:125-376); `architecture` first, then model_type (:822-836, :975-1007), default GPT-2
         std::string arch = str("architecture");
-        if (const LayeredArch* la = layered_arch(arch)) {       // sizes and constants come from the file; it names no longest sequence
+        if (const LayeredArch* la = layered_arch(arch)) {       // sizes and constants come from the file
             c.vocab_size = need_int(&raw, "vocab", "config: "); c.hidden = need_int(&raw, "width", "config: ");
             c.num_layers = (int)parse_layers(raw, *la).size();
             c.norm_eps = (float)need_num(raw.get("norm"), "eps", "config: norm: ");
-            c.max_seq_len = 4096;
-            c.attention_type = NVL_ATTN_GQA; c.norm_type = NVL_NORM_RMS; c.position_type = NVL_POS_NONE;
+            c.max_seq_len = raw.get("max_positions") ? need_int(&raw, "max_positions", "config: ") : 4096;
+            if (la->position_type == NVL_POS_LEARNED && !raw.get("max_positions")) throw std::runtime_error("config: number 'max_positions' expected");
+            c.attention_type = NVL_ATTN_GQA; c.norm_type = la->norm_type; c.position_type = la->position_type;
+            if (const JVal* ts = raw.get("token_side")) if (ts->kind == JVal::OBJ && la->block_style == NVL_BLOCK_PARALLEL) c.side_dim = need_int(ts, "dim", "config: token_side: ");
             c.activation_type = la->activation; c.block_style = la->block_style; c.norm_weight_offset = la->norm_offset;
             double cap;
             if (num("logit_softcap", cap)) c.logit_softcap = (float)cap;

@@ -16,6 +16,7 @@
 #include "sample.h"
 #include "gemm.h"
 #include "latent.h"
+#include "grouped.h"
 #include "delta.h"
 #include "linrec.h"
 #include "mamba.h"
@@ -46,7 +47,8 @@ enum KClass { KC_GEMM = 0, KC_ATTN = 1, KC_OTHER = 2 };
 enum KSite { KS_OTHER = 0, KS_QKV, KS_ATTN, KS_OPROJ, KS_FFN_UP, KS_FFN_DOWN, KS_LM_HEAD, KS_NORM, KS_MOE_ROUTER, KS_MOE_PLAN,
              KS_MOE_UP, KS_MOE_DOWN, KS_MOE_COMBINE, KS_EMBED, KS_ARGMAX, KS_ROPE, KS_MAMBA_IN, KS_MAMBA_CONV, KS_MAMBA_SCAN,
              KS_MAMBA_GATE, KS_MAMBA_OUT, KS_ALLREDUCE, KS_MIX_IN, KS_LAT_NORM, KS_LAT_UQ, KS_LAT_GATHER, KS_LAT_KV, KS_LAT_ABSORB,
-             KS_LAT_UV, KS_GLA_SCAN, KS_GLA_GATE, KS_SANDWICH, KS_DELTA_CONV, KS_DELTA_PACK, KS_DELTA_RANK, KS_DELTA_PREP, KS_DELTA_SCAN, KS_DELTA_GATE, KS_COUNT };
+             KS_LAT_UV, KS_GLA_SCAN, KS_GLA_GATE, KS_SANDWICH, KS_DELTA_CONV, KS_DELTA_PACK, KS_DELTA_RANK, KS_DELTA_PREP, KS_DELTA_SCAN, KS_DELTA_GATE,
+             KS_KV_PLACE, KS_SIDE_GATE, KS_SIDE_PROJ, KS_COUNT };
 
 // one layer of a model described by a list of layers: its configuration, padded sizes, where its tensors and its memory are
 struct LayerRun {
@@ -62,7 +64,12 @@ struct LayerRun {
     int Fp = 0;                  // feed-forward columns (padded), 0: none
     int conv_dim = 0;
     int win = -1;                // index into nvl_model::windows
-    int64_t cache_off = 0;       // latent attention: element offset inside a cache block
+    int64_t cache_off = 0;       // attention: element offset inside a cache block
+    int k_off = 0, v_off = 0, route_off = 0;     // grouped attention: columns of the fused input projection (keys, values, router)
+    int mix = 0;                 // grouped attention: GroupedArgs::mix
+    int kd = 0;                  // K of the joint output projection of a parallel block: ko, then the feed-forward's Fp columns
+    int act = 0;                 // activation of the feed-forward
+    int Ep = 0, Ip = 0, moe_slices = 0;          // experts (padded), their padded width, K slices of the decode down projection
     int64_t state_off = 0, ring_off = 0;     // recurrent layers: float offsets inside a slot
 };
 // its frozen tensors (owners only)
@@ -76,6 +83,10 @@ struct MixerW {
     void *a2m = nullptr, *g2m = nullptr;     // channel delta: the second decay / gate projections as GEMM operands ...
     void *a2r = nullptr, *g2r = nullptr;     // ... and row-major for the one-token step
     int grank = 0, a_rkp = 0, g_rkp = 0;
+    float *norm1_bias = nullptr, *r1 = nullptr, *r2 = nullptr, *v_lambda = nullptr;       // grouped attention, parallel blocks
+    void *moe_up = nullptr, *moe_down = nullptr, *moe_cat = nullptr;                      // experts: [E][2 Ip][H], [E][H][Ip], bf16: [H][Ep Ip]
+    float* route_bias = nullptr;
+    void *side_gate = nullptr, *side_proj = nullptr; float* side_norm = nullptr;
 };
 
 struct ProfRec { hipEvent_t a, b; int cls; double flops; int site, phase; double bytes; };
@@ -154,7 +165,10 @@ struct nvl_model {
     std::vector<nvl::LayerRun> runs;
     std::vector<nvl::MixerW> mixers;
     std::vector<void*> layered_allocs;
-    float *final_norm = nullptr;
+    float *final_norm = nullptr, *final_norm_b = nullptr;
+    float* lvf = nullptr; int64_t lvf_ld = 0;                       // grouped attention: the first mixing layer's values of the running batch
+    void *side_emb = nullptr, *lside = nullptr; int64_t side_ld = 0; int side_kp = 0;     // per-layer token inputs: table (rows of L * side4 entries), operand of the projection
+    float* grp_part = nullptr; int32_t* grp_cnt = nullptr; int64_t grp_cap = 0;           // grouped attention: key splits
     std::vector<int> windows;    // distinct windows of the latent attention layers (0: none)
     void* lat_cache = nullptr; int64_t lat_block_stride = 0;
     float* rec_state = nullptr; int64_t rec_slot_stride = 0;
@@ -171,6 +185,7 @@ struct nvl_model {
     std::vector<int64_t> key_rows; std::vector<int> key_max;       // per window: rows of the key workspace, longest key list
     int n_abs = 0; bool meta_dynamic = false;                      // tokens on the absorbed form; launch shapes depend on positions
     int min_len = 1;
+    std::vector<std::array<double, 2>> win_pairs, win_keys;       // per window: visible pairs and keys read by sequences with [one, several] new tokens
 
     // workspaces
     float* x = nullptr;          // residual stream fp32 [Mmax][H]

@@ -120,7 +120,7 @@ bool is_1d(int kind) {
         default: return false;
     }
 }
-bool is_global(int kind) { return kind < NVL_T_ATTN_NORM_W; }
+bool is_global(int kind) { return kind < NVL_T_ATTN_NORM_W || kind == NVL_T_SIDE_EMB; }
 
 DevTensor* tensor_slot(nvl_model* m, int kind, int layer) {
     if (kind < 0 || kind >= NVL_T_COUNT) return nullptr;
@@ -195,6 +195,8 @@ void gemm(nvl_model* m, int epi, bool out_f32, GemmArgs a, double flops = -1.0) 
             case EPI_GEGLU:  launch_gemm_bf16<EPI_GEGLU, bf16_t>(st, a); break;
             case EPI_CLAMP_GLU: launch_gemm_bf16<EPI_CLAMP_GLU, bf16_t>(st, a); break;
             case EPI_QKV:    launch_gemm_bf16<EPI_QKV, bf16_t>(st, a); break;
+            case EPI_RELU2:  launch_gemm_bf16<EPI_RELU2, bf16_t>(st, a); break;
+            case EPI_GELU_TOK: launch_gemm_bf16<EPI_GELU_TOK, bf16_t>(st, a); break;
             default: throw std::runtime_error("gemm: bad epilogue");
         }
     }
@@ -1505,7 +1507,7 @@ void ffn_up(nvl_model* m, const LayerW& l, int M, bool deferred_norm = false) {
             KScope ks(m, KC_OTHER);
             const int64_t n = (int64_t)M * m->F;
             hipLaunchKernelGGL((swiglu_kernel<float>), dim3(cdiv(n, 256)), dim3(256), 0, m->stream, m->h2,
-                               (float*)m->hbuf, (int64_t)M, m->F);
+                               (float*)m->hbuf, (int64_t)M, m->F, (int64_t)m->F, 0);
             NVL_HIP(hipGetLastError());
         } else {
             GemmArgs a = mk(m->xn, m->H, l.w1, m->hbuf, m->F, nullptr, 1.f, M, 2 * m->F, m->H);
@@ -1523,6 +1525,71 @@ void ffn_up(nvl_model* m, const LayerW& l, int M, bool deferred_norm = false) {
 // the (token, rank) pairs by expert -> ONE grouped gate/up GEMM and ONE grouped down GEMM over all experts
 // (m-tiles mapped to (expert, row segment) by a device table; token rows gathered by per-lane source address)
 // -> combine in rank order into x (with the residual multiplier).  The fp32 parity mode launches per expert.
+// one layer's experts: E SwiGLU feed-forwards of width I, top k of them per token; [E][2I][H] and [E][H][I] in the kernels' layouts
+struct MoeW { int E, k, I; const void *up, *down; };
+// prefill default: 256-row m-tiles on the ping-pong kernel (needs the rows copied into expert order and K >= 160)
+bool moe_pp_ok(const nvl_model* m, int I, bool small) {
+    return !m->f32 && !small && g_moe_bm == 0 && m->moe_xg && g_moe_gather && m->H >= 160 && I >= 160 && (2 * I) % 256 == 0 && m->H % 256 == 0;
+}
+// the (token, rank) pairs in m->expert_ids into expert order
+void moe_sort(nvl_model* m, int E, int k, int M, int BM) {
+    const int pairs = M * k;
+    KScope ks(m, KC_OTHER, 0, KS_MOE_PLAN);
+    hipLaunchKernelGGL(fill_i32_kernel, dim3(cdiv(E, 256)), dim3(256), 0, m->stream, m->moe_counts, 0, E);     // (a captured pass must hold no memset node)
+    hipLaunchKernelGGL(moe_hist_kernel, dim3(cdiv(pairs, MOE_PAIRS_PER_WG)), dim3(256), 0, m->stream, m->expert_ids, pairs, m->moe_counts);
+    hipLaunchKernelGGL(moe_scan_kernel, dim3(1), dim3(64), 0, m->stream, m->moe_counts, E, BM, m->seg_start, m->moe_cursor,
+                       m->moe_tile_map, m->moe_n_mtiles);
+    hipLaunchKernelGGL(moe_scatter_kernel, dim3(cdiv(pairs, MOE_PAIRS_PER_WG)), dim3(256), 0, m->stream, m->expert_ids, pairs, k,
+                       m->moe_cursor, m->perm_token, m->slot_of);
+    NVL_HIP(hipGetLastError());
+}
+// the experts' feed-forwards over the sorted pairs: rows of m->xn -> m->moe_eo (pair order of m->slot_of)
+void moe_expert_gemms(nvl_model* m, const MoeW& w, int M, int BM, bool pp, bool small) {
+    const int E = w.E, k = w.k, I = w.I, H = m->H, pairs = M * k;
+    const double e_touch = (double)std::min(E, pairs);
+    const int max_mtiles = cdiv(pairs, BM) + E;      // every expert may end on a partial tile
+    if (m->f32) {
+        for (int e = 0; e < E; e++) {   // grid bounded by M: a token picks an expert at most once; surplus blocks exit
+            const char* win = (const char*)w.up + (size_t)e * 2 * I * H * m->wsize;
+            GemmArgs a = mk(m->xn, H, win, m->h2, 2 * I, nullptr, 1.f, M, 2 * I, H);
+            a.a_rows = m->perm_token; a.seg = m->seg_start + e;
+            gemm(m, EPI_STORE, true, a);
+        }
+        {
+            KScope ks(m, KC_OTHER);
+            const int64_t n = (int64_t)pairs * I;
+            hipLaunchKernelGGL((swiglu_kernel<float>), dim3(cdiv(n, 256)), dim3(256), 0, m->stream, m->h2, (float*)m->hbuf,
+                               (int64_t)pairs, I, (int64_t)I, 0);
+            NVL_HIP(hipGetLastError());
+        }
+        for (int e = 0; e < E; e++) {
+            const char* wout = (const char*)w.down + (size_t)e * H * I * m->wsize;
+            GemmArgs a = mk(m->hbuf, I, wout, m->moe_eo, H, nullptr, 1.f, M, H, I);
+            a.seg = m->seg_start + e;
+            gemm(m, EPI_STORE, true, a);
+        }
+        return;
+    }
+    GemmArgs a = mk(m->xn, H, w.up, m->hbuf, I, nullptr, 1.f, max_mtiles, 2 * I, H);
+    a.a_rows = m->perm_token; a.tile_map = m->moe_tile_map; a.n_mtiles = m->moe_n_mtiles;
+    if (!small && m->moe_xg && g_moe_gather) {
+        // prefill: every m-tile's rows would be re-gathered 16 bytes at a time by each of its 2I/128 column tiles
+        // (64 cache lines per load instruction); copy them into expert order once, then the GEMM streams whole
+        // 1-KiB operand blocks (Granite-1B, 16384 tokens: expert-up 1119 -> ? us per layer)
+        KScope ks(m, KC_OTHER);
+        hipLaunchKernelGGL(moe_gather_fm_kernel, dim3(cdiv(pairs, 16)), dim3(256), 0, m->stream, (const bf16_t*)m->xn,
+                           m->perm_token, (bf16_t*)m->moe_xg, pairs, H);
+        NVL_HIP(hipGetLastError());
+        a.A = m->moe_xg; a.a_rows = nullptr;
+    }
+    a.w_expert_stride = (int64_t)2 * I * H; a.grp_bm = pp ? 512 : BM; a.grp_deep = small && g_moe_deep;
+    m->site = KS_MOE_UP; m->site_bytes = (e_touch * 2 * I * H + (double)pairs * H + (double)pairs * I) * (double)m->wsize;
+    gemm(m, EPI_SWIGLU, false, a, 2.0 * pairs * 2 * I * H);
+    GemmArgs d = mk(m->hbuf, I, w.down, m->moe_eo, H, nullptr, 1.f, max_mtiles, H, I);
+    d.tile_map = m->moe_tile_map; d.n_mtiles = m->moe_n_mtiles; d.w_expert_stride = (int64_t)H * I; d.grp_bm = pp ? 512 : BM; d.grp_deep = small && g_moe_deep;
+    m->site = KS_MOE_DOWN; m->site_bytes = (e_touch * H * I + (double)pairs * I) * (double)m->wsize + (double)pairs * H * 4.0;
+    gemm(m, EPI_STORE, true, d, 2.0 * pairs * H * I);
+}
 // can this call take the decode ("dense-masked") MoE form?  (also decides whether the O projection may carry the FFN norm)
 bool moe_dense_ok(const nvl_model* m, const LayerW& l, int M) {
     return !m->f32 && M <= 64 && g_moe_dense && l.moe_out_cat && m->moe_part && !m->keep_hidden && m->H % 4 == 0 &&
@@ -1593,8 +1660,7 @@ bool moe(nvl_model* m, const LayerW& l, int M, bool deferred_norm = false, const
     const bool small = !m->f32 && M <= 64 && pairs <= MOE_PLAN_MAX_PAIRS && E <= MOE_PLAN_MAX_E && g_moe_small;
     // m-tile height of the grouped GEMMs: 128 rows; the 256x128 three-stage instance stays a tuning option (Granite-1B,
     // 4096 rows per expert: 441 K vs 450 K prefill tok/s)
-    // prefill default: 256-row m-tiles on the ping-pong kernel (needs the rows copied into expert order and K >= 160)
-    const bool pp = !m->f32 && !small && g_moe_bm == 0 && m->moe_xg && g_moe_gather && H >= 160 && I >= 160 && (2 * I) % 256 == 0 && H % 256 == 0;
+    const bool pp = moe_pp_ok(m, I, small);
     const int BM = pp ? 256 : ((!m->f32 && !small && g_moe_bm == 256) ? 256 : 128);
     if (small) {
         KScope ks(m, KC_OTHER, 0, KS_MOE_PLAN);
@@ -1602,59 +1668,15 @@ bool moe(nvl_model* m, const LayerW& l, int M, bool deferred_norm = false, const
                            m->expert_w, m->seg_start, m->moe_tile_map, m->moe_n_mtiles, m->perm_token, m->slot_of);
         NVL_HIP(hipGetLastError());
     } else {
-        KScope ks(m, KC_OTHER, 0, KS_MOE_PLAN);
-        hipLaunchKernelGGL(fill_i32_kernel, dim3(cdiv(E, 256)), dim3(256), 0, m->stream, m->moe_counts, 0, E);     // (a captured pass must hold no memset node)
-        hipLaunchKernelGGL(moe_route_kernel, dim3(cdiv(M, 4)), dim3(256), 0, m->stream, m->router_logits, 128, M, E, k,
-                           m->expert_ids, m->expert_w);
-        hipLaunchKernelGGL(moe_hist_kernel, dim3(cdiv(pairs, MOE_PAIRS_PER_WG)), dim3(256), 0, m->stream, m->expert_ids, pairs, m->moe_counts);
-        hipLaunchKernelGGL(moe_scan_kernel, dim3(1), dim3(64), 0, m->stream, m->moe_counts, E, BM, m->seg_start, m->moe_cursor,
-                           m->moe_tile_map, m->moe_n_mtiles);
-        hipLaunchKernelGGL(moe_scatter_kernel, dim3(cdiv(pairs, MOE_PAIRS_PER_WG)), dim3(256), 0, m->stream, m->expert_ids, pairs, k,
-                           m->moe_cursor, m->perm_token, m->slot_of);
-        NVL_HIP(hipGetLastError());
-    }
-    const int max_mtiles = cdiv(pairs, BM) + E;      // every expert may end on a partial tile
-    if (m->f32) {
-        for (int e = 0; e < E; e++) {   // grid bounded by M: a token picks an expert at most once; surplus blocks exit
-            const char* win = (const char*)l.moe_in + (size_t)e * 2 * I * H * m->wsize;
-            GemmArgs a = mk(m->xn, H, win, m->h2, 2 * I, nullptr, 1.f, M, 2 * I, H);
-            a.a_rows = m->perm_token; a.seg = m->seg_start + e;
-            gemm(m, EPI_STORE, true, a);
-        }
         {
-            KScope ks(m, KC_OTHER);
-            const int64_t n = (int64_t)pairs * I;
-            hipLaunchKernelGGL((swiglu_kernel<float>), dim3(cdiv(n, 256)), dim3(256), 0, m->stream, m->h2, (float*)m->hbuf,
-                               (int64_t)pairs, I);
+            KScope ks(m, KC_OTHER, 0, KS_MOE_PLAN);
+            hipLaunchKernelGGL(moe_route_kernel, dim3(cdiv(M, 4)), dim3(256), 0, m->stream, m->router_logits, 128, M, E, k,
+                               m->expert_ids, m->expert_w);
             NVL_HIP(hipGetLastError());
         }
-        for (int e = 0; e < E; e++) {
-            const char* wout = (const char*)l.t[NVL_T_MOE_OUT].p + (size_t)e * H * I * m->wsize;
-            GemmArgs a = mk(m->hbuf, I, wout, m->moe_eo, H, nullptr, 1.f, M, H, I);
-            a.seg = m->seg_start + e;
-            gemm(m, EPI_STORE, true, a);
-        }
-    } else {
-        GemmArgs a = mk(m->xn, H, l.moe_in, m->hbuf, I, nullptr, 1.f, max_mtiles, 2 * I, H);
-        a.a_rows = m->perm_token; a.tile_map = m->moe_tile_map; a.n_mtiles = m->moe_n_mtiles;
-        if (!small && m->moe_xg && g_moe_gather) {
-            // prefill: every m-tile's rows would be re-gathered 16 bytes at a time by each of its 2I/128 column tiles
-            // (64 cache lines per load instruction); copy them into expert order once, then the GEMM streams whole
-            // 1-KiB operand blocks (Granite-1B, 16384 tokens: expert-up 1119 -> ? us per layer)
-            KScope ks(m, KC_OTHER);
-            hipLaunchKernelGGL(moe_gather_fm_kernel, dim3(cdiv(pairs, 16)), dim3(256), 0, m->stream, (const bf16_t*)m->xn,
-                               m->perm_token, (bf16_t*)m->moe_xg, pairs, H);
-            NVL_HIP(hipGetLastError());
-            a.A = m->moe_xg; a.a_rows = nullptr;
-        }
-        a.w_expert_stride = (int64_t)2 * I * H; a.grp_bm = pp ? 512 : BM; a.grp_deep = small && g_moe_deep;
-        m->site = KS_MOE_UP; m->site_bytes = (e_touch * 2 * I * H + (double)pairs * H + (double)pairs * I) * (double)m->wsize;
-        gemm(m, EPI_SWIGLU, false, a, 2.0 * pairs * 2 * I * H);
-        GemmArgs d = mk(m->hbuf, I, l.t[NVL_T_MOE_OUT].p, m->moe_eo, H, nullptr, 1.f, max_mtiles, H, I);
-        d.tile_map = m->moe_tile_map; d.n_mtiles = m->moe_n_mtiles; d.w_expert_stride = (int64_t)H * I; d.grp_bm = pp ? 512 : BM; d.grp_deep = small && g_moe_deep;
-        m->site = KS_MOE_DOWN; m->site_bytes = (e_touch * H * I + (double)pairs * I) * (double)m->wsize + (double)pairs * H * 4.0;
-        gemm(m, EPI_STORE, true, d, 2.0 * pairs * H * I);
+        moe_sort(m, E, k, M, BM);
     }
+    moe_expert_gemms(m, MoeW{E, k, I, l.moe_in, l.t[NVL_T_MOE_OUT].p}, M, BM, pp, small);
     if (small && !m->keep_hidden && m->pending_slices == 0 && H % 4 == 0 && H <= 1024 * NORM_ROW_MAXCH) {
         // x += rm * sum_k w[t][k] * eo[slot[t][k]] is completed by the next norm's read of x (PendingResid)
         m->pending_part = m->moe_eo; m->pending_slices = k; m->pending_rows = M; m->pending_alpha = c.residual_multiplier;
@@ -1957,7 +1979,7 @@ int enqueue_forward(nvl_model* m, const Meta& md, int n_seqs, int M, int max_len
         m->site = KS_LM_HEAD;
         gemm(m, EPI_STORE, true, al);
     } else if (m->layered) {
-        if (!xn_final) sandwich(m, nullptr, 0, 0, nullptr, m->final_norm, all ? nullptr : md.last_rows, m->xn_last, rows);
+        if (!xn_final) sandwich(m, SubOut{}, nullptr, {m->final_norm, m->final_norm_b, false}, m->xn_last, rows, all ? nullptr : md.last_rows);
         m->site = KS_LM_HEAD;
         gemm(m, EPI_STORE, true, mk(xn_final ? m->xn : m->xn_last, H, m->lm_head, m->logits, m->Vpad, nullptr, 1.f, rows, m->V, H));
     } else {
@@ -2343,7 +2365,7 @@ void decode_loop(nvl_model* m, const Meta& hm, int n_seqs, int n_steps, int32_t*
             const void* pe = (m->cfg.position_type == NVL_POS_LEARNED) ? m->g[NVL_T_POS_EMB].p : nullptr;
             const int pe_rows = pe ? (int)std::min<int64_t>(m->g[NVL_T_POS_EMB].rows, m->cfg.max_seq_len) : 0;
             const float* norm0 = m->layered ? m->mixers[(size_t)m->runs[0].owner].norm1 : (const float*)m->layers[0].t[NVL_T_ATTN_NORM_W].p;
-            const float* bias0 = m->layered ? nullptr : (const float*)m->layers[0].t[NVL_T_ATTN_NORM_B].p;
+            const float* bias0 = m->layered ? m->mixers[(size_t)m->runs[0].owner].norm1_bias : (const float*)m->layers[0].t[NVL_T_ATTN_NORM_B].p;
             hipLaunchKernelGGL(decode_seam_kernel, dim3(n_seqs), dim3(256), 0, m->stream, m->argmax_pval, m->argmax_pidx,
                                cdiv(m->V, ARGMAX_CHUNK), sp ? (const int32_t*)m->samp.out : (const int32_t*)nullptr, m->samp_hist,
                                (int64_t)m->cfg.max_seq_len, m->samp_hist_len, m->argmax_dev, m->ring, (const int32_t*)m->ring_pos0, n_seqs,
@@ -2713,7 +2735,8 @@ static const char* const k_site_names[KS_COUNT] = {
     "other", "qkv_proj", "attention", "o_proj", "ffn_up", "ffn_down", "lm_head", "norm", "moe_router", "moe_plan", "moe_up",
     "moe_down", "moe_combine", "embed", "argmax", "rope_kv", "mamba_in_proj", "mamba_conv", "mamba_scan", "mamba_gate_norm",
     "mamba_out_proj", "tp_allreduce", "mix_in_proj", "latent_norm", "latent_uq", "latent_gather", "latent_kv", "latent_absorb_q",
-    "latent_uv", "gla_scan", "gla_gate_norm", "sandwich_norm", "delta_conv", "delta_pack", "delta_rank_out", "delta_prep", "delta_scan", "delta_gate_norm"};
+    "latent_uv", "gla_scan", "gla_gate_norm", "sandwich_norm", "delta_conv", "delta_pack", "delta_rank_out", "delta_prep", "delta_scan", "delta_gate_norm",
+    "kv_place", "side_gate", "side_proj"};
 extern "C" const char* nvl_kernel_site_name(int site) { return site >= 0 && site < KS_COUNT ? k_site_names[site] : ""; }
 extern "C" int nvl_get_kernel_stats(nvl_model* m, nvl_kernel_stat* out, int cap) {
     if (!m || (cap > 0 && !out)) return NVL_ERR_INVALID;

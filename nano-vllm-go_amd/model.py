@@ -13,7 +13,7 @@ from . import _lib as L
 def _cfg_struct(cfg: dict) -> L.ModelConfigC:
     c = L.ModelConfigC()
     for k in ("vocab_size", "hidden", "num_layers", "num_heads", "num_kv_heads", "head_dim", "ffn_dim",
-              "max_seq_len", "num_experts", "num_experts_per_tok"):
+              "max_seq_len", "num_experts", "num_experts_per_tok", "side_dim"):
         setattr(c, k, int(cfg.get(k, 0)))
     c.attention_type = L.ATTN[cfg["attention_type"]]
     c.norm_type = L.NORM[cfg["norm_type"]]
@@ -111,8 +111,8 @@ class HipTransformerModel:
             L.check(L.lib().nvl_load_layers_json(cp.encode(), arr, n))
             names = {v: k for k, v in L.MIXER.items()}
             cfg["layers"] = [{k: names[getattr(a, k)] if k == "mixer" else getattr(a, k) for k, _ in a._fields_} for a in arr]
-        if max_seq_len is not None:
-            cfg["max_seq_len"] = int(max_seq_len)
+        if max_seq_len is not None:      # (a list of layers with learned positions: as far as those reach)
+            cfg["max_seq_len"] = min(int(max_seq_len), cfg["max_seq_len"]) if n and cfg["position_type"] == "learned" else int(max_seq_len)
         m = cls(cfg, None, **kw)
         L.check(m.lib.nvl_load_safetensors(m.h, path.encode()), m.h)
         m.finalize()
@@ -158,7 +158,7 @@ class HipTransformerModel:
         ptr, dtype, shape, keep = _as_pointer(arr)
         if slot in L.ONE_D:
             rows, cols = int(np.prod(shape)), 1
-        elif slot in ("moe_in", "moe_out"):
+        elif slot in ("moe_in", "moe_out") and len(shape) == 3:
             rows, cols = shape[0] * shape[1], shape[2]
         else:
             rows, cols = shape
