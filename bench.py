@@ -38,8 +38,8 @@ def parse():
     ap.add_argument("--gpus", type=int, default=1)
     ap.add_argument("--steps", type=int, default=3)
     ap.add_argument("--warmup", type=int, default=1)
-    ap.add_argument("--model", default="llama-3.2-1b", help="a synth.FULL_CONFIGS key; lufazen-2k / -4k and potuzen-2k / -4k are those designs at a real "
-                    "model's layer sizes, hybrid-2k / hybrid-4k the attention + Mamba-2 family at the same sizes")
+    ap.add_argument("--model", default="llama-3.2-1b", help="a synth.FULL_CONFIGS key; bolinex-2k / -4k, lufazen-2k / -4k and potuzen-2k / -4k are those designs at a real "
+                    "model's layer sizes, hybrid-2k / hybrid-4k the attention + Mamba-2 family at the same sizes, gqa[-moe]-2k / -4k the grouped-query attention families")
     ap.add_argument("--batch", type=int, default=32, help="sequences per GPU")
     ap.add_argument("--prompt", type=int, default=512, help="prompt tokens per sequence")
     ap.add_argument("--gen", type=int, default=128, help="decode steps per sequence")
@@ -85,7 +85,7 @@ def gen_weights_on_device(pkg, cfg, model, torch, device, keep_host: bool):
             t = torch.randn(*shape, device=device, generator=g)
             u = torch.rand(*shape, device=device, generator=g)
             t = {"matrix": lambda: t * shape[-1] ** -0.5, "norm": lambda: 1 + 0.02 * t, "norm0": lambda: 0.02 * t, "conv": lambda: 0.3 * t, "bias": lambda: 0.5 * t,
-                 "dt_bias": lambda: 3.5 * u - 3, "a_log": lambda: torch.log(1 + 7 * u)}[kind]()
+                 "dt_bias": lambda: 3.5 * u - 3, "decay": lambda: 0.5 * u, "a_log": lambda: torch.log(1 + 7 * u)}[kind]()
             model.upload(slot, layer, t.to(torch.bfloat16))
         return host
 
@@ -169,7 +169,9 @@ def flops_per_token(cfg):
     if cfg.get("layers"):
         from importlib import import_module
         shapes = import_module("nano-vllm-go_amd").synth.layered_shapes(cfg)
-        return 2.0 * sum(s[0] * s[1] for slot, _, s, _ in shapes if len(s) == 2 and slot not in ("tok_emb", "lm_head")), 2.0 * H * V
+        used = {i: c["top_k"] / c["experts"] for i, c in enumerate(cfg["layers"]) if c["experts"]}      # share of a layer's experts a token runs
+        return 2.0 * sum(s[0] * s[1] * (used[i] if slot in ("moe_in", "moe_out") else 1.0) for slot, i, s, _ in shapes
+                         if len(s) == 2 and slot not in ("tok_emb", "lm_head", "pos_emb", "side_emb")), 2.0 * H * V
     if cfg.get("hybrid_layers"):
         EH = cfg["mamba_expand"] * H
         n_m = sum(t.startswith("mamba") for t in cfg["hybrid_layers"])
@@ -338,12 +340,14 @@ def main():
     at = cfg["attention_type"]
     nKV = cfg["num_heads"] if at == "mha" else (1 if at == "mqa" else cfg["num_kv_heads"])
     kv_bytes = 2 * cfg["num_layers"] * nKV * cfg["head_dim"] * (S + G / 2) * 2 * B
+    if cfg.get("layers") and any(c["experts"] for c in cfg["layers"]):      # every expert a batch can touch, not a token's share
+        wbytes += (2 if args.precision == "bf16" else 4) * sum((min(c["experts"], B * c["top_k"]) - c["top_k"]) * 3 * cfg["hidden"] * c["expert_dim"] for c in cfg["layers"] if c["experts"])
     if cfg.get("hybrid_layers"):      # attention layers' K/V once, the Mamba-2 layers' fp32 states read and written
         n_m = sum(t.startswith("mamba") for t in cfg["hybrid_layers"])
         kv_bytes *= 1 - n_m / cfg["num_layers"]
         kv_bytes += n_m * B * 8.0 * cfg["mamba_expand"] * cfg["hidden"] * cfg["mamba_state_size"]
-    if cfg.get("layers"):             # cached latents once, fp32 states read and written
-        kv_bytes = sum(B * (2.0 * c["kv_rank"] * min(c["window"] or 1 << 30, S + G / 2) if c["mixer"] == "latent_attention" else
+    if cfg.get("layers"):             # cached latents (keys and values) once, fp32 states read and written
+        kv_bytes = sum(B * (2.0 * c["kv_heads"] * (c["dim"] + c["vdim"]) * min(c["window"] or 1 << 30, S + G / 2) if c["mixer"] == "attention" else 2.0 * c["kv_rank"] * min(c["window"] or 1 << 30, S + G / 2) if c["mixer"] == "latent_attention" else
                             8.0 * c["heads"] * c["vdim"] * (c["state"] or c["dim"])) for c in cfg["layers"])
     dec_gbs = (wbytes + kv_bytes) * G * args.steps / dec_s / 1e9
 

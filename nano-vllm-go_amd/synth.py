@@ -137,23 +137,36 @@ def tiny_config(family: str, **over) -> dict:
 
 def layered_shapes(cfg: dict, decay_rank: int = 16) -> list:
     """[(slot, layer, shape, kind)] of every tensor of a model described by a list of layers (cfg["layers"]: config.LAYER_FIELDS
-    dicts); kind: matrix | norm | norm0 (kept as a difference from one) | conv | bias | dt_bias | a_log — how a synthetic checkpoint
+    dicts); kind: matrix | norm | norm0 (kept as a difference from one) | conv | bias | dt_bias | a_log | decay (0 .. 0.5) — how a synthetic checkpoint
     should draw it.  decay_rank: of the low-rank decay (and gate) projections whose rank the configuration leaves open."""
-    H, V, post = cfg["hidden"], cfg["vocab_size"], cfg["block_style"] == "post"
+    H, V, post, par, side = cfg["hidden"], cfg["vocab_size"], cfg["block_style"] == "post", cfg["block_style"] == "parallel", cfg.get("side_dim", 0)
+    ln = cfg["norm_type"] == "layernorm"
     norm = "norm0" if cfg.get("norm_weight_offset") else "norm"
     out = [("tok_emb", 0, (V, H), "matrix"), ("lm_head", 0, (V, H), "matrix"), ("final_norm_w", 0, (H,), norm)]
+    if ln:
+        out.append(("final_norm_b", 0, (H,), "bias"))
+    if cfg["position_type"] == "learned":
+        out.append(("pos_emb", 0, (cfg["max_seq_len"], H), "matrix"))
+    if side:
+        out.append(("side_emb", 0, (V, len(cfg["layers"]) * side), "matrix"))
     for i, c in enumerate(cfg["layers"]):
         if c["weights_of"] >= 0:
             continue
         h, d, dv = c["heads"], c["dim"], c["vdim"]
         t = [("mix_scale", (H,), "norm")] if post else [("attn_norm_w", (H,), norm)]
-        t += [("mix_post_norm", (H,), norm)]
+        t += [("attn_norm_b", (H,), "bias")] if ln else []
+        t += [] if par else [("mix_post_norm", (H,), norm)]
+        t += [("side_gate", (side, H), "matrix"), ("side_proj", (H, side), "matrix"), ("side_norm", (H,), "norm")] if side else []
         if c["mixer"] == "latent_attention":
             qr, kr, rot = c["q_rank"], c["kv_rank"], c["rot_dim"]
             t += [("lat_dq", (qr, H), "matrix"), ("lat_dq_norm", (qr,), "norm"), ("lat_uq", (h * (d + rot), qr), "matrix"), ("lat_uk", (h * d, kr), "matrix"),
                   ("lat_uv", (h * dv, kr), "matrix"), ("mix_gate", (h if c["gate_per_head"] else h * dv, H), "matrix"), ("wo", (H, h * dv), "matrix")]
             if c["kv_from"] < 0:
                 t += [("lat_dkv", (kr + rot, H), "matrix"), ("lat_dkv_norm", (kr,), "norm")]
+        elif c["mixer"] == "attention":
+            g = c["kv_heads"]
+            t += [("wq", (h * d, H), "matrix"), ("wk", (g * d, H), "matrix"), ("wv", (g * dv, H), "matrix"), ("mix_gate", (h * dv, H), "matrix"),
+                  ("wo", (H, h * dv), "matrix"), ("bias_r1", (h,), "norm"), ("bias_r2", (h,), "decay")] + ([("v_mix", (1,), "decay")] if c["v_mix"] else [])
         elif c["mixer"] == "channel_delta":
             qk, r = c["kv_heads"] * d, c["decay_rank"] or decay_rank
             t += [("wq", (qk, H), "matrix"), ("wk", (qk, H), "matrix"), ("wv", (h * dv, H), "matrix"), ("wo", (H, h * dv), "matrix"),
@@ -169,7 +182,13 @@ def layered_shapes(cfg: dict, decay_rank: int = 16) -> list:
             t += [("wq", (h * d, H), "matrix"), ("wk", (h * d, H), "matrix"), ("wv", (h * dv, H), "matrix"), ("mix_gate", (h * dv, H), "matrix"),
                   ("wo", (H, h * dv), "matrix"), ("gla_norm", (dv,), "norm"), ("gla_a1", (decay_rank, H), "matrix"),
                   ("gla_a2", (h * d, decay_rank), "matrix"), ("gla_a2_b", (h * d,), "bias")]
-        if c["ffn_dim"]:
+        if c["experts"]:
+            E, I = c["experts"], c["expert_dim"]
+            t += [("router", (E, H), "matrix"), ("router_bias", (E,), "bias"), ("moe_in", (E * 2 * I, H), "matrix"), ("moe_out", (E * H, I), "matrix")]
+        if c["ffn_dim"] and par:
+            F, gated = c["ffn_dim"], c["ffn_act"] != 0 or cfg["activation_type"] != "relu2"      # (a layer's own activation here: SwiGLU)
+            t += [("w1", ((2 if gated else 1) * F, H), "matrix"), ("w2", (H, F), "matrix")]
+        elif c["ffn_dim"]:
             F = c["ffn_dim"]
             t += [("ffn_scale", (H,), "norm")] if post else [("ffn_norm_w", (H,), norm)]
             t += [("ffn_post_norm", (H,), norm), ("w1", (2 * F, H), "matrix"), ("w2", (H, F), "matrix")]
@@ -202,6 +221,23 @@ def _lufazen(width: int, layers: int, heads: int, q_rank: int, ff: int) -> dict:
     return dict(vocab_size=32000, hidden=width, num_layers=layers, num_heads=0, num_kv_heads=0, head_dim=0, ffn_dim=0, max_seq_len=4096,
                 attention_type="gqa", norm_type="rmsnorm", position_type="nope", activation_type="clamped_glu", block_style="post",
                 rope_base=0.0, norm_eps=1e-5, tied_embedding=False, norm_weight_offset=1.0, logit_softcap=30.0, layers=ls)
+
+
+def _bolinex(width: int, layers: int, heads: int, ff: int, expert_ff: int, window: int = 1024) -> dict:
+    """A Bolinex model at a real model's layer sizes: grouped attention with a window, dense and expert feed-forwards in turn."""
+    from .config import ACT_SWIGLU, LAYER_FIELDS
+    att = dict(mixer="attention", heads=heads, kv_heads=heads // 4, dim=128, vdim=128, window=window, scale=128 ** -0.5, softcap=30.0, v_mix=1)
+    kinds = [dict(ffn_dim=ff), dict(ffn_dim=expert_ff, ffn_act=ACT_SWIGLU, experts=32, top_k=8, expert_dim=expert_ff, expert_groups=8, groups_kept=4)]
+    return dict(vocab_size=32000, hidden=width, num_layers=layers, num_heads=0, num_kv_heads=0, head_dim=0, ffn_dim=0, max_seq_len=4096,
+                attention_type="gqa", norm_type="layernorm", position_type="learned", activation_type="relu2", block_style="parallel",
+                rope_base=0.0, norm_eps=1e-6, tied_embedding=False, side_dim=256, layers=[dict(LAYER_FIELDS, **att, **kinds[i % 2]) for i in range(layers)])
+
+
+def _gqa(hidden: int, layers: int, heads: int, ff: int, experts: bool = False) -> dict:
+    """The grouped-query attention families at the same sizes: dense feed-forwards (Llama), or 32 experts of which a token takes 8 (Granite)."""
+    return dict(vocab_size=32000, hidden=hidden, num_layers=layers, num_heads=heads, num_kv_heads=heads // 4, head_dim=128, ffn_dim=ff, max_seq_len=4096,
+                attention_type="gqa", norm_type="rmsnorm", position_type="rope", activation_type="swiglu", block_style="sequential", norm_eps=1e-6,
+                tied_embedding=False, **(dict(use_moe=True, num_experts=32, num_experts_per_tok=8) if experts else {}))
 
 
 def _hybrid(hidden: int, layers: int, heads: int, ff: int) -> dict:
@@ -238,6 +274,8 @@ FULL_CONFIGS = {
                        position_type="rope", activation_type="swiglu", block_style="sequential",
                        rope_base=500000.0, norm_eps=1e-5, tied_embedding=False),
     # designs described by a list of layers at a real model's layer sizes, and the closest other family at the same sizes
+    "bolinex-2k": _bolinex(2048, 12, 16, 6144, 512), "bolinex-4k": _bolinex(4096, 6, 32, 12288, 1024),
+    "gqa-2k": _gqa(2048, 12, 16, 6144), "gqa-moe-2k": _gqa(2048, 12, 16, 512, True), "gqa-4k": _gqa(4096, 6, 32, 12288), "gqa-moe-4k": _gqa(4096, 6, 32, 1024, True),
     "lufazen-2k": _lufazen(2048, 12, 16, 768, 6144), "lufazen-4k": _lufazen(4096, 6, 32, 1536, 12288),
     "potuzen-2k": _potuzen(2048, 12, 16, 768, 6144), "hybrid-2k": _hybrid(2048, 12, 16, 6144),
     "potuzen-4k": _potuzen(4096, 6, 32, 1536, 12288), "hybrid-4k": _hybrid(4096, 6, 32, 12288),

@@ -75,30 +75,43 @@ def gated_ff(h, w, name):
     return (silu(h @ w[name + ".gate"].T) * (h @ w[name + ".up"].T)) @ w[name + ".down"].T
 
 
+def group_scores(choice, groups):
+    return np.sort(choice.reshape(groups["count"], -1), axis=1)[:, -2:].sum(axis=1)
+
+
 def choose(choice, router):
-    """The chosen experts of one token."""
+    """The chosen experts of one token, best first, and how close the call was (the smallest gap that decided something)."""
     gr, E = router.get("groups"), router["experts"]
-    ok = np.ones(E, bool)
+    ok, gap = np.ones(E, bool), np.inf
     if gr is not None:
-        by_group = choice.reshape(gr["count"], -1)
-        score = np.sort(by_group, axis=1)[:, -2:].sum(axis=1)
-        ok = np.repeat(np.isin(np.arange(gr["count"]), np.argsort(-score, kind="stable")[:gr["keep"]]), E // gr["count"])
-    return np.argsort(-np.where(ok, choice, -np.inf), kind="stable")[:router["top"]]
+        score = group_scores(choice, gr)
+        order = np.argsort(-score, kind="stable")
+        ok = np.repeat(np.isin(np.arange(gr["count"]), order[:gr["keep"]]), E // gr["count"])
+        if gr["keep"] < gr["count"]:
+            gap = score[order[gr["keep"] - 1]] - score[order[gr["keep"]]]
+    c = np.where(ok, choice, -np.inf)
+    order = np.argsort(-c, kind="stable")
+    if router["top"] < ok.sum():
+        gap = min(gap, c[order[router["top"] - 1]] - c[order[router["top"]]])
+    return order[:router["top"]], gap
 
 
-def experts(h, w, mlp):
+def experts(h, w, mlp, margins=None):
     s = sigmoid(h @ w["router"].T)
-    out = np.zeros_like(h)
+    out, gaps = np.zeros_like(h), np.empty(h.shape[0])
     for t in range(h.shape[0]):
-        for e in choose(s[t] + w["correction"], mlp["router"]):
+        chosen, gaps[t] = choose(s[t] + w["correction"], mlp["router"])
+        for e in chosen:
             out[t] += s[t, e] * gated_ff(h[t], w, f"e{e}")
+    if margins is not None:
+        margins.append(gaps)
     return out if mlp.get("shared") is None else out + gated_ff(h, w, "shared")
 
 
-def feed_forward(h, w, mlp):
+def feed_forward(h, w, mlp, margins=None):
     if mlp is None:
         return 0.0
-    return squared_relu_ff(h, w["up"], w["down"]) if mlp["kind"] == "dense" else experts(h, w, mlp)
+    return squared_relu_ff(h, w["up"], w["down"]) if mlp["kind"] == "dense" else experts(h, w, mlp, margins)
 
 
 def token_side(x, e, w, eps):
@@ -109,8 +122,9 @@ def sub(weights, prefix):
     return {k[len(prefix):]: np.asarray(v, np.float64) for k, v in weights.items() if k.startswith(prefix)}
 
 
-def forward(cfg, weights, tokens, return_layers=False):
-    """Logits [T, vocab] of one sequence (and the residual stream after every layer [layers, T, width])."""
+def forward(cfg, weights, tokens, return_layers=False, margins=None):
+    """Logits [T, vocab] of one sequence (and the residual stream after every layer [layers, T, width]).  margins: a list that gets, for
+    every layer with experts, how close each token's choice was."""
     eps, tok = cfg["norm"]["eps"], np.asarray(tokens)
     x = np.asarray(weights["embed"], np.float64)[tok] + np.asarray(weights["pos"], np.float64)[:len(tok)]
     layers, first = [], None
@@ -120,7 +134,7 @@ def forward(cfg, weights, tokens, return_layers=False):
         y, v = attention(h, sub(weights, f"l{i}.mix."), ly["mixer"], first)
         if ly["mixer"].get("v_mix") and first is None:
             first = v
-        x = x + (y + feed_forward(h, sub(weights, f"l{i}.mlp."), ly["mlp"]))
+        x = x + (y + feed_forward(h, sub(weights, f"l{i}.mlp."), ly["mlp"], margins))
         n = cfg["token_side"]["dim"]
         x = x + token_side(x, np.asarray(weights["side.embed"], np.float64)[tok, i * n:(i + 1) * n], sub(weights, f"l{i}.side."), eps)
         layers.append(x)
