@@ -69,6 +69,14 @@ __device__ __forceinline__ void kv_locate(const int32_t* __restrict__ blk_table,
     row = pos - bi * bs;
 }
 
+// Grouped-query attention of models described by a list of layers (grouped.h) keeps keys as MFMA operand blocks whose rows are in the
+// order that makes the score accumulators the next product's operand: tile row 16 t + 4 a + r holds token 8 a + 4 t + r of its
+// 32-token unit.  Where token row `row` sits:
+__host__ __device__ __forceinline__ int grouped_k_row(int row) {
+    const int k = row & 31;
+    return (row & ~31) + 16 * ((k >> 2) & 1) + 4 * (k >> 3) + (k & 3);
+}
+
 __device__ __forceinline__ float gelu_tanh_f(float x) {
     // tensor.go:181-190: 0.5 x (1 + tanh(sqrt(2/pi) (x + 0.044715 x^3))), the tanh in float64 there.
     // tanh(u) = 1 - 2 / (exp(2u) + 1) on the hardware exp2 / rcp (both ~1 ulp): ABSOLUTE error ~1e-7, and only the absolute

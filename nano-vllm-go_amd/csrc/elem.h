@@ -627,13 +627,13 @@ __global__ void clamp_glu_kernel(const float* __restrict__ h, ActT* __restrict__
     const int64_t r = i / F; const int f = (int)(i - r * F);
     ActIO<ActT>::st(y + i, clamp_glu_f(h[r * 2 * F + f], h[r * 2 * F + F + f], limit, slope));
 }
-// h [rows][F] -> y [rows][ld] at column col: max(h, 0)^2
+// h [rows][F] (h_ld apart) -> y [rows][ld] at column col: max(h, 0)^2
 template <typename ActT>
-__global__ void relu2_kernel(const float* __restrict__ h, ActT* __restrict__ y, int64_t rows, int F, int64_t ld, int col) {
+__global__ void relu2_kernel(const float* __restrict__ h, int64_t h_ld, ActT* __restrict__ y, int64_t rows, int F, int64_t ld, int col) {
     const int64_t i = (int64_t)blockIdx.x * blockDim.x + threadIdx.x;
     if (i >= rows * F) return;
     const int64_t r = i / F; const int f = (int)(i - r * F);
-    const float v = fmaxf(h[i], 0.f);
+    const float v = fmaxf(h[r * h_ld + f], 0.f);
     ActIO<ActT>::st(y + act_index<ActT>(r, col + f, ld), v * v);
 }
 // h [rows][n] -> y [rows][ld]: gelu_tanh(h) * (the token's row of a table)

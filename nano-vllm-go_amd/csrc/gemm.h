@@ -42,6 +42,7 @@ enum GemmEpi {
     EPI_CLAMP_GLU = 6,   // C[m, f] = g sigmoid(slope g) (u + 1), g = min(gate, limit), u = clamp(up, -limit, limit); W as for EPI_SWIGLU
     EPI_GEGLU = 5,   // C[m, f] = gelu_tanh(gate) * up   W rows interleaved as for EPI_SWIGLU
     EPI_RELU2 = 7,   // C = max(acc, 0)^2
+    EPI_GROUPED = 9,     // fused input projection of grouped-query attention (grouped.h): every column range goes where it is used, GroupedEpi
     EPI_GELU_TOK = 8,    // C[m, n] = gelu_tanh(acc) * tok_table[tok_ids[m]][n]   (an input of the token's own, GemmArgs::tok_*)
 };
 
@@ -58,6 +59,16 @@ struct QkvEpi {             // EPI_QKV only
     bf16_t* vcache;
     int64_t slot_stride;
     int Tmax, nH, nKV, hd;
+};
+
+struct GroupedEpi {         // EPI_GROUPED: columns [q | k | v | gate | feed-forward | router], each range ending at a multiple of 32 (all but the last)
+    int k0, v0, gate0, ffn0, route0;
+    // q and gate -> C, side by side (ldc columns, fragment-major); keys and values -> their cache rows
+    const int32_t *tok_pos, *tok_tbl, *blk_table;
+    bf16_t* cache; int64_t block_stride; int bs, G, dp, vp;        // this layer's part of block 0 (grouped.h)
+    int mix; const float* lambda; float* vfirst; int64_t vfirst_ld;
+    bf16_t* ffn; int64_t ffn_ld;                                   // max(., 0)^2 -> the output projection's operand (fragment-major, shifted to its columns)
+    float* route; int64_t route_ld;                                // fp32 rows
 };
 
 struct GemmArgs {
@@ -85,6 +96,7 @@ struct GemmArgs {
     int grp_bm;             // rows per m-tile of the grouped launch (128, or 256: the 256x128 three-stage instance)
     int grp_deep;           // grouped launch on the four-stage 128x128 instance (decode-sized MoE batches)
     QkvEpi qkv;             // EPI_QKV
+    GroupedEpi grp;         // EPI_GROUPED
     // decode kernel, EPI_RESID only: K split over gridDim.y = sk_slices workgroups per column block.  Each
     // writes its fp32 partial tile to sk_part[slice][m][n] (ld = N) with plain stores; the NEXT kernel in the
     // stream — the norm that follows every residual add — folds x += alpha * sum(slices) into its read of x.
@@ -127,6 +139,42 @@ __device__ __forceinline__ bool moe_expert_live(const GemmArgs& p, int e) {
     return __any(g != 0.f);
 }
 
+// four columns n .. n + 3 of token `row`, inside one column range
+__device__ __forceinline__ void epilogue_grouped4(const GemmArgs& p, int64_t row, int n, f32x4 v) {
+    const GroupedEpi& e = p.grp;
+    if (n < e.k0) { act_store4<bf16_t>((bf16_t*)p.C, row, n, p.ldc, v); return; }
+    if (n >= e.route0) {
+        float* c = e.route + row * e.route_ld + (n - e.route0);
+#pragma unroll
+        for (int r = 0; r < 4; r++) if (n + r < p.N) c[r] = v[r];
+        return;
+    }
+    if (n >= e.ffn0) {
+#pragma unroll
+        for (int r = 0; r < 4; r++) { const float t = fmaxf(v[r], 0.f); v[r] = t * t; }
+        act_store4<bf16_t>(e.ffn, row, n - e.ffn0, e.ffn_ld, v);
+        return;
+    }
+    if (n >= e.gate0) { act_store4<bf16_t>((bf16_t*)p.C, row, e.k0 + n - e.gate0, p.ldc, v); return; }
+    int blk, crow;
+    kv_locate(e.blk_table, e.tok_tbl[row], e.tok_pos[row], e.bs, blk, crow);
+    bf16_t* base = e.cache + (int64_t)blk * e.block_stride;
+    if (n < e.v0) {
+        const int c = n - e.k0, g = c / e.dp;
+        act_store4<bf16_t>(base + (int64_t)g * e.bs * e.dp, grouped_k_row(crow), c - g * e.dp, e.dp, v);
+        return;
+    }
+    const int c = n - e.v0, g = c / e.vp;
+    if (e.mix) {
+        f32x4* f = (f32x4*)(e.vfirst + row * e.vfirst_ld + c);
+        if (e.mix == 1) *f = v;
+        else { const float lam = *e.lambda; v = (1.0f - lam) * v + lam * *f; }
+    }
+    bf16_t* d = base + (int64_t)e.G * e.bs * e.dp + (int64_t)g * e.bs * e.vp + fm_index(c - g * e.vp, crow, e.bs);      // (transposed: neighbouring channels are 8 apart)
+#pragma unroll
+    for (int r = 0; r < 4; r++) d[8 * r] = (bf16_t)v[r];
+}
+
 __device__ __forceinline__ float silu_f(float g) { return g / (1.0f + __expf(-g)); }
 __device__ __forceinline__ float deferred_rstd(const GemmArgs& p, int m);
 
@@ -152,6 +200,7 @@ __device__ __forceinline__ void epilogue4(const GemmArgs& p, int m, int n, f32x4
         for (int r = 0; r < 4; r++) { const float t = fmaxf(v[r], 0.f); v[r] = t * t; }
     }
     const int64_t row = (int64_t)p.c_row0 + m;
+    if (EPI == EPI_GROUPED) { epilogue_grouped4(p, row, n, v); return; }
     if (EPI == EPI_GELU_TOK) {
         const bf16x4 e = *(const bf16x4*)(p.tok_table + (int64_t)p.tok_ids[row] * p.tok_ld + n);
 #pragma unroll
@@ -1300,7 +1349,7 @@ static inline bool launch_gemm_skinny_bf16(hipStream_t st, const GemmArgs& a0) {
     if (skinny_rows(a0) > 64 || a0.a_rows || a0.seg || a0.tile_map) return false;
     GemmArgs a = a0;
     a.x_mask = (g_x_mask && a0.M % 16 != 0) ? 1 : 0;     // padded rows of the last 16-row activation tile are not fetched
-    if constexpr (epi_glu(EPI) || EPI == EPI_STORE || EPI == EPI_GELU || EPI == EPI_RELU2) {
+    if constexpr (epi_glu(EPI) || EPI == EPI_STORE || EPI == EPI_GELU || EPI == EPI_RELU2 || EPI == EPI_GROUPED) {
         // wide-N form once its 64-row groups fill the chip (g_force_ntw: 8 forces it, 1/2/4 force the narrow form)
         const bool wide_ok = skinny_rows(a) > 16 && cdiv(a.N, 64) >= 256 && !a.sk_part;   // M <= 16: the narrow form streams as fast
         if (g_force_ntw == 8 || (g_force_ntw == 0 && wide_ok)) { if (launch_gemm_skinny_wide<EPI, OutT>(st, a)) return true; }

@@ -27,8 +27,10 @@ struct GroupedArgs {
     int window;                                   // 0: every earlier token
     float scale, softcap;                         // softcap 0: none
     const float *r1, *r2;                         // [H] or NULL: no distance bias
-    const float* proj; int64_t proj_ld;           // [token][q : H dp | k : G dp | v : G vp | gate : H vp | ...] of the fused input projection
-    int k_off, v_off, gate_off;                   // gate_off < 0: no output gate
+    const void* q; int64_t q_ld;                  // queries of head h at column h dp, its gate at column gate_col + h vp: bf16 (fragment-major) or the fp32 rows of proj
+    int gate_col;
+    const float* proj; int64_t proj_ld;           // fp32 mode: [token][q : H dp | k : G dp | v : G vp | gate : H vp | ...] of the fused input projection
+    int k_off, v_off;
     int mix;                                      // values: 0 as they are, 1 also the model's first (kept in vfirst), 2 mixed with vfirst
     const float* lambda; float* vfirst; int64_t vfirst_ld;      // [token][G vp]
     void* cache; int64_t block_stride; int bs;    // this layer's part of block 0; elements between blocks
@@ -36,65 +38,32 @@ struct GroupedArgs {
     int tbl_stride;
     int short_rows;                               // sequences with up to this many query rows belong to grouped_short_kernel
     void* out; int64_t out_ld;                    // operand of W_o: [token][out_ld], head h at column h * vp
+    int table;                                    // grouped_prefill_kernel: the distance bias comes from a table in LDS (it has room for it)
     float* part; int32_t* part_cnt;               // keys split over workgroups: partial results, arrival tickets (zero between launches)
 };
 
-// where token row `row` of a block's keys sits: tile row 16 t + 4 a + r holds token 8 a + 4 t + r of its 32-token unit
-__host__ __device__ __forceinline__ int grouped_k_row(int row) {
-    const int k = row & 31;
-    return (row & ~31) + 16 * ((k >> 2) & 1) + 4 * (k >> 3) + (k & 3);
-}
-
-// ---- keys and values of the batch's tokens into the cache: grid (32-token units of a sequence's new positions, sequences, G) ----
-template <typename ActT>
+// ---- fp32 mode: keys and values of the batch's tokens into the cache (bf16: gemm.h EPI_GROUPED): grid (32-token units of a sequence's new positions, sequences, G) ----
 __global__ __launch_bounds__(256) void grouped_place_kernel(GroupedArgs p) {
     const int seq = blockIdx.y, g = blockIdx.z, n = p.seq_len[seq], pos0 = p.seq_pos[seq], tok0 = p.seq_tok_start[seq];
     const int u0 = (pos0 & ~31) + blockIdx.x * 32;                     // first position of the unit
     const int a = max(u0, pos0), b = min(u0 + 32, pos0 + n);           // positions [a, b) are written
     if (a >= b) return;
     const int bi = u0 / p.bs, row0 = u0 - bi * p.bs;
-    ActT* base = (ActT*)p.cache + (int64_t)p.blk_table[(int64_t)seq * p.tbl_stride + bi] * p.block_stride;
-    ActT* kc = base + (int64_t)g * p.bs * p.dp;
-    ActT* vc = base + (int64_t)p.G * p.bs * p.dp + (int64_t)g * p.bs * p.vp;
-    constexpr bool FM = sizeof(ActT) == 2;
-    const int q4 = p.dp >> 2;
-    for (int i = threadIdx.x; i < (b - a) * q4; i += 256) {
-        const int j = i / q4, c = (i - j * q4) * 4, row = row0 + a - u0 + j;
-        const f32x4 v = *(const f32x4*)(p.proj + (int64_t)(tok0 + a - pos0 + j) * p.proj_ld + p.k_off + g * p.dp + c);
-        act_store4<ActT>(kc, FM ? grouped_k_row(row) : row, c, p.dp, v);
-    }
+    float* base = (float*)p.cache + (int64_t)p.blk_table[(int64_t)seq * p.tbl_stride + bi] * p.block_stride;
+    float* kc = base + (int64_t)g * p.bs * p.dp;
+    float* vc = base + (int64_t)p.G * p.bs * p.dp + (int64_t)g * p.bs * p.vp;
     const float lam = p.mix == 2 ? *p.lambda : 0.f;
-    for (int i = threadIdx.x; i < 4 * p.vp; i += 256) {                // (eight positions, value channel)
-        const int o = i / p.vp, c = i - o * p.vp, p0 = u0 + 8 * o;
-        if (p0 + 8 <= a || p0 >= b) continue;
-        float v[8];
-#pragma unroll
-        for (int e = 0; e < 8; e++) {
-            v[e] = 0.f;
-            const int pos = p0 + e;
-            if (pos < a || pos >= b) continue;
-            const int64_t t = tok0 + pos - pos0;
-            v[e] = p.proj[t * p.proj_ld + p.v_off + g * p.vp + c];
-            if (p.mix) {
-                float* f = p.vfirst + t * p.vfirst_ld + g * p.vp + c;
-                if (p.mix == 1) *f = v[e];
-                else v[e] = (1.0f - lam) * v[e] + lam * *f;
-            }
-        }
-        if constexpr (FM) {
-            ActT* d = vc + fm_index(c, row0 + 8 * o, p.bs);            // eight consecutive positions of a channel are contiguous
-            if (p0 >= a && p0 + 8 <= b) {
-                bf16x8 w;
-#pragma unroll
-                for (int e = 0; e < 8; e++) w[e] = (bf16_t)v[e];
-                *(bf16x8*)d = w;
-            } else {
-#pragma unroll
-                for (int e = 0; e < 8; e++) if (p0 + e >= a && p0 + e < b) d[e] = (ActT)v[e];
-            }
-        } else {
-#pragma unroll
-            for (int e = 0; e < 8; e++) if (p0 + e >= a && p0 + e < b) vc[(int64_t)(row0 + 8 * o + e) * p.vp + c] = (ActT)v[e];
+    for (int pos = a; pos < b; pos++) {
+        const int64_t t = tok0 + pos - pos0;
+        const int row = row0 + pos - u0;
+        const float* pr = p.proj + t * p.proj_ld;
+        for (int c = threadIdx.x; c < p.dp; c += 256) kc[(int64_t)row * p.dp + c] = pr[p.k_off + g * p.dp + c];
+        for (int c = threadIdx.x; c < p.vp; c += 256) {
+            float v = pr[p.v_off + g * p.vp + c];
+            float* f = p.vfirst + t * p.vfirst_ld + g * p.vp + c;
+            if (p.mix == 1) *f = v;
+            else if (p.mix == 2) v = (1.0f - lam) * v + lam * *f;
+            vc[(int64_t)row * p.vp + c] = v;
         }
     }
 }
@@ -112,7 +81,8 @@ struct GroupedScore {       // constants of one query row
     }
 };
 // raw scores of one 64-key tile (tile-relative key 32 (t / 2) + 8 fg + 4 (t & 1) + r; `back`: the query's own place, tile-relative)
-__device__ __forceinline__ void grouped_scores(const GroupedScore& f, f32x4 (&s)[4], int back, int fg) {
+// tab: NULL, or the (negative) biases of this lane's keys in key order
+__device__ __forceinline__ void grouped_scores(const GroupedScore& f, f32x4 (&s)[4], int back, int fg, const float* tab = nullptr) {
     if (f.cap) {
 #pragma unroll
         for (int t = 0; t < 4; t++)
@@ -122,7 +92,12 @@ __device__ __forceinline__ void grouped_scores(const GroupedScore& f, f32x4 (&s)
 #pragma unroll
         for (int t = 0; t < 4; t++) s[t] *= f.sc;
     }
-    if (f.bias) {
+    if (tab) {
+#pragma unroll
+        for (int t = 0; t < 4; t++)
+#pragma unroll
+            for (int r = 0; r < 4; r++) s[t][r] += tab[32 * (t >> 1) + 4 * (t & 1) + r];
+    } else if (f.bias) {
         const float b = fmaf(f.r2, (float)(back - 8 * fg), 1.0f);
 #pragma unroll
         for (int t = 0; t < 4; t++)
@@ -140,25 +115,25 @@ __device__ __forceinline__ void grouped_mask(f32x4 (&s)[4], int back, int window
             if (k > back || k < from) s[t][r] = -INFINITY;
         }
 }
-__device__ __forceinline__ void grouped_load_q(const float* q, int ks, int fg, bf16x8& f) {
-    const f32x4 a = *(const f32x4*)(q + ks * 32 + fg * 8), b = *(const f32x4*)(q + ks * 32 + fg * 8 + 4);
-#pragma unroll
-    for (int e = 0; e < 4; e++) { f[e] = (bf16_t)a[e]; f[4 + e] = (bf16_t)b[e]; }
+__device__ __forceinline__ bf16x8 grouped_load_q(const GroupedArgs& p, int64_t tok, int head, int ks, int fg) {
+    return *(const bf16x8*)((const bf16_t*)p.q + fm_index(tok, (int64_t)head * p.dp + ks * 32 + fg * 8, p.q_ld));
 }
 // four channels of a finished row: gate, store
 __device__ __forceinline__ void grouped_store(const GroupedArgs& p, int64_t tok, int head, int c, f32x4 v) {
-    if (p.gate_off >= 0) {
-        const f32x4 g = *(const f32x4*)(p.proj + tok * p.proj_ld + p.gate_off + head * p.vp + c);
+    const bf16x4 g = *(const bf16x4*)((const bf16_t*)p.q + fm_index(tok, p.gate_col + (int64_t)head * p.vp + c, p.q_ld));
 #pragma unroll
-        for (int r = 0; r < 4; r++) v[r] *= lat_sigmoid(g[r]);
-    }
+    for (int r = 0; r < 4; r++) v[r] *= lat_sigmoid((float)g[r]);
     act_store4<bf16_t>((bf16_t*)p.out, tok, head * p.vp + c, p.out_ld, v);
 }
 
 template <int KS, int DT> constexpr int grouped_prefill_pieces() { return 4 * KS + 2 * DT; }       // 1-KiB operand blocks of a tile
 template <int KS, int DT> constexpr int grouped_prefill_ring_bytes() { return 3 * ((grouped_prefill_pieces<KS, DT>() + 7) / 8 * 8) * 1024; }
 
-// grid (G, sequences, 256-row tiles); dynamic LDS: the ring, then (block, row) of every key tile the workgroup walks
+// grid (G, sequences, 256-row tiles); dynamic LDS: the ring, (block, row) of every key tile the workgroup walks, and with p.table the
+// distance biases of the group's heads: [head][GROUPED_TAB_PAD + span + GROUPED_TAB_PAD], falling distances, so that consecutive keys are
+// consecutive.  A wave's tiles reach at most 31 rows + 63 keys beyond its rows' windows on either side: the padding.
+constexpr int GROUPED_TAB_PAD = 96;
+__host__ __device__ __forceinline__ int grouped_tab_span(int keys) { return keys + 2 * GROUPED_TAB_PAD; }
 template <int KS, int DT>
 __global__ __launch_bounds__(512, (KS <= 2 && DT <= 4) ? 4 : 2) void grouped_prefill_kernel(GroupedArgs p) {
     constexpr int TQ = 2, PIECES = grouped_prefill_pieces<KS, DT>(), PW = (PIECES + 7) / 8, TILE = PW * 8 * 1024, NBUF = 3;
@@ -193,9 +168,8 @@ __global__ __launch_bounds__(512, (KS <= 2 && DT <= 4) ? 4 : 2) void grouped_pre
         bool ok;
         const int row = row_of(i, ok), si = row / p.group, head = kvh * p.group + row - si * p.group;
         qpos[i] = pos0 + si;
-        const float* q = p.proj + (int64_t)(tok0 + si) * p.proj_ld + head * p.dp;
 #pragma unroll
-        for (int ks = 0; ks < KS; ks++) grouped_load_q(q, ks, fg, qf[i][ks]);
+        for (int ks = 0; ks < KS; ks++) qf[i][ks] = grouped_load_q(p, tok0 + si, head, ks, fg);
         const GroupedScore f(p, head);
         r1v[i] = f.nr1; r2v[i] = f.r2;
     }
@@ -207,7 +181,25 @@ __global__ __launch_bounds__(512, (KS <= 2 && DT <= 4) ? 4 : 2) void grouped_pre
         asm volatile("" : "+v"(r1v[i]), "+v"(r2v[i]));
     }
     asm volatile("" : "+v"(f.nr1), "+v"(f.r2));
-    __syncthreads();                      // stile is visible
+    // distances of visible keys: 0 .. dmax; entry x of a head's table belongs to distance dmax + PAD - x
+    float* const tabs = (float*)(stile + p.table);            // (p.table: entries of stile)
+    const int dmax = (p.window > 0 ? min(p.window - 1, wg_last) : wg_last), span = grouped_tab_span(dmax + 1);
+    if (p.table)
+        for (int h = 0; h < p.group; h++) {
+            const float nr1 = -p.r1[kvh * p.group + h], r2 = p.r2[kvh * p.group + h];
+            for (int x = tid; x < span; x += 512) {
+                const int d = dmax + GROUPED_TAB_PAD - x;
+                tabs[h * span + x] = d > 0 ? nr1 * __builtin_amdgcn_logf(fmaf(r2, (float)d, 1.0f)) : 0.f;
+            }
+        }
+    __syncthreads();                      // stile (and the table) are visible
+    const float* tab[TQ];
+#pragma unroll
+    for (int i = 0; i < TQ; i++) {
+        bool ok;
+        const int row = row_of(i, ok), h = row % p.group;
+        tab[i] = p.table ? tabs + h * span + dmax + GROUPED_TAB_PAD - qpos[i] + 8 * fg : nullptr;      // + key = the key's entry
+    }
     // LDS-DMA: wave w moves pieces w * PW .. of [K: 16-key tile, k-step | V^T: d, 32-key unit]; surplus pieces repeat the last one
     int64_t src[PW];
 #pragma unroll
@@ -274,7 +266,7 @@ __global__ __launch_bounds__(512, (KS <= 2 && DT <= 4) ? 4 : 2) void grouped_pre
         for (int i = 0; i < TQ; i++) {
             const int back = qpos[i] - kt * 64;
             f.nr1 = r1v[i]; f.r2 = r2v[i];
-            grouped_scores(f, s[i], back, fg);
+            grouped_scores(f, s[i], back, fg, p.table ? tab[i] + kt * 64 : nullptr);
             if (!whole) grouped_mask(s[i], back, p.window, fg);
             const float m_new = vmax2(m_run[i], rows_max(vmax16(s[i][0], s[i][1], s[i][2], s[i][3])));
             if (__any(m_new != m_run[i])) {
@@ -319,8 +311,22 @@ __global__ __launch_bounds__(512, (KS <= 2 && DT <= 4) ? 4 : 2) void grouped_pre
 
 // grid (G x 16-row tiles, sequences, key splits).  Wave w of workgroup z takes the key tiles z NW + w, + NW gridDim.z, ...; operands
 // come straight from the cache.  The waves' results are combined through LDS; with gridDim.z > 1 every workgroup leaves a partial
-// record {O^T [DT][64 lanes] f32x4, m[16], l[16]} and the one that draws the last ticket combines them in z order.
+// record {O^T [DT][64 lanes] f32x4, (m, l)[16]} (the lanes of live rows) and the one that draws the last ticket combines them in z order.
+constexpr int GROUPED_SPLITS = 16;          // most workgroups the keys of a row tile are split over
 template <int DT> constexpr int grouped_part_floats() { return DT * 256 + 32; }
+__device__ __forceinline__ void grouped_part_store2(float* p, float a, float b) {
+    __hip_atomic_store((unsigned long long*)p, __builtin_bit_cast(unsigned long long, f32x2{a, b}), __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
+}
+__device__ __forceinline__ void grouped_part_store(float* p, f32x4 v) { grouped_part_store2(p, v[0], v[1]); grouped_part_store2(p + 2, v[2], v[3]); }
+__device__ __forceinline__ void grouped_part_load2(const float* p, float& a, float& b) {
+    const f32x2 v = __builtin_bit_cast(f32x2, __hip_atomic_load((const unsigned long long*)p, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT));
+    a = v[0]; b = v[1];
+}
+__device__ __forceinline__ f32x4 grouped_part_load(const float* p) {
+    float a, b, c, d;
+    grouped_part_load2(p, a, b); grouped_part_load2(p + 2, c, d);
+    return f32x4{a, b, c, d};
+}
 template <int KS, int DT, int NW>
 __global__ __launch_bounds__(NW * 64) void grouped_short_kernel(GroupedArgs p) {
     extern __shared__ __attribute__((aligned(16))) char grp_sm[];       // [NW][DT][64] f32x4
@@ -341,9 +347,8 @@ __global__ __launch_bounds__(NW * 64) void grouped_short_kernel(GroupedArgs p) {
     const int full_lo = p.window > 0 ? last - p.window + 1 : 0, full_hi = first;
     const int64_t tok = tok0 + si;
     bf16x8 qf[KS], kf[4][KS], vf[DT][2];
-    const float* q = p.proj + tok * p.proj_ld + head * p.dp;
 #pragma unroll
-    for (int ks = 0; ks < KS; ks++) grouped_load_q(q, ks, fg, qf[ks]);
+    for (int ks = 0; ks < KS; ks++) qf[ks] = grouped_load_q(p, tok, head, ks, fg);
     const GroupedScore f(p, head);
     f32x4 o[DT];
 #pragma unroll
@@ -411,33 +416,39 @@ __global__ __launch_bounds__(NW * 64) void grouped_short_kernel(GroupedArgs p) {
         f32x4 a = f32x4{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
         for (int w = 0; w < NW; w++) a += po[(w * DT + d) * 64 + lane] * sc[w];
-        if (nz > 1) ((f32x4*)rec)[d * 64 + lane] = a;
-        else if (ok) grouped_store(p, tok, head, 16 * d + 4 * fg, a * (1.0f / L));
+        if (!ok) continue;
+        if (nz > 1) grouped_part_store(rec + (d * 64 + lane) * 4, a);
+        else grouped_store(p, tok, head, 16 * d + 4 * fg, a * (1.0f / L));
     }
     if (nz == 1) return;
-    if (wave == 0 && fg == 0) { rec[DT * 256 + fq] = ms; rec[DT * 256 + 16 + fq] = L; }
-    __threadfence();                       // release: the other workgroups may sit on other XCDs
+    if (wave == 0 && fg == 0 && ok) grouped_part_store2(rec + DT * 256 + 2 * fq, ms, L);
+    // Partial results go past the L2 of this XCD (agent-scope stores) and are read past the reader's, so no cache has to be written back
+    // or invalidated: it is enough that they have arrived when the ticket is drawn.
+    asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
     __syncthreads();
     if (tid == 0) ticket = __hip_atomic_fetch_add(p.part_cnt + pair, 1, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
     __syncthreads();
     if (ticket != nz - 1) return;
-    __threadfence();                       // acquire
+    if (tid == 0) __hip_atomic_store(p.part_cnt + pair, 0, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);      // for the next launch
+    if (!ok) return;
     const float* rec0 = p.part + (int64_t)pair * nz * grouped_part_floats<DT>();
-    float M = -1e30f, LL = 0.f;
-    for (int z = 0; z < nz; z++) M = fmaxf(M, rec0[(int64_t)z * grouped_part_floats<DT>() + DT * 256 + fq]);
-    for (int z = 0; z < nz; z++) {
-        const float* rz = rec0 + (int64_t)z * grouped_part_floats<DT>() + DT * 256;
-        LL += rz[16 + fq] * __builtin_amdgcn_exp2f(rz[fq] - M);
-    }
+    float M = -1e30f, LL = 0.f, mz[GROUPED_SPLITS];
+#pragma unroll
+    for (int z = 0; z < GROUPED_SPLITS; z++)
+        if (z < nz) {
+            float lz;
+            grouped_part_load2(rec0 + (int64_t)z * grouped_part_floats<DT>() + DT * 256 + 2 * fq, mz[z], lz);
+            const float mn = fmaxf(M, mz[z]);
+            LL = LL * __builtin_amdgcn_exp2f(M - mn) + lz * __builtin_amdgcn_exp2f(mz[z] - mn);
+            M = mn;
+        }
     for (int d = wave; d < DT; d += NW) {
         f32x4 a = f32x4{0.f, 0.f, 0.f, 0.f};
-        for (int z = 0; z < nz; z++) {
-            const float* rz = rec0 + (int64_t)z * grouped_part_floats<DT>();
-            a += ((const f32x4*)rz)[d * 64 + lane] * __builtin_amdgcn_exp2f(rz[DT * 256 + fq] - M);
-        }
-        if (ok) grouped_store(p, tok, head, 16 * d + 4 * fg, a * (1.0f / LL));
+#pragma unroll
+        for (int z = 0; z < GROUPED_SPLITS; z++)
+            if (z < nz) a += grouped_part_load(rec0 + (int64_t)z * grouped_part_floats<DT>() + (d * 64 + lane) * 4) * __builtin_amdgcn_exp2f(mz[z] - M);
+        grouped_store(p, tok, head, 16 * d + 4 * fg, a * (1.0f / LL));
     }
-    if (tid == 0) __hip_atomic_store(p.part_cnt + pair, 0, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);      // for the next launch
 }
 
 // ---- any size: one 256-thread workgroup per (token, head), online softmax over 256 keys at a time, plain fp32 arithmetic ----
@@ -452,7 +463,7 @@ __global__ __launch_bounds__(256) void grouped_plain_kernel(GroupedArgs p) {
     const int pos = p.seq_pos[seq] + r, lo = p.window > 0 && pos - p.window + 1 > 0 ? pos - p.window + 1 : 0;
     const int32_t* tbl = p.blk_table + (int64_t)seq * p.tbl_stride;
     float *sq = grp_f, *so = grp_f + p.dp;
-    for (int i = tid; i < p.dp; i += 256) sq[i] = p.proj[t * p.proj_ld + h * p.dp + i];
+    for (int i = tid; i < p.dp; i += 256) sq[i] = (float)((const T*)p.q)[act_index<T>(t, h * p.dp + i, p.q_ld)];
     for (int i = tid; i < p.vp; i += 256) so[i] = 0.f;
     const float r1 = p.r1 ? p.r1[h] : 0.f, r2 = p.r1 ? p.r2[h] : 0.f;
     float m = -1e30f, l = 0.f;
@@ -492,8 +503,7 @@ __global__ __launch_bounds__(256) void grouped_plain_kernel(GroupedArgs p) {
         __syncthreads();
     }
     for (int i = tid; i < p.vp; i += 256) {
-        float o = so[i] / l;
-        if (p.gate_off >= 0) o *= 1.0f / (1.0f + expf(-p.proj[t * p.proj_ld + p.gate_off + h * p.vp + i]));
+        const float o = so[i] / l * (1.0f / (1.0f + expf(-(float)((const T*)p.q)[act_index<T>(t, p.gate_col + h * p.vp + i, p.q_ld)])));
         ActIO<T>::st((T*)p.out + act_index<T>(t, h * p.vp + i, p.out_ld), o);
     }
 }

@@ -23,7 +23,7 @@ namespace {
 
 constexpr float CLAMPED_GLU_SLOPE = 1.702f;
 constexpr int LAT_ABSORB_MAX = 16, LAT_ABSORB_MAX_RP = 512, REC_STEP_MAX = 4;
-constexpr int GROUPED_SHORT_ROWS = 64, GROUPED_SPLITS = 16, GROUPED_SPLIT_WGS = 512;      // GROUPED_SPLIT_WGS: workgroups of a launch whose keys are split
+constexpr int GROUPED_SHORT_ROWS = 64, GROUPED_SPLIT_WGS = 512;      // GROUPED_SPLIT_WGS: workgroups of a launch whose keys are split
 
 bool same_rotation(const nvl_layer_config& a, const nvl_layer_config& b) {
     return a.rot_dim == b.rot_dim && a.rot_base == b.rot_base && a.rot_factor == b.rot_factor && a.rot_original == b.rot_original &&
@@ -164,7 +164,9 @@ int layered_create(const nvl_model_config& c, const nvl_layer_config* layers, co
             } else if (r.c.mixer == NVL_MIXER_ATTENTION) {
                 const int G = r.c.kv_heads;
                 r.dp = pad_head(r.c.dim, 64); r.vp = pad_head(r.c.vdim, 64);
-                r.k_off = H * r.dp; r.v_off = r.k_off + G * r.dp; r.gate_off = r.v_off + G * r.vp; r.route_off = r.gate_off + H * r.vp;
+                r.k_off = H * r.dp; r.v_off = r.k_off + G * r.dp; r.gate_off = r.v_off + G * r.vp; r.ffn_off = r.gate_off + H * r.vp;
+                r.ffn_in = par && r.c.ffn_dim && r.act == NVL_ACT_RELU2;
+                r.route_off = r.ffn_off + (r.ffn_in ? r.Fp : 0);
                 r.n_in = r.route_off + r.c.experts; r.ko = (int)round_up((int64_t)H * r.vp, 64);
                 r.cache_off = cache; cache += (int64_t)bs * G * (r.dp + r.vp);
                 if (r.c.v_mix) {
@@ -430,7 +432,7 @@ void layered_finalize(nvl_model* m) {
     m->g[NVL_T_POS_EMB].p = pos;
 
     int64_t ld_in = 0, q_cols = 0, cq_cols = 0, ko = 0, conv = 0, ocols = 0, Fmax = 0, abs_cols = 0, z_cols = 0, g_cols = 0, pa_cols = 0, pg_cols = 0;
-    int64_t moe_k = 0, moe_e = 0, moe_kI = 0, moe_ep = 0, moe_all = 0, moe_sl = 0, grp_vp = 0;
+    int64_t moe_k = 0, moe_e = 0, moe_kI = 0, moe_ep = 0, moe_all = 0, moe_sl = 0, grp_vp = 0, qg_cols = 0;
     for (int i = 0; i < m->L; i++) {
         LayerRun& r = m->runs[(size_t)i];
         const nvl_layer_config& c = r.c;
@@ -446,8 +448,9 @@ void layered_finalize(nvl_model* m) {
                 if (!post && !par) w.norm2 = lay_norm(m, T(NVL_T_FFN_NORM_W, "norm before the feed-forward"), H);
                 if (!par) w.norm2b = lay_norm(m, T(NVL_T_FFN_POST_NORM, "norm after the feed-forward"), H, &l.t[NVL_T_FFN_SCALE]);
                 const DevTensor& w1 = T(NVL_T_W1, "feed-forward gate / up");
-                w.w1 = lay_matrix(m, (r.act == NVL_ACT_RELU2 ? 1 : 2) * r.Fp, H);
-                if (r.act == NVL_ACT_RELU2) lay_place(m, w1, w.w1, H);
+                if (!r.ffn_in) w.w1 = lay_matrix(m, (r.act == NVL_ACT_RELU2 ? 1 : 2) * r.Fp, H);
+                if (r.ffn_in) {}
+                else if (r.act == NVL_ACT_RELU2) lay_place(m, w1, w.w1, H);
                 else if (m->f32) { lay_place(m, w1, w.w1, H, 0, 0, 0, 0, 0, 0, c.ffn_dim); lay_place(m, w1, w.w1, H, r.Fp, 0, 0, 0, 0, c.ffn_dim, c.ffn_dim); }
                 else { lay_place(m, w1, w.w1, H, 0, 16, 32, 0, 0, 0, c.ffn_dim); lay_place(m, w1, w.w1, H, 16, 16, 32, 0, 0, c.ffn_dim, c.ffn_dim); }
                 if (!par) {
@@ -581,6 +584,7 @@ void layered_finalize(nvl_model* m) {
                 w.o = lay_matrix(m, H, r.kd);
                 lay_place(m, T(NVL_T_WO, "output projection"), w.o, r.kd);
             }
+            if (r.ffn_in) lay_place(m, T(NVL_T_W1, "feed-forward up"), w.in, H, r.ffn_off);
             if (c.experts) lay_place(m, T(NVL_T_ROUTER, "router"), w.in, H, r.route_off);
             if (par && c.ffn_dim) lay_place(m, T(NVL_T_W2, "feed-forward down"), w.o, r.kd, 0, 0, 0, 0, 0, 0, -1, false, false, r.ko);
             NVL_HIP(hipStreamSynchronize(m->stream));
@@ -603,7 +607,9 @@ void layered_finalize(nvl_model* m) {
             pa_cols = std::max<int64_t>(pa_cols, w.a_rkp); pg_cols = std::max<int64_t>(pg_cols, w.g_rkp);
         }
         if (c.mixer == NVL_MIXER_GLA) r.n_in = 2 * c.heads * (c.dim + c.vdim) + m->mixers[(size_t)r.owner].rank;
-        ld_in = std::max(ld_in, round_up(r.n_in, 4));
+        const bool qg = c.mixer == NVL_MIXER_ATTENTION && !m->f32;           // (its projection goes to lqg, the cache and lmix; the router's columns stay)
+        ld_in = std::max(ld_in, round_up(qg ? r.n_in - r.route_off : r.n_in, 4));
+        if (qg) qg_cols = std::max<int64_t>(qg_cols, (int64_t)c.heads * (r.dp + r.vp));
         ko = std::max<int64_t>(ko, r.kd);
         Fmax = std::max<int64_t>(Fmax, r.Fp);
         if (c.experts) {
@@ -628,6 +634,7 @@ void layered_finalize(nvl_model* m) {
     m->lproj_ld = ld_in; m->lq_ld = q_cols; m->lo_ld = round_up(ocols, 4); m->lconv_ld = round_up(conv, 4);
     m->x = dmalloc<float>(Mmax * H);
     m->xn = dmalloc_bytes(Mp * H * ws);
+    ld_in = std::max<int64_t>(ld_in, 4);
     const int64_t hbuf = std::max(Mp * m->F, round_up(Mmax * std::max<int64_t>(moe_k, 1), 64) * (moe_k ? moe_kI / moe_k : 0) + 64 * moe_kI);
     m->hbuf = dmalloc_bytes(hbuf * ws);
     m->xn_last = dmalloc_bytes(round_up(S, 64) * H * ws);
@@ -650,6 +657,7 @@ void layered_finalize(nvl_model* m) {
         }
     }
     if (sd) m->lside = lay_alloc(m, Mp * m->side_kp * ws);
+    if (qg_cols) m->lqg = (bf16_t*)lay_alloc(m, Mp * qg_cols * 2);
     if (m->lvf_ld) m->lvf = (float*)lay_alloc(m, Mmax * m->lvf_ld * 4);
     if (grp_vp && !m->f32 && grp_vp <= 256) {
         m->grp_cap = GROUPED_SPLIT_WGS;
@@ -1243,34 +1251,44 @@ void tap_layer(nvl_model* m, int li, int M);
 // ---- grouped-query attention: m->xn -> m->lmix columns [0, ko) ----
 void mix_grouped(nvl_model* m, const LayerRun& r, const MixerW& w, const Meta& md, int n_seqs, int M, int max_len) {
     const nvl_layer_config& c = r.c;
-    in_proj(m, r, w, M);
     GroupedArgs a{};
     a.H = c.heads; a.G = c.kv_heads; a.group = c.heads / c.kv_heads; a.dim = c.dim; a.dp = r.dp; a.vdim = c.vdim; a.vp = r.vp;
     a.window = c.window; a.scale = c.scale; a.softcap = c.softcap; a.r1 = w.r1; a.r2 = w.r2;
-    a.proj = m->lproj; a.proj_ld = m->lproj_ld; a.k_off = r.k_off; a.v_off = r.v_off; a.gate_off = r.gate_off;
     a.mix = r.mix; a.lambda = w.v_lambda; a.vfirst = m->lvf; a.vfirst_ld = m->lvf_ld;
     a.cache = (char*)m->lat_cache + r.cache_off * (int64_t)m->wsize; a.block_stride = m->lat_block_stride; a.bs = m->Tmax;
     a.blk_table = md.blk_table; a.seq_tok_start = md.seq_tok_start; a.seq_len = md.seq_len; a.seq_pos = md.seq_pos; a.tbl_stride = m->blocks_per_seq;
     a.out = m->lmix; a.out_ld = r.kd;
     const double ws = (double)m->wsize;
-    {
+    if (m->f32) {
+        in_proj(m, r, w, M);
+        a.q = m->lproj; a.q_ld = m->lproj_ld; a.gate_col = r.gate_off;
+        a.proj = m->lproj; a.proj_ld = m->lproj_ld; a.k_off = r.k_off; a.v_off = r.v_off;
         KScope ks(m, KC_OTHER, 0, KS_KV_PLACE, (double)M * a.G * (c.dim + c.vdim) * (4.0 + ws) + (r.mix ? (double)M * a.G * c.vdim * 4.0 : 0.0));
-        const dim3 grid(cdiv(max_len + 31, 32), n_seqs, a.G);
-        if (m->f32) hipLaunchKernelGGL((grouped_place_kernel<float>), grid, dim3(256), 0, m->stream, a);
-        else hipLaunchKernelGGL((grouped_place_kernel<bf16_t>), grid, dim3(256), 0, m->stream, a);
+        hipLaunchKernelGGL(grouped_place_kernel, dim3(cdiv(max_len + 31, 32), n_seqs, a.G), dim3(256), 0, m->stream, a);
         NVL_HIP(hipGetLastError());
+    } else {
+        a.q = m->lqg; a.q_ld = (int64_t)a.H * (r.dp + r.vp); a.gate_col = a.H * r.dp;
+        GemmArgs g = mk(m->xn, m->H, w.in, m->lqg, (int)a.q_ld, nullptr, 1.f, M, r.n_in, m->H);
+        g.grp = GroupedEpi{r.k_off, r.v_off, r.gate_off, r.ffn_off, r.route_off, md.tok_pos, md.tok_tbl, md.blk_table, (bf16_t*)a.cache, a.block_stride, a.bs, a.G, r.dp, r.vp,
+                           r.mix, w.v_lambda, m->lvf, m->lvf_ld, (bf16_t*)m->lmix + (r.ko >> 5) * 512, r.kd, m->lproj, m->lproj_ld};
+        m->site = KS_MIX_IN;
+        gemm(m, EPI_GROUPED, false, g);
     }
     const bool plain = m->f32 || r.dp > 256 || r.vp > 256;
     const int ctx = m->ctx_hint > 0 ? m->ctx_hint : m->cfg.max_seq_len;
     int tiles = cdiv(ctx, 64) + 1;                              // most key tiles a 256-row workgroup walks
     if (c.window > 0) tiles = std::min(tiles, (c.window + cdiv(256, a.group) + 1) / 64 + 3);
-    const size_t ring = (size_t)3 * round_up(4 * (r.dp >> 5) + 2 * (r.vp >> 4), 8) * 1024, lds = ring + (size_t)tiles * 8;
+    const size_t ring = (size_t)3 * round_up(4 * (r.dp >> 5) + 2 * (r.vp >> 4), 8) * 1024;
+    size_t lds = ring + (size_t)tiles * 8;
+    // the distance biases of a workgroup's rows as a table in LDS, where they leave as many workgroups per CU as the ring does
+    const size_t tab = lds + (size_t)grouped_tab_span(std::min(ctx, c.window > 0 ? c.window : ctx)) * a.group * 4;
+    if (w.r1 && tab <= (size_t)(r.dp <= 64 && r.vp <= 64 ? 80 : 160) * 1024) { a.table = tiles; lds = tab; }
     a.short_rows = GROUPED_SHORT_ROWS;
     if ((r.dp == 256 && r.vp == 256) || lds > 160 * 1024) a.short_rows = 1 << 30;      // (three slots would not fit LDS)
     const bool any_short = m->min_len * a.group <= a.short_rows, any_long = max_len * a.group > a.short_rows;
     auto scope = [&](int several) {
         const double pairs = m->win_pairs[(size_t)r.win][(size_t)several], keys = m->win_keys[(size_t)r.win][(size_t)several];
-        return KScope(m, KC_ATTN, 2.0 * pairs * a.H * (c.dim + c.vdim), KS_ATTN, keys * a.G * (c.dim + c.vdim) * ws + (double)M * a.H * (4.0 * c.dim + (4.0 + ws) * c.vdim));
+        return KScope(m, KC_ATTN, 2.0 * pairs * a.H * (c.dim + c.vdim), KS_ATTN, (keys * a.G * (c.dim + c.vdim) + (double)M * a.H * (c.dim + 2.0 * c.vdim)) * ws);
     };
     if (plain) {
         KScope ks = scope(max_len > 1);
@@ -1300,19 +1318,24 @@ void mix_grouped(nvl_model* m, const LayerRun& r, const MixerW& w, const Meta& m
     if (any_short) {
         KScope scp = scope(any_long ? 0 : max_len > 1);
         const int64_t wgs = (int64_t)a.G * cdiv(std::min<int64_t>((int64_t)max_len * a.group, a.short_rows), 16);
+        // eight waves a workgroup when the row tiles alone come near the CUs' number; else four, and the keys split over workgroups
+        const int key_tiles = 1 << layered_kt_log2(m);
+        const bool wide = dt <= 8 && wgs * n_seqs >= 96;
         int z = 1;
-        while (z < GROUPED_SPLITS && wgs * n_seqs * z * 2 <= m->grp_cap && z * 2 * 4 <= (1 << layered_kt_log2(m))) z *= 2;
+        while (!wide && z < GROUPED_SPLITS && wgs * n_seqs * z * 2 <= 256 && z * 2 * 4 <= key_tiles) z *= 2;
         a.part = m->grp_part; a.part_cnt = m->grp_cnt;
         const dim3 grid((unsigned)wgs, n_seqs, z);
-#define NVL_GS(KSv, DTv)                                                                                                     \
+#define NVL_GSW(KSv, DTv, NWv)                                                                                               \
         do {                                                                                                                 \
-            NVL_LDS_ATTR((grouped_short_kernel<KSv, DTv, 4>), 4 * DTv * 1024);                                               \
-            hipLaunchKernelGGL((grouped_short_kernel<KSv, DTv, 4>), grid, dim3(256), 4 * DTv * 1024, m->stream, a);          \
+            NVL_LDS_ATTR((grouped_short_kernel<KSv, DTv, NWv>), NWv * DTv * 1024);                                           \
+            hipLaunchKernelGGL((grouped_short_kernel<KSv, DTv, NWv>), grid, dim3(NWv * 64), NWv * DTv * 1024, m->stream, a); \
         } while (0)
+#define NVL_GS(KSv, DTv) do { if (wide) NVL_GSW(KSv, DTv, (DTv <= 8 ? 8 : 4)); else NVL_GSW(KSv, DTv, 4); } while (0)
 #define NVL_GSK(KSv) do { if (dt == 2) NVL_GS(KSv, 2); else if (dt == 4) NVL_GS(KSv, 4); else if (dt == 8) NVL_GS(KSv, 8); else NVL_GS(KSv, 16); } while (0)
         if (ks == 1) NVL_GSK(1); else if (ks == 2) NVL_GSK(2); else if (ks == 4) NVL_GSK(4); else NVL_GSK(8);
 #undef NVL_GSK
 #undef NVL_GS
+#undef NVL_GSW
         NVL_HIP(hipGetLastError());
     }
 }
@@ -1320,7 +1343,12 @@ void mix_grouped(nvl_model* m, const LayerRun& r, const MixerW& w, const Meta& m
 // ---- feed-forward of a parallel block: m->xn -> m->lmix columns [ko, kd); the experts' results for the join ----
 ExpertOut parallel_ffn(nvl_model* m, const LayerRun& r, const MixerW& w, int M) {
     const nvl_layer_config& c = r.c;
-    if (c.ffn_dim) {
+    if (r.ffn_in && m->f32) {       // (bf16: the input projection's epilogue has written them)
+        const int64_t n = (int64_t)M * r.Fp;
+        KScope ks(m, KC_OTHER);
+        hipLaunchKernelGGL((relu2_kernel<float>), dim3(cdiv(n, 256)), dim3(256), 0, m->stream, m->lproj + r.ffn_off, m->lproj_ld, (float*)m->lmix, (int64_t)M, r.Fp, (int64_t)r.kd, r.ko);
+        NVL_HIP(hipGetLastError());
+    } else if (c.ffn_dim && !r.ffn_in) {
         m->site = KS_FFN_UP;
         const bool relu2 = r.act == NVL_ACT_RELU2;
         const int N = relu2 ? r.Fp : 2 * r.Fp;
@@ -1328,7 +1356,7 @@ ExpertOut parallel_ffn(nvl_model* m, const LayerRun& r, const MixerW& w, int M) 
             gemm(m, EPI_STORE, true, mk(m->xn, m->H, w.w1, m->h2, N, nullptr, 1.f, M, N, m->H));
             const int64_t n = (int64_t)M * r.Fp;
             KScope ks(m, KC_OTHER);
-            if (relu2) hipLaunchKernelGGL((relu2_kernel<float>), dim3(cdiv(n, 256)), dim3(256), 0, m->stream, m->h2, (float*)m->lmix, (int64_t)M, r.Fp, (int64_t)r.kd, r.ko);
+            if (relu2) hipLaunchKernelGGL((relu2_kernel<float>), dim3(cdiv(n, 256)), dim3(256), 0, m->stream, m->h2, (int64_t)N, (float*)m->lmix, (int64_t)M, r.Fp, (int64_t)r.kd, r.ko);
             else hipLaunchKernelGGL((swiglu_kernel<float>), dim3(cdiv(n, 256)), dim3(256), 0, m->stream, m->h2, (float*)m->lmix, (int64_t)M, r.Fp, (int64_t)r.kd, r.ko);
             NVL_HIP(hipGetLastError());
         } else      // (the operand's column blocks are 32 wide: a shift by ko columns is a shift of the base)
@@ -1338,7 +1366,7 @@ ExpertOut parallel_ffn(nvl_model* m, const LayerRun& r, const MixerW& w, int M) 
     const int E = c.experts, k = c.top_k, pairs = M * k;
     // decode: all experts as one projection each way with the routing weights as a mask (gemm.h GemmArgs::moe_gate)
     const bool dense = !m->f32 && M <= 64 && r.Ip <= 2048;
-    GroupRouteArgs ra{m->lproj + r.route_off, m->lproj_ld, w.route_bias, M, E, k, c.expert_groups, c.groups_kept, m->expert_ids, m->expert_w, dense ? m->moe_gate : nullptr, r.Ep};
+    GroupRouteArgs ra{m->lproj + (m->f32 ? r.route_off : 0), m->lproj_ld, w.route_bias, M, E, k, c.expert_groups, c.groups_kept, m->expert_ids, m->expert_w, dense ? m->moe_gate : nullptr, r.Ep};
     {
         KScope ks(m, KC_OTHER, 0, KS_MOE_ROUTER, (double)M * (E + 2.0 * k) * 4.0);
         hipLaunchKernelGGL(moe_route_grouped_kernel, dim3(cdiv(M, 4)), dim3(256), 0, m->stream, ra);

@@ -65,7 +65,8 @@ struct LayerRun {
     int conv_dim = 0;
     int win = -1;                // index into nvl_model::windows
     int64_t cache_off = 0;       // attention: element offset inside a cache block
-    int k_off = 0, v_off = 0, route_off = 0;     // grouped attention: columns of the fused input projection (keys, values, router)
+    int k_off = 0, v_off = 0, ffn_off = 0, route_off = 0;     // grouped attention: columns of the fused input projection (keys, values, feed-forward, router)
+    bool ffn_in = false;         // ... whose feed-forward columns are the whole up projection (ungated activations)
     int mix = 0;                 // grouped attention: GroupedArgs::mix
     int kd = 0;                  // K of the joint output projection of a parallel block: ko, then the feed-forward's Fp columns
     int act = 0;                 // activation of the feed-forward
@@ -166,6 +167,7 @@ struct nvl_model {
     std::vector<nvl::MixerW> mixers;
     std::vector<void*> layered_allocs;
     float *final_norm = nullptr, *final_norm_b = nullptr;
+    nvl::bf16_t* lqg = nullptr;          // grouped attention, bf16: [token][queries | gates] (fragment-major)
     float* lvf = nullptr; int64_t lvf_ld = 0;                       // grouped attention: the first mixing layer's values of the running batch
     void *side_emb = nullptr, *lside = nullptr; int64_t side_ld = 0; int side_kp = 0;     // per-layer token inputs: table (rows of L * side4 entries), operand of the projection
     float* grp_part = nullptr; int32_t* grp_cnt = nullptr; int64_t grp_cap = 0;           // grouped attention: key splits

@@ -195,6 +195,7 @@ void gemm(nvl_model* m, int epi, bool out_f32, GemmArgs a, double flops = -1.0) 
             case EPI_GEGLU:  launch_gemm_bf16<EPI_GEGLU, bf16_t>(st, a); break;
             case EPI_CLAMP_GLU: launch_gemm_bf16<EPI_CLAMP_GLU, bf16_t>(st, a); break;
             case EPI_QKV:    launch_gemm_bf16<EPI_QKV, bf16_t>(st, a); break;
+            case EPI_GROUPED: launch_gemm_bf16<EPI_GROUPED, bf16_t>(st, a); break;
             case EPI_RELU2:  launch_gemm_bf16<EPI_RELU2, bf16_t>(st, a); break;
             case EPI_GELU_TOK: launch_gemm_bf16<EPI_GELU_TOK, bf16_t>(st, a); break;
             default: throw std::runtime_error("gemm: bad epilogue");
