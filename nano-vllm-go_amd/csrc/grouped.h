@@ -81,8 +81,17 @@ struct GroupedScore {       // constants of one query row
     }
 };
 // raw scores of one 64-key tile (tile-relative key 32 (t / 2) + 8 fg + 4 (t & 1) + r; `back`: the query's own place, tile-relative)
-// tab: NULL, or the (negative) biases of this lane's keys in key order
+// tab: NULL, or the (negative) biases of this lane's keys in key order; FAST: capped, with a table that holds softcap - bias
+template <bool FAST = false>
 __device__ __forceinline__ void grouped_scores(const GroupedScore& f, f32x4 (&s)[4], int back, int fg, const float* tab = nullptr) {
+    if constexpr (FAST) {
+#pragma unroll
+        for (int t = 0; t < 4; t++)
+#pragma unroll
+            for (int r = 0; r < 4; r++)
+                s[t][r] = fmaf(f.c2, __builtin_amdgcn_rcpf(__builtin_amdgcn_exp2f(s[t][r] * f.sc) + 1.0f), tab[32 * (t >> 1) + 4 * (t & 1) + r]);
+        return;
+    }
     if (f.cap) {
 #pragma unroll
         for (int t = 0; t < 4; t++)
@@ -133,8 +142,13 @@ template <int KS, int DT> constexpr int grouped_prefill_ring_bytes() { return 3 
 // distance biases of the group's heads: [head][GROUPED_TAB_PAD + span + GROUPED_TAB_PAD], falling distances, so that consecutive keys are
 // consecutive.  A wave's tiles reach at most 31 rows + 63 keys beyond its rows' windows on either side: the padding.
 constexpr int GROUPED_TAB_PAD = 96;
-__host__ __device__ __forceinline__ int grouped_tab_span(int keys) { return keys + 2 * GROUPED_TAB_PAD; }
-template <int KS, int DT>
+// (20 modulo 64: the heads of a group then read from different banks; never less than keys + 2 PAD)
+__host__ __device__ __forceinline__ int grouped_tab_span(int keys) { return ((keys + 2 * GROUPED_TAB_PAD + 43) & ~63) + 20; }
+// FAST: scores that the cap bounds from both sides and biases that only lower them, from the table.  Their exponentials are taken as
+// they are: no running maximum, no rescaling.  (GROUPED_FAST_CAP: the sum of 2^20 weights stays finite; a query sees its own key, so a
+// weight that underflows is below 2^-30 of the sum.)  The other modes share the other instance.
+constexpr float GROUPED_FAST_CAP = 60.0f;
+template <int KS, int DT, bool FAST>
 __global__ __launch_bounds__(512, (KS <= 2 && DT <= 4) ? 4 : 2) void grouped_prefill_kernel(GroupedArgs p) {
     constexpr int TQ = 2, PIECES = grouped_prefill_pieces<KS, DT>(), PW = (PIECES + 7) / 8, TILE = PW * 8 * 1024, NBUF = 3;
     extern __shared__ __attribute__((aligned(16))) char grp_sm[];
@@ -186,10 +200,10 @@ __global__ __launch_bounds__(512, (KS <= 2 && DT <= 4) ? 4 : 2) void grouped_pre
     const int dmax = (p.window > 0 ? min(p.window - 1, wg_last) : wg_last), span = grouped_tab_span(dmax + 1);
     if (p.table)
         for (int h = 0; h < p.group; h++) {
-            const float nr1 = -p.r1[kvh * p.group + h], r2 = p.r2[kvh * p.group + h];
+            const float nr1 = -p.r1[kvh * p.group + h], r2 = p.r2[kvh * p.group + h], top = FAST ? p.softcap * 1.4426950408889634f : 0.f;
             for (int x = tid; x < span; x += 512) {
                 const int d = dmax + GROUPED_TAB_PAD - x;
-                tabs[h * span + x] = d > 0 ? nr1 * __builtin_amdgcn_logf(fmaf(r2, (float)d, 1.0f)) : 0.f;
+                tabs[h * span + x] = d > 0 ? fmaf(nr1, __builtin_amdgcn_logf(fmaf(r2, (float)d, 1.0f)), top) : top;
             }
         }
     __syncthreads();                      // stile (and the table) are visible
@@ -198,7 +212,7 @@ __global__ __launch_bounds__(512, (KS <= 2 && DT <= 4) ? 4 : 2) void grouped_pre
     for (int i = 0; i < TQ; i++) {
         bool ok;
         const int row = row_of(i, ok), h = row % p.group;
-        tab[i] = p.table ? tabs + h * span + dmax + GROUPED_TAB_PAD - qpos[i] + 8 * fg : nullptr;      // + key = the key's entry
+        tab[i] = FAST || p.table ? tabs + h * span + dmax + GROUPED_TAB_PAD - qpos[i] + 8 * fg : nullptr;      // + key = the key's entry
     }
     // LDS-DMA: wave w moves pieces w * PW .. of [K: 16-key tile, k-step | V^T: d, 32-key unit]; surplus pieces repeat the last one
     int64_t src[PW];
@@ -264,23 +278,37 @@ __global__ __launch_bounds__(512, (KS <= 2 && DT <= 4) ? 4 : 2) void grouped_pre
         const bool whole = kt * 64 >= full_lo && kt * 64 + 63 <= full_hi;
 #pragma unroll
         for (int i = 0; i < TQ; i++) {
-            const int back = qpos[i] - kt * 64;
-            f.nr1 = r1v[i]; f.r2 = r2v[i];
-            grouped_scores(f, s[i], back, fg, p.table ? tab[i] + kt * 64 : nullptr);
-            if (!whole) grouped_mask(s[i], back, p.window, fg);
-            const float m_new = vmax2(m_run[i], rows_max(vmax16(s[i][0], s[i][1], s[i][2], s[i][3])));
-            if (__any(m_new != m_run[i])) {
-                const float alpha = __builtin_amdgcn_exp2f(m_run[i] - m_new);
-                lacc[i] *= alpha;
+            if constexpr (!FAST) { f.nr1 = r1v[i]; f.r2 = r2v[i]; }
+            grouped_scores<FAST>(f, s[i], qpos[i] - kt * 64, fg, FAST || p.table ? tab[i] + kt * 64 : nullptr);
+        }
+        if (!whole)
 #pragma unroll
-                for (int d = 0; d < DT; d++) o[i][d] *= alpha;
-                m_run[i] = m_new;
+            for (int i = 0; i < TQ; i++) grouped_mask(s[i], qpos[i] - kt * 64, p.window, fg);
+        if constexpr (!FAST) {
+            float m_new[TQ];
+            bool moved = false;
+#pragma unroll
+            for (int i = 0; i < TQ; i++) {
+                m_new[i] = vmax2(m_run[i], rows_max(vmax16(s[i][0], s[i][1], s[i][2], s[i][3])));
+                moved |= m_new[i] > m_run[i] + 8.0f;            // (weights up to 2^8 over the reference do no harm)
             }
+            if (__any(moved)) {
+#pragma unroll
+                for (int i = 0; i < TQ; i++) {
+                    const float alpha = __builtin_amdgcn_exp2f(m_run[i] - m_new[i]);
+                    lacc[i] *= alpha;
+#pragma unroll
+                    for (int d = 0; d < DT; d++) o[i][d] *= alpha;
+                    m_run[i] = m_new[i];
+                }
+            }
+        }
+#pragma unroll
+        for (int i = 0; i < TQ; i++)
 #pragma unroll
             for (int t = 0; t < 4; t++)
 #pragma unroll
-                for (int r = 0; r < 4; r++) s[i][t][r] = __builtin_amdgcn_exp2f(s[i][t][r] - m_new);
-        }
+                for (int r = 0; r < 4; r++) s[i][t][r] = __builtin_amdgcn_exp2f(FAST ? s[i][t][r] : s[i][t][r] - m_run[i]);
 #pragma unroll
         for (int u = 0; u < 2; u++) {
             bf16x8 pf[TQ];

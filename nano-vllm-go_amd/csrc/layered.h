@@ -520,6 +520,11 @@ void layered_finalize(nvl_model* m) {
                 if (l.t[NVL_T_BIAS_R1].present()) {
                     w.r1 = lay_vector(m, l.t[NVL_T_BIAS_R1], c.heads);
                     w.r2 = lay_vector(m, T(NVL_T_BIAS_R2, "distance bias (r2)"), c.heads);
+                    std::vector<float> v((size_t)c.heads * 2);
+                    NVL_HIP(hipMemcpyAsync(v.data(), w.r1, (size_t)c.heads * 4, hipMemcpyDeviceToHost, m->stream));
+                    NVL_HIP(hipMemcpyAsync(v.data() + c.heads, w.r2, (size_t)c.heads * 4, hipMemcpyDeviceToHost, m->stream));
+                    NVL_HIP(hipStreamSynchronize(m->stream));
+                    w.bias_lowers = std::all_of(v.begin(), v.end(), [](float x) { return x >= 0.f; });
                 }
                 if (c.v_mix) w.v_lambda = lay_vector(m, T(NVL_T_V_MIX, "value mixing"), 1);
                 w.o = lay_matrix(m, H, r.kd);
@@ -1303,16 +1308,18 @@ void mix_grouped(nvl_model* m, const LayerRun& r, const MixerW& w, const Meta& m
     if (any_long) {
         KScope scp = scope(1);
         const dim3 grid(a.G, n_seqs, cdiv((int64_t)max_len * a.group, 256));
-#define NVL_GP(KSv, DTv)                                                                                                     \
+#define NVL_GPF(KSv, DTv, FASTv)                                                                                             \
         do {                                                                                                                 \
-            NVL_LDS_ATTR((grouped_prefill_kernel<KSv, DTv>), 160 * 1024);                                                    \
-            hipLaunchKernelGGL((grouped_prefill_kernel<KSv, DTv>), grid, dim3(512), lds, m->stream, a);                      \
+            NVL_LDS_ATTR((grouped_prefill_kernel<KSv, DTv, FASTv>), 160 * 1024);                                             \
+            hipLaunchKernelGGL((grouped_prefill_kernel<KSv, DTv, FASTv>), grid, dim3(512), lds, m->stream, a);               \
         } while (0)
+#define NVL_GP(KSv, DTv) do { if (a.table && w.bias_lowers && c.softcap > 0.f && c.softcap <= GROUPED_FAST_CAP) NVL_GPF(KSv, DTv, true); else NVL_GPF(KSv, DTv, false); } while (0)
 #define NVL_GPK(KSv) do { if (dt == 2) NVL_GP(KSv, 2); else if (dt == 4) NVL_GP(KSv, 4); else if (dt == 8) NVL_GP(KSv, 8); else NVL_GP(KSv, 16); } while (0)
         if (ks == 1) NVL_GPK(1); else if (ks == 2) NVL_GPK(2); else if (ks == 4) NVL_GPK(4);
         else if (dt == 2) NVL_GP(8, 2); else if (dt == 4) NVL_GP(8, 4); else NVL_GP(8, 8);
 #undef NVL_GPK
 #undef NVL_GP
+#undef NVL_GPF
         NVL_HIP(hipGetLastError());
     }
     if (any_short) {

@@ -84,6 +84,7 @@ struct MixerW {
     void *a2m = nullptr, *g2m = nullptr;     // channel delta: the second decay / gate projections as GEMM operands ...
     void *a2r = nullptr, *g2r = nullptr;     // ... and row-major for the one-token step
     int grank = 0, a_rkp = 0, g_rkp = 0;
+    bool bias_lowers = false;    // r1, r2 >= 0 for every head
     float *norm1_bias = nullptr, *r1 = nullptr, *r2 = nullptr, *v_lambda = nullptr;       // grouped attention, parallel blocks
     void *moe_up = nullptr, *moe_down = nullptr, *moe_cat = nullptr;                      // experts: [E][2 Ip][H], [E][H][Ip], bf16: [H][Ep Ip]
     float* route_bias = nullptr;

@@ -26,7 +26,8 @@ att, moe = BM.attention, BM.moe
 SINGLE = {      # layer, width, side
     "odd": (att(), 96, 20), "no-window": (att(window=None), 96, 20), "window-1": (att(window=1), 64, 20), "window-63": (att(window=63), 64, 20),
     "window-64": (att(window=64), 64, 20), "window-65": (att(window=65), 64, 20), "no-cap": (att(cap=None), 64, 20), "tight-cap": (att(cap=0.7, scale=0.6), 64, 20),
-    "negative-scale": (att(scale=-0.3), 64, 20), "one-head-each": (att(heads=3, kv_heads=3), 96, 20), "one-kv-head": (att(heads=5, kv_heads=1), 96, 20),
+    "negative-scale": (att(scale=-0.3), 64, 20), "wide-cap": (att(cap=59.0, scale=9.0), 64, 20), "wider-cap": (att(cap=200.0, scale=9.0), 64, 20),
+    "no-cap-long-table": (att(cap=None, window=None, heads=24, kv_heads=1, dim=64, vdim=64), 64, 20), "one-head-each": (att(heads=3, kv_heads=3), 96, 20), "one-kv-head": (att(heads=5, kv_heads=1), 96, 20),
     "group-17": (att(heads=34, kv_heads=2, dim=16, vdim=8, window=100), 96, 20), "group-70": (att(heads=70, kv_heads=1, dim=12, vdim=5), 64, 20),
     "32-32": (att(dim=32, vdim=32), 64, 20), "64-64": (att(heads=4, kv_heads=1, dim=64, vdim=64, window=None), 128, 64), "128-128": (att(heads=4, kv_heads=2, dim=128, vdim=128), 128, 20),
     "20-160": (att(heads=2, kv_heads=1, dim=20, vdim=160), 64, 20), "200-40": (att(heads=2, kv_heads=2, dim=200, vdim=40), 64, 20), "150-100": (att(heads=2, kv_heads=1, dim=150, vdim=100), 64, 20),
@@ -224,6 +225,20 @@ def test_distance_bias_places_the_keys(gpu, tmp_path, precision):
         assert err(O.forward(cfg, w, tok), want) > 0.1
     finally:
         O.distance_bias = keep
+    m = build(gpu, tmp_path, cfg, w, precision)
+    for s, cuts in enumerate(([300], [250] + [1] * 50, cut(300, 33))):
+        assert err(feed(m, s, tok, cuts), want, precision) < ONE[precision]
+    m.close()
+
+
+@pytest.mark.parametrize("precision", ["f32", "bf16"])
+@pytest.mark.parametrize("r1,r2", [((-1.5, -0.5), (0.1, 0.4)), ((0.0, 0.0), (0.0, 0.0)), ((20.0, 40.0), (1.0, 3.0))])
+def test_distance_bias_of_any_sign_and_size(gpu, tmp_path, r1, r2, precision):
+    """Biases that raise far scores (a running maximum is needed), that are zero, and that bury everything but the nearest keys."""
+    cfg = BM.config([att(heads=4, kv_heads=2, dim=32, vdim=32, window=None, mlp=None)], width=64, vocab=70, side=4, positions=300)
+    w = BM.weights(cfg, 48, r1=r1, r2=r2)
+    tok = np.random.default_rng(10).integers(0, 70, 300).tolist()
+    want = O.forward(cfg, w, tok)
     m = build(gpu, tmp_path, cfg, w, precision)
     for s, cuts in enumerate(([300], [250] + [1] * 50, cut(300, 33))):
         assert err(feed(m, s, tok, cuts), want, precision) < ONE[precision]
