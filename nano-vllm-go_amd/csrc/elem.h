@@ -974,12 +974,26 @@ __global__ __launch_bounds__(1024) void moe_plan_kernel(const float* __restrict_
 // Group-limited routing on sigmoid scores.  s = sigmoid(z); the choice goes by s + correction, the weights are the s of the chosen
 // experts as they are.  Experts form `groups` equal groups of neighbours; a group counts as much as its two largest choice scores
 // together, and only the experts of the best `keep` groups can be chosen.  Ties go to the lower index.  One wave per token, E <= 256;
-// writes (id, weight) in rank order, or with `gate` the dense [rows][gate_ld] matrix of weights (0: not chosen).
+// writes (id, weight) in rank order, or with `gate` the dense [rows][gate_ld] matrix of weights (0: not chosen).  Workgroups with
+// blockIdx.y > 0 finish a SwiGLU feed-forward whose fp32 gate and up columns the same projection made (a small shared expert):
+// grid (ceil(rows / 4), 1 + ceil(F / 256)).
 constexpr int ROUTE_MAX_E = 256;
-struct GroupRouteArgs { const float* logits; int64_t ld; const float* correction; int rows, E, top, groups, keep; int32_t* ids; float* w; float* gate; int gate_ld; };
+struct GroupRouteArgs { const float* logits; int64_t ld; const float* correction; int rows, E, top, groups, keep; int32_t* ids; float* w; float* gate; int gate_ld;
+                        const float* glu; int F; void* out; int64_t out_ld; int out_col; };      // glu: [rows][ld] = [gate F | up F]; out: columns out_col ..
+template <typename ActT>
 __global__ __launch_bounds__(256) void moe_route_grouped_kernel(GroupRouteArgs p) {
     __shared__ float choice_s[4][ROUTE_MAX_E], group_s[4][ROUTE_MAX_E];
     const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, r = blockIdx.x * 4 + wave;
+    if (blockIdx.y > 0) {
+        const int f = (blockIdx.y - 1) * 256 + lane * 4;
+        if (r >= p.rows || f >= p.F) return;
+        const float* g = p.glu + (int64_t)r * p.ld + f;
+        f32x4 v;
+#pragma unroll
+        for (int k = 0; k < 4; k++) v[k] = g[k] / (1.0f + expf(-g[k])) * g[p.F + k];
+        act_store4<ActT>((ActT*)p.out, r, p.out_col + f, p.out_ld, v);
+        return;
+    }
     const int size = p.E / p.groups;
     float *choice = choice_s[wave], *group = group_s[wave];
     float s[ROUTE_MAX_E / 64];

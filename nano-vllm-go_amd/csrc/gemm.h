@@ -67,8 +67,8 @@ struct GroupedEpi {         // EPI_GROUPED: columns [q | k | v | gate | feed-for
     const int32_t *tok_pos, *tok_tbl, *blk_table;
     bf16_t* cache; int64_t block_stride; int bs, G, dp, vp;        // this layer's part of block 0 (grouped.h)
     int mix; const float* lambda; float* vfirst; int64_t vfirst_ld;
-    bf16_t* ffn; int64_t ffn_ld;                                   // max(., 0)^2 -> the output projection's operand (fragment-major, shifted to its columns)
-    float* route; int64_t route_ld;                                // fp32 rows
+    bf16_t* ffn; int64_t ffn_ld;                                   // [ffn0, route0): max(., 0)^2 -> the output projection's operand (fragment-major, shifted to its columns)
+    float* route; int64_t route_ld;                                // from route0 on: fp32 rows
 };
 
 struct GemmArgs {
@@ -145,6 +145,7 @@ __device__ __forceinline__ void epilogue_grouped4(const GemmArgs& p, int64_t row
     if (n < e.k0) { act_store4<bf16_t>((bf16_t*)p.C, row, n, p.ldc, v); return; }
     if (n >= e.route0) {
         float* c = e.route + row * e.route_ld + (n - e.route0);
+        if (n + 3 < p.N) { *(f32x4*)c = v; return; }      // (rows of 4 k floats)
 #pragma unroll
         for (int r = 0; r < 4; r++) if (n + r < p.N) c[r] = v[r];
         return;

@@ -23,6 +23,7 @@ namespace {
 
 constexpr float CLAMPED_GLU_SLOPE = 1.702f;
 constexpr int LAT_ABSORB_MAX = 16, LAT_ABSORB_MAX_RP = 512, REC_STEP_MAX = 4;
+constexpr int GLU_IN_MAX = 1024;       // widest shared expert whose gate and up columns pass through fp32 rows instead of a launch of their own
 constexpr int GROUPED_SHORT_ROWS = 64, GROUPED_SPLIT_WGS = 512;      // GROUPED_SPLIT_WGS: workgroups of a launch whose keys are split
 
 bool same_rotation(const nvl_layer_config& a, const nvl_layer_config& b) {
@@ -166,7 +167,8 @@ int layered_create(const nvl_model_config& c, const nvl_layer_config* layers, co
                 r.dp = pad_head(r.c.dim, 64); r.vp = pad_head(r.c.vdim, 64);
                 r.k_off = H * r.dp; r.v_off = r.k_off + G * r.dp; r.gate_off = r.v_off + G * r.vp; r.ffn_off = r.gate_off + H * r.vp;
                 r.ffn_in = par && r.c.ffn_dim && r.act == NVL_ACT_RELU2;
-                r.route_off = r.ffn_off + (r.ffn_in ? r.Fp : 0);
+                r.glu_in = par && r.c.experts && r.c.ffn_dim && r.act == NVL_ACT_SWIGLU && r.Fp <= GLU_IN_MAX;
+                r.route_off = r.ffn_off + (r.ffn_in ? r.Fp : r.glu_in ? 2 * r.Fp : 0);
                 r.n_in = r.route_off + r.c.experts; r.ko = (int)round_up((int64_t)H * r.vp, 64);
                 r.cache_off = cache; cache += (int64_t)bs * G * (r.dp + r.vp);
                 if (r.c.v_mix) {
@@ -448,8 +450,8 @@ void layered_finalize(nvl_model* m) {
                 if (!post && !par) w.norm2 = lay_norm(m, T(NVL_T_FFN_NORM_W, "norm before the feed-forward"), H);
                 if (!par) w.norm2b = lay_norm(m, T(NVL_T_FFN_POST_NORM, "norm after the feed-forward"), H, &l.t[NVL_T_FFN_SCALE]);
                 const DevTensor& w1 = T(NVL_T_W1, "feed-forward gate / up");
-                if (!r.ffn_in) w.w1 = lay_matrix(m, (r.act == NVL_ACT_RELU2 ? 1 : 2) * r.Fp, H);
-                if (r.ffn_in) {}
+                if (!r.ffn_in && !r.glu_in) w.w1 = lay_matrix(m, (r.act == NVL_ACT_RELU2 ? 1 : 2) * r.Fp, H);
+                if (r.ffn_in || r.glu_in) {}      // (rows of the fused input projection)
                 else if (r.act == NVL_ACT_RELU2) lay_place(m, w1, w.w1, H);
                 else if (m->f32) { lay_place(m, w1, w.w1, H, 0, 0, 0, 0, 0, 0, c.ffn_dim); lay_place(m, w1, w.w1, H, r.Fp, 0, 0, 0, 0, c.ffn_dim, c.ffn_dim); }
                 else { lay_place(m, w1, w.w1, H, 0, 16, 32, 0, 0, 0, c.ffn_dim); lay_place(m, w1, w.w1, H, 16, 16, 32, 0, 0, c.ffn_dim, c.ffn_dim); }
@@ -590,6 +592,7 @@ void layered_finalize(nvl_model* m) {
                 lay_place(m, T(NVL_T_WO, "output projection"), w.o, r.kd);
             }
             if (r.ffn_in) lay_place(m, T(NVL_T_W1, "feed-forward up"), w.in, H, r.ffn_off);
+            if (r.glu_in) lay_place(m, T(NVL_T_W1, "feed-forward gate / up"), w.in, H, r.ffn_off, c.ffn_dim, r.Fp);
             if (c.experts) lay_place(m, T(NVL_T_ROUTER, "router"), w.in, H, r.route_off);
             if (par && c.ffn_dim) lay_place(m, T(NVL_T_W2, "feed-forward down"), w.o, r.kd, 0, 0, 0, 0, 0, 0, -1, false, false, r.ko);
             NVL_HIP(hipStreamSynchronize(m->stream));
@@ -613,7 +616,7 @@ void layered_finalize(nvl_model* m) {
         }
         if (c.mixer == NVL_MIXER_GLA) r.n_in = 2 * c.heads * (c.dim + c.vdim) + m->mixers[(size_t)r.owner].rank;
         const bool qg = c.mixer == NVL_MIXER_ATTENTION && !m->f32;           // (its projection goes to lqg, the cache and lmix; the router's columns stay)
-        ld_in = std::max(ld_in, round_up(qg ? r.n_in - r.route_off : r.n_in, 4));
+        ld_in = std::max(ld_in, round_up(qg ? r.n_in - (r.ffn_in ? r.route_off : r.ffn_off) : r.n_in, 4));
         if (qg) qg_cols = std::max<int64_t>(qg_cols, (int64_t)c.heads * (r.dp + r.vp));
         ko = std::max<int64_t>(ko, r.kd);
         Fmax = std::max<int64_t>(Fmax, r.Fp);
@@ -1274,7 +1277,7 @@ void mix_grouped(nvl_model* m, const LayerRun& r, const MixerW& w, const Meta& m
     } else {
         a.q = m->lqg; a.q_ld = (int64_t)a.H * (r.dp + r.vp); a.gate_col = a.H * r.dp;
         GemmArgs g = mk(m->xn, m->H, w.in, m->lqg, (int)a.q_ld, nullptr, 1.f, M, r.n_in, m->H);
-        g.grp = GroupedEpi{r.k_off, r.v_off, r.gate_off, r.ffn_off, r.route_off, md.tok_pos, md.tok_tbl, md.blk_table, (bf16_t*)a.cache, a.block_stride, a.bs, a.G, r.dp, r.vp,
+        g.grp = GroupedEpi{r.k_off, r.v_off, r.gate_off, r.ffn_off, r.ffn_in ? r.route_off : r.ffn_off, md.tok_pos, md.tok_tbl, md.blk_table, (bf16_t*)a.cache, a.block_stride, a.bs, a.G, r.dp, r.vp,
                            r.mix, w.v_lambda, m->lvf, m->lvf_ld, (bf16_t*)m->lmix + (r.ko >> 5) * 512, r.kd, m->lproj, m->lproj_ld};
         m->site = KS_MIX_IN;
         gemm(m, EPI_GROUPED, false, g);
@@ -1355,7 +1358,7 @@ ExpertOut parallel_ffn(nvl_model* m, const LayerRun& r, const MixerW& w, int M) 
         KScope ks(m, KC_OTHER);
         hipLaunchKernelGGL((relu2_kernel<float>), dim3(cdiv(n, 256)), dim3(256), 0, m->stream, m->lproj + r.ffn_off, m->lproj_ld, (float*)m->lmix, (int64_t)M, r.Fp, (int64_t)r.kd, r.ko);
         NVL_HIP(hipGetLastError());
-    } else if (c.ffn_dim && !r.ffn_in) {
+    } else if (c.ffn_dim && !r.ffn_in && !r.glu_in) {
         m->site = KS_FFN_UP;
         const bool relu2 = r.act == NVL_ACT_RELU2;
         const int N = relu2 ? r.Fp : 2 * r.Fp;
@@ -1373,10 +1376,14 @@ ExpertOut parallel_ffn(nvl_model* m, const LayerRun& r, const MixerW& w, int M) 
     const int E = c.experts, k = c.top_k, pairs = M * k;
     // decode: all experts as one projection each way with the routing weights as a mask (gemm.h GemmArgs::moe_gate)
     const bool dense = !m->f32 && M <= 64 && r.Ip <= 2048;
-    GroupRouteArgs ra{m->lproj + (m->f32 ? r.route_off : 0), m->lproj_ld, w.route_bias, M, E, k, c.expert_groups, c.groups_kept, m->expert_ids, m->expert_w, dense ? m->moe_gate : nullptr, r.Ep};
+    const float* tail = m->lproj + (m->f32 ? r.ffn_off : 0);          // [a small shared expert's gate | up |] router logits
+    GroupRouteArgs ra{m->f32 ? m->lproj + r.route_off : tail + (r.glu_in ? 2 * r.Fp : 0), m->lproj_ld, w.route_bias, M, E, k, c.expert_groups, c.groups_kept, m->expert_ids, m->expert_w, dense ? m->moe_gate : nullptr, r.Ep,
+                      tail, r.Fp, m->lmix, r.kd, r.ko};
     {
-        KScope ks(m, KC_OTHER, 0, KS_MOE_ROUTER, (double)M * (E + 2.0 * k) * 4.0);
-        hipLaunchKernelGGL(moe_route_grouped_kernel, dim3(cdiv(M, 4)), dim3(256), 0, m->stream, ra);
+        KScope ks(m, KC_OTHER, 0, KS_MOE_ROUTER, (double)M * ((E + 2.0 * k) * 4.0 + (r.glu_in ? c.ffn_dim * (8.0 + (double)m->wsize) : 0.0)));
+        const dim3 grid(cdiv(M, 4), 1 + (r.glu_in ? cdiv(r.Fp, 256) : 0));
+        if (m->f32) hipLaunchKernelGGL((moe_route_grouped_kernel<float>), grid, dim3(256), 0, m->stream, ra);
+        else hipLaunchKernelGGL((moe_route_grouped_kernel<bf16_t>), grid, dim3(256), 0, m->stream, ra);
         NVL_HIP(hipGetLastError());
     }
     const double touch = (double)std::min(E, pairs);

@@ -66,7 +66,8 @@ struct LayerRun {
     int win = -1;                // index into nvl_model::windows
     int64_t cache_off = 0;       // attention: element offset inside a cache block
     int k_off = 0, v_off = 0, ffn_off = 0, route_off = 0;     // grouped attention: columns of the fused input projection (keys, values, feed-forward, router)
-    bool ffn_in = false;         // ... whose feed-forward columns are the whole up projection (ungated activations)
+    bool ffn_in = false;         // ... whose feed-forward columns are the whole up projection (ungated activations),
+    bool glu_in = false;         // or gate and up of a small shared expert, finished by the router's launch
     int mix = 0;                 // grouped attention: GroupedArgs::mix
     int kd = 0;                  // K of the joint output projection of a parallel block: ko, then the feed-forward's Fp columns
     int act = 0;                 // activation of the feed-forward

@@ -25,13 +25,13 @@ def attention(heads=6, kv_heads=2, dim=40, vdim=24, window=50, scale=0.2, cap=9.
 
 
 def config(layers, width=160, vocab=331, eps=1e-5, side=20, positions=700):
-    return dict(architecture="Bolinex", vocab=vocab, width=width, norm=dict(eps=eps), token_side=dict(dim=side), max_positions=positions, layers=layers)
+    return dict(architecture="Bolinex", vocab=vocab, width=width, norm=dict(eps=eps), token_side=None if side is None else dict(dim=side), max_positions=positions, layers=layers)
 
 
 def weights(cfg, seed=0, r1=(0.02, 2.0), r2=(0.05, 0.5), correction=(-2.2, 0.7)):
     """{tensor name: fp32 array whose values are bf16}.  r1, r2: ranges; correction: mean and spread."""
     g = np.random.default_rng(seed)
-    W, V, sd, L = cfg["width"], cfg["vocab"], cfg["token_side"]["dim"], len(cfg["layers"])
+    W, V, sd, L = cfg["width"], cfg["vocab"], (cfg["token_side"] or {}).get("dim", 0), len(cfg["layers"])
     t = {}
 
     def mat(name, out, inn, s=1.0):
@@ -47,7 +47,8 @@ def weights(cfg, seed=0, r1=(0.02, 2.0), r2=(0.05, 0.5), correction=(-2.2, 0.7))
 
     t["embed"] = bf16(g.standard_normal((V, W)))
     t["pos"] = bf16(0.4 * g.standard_normal((cfg["max_positions"], W)))
-    t["side.embed"] = bf16(g.standard_normal((V, L * sd)))
+    if sd:
+        t["side.embed"] = bf16(g.standard_normal((V, L * sd)))
     mat("head", V, W, 2.0)
     norm("final.norm", W)
     for i, ly in enumerate(cfg["layers"]):
@@ -58,7 +59,8 @@ def weights(cfg, seed=0, r1=(0.02, 2.0), r2=(0.05, 0.5), correction=(-2.2, 0.7))
         t[m + "r1"], t[m + "r2"] = bf16(g.uniform(*r1, H)), bf16(g.uniform(*r2, H))
         if mx["v_mix"]:
             t[m + "vmix"] = bf16(np.float32(g.uniform(0.2, 0.8)))
-        mat(p + "side.gate", sd, W); mat(p + "side.proj", W, sd); norm(p + "side.norm", W, False)
+        if sd:
+            mat(p + "side.gate", sd, W); mat(p + "side.proj", W, sd); norm(p + "side.norm", W, False)
         if mlp is None:
             continue
         if mlp["kind"] == "dense":

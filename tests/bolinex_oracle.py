@@ -135,8 +135,9 @@ def forward(cfg, weights, tokens, return_layers=False, margins=None):
         if ly["mixer"].get("v_mix") and first is None:
             first = v
         x = x + (y + feed_forward(h, sub(weights, f"l{i}.mlp."), ly["mlp"], margins))
-        n = cfg["token_side"]["dim"]
-        x = x + token_side(x, np.asarray(weights["side.embed"], np.float64)[tok, i * n:(i + 1) * n], sub(weights, f"l{i}.side."), eps)
+        if cfg.get("token_side"):
+            n = cfg["token_side"]["dim"]
+            x = x + token_side(x, np.asarray(weights["side.embed"], np.float64)[tok, i * n:(i + 1) * n], sub(weights, f"l{i}.side."), eps)
         layers.append(x)
     logits = layer_norm(x, *(np.asarray(weights["final.norm" + b], np.float64) for b in ("", ".b")), eps) @ np.asarray(weights["head"], np.float64).T
     return (logits, np.stack(layers)) if return_layers else logits

@@ -33,7 +33,8 @@ SINGLE = {      # layer, width, side
     "20-160": (att(heads=2, kv_heads=1, dim=20, vdim=160), 64, 20), "200-40": (att(heads=2, kv_heads=2, dim=200, vdim=40), 64, 20), "150-100": (att(heads=2, kv_heads=1, dim=150, vdim=100), 64, 20),
     "256-256": (att(heads=4, kv_heads=2, dim=250, vdim=256, scale=0.06), 96, 20), "big-heads": (att(heads=2, kv_heads=1, dim=272, vdim=264, scale=0.05), 64, 20),
     "narrow": (att(heads=1, kv_heads=1, dim=4, vdim=4, mlp=BM.dense(5)), 12, 3), "wide-row": (att(heads=2, kv_heads=1, mlp=BM.dense(16)), 1100, 20),
-    "no-feed-forward": (att(mlp=None), 96, 20), "dense-200": (att(mlp=BM.dense(200)), 70, 100), "side-5": (att(mlp=None), 64, 5), "side-300": (att(mlp=None), 64, 300),
+    "no-feed-forward": (att(mlp=None), 96, 20), "dense-200": (att(mlp=BM.dense(200)), 70, 100), "side-5": (att(mlp=None), 64, 5), "side-300": (att(mlp=None), 64, 300), "no-side": (att(mlp=moe()), 64, None),
+    "shared-1100": (att(mlp=moe(4, 2, None, 24, 1100)), 64, 20),
     "experts": (att(mlp=moe()), 96, 20), "experts-5-of-one-group": (att(mlp=moe(5, 2, None, 24, None)), 64, 20), "one-expert": (att(mlp=moe(1, 1, None, 24, 30)), 64, 20),
     "experts-40": (att(mlp=moe(40, 6, (8, 3), 16, 8)), 64, 20), "experts-72": (att(mlp=moe(72, 5, (9, 4), 12, None)), 64, 20), "groups-of-one": (att(mlp=moe(6, 2, (6, 3), 24)), 64, 20),
     "all-of-the-kept": (att(mlp=moe(8, 4, (4, 2), 24)), 64, 20), "every-expert": (att(mlp=moe(6, 6, (3, 3), 24)), 64, 20), "wide-experts": (att(mlp=moe(6, 2, (2, 1), 200, 136)), 256, 20),
