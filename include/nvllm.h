@@ -541,8 +541,9 @@ int nvl_bench_gemm(int device, int M, int N, int K, int epi, int force_bnt, int 
  * fills the chip (>= 160 workgroups) or the batch is one sequence; 0 never; 2 always.
  * key 36: weight tiles per wave of the wide decode projections (FFN-up, LM head): 0 (default) 2 for 17..32 rows and N < 65536, else 4;
  * 2 / 4 forced.
+ * key 37: workgroups the keys of a row tile are split over in the short grouped attention (lists of layers): 0 (default) from the context.
  * key 33: MoE decode: the experts' down projection carries the next RMSNorm (no K slices, no norm launch before the next QKV);
- * 0 (default): measured slower (rejected list (27)).
+ * 0 (default): measured slower.
  * The settings are PROCESS-GLOBAL and unsynchronised (every model in the process sees them): set them from one thread
  * while no forward call is running.  Every call starts a new tuning epoch: captured decode graphs bake the tuning in and are re-captured.
  * Returns the previous value. */

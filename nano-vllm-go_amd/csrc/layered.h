@@ -19,6 +19,8 @@
 //     query rows; recurrences go token by token up to REC_STEP_MAX.
 #pragma once
 
+static int g_grouped_split = 0;      // nvl_set_tuning key 37: key splits of the short grouped attention (1 .. 16); 0 = automatic
+
 namespace {
 
 constexpr float CLAMPED_GLU_SLOPE = 1.702f;
@@ -463,8 +465,9 @@ void layered_finalize(nvl_model* m) {
             if (c.experts) {
                 const int64_t E = c.experts, I = c.expert_dim, Ip = r.Ip;
                 const DevTensor &up = T(NVL_T_MOE_IN, "experts' gate / up"), &down = T(NVL_T_MOE_OUT, "experts' down");
-                w.moe_up = lay_matrix(m, E * 2 * Ip, H);
-                w.moe_down = lay_matrix(m, E * H, Ip);
+                // (a grouped launch reads whole column tiles of its expert's rows: the last expert's need rows behind them)
+                w.moe_up = lay_matrix(m, (E - 1) * 2 * Ip + round_up(2 * Ip, W_ROW_PAD), H);
+                w.moe_down = lay_matrix(m, (E - 1) * H + round_up(H, W_ROW_PAD), Ip);
                 if (!m->f32) w.moe_cat = lay_matrix(m, H, r.Ep * Ip);
                 for (int64_t e = 0; e < E; e++) {
                     const int64_t row = e * 2 * Ip, from = e * 2 * I;
@@ -643,7 +646,7 @@ void layered_finalize(nvl_model* m) {
     m->x = dmalloc<float>(Mmax * H);
     m->xn = dmalloc_bytes(Mp * H * ws);
     ld_in = std::max<int64_t>(ld_in, 4);
-    const int64_t hbuf = std::max(Mp * m->F, round_up(Mmax * std::max<int64_t>(moe_k, 1), 64) * (moe_k ? moe_kI / moe_k : 0) + 64 * moe_kI);
+    const int64_t hbuf = std::max(Mp * m->F, (Mmax + 64) * moe_kI);      // (pairs, rounded up to whole tiles, x the experts' width)
     m->hbuf = dmalloc_bytes(hbuf * ws);
     m->xn_last = dmalloc_bytes(round_up(S, 64) * H * ws);
     NVL_HIP(hipMemsetAsync(m->xn, 0, (size_t)(Mp * H * ws), m->stream));
@@ -1328,24 +1331,24 @@ void mix_grouped(nvl_model* m, const LayerRun& r, const MixerW& w, const Meta& m
     if (any_short) {
         KScope scp = scope(any_long ? 0 : max_len > 1);
         const int64_t wgs = (int64_t)a.G * cdiv(std::min<int64_t>((int64_t)max_len * a.group, a.short_rows), 16);
-        // eight waves a workgroup when the row tiles alone come near the CUs' number; else four, and the keys split over workgroups
-        const int key_tiles = 1 << layered_kt_log2(m);
-        const bool wide = dt <= 8 && wgs * n_seqs >= 96;
+        // Key tiles are split over workgroups once a wave would walk more than two: a split costs a round trip to memory and back (one
+        // sequence of 2048 tokens with a window of 1024: 13.1 us unsplit, 13.7 in four; without a window, 3900 tokens: 27.8 -> 16.6 us)
+        const int key_tiles = 1 << layered_kt_log2(m), nw = dt <= 8 ? 8 : 4;
         int z = 1;
-        while (!wide && z < GROUPED_SPLITS && wgs * n_seqs * z * 2 <= 256 && z * 2 * 4 <= key_tiles) z *= 2;
+        while (z < GROUPED_SPLITS && wgs * n_seqs * z * 2 <= 256 && z * 2 * 2 * nw <= key_tiles) z *= 2;
+        if (g_grouped_split) z = (int)std::min<int64_t>(g_grouped_split, std::max<int64_t>(1, m->grp_cap / (wgs * n_seqs)));
         a.part = m->grp_part; a.part_cnt = m->grp_cnt;
         const dim3 grid((unsigned)wgs, n_seqs, z);
-#define NVL_GSW(KSv, DTv, NWv)                                                                                               \
+#define NVL_GS(KSv, DTv)                                                                                                     \
         do {                                                                                                                 \
-            NVL_LDS_ATTR((grouped_short_kernel<KSv, DTv, NWv>), NWv * DTv * 1024);                                           \
-            hipLaunchKernelGGL((grouped_short_kernel<KSv, DTv, NWv>), grid, dim3(NWv * 64), NWv * DTv * 1024, m->stream, a); \
+            constexpr int nw_ = DTv <= 8 ? 8 : 4;                                                                            \
+            NVL_LDS_ATTR((grouped_short_kernel<KSv, DTv, nw_>), nw_ * DTv * 1024);                                           \
+            hipLaunchKernelGGL((grouped_short_kernel<KSv, DTv, nw_>), grid, dim3(nw_ * 64), nw_ * DTv * 1024, m->stream, a); \
         } while (0)
-#define NVL_GS(KSv, DTv) do { if (wide) NVL_GSW(KSv, DTv, (DTv <= 8 ? 8 : 4)); else NVL_GSW(KSv, DTv, 4); } while (0)
 #define NVL_GSK(KSv) do { if (dt == 2) NVL_GS(KSv, 2); else if (dt == 4) NVL_GS(KSv, 4); else if (dt == 8) NVL_GS(KSv, 8); else NVL_GS(KSv, 16); } while (0)
         if (ks == 1) NVL_GSK(1); else if (ks == 2) NVL_GSK(2); else if (ks == 4) NVL_GSK(4); else NVL_GSK(8);
 #undef NVL_GSK
 #undef NVL_GS
-#undef NVL_GSW
         NVL_HIP(hipGetLastError());
     }
 }

@@ -532,7 +532,9 @@ extern "C" int nvl_upload_tensor(nvl_model* m, int kind, int layer, const void* 
                      (long long)cols, (long long)out, (long long)in);
             return fail(m, NVL_ERR_INVALID, buf);
         }
-        upload_2d(m, t, data, dtype, rows, cols, false, Slice2D{rows, cols, 0, 0, 0}, rows, true);
+        // (a grouped launch reads whole column tiles of its expert's rows: the last expert's need rows behind them)
+        upload_2d(m, t, data, dtype, rows, cols, false, Slice2D{rows, cols, 0, 0, 0}, (E - 1) * out + round_up(out, W_ROW_PAD), true);
+        t->rows = rows;
         return NVL_OK;
     }
     if (kind >= NVL_T_MAMBA_IN_PROJ && !m->n_mamba) return fail(m, NVL_ERR_INVALID, "nvl_upload_tensor: the model has no Mamba2 layers");

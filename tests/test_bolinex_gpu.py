@@ -271,6 +271,25 @@ def test_expert_forms_agree(gpu, tmp_path, rows):
     m.close()
 
 
+@pytest.mark.parametrize("heads,kv_heads,dim,vdim,window", [(6, 2, 40, 24, None), (4, 1, 64, 128, 300), (20, 1, 20, 200, None)])
+def test_key_splits(gpu, tmp_path, heads, kv_heads, dim, vdim, window):
+    """Decoding and short portions with the keys split over workgroups: any number of splits, captured passes included."""
+    cfg = BM.config([att(heads=heads, kv_heads=kv_heads, dim=dim, vdim=vdim, window=window), att(heads=heads, kv_heads=kv_heads, dim=dim, vdim=vdim, window=window, mlp=None)],
+                    width=128, vocab=90, positions=460)
+    w = BM.weights(cfg, 16)
+    tok, want, _ = BM.clear_tokens(cfg, w, 450, 6)
+    m = build(gpu, tmp_path, cfg, w, "bf16")
+    lib = gpu.lib()
+    try:
+        for i, n in enumerate((1, 2, 3, 7, 16)):
+            lib.nvl_set_tuning(37, n)
+            assert err(feed(m, i, tok, [400] + [1] * 20 + [3] * 10), want, "bf16") < ONE["bf16"], n
+            m.seq_close(i)
+    finally:
+        lib.nvl_set_tuning(37, 0)
+    m.close()
+
+
 # ---- the framework's own entry points ----
 def test_greedy_generation(gpu, tmp_path, stack):
     """Stepwise, fused on the device, and through the runner give the restatement's tokens (fp32)."""
