@@ -636,13 +636,16 @@ __global__ void relu2_kernel(const float* __restrict__ h, int64_t h_ld, ActT* __
     const float v = fmaxf(h[r * h_ld + f], 0.f);
     ActIO<ActT>::st(y + act_index<ActT>(r, col + f, ld), v * v);
 }
-// h [rows][n] -> y [rows][ld]: gelu_tanh(h) * (the token's row of a table)
+// h [slices][rows][h_ld], summed -> y [rows][ld]: gelu_tanh(h) * (the token's row of a table)
 template <typename ActT, typename TabT>
-__global__ void gelu_token_kernel(const float* __restrict__ h, int64_t h_ld, const TabT* __restrict__ table, int64_t table_ld, const int32_t* __restrict__ ids,
+__global__ void gelu_token_kernel(const float* __restrict__ h, int64_t h_ld, int slices, int64_t stride, const TabT* __restrict__ table, int64_t table_ld, const int32_t* __restrict__ ids,
                                   ActT* __restrict__ y, int64_t ld, int n) {
     const int64_t r = blockIdx.x;
-    for (int i = threadIdx.x; i < n; i += blockDim.x)
-        ActIO<ActT>::st(y + act_index<ActT>(r, i, ld), gelu_tanh_f(h[r * h_ld + i]) * (float)table[(int64_t)ids[r] * table_ld + i]);
+    for (int i = threadIdx.x; i < n; i += blockDim.x) {
+        float v = h[r * h_ld + i];
+        for (int s = 1; s < slices; s++) v += h[s * stride + r * h_ld + i];
+        ActIO<ActT>::st(y + act_index<ActT>(r, i, ld), gelu_tanh_f(v) * (float)table[(int64_t)ids[r] * table_ld + i]);
+    }
 }
 __global__ void gelu_kernel(const float* __restrict__ x, float* __restrict__ y, int64_t n) {
     const int64_t i = (int64_t)blockIdx.x * blockDim.x + threadIdx.x;

@@ -1412,16 +1412,29 @@ ExpertOut parallel_ffn(nvl_model* m, const LayerRun& r, const MixerW& w, int M) 
 SubOut side_input(nvl_model* m, const MixerW& w, const Meta& md, int li, int M) {
     const int sd = m->cfg.side_dim, kp = m->side_kp;
     const int64_t col = (int64_t)li * round_up(sd, 4);
+    const int sd4 = (int)round_up(sd, 4);
     m->site = KS_SIDE_GATE;
     if (m->f32) {
-        gemm(m, EPI_STORE, true, mk(m->xn, m->H, w.side_gate, m->h2, (int)round_up(sd, 4), nullptr, 1.f, M, sd, m->H));
+        gemm(m, EPI_STORE, true, mk(m->xn, m->H, w.side_gate, m->h2, sd4, nullptr, 1.f, M, sd, m->H));
         KScope ks(m, KC_OTHER);
-        hipLaunchKernelGGL((gelu_token_kernel<float, float>), dim3(M), dim3(256), 0, m->stream, m->h2, round_up(sd, 4), (const float*)m->side_emb + col, m->side_ld, md.tokens, (float*)m->lside, (int64_t)kp, sd);
+        hipLaunchKernelGGL((gelu_token_kernel<float, float>), dim3(M), dim3(256), 0, m->stream, m->h2, (int64_t)sd4, 1, (int64_t)0, (const float*)m->side_emb + col, m->side_ld, md.tokens, (float*)m->lside, (int64_t)kp, sd);
         NVL_HIP(hipGetLastError());
     } else {
         GemmArgs a = mk(m->xn, m->H, w.side_gate, m->lside, kp, nullptr, 1.f, M, sd, m->H);
-        a.tok_ids = md.tokens; a.tok_table = (const bf16_t*)m->side_emb + col; a.tok_ld = m->side_ld;
-        gemm(m, EPI_GELU_TOK, false, a);
+        // a few hundred rows: the narrow projection has too few tiles for the chip; split along K, the activation in a launch of its own
+        int slices = 1;
+        const int tiles = cdiv(M, 128) * cdiv(sd, 128);
+        if (M > 512 && M <= m->sk_rows && sd4 <= m->H) while (slices < SK_TILE_MAX_SLICES && tiles * slices < 256 && m->H / (slices * 2) >= 256) slices *= 2;
+        if (slices > 1) {
+            a.C = m->x; a.N = sd4; a.sk_part = m->sk_part; a.sk_slices = slices;      // (x is not touched)
+            gemm(m, EPI_RESID, true, a);
+            KScope ks(m, KC_OTHER, 0, KS_SIDE_GATE, (double)M * sd * (4.0 * slices + 4.0));
+            hipLaunchKernelGGL((gelu_token_kernel<bf16_t, bf16_t>), dim3(M), dim3(256), 0, m->stream, m->sk_part, (int64_t)sd4, slices, (int64_t)M * sd4, (const bf16_t*)m->side_emb + col, m->side_ld, md.tokens, (bf16_t*)m->lside, (int64_t)kp, sd);
+            NVL_HIP(hipGetLastError());
+        } else {
+            a.tok_ids = md.tokens; a.tok_table = (const bf16_t*)m->side_emb + col; a.tok_ld = m->side_ld;
+            gemm(m, EPI_GELU_TOK, false, a);
+        }
     }
     return sub_out(m, KS_SIDE_PROJ, m->lside, w.side_proj, M, kp);
 }

@@ -290,6 +290,17 @@ def test_key_splits(gpu, tmp_path, heads, kv_heads, dim, vdim, window):
     m.close()
 
 
+def test_prompt_of_many_hundred_tokens(gpu, tmp_path):
+    """Long enough that the narrow projections are split along K."""
+    cfg = BM.config([att(window=40, mlp=None), att(window=40, mlp=moe(6, 2, None, 24))], width=520, vocab=90, side=30, positions=700)
+    w = BM.weights(cfg, 18)
+    tok, want, _ = BM.clear_tokens(cfg, w, 690, 6)
+    m = build(gpu, tmp_path, cfg, w, "bf16")
+    for i, cuts in enumerate(([690], [530, 160], [64, 600, 26])):
+        assert err(feed(m, i, tok, cuts), want, "bf16") < ONE["bf16"], cuts
+    m.close()
+
+
 # ---- the framework's own entry points ----
 def test_greedy_generation(gpu, tmp_path, stack):
     """Stepwise, fused on the device, and through the runner give the restatement's tokens (fp32)."""
