@@ -322,7 +322,7 @@ def main():
             tf = k["flops"] / (k["ms"] * 1e-3) / 1e12 if k["ms"] > 0 else 0.0
             gbs = k["bytes"] / (k["ms"] * 1e-3) / 1e9 if k["ms"] > 0 else 0.0
             mfma_bound = k["phase"] == "prefill" and k["site"] in ("qkv_proj", "o_proj", "ffn_up", "ffn_down", "attention",
-                                                                   "moe_up", "moe_down", "lm_head") and tf / MFMA_BF16_PEAK_TFLOPS > gbs / HBM_PEAK_GBS
+                                                                   "moe_up", "moe_down", "lm_head", "mix_in_proj", "side_gate", "side_proj") and tf / MFMA_BF16_PEAK_TFLOPS > gbs / HBM_PEAK_GBS
             e = {"site": k["site"], "phase": k["phase"], "launches": k["launches"], "avg_launch_us": round(us, 2),
                  "share_of_step": round(k["ms"] / tot_ms, 4), "bound": "mfma" if mfma_bound else "hbm",
                  "flops_per_launch": round(k["flops"] / k["launches"]), "bytes_per_launch": round(k["bytes"] / k["launches"]),
