@@ -782,7 +782,7 @@ __global__ __launch_bounds__(NW * 64) void attn_decode_bf16_kernel(const int32_t
 // ------------------------------------------------------------------------------------------
 // fp32 parity kernel: block = (query position, head), 256 threads, T <= 8192
 // ------------------------------------------------------------------------------------------
-__global__ __launch_bounds__(256) void attn_f32_kernel(AttnArgs p, int HD) {
+static __global__ __launch_bounds__(256) void attn_f32_kernel(AttnArgs p, int HD) {
     extern __shared__ float sc[];                 // [T_max_needed] scores then probs
     __shared__ float red[8];
     const int seq = blockIdx.z, head = blockIdx.y, s_idx = blockIdx.x;

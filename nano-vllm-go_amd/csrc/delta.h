@@ -681,4 +681,9 @@ __global__ __launch_bounds__(64) void pack_rows_kernel(PackArgs p) {
     }
 }
 
+// launches (delta_inst.hip); nk: template argument of the chunk kernels
+void delta_step_launch(hipStream_t st, const DeltaArgs& p, int n_seqs, bool fused, bool f32);
+void delta_prep_launch(hipStream_t st, const DeltaArgs& p, dim3 grid, int nk);
+void delta_scan_launch(hipStream_t st, const DeltaArgs& p, int n_seqs, int nk);
+
 }  // namespace nvl

@@ -27,6 +27,7 @@
 // the tight-tolerance parity mode, not a performance path.
 #pragma once
 #include <stdexcept>
+#include <type_traits>
 #include "common.h"
 
 namespace nvl {
@@ -911,6 +912,7 @@ __global__ __launch_bounds__(1024) void gemm_skinny_bf16_kernel(GemmArgs p) {
     }
 }
 
+#ifndef NVL_GEMM_INST
 // ------------------------------------------------------------------------------------------
 // MoE decode routing in ONE launch (moe.go:57-103): router logits of a 16-row activation tile (E <= 64 experts, all of K),
 // softmax, top-k, renormalised weights as the dense gate matrix GemmArgs::moe_gate of the expert projections.  Before:
@@ -919,7 +921,7 @@ __global__ __launch_bounds__(1024) void gemm_skinny_bf16_kernel(GemmArgs p) {
 // the K slices are summed through LDS in wave order, then wave r routes row r of the tile with a lane per expert.
 // p: A (fragment-major operand, possibly the deferred-norm raw form with rs_in), W (router, fragment-major), M, N = E, K.
 // ------------------------------------------------------------------------------------------
-__global__ __launch_bounds__(1024) void moe_router_gate_kernel(GemmArgs p, int top_k, float* __restrict__ gate, float* __restrict__ logits_out, int ld_logits) {
+static __global__ __launch_bounds__(1024) void moe_router_gate_kernel(GemmArgs p, int top_k, float* __restrict__ gate, float* __restrict__ logits_out, int ld_logits) {
     __shared__ f32x4 red[16][64];
     __shared__ float lg[16][64];
     const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
@@ -994,6 +996,7 @@ __global__ __launch_bounds__(1024) void moe_router_gate_kernel(GemmArgs p, int t
     }
     if (lane < E) gate[(int64_t)m * E + lane] = rank < top_k ? prob / wsum : 0.f;      // moe.go:103
 }
+#endif
 
 // ------------------------------------------------------------------------------------------
 // fp32 kernel (parity mode): 64x64 tile, BK=16, 256 threads, 4x4 outputs per thread, k ascending.
@@ -1179,20 +1182,20 @@ __global__ __launch_bounds__(512) void gemm_skinny_wide_bf16_kernel(GemmArgs p) 
     }
 }
 
-static int g_chunk_max_m = 512;    // largest M that uses 64-row passes of the decode form at all (nvl_set_tuning key 11; 64 = off)
-static int g_chunk_all_m = 64;     // up to here every projection does; above, only those whose 128x128 tile grid would
+inline int g_chunk_max_m = 512;    // largest M that uses 64-row passes of the decode form at all (nvl_set_tuning key 11; 64 = off)
+inline int g_chunk_all_m = 64;     // up to here every projection does; above, only those whose 128x128 tile grid would
                                    // have fewer than g_chunk_min_tiles workgroups (keys 14, 12).  Measured: the mix wins
                                    // from 96 rows on (profiles/r01g_large_decode_batches.txt)
-static int g_pass_interleave = 1;   // 64-row groups of one projection in ONE launch (key 13; 0 = one launch per group)
-static int g_chunk_min_tiles = 160;
-static int g_msplit_ks = 8;         // K split of the deferred-norm residual projections (nvl_set_tuning key 6)
-static int g_narrow_waves = 2048;   // waves per narrow-form launch (nvl_set_tuning key 5).  Round-2 sweep on the final kernels
+inline int g_pass_interleave = 1;   // 64-row groups of one projection in ONE launch (key 13; 0 = one launch per group)
+inline int g_chunk_min_tiles = 160;
+inline int g_msplit_ks = 8;         // K split of the deferred-norm residual projections (nvl_set_tuning key 6)
+inline int g_narrow_waves = 2048;   // waves per narrow-form launch (nvl_set_tuning key 5).  Round-2 sweep on the final kernels
                                     // (profiles/r02_narrow_waves_sweep.txt): 2048 vs 1024: B=1 +5.4 %, B=8 +5.0 %, B=16 +2.4 %,
                                     // B=32 flat; 4096 = 2048.  (Round 1, before the activation-row mask: 1024 beat 4096 by 3-8 %.)
-static int g_wide_ksplit = 0;   // experiment (nvl_set_tuning key 4): K split of the wide form when groups <= 512
-static int g_x_mask = 1;            // nvl_set_tuning key 24: decode kernels skip the activation fetch of padded rows (M % 16 != 0)
-static int g_force_ntw = 0, g_force_ksplit = 0;   // tuning overrides (nvl_bench_gemm only)
-static int g_force_tile = 0;                      // 0 automatic, 1: 128x128x2st, 2: 256x128x3st, 3: 256x256x2st, 5: ping-pong 256x256
+inline int g_wide_ksplit = 0;   // experiment (nvl_set_tuning key 4): K split of the wide form when groups <= 512
+inline int g_x_mask = 1;            // nvl_set_tuning key 24: decode kernels skip the activation fetch of padded rows (M % 16 != 0)
+inline int g_force_ntw = 0, g_force_ksplit = 0;   // tuning overrides (nvl_bench_gemm only)
+inline int g_force_tile = 0;                      // 0 automatic, 1: 128x128x2st, 2: 256x128x3st, 3: 256x256x2st, 5: ping-pong 256x256
 
 template <int EPI, typename OutT>
 static inline bool launch_gemm_skinny_bf16(hipStream_t st, const GemmArgs& a);
@@ -1300,7 +1303,7 @@ static inline bool launch_gemm_skinny_ntw(hipStream_t st, const GemmArgs& a) {
 // flight per CU.  Two tiles per wave (512 workgroups) for batches of 17..32 rows: Llama-3.2-1B B=32 decode 33.7 K -> 34.5 K
 // tok/s (+2.4 %), B=20 +3.1 %, Falcon-7B B=32 +4.7 %, Llama-3-8B / Granite B=32 +0.8 %; the LM head (thousands of groups
 // either way) is indifferent, and 64-row launches (MT = 4) lose 2 % (profiles/r03_wide_tiles_per_wave.txt).
-static int g_wide_ntb = 0;
+inline int g_wide_ntb = 0;
 template <int EPI, typename OutT, int NTB = 4>
 static inline bool launch_gemm_skinny_wide(hipStream_t st, const GemmArgs& a) {
     if constexpr (NTB == 4) {
@@ -1404,7 +1407,7 @@ static inline void launch_gemm_grouped(hipStream_t st, const GemmArgs& a, int ma
 }
 
 template <int EPI, typename OutT>
-static inline void launch_gemm_bf16(hipStream_t st, const GemmArgs& a) {
+void launch_gemm_bf16(hipStream_t st, const GemmArgs& a) {
     if (a.tile_map) { launch_gemm_grouped<EPI, OutT>(st, a, a.M); return; }   // a.M carries the m-tile bound
     if (launch_gemm_skinny_bf16<EPI, OutT>(st, a)) return;
     if constexpr (EPI != EPI_QKV) {
@@ -1462,9 +1465,23 @@ static inline void launch_gemm_bf16(hipStream_t st, const GemmArgs& a) {
 }
 
 template <int EPI, typename OutT>
-static inline void launch_gemm_f32(hipStream_t st, const GemmArgs& a) {
+void launch_gemm_f32(hipStream_t st, const GemmArgs& a) {
     const int tiles = cdiv(a.M, 64) * cdiv(a.N, 64);
     hipLaunchKernelGGL((gemm_f32_kernel<EPI, OutT>), dim3(tiles), dim3(256), 0, st, a);
 }
+
+// The projections' kernels are compiled per epilogue, side by side (gemm_inst.hip): (epilogue, output type)
+#define NVL_GEMM_BF16_INSTANCES(X)                                                                                              \
+    X(EPI_STORE, float) X(EPI_STORE, bf16_t) X(EPI_RESID, float) X(EPI_SWIGLU, bf16_t) X(EPI_GELU, bf16_t) X(EPI_GEGLU, bf16_t) \
+    X(EPI_CLAMP_GLU, bf16_t) X(EPI_QKV, bf16_t) X(EPI_GROUPED, bf16_t) X(EPI_RELU2, bf16_t) X(EPI_GELU_TOK, bf16_t)
+#define NVL_GEMM_F32_INSTANCES(X) X(EPI_STORE) X(EPI_RESID) X(EPI_GELU)
+#ifndef NVL_GEMM_INST
+#define NVL_X(E, T) extern template void launch_gemm_bf16<E, T>(hipStream_t, const GemmArgs&);
+NVL_GEMM_BF16_INSTANCES(NVL_X)
+#undef NVL_X
+#define NVL_X(E) extern template void launch_gemm_f32<E, float>(hipStream_t, const GemmArgs&);
+NVL_GEMM_F32_INSTANCES(NVL_X)
+#undef NVL_X
+#endif
 
 }  // namespace nvl

@@ -43,7 +43,7 @@ struct GroupedArgs {
 };
 
 // ---- fp32 mode: keys and values of the batch's tokens into the cache (bf16: gemm.h EPI_GROUPED): grid (32-token units of a sequence's new positions, sequences, G) ----
-__global__ __launch_bounds__(256) void grouped_place_kernel(GroupedArgs p) {
+static __global__ __launch_bounds__(256) void grouped_place_kernel(GroupedArgs p) {
     const int seq = blockIdx.y, g = blockIdx.z, n = p.seq_len[seq], pos0 = p.seq_pos[seq], tok0 = p.seq_tok_start[seq];
     const int u0 = (pos0 & ~31) + blockIdx.x * 32;                     // first position of the unit
     const int a = max(u0, pos0), b = min(u0 + 32, pos0 + n);           // positions [a, b) are written
@@ -535,5 +535,9 @@ __global__ __launch_bounds__(256) void grouped_plain_kernel(GroupedArgs p) {
         ActIO<T>::st((T*)p.out + act_index<T>(t, h * p.vp + i, p.out_ld), o);
     }
 }
+
+// launches (grouped_inst.hip): the instance follows from p.dp and p.vp
+void grouped_prefill_launch(hipStream_t st, const GroupedArgs& p, dim3 grid, size_t lds, bool fast);
+void grouped_short_launch(hipStream_t st, const GroupedArgs& p, dim3 grid);
 
 }  // namespace nvl

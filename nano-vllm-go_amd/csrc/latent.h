@@ -106,7 +106,7 @@ __global__ __launch_bounds__(256) void latent_norm_kernel(LatentArgs p) {
 }
 
 // ---- q's rotated part in place, for sizes its readers do not turn themselves: grid (tokens, heads) ----
-__global__ __launch_bounds__(64) void latent_turn_q_kernel(LatentArgs p) {
+static __global__ __launch_bounds__(64) void latent_turn_q_kernel(LatentArgs p) {
     const int64_t t = blockIdx.x;
     float* q = (float*)p.q + t * p.q_ld + (int64_t)blockIdx.y * p.dp + p.dn;
     const int half = p.rot >> 1;
@@ -672,5 +672,9 @@ static __global__ __launch_bounds__(1024) void latent_uv_kernel(LatentArgs p) {
     for (int r = 0; r < 4; r++) acc[r] *= lat_sigmoid(g[r]);
     act_store4<bf16_t>((bf16_t*)p.out, t, col, p.out_ld, acc);
 }
+
+// launches (latent_inst.hip): the instance follows from the padded sizes
+void latent_prefill_launch(hipStream_t st, const LatentArgs& p, int n_seqs, int max_len);
+void latent_decode_launch(hipStream_t st, const LatentArgs& p, dim3 grid);
 
 }  // namespace nvl

@@ -917,27 +917,7 @@ void mix_latent(nvl_model* m, const LayerRun& r, const MixerW& w, const Meta& md
                 if (m->f32) hipLaunchKernelGGL((latent_plain_kernel<float>), grid, dim3(256), lds, m->stream, a);
                 else hipLaunchKernelGGL((latent_plain_kernel<bf16_t>), grid, dim3(256), lds, m->stream, a);
             } else {
-                const dim3 grid(H, n_seqs, cdiv(max_len, 256));
-#define NVL_LP(KSv, DTv)                                                                                                      \
-                do {                                                                                                         \
-                    constexpr int lds_ = latent_prefill_lds_bytes<KSv, DTv>();                                               \
-                    NVL_LDS_ATTR((latent_prefill_kernel<KSv, DTv>), lds_);                                                   \
-                    hipLaunchKernelGGL((latent_prefill_kernel<KSv, DTv>), grid, dim3(512), lds_, m->stream, a);              \
-                } while (0)
-#define NVL_LPK(KSv)                                                                                        \
-                do {                                                                                         \
-                    if (r.vp == 32) NVL_LP(KSv, 2); else if (r.vp == 64) NVL_LP(KSv, 4);                      \
-                    else if (r.vp == 128) NVL_LP(KSv, 8); else NVL_LP(KSv, 16);                               \
-                } while (0)
-                if (r.dp == 256 && r.vp == 256) hipLaunchKernelGGL((latent_prefill_wide_kernel<8, 16>), dim3(H, n_seqs, cdiv(max_len, 64)), dim3(256), 0, m->stream, a);
-                else if (r.dp == 32) NVL_LPK(1);
-                else if (r.dp == 64) NVL_LPK(2);
-                else if (r.dp == 96) NVL_LPK(3);
-                else if (r.dp == 128) NVL_LPK(4);
-                else if (r.dp == 192) { if (r.vp == 32) NVL_LP(6, 2); else if (r.vp == 64) NVL_LP(6, 4); else NVL_LP(6, 8); }
-                else if (r.vp == 32) NVL_LP(8, 2); else if (r.vp == 64) NVL_LP(8, 4); else NVL_LP(8, 8);
-#undef NVL_LPK
-#undef NVL_LP
+                latent_prefill_launch(m->stream, a, n_seqs, max_len);
             }
             NVL_HIP(hipGetLastError());
         }
@@ -959,20 +939,7 @@ void mix_latent(nvl_model* m, const LayerRun& r, const MixerW& w, const Meta& md
             const double keys = m->kv_tok > 0 && c.window > 0 ? std::min(m->kv_tok, (double)n * c.window) : (m->kv_tok > 0 ? m->kv_tok : (double)n * std::max(1, c.window));
             KScope ks(m, KC_ATTN, keys * H * (4.0 * c.kv_rank + 2.0 * c.rot_dim), KS_ATTN, keys * (c.kv_rank + c.rot_dim) * 2.0 + (double)n * H * c.kv_rank * (2.0 + 4.0 * split));
             const dim3 grid(ht, n, split);
-#define NVL_LDR(NRv, KRv)                                                                                                  \
-            do {                                                                                                            \
-                constexpr int lds_ = latent_decode_lds_bytes<NRv>();                                                        \
-                NVL_LDS_ATTR((latent_decode_kernel<NRv, KRv>), lds_);                                                       \
-                hipLaunchKernelGGL((latent_decode_kernel<NRv, KRv>), grid, dim3(256), lds_, m->stream, a);                  \
-            } while (0)
-#define NVL_LD(NRv) do { if (r.rotp == 0) NVL_LDR(NRv, 0); else if (r.rotp == 32) NVL_LDR(NRv, 1); else if (r.rotp == 64) NVL_LDR(NRv, 2); else NVL_LDR(NRv, 4); } while (0)
-            switch (r.rp / 64) {
-                case 1: NVL_LD(1); break; case 2: NVL_LD(2); break; case 3: NVL_LD(3); break; case 4: NVL_LD(4); break;
-                case 6: NVL_LD(6); break; case 8: NVL_LD(8); break;
-                default: throw std::runtime_error("latent attention: no absorbed instance for this latent size");
-            }
-#undef NVL_LD
-#undef NVL_LDR
+            latent_decode_launch(m->stream, a, grid);
             NVL_HIP(hipGetLastError());
         }
         {
@@ -989,23 +956,9 @@ void linrec(nvl_model* m, LinRecArgs a, int n_seqs, int M, int max_len, bool fus
     const double elems = (double)a.H * a.DK * a.DVp;
     const double bytes = (double)M * a.H * (2.0 * a.DK / a.kdiv + 2.0 * a.DV) * 4.0 + 2.0 * n_seqs * elems * 4.0;
     KScope ks(m, KC_OTHER, 4.0 * (double)M * a.H * a.DK * a.DV, site, bytes);
-    const int lds = linrec_step_lds_bytes(a.DK, a.DVp);
-    const dim3 sgrid(a.H, n_seqs);
     a.len_lo = 1; a.len_hi = 1 << 30;
-    auto step = [&](auto kind, auto act) {
-        constexpr int KIND = decltype(kind)::value;
-        using ActT = decltype(act);
-        int tv = 1;
-        while (tv < a.DVp / 4) tv <<= 1;
-        const int rows = cdiv(a.DK, LR_STEP_THREADS / tv);        // state rows per thread
-        if (rows <= 4) hipLaunchKernelGGL((linrec_step_kernel<KIND, 4, ActT>), sgrid, dim3(LR_STEP_THREADS), lds, m->stream, a);
-        else if (rows <= 8) hipLaunchKernelGGL((linrec_step_kernel<KIND, 8, ActT>), sgrid, dim3(LR_STEP_THREADS), lds, m->stream, a);
-        else hipLaunchKernelGGL((linrec_step_kernel<KIND, 16, ActT>), sgrid, dim3(LR_STEP_THREADS), lds, m->stream, a);
-        NVL_HIP(hipGetLastError());
-    };
     if (fused) {
-        if (m->f32) step(std::integral_constant<int, (CH ? 1 : 0) + 2>{}, float{});
-        else step(std::integral_constant<int, (CH ? 1 : 0) + 2>{}, bf16_t{});
+        linrec_step_launch(m->stream, a, n_seqs, CH, true, m->f32);
         return;
     }
     const int nk = a.DK <= 32 ? 2 : (a.DK <= 64 ? 4 : (a.DK <= 128 ? 8 : 16)), nw = a.DV <= 64 ? 4 : 8;
@@ -1013,7 +966,7 @@ void linrec(nvl_model* m, LinRecArgs a, int n_seqs, int M, int max_len, bool fus
     const bool steps = !chunks || m->min_len <= REC_STEP_MAX;
     if (steps) {
         a.len_hi = chunks ? REC_STEP_MAX : 1 << 30;
-        step(std::integral_constant<int, CH ? 1 : 0>{}, float{});
+        linrec_step_launch(m->stream, a, n_seqs, CH, false, m->f32);
     }
     if (!chunks || max_len <= REC_STEP_MAX) return;
     a.len_lo = REC_STEP_MAX + 1; a.len_hi = 1 << 30;
@@ -1033,25 +986,7 @@ void linrec(nvl_model* m, LinRecArgs a, int n_seqs, int M, int max_len, bool fus
         grow(m, m->rec_decay, m->rec_decay_floats, (int64_t)n_seqs * a.n_super * a.H * (CH ? a.DK : 1));
         a.z = m->rec_z; a.zdecay = m->rec_decay;
     }
-#define NVL_LC(NKv, NWv, MODEv)                                                                                              \
-    do {                                                                                                                     \
-        NVL_LDS_ATTR((linrec_chunk_kernel<NKv, NWv, CH, MODEv>), 160 * 1024);                                                \
-        hipLaunchKernelGGL((linrec_chunk_kernel<NKv, NWv, CH, MODEv>), dim3(a.H, n_seqs, a.n_slices * (MODEv ? a.n_super : 1)), dim3(NWv * 64), \
-                           (linrec_chunk_lds_bytes<NKv, NWv, CH>(a.rank)), m->stream, a);                                    \
-    } while (0)
-#define NVL_LCM(NKv, NWv)                                                                                                    \
-    do {                                                                                                                     \
-        if (par) {                                                                                                           \
-            NVL_LC(NKv, NWv, 1);                                                                                             \
-            hipLaunchKernelGGL((linrec_prefix_kernel<CH>), dim3(a.H, n_seqs, cdiv((int64_t)a.DK * a.DVp, 1024)), dim3(256), 0, m->stream, a); \
-            NVL_LC(NKv, NWv, 2);                                                                                             \
-        } else NVL_LC(NKv, NWv, 0);                                                                                          \
-    } while (0)
-#define NVL_LCN(NKv) do { if (nw == 4) NVL_LCM(NKv, 4); else NVL_LCM(NKv, 8); } while (0)
-    if (nk == 2) NVL_LCN(2); else if (nk == 4) NVL_LCN(4); else if (nk == 8) NVL_LCN(8); else NVL_LCN(16);
-#undef NVL_LCN
-#undef NVL_LCM
-#undef NVL_LC
+    linrec_chunk_launch(m->stream, a, n_seqs, CH, nk, nw, par);
     NVL_HIP(hipGetLastError());
 }
 
@@ -1140,26 +1075,6 @@ void mix_gla(nvl_model* m, const LayerRun& r, const MixerW& w, const Meta& md, i
     gated_norm<false>(m, g, KS_GLA_GATE);
 }
 
-void delta_step(nvl_model* m, const DeltaArgs& a, int n_seqs, bool fused) {
-    const int lds = delta_step_lds_bytes(a.DK, a.DVp, fused ? a.a_rkp + a.g_rkp : 0);
-    const dim3 grid(a.H, n_seqs);
-    int tv = 1;
-    while (tv < a.DVp / 4) tv <<= 1;
-    const int rows = cdiv(a.DK, LR_STEP_THREADS / tv);        // state rows per thread
-#define NVL_DS(FU, RO, ACT)                                                                                                  \
-    do {                                                                                                                     \
-        NVL_LDS_ATTR((delta_step_kernel<FU, RO, ACT>), 128 * 1024);                                                          \
-        hipLaunchKernelGGL((delta_step_kernel<FU, RO, ACT>), grid, dim3(LR_STEP_THREADS), lds, m->stream, a);                \
-    } while (0)
-#define NVL_DSR(FU, ACT) do { if (rows <= 4) NVL_DS(FU, 4, ACT); else if (rows <= 8) NVL_DS(FU, 8, ACT); else NVL_DS(FU, 16, ACT); } while (0)
-    if (!fused) NVL_DSR(false, float);
-    else if (m->f32) NVL_DSR(true, float);
-    else NVL_DSR(true, bf16_t);
-#undef NVL_DSR
-#undef NVL_DS
-    NVL_HIP(hipGetLastError());
-}
-
 void mix_delta(nvl_model* m, const LayerRun& r, const MixerW& w, const Meta& md, int n_seqs, int M, int max_len) {
     const nvl_layer_config& c = r.c;
     const int64_t qk = (int64_t)c.kv_heads * c.dim, hd = (int64_t)c.heads * c.dim, hv = (int64_t)c.heads * c.vdim;
@@ -1183,7 +1098,7 @@ void mix_delta(nvl_model* m, const LayerRun& r, const MixerW& w, const Meta& md,
         a.norm_w = w.mix_norm; a.eps = m->cfg.norm_eps; a.out = m->lmix; a.out_ld = r.kd;
         KScope ks(m, KC_OTHER, 6.0 * M * elems, KS_DELTA_SCAN, 2.0 * n_seqs * elems * 4.0 + (double)M * (r.conv_dim * 4.0 * (c.conv_taps + 1) + hv * (double)m->wsize) +
                                                                    ((double)hd * w.rank + (double)hv * w.grank) * (double)m->wsize);
-        delta_step(m, a, n_seqs, true);
+        delta_step_launch(m->stream, a, n_seqs, true, m->f32);
         return;
     }
     {
@@ -1208,7 +1123,7 @@ void mix_delta(nvl_model* m, const LayerRun& r, const MixerW& w, const Meta& md,
     if (!chunks || m->min_len <= REC_STEP_MAX) {
         a.len_hi = chunks ? REC_STEP_MAX : 1 << 30;
         KScope ks(m, KC_OTHER, chunks ? 0.0 : 6.0 * M * elems, KS_DELTA_SCAN, chunks ? 0.0 : io + 2.0 * n_seqs * elems * 4.0);
-        delta_step(m, a, n_seqs, false);
+        delta_step_launch(m->stream, a, n_seqs, false, m->f32);
     }
     if (chunks && max_len > REC_STEP_MAX) {
         a.len_lo = REC_STEP_MAX + 1; a.len_hi = 1 << 30;
@@ -1221,35 +1136,12 @@ void mix_delta(nvl_model* m, const LayerRun& r, const MixerW& w, const Meta& md,
         const double scratch = (double)M * c.heads * (3.0 * nk * 16 + 2.0 * c.vdim) * 4.0;
         {
             KScope ks(m, KC_OTHER, 0, KS_DELTA_PREP, io + scratch);
-#define NVL_DP(NKv)                                                                                                           \
-            do {                                                                                                              \
-                constexpr int lds_ = delta_prep_lds_bytes<NKv>();                                                              \
-                NVL_LDS_ATTR((delta_prep_kernel<NKv>), lds_);                                                                  \
-                hipLaunchKernelGGL((delta_prep_kernel<NKv>), pgrid, dim3(512), lds_, m->stream, a);                            \
-            } while (0)
-            if (nk == 2) NVL_DP(2); else if (nk == 4) NVL_DP(4); else if (nk == 8) NVL_DP(8); else NVL_DP(16);
-#undef NVL_DP
+            delta_prep_launch(m->stream, a, pgrid, nk);
             NVL_HIP(hipGetLastError());
         }
         {
             KScope ks(m, KC_OTHER, 6.0 * M * elems, KS_DELTA_SCAN, scratch + 2.0 * n_seqs * elems * 4.0);
-            // columns per workgroup, and with few of them the key channels split over the waves too
-            const int pairs = c.heads * n_seqs;
-#define NVL_DC(NKv, NWv, KSPv)                                                                                                \
-            do {                                                                                                              \
-                constexpr int lds_ = delta_scan_lds_bytes<NKv, NWv, KSPv>();                                                   \
-                NVL_LDS_ATTR((delta_scan_kernel<NKv, NWv, KSPv>), lds_);                                                       \
-                hipLaunchKernelGGL((delta_scan_kernel<NKv, NWv, KSPv>), dim3(c.heads, n_seqs, cdiv(c.vdim, 16 * NWv / KSPv)), dim3(NWv * 64), lds_, m->stream, a); \
-            } while (0)
-#define NVL_DCK(NKv, LOW)                                                                                                     \
-            do {                                                                                                              \
-                if (pairs * cdiv(c.vdim, 64) < 128) NVL_DC(NKv, 4, LOW);                                                       \
-                else if (c.vdim <= 64 || pairs * cdiv(c.vdim, 128) < 256) NVL_DC(NKv, 4, 1);                                                                      \
-                else NVL_DC(NKv, 8, 1);                                                                                        \
-            } while (0)
-            if (nk == 2) NVL_DC(2, 4, 1); else if (nk == 4) NVL_DCK(4, 2); else if (nk == 8) NVL_DCK(8, 4); else NVL_DCK(16, 4);
-#undef NVL_DCK
-#undef NVL_DC
+            delta_scan_launch(m->stream, a, n_seqs, nk);
             NVL_HIP(hipGetLastError());
         }
     }
@@ -1310,22 +1202,11 @@ void mix_grouped(nvl_model* m, const LayerRun& r, const MixerW& w, const Meta& m
         NVL_HIP(hipGetLastError());
         return;
     }
-    const int ks = r.dp == 32 ? 1 : r.dp >> 5, dt = r.vp >> 4;
+    const int dt = r.vp >> 4;
     if (any_long) {
         KScope scp = scope(1);
         const dim3 grid(a.G, n_seqs, cdiv((int64_t)max_len * a.group, 256));
-#define NVL_GPF(KSv, DTv, FASTv)                                                                                             \
-        do {                                                                                                                 \
-            NVL_LDS_ATTR((grouped_prefill_kernel<KSv, DTv, FASTv>), 160 * 1024);                                             \
-            hipLaunchKernelGGL((grouped_prefill_kernel<KSv, DTv, FASTv>), grid, dim3(512), lds, m->stream, a);               \
-        } while (0)
-#define NVL_GP(KSv, DTv) do { if (a.table && w.bias_lowers && c.softcap > 0.f && c.softcap <= GROUPED_FAST_CAP) NVL_GPF(KSv, DTv, true); else NVL_GPF(KSv, DTv, false); } while (0)
-#define NVL_GPK(KSv) do { if (dt == 2) NVL_GP(KSv, 2); else if (dt == 4) NVL_GP(KSv, 4); else if (dt == 8) NVL_GP(KSv, 8); else NVL_GP(KSv, 16); } while (0)
-        if (ks == 1) NVL_GPK(1); else if (ks == 2) NVL_GPK(2); else if (ks == 4) NVL_GPK(4);
-        else if (dt == 2) NVL_GP(8, 2); else if (dt == 4) NVL_GP(8, 4); else NVL_GP(8, 8);
-#undef NVL_GPK
-#undef NVL_GP
-#undef NVL_GPF
+        grouped_prefill_launch(m->stream, a, grid, lds, a.table && w.bias_lowers && c.softcap > 0.f && c.softcap <= GROUPED_FAST_CAP);
         NVL_HIP(hipGetLastError());
     }
     if (any_short) {
@@ -1339,16 +1220,7 @@ void mix_grouped(nvl_model* m, const LayerRun& r, const MixerW& w, const Meta& m
         if (g_grouped_split) z = (int)std::min<int64_t>(g_grouped_split, std::max<int64_t>(1, m->grp_cap / (wgs * n_seqs)));
         a.part = m->grp_part; a.part_cnt = m->grp_cnt;
         const dim3 grid((unsigned)wgs, n_seqs, z);
-#define NVL_GS(KSv, DTv)                                                                                                     \
-        do {                                                                                                                 \
-            constexpr int nw_ = DTv <= 8 ? 8 : 4;                                                                            \
-            NVL_LDS_ATTR((grouped_short_kernel<KSv, DTv, nw_>), nw_ * DTv * 1024);                                           \
-            hipLaunchKernelGGL((grouped_short_kernel<KSv, DTv, nw_>), grid, dim3(nw_ * 64), nw_ * DTv * 1024, m->stream, a); \
-        } while (0)
-#define NVL_GSK(KSv) do { if (dt == 2) NVL_GS(KSv, 2); else if (dt == 4) NVL_GS(KSv, 4); else if (dt == 8) NVL_GS(KSv, 8); else NVL_GS(KSv, 16); } while (0)
-        if (ks == 1) NVL_GSK(1); else if (ks == 2) NVL_GSK(2); else if (ks == 4) NVL_GSK(4); else NVL_GSK(8);
-#undef NVL_GSK
-#undef NVL_GS
+        grouped_short_launch(m->stream, a, grid);
         NVL_HIP(hipGetLastError());
     }
 }

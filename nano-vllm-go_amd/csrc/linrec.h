@@ -602,7 +602,7 @@ __global__ __launch_bounds__(256) void conv_silu_kernel(ConvArgs p, int n_tok) {
         for (int e = 0; e < 4; e++) if (c + e < p.channels) p.out[(int64_t)t * p.out_ld + c + e] = conv_at(p, ring, t, pos, first, c + e);
     }
 }
-__global__ __launch_bounds__(256) void conv_ring_kernel(ConvArgs p) {      // grid (sequences, ceil(channels / 256))
+static __global__ __launch_bounds__(256) void conv_ring_kernel(ConvArgs p) {      // grid (sequences, ceil(channels / 256))
     const int seq = blockIdx.x, n = p.seq_len[seq], c = blockIdx.y * 256 + threadIdx.x;
     if (c >= p.channels) return;
     float* ring = p.ring + (int64_t)p.seq_slot[seq] * p.ring_slot_stride;
@@ -695,5 +695,9 @@ __global__ __launch_bounds__(256) void gated_norm_kernel(GatedNormArgs p, ActT* 
     for (int i = 0; i < KEEP; i++) { const int c = (l + i * nt) * E; if (c < part) put(c, u[i]); }
     for (int c = (l + KEEP * nt) * E; c < part; c += nt * E) put(c, load(c));
 }
+
+// launches (linrec_inst.hip).  ch: a decay per key channel; nk, nw: template arguments of the chunk kernel; par: pieces in parallel
+void linrec_step_launch(hipStream_t st, const LinRecArgs& p, int n_seqs, bool ch, bool fused, bool f32);
+void linrec_chunk_launch(hipStream_t st, const LinRecArgs& p, int n_seqs, bool ch, int nk, int nw, bool par);
 
 }  // namespace nvl

@@ -12,7 +12,10 @@
 set -e
 S=${TMPDIR:-/tmp}/nvllm_check.s
 cd "$(dirname "$0")/.."
-/opt/rocm/bin/hipcc -O3 -std=c++17 --offload-arch=gfx950 -mllvm -amdgpu-kernarg-preload-count=6 -Xclang -target-feature -Xclang -packed-fp32-ops -Wno-unused-function -Wno-unused-variable --cuda-device-only -S nano-vllm-go_amd/csrc/nvllm.hip -o $S 2>/dev/null
+asm() { /opt/rocm/bin/hipcc -O3 -std=c++17 --offload-arch=gfx950 -mllvm -amdgpu-kernarg-preload-count=6 -Xclang -target-feature -Xclang -packed-fp32-ops -Wno-unused-function -Wno-unused-variable --cuda-device-only -S "$@" 2>/dev/null; }
+(asm nano-vllm-go_amd/csrc/nvllm.hip -o $S) & pids=$!
+for i in 1 2 3 4 5 6 7 8 9 10; do (asm -DNVL_GEMM_INST=$i nano-vllm-go_amd/csrc/gemm_inst.hip -o $S.gemm$i) & pids="$pids $!"; done
+for p in $pids; do wait $p; done
 rc=0
 for hd in 64 128; do
   K=$S.attn$hd
@@ -24,7 +27,8 @@ for hd in 64 128; do
   echo "attn_prefill<$hd>: m0 outside asm=$m0  vmcnt(0) after loop entry: $all0 (of them hand-written: $loop0)  vgpr spills=$spills"
   [ "$m0" = 0 ] && [ "$spills" = 0 ] && [ "$all0" = "$loop0" ] || rc=1
 done
-python3 - $S <<'PY' || rc=1
+cat $S $S.gemm* > $S.all
+python3 - $S.all <<'PY' || rc=1
 import re, sys
 meta = open(sys.argv[1]).read()
 kern = {}
