@@ -27,11 +27,13 @@
 extern "C" {
 #endif
 
-#define NVL_ABI_VERSION 6      /* 2: Mamba2 / hybrid layers (config fields, tensor kinds), nvl_stats.evictions, kernel stats;
+#define NVL_ABI_VERSION 7      /* 2: Mamba2 / hybrid layers (config fields, tensor kinds), nvl_stats.evictions, kernel stats;
                                   3: nvl_get_weight, nvl_get_stamps, nvl_tp_p2p_rearm, debug modes 2 / 4 (additions only);
                                   4: models described by a list of layers, library-owned block pool, nvl_forward_rows (additions only);
                                   5: rotated latent attention, channel-wise gated delta rule, output-only norms (new config fields at the end);
-                                  6: grouped-query attention, parallel blocks, experts and per-layer token inputs in lists of layers (new config fields at the end) */
+                                  6: grouped-query attention, parallel blocks, experts and per-layer token inputs in lists of layers (new config fields at the end);
+                                  7: norms of sums, token shift, normed and rotated grouped attention with chunks, kept tokens and sinks, lightning
+                                     attention beside it, softmax-routed clamped experts (new config fields at the end) */
 
 typedef enum nvl_status {
     NVL_OK = 0,
@@ -47,15 +49,18 @@ typedef enum nvl_status {
 
 /* ---- model description: flat mirror of tensor.ModelConfig (purego/tensor/config.go:58-122) ---- */
 enum { NVL_ATTN_MHA = 0, NVL_ATTN_MQA = 1, NVL_ATTN_GQA = 2 };        /* config.go:18-22 */
-enum { NVL_NORM_LAYER = 0, NVL_NORM_RMS = 1 };                        /* config.go:27-30 */
+enum { NVL_NORM_LAYER = 0, NVL_NORM_RMS = 1,                          /* config.go:27-30 */
+       NVL_NORM_RMS_SCALAR = 2 };  /* RMS norms with one weight for all coordinates (lists of layers) */
 enum { NVL_POS_LEARNED = 0, NVL_POS_ROPE = 1, NVL_POS_NONE = 2 };     /* config.go:35-40 */
 enum { NVL_ACT_GELU = 0, NVL_ACT_SWIGLU = 1,                          /* config.go:45-48 */
        NVL_ACT_GEGLU = 2,                                             /* gelu_tanh(gate) * up */
        NVL_ACT_CLAMPED_GLU = 3 };   /* g sigmoid(1.702 g) (u + 1), g = min(gate, limit), u = clamp(up, -limit, limit): nvl_layer_config.ffn_limit */
-enum { NVL_ACT_RELU2 = 4 };         /* max(z, 0)^2, no gate (lists of layers) */
+enum { NVL_ACT_RELU2 = 4,          /* max(z, 0)^2, no gate (lists of layers) */
+       NVL_ACT_REGLU = 5 };        /* max(gate, 0) * up (lists of layers) */
 enum { NVL_BLOCK_SEQUENTIAL = 0, NVL_BLOCK_PARALLEL = 1,              /* config.go:53-56 (parallel: with a list of layers too) */
        NVL_BLOCK_SANDWICH = 2,     /* a norm before AND after each sublayer, x += norm_b(f(norm_a(x)))  } the model is described by a list */
-       NVL_BLOCK_POST = 3 };       /* a norm after each sublayer only, x += scale * norm(f(x))           } of layers (nvl_create_layers)    */
+       NVL_BLOCK_POST = 3,         /* a norm after each sublayer only, x += scale * norm(f(x))           } of layers (nvl_create_layers)    */
+       NVL_BLOCK_SUM_NORM = 4 };   /* a norm of the sum, x <- norm(stream_scale * x + f(x))              }                                  */
 
 typedef struct nvl_model_config {
     int32_t vocab_size, hidden, num_layers, num_heads, num_kv_heads, head_dim;
@@ -75,6 +80,8 @@ typedef struct nvl_model_config {
     float   norm_weight_offset;     /* added to every stored weight of the model's norm (1: weights are kept as differences from one)     */
     float   logit_softcap;          /* logits <- cap tanh(logits / cap); 0: none                                                          */
     int32_t side_dim;               /* per-layer token inputs: columns of NVL_T_SIDE_EMB a layer takes; 0: none (NVL_BLOCK_PARALLEL)        */
+    float   stream_scale;           /* NVL_BLOCK_SUM_NORM: factor of the residual stream in the sum                                       */
+    int32_t token_shift;            /* 1: mixers read h + (h_previous_token - h) * NVL_T_SHIFT (NVL_BLOCK_POST, NVL_BLOCK_SUM_NORM)        */
 } nvl_model_config;
 
 /* ---- models described by a list of layers: every layer names its mixer, the mixer's sizes and its feed-forward ---- */
@@ -83,8 +90,13 @@ enum {
     NVL_MIXER_MAMBA2 = 1,           /* causal convolution + selective state space, gate before a grouped norm                     */
     NVL_MIXER_GLA = 2,              /* gated linear attention: a decay per key channel                                            */
     NVL_MIXER_CHANNEL_DELTA = 3,    /* delta rule with a decay per key channel, short convolutions on q, k and v                  */
-    NVL_MIXER_ATTENTION = 4         /* grouped-query attention: capped scores, logarithmic distance bias, value mixing, output gate */
+    NVL_MIXER_ATTENTION = 4,        /* grouped-query attention: query/key norms, rotation, capped scores, logarithmic distance bias, windows
+                                       with kept first tokens or chunks, sinks, value mixing, output gate                          */
+    NVL_MIXER_LIGHTNING = 5         /* linear attention with a fixed decay per head: beside attention only (nvl_layer_config.mixer2) */
 };
+enum { NVL_QK_NORM_NONE = 0, NVL_QK_NORM_HEAD = 1, NVL_QK_NORM_ROW = 2 };      /* RMS norm of every query / key head, or of the whole projections */
+enum { NVL_SINK_NONE = 0, NVL_SINK_ZERO = 1, NVL_SINK_LEARNED = 2 };           /* an entry of the softmax's denominator: score 0, or NVL_T_SINK  */
+#define NVL_MAX_DECAYS 128
 typedef struct nvl_layer_config {
     int32_t mixer;                  /* NVL_MIXER_*                                                                         */
     int32_t weights_of;             /* the layer whose tensors this one uses (its cache / state is its own); -1: its own   */
@@ -98,16 +110,30 @@ typedef struct nvl_layer_config {
     int32_t ffn_dim;                /* 0: no feed-forward (with experts: the shared expert, 0: none)                       */
     float   ffn_limit;              /* NVL_ACT_CLAMPED_GLU                                                                 */
     int32_t kv_from;                /* latent attention: use this earlier layer's cached latents and rotated keys; -1: own */
-    int32_t rot_dim;                /* latent attention: rotated query/key dimensions per head beside `dim`; 0: none       */
+    int32_t rot_dim;                /* rotated query/key dimensions per head (latent attention: beside `dim`; attention: the first of them); 0: none */
     int32_t gate_per_head;          /* latent attention: 1: one output gate per head; 0: one per channel                   */
     int32_t kv_heads;               /* channel delta: heads of q and k; attention: heads of k and v (heads is a multiple)  */
     double  rot_base;               /* rotation: pair i turns by base^(-2 i / rot_dim) per position                        */
-    double  rot_factor, rot_original, rot_fast, rot_slow;       /* YaRN context extension; rot_factor 0: none              */
+    double  rot_factor, rot_original, rot_fast, rot_slow;       /* YaRN context extension; rot_factor 0: none (rot_low, rot_high: Llama 3.1's) */
     float   softcap;                /* attention: score <- cap tanh(score / cap); 0: none                                  */
     int32_t v_mix;                  /* attention: 1: v <- (1 - lambda) v + lambda v_first, v_first the values of the first such layer */
     int32_t ffn_act;                /* activation of ffn_dim's feed-forward: NVL_ACT_*; 0: the model's activation_type     */
-    int32_t experts, top_k, expert_dim;        /* mixture of experts (SwiGLU, sigmoid scores); experts 0: none             */
+    int32_t experts, top_k, expert_dim;        /* mixture of experts (SwiGLU, sigmoid scores unless said otherwise below); experts 0: none */
     int32_t expert_groups, groups_kept;        /* only experts of the best groups_kept of expert_groups equal groups can be chosen */
+    int32_t chunk;                  /* attention: a query sees the earlier tokens of its own chunk of this many positions; 0: none (not with window) */
+    int32_t keep_first;             /* attention with a window: the first keep_first tokens stay visible                   */
+    int32_t qk_norm;                /* attention: NVL_QK_NORM_*                                                            */
+    int32_t sink;                   /* attention: NVL_SINK_*                                                               */
+    int32_t qkv_bias;               /* attention: 1: NVL_T_BQ / BK / BV are added in the projections                       */
+    int32_t ungated;                /* attention: 1: no output gate                                                        */
+    double  rot_low, rot_high;      /* Llama 3.1 frequency scaling (with rot_factor, rot_original); rot_high 0: not this one */
+    float   out_scale;              /* attention: factor of the mixer's result; 0: one                                     */
+    int32_t route_softmax;          /* experts: weights are the softmax over the chosen experts' logits (bias included)    */
+    float   expert_limit;           /* experts: > 0: NVL_ACT_CLAMPED_GLU with this limit; 0: SwiGLU                        */
+    int32_t mixer2;                 /* a second mixer that reads the same input, its result added: NVL_MIXER_LIGHTNING; 0: none */
+    int32_t heads2, dim2, vdim2;
+    float   out_scale2;             /* factor of its result                                                                */
+    double  decay[NVL_MAX_DECAYS];  /* NVL_MIXER_LIGHTNING: per head                                                       */
 } nvl_layer_config;
 
 /* Arithmetic the device path computes in. */
@@ -208,6 +234,16 @@ typedef enum nvl_tensor_kind {
     NVL_T_SIDE_PROJ,       /* [H, side_dim]                                                           */
     NVL_T_SIDE_NORM,       /* [H]                                                                     */
     NVL_T_SIDE_EMB,        /* model: [V, layers*side_dim] e of every token and layer                  */
+    NVL_T_Q_NORM,          /* [dim] (NVL_QK_NORM_HEAD) or [heads*dim] (NVL_QK_NORM_ROW)               */
+    NVL_T_K_NORM,          /* [dim] or [kv_heads*dim]                                                 */
+    NVL_T_SINK,            /* [heads] scores of NVL_SINK_LEARNED                                      */
+    NVL_T_SHIFT,           /* [H] token shift                                                         */
+    NVL_T_LIN_Q,           /* [heads2*dim2, H]    lightning attention                                 */
+    NVL_T_LIN_K,           /* [heads2*dim2, H]                                                        */
+    NVL_T_LIN_V,           /* [heads2*vdim2, H]                                                       */
+    NVL_T_LIN_GATE,        /* [heads2*vdim2, H]                                                       */
+    NVL_T_LIN_NORM,        /* [heads2*vdim2]      norm of the concatenated heads                      */
+    NVL_T_LIN_O,           /* [H, heads2*vdim2]                                                       */
     NVL_T_COUNT
 } nvl_tensor_kind;
 
@@ -222,11 +258,12 @@ enum {
 /* Replaces tensor.NewTransformerModel (generic_model.go:41-61) + the runner's model ownership
  * (tensor_model_runner.go:21-33).  Fails with NVL_ERR_NO_DEVICE when no GPU is present. */
 int nvl_create(const nvl_model_config* cfg, const nvl_runtime_opts* opts, nvl_model** out);
-/* nvl_create for a model described by a list of layers (cfg->block_style NVL_BLOCK_SANDWICH, NVL_BLOCK_POST or NVL_BLOCK_PARALLEL): `layers`
+/* nvl_create for a model described by a list of layers (cfg->block_style NVL_BLOCK_SANDWICH, _POST, _PARALLEL or _SUM_NORM): `layers`
  * has cfg->num_layers entries; of cfg only vocab_size, hidden, num_layers, max_seq_len, norm_eps, norm_type, norm_weight_offset, position_type
- * (learned or none), activation_type (NVL_ACT_GEGLU, NVL_ACT_CLAMPED_GLU; NVL_ACT_RELU2 or NVL_ACT_SWIGLU in parallel blocks),
- * embedding_multiplier, logits_scaling, logit_softcap, side_dim and tied_embedding are read.  Layer norms, learned positions, NVL_MIXER_ATTENTION,
- * experts and side_dim belong to NVL_BLOCK_PARALLEL: x += mixer(h) + ff(h), h = norm(x). */
+ * (learned or none), activation_type (NVL_ACT_GEGLU, NVL_ACT_CLAMPED_GLU; NVL_ACT_RELU2 or NVL_ACT_SWIGLU in parallel blocks, NVL_ACT_REGLU or
+ * NVL_ACT_CLAMPED_GLU in NVL_BLOCK_SUM_NORM), embedding_multiplier, logits_scaling, logit_softcap, side_dim, stream_scale, token_shift and
+ * tied_embedding are read.  Layer norms, learned positions and side_dim belong to NVL_BLOCK_PARALLEL: x += mixer(h) + ff(h), h = norm(x);
+ * experts to it and NVL_BLOCK_SUM_NORM. */
 int nvl_create_layers(const nvl_model_config* cfg, const nvl_layer_config* layers, const nvl_runtime_opts* opts, nvl_model** out);
 
 /* Replaces loadTensorFromData + the per-kind placement in loadAttention/loadFFN/loadMoE/loadNorm
@@ -247,7 +284,7 @@ int nvl_load_safetensors(nvl_model* m, const char* path);
  * the reference's model_info.json) -> nvl_model_config.  Reference quirks kept: max_position_embeddings and
  * rope_scaling are not read.  Errors are reported through nvl_last_error(NULL). */
 int nvl_load_config_json(const char* path, nvl_model_config* cfg);
-/* The layer list of a config.json whose architecture is described by one ("Potuzen", "Lufazen", "Bolinex"): writes up to `cap` entries, returns
+/* The layer list of a config.json whose architecture is described by one ("Potuzen", "Lufazen", "Bolinex", "Medulorn"): writes up to `cap` entries, returns
  * how many the file has; 0 for every other architecture.  A file that names no longest sequence (max_positions): nvl_load_config_json
  * sets max_seq_len to 4096, the caller may change it before nvl_create_layers (a smaller one always). */
 int nvl_load_layers_json(const char* path, nvl_layer_config* layers, int cap);

@@ -22,21 +22,23 @@ SLOTS = [
     "mix_post_norm", "ffn_post_norm", "mix_gate", "lat_dq", "lat_dq_norm", "lat_uq", "lat_dkv", "lat_dkv_norm", "lat_uk", "lat_uv",
     "gla_norm", "gla_a1", "gla_a2", "gla_a2_b", "mix_scale", "ffn_scale", "delta_conv", "delta_beta", "delta_g1", "delta_g2",
     "bias_r1", "bias_r2", "v_mix", "router_bias", "side_gate", "side_proj", "side_norm", "side_emb",
+    "q_norm", "k_norm", "sink", "shift", "lin_q", "lin_k", "lin_v", "lin_gate", "lin_norm", "lin_o",
 ]
 SLOT_ID = {n: i for i, n in enumerate(SLOTS)}
 ONE_D = {"final_norm_w", "final_norm_b", "attn_norm_w", "attn_norm_b", "ffn_norm_w", "ffn_norm_b",
          "bq", "bk", "bv", "bo", "b1", "b2",
          "mamba_conv_w", "mamba_conv_b", "mamba_a_log", "mamba_d", "mamba_dt_bias", "mamba_norm",
          "mix_post_norm", "ffn_post_norm", "lat_dq_norm", "lat_dkv_norm", "gla_norm", "gla_a2_b", "mix_scale", "ffn_scale", "delta_conv",
-         "bias_r1", "bias_r2", "v_mix", "router_bias", "side_norm"}
+         "bias_r1", "bias_r2", "v_mix", "router_bias", "side_norm", "q_norm", "k_norm", "sink", "shift", "lin_norm"}
 OUT_IN_SLOTS = {"mamba_in_proj", "mamba_out_proj"}      # kept in the checkpoint's [out, in] layout by the reference's loader
 
 ATTN = {"mha": 0, "mqa": 1, "gqa": 2}
-NORM = {"layernorm": 0, "rmsnorm": 1}
+NORM = {"layernorm": 0, "rmsnorm": 1, "rmsnorm_scalar": 2}
 POS = {"learned": 0, "rope": 1, "nope": 2}
-ACT = {"gelu": 0, "swiglu": 1, "geglu": 2, "clamped_glu": 3, "relu2": 4}
-BLOCK = {"sequential": 0, "parallel": 1, "sandwich": 2, "post": 3}
-MIXER = {"latent_attention": 0, "mamba2": 1, "gla": 2, "channel_delta": 3, "attention": 4}
+ACT = {"gelu": 0, "swiglu": 1, "geglu": 2, "clamped_glu": 3, "relu2": 4, "reglu": 5}
+BLOCK = {"sequential": 0, "parallel": 1, "sandwich": 2, "post": 3, "sum_norm": 4}
+MIXER = {"latent_attention": 0, "mamba2": 1, "gla": 2, "channel_delta": 3, "attention": 4, "lightning": 5}
+MAX_DECAYS = 128                        # NVL_MAX_DECAYS
 PRECISION = {"bf16": 0, "f32": 1}
 DTYPE_F32, DTYPE_BF16, DTYPE_F16 = 0, 1, 2
 LAYOUT_IN_OUT, LAYOUT_OUT_IN = 0, 1
@@ -68,6 +70,7 @@ class ModelConfigC(C.Structure):
         ("mamba_head_dim", C.c_int32), ("mamba_n_groups", C.c_int32), ("mamba_conv_kernel", C.c_int32),
         ("mamba_layer_mask", C.c_uint64 * 2),
         ("norm_weight_offset", C.c_float), ("logit_softcap", C.c_float), ("side_dim", C.c_int32),
+        ("stream_scale", C.c_float), ("token_shift", C.c_int32),
     ]
 
 
@@ -79,7 +82,11 @@ class LayerConfigC(C.Structure):        # nvl_layer_config
                 ("ffn_limit", C.c_float), ("kv_from", C.c_int32), ("rot_dim", C.c_int32), ("gate_per_head", C.c_int32), ("kv_heads", C.c_int32),
                 ("rot_base", C.c_double), ("rot_factor", C.c_double), ("rot_original", C.c_double), ("rot_fast", C.c_double), ("rot_slow", C.c_double),
                 ("softcap", C.c_float), ("v_mix", C.c_int32), ("ffn_act", C.c_int32), ("experts", C.c_int32), ("top_k", C.c_int32),
-                ("expert_dim", C.c_int32), ("expert_groups", C.c_int32), ("groups_kept", C.c_int32)]
+                ("expert_dim", C.c_int32), ("expert_groups", C.c_int32), ("groups_kept", C.c_int32),
+                ("chunk", C.c_int32), ("keep_first", C.c_int32), ("qk_norm", C.c_int32), ("sink", C.c_int32), ("qkv_bias", C.c_int32), ("ungated", C.c_int32),
+                ("rot_low", C.c_double), ("rot_high", C.c_double), ("out_scale", C.c_float), ("route_softmax", C.c_int32), ("expert_limit", C.c_float),
+                ("mixer2", C.c_int32), ("heads2", C.c_int32), ("dim2", C.c_int32), ("vdim2", C.c_int32), ("out_scale2", C.c_float),
+                ("decay", C.c_double * MAX_DECAYS)]
 
 
 class RuntimeOptsC(C.Structure):

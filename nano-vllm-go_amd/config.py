@@ -49,6 +49,8 @@ class ModelConfig:
     norm_weight_offset: float = 0.0
     logit_softcap: float = 0.0
     side_dim: int = 0                 # per-layer token inputs
+    stream_scale: float = 0.0         # norms of sums: factor of the residual stream
+    token_shift: int = 0
 
     @property
     def mamba_layer_mask(self):
@@ -140,8 +142,12 @@ def new_granite_config(size: str = "350m") -> ModelConfig:   # config.go:241-330
 LAYER_FIELDS = dict(mixer="", weights_of=-1, heads=0, dim=0, vdim=0, q_rank=0, kv_rank=0, window=0, scale=0.0, state=0, groups=0,
                     norm_groups=0, conv_taps=0, tau=0.0, decay_rank=0, ffn_dim=0, ffn_limit=0.0, kv_from=-1, rot_dim=0, gate_per_head=0, kv_heads=0,
                     rot_base=0.0, rot_factor=0.0, rot_original=0.0, rot_fast=0.0, rot_slow=0.0, softcap=0.0, v_mix=0, ffn_act=0, experts=0, top_k=0,
-                    expert_dim=0, expert_groups=0, groups_kept=0)      # nvl_layer_config
-ACT_SWIGLU = 1                                                         # NVL_ACT_SWIGLU (ffn_act)
+                    expert_dim=0, expert_groups=0, groups_kept=0, chunk=0, keep_first=0, qk_norm=0, sink=0, qkv_bias=0, ungated=0, rot_low=0.0, rot_high=0.0,
+                    out_scale=0.0, route_softmax=0, expert_limit=0.0, mixer2=0, heads2=0, dim2=0, vdim2=0, out_scale2=0.0, decay=())      # nvl_layer_config
+ACT_SWIGLU, ACT_CLAMPED_GLU = 1, 3                                     # NVL_ACT_* (ffn_act)
+QK_NORM_HEAD, QK_NORM_ROW = 1, 2                                       # NVL_QK_NORM_*
+SINK_ZERO, SINK_LEARNED = 1, 2                                         # NVL_SINK_*
+MIXER_LIGHTNING = 5                                                    # NVL_MIXER_LIGHTNING (mixer2)
 
 
 def _potuzen_layer(e: dict) -> dict:
@@ -237,7 +243,60 @@ def bolinex_config(raw: dict) -> ModelConfig:
                        side_dim=(raw.get("token_side") or {}).get("dim", 0), layers=[_bolinex_layer(e) for e in raw["layers"]])
 
 
-LAYERED = {"Potuzen": potuzen_config, "Lufazen": lufazen_config, "Bolinex": bolinex_config}      # architectures described by a list of layers
+def _medulorn_attention(mx: dict) -> dict:
+    """What the two attentions of the Medulorn design have in common."""
+    out = dict(heads=mx["heads"], kv_heads=mx["kv_heads"], dim=mx["dim"], vdim=mx["vdim"], scale=float(mx["scale"]), ungated=1)
+    rot = mx.get("rot")
+    if rot is not None:
+        out.update(rot_dim=rot["dims"], rot_base=float(rot["base"]))
+        sc = rot.get("scaling")
+        if sc is not None:
+            out.update({"rot_" + k: float(sc[k]) for k in ("factor", "original", "low", "high")})
+    return out
+
+
+def _medulorn_layer(e: dict) -> dict:
+    """One entry of a Medulorn config.json's layer list -> the fields of nvl_layer_config."""
+    mx, mlp, ty = e["mixer"], e.get("mlp"), e["type"]
+    out = dict(LAYER_FIELDS, mixer="attention")
+    if ty == "attention":
+        out.update(_medulorn_attention(mx), qk_norm=QK_NORM_HEAD, sink=SINK_ZERO, qkv_bias=1, chunk=(mx.get("mask") or {}).get("size", 0))
+    elif ty == "parallel":
+        left, right = mx["left"], mx["right"]
+        mask = left.get("mask") or {}
+        if len(right["decay"]) != right["heads"]:
+            raise ValueError("as many decays as heads expected")
+        out.update(_medulorn_attention(left), qk_norm=QK_NORM_ROW, sink=SINK_LEARNED, window=mask.get("size", 0), keep_first=mask.get("keep_first", 0),
+                   out_scale=float(mx["left_scale"]), mixer2=MIXER_LIGHTNING, heads2=right["heads"], dim2=right["dim"], vdim2=right["vdim"],
+                   out_scale2=float(mx["right_scale"]), decay=[float(d) for d in right["decay"]])
+    else:
+        raise ValueError(f"unknown mixer {ty!r}")
+    if mlp is None:
+        return out
+    kind = mlp.get("kind", "dense")
+    if kind == "moe":
+        out.update(expert_dim=mlp["expert"]["ff"], expert_limit=float(mlp["expert"]["limit"]), experts=mlp["router"]["experts"], top_k=mlp["router"]["top"],
+                   expert_groups=1, groups_kept=1, route_softmax=1)
+        if mlp.get("shared") is not None:
+            out.update(ffn_dim=mlp["shared"]["ff"], ffn_limit=float(mlp["shared"]["limit"]), ffn_act=ACT_CLAMPED_GLU)
+    elif kind == "dense":
+        out["ffn_dim"] = mlp["ff"]
+    else:
+        raise ValueError(f"unknown feed-forward kind {kind!r}")
+    return out
+
+
+def medulorn_config(raw: dict) -> ModelConfig:
+    """The Medulorn design: norms (one weight each) of alpha x + f(x), token shift in front of every mixer, chunked attention, and windowed
+    attention beside lightning attention; ReLU-gated or expert feed-forwards, capped logits."""
+    return ModelConfig(architecture="Medulorn", model_name="medulorn", vocab_size=raw["vocab"], hidden=raw["width"],
+                       num_layers=len(raw["layers"]), max_seq_len=4096, attention_type="gqa", norm_type="rmsnorm_scalar", position_type="nope",
+                       activation_type="reglu", block_style="sum_norm", rope_base=0.0, norm_eps=float(raw["norm"]["eps"]),
+                       embedding_multiplier=float(raw["embedding"]["scale"]), stream_scale=float(raw["postln_alpha"]), token_shift=1,
+                       logit_softcap=float(raw.get("logit_softcap") or 0.0), layers=[_medulorn_layer(e) for e in raw["layers"]])
+
+
+LAYERED = {"Medulorn": medulorn_config, "Potuzen": potuzen_config, "Lufazen": lufazen_config, "Bolinex": bolinex_config}      # architectures described by a list of layers
 
 
 def load_model_config(raw: dict | str) -> ModelConfig:

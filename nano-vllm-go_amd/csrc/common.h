@@ -77,6 +77,18 @@ __host__ __device__ __forceinline__ int grouped_k_row(int row) {
     return (row & ~31) + 16 * ((k >> 2) & 1) + 4 * (k >> 3) + (k & 3);
 }
 
+// Which keys a query sees, itself included: all earlier ones, those of its window (and the sequence's first `keep` tokens), or those of its
+// chunk of positions (chunks are counted from position 0).
+struct KeyMask {
+    int window, chunk, keep;          // 0: none; not both window and chunk; keep only with a window
+    __host__ __device__ __forceinline__ int lo(int pos) const {       // first key of the contiguous range that ends with the query
+        if (chunk > 0) return pos - pos % chunk;
+        return window > 0 && pos - window + 1 > 0 ? pos - window + 1 : 0;
+    }
+    __host__ __device__ __forceinline__ int span() const { return chunk > 0 ? chunk : window; }      // longest such range; 0: unlimited
+    bool operator==(const KeyMask& o) const { return window == o.window && chunk == o.chunk && keep == o.keep; }
+};
+
 __device__ __forceinline__ float gelu_tanh_f(float x) {
     // tensor.go:181-190: 0.5 x (1 + tanh(sqrt(2/pi) (x + 0.044715 x^3))), the tanh in float64 there.
     // tanh(u) = 1 - 2 / (exp(2u) + 1) on the hardware exp2 / rcp (both ~1 ulp): ABSOLUTE error ~1e-7, and only the absolute

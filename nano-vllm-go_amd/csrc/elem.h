@@ -321,6 +321,9 @@ struct SandwichArgs {
     int raw_next;             // w_next == NULL: xn = x
     // EXT instances
     const float* b_next;      // not NULL: the norm that follows is a layer norm with this bias
+    float sum_scale;          // not 0: the norm is of the sum, x = rms(sum_scale x + y) * w_post
+    // row kernel, one token per sequence (row r = sequence r), with raw_next: xn = x + (h - x) * shift, h the sequence's row before this one
+    const float* shift; float* before; int64_t before_stride; const int32_t *seq_slot, *seq_pos;      // kept in its slot: read, then replaced
     const float* y2;          // a second source, added as it is: [slices2][.][H], or with slot_of the rows slot_of[r * slices2 + k], weighted by gate_w
     int slices2; int64_t stride2;
     const int32_t* slot_of; const float* gate_w;
@@ -369,7 +372,25 @@ __global__ __launch_bounds__(256) void sandwich_row_kernel(SandwichArgs p, ActT*
         }
         ss += y[c][0] * y[c][0] + y[c][1] * y[c][1] + y[c][2] * y[c][2] + y[c][3] * y[c][3];
     }
-    if (EXT && p.y && !p.w_post) {
+    if (EXT && p.sum_scale != 0.f && p.y) {
+        ss = 0.f;
+#pragma unroll
+        for (int c = 0; c < MAXCH; c++) {
+            x[c] = p.sum_scale * x[c] + y[c];
+            ss += x[c][0] * x[c][0] + x[c][1] * x[c][1] + x[c][2] * x[c][2] + x[c][3] * x[c][3];
+        }
+        const float rms = sqrtf(block256_sum(ss, red) / (float)p.width + p.eps);
+#pragma unroll
+        for (int c = 0; c < MAXCH; c++) {
+            const int j = threadIdx.x + c * 256;
+            if (j < H4) {
+                const f32x4 w = *(const f32x4*)(p.w_post + j * 4);
+#pragma unroll
+                for (int k = 0; k < 4; k++) x[c][k] = (x[c][k] / rms) * w[k];
+                *(f32x4*)(xr + j * 4) = x[c];
+            }
+        }
+    } else if (EXT && p.y && !p.w_post) {
 #pragma unroll
         for (int c = 0; c < MAXCH; c++) {
             const int j = threadIdx.x + c * 256;
@@ -390,7 +411,21 @@ __global__ __launch_bounds__(256) void sandwich_row_kernel(SandwichArgs p, ActT*
         }
     }
     if (!p.w_next) {
-        if (p.raw_next)
+        if (EXT && p.shift) {
+            float* before = p.before + (int64_t)p.seq_slot[r] * p.before_stride;
+            const bool any = p.seq_pos[r] > 0;
+#pragma unroll
+            for (int c = 0; c < MAXCH; c++) {
+                const int j = threadIdx.x + c * 256;
+                if (j < H4) {
+                    const f32x4 mu = *(const f32x4*)(p.shift + j * 4);
+                    f32x4 h = f32x4{0.f, 0.f, 0.f, 0.f};
+                    if (any) h = *(const f32x4*)(before + j * 4);
+                    *(f32x4*)(before + j * 4) = x[c];
+                    act_store4<ActT>(xn, r, j * 4, p.H, x[c] + (h - x[c]) * mu);
+                }
+            }
+        } else if (p.raw_next)
 #pragma unroll
             for (int c = 0; c < MAXCH; c++) { const int j = threadIdx.x + c * 256; if (j < H4) act_store4<ActT>(xn, r, j * 4, p.H, x[c]); }
         return;
@@ -445,7 +480,29 @@ __global__ __launch_bounds__(1024) void sandwich_tile16_kernel(SandwichArgs p, b
             const int j = lane + c * 64;
             x[c] = j < H4 ? *(const f32x4*)(xr + j * 4) : f32x4{0.f, 0.f, 0.f, 0.f};
         }
-        if (EXT && p.y && !p.w_post) {
+        if (EXT && p.sum_scale != 0.f && p.y) {
+            float ss = 0.f;
+#pragma unroll
+            for (int c = 0; c < MAXCH; c++) {
+                const int j = lane + c * 64;
+                if (j < H4) {
+                    x[c] = p.sum_scale * x[c] + *(const f32x4*)(p.y + (int64_t)r * p.H + j * 4);
+                    if (p.y2) x[c] += sandwich_more(p, r, j * 4);
+                }
+                ss += x[c][0] * x[c][0] + x[c][1] * x[c][1] + x[c][2] * x[c][2] + x[c][3] * x[c][3];
+            }
+            const float rms = sqrtf(wave_sum(ss) / (float)p.width + p.eps);
+#pragma unroll
+            for (int c = 0; c < MAXCH; c++) {
+                const int j = lane + c * 64;
+                if (j < H4) {
+                    const f32x4 w = *(const f32x4*)(p.w_post + j * 4);
+#pragma unroll
+                    for (int k = 0; k < 4; k++) x[c][k] = (x[c][k] / rms) * w[k];
+                    *(f32x4*)(xr + j * 4) = x[c];
+                }
+            }
+        } else if (EXT && p.y && !p.w_post) {
 #pragma unroll
             for (int c = 0; c < MAXCH; c++) {
                 const int j = lane + c * 64;
@@ -527,6 +584,55 @@ __global__ __launch_bounds__(1024) void sandwich_tile16_kernel(SandwichArgs p, b
     if (blockIdx.x * 16 + lr < p.rows)
         for (int kb = wave; kb < nkb; kb += 16)
             *(bf16x8*)(xn + (((int64_t)blockIdx.x * nkb + kb) * 64 + lane) * 8) = *(const bf16x8*)(tile + lr * p.H + kb * 32 + lc * 8);
+}
+
+// ---------------------------------------------------------------------------------------
+// Token shift of batches with more than one token per sequence: xn[t] = x[t] + (x[t - 1] - x[t]) * mu.  The row before a sequence's first
+// token of this call is its slot's (zeros at position 0), taken from a copy made when the pass began (shift_copy_kernel: one row per layer
+// and sequence), because the launch also leaves the sequence's last row in its slot.  bf16: one workgroup per 16 rows, a lane is a row of
+// the operand block it writes; fp32 mode: one workgroup per row.
+// ---------------------------------------------------------------------------------------
+struct ShiftArgs {
+    const float* x; const float* mu;
+    const float* copy;                // [sequence][H] of this layer
+    float* state; int64_t slot_stride;      // slot s keeps its row at state + s * slot_stride
+    const int32_t *tok_seq, *tok_pos, *seq_tok_start, *seq_len, *seq_pos, *seq_slot;
+    int rows, H;
+};
+__device__ __forceinline__ f32x4 token_shift4(const ShiftArgs& p, int t, int seq, int c) {
+    const int first = p.seq_tok_start[seq];
+    const f32x4 x = *(const f32x4*)(p.x + (int64_t)t * p.H + c), mu = *(const f32x4*)(p.mu + c);
+    f32x4 h = f32x4{0.f, 0.f, 0.f, 0.f};
+    if (t > first) h = *(const f32x4*)(p.x + (int64_t)(t - 1) * p.H + c);
+    else if (p.seq_pos[seq] > 0) h = *(const f32x4*)(p.copy + (int64_t)seq * p.H + c);
+    if (t == first + p.seq_len[seq] - 1) *(f32x4*)(p.state + (int64_t)p.seq_slot[seq] * p.slot_stride + c) = x;
+    return x + (h - x) * mu;
+}
+template <typename ActT>
+__global__ __launch_bounds__(1024) void token_shift_kernel(ShiftArgs p, ActT* __restrict__ xn) {
+    if constexpr (sizeof(ActT) == 4) {
+        const int t = blockIdx.x, seq = p.tok_seq[t];
+        for (int c = threadIdx.x * 4; c < p.H; c += blockDim.x * 4) act_store4<ActT>(xn, t, c, p.H, token_shift4(p, t, seq, c));
+    } else {
+        const int lane = threadIdx.x & 63, t = blockIdx.x * 16 + (lane & 15), NW = blockDim.x >> 6;
+        if (t >= p.rows) return;
+        const int seq = p.tok_seq[t];
+        for (int kb = threadIdx.x >> 6; kb < (p.H >> 5); kb += NW) {
+            const int c = kb * 32 + (lane >> 4) * 8;
+            const f32x4 a = token_shift4(p, t, seq, c), b = token_shift4(p, t, seq, c + 4);
+            bf16x8 o;
+#pragma unroll
+            for (int r = 0; r < 4; r++) { o[r] = (bf16_t)a[r]; o[4 + r] = (bf16_t)b[r]; }
+            *(bf16x8*)(xn + (((int64_t)blockIdx.x * (p.H >> 5) + kb) * 64 + lane) * 8) = o;
+        }
+    }
+}
+// grid (sequences, layers): every layer's kept row -> copy [layer][max_seqs][H]; layer l's row lies at off[l] in a slot
+__global__ __launch_bounds__(256) void shift_copy_kernel(const float* __restrict__ state, int64_t slot_stride, const int64_t* __restrict__ off,
+                                                         const int32_t* __restrict__ seq_slot, float* __restrict__ copy, int max_seqs, int H) {
+    const float* s = state + (int64_t)seq_slot[blockIdx.x] * slot_stride + off[blockIdx.y];
+    float* d = copy + ((int64_t)blockIdx.y * max_seqs + blockIdx.x) * H;
+    for (int c = threadIdx.x * 4; c < H; c += 1024) *(f32x4*)(d + c) = *(const f32x4*)(s + c);
 }
 
 // Debug tap (nvl_set_debug mode 2): the residual stream after a layer as the NEXT kernel will see it — x plus whatever a
@@ -619,6 +725,19 @@ __global__ void swiglu_kernel(const float* __restrict__ h, ActT* __restrict__ y,
     const int64_t r = i / F; const int f = (int)(i - r * F);
     const float g = h[r * 2 * F + f], u = h[r * 2 * F + F + f];
     ActIO<ActT>::st(y + r * ld + col + f, (GELU ? gelu_tanh_f(g) : g / (1.0f + expf(-g))) * u);
+}
+// h [rows][2F] (gate | up) -> y [rows][F]: max(gate, 0) * up
+template <typename ActT>
+__global__ void reglu_kernel(const float* __restrict__ h, ActT* __restrict__ y, int64_t rows, int F) {
+    const int64_t i = (int64_t)blockIdx.x * blockDim.x + threadIdx.x;
+    if (i >= rows * F) return;
+    const int64_t r = i / F; const int f = (int)(i - r * F);
+    ActIO<ActT>::st(y + i, fmaxf(h[r * 2 * F + f], 0.f) * h[r * 2 * F + F + f]);
+}
+// columns [c0, c0 + n) of fp32 rows through silu, in place
+static __global__ __launch_bounds__(256) void silu_cols_kernel(float* __restrict__ x, int64_t ld, int c0, int n) {
+    float* r = x + (int64_t)blockIdx.x * ld + c0;
+    for (int i = threadIdx.x; i < n; i += 256) r[i] = r[i] / (1.0f + expf(-r[i]));
 }
 template <typename ActT>
 __global__ void clamp_glu_kernel(const float* __restrict__ h, ActT* __restrict__ y, int64_t rows, int F, float limit, float slope) {
@@ -761,6 +880,8 @@ __global__ void scale_rows_kernel(float* __restrict__ x, int ld, int n, float di
 // position advanced by one (cmd/ask/main.go:315-320), the embedding gather of that token (embed_kernel,
 // generic_model.go:567-592) and layer 0's norm of the row (norm_row_kernel) — same arithmetic, same summation order.
 // ---------------------------------------------------------------------------------------
+// token shift in front of layer 0 (mu not NULL): the row before is the embedding of the token this step ran, which the slot keeps too
+struct SeamShift { const float* mu; float* state; int64_t slot_stride; const int32_t* seq_slot; };
 __global__ __launch_bounds__(256) void decode_seam_kernel(const float* __restrict__ pval, const int32_t* __restrict__ pidx,
                                                           int chunks, const int32_t* __restrict__ sampled,
                                                           int32_t* __restrict__ hist, int64_t hist_stride,
@@ -771,9 +892,9 @@ __global__ __launch_bounds__(256) void decode_seam_kernel(const float* __restric
                                                           const bf16_t* __restrict__ emb, const bf16_t* __restrict__ pos_emb,
                                                           int max_seq, float mult, float* __restrict__ x,
                                                           const float* __restrict__ w, const float* __restrict__ b,
-                                                          float eps, bf16_t* __restrict__ y, int H, int width) {
+                                                          float eps, bf16_t* __restrict__ y, int H, int width, SeamShift sh) {
     __shared__ float red[4];
-    __shared__ int tok_s, pos_s;
+    __shared__ int tok_s, pos_s, old_s;
     const int r = blockIdx.x;
     if (threadIdx.x < 64) {
         float best = -INFINITY;
@@ -792,6 +913,7 @@ __global__ __launch_bounds__(256) void decode_seam_kernel(const float* __restric
                 hist_len[r] = n + 1;
             }
             const int pos = tok_pos[r] + 1;
+            old_s = tokens[r];
             // ring row = steps since the loop started (from the positions, so every step's launch has the same arguments)
             argmax_out[r] = t; ring_out[(int64_t)(pos - 1 - ring_pos0[r]) * ring_rows + r] = t; tokens[r] = t;
             tok_pos[r] = pos; seq_pos[r] = pos;          // (one token per sequence: row r IS sequence r)
@@ -821,7 +943,15 @@ __global__ __launch_bounds__(256) void decode_seam_kernel(const float* __restric
             }
             *(f32x4*)(xr + j * 4) = v[c];
             if (w) ww[c] = *(const f32x4*)(w + j * 4);
-            else act_store4<bf16_t>(y, r, j * 4, H, v[c]);           // no norm in front of layer 0
+            else if (sh.mu) {
+                const bf16x4 o = *(const bf16x4*)(emb + fm_index(old_s, j * 4, H));
+                const f32x4 mu = *(const f32x4*)(sh.mu + j * 4);
+                f32x4 h;
+#pragma unroll
+                for (int k = 0; k < 4; k++) h[k] = mult != 0.f ? (float)o[k] * mult : (float)o[k];
+                *(f32x4*)(sh.state + (int64_t)sh.seq_slot[r] * sh.slot_stride + j * 4) = h;
+                act_store4<bf16_t>(y, r, j * 4, H, v[c] + (h - v[c]) * mu);
+            } else act_store4<bf16_t>(y, r, j * 4, H, v[c]);           // no norm in front of layer 0
             if (b) bb[c] = *(const f32x4*)(b + j * 4);
         }
     }
@@ -977,12 +1107,14 @@ __global__ __launch_bounds__(1024) void moe_plan_kernel(const float* __restrict_
 // Group-limited routing on sigmoid scores.  s = sigmoid(z); the choice goes by s + correction, the weights are the s of the chosen
 // experts as they are.  Experts form `groups` equal groups of neighbours; a group counts as much as its two largest choice scores
 // together, and only the experts of the best `keep` groups can be chosen.  Ties go to the lower index.  One wave per token, E <= 256;
+// `softmax`: the choice goes by z + correction, and the weights are the softmax over the chosen ones of these (no groups).
 // writes (id, weight) in rank order, or with `gate` the dense [rows][gate_ld] matrix of weights (0: not chosen).  Workgroups with
 // blockIdx.y > 0 finish a SwiGLU feed-forward whose fp32 gate and up columns the same projection made (a small shared expert):
 // grid (ceil(rows / 4), 1 + ceil(F / 256)).
 constexpr int ROUTE_MAX_E = 256;
 struct GroupRouteArgs { const float* logits; int64_t ld; const float* correction; int rows, E, top, groups, keep; int32_t* ids; float* w; float* gate; int gate_ld;
-                        const float* glu; int F; void* out; int64_t out_ld; int out_col; };      // glu: [rows][ld] = [gate F | up F]; out: columns out_col ..
+                        const float* glu; int F; void* out; int64_t out_ld; int out_col;         // glu: [rows][ld] = [gate F | up F]; out: columns out_col ..
+                        int softmax, n_always; };                                                // n_always: gate columns E .. that are one
 template <typename ActT>
 __global__ __launch_bounds__(256) void moe_route_grouped_kernel(GroupRouteArgs p) {
     __shared__ float choice_s[4][ROUTE_MAX_E], group_s[4][ROUTE_MAX_E];
@@ -1006,8 +1138,9 @@ __global__ __launch_bounds__(256) void moe_route_grouped_kernel(GroupRouteArgs p
             const int e = lane + 64 * i;
             s[i] = 0.f;
             if (e < p.E) {
-                s[i] = 1.0f / (1.0f + expf(-p.logits[r * p.ld + e]));
-                choice[e] = s[i] + (p.correction ? p.correction[e] : 0.f);
+                const float z = p.logits[r * p.ld + e];
+                s[i] = p.softmax ? z + (p.correction ? p.correction[e] : 0.f) : 1.0f / (1.0f + expf(-z));
+                choice[e] = p.softmax ? s[i] : s[i] + (p.correction ? p.correction[e] : 0.f);
             }
         }
     __syncthreads();
@@ -1037,13 +1170,32 @@ __global__ __launch_bounds__(256) void moe_route_grouped_kernel(GroupRouteArgs p
         if (r < p.rows && e < p.E && !in[i]) choice[e] = -INFINITY;       // (read by nobody but this lane so far)
     }
     __syncthreads();
+    int ranks[ROUTE_MAX_E / 64];
+    float top_z = -INFINITY, sum = 0.f;
 #pragma unroll
     for (int i = 0; i < ROUTE_MAX_E / 64; i++) {
         const int e = lane + 64 * i;
-        if (r < p.rows && p.gate && e >= p.E && e < p.gate_ld) p.gate[(int64_t)r * p.gate_ld + e] = 0.f;       // padding experts
+        ranks[i] = p.top;
+        if (in[i]) { ranks[i] = 0; for (int j = 0; j < p.E; j++) { const float v = choice[j]; ranks[i] += v > c[i] || (v == c[i] && j < e); } }
+        if (in[i]) top_z = fmaxf(top_z, c[i]);
+    }
+    if (p.softmax) {
+        top_z = wave_max(top_z);
+#pragma unroll
+        for (int i = 0; i < ROUTE_MAX_E / 64; i++) {
+            s[i] = in[i] && ranks[i] < p.top ? expf(s[i] - top_z) : 0.f;
+            sum += s[i];
+        }
+        sum = wave_sum(sum);
+#pragma unroll
+        for (int i = 0; i < ROUTE_MAX_E / 64; i++) s[i] /= sum;
+    }
+    if (r < p.rows && p.gate) for (int e = p.E + lane; e < p.gate_ld; e += 64) p.gate[(int64_t)r * p.gate_ld + e] = e < p.E + p.n_always ? 1.0f : 0.f;       // the others are padding
+#pragma unroll
+    for (int i = 0; i < ROUTE_MAX_E / 64; i++) {
+        const int e = lane + 64 * i;
         if (r >= p.rows || e >= p.E) continue;
-        int rank = 0;
-        if (in[i]) for (int j = 0; j < p.E; j++) { const float v = choice[j]; rank += v > c[i] || (v == c[i] && j < e); }
+        const int rank = ranks[i];
         const bool chosen = in[i] && rank < p.top;
         if (p.gate) p.gate[(int64_t)r * p.gate_ld + e] = chosen ? s[i] : 0.f;
         else if (chosen) { p.ids[(int64_t)r * p.top + rank] = e; p.w[(int64_t)r * p.top + rank] = s[i]; }

@@ -44,10 +44,13 @@ enum GemmEpi {
     EPI_GEGLU = 5,   // C[m, f] = gelu_tanh(gate) * up   W rows interleaved as for EPI_SWIGLU
     EPI_RELU2 = 7,   // C = max(acc, 0)^2
     EPI_GROUPED = 9,     // fused input projection of grouped-query attention (grouped.h): every column range goes where it is used, GroupedEpi
+    EPI_GROUPED_RAW = 11,    // ... of attention whose queries and keys are normed or rotated first: those go to fp32 rows, as does what lies behind the gate
+    EPI_REGLU = 10,      // C[m, f] = max(gate, 0) * up   W rows interleaved as for EPI_SWIGLU
     EPI_GELU_TOK = 8,    // C[m, n] = gelu_tanh(acc) * tok_table[tok_ids[m]][n]   (an input of the token's own, GemmArgs::tok_*)
 };
 
-constexpr bool epi_glu(int epi) { return epi == 2 || epi == 5 || epi == 6; }      // gate | up pairs in, one column out
+constexpr bool epi_moe(int epi) { return epi == 2 || epi == 6; }      // ... with instances for masked experts
+constexpr bool epi_glu(int epi) { return epi == 2 || epi == 5 || epi == 6 || epi == 10; }      // gate | up pairs in, one column out
 
 struct QkvEpi {             // EPI_QKV only
     const int32_t* tok_pos;
@@ -70,6 +73,8 @@ struct GroupedEpi {         // EPI_GROUPED: columns [q | k | v | gate | feed-for
     int mix; const float* lambda; float* vfirst; int64_t vfirst_ld;
     bf16_t* ffn; int64_t ffn_ld;                                   // [ffn0, route0): max(., 0)^2 -> the output projection's operand (fragment-major, shifted to its columns)
     float* route; int64_t route_ld;                                // from route0 on: fp32 rows
+    // EPI_GROUPED_RAW: queries and keys, and everything from raw0 on, to fp32 rows at their own columns; [raw0, silu1): through silu
+    float* raw; int64_t raw_ld; int raw0, silu1;
 };
 
 struct GemmArgs {
@@ -82,6 +87,7 @@ struct GemmArgs {
     const float* bias;      // [N] or NULL
     float alpha;            // EPI_RESID multiplier
     float glu_limit, glu_slope;     // EPI_CLAMP_GLU
+    float glu_limit2; int glu_from2;      // ... masked experts: the limit of output columns from glu_from2 on
     const int32_t* tok_ids; const bf16_t* tok_table; int64_t tok_ld;      // EPI_GELU_TOK: row-major, rows of 4 k entries
     int M, N, K;            // logical sizes
     const int32_t* seg;     // optional device {start,end}: rows [start,end) of A (via a_rows if set)
@@ -177,6 +183,20 @@ __device__ __forceinline__ void epilogue_grouped4(const GemmArgs& p, int64_t row
     for (int r = 0; r < 4; r++) d[8 * r] = (bf16_t)v[r];
 }
 
+// EPI_GROUPED_RAW
+__device__ __forceinline__ float silu_f(float g);
+__device__ __forceinline__ void epilogue_grouped_raw4(const GemmArgs& p, int64_t row, int n, f32x4 v) {
+    const GroupedEpi& e = p.grp;
+    if (n >= e.v0 && n < e.raw0) { epilogue_grouped4(p, row, n, v); return; }        // values and gates
+    if (n < e.silu1 && n >= e.raw0)
+#pragma unroll
+        for (int r = 0; r < 4; r++) v[r] = silu_f(v[r]);
+    float* c = e.raw + row * e.raw_ld + n;
+    if (n + 3 < p.N) { *(f32x4*)c = v; return; }      // (rows of 4 k floats)
+#pragma unroll
+    for (int r = 0; r < 4; r++) if (n + r < p.N) c[r] = v[r];
+}
+
 __device__ __forceinline__ float silu_f(float g) { return g / (1.0f + __expf(-g)); }
 __device__ __forceinline__ float deferred_rstd(const GemmArgs& p, int m);
 
@@ -203,6 +223,7 @@ __device__ __forceinline__ void epilogue4(const GemmArgs& p, int m, int n, f32x4
     }
     const int64_t row = (int64_t)p.c_row0 + m;
     if (EPI == EPI_GROUPED) { epilogue_grouped4(p, row, n, v); return; }
+    if (EPI == EPI_GROUPED_RAW) { epilogue_grouped_raw4(p, row, n, v); return; }
     if (EPI == EPI_GELU_TOK) {
         const bf16x4 e = *(const bf16x4*)(p.tok_table + (int64_t)p.tok_ids[row] * p.tok_ld + n);
 #pragma unroll
@@ -264,7 +285,8 @@ __device__ __forceinline__ void epilogue_glu4(const GemmArgs& p, int m, int f, f
     f32x4 v;
 #pragma unroll
     for (int r = 0; r < 4; r++) {
-        if constexpr (EPI == EPI_CLAMP_GLU) v[r] = clamp_glu_f(g[r], u[r], p.glu_limit, p.glu_slope);
+        if constexpr (EPI == EPI_CLAMP_GLU) v[r] = clamp_glu_f(g[r], u[r], MOE && f >= p.glu_from2 ? p.glu_limit2 : p.glu_limit, p.glu_slope);
+        else if constexpr (EPI == EPI_REGLU) v[r] = fmaxf(g[r], 0.f) * u[r];
         else v[r] = (EPI == EPI_GEGLU ? gelu_tanh_f(g[r]) : silu_f(g[r])) * u[r];
     }
     if constexpr (MOE) v *= p.moe_gate[m * p.moe_E + f / p.moe_I];      // routing weight of (token, expert); 0 = not routed
@@ -748,7 +770,7 @@ __global__ __launch_bounds__(1024) void gemm_skinny_bf16_kernel(GemmArgs p) {
     uint32_t blk_live = 0xffffffffu;
     bool tail_live = true;                 // the ragged tail (fewer than U k-steps; it lies inside the range's last expert)
     if constexpr (MOE) {
-        if (EPI == EPI_SWIGLU) { if (!moe_expert_live(p, (nt0 * 16) / (2 * p.moe_I))) return; }          // (whole workgroup: uniform)
+        if (epi_moe(EPI)) { if (!moe_expert_live(p, (nt0 * 16) / (2 * p.moe_I))) return; }          // (whole workgroup: uniform)
         else {
             const int spe = p.moe_I >> 5, e0 = ks0 / spe, e1 = (ks0 + my_steps - 1) / spe;      // k-steps per expert; this wave's experts
             float g[4];
@@ -919,9 +941,11 @@ __global__ __launch_bounds__(1024) void gemm_skinny_bf16_kernel(GemmArgs p) {
 // the router as a skinny GEMM launch (4.6 us) + moe_gate_kernel (4.5 us).  grid = 16-row tiles of the batch, 1024
 // threads: wave w takes expert tile w % ET over K slice w / ET (fragments straight from L2 / HBM, as the skinny kernel),
 // the K slices are summed through LDS in wave order, then wave r routes row r of the tile with a lane per expert.
-// p: A (fragment-major operand, possibly the deferred-norm raw form with rs_in), W (router, fragment-major), M, N = E, K.
+// p: A (fragment-major operand, possibly the deferred-norm raw form with rs_in), W (router, fragment-major), bias, M, N = E, K.
+// The gate's columns E .. E + n_always - 1 are one (experts every token takes), those up to gate_ld zero.
 // ------------------------------------------------------------------------------------------
-static __global__ __launch_bounds__(1024) void moe_router_gate_kernel(GemmArgs p, int top_k, float* __restrict__ gate, float* __restrict__ logits_out, int ld_logits) {
+static __global__ __launch_bounds__(1024) void moe_router_gate_kernel(GemmArgs p, int top_k, float* __restrict__ gate, float* __restrict__ logits_out, int ld_logits,
+                                                                      int gate_ld, int n_always) {
     __shared__ f32x4 red[16][64];
     __shared__ float lg[16][64];
     const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
@@ -972,7 +996,7 @@ static __global__ __launch_bounds__(1024) void moe_router_gate_kernel(GemmArgs p
     const int m = row0 + wave;
     if (m >= p.M) return;
     const float rstd = p.rs_in ? 1.0f / sqrtf(ssq * p.rs_inv_h + p.rs_eps) : 1.0f;
-    const float v = (lane < E) ? lg[wave][lane] * rstd : -INFINITY;
+    const float v = (lane < E) ? lg[wave][lane] * rstd + (p.bias ? p.bias[lane] : 0.f) : -INFINITY;
     if (logits_out && lane < E) logits_out[(int64_t)m * ld_logits + lane] = v;
     float mx = v;
 #pragma unroll
@@ -994,13 +1018,14 @@ static __global__ __launch_bounds__(1024) void moe_router_gate_kernel(GemmArgs p
         const int src = __ffsll((unsigned long long)__ballot(rank == k)) - 1;
         wsum += __builtin_bit_cast(float, __builtin_amdgcn_readlane(pbits, src));
     }
-    if (lane < E) gate[(int64_t)m * E + lane] = rank < top_k ? prob / wsum : 0.f;      // moe.go:103
+    if (lane < E) gate[(int64_t)m * gate_ld + lane] = rank < top_k ? prob / wsum : 0.f;      // moe.go:103
+    for (int e = E + lane; e < gate_ld; e += 64) gate[(int64_t)m * gate_ld + e] = e < E + n_always ? 1.0f : 0.f;
 }
 #endif
 
 // ------------------------------------------------------------------------------------------
 // fp32 kernel (parity mode): 64x64 tile, BK=16, 256 threads, 4x4 outputs per thread, k ascending.
-// EPI_SWIGLU / EPI_GEGLU / EPI_CLAMP_GLU are not instantiated: the f32 path keeps W1 un-interleaved and applies the
+// The gated epilogues are not instantiated: the f32 path keeps W1 un-interleaved and applies the
 // activation with swiglu_kernel.
 // ------------------------------------------------------------------------------------------
 template <int EPI, typename OutT>
@@ -1270,7 +1295,7 @@ static inline bool launch_gemm_skinny_ntw(hipStream_t st, const GemmArgs& a) {
     else {
         // (the MoE gate/up projection counts every expert's workgroups, but those of experts no token picked exit at once:
         //  twice the budget — Granite-1B B=8 decode 6.50 K -> 6.60 K tok/s, profiles/r03_moe_decode_experiments.txt)
-        const int64_t budget = (int64_t)g_narrow_waves * ((a.moe_gate && EPI == EPI_SWIGLU) ? 2 : 1);
+        const int64_t budget = (int64_t)g_narrow_waves * ((a.moe_gate && epi_moe(EPI)) ? 2 : 1);
         while (ksplit > 1 && (int64_t)nblocks * KS * NTW * ksplit > budget) ksplit >>= 1;
     }
     while (ksplit > 1 && ((a.K >> 5) / (ksplit * KS) < U || ksplit * NTW > 16)) ksplit >>= 1;   // >= one block of U k-steps per wave
@@ -1285,7 +1310,7 @@ static inline bool launch_gemm_skinny_ntw(hipStream_t st, const GemmArgs& a) {
     if (a.grid_y != KS) { GemmArgs c = a; c.grid_y = KS; return launch_gemm_skinny_ntw<NTW, EPI, OutT>(st, c); }
 #define NVL_SK(MTv, Uv) hipLaunchKernelGGL((gemm_skinny_bf16_kernel<MTv, NTW, Uv, EPI, OutT>), grid, block, lds, st, a)
 #define NVL_SKM(MTv, Uv) hipLaunchKernelGGL((gemm_skinny_bf16_kernel<MTv, NTW, Uv, EPI, OutT, false, true>), grid, block, lds, st, a)
-    if constexpr (EPI == EPI_SWIGLU || EPI == EPI_RESID) {
+    if constexpr (epi_moe(EPI) || EPI == EPI_RESID) {
         if (a.moe_gate) {                                 // MoE decode instantiation (expert skip + gate weight)
             if (a.m_passes > 1) return false;
             if (MT == 1) NVL_SKM(1, 4); else if (MT == 2) NVL_SKM(2, 4); else NVL_SKM(4, 2);
@@ -1335,7 +1360,7 @@ static inline bool launch_gemm_skinny_wide(hipStream_t st, const GemmArgs& a) {
         hipLaunchKernelGGL((gemm_skinny_wide_bf16_kernel<MTv, NTB, Uv, EPI, OutT, false, true>), dim3(wgs), dim3(ksplit * 64), \
                            lds, st, a);                                                                                \
     } while (0)
-    if constexpr (EPI == EPI_SWIGLU) {
+    if constexpr (epi_moe(EPI)) {
         if (a.moe_gate) {
             if (a.m_passes > 1) return false;
             if (MT == 1) NVL_SKWM(1, 4); else if (MT == 2) NVL_SKWM(2, 4); else NVL_SKWM(4, 2);
@@ -1353,7 +1378,7 @@ static inline bool launch_gemm_skinny_bf16(hipStream_t st, const GemmArgs& a0) {
     if (skinny_rows(a0) > 64 || a0.a_rows || a0.seg || a0.tile_map) return false;
     GemmArgs a = a0;
     a.x_mask = (g_x_mask && a0.M % 16 != 0) ? 1 : 0;     // padded rows of the last 16-row activation tile are not fetched
-    if constexpr (epi_glu(EPI) || EPI == EPI_STORE || EPI == EPI_GELU || EPI == EPI_RELU2 || EPI == EPI_GROUPED) {
+    if constexpr (epi_glu(EPI) || EPI == EPI_STORE || EPI == EPI_GELU || EPI == EPI_RELU2 || EPI == EPI_GROUPED || EPI == EPI_GROUPED_RAW) {
         // wide-N form once its 64-row groups fill the chip (g_force_ntw: 8 forces it, 1/2/4 force the narrow form)
         const bool wide_ok = skinny_rows(a) > 16 && cdiv(a.N, 64) >= 256 && !a.sk_part;   // M <= 16: the narrow form streams as fast
         if (g_force_ntw == 8 || (g_force_ntw == 0 && wide_ok)) { if (launch_gemm_skinny_wide<EPI, OutT>(st, a)) return true; }
@@ -1473,7 +1498,8 @@ void launch_gemm_f32(hipStream_t st, const GemmArgs& a) {
 // The projections' kernels are compiled per epilogue, side by side (gemm_inst.hip): (epilogue, output type)
 #define NVL_GEMM_BF16_INSTANCES(X)                                                                                              \
     X(EPI_STORE, float) X(EPI_STORE, bf16_t) X(EPI_RESID, float) X(EPI_SWIGLU, bf16_t) X(EPI_GELU, bf16_t) X(EPI_GEGLU, bf16_t) \
-    X(EPI_CLAMP_GLU, bf16_t) X(EPI_QKV, bf16_t) X(EPI_GROUPED, bf16_t) X(EPI_RELU2, bf16_t) X(EPI_GELU_TOK, bf16_t)
+    X(EPI_CLAMP_GLU, bf16_t) X(EPI_QKV, bf16_t) X(EPI_GROUPED, bf16_t) X(EPI_RELU2, bf16_t) X(EPI_GELU_TOK, bf16_t) \
+    X(EPI_REGLU, bf16_t) X(EPI_GROUPED_RAW, bf16_t)
 #define NVL_GEMM_F32_INSTANCES(X) X(EPI_STORE) X(EPI_RESID) X(EPI_GELU)
 #ifndef NVL_GEMM_INST
 #define NVL_X(E, T) extern template void launch_gemm_bf16<E, T>(hipStream_t, const GemmArgs&);

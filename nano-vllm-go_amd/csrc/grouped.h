@@ -1,9 +1,11 @@
 // grouped.h — grouped-query attention of models described by a list of layers: H query heads share G key/value heads, query/key and
 // value sizes differ freely, and every score passes through
 //     s = q . k * scale;   s <- softcap tanh(s / softcap);   s <- s - r1 ln(1 + r2 (i - j))
-// (cap and bias are optional, r1 and r2 belong to the query head) before an ordinary softmax over an optional sliding window.  The
-// values may be mixed with those of an earlier layer before they are cached; the concatenated heads are multiplied by sigmoid(gate).
-// Scores, cap, bias, softmax and their sums are fp32.
+// (cap and bias are optional, r1 and r2 belong to the query head) before a softmax over the keys of a KeyMask (common.h) and, with a sink,
+// one more entry of the denominator that has a score of its own and neither key nor value.  Queries and keys may be normed (per head or
+// over the whole projection) and rotated first: grouped_qk_*_kernel, on the fp32 rows the projection leaves.  The values may be mixed with
+// those of an earlier layer before they are cached; the concatenated heads are multiplied by sigmoid(gate) where there is a gate.
+// Norms, angles, scores, cap, bias, softmax and their sums are fp32.
 //
 // Cache: blocks of `bs` tokens (64 | bs) named by block tables.  A layer's part of a block is [G][bs][dp] keys, then [G][vp][bs] values,
 // dp / vp = padded head sizes (the padding is zero).  bf16: both are stored as the MFMA operand blocks they are read as (common.h
@@ -24,13 +26,22 @@ namespace nvl {
 
 struct GroupedArgs {
     int H, G, group, dim, dp, vdim, vp;
-    int window;                                   // 0: every earlier token
+    KeyMask mask;
     float scale, softcap;                         // softcap 0: none
     const float *r1, *r2;                         // [H] or NULL: no distance bias
+    const float* sink;                            // [H] scores of the denominator's own entry, or NULL
+    float out_scale;
     const void* q; int64_t q_ld;                  // queries of head h at column h dp, its gate at column gate_col + h vp: bf16 (fragment-major) or the fp32 rows of proj
-    int gate_col;
+    int gate_col;                                 // < 0: no gate
     const float* proj; int64_t proj_ld;           // fp32 mode: [token][q : H dp | k : G dp | v : G vp | gate : H vp | ...] of the fused input projection
-    int k_off, v_off;
+    int k_off, v_off;                             // k_off < 0: the keys are in the cache already
+    // normed and / or rotated queries and keys (grouped_qk_*_kernel): fp32 columns [0, H dp) and [qk_koff, + G dp) of proj
+    int qk_koff, qk_norm, rot;                    // qk_norm: 0 none, 1 per head, 2 over the projection; rot: rotated dimensions
+    const float *q_norm, *k_norm;                 // [dim] or [heads dim]
+    const f32x2* turn;                            // [position][rot / 2] (cos, sin)
+    float eps;
+    void* q_out;                                  // what `q` is read from: [token][q_ld]
+    const int32_t *tok_pos, *tok_tbl; int rows;
     int mix;                                      // values: 0 as they are, 1 also the model's first (kept in vfirst), 2 mixed with vfirst
     const float* lambda; float* vfirst; int64_t vfirst_ld;      // [token][G vp]
     void* cache; int64_t block_stride; int bs;    // this layer's part of block 0; elements between blocks
@@ -57,13 +68,152 @@ static __global__ __launch_bounds__(256) void grouped_place_kernel(GroupedArgs p
         const int64_t t = tok0 + pos - pos0;
         const int row = row0 + pos - u0;
         const float* pr = p.proj + t * p.proj_ld;
-        for (int c = threadIdx.x; c < p.dp; c += 256) kc[(int64_t)row * p.dp + c] = pr[p.k_off + g * p.dp + c];
+        if (p.k_off >= 0) for (int c = threadIdx.x; c < p.dp; c += 256) kc[(int64_t)row * p.dp + c] = pr[p.k_off + g * p.dp + c];
         for (int c = threadIdx.x; c < p.vp; c += 256) {
             float v = pr[p.v_off + g * p.vp + c];
             float* f = p.vfirst + t * p.vfirst_ld + g * p.vp + c;
             if (p.mix == 1) *f = v;
             else if (p.mix == 2) v = (1.0f - lam) * v + lam * *f;
             vc[(int64_t)row * p.vp + c] = v;
+        }
+    }
+}
+
+// ---- queries and keys of the batch's tokens: RMS norm, rotation; queries to q_out, keys to their cache rows ----
+// where the key of token t and head g goes (its channel 0): bf16 an operand block's row, fp32 mode a plain row
+template <typename T>
+__device__ __forceinline__ T* grouped_key_row(const GroupedArgs& p, int64_t t, int g, int& row) {
+    int blk;
+    kv_locate(p.blk_table, p.tok_tbl[t], p.tok_pos[t], p.bs, blk, row);
+    if (sizeof(T) == 2) row = grouped_k_row(row);
+    return (T*)p.cache + (int64_t)blk * p.block_stride + (int64_t)g * p.bs * p.dp;
+}
+// channel c of a head whose fp32 row is x and norm weight w (NULL: none), already scaled by inv: rotated
+__device__ __forceinline__ float grouped_turn(const GroupedArgs& p, const float* x, const float* w, float inv, const f32x2* turn, int c) {
+    auto at = [&](int i) { return w ? x[i] * inv * w[i] : x[i]; };
+    if (c >= p.dim) return 0.f;
+    if (c >= p.rot) return at(c);
+    const int half = p.rot >> 1;
+    const f32x2 cs = turn[c < half ? c : c - half];
+    return c < half ? at(c) * cs[0] - at(c + half) * cs[1] : at(c) * cs[0] + at(c - half) * cs[1];
+}
+// one workgroup per token, a wave per head: small batches, fp32 mode
+template <typename T>
+__global__ __launch_bounds__(1024) void grouped_qk_row_kernel(GroupedArgs p) {
+    __shared__ float sums[2][16];
+    const int64_t t = blockIdx.x;
+    const int lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), NW = blockDim.x >> 6;
+    const float* row = p.proj + t * p.proj_ld;
+    auto head_x = [&](int h) { return row + (h < p.H ? (int64_t)h * p.dp : p.qk_koff + (int64_t)(h - p.H) * p.dp); };
+    auto squares = [&](const float* x) {
+        float a = 0.f;
+        for (int c = lane * 4; c < p.dp; c += 256) { const f32x4 v = *(const f32x4*)(x + c); a += v[0] * v[0] + v[1] * v[1] + v[2] * v[2] + v[3] * v[3]; }      // (padding is zero)
+        return wave_sum(a);
+    };
+    if (p.qk_norm == 2) {
+        float sq = 0.f, sk = 0.f;
+        for (int h = wave; h < p.H + p.G; h += NW) (h < p.H ? sq : sk) += squares(head_x(h));
+        if (lane == 0) { sums[0][wave] = sq; sums[1][wave] = sk; }
+        __syncthreads();
+    }
+    const f32x2* turn = p.rot ? p.turn + (int64_t)p.tok_pos[t] * (p.rot >> 1) : nullptr;
+    for (int h = wave; h < p.H + p.G; h += NW) {
+        const bool is_q = h < p.H;
+        const float* x = head_x(h);
+        const float* w = is_q ? p.q_norm : p.k_norm;
+        float inv = 1.f;
+        if (p.qk_norm == 1) inv = 1.0f / sqrtf(squares(x) / (float)p.dim + p.eps);
+        else if (p.qk_norm == 2) {
+            float s = 0.f;
+            for (int i = 0; i < NW; i++) s += sums[!is_q][i];
+            inv = 1.0f / sqrtf(s / ((float)p.dim * (is_q ? p.H : p.G)) + p.eps);
+            w += (int64_t)(is_q ? h : h - p.H) * p.dim;
+        }
+        int krow = 0;
+        T* dst = is_q ? (T*)p.q_out : grouped_key_row<T>(p, t, h - p.H, krow);
+        for (int c = lane * 4; c < p.dp; c += 256) {
+            f32x4 v;
+#pragma unroll
+            for (int r = 0; r < 4; r++) v[r] = grouped_turn(p, x, p.qk_norm ? w : nullptr, inv, turn, c + r);
+            if (is_q) act_store4<T>(dst, t, h * p.dp + c, p.q_ld, v);
+            else act_store4<T>(dst, krow, c, p.dp, v);
+        }
+    }
+}
+// Prompts, bf16: one workgroup per 16 tokens, a wave per head.  A lane is a row of the operand blocks it writes (token l & 15, channels
+// 8 (l >> 4) ..), so a query head's stores are whole KiB; rows of keys are 16-byte pieces of the cache's blocks.
+static __global__ __launch_bounds__(1024) void grouped_qk_tile_kernel(GroupedArgs p) {
+    __shared__ float sums[2][16][16];                 // [q, k][wave][token]
+    const int lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
+    const int tok = blockIdx.x * 16 + (lane & 15), c0 = (lane >> 4) * 8;
+    const bool ok = tok < p.rows;
+    const int64_t t = ok ? tok : p.rows - 1;
+    const float* row = p.proj + t * p.proj_ld + c0;
+    auto head_x = [&](int h) { return row + (h < p.H ? (int64_t)h * p.dp : p.qk_koff + (int64_t)(h - p.H) * p.dp); };
+    auto squares = [&](const float* x) {              // of this lane's token
+        float a = 0.f;
+        for (int b = 0; b < p.dp; b += 32) {
+            const f32x4 u = *(const f32x4*)(x + b), v = *(const f32x4*)(x + b + 4);
+            a += (u[0] * u[0] + u[1] * u[1]) + (u[2] * u[2] + u[3] * u[3]) + (v[0] * v[0] + v[1] * v[1]) + (v[2] * v[2] + v[3] * v[3]);
+        }
+        a += __shfl_xor(a, 16, 64);
+        return a + __shfl_xor(a, 32, 64);
+    };
+    if (p.qk_norm == 2) {
+        float sq = 0.f, sk = 0.f;
+        for (int h = wave; h < p.H + p.G; h += 16) (h < p.H ? sq : sk) += squares(head_x(h));
+        if (lane < 16) { sums[0][wave][lane] = sq; sums[1][wave][lane] = sk; }
+        __syncthreads();
+    }
+    const f32x2* turn = p.rot ? p.turn + (int64_t)p.tok_pos[t] * (p.rot >> 1) : nullptr;
+    const bool whole8 = (p.rot >> 1) % 8 == 0 && p.dim % 8 == 0;      // a lane's eight channels turn, and pair, as one
+    for (int h = wave; h < p.H + p.G; h += 16) {
+        const bool is_q = h < p.H;
+        const float* x = head_x(h);
+        const float* w = is_q ? p.q_norm : p.k_norm;
+        float inv = 1.f;
+        if (p.qk_norm == 1) inv = 1.0f / sqrtf(squares(x) / (float)p.dim + p.eps);
+        else if (p.qk_norm == 2) {
+            float s = 0.f;
+#pragma unroll
+            for (int i = 0; i < 16; i++) s += sums[!is_q][i][lane & 15];
+            inv = 1.0f / sqrtf(s / ((float)p.dim * (is_q ? p.H : p.G)) + p.eps);
+            w += (int64_t)(is_q ? h : h - p.H) * p.dim;
+        }
+        int krow = 0;
+        bf16_t* dst = is_q ? (bf16_t*)p.q_out : grouped_key_row<bf16_t>(p, t, h - p.H, krow);
+        for (int b = 0; b < p.dp; b += 32) {
+            const int c = b + c0, half = p.rot >> 1;
+            float v[8];
+            if (whole8) {
+                auto take = [&](int i, float (&y)[8]) {       // eight normed channels
+                    const f32x4 u0 = *(const f32x4*)(x - c0 + i), u1 = *(const f32x4*)(x - c0 + i + 4);
+#pragma unroll
+                    for (int r = 0; r < 8; r++) { y[r] = r < 4 ? u0[r] : u1[r - 4]; if (p.qk_norm) y[r] *= inv * w[i + r]; }
+                };
+                if (c >= p.dim) {
+#pragma unroll
+                    for (int r = 0; r < 8; r++) v[r] = 0.f;
+                } else {
+                    take(c, v);
+                    if (c < p.rot) {
+                        float y[8];
+                        take(c < half ? c + half : c - half, y);
+                        const f32x2* cs = turn + (c < half ? c : c - half);
+#pragma unroll
+                        for (int r = 0; r < 8; r++) v[r] = c < half ? v[r] * cs[r][0] - y[r] * cs[r][1] : v[r] * cs[r][0] + y[r] * cs[r][1];
+                    }
+                }
+            } else {
+#pragma unroll
+                for (int r = 0; r < 8; r++) v[r] = grouped_turn(p, x - c0, p.qk_norm ? w : nullptr, inv, turn, c + r);
+            }
+            bf16x8 out;
+#pragma unroll
+            for (int r = 0; r < 8; r++) out[r] = (bf16_t)v[r];
+            if (!ok) continue;
+            if (is_q) *(bf16x8*)(dst + fm_index(t, (int64_t)h * p.dp + c, p.q_ld)) = out;
+            else *(bf16x8*)(dst + fm_index(krow, c, p.dp)) = out;
         }
     }
 }
@@ -114,24 +264,29 @@ __device__ __forceinline__ void grouped_scores(const GroupedScore& f, f32x4 (&s)
             for (int r = 0; r < 4; r++) s[t][r] = fmaf(f.nr1, __builtin_amdgcn_logf(fmaf(-f.r2, (float)(32 * (t >> 1) + 4 * (t & 1) + r), b)), s[t][r]);
     }
 }
-__device__ __forceinline__ void grouped_mask(f32x4 (&s)[4], int back, int window, int fg) {
-    const int from = window > 0 ? back - window + 1 : 0;
+// from, keep: the query's first key (KeyMask::lo) and the end of the kept tokens, tile-relative
+__device__ __forceinline__ void grouped_mask(f32x4 (&s)[4], int back, int from, int keep, int fg) {
 #pragma unroll
     for (int t = 0; t < 4; t++)
 #pragma unroll
         for (int r = 0; r < 4; r++) {
             const int k = 32 * (t >> 1) + 8 * fg + 4 * (t & 1) + r;
-            if (k > back || k < from) s[t][r] = -INFINITY;
+            if (k > back || (k < from && k >= keep)) s[t][r] = -INFINITY;
         }
 }
 __device__ __forceinline__ bf16x8 grouped_load_q(const GroupedArgs& p, int64_t tok, int head, int ks, int fg) {
     return *(const bf16x8*)((const bf16_t*)p.q + fm_index(tok, (int64_t)head * p.dp + ks * 32 + fg * 8, p.q_ld));
 }
+// the sink's score in the exp2 domain
+__device__ __forceinline__ float grouped_sink(const GroupedArgs& p, int head) { return p.sink ? p.sink[head] * 1.4426950408889634f : -INFINITY; }
 // four channels of a finished row: gate, store
 __device__ __forceinline__ void grouped_store(const GroupedArgs& p, int64_t tok, int head, int c, f32x4 v) {
-    const bf16x4 g = *(const bf16x4*)((const bf16_t*)p.q + fm_index(tok, p.gate_col + (int64_t)head * p.vp + c, p.q_ld));
+    if (p.gate_col >= 0) {
+        const bf16x4 g = *(const bf16x4*)((const bf16_t*)p.q + fm_index(tok, p.gate_col + (int64_t)head * p.vp + c, p.q_ld));
 #pragma unroll
-    for (int r = 0; r < 4; r++) v[r] *= lat_sigmoid((float)g[r]);
+        for (int r = 0; r < 4; r++) v[r] *= lat_sigmoid((float)g[r]);
+    }
+    v *= p.out_scale;
     act_store4<bf16_t>((bf16_t*)p.out, tok, head * p.vp + c, p.out_ld, v);
 }
 
@@ -160,28 +315,31 @@ __global__ __launch_bounds__(512, (KS <= 2 && DT <= 4) ? 4 : 2) void grouped_pre
     const int tok0 = p.seq_tok_start[seq], pos0 = p.seq_pos[seq];
     const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6);
     const int fq = lane & 15, fg = lane >> 4;
-    auto key_lo = [&](int pos) { const int lo = p.window > 0 ? pos - p.window + 1 : 0; return lo > 0 ? lo : 0; };
     // key tiles of the workgroup, and of this wave (rows w_row0 .. + 31)
     const int wg_first = pos0 + qt * 256 / p.group, wg_last = pos0 + (min(qt * 256 + 255, R - 1)) / p.group;
-    const int t0 = key_lo(wg_first) >> 6, n_kt = (wg_last >> 6) + 1;
+    const int t0 = p.mask.lo(wg_first) >> 6, n_kt = (wg_last >> 6) + 1;
+    const int keep_kt = (p.mask.keep + 63) >> 6, n_pre = min(t0, keep_kt), n_tiles = n_pre + n_kt - t0;      // (tiles of kept tokens before the window's)
+    auto tile_at = [&](int i) { return i < n_pre ? i : t0 + i - n_pre; };
     const int w_row0 = qt * 256 + wave * 32;
     const bool w_live = w_row0 < R;
     const int first = pos0 + min(w_row0, R - 1) / p.group, last = pos0 + min(w_row0 + 31, R - 1) / p.group;
-    const int wt0 = w_live ? key_lo(first) >> 6 : n_kt, wt1 = w_live ? (last >> 6) + 1 : 0;
-    const int full_lo = p.window > 0 ? last - p.window + 1 : 0, full_hi = first;
-    for (int i = tid; i < n_kt - t0; i += 512) {
-        const int key = (t0 + i) * 64, bi = key / p.bs;
+    const int wt0 = w_live ? p.mask.lo(first) >> 6 : n_kt, wt1 = w_live ? (last >> 6) + 1 : 0;
+    const int full_lo = p.mask.lo(last), full_hi = first;
+    for (int i = tid; i < n_tiles; i += 512) {
+        const int key = tile_at(i) * 64, bi = key / p.bs;
         stile[i] = make_int2(p.blk_table[(int64_t)seq * p.tbl_stride + bi], key - bi * p.bs);
     }
     auto row_of = [&](int i, bool& ok) { const int r = w_row0 + 16 * i + fq; ok = r < R; return ok ? r : R - 1; };
     bf16x8 qf[TQ][KS];
-    int qpos[TQ];
-    float r1v[TQ], r2v[TQ];
+    int qpos[TQ], qlo[TQ];
+    float r1v[TQ], r2v[TQ], m_run[TQ];
 #pragma unroll
     for (int i = 0; i < TQ; i++) {
         bool ok;
         const int row = row_of(i, ok), si = row / p.group, head = kvh * p.group + row - si * p.group;
         qpos[i] = pos0 + si;
+        qlo[i] = p.mask.lo(qpos[i]);
+        m_run[i] = p.sink ? grouped_sink(p, head) : -1e30f;
 #pragma unroll
         for (int ks = 0; ks < KS; ks++) qf[i][ks] = grouped_load_q(p, tok0 + si, head, ks, fg);
         const GroupedScore f(p, head);
@@ -192,12 +350,12 @@ __global__ __launch_bounds__(512, (KS <= 2 && DT <= 4) ? 4 : 2) void grouped_pre
     for (int i = 0; i < TQ; i++) {
 #pragma unroll
         for (int ks = 0; ks < KS; ks++) asm volatile("" : "+v"(qf[i][ks]));      // complete before the first DMA is issued (attn.h)
-        asm volatile("" : "+v"(r1v[i]), "+v"(r2v[i]));
+        asm volatile("" : "+v"(r1v[i]), "+v"(r2v[i]), "+v"(m_run[i]));
     }
     asm volatile("" : "+v"(f.nr1), "+v"(f.r2));
     // distances of visible keys: 0 .. dmax; entry x of a head's table belongs to distance dmax + PAD - x
     float* const tabs = (float*)(stile + p.table);            // (p.table: entries of stile)
-    const int dmax = (p.window > 0 ? min(p.window - 1, wg_last) : wg_last), span = grouped_tab_span(dmax + 1);
+    const int dmax = (p.mask.span() > 0 ? min(p.mask.span() - 1, wg_last) : wg_last), span = grouped_tab_span(dmax + 1);
     if (p.table)
         for (int h = 0; h < p.group; h++) {
             const float nr1 = -p.r1[kvh * p.group + h], r2 = p.r2[kvh * p.group + h], top = FAST ? p.softcap * 1.4426950408889634f : 0.f;
@@ -227,8 +385,8 @@ __global__ __launch_bounds__(512, (KS <= 2 && DT <= 4) ? 4 : 2) void grouped_pre
         }
     }
     const uint32_t smem_lds = (uint32_t)(size_t)(__attribute__((address_space(3))) char*)grp_sm;
-    auto issue = [&](int kt, int buf) {
-        const int2 tl = stile[kt - t0];
+    auto issue = [&](int it, int buf) {
+        const int2 tl = stile[it];
         const int blk = __builtin_amdgcn_readfirstlane(tl.x), row = __builtin_amdgcn_readfirstlane(tl.y);
         const bf16_t* base = (const bf16_t*)p.cache + (int64_t)blk * p.block_stride;
         const uint32_t dst = smem_lds + buf * TILE + wave * (PW * 1024);
@@ -241,27 +399,28 @@ __global__ __launch_bounds__(512, (KS <= 2 && DT <= 4) ? 4 : 2) void grouped_pre
         }
     };
     f32x4 o[TQ][DT], lacc[TQ];
-    float m_run[TQ];
+    const float l0 = p.sink ? 1.0f : 0.0f;                    // (the sink's own weight, relative to m_run)
 #pragma unroll
     for (int i = 0; i < TQ; i++) {
-        m_run[i] = -1e30f; lacc[i] = f32x4{0.f, 0.f, 0.f, 0.f};
+        lacc[i] = f32x4{l0, l0, l0, l0};
 #pragma unroll
         for (int d = 0; d < DT; d++) o[i][d] = f32x4{0.f, 0.f, 0.f, 0.f};
     }
     bf16x8 ones;
 #pragma unroll
     for (int e = 0; e < 8; e++) ones[e] = (bf16_t)1.0f;
-    issue(t0, 0);
-    if (t0 + 1 < n_kt) issue(t0 + 1, 1);
+    issue(0, 0);
+    if (1 < n_tiles) issue(1, 1);
     int buf = 0;
-    for (int kt = t0; kt < n_kt; kt++) {
-        if (kt + 1 < n_kt) wait_vm<PW>(); else wait_vm<0>();      // my pieces of tile kt have landed
+    for (int it = 0; it < n_tiles; it++) {
+        if (it + 1 < n_tiles) wait_vm<PW>(); else wait_vm<0>();      // my pieces of this tile have landed
         __builtin_amdgcn_s_barrier();
-        if (kt + 2 < n_kt) { int nb = buf + 2; if (nb >= NBUF) nb -= NBUF; issue(kt + 2, nb); }
+        if (it + 2 < n_tiles) { int nb = buf + 2; if (nb >= NBUF) nb -= NBUF; issue(it + 2, nb); }
+        const int kt = tile_at(it);
         const char* kimg = grp_sm + buf * TILE + lane * 16;
         const char* vimg = kimg + 4 * KS * 1024;
         buf = buf + 1 == NBUF ? 0 : buf + 1;
-        if (kt < wt0 || kt >= wt1) continue;                      // (wave-uniform)
+        if ((kt < wt0 && kt >= keep_kt) || kt >= wt1) continue;      // (wave-uniform)
         f32x4 s[TQ][4];
 #pragma unroll
         for (int i = 0; i < TQ; i++)
@@ -275,7 +434,7 @@ __global__ __launch_bounds__(512, (KS <= 2 && DT <= 4) ? 4 : 2) void grouped_pre
 #pragma unroll
                 for (int i = 0; i < TQ; i++) s[i][t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf, qf[i][ks], s[i][t], 0, 0, 0);
             }
-        const bool whole = kt * 64 >= full_lo && kt * 64 + 63 <= full_hi;
+        const bool whole = (kt * 64 >= full_lo || kt * 64 + 63 < p.mask.keep) && kt * 64 + 63 <= full_hi;
 #pragma unroll
         for (int i = 0; i < TQ; i++) {
             if constexpr (!FAST) { f.nr1 = r1v[i]; f.r2 = r2v[i]; }
@@ -283,7 +442,7 @@ __global__ __launch_bounds__(512, (KS <= 2 && DT <= 4) ? 4 : 2) void grouped_pre
         }
         if (!whole)
 #pragma unroll
-            for (int i = 0; i < TQ; i++) grouped_mask(s[i], qpos[i] - kt * 64, p.window, fg);
+            for (int i = 0; i < TQ; i++) grouped_mask(s[i], qpos[i] - kt * 64, qlo[i] - kt * 64, p.mask.keep - kt * 64, fg);
         if constexpr (!FAST) {
             float m_new[TQ];
             bool moved = false;
@@ -370,9 +529,9 @@ __global__ __launch_bounds__(NW * 64) void grouped_short_kernel(GroupedArgs p) {
     const bool ok = rt * 16 + fq < R;
     const int row = ok ? rt * 16 + fq : R - 1, si = row / p.group, head = kvh * p.group + row - si * p.group;
     const int first = pos0 + rt * 16 / p.group, last = pos0 + min(rt * 16 + 15, R - 1) / p.group, qpos = pos0 + si;
-    const int lo = p.window > 0 && first - p.window + 1 > 0 ? first - p.window + 1 : 0;
-    const int t0 = lo >> 6, n_kt = (last >> 6) + 1;
-    const int full_lo = p.window > 0 ? last - p.window + 1 : 0, full_hi = first;
+    const int t0 = p.mask.lo(first) >> 6, n_kt = (last >> 6) + 1, qlo = p.mask.lo(qpos);
+    const int n_pre = min(t0, (p.mask.keep + 63) >> 6), n_tiles = n_pre + n_kt - t0;      // (tiles of kept tokens before the window's)
+    const int full_lo = p.mask.lo(last), full_hi = first;
     const int64_t tok = tok0 + si;
     bf16x8 qf[KS], kf[4][KS], vf[DT][2];
 #pragma unroll
@@ -383,7 +542,8 @@ __global__ __launch_bounds__(NW * 64) void grouped_short_kernel(GroupedArgs p) {
     for (int d = 0; d < DT; d++) o[d] = f32x4{0.f, 0.f, 0.f, 0.f};
     float m = -1e30f, l = 0.f;
     const int64_t v_ld = p.bs >> 5;
-    for (int kt = t0 + blockIdx.z * NW + wave; kt < n_kt; kt += NW * gridDim.z) {
+    for (int it = blockIdx.z * NW + wave; it < n_tiles; it += NW * gridDim.z) {
+        const int kt = it < n_pre ? it : t0 + it - n_pre;
         const int bi = kt * 64 / p.bs, r0 = kt * 64 - bi * p.bs;
         const bf16_t* base = (const bf16_t*)p.cache + (int64_t)__builtin_amdgcn_readfirstlane(tbl[bi]) * p.block_stride + lane * 8;
         const bf16_t* kp = base + ((int64_t)kvh * p.bs + r0) * p.dp;
@@ -405,7 +565,7 @@ __global__ __launch_bounds__(NW * 64) void grouped_short_kernel(GroupedArgs p) {
         }
         const int back = qpos - kt * 64;
         grouped_scores(f, s, back, fg);
-        if (!(kt * 64 >= full_lo && kt * 64 + 63 <= full_hi)) grouped_mask(s, back, p.window, fg);
+        if (!((kt * 64 >= full_lo || kt * 64 + 63 < p.mask.keep) && kt * 64 + 63 <= full_hi)) grouped_mask(s, back, qlo - kt * 64, p.mask.keep - kt * 64, fg);
         float mx = -INFINITY;
 #pragma unroll
         for (int t = 0; t < 4; t++)
@@ -439,6 +599,8 @@ __global__ __launch_bounds__(NW * 64) void grouped_short_kernel(GroupedArgs p) {
 #pragma unroll
     for (int w = 0; w < NW; w++) { sc[w] = __builtin_amdgcn_exp2f(red_m[w][fq] - ms); L += red_l[w][fq] * sc[w]; }      // (a wave without a tile: l = 0, O = 0)
     const int nz = gridDim.z, pair = seq * gridDim.x + blockIdx.x;
+    const float sink = grouped_sink(p, head);
+    if (nz == 1 && p.sink) L += __builtin_amdgcn_exp2f(sink - ms);       // (a sink far above every score: inf, and the row is zero)
     float* rec = p.part + ((int64_t)pair * nz + blockIdx.z) * grouped_part_floats<DT>();
     for (int d = wave; d < DT; d += NW) {
         f32x4 a = f32x4{0.f, 0.f, 0.f, 0.f};
@@ -460,7 +622,7 @@ __global__ __launch_bounds__(NW * 64) void grouped_short_kernel(GroupedArgs p) {
     if (tid == 0) __hip_atomic_store(p.part_cnt + pair, 0, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);      // for the next launch
     if (!ok) return;
     const float* rec0 = p.part + (int64_t)pair * nz * grouped_part_floats<DT>();
-    float M = -1e30f, LL = 0.f, mz[GROUPED_SPLITS];
+    float M = p.sink ? sink : -1e30f, LL = p.sink ? 1.0f : 0.f, mz[GROUPED_SPLITS];
 #pragma unroll
     for (int z = 0; z < GROUPED_SPLITS; z++)
         if (z < nz) {
@@ -488,21 +650,23 @@ __global__ __launch_bounds__(256) void grouped_plain_kernel(GroupedArgs p) {
     if (r >= p.seq_len[seq]) return;
     constexpr bool FM = sizeof(T) == 2;
     const int64_t t = p.seq_tok_start[seq] + r;
-    const int pos = p.seq_pos[seq] + r, lo = p.window > 0 && pos - p.window + 1 > 0 ? pos - p.window + 1 : 0;
+    const int pos = p.seq_pos[seq] + r, lo = p.mask.lo(pos), n_pre = min(lo, p.mask.keep), n_keys = n_pre + pos - lo + 1;
+    auto key_at = [&](int i) { return i < n_pre ? i : lo + i - n_pre; };
     const int32_t* tbl = p.blk_table + (int64_t)seq * p.tbl_stride;
     float *sq = grp_f, *so = grp_f + p.dp;
     for (int i = tid; i < p.dp; i += 256) sq[i] = (float)((const T*)p.q)[act_index<T>(t, h * p.dp + i, p.q_ld)];
     for (int i = tid; i < p.vp; i += 256) so[i] = 0.f;
     const float r1 = p.r1 ? p.r1[h] : 0.f, r2 = p.r1 ? p.r2[h] : 0.f;
-    float m = -1e30f, l = 0.f;
+    float m = p.sink ? p.sink[h] : -1e30f, l = p.sink ? 1.f : 0.f;
     __syncthreads();
     auto bmax = [&](float v) { v = wave_max(v); if ((tid & 63) == 0) red[tid >> 6] = v; __syncthreads(); v = fmaxf(fmaxf(red[0], red[1]), fmaxf(red[2], red[3])); __syncthreads(); return v; };
     auto bsum = [&](float v) { v = wave_sum(v); if ((tid & 63) == 0) red[tid >> 6] = v; __syncthreads(); v = red[0] + red[1] + red[2] + red[3]; __syncthreads(); return v; };
     auto part = [&](int key, int& row) { const int bi = key / p.bs; row = key - bi * p.bs; return (const T*)p.cache + (int64_t)tbl[bi] * p.block_stride; };
-    for (int base = lo; base <= pos; base += 256) {
-        const int key = base + tid;
+    for (int base = 0; base < n_keys; base += 256) {
+        const bool live = base + tid < n_keys;
+        const int key = key_at(base + tid);
         float s = -INFINITY;
-        if (key <= pos) {
+        if (live) {
             int row;
             const T* k = part(key, row) + (int64_t)kvh * p.bs * p.dp;
             if (FM) row = grouped_k_row(row);
@@ -513,17 +677,17 @@ __global__ __launch_bounds__(256) void grouped_plain_kernel(GroupedArgs p) {
             if (p.r1) s -= r1 * log1pf(r2 * (float)(pos - key));
         }
         const float mn = fmaxf(m, bmax(s)), alpha = expf(m - mn);
-        const float e = key <= pos ? expf(s - mn) : 0.f;
+        const float e = live ? expf(s - mn) : 0.f;
         m = mn;
         l = l * alpha + bsum(e);
         sp[tid] = e;
         __syncthreads();
-        const int nk = min(256, pos - base + 1);
+        const int nk = min(256, n_keys - base);
         for (int i = tid; i < p.vp; i += 256) {
             float a = so[i] * alpha;
             for (int j = 0; j < nk; j++) {
                 int row;
-                const T* v = part(base + j, row) + (int64_t)p.G * p.bs * p.dp + (int64_t)kvh * p.bs * p.vp;
+                const T* v = part(key_at(base + j), row) + (int64_t)p.G * p.bs * p.dp + (int64_t)kvh * p.bs * p.vp;
                 a = fmaf(sp[j], (float)(FM ? v[fm_index(i, row, p.bs)] : v[(int64_t)row * p.vp + i]), a);
             }
             so[i] = a;
@@ -531,7 +695,8 @@ __global__ __launch_bounds__(256) void grouped_plain_kernel(GroupedArgs p) {
         __syncthreads();
     }
     for (int i = tid; i < p.vp; i += 256) {
-        const float o = so[i] / l * (1.0f / (1.0f + expf(-(float)((const T*)p.q)[act_index<T>(t, p.gate_col + h * p.vp + i, p.q_ld)])));
+        float o = so[i] / l * p.out_scale;
+        if (p.gate_col >= 0) o *= 1.0f / (1.0f + expf(-(float)((const T*)p.q)[act_index<T>(t, p.gate_col + h * p.vp + i, p.q_ld)]));
         ActIO<T>::st((T*)p.out + act_index<T>(t, h * p.vp + i, p.out_ld), o);
     }
 }

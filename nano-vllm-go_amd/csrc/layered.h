@@ -1,6 +1,7 @@
 // layered.h — models described by a list of layers (nvl_layer_config): every layer names a mixer (latent attention, Mamba-2, gated
-// linear attention, channel-wise delta rule, grouped-query attention), its sizes and its feed-forward, with a norm before and after each
-// sublayer (NVL_BLOCK_SANDWICH), after it only (NVL_BLOCK_POST: the sublayers read the residual stream itself), or one norm that both
+// linear attention, channel-wise delta rule, grouped-query attention, the last also with lightning attention beside it), its sizes and its
+// feed-forward, with a norm before and after each sublayer (NVL_BLOCK_SANDWICH), after it only (NVL_BLOCK_POST: the sublayers read the
+// residual stream itself), of the scaled stream and the sublayer's result together (NVL_BLOCK_SUM_NORM: likewise), or one norm that both
 // sublayers read (NVL_BLOCK_PARALLEL).  Host side: creation, tensor staging, freezing into the kernels' layouts, the layer stack of one
 // forward pass.  Included by nvllm.hip.
 //
@@ -8,6 +9,9 @@
 // and W_down side by side in one matrix.  The feed-forward is dense, or a mixture of experts whose shared expert takes the dense one's
 // place; the experts' sum joins in the launch that completes the residual.  A per-layer token input (side_dim) follows:
 // x += rms(P (gelu(G x) * e_token)) * w.
+//
+// Two mixers side by side (mixer2) share ONE projection in and ONE out: their operands sit side by side in m->lmix, W_o and W_o2 side by
+// side in one matrix, and the factors of their results are applied, in fp32, as the operands are written.
 //
 // What differs from the fixed-shape models around it:
 //   * widths need not be multiples of 64: rows, heads and latents are padded with zeros when the tensors are frozen (m->H is the
@@ -23,14 +27,15 @@ static int g_grouped_split = 0;      // nvl_set_tuning key 37: key splits of the
 
 namespace {
 
-constexpr float CLAMPED_GLU_SLOPE = 1.702f;
 constexpr int LAT_ABSORB_MAX = 16, LAT_ABSORB_MAX_RP = 512, REC_STEP_MAX = 4;
 constexpr int GLU_IN_MAX = 1024;       // widest shared expert whose gate and up columns pass through fp32 rows instead of a launch of their own
+constexpr int QK_ROW_MAX = 256;        // batches whose queries and keys are normed and rotated by a workgroup per token
+constexpr int SHARED_PARTS_MAX = 16;   // widest shared expert, in experts, that joins the masked experts of a decode step
 constexpr int GROUPED_SHORT_ROWS = 64, GROUPED_SPLIT_WGS = 512;      // GROUPED_SPLIT_WGS: workgroups of a launch whose keys are split
 
 bool same_rotation(const nvl_layer_config& a, const nvl_layer_config& b) {
     return a.rot_dim == b.rot_dim && a.rot_base == b.rot_base && a.rot_factor == b.rot_factor && a.rot_original == b.rot_original &&
-           a.rot_fast == b.rot_fast && a.rot_slow == b.rot_slow;
+           a.rot_fast == b.rot_fast && a.rot_slow == b.rot_slow && a.rot_low == b.rot_low && a.rot_high == b.rot_high;
 }
 // unrotated (padded to 32) + rotated part; d + rot = 192 with 256 value channels has no LDS left for its ring of tiles
 int pad_rotated(int d, int vp) {
@@ -47,12 +52,14 @@ int pad_head(int d, int unit) {       // head sizes the attention instances exis
 // ------------------------------------------------------------------------------------------
 int layered_create(const nvl_model_config& c, const nvl_layer_config* layers, const nvl_runtime_opts& opts, nvl_model** out) {
     auto bad = [&](const std::string& why) { return fail(nullptr, NVL_ERR_INVALID, "nvl_create_layers: " + why); };
-    const bool par = c.block_style == NVL_BLOCK_PARALLEL;
-    if (c.block_style != NVL_BLOCK_SANDWICH && c.block_style != NVL_BLOCK_POST && !par) return bad("block_style NVL_BLOCK_SANDWICH, NVL_BLOCK_POST or NVL_BLOCK_PARALLEL expected");
-    auto act_ok = [&](int a) { return par ? a == NVL_ACT_RELU2 || a == NVL_ACT_SWIGLU : a == NVL_ACT_GEGLU || a == NVL_ACT_CLAMPED_GLU; };
-    if (!act_ok(c.activation_type)) return bad("activation_type does not fit the block style (NVL_ACT_GEGLU, NVL_ACT_CLAMPED_GLU; parallel: NVL_ACT_RELU2, NVL_ACT_SWIGLU)");
-    if (!par && (c.norm_type != NVL_NORM_RMS || c.position_type != NVL_POS_NONE || c.side_dim)) return bad("layer norms, learned positions and side_dim need NVL_BLOCK_PARALLEL");
-    if ((c.norm_type != NVL_NORM_RMS && c.norm_type != NVL_NORM_LAYER) || (c.position_type != NVL_POS_NONE && c.position_type != NVL_POS_LEARNED)) return bad("bad norm_type / position_type");
+    const bool par = c.block_style == NVL_BLOCK_PARALLEL, sum = c.block_style == NVL_BLOCK_SUM_NORM;
+    if (c.block_style != NVL_BLOCK_SANDWICH && c.block_style != NVL_BLOCK_POST && !par && !sum) return bad("block_style NVL_BLOCK_SANDWICH, _POST, _PARALLEL or _SUM_NORM expected");
+    auto act_ok = [&](int a) { return par ? a == NVL_ACT_RELU2 || a == NVL_ACT_SWIGLU : a == (sum ? NVL_ACT_REGLU : NVL_ACT_GEGLU) || a == NVL_ACT_CLAMPED_GLU; };
+    if (!act_ok(c.activation_type)) return bad("activation_type does not fit the block style (NVL_ACT_GEGLU, NVL_ACT_CLAMPED_GLU; parallel: NVL_ACT_RELU2, NVL_ACT_SWIGLU; norms of sums: NVL_ACT_REGLU, NVL_ACT_CLAMPED_GLU)");
+    if (sum && !(c.stream_scale != 0.f)) return bad("stream_scale is zero");
+    if (c.token_shift && !sum && c.block_style != NVL_BLOCK_POST) return bad("token_shift needs mixers that read the residual stream itself");
+    if (!par && ((c.norm_type != NVL_NORM_RMS && c.norm_type != NVL_NORM_RMS_SCALAR) || c.position_type != NVL_POS_NONE || c.side_dim)) return bad("layer norms, learned positions and side_dim need NVL_BLOCK_PARALLEL");
+    if ((c.norm_type != NVL_NORM_RMS && c.norm_type != NVL_NORM_RMS_SCALAR && c.norm_type != NVL_NORM_LAYER) || (c.position_type != NVL_POS_NONE && c.position_type != NVL_POS_LEARNED)) return bad("bad norm_type / position_type");
     if (c.norm_type == NVL_NORM_LAYER && c.norm_weight_offset != 0.f) return bad("layer norms take their weights as they are");
     if (c.side_dim < 0 || c.side_dim > 8192) return bad("bad side_dim");
     if (!(c.logit_softcap >= 0.f)) return bad("logit_softcap is negative");
@@ -66,17 +73,21 @@ int layered_create(const nvl_model_config& c, const nvl_layer_config* layers, co
         const nvl_layer_config& l = layers[i];
         const std::string at = "layer " + std::to_string(i) + ": ";
         if (l.heads <= 0 || l.vdim <= 0 || l.vdim > 2048 || l.ffn_dim < 0) return bad(at + "bad heads / vdim / ffn_dim");
-        if (l.ffn_dim && c.activation_type == NVL_ACT_CLAMPED_GLU && !(l.ffn_limit > 0.f)) return bad(at + "ffn_limit is not positive");
+        if (l.ffn_dim && (l.ffn_act ? l.ffn_act : c.activation_type) == NVL_ACT_CLAMPED_GLU && !(l.ffn_limit > 0.f)) return bad(at + "ffn_limit is not positive");
         if (l.ffn_act && !act_ok(l.ffn_act)) return bad(at + "ffn_act does not fit the block style");
         if (l.experts) {
-            if (!par) return bad(at + "experts need NVL_BLOCK_PARALLEL");
+            if (!par && !sum) return bad(at + "experts need NVL_BLOCK_PARALLEL or NVL_BLOCK_SUM_NORM");
+            if (!(l.expert_limit >= 0.f)) return bad(at + "expert_limit is negative");
+            if (l.route_softmax && l.expert_groups != 1) return bad(at + "softmax routing has no expert groups");
+            if (par && (l.route_softmax || l.expert_limit > 0.f)) return bad(at + "softmax routing and clamped experts need NVL_BLOCK_SUM_NORM");
             if (l.experts < 0 || l.experts > std::min(MOE_MAX_E, ROUTE_MAX_E) || l.expert_dim <= 0 || l.expert_groups <= 0 || l.experts % l.expert_groups || l.groups_kept <= 0 ||
                 l.groups_kept > l.expert_groups || l.top_k <= 0 || l.top_k > l.groups_kept * (l.experts / l.expert_groups)) return bad(at + "bad expert sizes");
         }
+        if (l.mixer != NVL_MIXER_ATTENTION && (l.chunk || l.keep_first || l.qk_norm || l.sink || l.qkv_bias || l.ungated || l.mixer2)) return bad(at + "chunks, kept tokens, query/key norms, sinks, biases and a second mixer belong to NVL_MIXER_ATTENTION");
+        if (l.rot_dim < 0 || l.rot_dim % 2 || l.rot_dim > 1024 || (l.rot_dim && !(l.rot_base > 1.0)) || (l.rot_factor != 0.0 && !(l.rot_factor > 0.0 && l.rot_original > 0.0)) ||
+            (l.rot_high != 0.0 ? !(l.rot_factor > 0.0 && l.rot_low > 0.0 && l.rot_high > l.rot_low) : l.rot_factor != 0.0 && !(l.rot_fast > 0.0 && l.rot_slow > 0.0))) return bad(at + "bad rotation");
         switch (l.mixer) {
             case NVL_MIXER_LATENT_ATTENTION:
-                if (l.rot_dim < 0 || l.rot_dim % 2 || l.rot_dim > 1024 || (l.rot_dim && !(l.rot_base > 1.0)) ||
-                    (l.rot_factor != 0.0 && !(l.rot_factor > 0.0 && l.rot_original > 0.0 && l.rot_fast > 0.0 && l.rot_slow > 0.0))) return bad(at + "bad rotation");
                 if (l.kv_from >= 0) {
                     if (l.kv_from >= i) return bad(at + "kv_from names no earlier layer");
                     const nvl_layer_config& s = layers[l.kv_from];
@@ -97,6 +108,14 @@ int layered_create(const nvl_model_config& c, const nvl_layer_config* layers, co
                 break;
             case NVL_MIXER_ATTENTION: {
                 if (l.dim <= 0 || l.dim > 2048 || l.kv_heads <= 0 || l.heads % l.kv_heads || l.window < 0 || !(l.softcap >= 0.f)) return bad(at + "bad attention sizes");
+                if (l.chunk < 0 || l.keep_first < 0 || (l.chunk && l.window) || (l.keep_first && !l.window) || l.rot_dim > l.dim || l.qk_norm < 0 || l.qk_norm > NVL_QK_NORM_ROW || l.sink < 0 || l.sink > NVL_SINK_LEARNED)
+                    return bad(at + "bad key mask, rotation, query/key norm or sink");
+                if (!l.ungated && (l.qk_norm || l.rot_dim || l.mixer2 || l.qkv_bias)) return bad(at + "normed, rotated or biased attention, and attention beside a second mixer, has no output gate");
+                if (l.mixer2) {
+                    if (l.mixer2 != NVL_MIXER_LIGHTNING || par) return bad(at + "the second mixer is not NVL_MIXER_LIGHTNING (or in a parallel block)");
+                    if (l.heads2 <= 0 || l.heads2 > NVL_MAX_DECAYS || l.dim2 <= 0 || l.dim2 > 2048 || l.vdim2 <= 0 || l.vdim2 > 2048) return bad(at + "bad lightning attention sizes");
+                    for (int h = 0; h < l.heads2; h++) if (!(l.decay[h] >= 0.0 && l.decay[h] <= 1.0)) return bad(at + "a decay is not between 0 and 1");
+                }
                 for (int j = 0; j < i && l.v_mix; j++)
                     if (layers[j].mixer == l.mixer && layers[j].v_mix && (layers[j].kv_heads != l.kv_heads || layers[j].vdim != l.vdim)) return bad(at + "mixes values of another shape");
                 break;
@@ -113,7 +132,8 @@ int layered_create(const nvl_model_config& c, const nvl_layer_config* layers, co
         const nvl_layer_config &a = layers[i], &b = layers[o];
         if (a.mixer != b.mixer || a.heads != b.heads || a.dim != b.dim || a.vdim != b.vdim || a.q_rank != b.q_rank || a.kv_rank != b.kv_rank ||
             a.state != b.state || a.groups != b.groups || a.conv_taps != b.conv_taps || a.ffn_dim != b.ffn_dim || a.rot_dim != b.rot_dim ||
-            a.kv_heads != b.kv_heads || a.gate_per_head != b.gate_per_head || a.experts != b.experts || a.expert_dim != b.expert_dim || a.v_mix != b.v_mix || a.ffn_act != b.ffn_act || (i != o && a.mixer == NVL_MIXER_LATENT_ATTENTION && (a.kv_from >= 0) != (b.kv_from >= 0)))
+            a.kv_heads != b.kv_heads || a.qk_norm != b.qk_norm || a.sink != b.sink || a.qkv_bias != b.qkv_bias || a.ungated != b.ungated || a.out_scale2 != b.out_scale2 ||
+            a.mixer2 != b.mixer2 || a.heads2 != b.heads2 || a.dim2 != b.dim2 || a.vdim2 != b.vdim2 || memcmp(a.decay, b.decay, sizeof a.decay) || a.gate_per_head != b.gate_per_head || a.experts != b.experts || a.expert_dim != b.expert_dim || a.v_mix != b.v_mix || a.ffn_act != b.ffn_act || (i != o && a.mixer == NVL_MIXER_LATENT_ATTENTION && (a.kv_from >= 0) != (b.kv_from >= 0)))
             return bad("layer " + std::to_string(i) + " does not have the shape of the layer whose tensors it uses");
     }
     if (opts.device < 0 || nvl_device_count() <= opts.device) return fail(nullptr, NVL_ERR_NO_DEVICE, "nvl_create_layers: no HIP device (this library has no CPU fallback)");
@@ -141,14 +161,18 @@ int layered_create(const nvl_model_config& c, const nvl_layer_config* layers, co
             r.c = layers[i]; r.owner = owner[(size_t)i];
             r.Fp = (int)round_up(r.c.ffn_dim, 64);
             r.act = r.c.ffn_act ? r.c.ffn_act : c.activation_type;
+            if (c.token_shift) { r.shift_off = state; state += m->H; }
             if (r.c.experts) {      // padded so that a wave of the decode down projection owns one expert, at most 16 of them a workgroup
-                r.Ep = (int)round_up(r.c.experts, r.c.experts <= 32 ? 2 : 16); r.moe_slices = r.Ep <= 32 ? 2 : r.Ep / 16;
                 r.Ip = (int)round_up(r.c.expert_dim, 64);
+                if (sum && r.c.ffn_dim && r.act == NVL_ACT_CLAMPED_GLU && r.c.expert_limit > 0.f && cdiv(r.Fp, r.Ip) <= SHARED_PARTS_MAX) r.shared_parts = cdiv(r.Fp, r.Ip);
+                const int all = r.c.experts + r.shared_parts;
+                r.Ep = (int)round_up(all, all <= 32 ? 2 : 16); r.moe_slices = r.Ep <= 32 ? 2 : r.Ep / 16;
             }
             if (r.c.mixer == NVL_MIXER_LATENT_ATTENTION || r.c.mixer == NVL_MIXER_ATTENTION) {
+                const KeyMask mask{r.c.window, r.c.chunk, r.c.keep_first};
                 size_t w = 0;
-                while (w < m->windows.size() && m->windows[w] != r.c.window) w++;
-                if (w == m->windows.size()) m->windows.push_back(r.c.window);
+                while (w < m->masks.size() && !(m->masks[w] == mask)) w++;
+                if (w == m->masks.size()) m->masks.push_back(mask);
                 r.win = (int)w;
             }
             const int H = r.c.heads;
@@ -167,11 +191,19 @@ int layered_create(const nvl_model_config& c, const nvl_layer_config* layers, co
             } else if (r.c.mixer == NVL_MIXER_ATTENTION) {
                 const int G = r.c.kv_heads;
                 r.dp = pad_head(r.c.dim, 64); r.vp = pad_head(r.c.vdim, 64);
-                r.k_off = H * r.dp; r.v_off = r.k_off + G * r.dp; r.gate_off = r.v_off + G * r.vp; r.ffn_off = r.gate_off + H * r.vp;
+                r.k_off = H * r.dp; r.v_off = r.k_off + G * r.dp; r.gate_off = r.v_off + G * r.vp; r.ffn_off = r.gate_off + (r.c.ungated ? 0 : H * r.vp);
+                r.raw = r.c.qk_norm || r.c.rot_dim || r.c.mixer2;
                 r.ffn_in = par && r.c.ffn_dim && r.act == NVL_ACT_RELU2;
                 r.glu_in = par && r.c.experts && r.c.ffn_dim && r.act == NVL_ACT_SWIGLU && r.Fp <= GLU_IN_MAX;
                 r.route_off = r.ffn_off + (r.ffn_in ? r.Fp : r.glu_in ? 2 * r.Fp : 0);
-                r.n_in = r.route_off + r.c.experts; r.ko = (int)round_up((int64_t)H * r.vp, 64);
+                r.n_in = r.route_off + (par ? r.c.experts : 0); r.ko = (int)round_up((int64_t)H * r.vp, 64);
+                if (r.c.mixer2) {
+                    const int qk = (int)round_up(r.c.heads2 * r.c.dim2, 4), v = (int)round_up(r.c.heads2 * r.c.vdim2, 4);
+                    r.lq_off = r.ffn_off; r.lk_off = r.lq_off + qk; r.lv_off = r.lk_off + qk; r.lg_off = r.lv_off + v;
+                    r.n_in = r.lg_off + r.c.heads2 * r.c.vdim2;
+                    r.ko2 = (int)round_up((int64_t)r.c.heads2 * r.c.vdim2, 64);
+                    r.state_off = state; state += round_up((int64_t)r.c.heads2 * r.c.dim2 * round_up(r.c.vdim2, 4), 64);
+                }
                 r.cache_off = cache; cache += (int64_t)bs * G * (r.dp + r.vp);
                 if (r.c.v_mix) {
                     r.mix = m->lvf_ld ? 2 : 1;
@@ -190,7 +222,7 @@ int layered_create(const nvl_model_config& c, const nvl_layer_config* layers, co
                     r.ring_off = state; state += round_up((int64_t)r.c.conv_taps * r.conv_dim, 64);
                 }       // (GLA, channel delta: n_in follows from the decay rank, layered_finalize)
             }
-            r.kd = r.ko + (par ? r.Fp : 0);
+            r.kd = r.ko + r.ko2 + (par ? r.Fp : 0);
         }
         m->lat_block_stride = cache; m->rec_slot_stride = state;
         m->pool = 1; m->Tmax = bs; m->blocks_per_seq = cdiv(c.max_seq_len, bs);
@@ -199,7 +231,7 @@ int layered_create(const nvl_model_config& c, const nvl_layer_config* layers, co
             int64_t span = c.max_seq_len;
             int w = 0;
             bool windowed = true;
-            for (int x : m->windows) { w = std::max(w, x); windowed &= x > 0; }
+            for (const KeyMask& x : m->masks) { w = std::max(w, x.span() + (int)round_up(x.keep, bs)); windowed &= x.span() > 0; }
             if (windowed) span = std::min<int64_t>(span, (int64_t)w + m->opts.max_batch_tokens + 2 * bs);
             m->num_blocks = opts.max_seqs * cdiv(span, bs);
         }
@@ -221,11 +253,11 @@ int layered_create(const nvl_model_config& c, const nvl_layer_config* layers, co
 // tensors: staged on the device in the checkpoint's dtype, placed into the kernels' layouts by layered_finalize
 // ------------------------------------------------------------------------------------------
 void layered_shape(const nvl_model* m, int kind, int layer, int64_t& N, int64_t& K) {     // N = 0: the model has no such tensor; K = 1: a vector
-    const int64_t W = m->Hn;
+    const int64_t W = m->Hn, W1 = m->cfg.norm_type == NVL_NORM_RMS_SCALAR ? 1 : W;
     N = 0; K = 1;
     switch (kind) {
         case NVL_T_TOK_EMB: case NVL_T_LM_HEAD: N = m->V; K = W; return;
-        case NVL_T_FINAL_NORM_W: N = W; return;
+        case NVL_T_FINAL_NORM_W: N = W1; return;
         case NVL_T_FINAL_NORM_B: if (m->cfg.norm_type == NVL_NORM_LAYER) N = W; return;
         case NVL_T_POS_EMB: if (m->cfg.position_type == NVL_POS_LEARNED) { N = -1; K = W; } return;
         case NVL_T_SIDE_EMB: if (m->cfg.side_dim) { N = m->V; K = (int64_t)m->L * m->cfg.side_dim; } return;
@@ -234,14 +266,15 @@ void layered_shape(const nvl_model* m, int kind, int layer, int64_t& N, int64_t&
     const LayerRun& r = m->runs[(size_t)layer];
     const nvl_layer_config& c = r.c;
     if (r.owner != layer) return;
-    const bool post = m->cfg.block_style == NVL_BLOCK_POST, par = m->cfg.block_style == NVL_BLOCK_PARALLEL, delta = c.mixer == NVL_MIXER_CHANNEL_DELTA;
+    const bool sum = m->cfg.block_style == NVL_BLOCK_SUM_NORM, post = m->cfg.block_style == NVL_BLOCK_POST, par = m->cfg.block_style == NVL_BLOCK_PARALLEL, delta = c.mixer == NVL_MIXER_CHANNEL_DELTA;
     const bool att = c.mixer == NVL_MIXER_ATTENTION, lat = c.mixer == NVL_MIXER_LATENT_ATTENTION, mam = c.mixer == NVL_MIXER_MAMBA2, gla = c.mixer == NVL_MIXER_GLA;
     const int64_t hv = (int64_t)c.heads * c.vdim, hd = (int64_t)c.heads * c.dim;
     switch (kind) {
-        case NVL_T_ATTN_NORM_W: if (!post) N = W; return;
-        case NVL_T_FFN_NORM_W: if (!post && !par) N = W; return;
+        case NVL_T_ATTN_NORM_W: if (!post && !sum) N = W1; return;
+        case NVL_T_FFN_NORM_W: if (!post && !par && !sum) N = W1; return;
         case NVL_T_ATTN_NORM_B: if (m->cfg.norm_type == NVL_NORM_LAYER) N = W; return;
-        case NVL_T_MIX_POST_NORM: case NVL_T_FFN_POST_NORM: if (!par) N = W; return;
+        case NVL_T_MIX_POST_NORM: case NVL_T_FFN_POST_NORM: if (!par) N = W1; return;
+        case NVL_T_SHIFT: if (m->cfg.token_shift) N = W; return;
         case NVL_T_SIDE_GATE: if (m->cfg.side_dim) { N = m->cfg.side_dim; K = W; } return;
         case NVL_T_SIDE_PROJ: if (m->cfg.side_dim) { N = W; K = m->cfg.side_dim; } return;
         case NVL_T_SIDE_NORM: if (m->cfg.side_dim) N = W; return;
@@ -255,7 +288,17 @@ void layered_shape(const nvl_model* m, int kind, int layer, int64_t& N, int64_t&
         case NVL_T_W1: N = (r.act == NVL_ACT_RELU2 ? 1 : 2) * (int64_t)c.ffn_dim; K = W; return;
         case NVL_T_W2: if (c.ffn_dim) { N = W; K = c.ffn_dim; } return;
         case NVL_T_WO: if (!mam) { N = W; K = hv; } return;
-        case NVL_T_MIX_GATE: if (lat || gla || att) { N = c.gate_per_head && lat ? c.heads : hv; K = W; } return;
+        case NVL_T_BQ: if (att && c.qkv_bias) N = hd; return;
+        case NVL_T_BK: if (att && c.qkv_bias) N = (int64_t)c.kv_heads * c.dim; return;
+        case NVL_T_BV: if (att && c.qkv_bias) N = (int64_t)c.kv_heads * c.vdim; return;
+        case NVL_T_Q_NORM: if (c.qk_norm) N = c.qk_norm == NVL_QK_NORM_HEAD ? c.dim : hd; return;
+        case NVL_T_K_NORM: if (c.qk_norm) N = c.qk_norm == NVL_QK_NORM_HEAD ? c.dim : (int64_t)c.kv_heads * c.dim; return;
+        case NVL_T_SINK: if (c.sink == NVL_SINK_LEARNED) N = c.heads; return;
+        case NVL_T_LIN_Q: case NVL_T_LIN_K: if (c.mixer2) { N = (int64_t)c.heads2 * c.dim2; K = W; } return;
+        case NVL_T_LIN_V: case NVL_T_LIN_GATE: if (c.mixer2) { N = (int64_t)c.heads2 * c.vdim2; K = W; } return;
+        case NVL_T_LIN_NORM: if (c.mixer2) N = (int64_t)c.heads2 * c.vdim2; return;
+        case NVL_T_LIN_O: if (c.mixer2) { N = W; K = (int64_t)c.heads2 * c.vdim2; } return;
+        case NVL_T_MIX_GATE: if (lat || gla || (att && !c.ungated)) { N = c.gate_per_head && lat ? c.heads : hv; K = W; } return;
         case NVL_T_LAT_DQ: if (lat) { N = c.q_rank; K = W; } return;
         case NVL_T_LAT_DQ_NORM: if (lat) N = c.q_rank; return;
         case NVL_T_LAT_UQ: if (lat) { N = hd + (int64_t)c.heads * c.rot_dim; K = c.q_rank; } return;
@@ -288,7 +331,7 @@ bool layered_1d(int kind) {
     if (is_1d(kind)) return true;
     return kind == NVL_T_MIX_POST_NORM || kind == NVL_T_FFN_POST_NORM || kind == NVL_T_LAT_DQ_NORM || kind == NVL_T_LAT_DKV_NORM ||
            kind == NVL_T_BIAS_R1 || kind == NVL_T_BIAS_R2 || kind == NVL_T_V_MIX || kind == NVL_T_ROUTER_BIAS || kind == NVL_T_SIDE_NORM ||
-           kind == NVL_T_GLA_NORM || kind == NVL_T_GLA_A2_B || kind == NVL_T_MIX_SCALE || kind == NVL_T_FFN_SCALE || kind == NVL_T_DELTA_CONV;
+           kind == NVL_T_Q_NORM || kind == NVL_T_K_NORM || kind == NVL_T_SINK || kind == NVL_T_SHIFT || kind == NVL_T_LIN_NORM || kind == NVL_T_GLA_NORM || kind == NVL_T_GLA_A2_B || kind == NVL_T_MIX_SCALE || kind == NVL_T_FFN_SCALE || kind == NVL_T_DELTA_CONV;
 }
 int layered_upload(nvl_model* m, int kind, int layer, const void* data, int dtype, int64_t rows, int64_t cols, int layout) {
     int64_t N, K;
@@ -340,11 +383,22 @@ __global__ void norm_weight_kernel(float* w, const void* scale, int scale_dtype,
     const int64_t i = (int64_t)blockIdx.x * 256 + threadIdx.x;
     if (i < n) w[i] = (w[i] + offset) * (scale ? ld_as_f32(scale, scale_dtype, i) : 1.0f);
 }
+// w[i] *= f; with `spread`, every w[i] <- w[0] * f
+__global__ void scale_weight_kernel(float* w, float f, int64_t n, bool spread) {
+    const float first = w[0];
+    __syncthreads();
+    for (int64_t i = threadIdx.x; i < n; i += blockDim.x) w[i] = (spread ? first : w[i]) * f;
+}
+void lay_scale(nvl_model* m, float* w, float f, int64_t n, bool spread = false) {
+    hipLaunchKernelGGL(scale_weight_kernel, dim3(1), dim3(1024), 0, m->stream, w, f, n, spread);
+    NVL_HIP(hipGetLastError());
+}
 float* lay_norm(nvl_model* m, const DevTensor& t, int64_t padded, const DevTensor* scale = nullptr) {
     float* p = lay_vector(m, t, padded);
-    const bool sc = scale && scale->present();
+    const bool sc = scale && scale->present(), one = m->cfg.norm_type == NVL_NORM_RMS_SCALAR;
+    if (one) lay_scale(m, p, 1.0f, m->Hn, true);          // one weight for all coordinates
     if (m->cfg.norm_weight_offset != 0.f || sc) {
-        const int64_t n = t.rows * t.cols;
+        const int64_t n = one ? m->Hn : t.rows * t.cols;
         hipLaunchKernelGGL(norm_weight_kernel, dim3(cdiv(n, 256)), dim3(256), 0, m->stream, p, sc ? (const void*)scale->p : nullptr, sc ? scale->raw_dtype : 0, m->cfg.norm_weight_offset, n);
         NVL_HIP(hipGetLastError());
     }
@@ -356,7 +410,13 @@ f32x2* lay_rotation(nvl_model* m, const nvl_layer_config& c) {
     std::vector<double> f((size_t)half);
     double mag = 1.0;
     for (int i = 0; i < half; i++) f[(size_t)i] = std::pow(c.rot_base, -2.0 * i / c.rot_dim);
-    if (c.rot_factor > 0.0) {      // YaRN: pairs that turn often over the original length keep their frequency, the others are slowed down
+    if (c.rot_high > 0.0) {        // Llama 3.1: waves longer than original / low are slowed down, those shorter than original / high are not, in between a blend
+        for (double& v : f) {
+            const double wave = 2.0 * M_PI / v, s = (c.rot_original / wave - c.rot_low) / (c.rot_high - c.rot_low);
+            if (wave > c.rot_original / c.rot_low) v /= c.rot_factor;
+            else if (!(wave < c.rot_original / c.rot_high)) v = (1.0 - s) * v / c.rot_factor + s * v;
+        }
+    } else if (c.rot_factor > 0.0) {      // YaRN: pairs that turn often over the original length keep their frequency, the others are slowed down
         auto place = [&](double turns) { return c.rot_dim * std::log(c.rot_original / (2.0 * M_PI * turns)) / (2.0 * std::log(c.rot_base)); };
         const double lo = std::max(std::floor(place(c.rot_fast)), 0.0), hi = std::min(std::ceil(place(c.rot_slow)), c.rot_dim - 1.0);
         for (int i = 0; i < half; i++) {
@@ -405,7 +465,7 @@ void layered_finalize(nvl_model* m) {
     };
     const int64_t H = m->H;
     need(m->g[NVL_T_TOK_EMB], "token embedding"); need(m->g[NVL_T_FINAL_NORM_W], "final norm");
-    const bool post = m->cfg.block_style == NVL_BLOCK_POST;
+    const bool sum = m->cfg.block_style == NVL_BLOCK_SUM_NORM, post = sum || m->cfg.block_style == NVL_BLOCK_POST;      // post: sublayers read the stream itself
     const bool par = m->cfg.block_style == NVL_BLOCK_PARALLEL, ln = m->cfg.norm_type == NVL_NORM_LAYER, learned = m->cfg.position_type == NVL_POS_LEARNED;
     m->final_norm = lay_norm(m, m->g[NVL_T_FINAL_NORM_W], H);
     if (ln) m->final_norm_b = lay_vector(m, need(m->g[NVL_T_FINAL_NORM_B], "final norm bias"), H);
@@ -448,12 +508,15 @@ void layered_finalize(nvl_model* m) {
             if (!post) w.norm1 = lay_norm(m, T(NVL_T_ATTN_NORM_W, "norm before the mixer"), H);
             if (ln) w.norm1_bias = lay_vector(m, T(NVL_T_ATTN_NORM_B, "bias of the norm before the mixer"), H);
             if (!par) w.norm1b = lay_norm(m, T(NVL_T_MIX_POST_NORM, "norm after the mixer"), H, &l.t[NVL_T_MIX_SCALE]);
+            if (m->cfg.token_shift) w.shift = lay_vector(m, T(NVL_T_SHIFT, "token shift"), H);
+            if (sum && (c.ffn_dim || c.experts)) w.norm2b = lay_norm(m, T(NVL_T_FFN_POST_NORM, "norm after the feed-forward"), H);
             if (c.ffn_dim) {
                 if (!post && !par) w.norm2 = lay_norm(m, T(NVL_T_FFN_NORM_W, "norm before the feed-forward"), H);
-                if (!par) w.norm2b = lay_norm(m, T(NVL_T_FFN_POST_NORM, "norm after the feed-forward"), H, &l.t[NVL_T_FFN_SCALE]);
+                if (!par && !sum) w.norm2b = lay_norm(m, T(NVL_T_FFN_POST_NORM, "norm after the feed-forward"), H, &l.t[NVL_T_FFN_SCALE]);
                 const DevTensor& w1 = T(NVL_T_W1, "feed-forward gate / up");
-                if (!r.ffn_in && !r.glu_in) w.w1 = lay_matrix(m, (r.act == NVL_ACT_RELU2 ? 1 : 2) * r.Fp, H);
-                if (r.ffn_in || r.glu_in) {}      // (rows of the fused input projection)
+                const bool in_experts = r.shared_parts && !m->f32;        // (rows of the experts' matrix)
+                if (!r.ffn_in && !r.glu_in && !in_experts) w.w1 = lay_matrix(m, (r.act == NVL_ACT_RELU2 ? 1 : 2) * r.Fp, H);
+                if (r.ffn_in || r.glu_in || in_experts) {}      // (or rows of the fused input projection)
                 else if (r.act == NVL_ACT_RELU2) lay_place(m, w1, w.w1, H);
                 else if (m->f32) { lay_place(m, w1, w.w1, H, 0, 0, 0, 0, 0, 0, c.ffn_dim); lay_place(m, w1, w.w1, H, r.Fp, 0, 0, 0, 0, c.ffn_dim, c.ffn_dim); }
                 else { lay_place(m, w1, w.w1, H, 0, 16, 32, 0, 0, 0, c.ffn_dim); lay_place(m, w1, w.w1, H, 16, 16, 32, 0, 0, c.ffn_dim, c.ffn_dim); }
@@ -463,10 +526,10 @@ void layered_finalize(nvl_model* m) {
                 }
             }
             if (c.experts) {
-                const int64_t E = c.experts, I = c.expert_dim, Ip = r.Ip;
+                const int64_t E = c.experts, I = c.expert_dim, Ip = r.Ip, Es = E + (m->f32 ? 0 : r.shared_parts);
                 const DevTensor &up = T(NVL_T_MOE_IN, "experts' gate / up"), &down = T(NVL_T_MOE_OUT, "experts' down");
                 // (a grouped launch reads whole column tiles of its expert's rows: the last expert's need rows behind them)
-                w.moe_up = lay_matrix(m, (E - 1) * 2 * Ip + round_up(2 * Ip, W_ROW_PAD), H);
+                w.moe_up = lay_matrix(m, (Es - 1) * 2 * Ip + round_up(2 * Ip, W_ROW_PAD), H);
                 w.moe_down = lay_matrix(m, (E - 1) * H + round_up(H, W_ROW_PAD), Ip);
                 if (!m->f32) w.moe_cat = lay_matrix(m, H, r.Ep * Ip);
                 for (int64_t e = 0; e < E; e++) {
@@ -476,6 +539,13 @@ void layered_finalize(nvl_model* m) {
                     lay_place(m, down, w.moe_down, Ip, e * H, 0, 0, 0, 0, e * m->Hn, m->Hn);
                     if (!m->f32) lay_place(m, down, w.moe_cat, r.Ep * Ip, 0, 0, 0, 0, 0, e * m->Hn, m->Hn, false, false, e * Ip);
                 }
+                if (Es > E) {        // the shared expert behind them: the same 16 + 16 rows, its columns of the down projection
+                    const DevTensor& w1 = T(NVL_T_W1, "shared expert's gate / up");
+                    lay_place(m, w1, w.moe_up, H, E * 2 * Ip, 16, 32, 0, 0, 0, c.ffn_dim);
+                    lay_place(m, w1, w.moe_up, H, E * 2 * Ip + 16, 16, 32, 0, 0, c.ffn_dim, c.ffn_dim);
+                    lay_place(m, T(NVL_T_W2, "shared expert's down"), w.moe_cat, r.Ep * Ip, 0, 0, 0, 0, 0, 0, -1, false, false, E * Ip);
+                }
+                if (!par) { w.router = lay_matrix(m, E, H); lay_place(m, T(NVL_T_ROUTER, "router"), w.router, H); }
                 if (l.t[NVL_T_ROUTER_BIAS].present()) w.route_bias = lay_vector(m, l.t[NVL_T_ROUTER_BIAS], E);
             }
             if (sd) {
@@ -521,7 +591,20 @@ void layered_finalize(nvl_model* m) {
                 lay_place(m, T(NVL_T_WQ, "query projection"), w.in, H, 0, c.dim, r.dp);
                 lay_place(m, T(NVL_T_WK, "key projection"), w.in, H, r.k_off, c.dim, r.dp);
                 lay_place(m, T(NVL_T_WV, "value projection"), w.in, H, r.v_off, c.vdim, r.vp);
-                lay_place(m, T(NVL_T_MIX_GATE, "output gate"), w.in, H, r.gate_off, c.vdim, r.vp);
+                if (!c.ungated) lay_place(m, T(NVL_T_MIX_GATE, "output gate"), w.in, H, r.gate_off, c.vdim, r.vp);
+                if (c.qkv_bias) {
+                    w.in_bias = (float*)lay_alloc(m, round_up(r.n_in, W_ROW_PAD) * 4);
+                    auto bias = [&](int kind, const char* what, int off, int d, int dp) {
+                        const DevTensor& t = T(kind, what);
+                        const Place2D pl{1, t.rows, round_up(r.n_in, W_ROW_PAD), 0, 1, 1, d, dp, off};
+                        hipLaunchKernelGGL((place_2d_kernel<float, false, false>), dim3((unsigned)std::min<int64_t>(cdiv(t.rows, 256), 64), 1, 1), dim3(256), 0, m->stream, t.p, t.raw_dtype, 0, w.in_bias, pl);
+                        NVL_HIP(hipGetLastError());
+                    };
+                    bias(NVL_T_BQ, "query bias", 0, c.dim, r.dp); bias(NVL_T_BK, "key bias", r.k_off, c.dim, r.dp); bias(NVL_T_BV, "value bias", r.v_off, c.vdim, r.vp);
+                }
+                if (c.qk_norm) { w.q_norm = lay_vector(m, T(NVL_T_Q_NORM, "query norm"), l.t[NVL_T_Q_NORM].rows); w.k_norm = lay_vector(m, T(NVL_T_K_NORM, "key norm"), l.t[NVL_T_K_NORM].rows); }
+                if (c.sink == NVL_SINK_LEARNED) w.sink = lay_vector(m, T(NVL_T_SINK, "sinks"), c.heads);
+                else if (c.sink) w.sink = (float*)lay_alloc(m, (int64_t)c.heads * 4);
                 if (l.t[NVL_T_BIAS_R1].present()) {
                     w.r1 = lay_vector(m, l.t[NVL_T_BIAS_R1], c.heads);
                     w.r2 = lay_vector(m, T(NVL_T_BIAS_R2, "distance bias (r2)"), c.heads);
@@ -534,6 +617,19 @@ void layered_finalize(nvl_model* m) {
                 if (c.v_mix) w.v_lambda = lay_vector(m, T(NVL_T_V_MIX, "value mixing"), 1);
                 w.o = lay_matrix(m, H, r.kd);
                 lay_place(m, T(NVL_T_WO, "output projection"), w.o, r.kd, 0, 0, 0, c.vdim, r.vp);
+                if (c.mixer2) {
+                    lay_place(m, T(NVL_T_LIN_Q, "lightning query projection"), w.in, H, r.lq_off); lay_place(m, T(NVL_T_LIN_K, "lightning key projection"), w.in, H, r.lk_off);
+                    lay_place(m, T(NVL_T_LIN_V, "lightning value projection"), w.in, H, r.lv_off); lay_place(m, T(NVL_T_LIN_GATE, "lightning gate"), w.in, H, r.lg_off);
+                    const int64_t hv = (int64_t)c.heads2 * c.vdim2;
+                    w.lin_norm = lay_vector(m, T(NVL_T_LIN_NORM, "lightning norm"), hv);
+                    lay_scale(m, w.lin_norm, c.out_scale2, hv);
+                    lay_place(m, T(NVL_T_LIN_O, "lightning output projection"), w.o, r.kd, 0, 0, 0, 0, 0, 0, -1, false, false, r.ko);
+                    std::vector<float> d((size_t)c.heads2 * 2);       // decays, then their logarithms (a decay of zero: finite, and far below every sum)
+                    for (int h = 0; h < c.heads2; h++) { d[(size_t)h] = (float)c.decay[h]; d[(size_t)(c.heads2 + h)] = (float)std::max(std::log2(c.decay[h]), -1e30); }
+                    w.decay = (float*)lay_alloc(m, (int64_t)d.size() * 4); w.log2_decay = w.decay + c.heads2;
+                    NVL_HIP(hipMemcpyAsync(w.decay, d.data(), d.size() * 4, hipMemcpyHostToDevice, m->stream));
+                    NVL_HIP(hipStreamSynchronize(m->stream));
+                }
             } else if (c.mixer == NVL_MIXER_MAMBA2) {
                 w.in = lay_matrix(m, r.n_in, H);
                 lay_place(m, T(NVL_T_MAMBA_IN_PROJ, "input projection"), w.in, H);
@@ -596,7 +692,7 @@ void layered_finalize(nvl_model* m) {
             }
             if (r.ffn_in) lay_place(m, T(NVL_T_W1, "feed-forward up"), w.in, H, r.ffn_off);
             if (r.glu_in) lay_place(m, T(NVL_T_W1, "feed-forward gate / up"), w.in, H, r.ffn_off, c.ffn_dim, r.Fp);
-            if (c.experts) lay_place(m, T(NVL_T_ROUTER, "router"), w.in, H, r.route_off);
+            if (c.experts && par) lay_place(m, T(NVL_T_ROUTER, "router"), w.in, H, r.route_off);
             if (par && c.ffn_dim) lay_place(m, T(NVL_T_W2, "feed-forward down"), w.o, r.kd, 0, 0, 0, 0, 0, 0, -1, false, false, r.ko);
             NVL_HIP(hipStreamSynchronize(m->stream));
             for (auto& t : l.t) { dfree(t.p); t.p = nullptr; }
@@ -605,7 +701,7 @@ void layered_finalize(nvl_model* m) {
     for (int i = 0; i < m->L; i++) {
         LayerRun& r = m->runs[(size_t)i];
         const nvl_layer_config& c = r.c;
-        if (c.mixer == NVL_MIXER_LATENT_ATTENTION && c.rot_dim) {
+        if (c.rot_dim) {
             for (int j = 0; j < i && !r.turn; j++)
                 if (m->runs[(size_t)j].turn && same_rotation(m->runs[(size_t)j].c, c)) r.turn = m->runs[(size_t)j].turn;
             if (!r.turn) r.turn = lay_rotation(m, c);
@@ -618,9 +714,10 @@ void layered_finalize(nvl_model* m) {
             pa_cols = std::max<int64_t>(pa_cols, w.a_rkp); pg_cols = std::max<int64_t>(pg_cols, w.g_rkp);
         }
         if (c.mixer == NVL_MIXER_GLA) r.n_in = 2 * c.heads * (c.dim + c.vdim) + m->mixers[(size_t)r.owner].rank;
-        const bool qg = c.mixer == NVL_MIXER_ATTENTION && !m->f32;           // (its projection goes to lqg, the cache and lmix; the router's columns stay)
+        const bool qg = c.mixer == NVL_MIXER_ATTENTION && !m->f32 && !r.raw;           // (its projection goes to lqg, the cache and lmix; the router's columns stay)
         ld_in = std::max(ld_in, round_up(qg ? r.n_in - (r.ffn_in ? r.route_off : r.ffn_off) : r.n_in, 4));
-        if (qg) qg_cols = std::max<int64_t>(qg_cols, (int64_t)c.heads * (r.dp + r.vp));
+        if (c.experts && !par) ld_in = std::max(ld_in, round_up(c.experts, 4));         // (the router's scores, once the mixer is done)
+        if (qg || r.raw) qg_cols = std::max<int64_t>(qg_cols, (int64_t)c.heads * (r.dp + (c.ungated ? 0 : r.vp)));
         ko = std::max<int64_t>(ko, r.kd);
         Fmax = std::max<int64_t>(Fmax, r.Fp);
         if (c.experts) {
@@ -634,6 +731,7 @@ void layered_finalize(nvl_model* m) {
             if (lat_absorb_ok(m, r)) abs_cols = std::max(abs_cols, round_up(c.heads, 16) * (r.rp + r.rotp));
         } else if (c.mixer == NVL_MIXER_ATTENTION) {
             grp_vp = std::max<int64_t>(grp_vp, r.vp);
+            if (c.mixer2) ocols = std::max<int64_t>(ocols, (int64_t)c.heads2 * c.vdim2);
         } else {
             ocols = std::max<int64_t>(ocols, (int64_t)c.heads * c.vdim);
             conv = std::max<int64_t>(conv, r.conv_dim);
@@ -668,7 +766,7 @@ void layered_finalize(nvl_model* m) {
         }
     }
     if (sd) m->lside = lay_alloc(m, Mp * m->side_kp * ws);
-    if (qg_cols) m->lqg = (bf16_t*)lay_alloc(m, Mp * qg_cols * 2);
+    if (qg_cols) m->lqg = lay_alloc(m, Mp * qg_cols * ws);
     if (m->lvf_ld) m->lvf = (float*)lay_alloc(m, Mmax * m->lvf_ld * 4);
     if (grp_vp && !m->f32 && grp_vp <= 256) {
         m->grp_cap = GROUPED_SPLIT_WGS;
@@ -688,6 +786,14 @@ void layered_finalize(nvl_model* m) {
     if (conv) m->lconv = f32buf(Mmax * m->lconv_ld);
     if (m->lat_block_stride) m->lat_cache = lay_alloc(m, m->lat_block_stride * m->num_blocks * ws);
     if (m->rec_slot_stride) m->rec_state = f32buf(m->rec_slot_stride * S);
+    if (m->cfg.token_shift) {
+        m->lshift = f32buf((int64_t)m->L * S * H);
+        std::vector<int64_t> off;
+        for (const LayerRun& r : m->runs) off.push_back(r.shift_off);
+        m->shift_offs = (int64_t*)lay_alloc(m, (int64_t)off.size() * 8);
+        NVL_HIP(hipMemcpyAsync(m->shift_offs, off.data(), off.size() * 8, hipMemcpyHostToDevice, m->stream));
+        NVL_HIP(hipStreamSynchronize(m->stream));
+    }
     if (abs_cols) {     // tokens on the absorbed form, and their partial results: splits x tokens <= max(tokens, LAT_PART)
         m->lat_abs_cap = (int)std::max<int64_t>(std::min(Mmax, S * LAT_ABSORB_MAX), 512);
         m->lat_qa = (bf16_t*)lay_alloc(m, (int64_t)m->lat_abs_cap * abs_cols * 2);
@@ -701,7 +807,7 @@ void layered_finalize(nvl_model* m) {
     m->argmax_pidx = dmalloc<int32_t>(std::max<int64_t>(S, Mmax) * cdiv(m->V, ARGMAX_CHUNK));
     m->sk_rows = (int)std::min<int64_t>(std::max<int64_t>(Mmax, 64), SK_TILE_MAX_M);
     if (!m->f32) m->sk_part = dmalloc<float>((int64_t)std::max(m->sk_max_slices, SK_TILE_MAX_SLICES) * m->sk_rows * H);
-    m->key_rows.assign(m->windows.size(), 0); m->key_max.assign(m->windows.size(), 0);
+    m->key_rows.assign(m->masks.size(), 0); m->key_max.assign(m->masks.size(), 0);
     init_slots(m);
     init_meta(m);
     NVL_HIP(hipStreamSynchronize(m->stream));
@@ -721,17 +827,25 @@ void layered_free(nvl_model* m) {
 // Which tokens take the absorbed attention, and where every other sequence's keys sit in the key workspace.  hm: host metadata with
 // the sequences filled in; `steps` one-token passes will run on it (the positions advance on the device).
 void layered_meta(nvl_model* m, const Meta& hm, int n_seqs, int steps) {
-    bool absorb = !m->windows.empty();
+    bool absorb = !m->masks.empty();
     for (const LayerRun& r : m->runs) if (r.c.mixer == NVL_MIXER_LATENT_ATTENTION) absorb &= lat_absorb_ok(m, r);
     m->n_abs = 0; m->meta_dynamic = false;
     m->min_len = hm.seq_len[0];
-    for (size_t w = 0; w < m->windows.size(); w++) { m->key_rows[w] = 0; m->key_max[w] = 0; }
+    for (size_t w = 0; w < m->masks.size(); w++) { m->key_rows[w] = 0; m->key_max[w] = 0; }
     const int64_t S = m->opts.max_seqs;
-    m->win_pairs.assign(m->windows.size(), {0.0, 0.0}); m->win_keys.assign(m->windows.size(), {0.0, 0.0});
+    m->win_pairs.assign(m->masks.size(), {0.0, 0.0}); m->win_keys.assign(m->masks.size(), {0.0, 0.0});
     for (int i = 0; i < n_seqs; i++) {
         const int n = hm.seq_len[i], pos = hm.seq_pos[i];
-        for (size_t w = 0; w < m->windows.size(); w++) {       // visible (query, key) pairs, keys read: [several new tokens]
-            const double W = m->windows[w] > 0 ? m->windows[w] : 1e18, full = std::min<double>(n, std::max(0.0, pos + n - W));      // tokens whose window is full
+        for (size_t w = 0; w < m->masks.size(); w++) {       // visible (query, key) pairs, keys read: [several new tokens]
+            const KeyMask& k = m->masks[w];
+            if (k.chunk > 0) {                                // a first part of a chunk, whole chunks, a last part
+                auto upto = [&](double p) { const double c = std::floor(p / k.chunk), x = p - c * k.chunk; return c * k.chunk * (k.chunk + 1.0) / 2 + x * (x + 1) / 2; };
+                m->win_pairs[w][n > 1] += upto(pos + n) - upto(pos);
+                m->win_keys[w][n > 1] += pos + n - k.lo(pos);
+                continue;
+            }
+            m->win_pairs[w][n > 1] += (double)n * std::min<double>(k.keep, std::max(0, pos - k.window)); m->win_keys[w][n > 1] += std::min<double>(k.keep, std::max(0, pos - k.window));      // (kept tokens behind the window, nearly)
+            const double W = k.window > 0 ? k.window : 1e18, full = std::min<double>(n, std::max(0.0, pos + n - W));      // tokens whose window is full
             const double part = n - full;                       // the others are the first ones: they see pos + 1 .. pos + part keys
             m->win_pairs[w][n > 1] += full * std::min(W, 1e17) * (full > 0) + part * pos + part * (part + 1) / 2;
             m->win_keys[w][n > 1] += std::min<double>(pos + n, W + n - 1);
@@ -739,12 +853,12 @@ void layered_meta(nvl_model* m, const Meta& hm, int n_seqs, int steps) {
         m->min_len = std::min(m->min_len, n);
         const bool abs = absorb && n <= LAT_ABSORB_MAX;
         if (abs) for (int j = 0; j < n; j++) { hm.abs_tok[m->n_abs] = hm.seq_tok_start[i] + j; hm.abs_seq[m->n_abs] = i; m->n_abs++; }
-        for (size_t w = 0; w < m->windows.size(); w++) {
+        for (size_t w = 0; w < m->masks.size(); w++) {
             if (abs) { hm.kbase[(int64_t)w * S + i] = -1; continue; }
-            int64_t nk = (int64_t)pos + n - latent_key0(pos, m->windows[w]);
+            int64_t nk = (int64_t)pos + n - latent_key0(pos, m->masks[w].window);
             if (steps > 1) {
                 nk = (int64_t)pos + n + steps;
-                if (m->windows[w] > 0) nk = std::min<int64_t>(nk, m->windows[w] + n + 31);
+                if (m->masks[w].window > 0) nk = std::min<int64_t>(nk, m->masks[w].window + n + 31);
             }
             hm.kbase[(int64_t)w * S + i] = (int32_t)m->key_rows[w];
             m->key_rows[w] += round_up(nk, 32);
@@ -759,8 +873,8 @@ int layered_kt_log2(const nvl_model* m) {
     int64_t ctx = m->ctx_hint > 0 ? m->ctx_hint : m->cfg.max_seq_len;
     bool windowed = true;
     int w = 0;
-    for (int x : m->windows) { windowed &= x > 0; w = std::max(w, x); }
-    if (windowed && !m->windows.empty()) ctx = std::min<int64_t>(ctx, w);
+    for (const KeyMask& x : m->masks) { windowed &= x.span() > 0; w = std::max(w, x.span() + (x.keep ? 64 : 0)); }
+    if (windowed && !m->masks.empty()) ctx = std::min<int64_t>(ctx, w);
     int b = 0;
     while ((64ll << b) < ctx) b++;
     return b;
@@ -773,16 +887,21 @@ struct SubOut { const float* y; int slices; int64_t stride; };
 struct NextNorm { const float *w, *b; bool raw; };
 // experts' results that join the stream beside a sublayer's: K slices, or rows of pairs to be gathered and weighted
 struct ExpertOut { const float* y = nullptr; int slices = 0; int64_t stride = 0; const int32_t* slot_of = nullptr; const float* gate_w = nullptr; };
+// token shift of the next mixer's input: its weights, the rows kept in the slots (one token per sequence: done by the same launch)
+struct ShiftOut { const float* mu = nullptr; float* state = nullptr; const Meta* md = nullptr; };
 
-// x += rms(y) * w_post (w_post NULL: x += y + experts) and / or xn = next(x) (elem.h SandwichArgs)
-void sandwich(nvl_model* m, SubOut y, const float* w_post, NextNorm next, void* xn, int rows, const int32_t* rows_idx = nullptr, ExpertOut ex = {}) {
+// x += rms(y) * w_post (w_post NULL: x += y + experts; NVL_BLOCK_SUM_NORM: x = rms(stream_scale x + y + experts) * w_post) and / or
+// xn = next(x) (elem.h SandwichArgs)
+void sandwich(nvl_model* m, SubOut y, const float* w_post, NextNorm next, void* xn, int rows, const int32_t* rows_idx = nullptr, ExpertOut ex = {}, ShiftOut sh = {}) {
     KScope ks(m, KC_OTHER, 0, KS_SANDWICH, (double)rows * m->Hn * ((y.y ? 8.0 + 4.0 * (std::max(y.slices, 1) + ex.slices) : 4.0) + (next.w || next.raw ? (double)m->wsize : 0.0)));
     SandwichArgs a{};
     a.x = m->x; a.y = y.y; a.slices = y.slices; a.slice_stride = y.stride; a.w_post = w_post; a.w_next = next.w; a.b_next = next.b; a.rows_idx = rows_idx;
     a.rows = rows; a.H = m->H; a.width = m->Hn; a.eps = m->cfg.norm_eps; a.raw_next = next.raw;
     a.y2 = ex.y; a.slices2 = ex.slices; a.stride2 = ex.stride; a.slot_of = ex.slot_of; a.gate_w = ex.gate_w;
-    const bool ext = (y.y && !w_post) || next.b;
-    if (!m->f32 && rows > 512 && m->H <= 4096 && y.slices <= 1) {
+    if (m->cfg.block_style == NVL_BLOCK_SUM_NORM && w_post) a.sum_scale = m->cfg.stream_scale;
+    if (sh.mu) { a.shift = sh.mu; a.before = sh.state; a.before_stride = m->rec_slot_stride; a.seq_slot = sh.md->seq_slot; a.seq_pos = sh.md->seq_pos; }
+    const bool ext = (y.y && !w_post) || next.b || a.sum_scale != 0.f || sh.mu;
+    if (!m->f32 && rows > 512 && !sh.mu && m->H <= 4096 && y.slices <= 1) {
         const size_t lds = (size_t)16 * m->H * 2;
 #define NVL_SW16E(CH, EXT)                                                                                                  \
         do {                                                                                                                \
@@ -842,7 +961,7 @@ void grow(nvl_model* m, float*& p, int64_t& have, int64_t want) {
 // ------------------------------------------------------------------------------------------
 void in_proj(nvl_model* m, const LayerRun& r, const MixerW& w, int M) {
     m->site = KS_MIX_IN;
-    gemm(m, EPI_STORE, true, mk(m->xn, m->H, w.in, m->lproj, (int)m->lproj_ld, nullptr, 1.f, M, r.n_in, m->H));
+    gemm(m, EPI_STORE, true, mk(m->xn, m->H, w.in, m->lproj, (int)m->lproj_ld, w.in_bias, 1.f, M, r.n_in, m->H));
 }
 
 void mix_latent(nvl_model* m, const LayerRun& r, const MixerW& w, const Meta& md, int n_seqs, int M, int max_len) {
@@ -991,23 +1110,23 @@ void linrec(nvl_model* m, LinRecArgs a, int n_seqs, int M, int max_len, bool fus
 }
 
 template <typename ActT, bool GATE_FIRST>
-void gated_norm_launch(nvl_model* m, GatedNormArgs a) {
+void gated_norm_launch(nvl_model* m, GatedNormArgs a, int col) {
     const bool v4 = a.part % 4 == 0 && a.y_ld % 4 == 0 && a.gate_ld % 4 == 0 && (((uintptr_t)a.y | (uintptr_t)a.gate) & 15) == 0;
     const bool wide = a.part > 1024;
     a.lanes = 4;
     while (a.lanes < 64 && a.lanes * (v4 ? 4 : 1) < a.part) a.lanes *= 2;
     const dim3 grid(wide ? a.rows * a.parts : cdiv((int64_t)a.rows * a.parts, 256 / a.lanes));
-    ActT* out = (ActT*)m->lmix;
+    ActT* out = (ActT*)m->lmix + (sizeof(ActT) == 2 ? (int64_t)(col >> 5) * 512 : col);      // (the operand's column blocks are 32 wide: a shift by columns is a shift of the base)
     if (wide && v4) hipLaunchKernelGGL((gated_norm_kernel<ActT, GATE_FIRST, true, true>), grid, dim3(256), 0, m->stream, a, out);
     else if (wide) hipLaunchKernelGGL((gated_norm_kernel<ActT, GATE_FIRST, true, false>), grid, dim3(256), 0, m->stream, a, out);
     else if (v4) hipLaunchKernelGGL((gated_norm_kernel<ActT, GATE_FIRST, false, true>), grid, dim3(256), 0, m->stream, a, out);
     else hipLaunchKernelGGL((gated_norm_kernel<ActT, GATE_FIRST, false, false>), grid, dim3(256), 0, m->stream, a, out);
 }
 template <bool GATE_FIRST>
-void gated_norm(nvl_model* m, const GatedNormArgs& a, int site) {
+void gated_norm(nvl_model* m, const GatedNormArgs& a, int site, int col = 0) {
     KScope ks(m, KC_OTHER, 0, site, (double)a.rows * a.parts * a.part * (8.0 + (double)m->wsize));
-    if (m->f32) gated_norm_launch<float, GATE_FIRST>(m, a);
-    else gated_norm_launch<bf16_t, GATE_FIRST>(m, a);
+    if (m->f32) gated_norm_launch<float, GATE_FIRST>(m, a, col);
+    else gated_norm_launch<bf16_t, GATE_FIRST>(m, a, col);
     NVL_HIP(hipGetLastError());
 }
 
@@ -1151,12 +1270,24 @@ void mix_delta(nvl_model* m, const LayerRun& r, const MixerW& w, const Meta& md,
 
 void tap_layer(nvl_model* m, int li, int M);
 
+// ---- lightning attention beside another mixer: columns of the joint input projection -> m->lmix columns [ko, ko + ko2) ----
+void mix_lightning(nvl_model* m, const LayerRun& r, const MixerW& w, const Meta& md, int n_seqs, int M, int max_len) {
+    const nvl_layer_config& c = r.c;
+    LinRecArgs a = linrec_args(m, r, md);
+    a.H = c.heads2; a.DK = c.dim2; a.DV = c.vdim2; a.DVp = (int)round_up(c.vdim2, 4); a.kdiv = 1; a.q_scale = 1.f;
+    a.q = m->lproj + r.lq_off; a.k = m->lproj + r.lk_off; a.v = m->lproj + r.lv_off; a.ld = m->lproj_ld;
+    a.decay = w.decay; a.log2_decay = w.log2_decay;
+    linrec<false>(m, a, n_seqs, M, max_len, false, KS_LIN_SCAN);
+    GatedNormArgs g{m->lo, m->lo_ld, m->lproj + r.lg_off, m->lproj_ld, w.lin_norm, M, 1, c.heads2 * c.vdim2, m->cfg.norm_eps, r.kd, 0, 1};
+    gated_norm<false>(m, g, KS_LIN_GATE, r.ko);
+}
+
 // ---- grouped-query attention: m->xn -> m->lmix columns [0, ko) ----
 void mix_grouped(nvl_model* m, const LayerRun& r, const MixerW& w, const Meta& md, int n_seqs, int M, int max_len) {
     const nvl_layer_config& c = r.c;
     GroupedArgs a{};
     a.H = c.heads; a.G = c.kv_heads; a.group = c.heads / c.kv_heads; a.dim = c.dim; a.dp = r.dp; a.vdim = c.vdim; a.vp = r.vp;
-    a.window = c.window; a.scale = c.scale; a.softcap = c.softcap; a.r1 = w.r1; a.r2 = w.r2;
+    a.mask = m->masks[(size_t)r.win]; a.scale = c.scale; a.softcap = c.softcap; a.r1 = w.r1; a.r2 = w.r2; a.sink = w.sink; a.out_scale = c.out_scale != 0.f ? c.out_scale : 1.f;
     a.mix = r.mix; a.lambda = w.v_lambda; a.vfirst = m->lvf; a.vfirst_ld = m->lvf_ld;
     a.cache = (char*)m->lat_cache + r.cache_off * (int64_t)m->wsize; a.block_stride = m->lat_block_stride; a.bs = m->Tmax;
     a.blk_table = md.blk_table; a.seq_tok_start = md.seq_tok_start; a.seq_len = md.seq_len; a.seq_pos = md.seq_pos; a.tbl_stride = m->blocks_per_seq;
@@ -1164,28 +1295,47 @@ void mix_grouped(nvl_model* m, const LayerRun& r, const MixerW& w, const Meta& m
     const double ws = (double)m->wsize;
     if (m->f32) {
         in_proj(m, r, w, M);
-        a.q = m->lproj; a.q_ld = m->lproj_ld; a.gate_col = r.gate_off;
-        a.proj = m->lproj; a.proj_ld = m->lproj_ld; a.k_off = r.k_off; a.v_off = r.v_off;
+        a.q = m->lproj; a.q_ld = m->lproj_ld; a.gate_col = c.ungated ? -1 : r.gate_off;
+        a.proj = m->lproj; a.proj_ld = m->lproj_ld; a.k_off = r.raw ? -1 : r.k_off; a.v_off = r.v_off;
+        if (c.mixer2) {
+            KScope ks(m, KC_OTHER);
+            hipLaunchKernelGGL(silu_cols_kernel, dim3(M), dim3(256), 0, m->stream, m->lproj, m->lproj_ld, r.lq_off, r.lg_off - r.lq_off);
+            NVL_HIP(hipGetLastError());
+        }
         KScope ks(m, KC_OTHER, 0, KS_KV_PLACE, (double)M * a.G * (c.dim + c.vdim) * (4.0 + ws) + (r.mix ? (double)M * a.G * c.vdim * 4.0 : 0.0));
         hipLaunchKernelGGL(grouped_place_kernel, dim3(cdiv(max_len + 31, 32), n_seqs, a.G), dim3(256), 0, m->stream, a);
         NVL_HIP(hipGetLastError());
     } else {
-        a.q = m->lqg; a.q_ld = (int64_t)a.H * (r.dp + r.vp); a.gate_col = a.H * r.dp;
-        GemmArgs g = mk(m->xn, m->H, w.in, m->lqg, (int)a.q_ld, nullptr, 1.f, M, r.n_in, m->H);
-        g.grp = GroupedEpi{r.k_off, r.v_off, r.gate_off, r.ffn_off, r.ffn_in ? r.route_off : r.ffn_off, md.tok_pos, md.tok_tbl, md.blk_table, (bf16_t*)a.cache, a.block_stride, a.bs, a.G, r.dp, r.vp,
-                           r.mix, w.v_lambda, m->lvf, m->lvf_ld, (bf16_t*)m->lmix + (r.ko >> 5) * 512, r.kd, m->lproj, m->lproj_ld};
+        a.q = m->lqg; a.q_ld = (int64_t)a.H * (r.dp + (c.ungated ? 0 : r.vp)); a.gate_col = c.ungated ? -1 : a.H * r.dp;
+        GemmArgs g = mk(m->xn, m->H, w.in, m->lqg, (int)a.q_ld, w.in_bias, 1.f, M, r.n_in, m->H);
+        g.grp = GroupedEpi{r.k_off, r.v_off, r.gate_off, r.raw ? 1 << 30 : r.ffn_off, r.raw ? 1 << 30 : r.ffn_in ? r.route_off : r.ffn_off, md.tok_pos, md.tok_tbl, md.blk_table, (bf16_t*)a.cache, a.block_stride, a.bs, a.G, r.dp, r.vp,
+                           r.mix, w.v_lambda, m->lvf, m->lvf_ld, (bf16_t*)m->lmix + (r.ko >> 5) * 512, r.kd, m->lproj, m->lproj_ld,
+                           m->lproj, m->lproj_ld, r.ffn_off, c.mixer2 ? r.lg_off : 0};
         m->site = KS_MIX_IN;
-        gemm(m, EPI_GROUPED, false, g);
+        gemm(m, r.raw ? EPI_GROUPED_RAW : EPI_GROUPED, false, g);
     }
+    if (r.raw) {          // norms and rotation of the fp32 queries and keys
+        a.proj = m->lproj; a.proj_ld = m->lproj_ld; a.qk_koff = r.k_off; a.qk_norm = c.qk_norm; a.q_norm = w.q_norm; a.k_norm = w.k_norm; a.eps = m->cfg.norm_eps;
+        a.rot = c.rot_dim; a.turn = r.turn; a.tok_pos = md.tok_pos; a.tok_tbl = md.tok_tbl; a.rows = M;
+        a.q = a.q_out = m->lqg; a.q_ld = (int64_t)a.H * r.dp;
+        KScope ks(m, KC_OTHER, 0, KS_QK_TURN, (double)M * (a.H + a.G) * c.dim * (4.0 + ws));
+        const int threads = std::min(1024, (a.H + a.G) * 64);
+        if (m->f32) hipLaunchKernelGGL((grouped_qk_row_kernel<float>), dim3(M), dim3(threads), 0, m->stream, a);
+        else if (M <= QK_ROW_MAX) hipLaunchKernelGGL((grouped_qk_row_kernel<bf16_t>), dim3(M), dim3(threads), 0, m->stream, a);
+        else hipLaunchKernelGGL(grouped_qk_tile_kernel, dim3(cdiv(M, 16)), dim3(1024), 0, m->stream, a);
+        NVL_HIP(hipGetLastError());
+    }
+    if (c.mixer2) mix_lightning(m, r, w, md, n_seqs, M, max_len);
     const bool plain = m->f32 || r.dp > 256 || r.vp > 256;
     const int ctx = m->ctx_hint > 0 ? m->ctx_hint : m->cfg.max_seq_len;
     int tiles = cdiv(ctx, 64) + 1;                              // most key tiles a 256-row workgroup walks
-    if (c.window > 0) tiles = std::min(tiles, (c.window + cdiv(256, a.group) + 1) / 64 + 3);
+    const int span = a.mask.span();
+    if (span > 0) tiles = std::min(tiles, (span + cdiv(256, a.group) + 1) / 64 + 3 + cdiv(a.mask.keep, 64));
     const size_t ring = (size_t)3 * round_up(4 * (r.dp >> 5) + 2 * (r.vp >> 4), 8) * 1024;
     size_t lds = ring + (size_t)tiles * 8;
     // the distance biases of a workgroup's rows as a table in LDS, where they leave as many workgroups per CU as the ring does
-    const size_t tab = lds + (size_t)grouped_tab_span(std::min(ctx, c.window > 0 ? c.window : ctx)) * a.group * 4;
-    if (w.r1 && tab <= (size_t)(r.dp <= 64 && r.vp <= 64 ? 80 : 160) * 1024) { a.table = tiles; lds = tab; }
+    const size_t tab = lds + (size_t)grouped_tab_span(std::min(ctx, span > 0 ? span : ctx)) * a.group * 4;
+    if (w.r1 && !a.mask.keep && tab <= (size_t)(r.dp <= 64 && r.vp <= 64 ? 80 : 160) * 1024) { a.table = tiles; lds = tab; }
     a.short_rows = GROUPED_SHORT_ROWS;
     if ((r.dp == 256 && r.vp == 256) || lds > 160 * 1024) a.short_rows = 1 << 30;      // (three slots would not fit LDS)
     const bool any_short = m->min_len * a.group <= a.short_rows, any_long = max_len * a.group > a.short_rows;
@@ -1280,6 +1430,78 @@ ExpertOut parallel_ffn(nvl_model* m, const LayerRun& r, const MixerW& w, int M) 
     return {m->moe_eo, k, 0, m->slot_of, m->expert_w};
 }
 
+// ---- gate and up of a gated feed-forward, m->xn -> m->hbuf (fp32 mode: W [gate rows | up rows], the activation in a launch of its own) ----
+void glu_up(nvl_model* m, const void* W, int M, int Fp, int act, float limit) {
+    m->site = KS_FFN_UP;
+    if (m->f32) {
+        gemm(m, EPI_STORE, true, mk(m->xn, m->H, W, m->h2, 2 * Fp, nullptr, 1.f, M, 2 * Fp, m->H));
+        const int64_t n = (int64_t)M * Fp;
+        KScope ks(m, KC_OTHER);
+        if (act == NVL_ACT_CLAMPED_GLU) hipLaunchKernelGGL((clamp_glu_kernel<float>), dim3(cdiv(n, 256)), dim3(256), 0, m->stream, m->h2, (float*)m->hbuf, (int64_t)M, Fp, limit, CLAMPED_GLU_SLOPE);
+        else if (act == NVL_ACT_REGLU) hipLaunchKernelGGL((reglu_kernel<float>), dim3(cdiv(n, 256)), dim3(256), 0, m->stream, m->h2, (float*)m->hbuf, (int64_t)M, Fp);
+        else hipLaunchKernelGGL((swiglu_kernel<float, true>), dim3(cdiv(n, 256)), dim3(256), 0, m->stream, m->h2, (float*)m->hbuf, (int64_t)M, Fp, (int64_t)Fp, 0);
+        NVL_HIP(hipGetLastError());
+        return;
+    }
+    GemmArgs up = mk(m->xn, m->H, W, m->hbuf, Fp, nullptr, 1.f, M, 2 * Fp, m->H);
+    up.glu_limit = limit; up.glu_slope = CLAMPED_GLU_SLOPE;
+    gemm(m, act == NVL_ACT_CLAMPED_GLU ? EPI_CLAMP_GLU : act == NVL_ACT_REGLU ? EPI_REGLU : EPI_GEGLU, false, up);
+}
+// ---- experts that read m->xn by themselves (their shared expert too); returns the shared expert's result, or in `joined` cases everything ----
+SubOut expert_ffn(nvl_model* m, const LayerRun& r, const MixerW& w, int M, ExpertOut& ex) {
+    const nvl_layer_config& c = r.c;
+    const int E = c.experts, k = c.top_k, pairs = M * k;
+    const bool dense = !m->f32 && M <= 64 && r.Ip <= 2048;          // decode: masked projections over all experts (gemm.h GemmArgs::moe_gate)
+    const int parts = dense ? r.shared_parts : 0;
+    SubOut y{nullptr, 1, 0};
+    if (c.ffn_dim && !parts) {
+        const void* W = r.shared_parts && !m->f32 ? (const void*)((const char*)w.moe_up + (int64_t)E * 2 * r.Ip * m->H * (int64_t)m->wsize) : w.w1;
+        glu_up(m, W, M, r.Fp, r.act, c.ffn_limit);
+        y = sub_out(m, KS_FFN_DOWN, m->hbuf, w.w2, M, r.Fp);
+    }
+    if (dense && E <= 64 && c.route_softmax) {
+        GemmArgs a = mk(m->xn, m->H, w.router, nullptr, E, w.route_bias, 1.f, M, E, m->H);
+        KScope ks(m, KC_OTHER, 2.0 * M * E * m->Hn, KS_MOE_ROUTER, ((double)E * m->Hn + (double)M * m->Hn) * (double)m->wsize + (double)M * E * 4.0);
+        hipLaunchKernelGGL(moe_router_gate_kernel, dim3(cdiv(M, 16)), dim3(1024), 0, m->stream, a, k, m->moe_gate, (float*)nullptr, 0, r.Ep, parts);
+        NVL_HIP(hipGetLastError());
+    } else {
+        m->site = KS_MOE_ROUTER;
+        gemm(m, EPI_STORE, true, mk(m->xn, m->H, w.router, m->lproj, (int)m->lproj_ld, nullptr, 1.f, M, E, m->H));
+        GroupRouteArgs ra{};
+        ra.logits = m->lproj; ra.ld = m->lproj_ld; ra.correction = w.route_bias; ra.rows = M; ra.E = E; ra.top = k; ra.groups = c.expert_groups; ra.keep = c.groups_kept;
+        ra.ids = m->expert_ids; ra.w = m->expert_w; ra.gate = dense ? m->moe_gate : nullptr; ra.gate_ld = r.Ep; ra.softmax = c.route_softmax; ra.n_always = parts;
+        KScope ks(m, KC_OTHER, 0, KS_MOE_ROUTER, (double)M * (E + 2.0 * k) * 4.0);
+        hipLaunchKernelGGL((moe_route_grouped_kernel<float>), dim3(cdiv(M, 4)), dim3(256), 0, m->stream, ra);
+        NVL_HIP(hipGetLastError());
+    }
+    if (dense) {
+        const double touch = (double)std::min(E, pairs) * c.expert_dim + (parts ? c.ffn_dim : 0), work = (double)pairs * c.expert_dim + (parts ? (double)M * c.ffn_dim : 0.0);
+        GemmArgs u = mk(m->xn, m->H, w.moe_up, m->moe_hall, r.Ep * r.Ip, nullptr, 1.f, M, (E + parts) * 2 * r.Ip, m->H);
+        u.moe_gate = m->moe_gate; u.moe_E = r.Ep; u.moe_I = r.Ip;
+        u.glu_limit = c.expert_limit; u.glu_limit2 = c.ffn_limit; u.glu_from2 = E * r.Ip; u.glu_slope = CLAMPED_GLU_SLOPE;
+        m->site = KS_MOE_UP; m->site_bytes = (2 * touch * m->Hn + (double)M * m->Hn + work) * (double)m->wsize;
+        gemm(m, c.expert_limit > 0.f ? EPI_CLAMP_GLU : EPI_SWIGLU, false, u, 4.0 * work * m->Hn);
+        GemmArgs d = mk(m->moe_hall, r.Ep * r.Ip, w.moe_cat, m->x, m->H, nullptr, 1.f, M, m->H, r.Ep * r.Ip);      // (K slices: plain stores into moe_part)
+        d.moe_gate = m->moe_gate; d.moe_E = r.Ep; d.moe_I = r.Ip; d.sk_part = m->moe_part; d.sk_slices = r.moe_slices;
+        m->site = KS_MOE_DOWN; m->site_bytes = (touch * m->Hn + work) * (double)m->wsize + (double)r.moe_slices * M * m->Hn * 4.0;
+        gemm(m, EPI_RESID, true, d, 2.0 * work * m->Hn);
+        if (!y.y) return {m->moe_part, r.moe_slices, (int64_t)M * m->H};
+        ex = {m->moe_part, r.moe_slices, (int64_t)M * m->H, nullptr, nullptr};
+        return y;
+    }
+    const bool pp = moe_pp_ok(m, r.Ip, false);
+    const int BM = pp ? 256 : ((!m->f32 && g_moe_bm == 256) ? 256 : 128);
+    moe_sort(m, E, k, M, BM);
+    moe_expert_gemms(m, MoeW{E, k, r.Ip, w.moe_up, w.moe_down, c.expert_limit}, M, BM, pp, false);
+    ex = {m->moe_eo, k, 0, m->slot_of, m->expert_w};
+    if (!y.y) {          // no shared expert: nothing but the experts joins
+        y = {m->ly, 1, 0};
+        hipLaunchKernelGGL(fill_i32_kernel, dim3(cdiv((int64_t)M * m->H, 256)), dim3(256), 0, m->stream, (int32_t*)m->ly, 0, M * m->H);
+        NVL_HIP(hipGetLastError());
+    }
+    return y;
+}
+
 // ---- per-layer token input: x (as m->xn) -> m->ly or its K slices ----
 SubOut side_input(nvl_model* m, const MixerW& w, const Meta& md, int li, int M) {
     const int sd = m->cfg.side_dim, kp = m->side_kp;
@@ -1315,10 +1537,26 @@ SubOut side_input(nvl_model* m, const MixerW& w, const Meta& md, int li, int M) 
 // in order: the last sandwich norm then leaves the final norm of every row in m->xn; returns whether it did.
 bool layered_stack(nvl_model* m, const Meta& md, int n_seqs, int M, int max_len, bool have_xn, bool all_rows) {
     auto W = [&](int li) -> const MixerW& { return m->mixers[(size_t)m->runs[(size_t)li].owner]; };
-    const bool post = m->cfg.block_style == NVL_BLOCK_POST;        // sublayers read x itself
+    const bool sum = m->cfg.block_style == NVL_BLOCK_SUM_NORM, post = sum || m->cfg.block_style == NVL_BLOCK_POST;        // post: sublayers read x itself
+    const bool shift = m->cfg.token_shift != 0, ones = max_len == 1;       // ones: token shift in the launch that makes x, else in one of its own
     const bool par = m->cfg.block_style == NVL_BLOCK_PARALLEL;
     m->key_src = m->key_win = -1;
-    if (!have_xn) sandwich(m, SubOut{}, nullptr, {W(0).norm1, W(0).norm1_bias, post}, m->xn, M);
+    auto shift_out = [&](int li) { return shift && ones && li < m->L ? ShiftOut{W(li).shift, m->rec_state + m->runs[(size_t)li].shift_off, &md} : ShiftOut{}; };
+    auto shift_rows = [&](int li) {          // x -> m->xn, the shifted input of layer li's mixer
+        ShiftArgs a{m->x, W(li).shift, m->lshift + (int64_t)li * m->opts.max_seqs * m->H, m->rec_state + m->runs[(size_t)li].shift_off, m->rec_slot_stride,
+                    md.tok_seq, md.tok_pos, md.seq_tok_start, md.seq_len, md.seq_pos, md.seq_slot, M, m->H};
+        KScope ks(m, KC_OTHER, 0, KS_SHIFT, (double)M * m->Hn * (4.0 + (double)m->wsize));
+        if (m->f32) hipLaunchKernelGGL((token_shift_kernel<float>), dim3(M), dim3(256), 0, m->stream, a, (float*)m->xn);
+        else hipLaunchKernelGGL((token_shift_kernel<bf16_t>), dim3(cdiv(M, 16)), dim3(std::min(1024, m->H * 2)), 0, m->stream, a, (bf16_t*)m->xn);
+        NVL_HIP(hipGetLastError());
+    };
+    if (shift && !ones) {
+        KScope ks(m, KC_OTHER, 0, KS_SHIFT);
+        hipLaunchKernelGGL(shift_copy_kernel, dim3(n_seqs, m->L), dim3(256), 0, m->stream, m->rec_state, m->rec_slot_stride, m->shift_offs, md.seq_slot, m->lshift, m->opts.max_seqs, m->H);
+        NVL_HIP(hipGetLastError());
+    }
+    if (!have_xn && shift && !ones) shift_rows(0);
+    else if (!have_xn) sandwich(m, SubOut{}, nullptr, {W(0).norm1, W(0).norm1_bias, post}, m->xn, M, nullptr, {}, shift_out(0));
     for (int li = 0; li < m->L; li++) {
         const LayerRun& r = m->runs[(size_t)li];
         const MixerW& w = W(li);
@@ -1343,22 +1581,23 @@ bool layered_stack(nvl_model* m, const Meta& md, int n_seqs, int M, int max_len,
             continue;
         }
         SubOut y = sub_out(m, KS_OPROJ, m->lmix, w.o, M, r.kd);
+        if (sum || shift) {
+            const bool apart = shift && !ones && li + 1 < m->L, ff = r.c.ffn_dim || r.c.experts;      // apart: the next mixer's input comes from shift_rows
+            const NextNorm own{nullptr, nullptr, true}, close = apart ? NextNorm{nullptr, nullptr, false} : after;
+            sandwich(m, y, w.norm1b, ff ? own : close, m->xn, M, nullptr, {}, ff ? ShiftOut{} : shift_out(li + 1));
+            if (ff) {
+                ExpertOut ex;
+                if (r.c.experts) y = expert_ffn(m, r, w, M, ex);
+                else { glu_up(m, w.w1, M, r.Fp, r.act, r.c.ffn_limit); y = sub_out(m, KS_FFN_DOWN, m->hbuf, w.w2, M, r.Fp); }
+                sandwich(m, y, w.norm2b, close, m->xn, M, nullptr, ex, shift_out(li + 1));
+            }
+            if (apart) shift_rows(li + 1);
+            tap_layer(m, li, M);
+            continue;
+        }
         sandwich(m, y, w.norm1b, r.c.ffn_dim ? NextNorm{w.norm2, nullptr, post} : after, m->xn, M);
         if (r.c.ffn_dim) {
-            m->site = KS_FFN_UP;
-            const bool clamped = m->cfg.activation_type == NVL_ACT_CLAMPED_GLU;
-            if (m->f32) {
-                gemm(m, EPI_STORE, true, mk(m->xn, m->H, w.w1, m->h2, 2 * r.Fp, nullptr, 1.f, M, 2 * r.Fp, m->H));
-                const int64_t n = (int64_t)M * r.Fp;
-                KScope ks(m, KC_OTHER);
-                if (clamped) hipLaunchKernelGGL((clamp_glu_kernel<float>), dim3(cdiv(n, 256)), dim3(256), 0, m->stream, m->h2, (float*)m->hbuf, (int64_t)M, r.Fp, r.c.ffn_limit, CLAMPED_GLU_SLOPE);
-                else hipLaunchKernelGGL((swiglu_kernel<float, true>), dim3(cdiv(n, 256)), dim3(256), 0, m->stream, m->h2, (float*)m->hbuf, (int64_t)M, r.Fp, (int64_t)r.Fp, 0);
-                NVL_HIP(hipGetLastError());
-            } else {
-                GemmArgs up = mk(m->xn, m->H, w.w1, m->hbuf, r.Fp, nullptr, 1.f, M, 2 * r.Fp, m->H);
-                up.glu_limit = r.c.ffn_limit; up.glu_slope = CLAMPED_GLU_SLOPE;
-                gemm(m, clamped ? EPI_CLAMP_GLU : EPI_GEGLU, false, up);
-            }
+            glu_up(m, w.w1, M, r.Fp, m->cfg.activation_type, r.c.ffn_limit);
             y = sub_out(m, KS_FFN_DOWN, m->hbuf, w.w2, M, r.Fp);
             sandwich(m, y, w.norm2b, after, m->xn, M);
         }

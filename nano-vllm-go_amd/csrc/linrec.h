@@ -1,10 +1,11 @@
 // linrec.h — gated linear recurrences with a matrix state per head, in fp32 throughout:
 //     S_t = diag(alpha_t) S_{t-1} + k_t v_t^T        S [DK][DV], alpha_t in (0, 1]
 //     o_t = S_t^T q_t
-// Two designs of the family run on the same kernels:
+// Three designs of the family run on the same kernels:
 //   per-channel decay (gated linear attention): alpha = sigmoid(z)^(1/tau), z = A2 (A1 h) + b per key channel;
 //   one decay per head (Mamba-2, state-space duality): q = C, k = dt B, v = x, alpha = exp(-exp(A_log) dt), o += D x; a group
-//     of heads shares q and k.
+//     of heads shares q and k;
+//   one fixed decay per head (lightning attention): alpha given, dt = 1, D = 0.
 //
 //   linrec_step_kernel   token by token, the state streamed once per token (decode; the convolution of a Mamba-2 decode token,
 //                        and GLA's head norm + output gate, are fused in)
@@ -32,6 +33,7 @@ struct LinRecArgs {
     // one decay per head
     const float* dt; int64_t dt_ld;    // raw step sizes (before bias and softplus), one column per head
     const float *dt_bias, *a_log, *Dskip;
+    const float *decay, *log2_decay;   // not NULL: fixed decays instead, and their base-2 logarithms
     // a decay per key channel
     const float* a1; int64_t a1_ld;    // [token][rank]
     int rank;
@@ -107,7 +109,9 @@ __global__ __launch_bounds__(LR_STEP_THREADS, LR_STEP_ROWS <= 8 ? 4 : 2) void li
     for (int it = 0; it < n; it++) {
         const int64_t t = t0 + it;
         if constexpr (!CH) {
-            if (tid == 0) {
+            if (p.decay) {
+                if (tid == 0) { s_sc[0] = 1.0f; s_sc[1] = p.decay[h]; }
+            } else if (tid == 0) {
                 const float d = lr_softplus(p.dt[t * p.dt_ld + h] + p.dt_bias[h]);
                 s_sc[0] = d;
                 s_sc[1] = expf(-expf(p.a_log[h]) * d);
@@ -186,7 +190,7 @@ __global__ __launch_bounds__(LR_STEP_THREADS, LR_STEP_ROWS <= 8 ? 4 : 2) void li
                 float a = 0.f;
 #pragma unroll 4
                 for (int r = 0; r < NRED; r++) a += red[(int64_t)r * p.DVp + i];
-                if (!CH) a = fmaf(p.Dskip[h], sv[i], a);
+                if (!CH && p.Dskip) a = fmaf(p.Dskip[h], sv[i], a);
                 ov[c] = a;
                 ss = fmaf(a, a, ss);
                 if (!(CH && FUSED)) p.o[t * p.o_ld + (int64_t)h * p.DV + i] = a;
@@ -268,7 +272,7 @@ __global__ __launch_bounds__(NW * 64, NK > 8 ? 1 : (NW == 8 ? 4 : 3)) void linre
         }
     for (int i = tid; i < C * LA; i += NT) As[i] = 0.f;          // (the blocks above the diagonal stay zero)
     float btot = 0.f;                                            // MODE 1: log2 of the decay over all chunks (one channel per thread)
-    const float A = CH ? 0.f : -expf(p.a_log[h]), Dh = CH ? 0.f : p.Dskip[h];
+    const float A = CH ? 0.f : (p.decay ? p.log2_decay[h] : -expf(p.a_log[h])), Dh = CH || !p.Dskip ? 0.f : p.Dskip[h];
     // the next chunk's rows are fetched into registers while the current one is worked on
     constexpr int RQ = NT / (DKP / 4), RV = NT / (DVS / 4), NQ = (C + RQ - 1) / RQ, NV = (C + RV - 1) / RV, NA1 = 2;      // rows per pass, passes
     const int tq = tid / (DKP / 4), dq = tid % (DKP / 4) * 4, tv_ = tid / (DVS / 4), dv_ = tid % (DVS / 4) * 4;
@@ -304,7 +308,7 @@ __global__ __launch_bounds__(NW * 64, NK > 8 ? 1 : (NW == 8 ? 4 : 3)) void linre
                 const int e = tid + i * NT, t = e / p.rank;
                 ra[i] = t < nv ? p.a1[(tb + t) * p.a1_ld + (e - t * p.rank)] : 0.f;      // (t < nv <= 32: inside the chunk)
             }
-        } else if (tid < nv) rdt = p.dt[(tb + tid) * p.dt_ld + h];
+        } else if (!p.decay && tid < nv) rdt = p.dt[(tb + tid) * p.dt_ld + h];
     };
     fetch(c_first);
 
@@ -363,8 +367,8 @@ __global__ __launch_bounds__(NW * 64, NK > 8 ? 1 : (NW == 8 ? 4 : 3)) void linre
                 for (int j = 0; j < TPG; j++) bs[(grp * TPG + j) * LQ + d] = off + pre[j];
             }
         } else if (wave == 0 && lane < 32) {
-            const float dt = lane < nv ? lr_softplus(dt_raw + p.dt_bias[h]) : 0.f;
-            float s = A * dt * LOG2E;
+            const float dt = lane < nv ? (p.decay ? 1.0f : lr_softplus(dt_raw + p.dt_bias[h])) : 0.f;
+            float s = p.decay ? A * dt : A * dt * LOG2E;
 #pragma unroll
             for (int o = 1; o < 32; o <<= 1) { const float v = __shfl_up(s, o, 32); if (lane >= o) s += v; }
             aux[lane] = s; aux[32 + lane] = dt;

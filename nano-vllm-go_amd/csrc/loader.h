@@ -286,7 +286,8 @@ std::vector<float> to_f32(const StTensor& t) {
 struct LayeredArch { const char* name; int block_style, activation; float norm_offset; int norm_type, position_type; };
 const LayeredArch LAYERED_ARCHS[] = {{"Potuzen", NVL_BLOCK_SANDWICH, NVL_ACT_GEGLU, 0.f, NVL_NORM_RMS, NVL_POS_NONE},
                                      {"Lufazen", NVL_BLOCK_POST, NVL_ACT_CLAMPED_GLU, 1.f, NVL_NORM_RMS, NVL_POS_NONE},
-                                     {"Bolinex", NVL_BLOCK_PARALLEL, NVL_ACT_RELU2, 0.f, NVL_NORM_LAYER, NVL_POS_LEARNED}};
+                                     {"Bolinex", NVL_BLOCK_PARALLEL, NVL_ACT_RELU2, 0.f, NVL_NORM_LAYER, NVL_POS_LEARNED},
+                                     {"Medulorn", NVL_BLOCK_SUM_NORM, NVL_ACT_REGLU, 0.f, NVL_NORM_RMS_SCALAR, NVL_POS_NONE}};
 const LayeredArch* layered_arch(const std::string& name) {
     for (const LayeredArch& a : LAYERED_ARCHS) if (name == a.name) return &a;
     return nullptr;
@@ -335,6 +336,71 @@ void parse_experts(const JVal* mlp, nvl_layer_config& c, const std::string& at) 
     if (sh && sh->kind == JVal::OBJ) c.ffn_dim = need_int(sh, "ff", at);
     if (c.experts <= 0 || c.expert_dim <= 0 || c.ffn_dim < 0) throw std::runtime_error(at + "an expert size is not positive");
 }
+// a key mask {size, keep_first} (null: none); returns the size
+int parse_mask(const JVal* mx, int* keep_first, const std::string& at) {
+    const JVal* mask = mx->get("mask");
+    if (!mask || mask->kind != JVal::OBJ) return 0;
+    const int size = need_int(mask, "size", at);
+    if (size <= 0) throw std::runtime_error(at + "the mask's size is not positive");
+    if (keep_first && mask->get("keep_first")) *keep_first = need_int(mask, "keep_first", at);
+    return size;
+}
+// what the two attentions of the design with norms of sums share: sizes, scale, rotation {dims, base, scaling: null | {factor, original, low, high}}
+void parse_plain_attention(const JVal* mx, nvl_layer_config& c, const std::string& at) {
+    c.mixer = NVL_MIXER_ATTENTION;
+    c.heads = need_int(mx, "heads", at); c.kv_heads = need_int(mx, "kv_heads", at); c.dim = need_int(mx, "dim", at); c.vdim = need_int(mx, "vdim", at);
+    c.scale = (float)need_num(mx, "scale", at);
+    c.ungated = 1;
+    const JVal* rot = mx->get("rot");
+    if (!rot || rot->kind != JVal::OBJ) return;
+    c.rot_dim = need_int(rot, "dims", at); c.rot_base = need_num(rot, "base", at);
+    const JVal* sc = rot->get("scaling");
+    if (sc && sc->kind == JVal::OBJ) {
+        c.rot_factor = need_num(sc, "factor", at); c.rot_original = need_num(sc, "original", at);
+        c.rot_low = need_num(sc, "low", at); c.rot_high = need_num(sc, "high", at);
+    }
+}
+// a layer of that design
+nvl_layer_config parse_sum_norm_layer(const std::string& type, const JVal* mx, const JVal* mlp, const std::string& at) {
+    nvl_layer_config c;
+    memset(&c, 0, sizeof c);
+    c.kv_from = c.weights_of = -1;
+    if (type == "attention") {
+        parse_plain_attention(mx, c, at);
+        c.qk_norm = NVL_QK_NORM_HEAD; c.sink = NVL_SINK_ZERO; c.qkv_bias = 1;
+        c.chunk = parse_mask(mx, nullptr, at);
+    } else if (type == "parallel") {
+        const JVal *left = mx->get("left"), *right = mx->get("right");
+        if (!left || left->kind != JVal::OBJ || !right || right->kind != JVal::OBJ) throw std::runtime_error(at + "'left' and 'right' expected");
+        parse_plain_attention(left, c, at);
+        c.qk_norm = NVL_QK_NORM_ROW; c.sink = NVL_SINK_LEARNED;
+        c.window = parse_mask(left, &c.keep_first, at);
+        c.out_scale = (float)need_num(mx, "left_scale", at); c.out_scale2 = (float)need_num(mx, "right_scale", at);
+        c.mixer2 = NVL_MIXER_LIGHTNING;
+        c.heads2 = need_int(right, "heads", at); c.dim2 = need_int(right, "dim", at); c.vdim2 = need_int(right, "vdim", at);
+        const JVal* decay = right->get("decay");
+        if (!decay || decay->kind != JVal::ARR || c.heads2 <= 0 || decay->arr.size() != (size_t)c.heads2) throw std::runtime_error(at + "as many decays as heads expected");
+        if (c.heads2 > NVL_MAX_DECAYS) throw std::runtime_error(at + "too many heads of lightning attention");
+        for (size_t h = 0; h < decay->arr.size(); h++) {
+            if (decay->arr[h].kind != JVal::NUM) throw std::runtime_error(at + "a decay is not a number");
+            c.decay[h] = decay->arr[h].num;
+        }
+    } else throw std::runtime_error(at + "unknown mixer '" + type + "'");
+    if (!mlp || mlp->kind != JVal::OBJ) return c;
+    const JVal* kind = mlp->get("kind");
+    const std::string k = kind && kind->kind == JVal::STR ? kind->str : kind ? "?" : "dense";
+    if (k == "moe") {
+        parse_experts(mlp, c, at);
+        c.expert_limit = (float)need_num(mlp->get("expert"), "limit", at);
+        c.route_softmax = 1;
+        c.ffn_act = 0;
+        if (c.ffn_dim) { c.ffn_act = NVL_ACT_CLAMPED_GLU; c.ffn_limit = (float)need_num(mlp->get("shared"), "limit", at); }
+    } else if (k == "dense") {
+        c.ffn_dim = need_int(mlp, "ff", at);
+        if (c.ffn_dim <= 0) throw std::runtime_error(at + "the feed-forward size is not positive");
+    } else throw std::runtime_error(at + "unknown feed-forward kind");
+    return c;
+}
 std::vector<nvl_layer_config> parse_layers(const JVal& raw, const LayeredArch& arch) {
     const bool post = arch.block_style == NVL_BLOCK_POST, par = arch.block_style == NVL_BLOCK_PARALLEL;
     const JVal* ls = raw.get("layers");
@@ -348,6 +414,7 @@ std::vector<nvl_layer_config> parse_layers(const JVal& raw, const LayeredArch& a
         c.kv_from = -1;
         const JVal *ty = e.get("type"), *mx = e.get("mixer"), *mlp = e.get("mlp"), *wo = e.get("weights_of");
         if (!ty || ty->kind != JVal::STR || !mx || mx->kind != JVal::OBJ) throw std::runtime_error(at + "'type' and 'mixer' expected");
+        if (arch.block_style == NVL_BLOCK_SUM_NORM) { out.push_back(parse_sum_norm_layer(ty->str, mx, mlp, at)); continue; }
         c.weights_of = wo && wo->kind == JVal::NUM ? need_int(&e, "weights_of", at) : -1;
         c.heads = need_int(mx, "heads", at); c.vdim = need_int(mx, "vdim", at);
         if (ty->str == "attention" && par) parse_attention(mx, c, at);
@@ -405,7 +472,7 @@ void load_layered(nvl_model* m, const StSet& st) {
         }
         if (nvl_upload_tensor(m, kind, layer, all.data(), a.dtype, rows, a.shape[1], OI)) throw std::runtime_error(nvl_last_error(m));
     };
-    const bool post = m->cfg.block_style == NVL_BLOCK_POST, par = m->cfg.block_style == NVL_BLOCK_PARALLEL;
+    const bool post = m->cfg.block_style == NVL_BLOCK_POST, par = m->cfg.block_style == NVL_BLOCK_PARALLEL, sum = m->cfg.block_style == NVL_BLOCK_SUM_NORM;
     if (m->cfg.norm_type == NVL_NORM_LAYER) vec(NVL_T_FINAL_NORM_B, 0, "final.norm.b");
     if (m->cfg.position_type == NVL_POS_LEARNED) mat(NVL_T_POS_EMB, 0, "pos");
     if (m->cfg.side_dim) mat(NVL_T_SIDE_EMB, 0, "side.embed");
@@ -420,6 +487,9 @@ void load_layered(nvl_model* m, const StSet& st) {
             vec(NVL_T_ATTN_NORM_W, i, l + "norm1");
             if (m->cfg.norm_type == NVL_NORM_LAYER) vec(NVL_T_ATTN_NORM_B, i, l + "norm1.b");
             if (m->cfg.side_dim) { mat(NVL_T_SIDE_GATE, i, l + "side.gate"); mat(NVL_T_SIDE_PROJ, i, l + "side.proj"); vec(NVL_T_SIDE_NORM, i, l + "side.norm"); }
+        } else if (sum) {
+            vec(NVL_T_MIX_POST_NORM, i, l + "norm1");
+            if (r.c.ffn_dim || r.c.experts) vec(NVL_T_FFN_POST_NORM, i, l + "norm2");
         } else if (post) {
             vec(NVL_T_MIX_POST_NORM, i, l + "norm1"); vec(NVL_T_MIX_SCALE, i, l + "ls1");
             if (r.c.ffn_dim) { vec(NVL_T_FFN_POST_NORM, i, l + "norm2"); vec(NVL_T_FFN_SCALE, i, l + "ls2"); }
@@ -427,6 +497,7 @@ void load_layered(nvl_model* m, const StSet& st) {
             vec(NVL_T_ATTN_NORM_W, i, l + "norm1"); vec(NVL_T_MIX_POST_NORM, i, l + "norm1b");
             if (r.c.ffn_dim) { vec(NVL_T_FFN_NORM_W, i, l + "norm2"); vec(NVL_T_FFN_POST_NORM, i, l + "norm2b"); }
         }
+        if (m->cfg.token_shift) vec(NVL_T_SHIFT, i, l + "shift");
         if (r.c.ffn_dim) {
             const std::string f = l + (r.c.experts ? "mlp.shared." : "mlp.");
             if (r.act == NVL_ACT_RELU2) mat(NVL_T_W1, i, f + "up"); else cat(NVL_T_W1, i, {f + "gate", f + "up"});
@@ -439,7 +510,7 @@ void load_layered(nvl_model* m, const StSet& st) {
                 up.push_back(x + "gate"); up.push_back(x + "up"); down.push_back(x + "down");
             }
             cat(NVL_T_MOE_IN, i, up); cat(NVL_T_MOE_OUT, i, down);
-            mat(NVL_T_ROUTER, i, l + "mlp.router"); vec(NVL_T_ROUTER_BIAS, i, l + "mlp.correction");
+            mat(NVL_T_ROUTER, i, l + "mlp.router"); vec(NVL_T_ROUTER_BIAS, i, l + (r.c.route_softmax ? "mlp.router.b" : "mlp.correction"));
         }
         switch (r.c.mixer) {
             case NVL_MIXER_LATENT_ATTENTION:
@@ -448,11 +519,20 @@ void load_layered(nvl_model* m, const StSet& st) {
                 mat(NVL_T_LAT_UK, i, x + "uk"); mat(NVL_T_LAT_UV, i, x + "uv");
                 mat(NVL_T_MIX_GATE, i, x + "g"); mat(NVL_T_WO, i, x + "o");
                 break;
-            case NVL_MIXER_ATTENTION:
-                mat(NVL_T_WQ, i, x + "q"); mat(NVL_T_WK, i, x + "k"); mat(NVL_T_WV, i, x + "v"); mat(NVL_T_MIX_GATE, i, x + "g"); mat(NVL_T_WO, i, x + "o");
-                vec(NVL_T_BIAS_R1, i, x + "r1"); vec(NVL_T_BIAS_R2, i, x + "r2");
-                if (r.c.v_mix) vec(NVL_T_V_MIX, i, x + "vmix");
+            case NVL_MIXER_ATTENTION: {
+                const std::string a = r.c.mixer2 ? x + "left." : x, b = x + "right.";
+                mat(NVL_T_WQ, i, a + "q"); mat(NVL_T_WK, i, a + "k"); mat(NVL_T_WV, i, a + "v"); mat(NVL_T_WO, i, a + "o");
+                if (r.c.qkv_bias) { vec(NVL_T_BQ, i, a + "q.b"); vec(NVL_T_BK, i, a + "k.b"); vec(NVL_T_BV, i, a + "v.b"); }
+                if (r.c.qk_norm) { vec(NVL_T_Q_NORM, i, a + "q.norm"); vec(NVL_T_K_NORM, i, a + "k.norm"); }
+                if (r.c.sink == NVL_SINK_LEARNED) vec(NVL_T_SINK, i, a + "sink");
+                if (par) { mat(NVL_T_MIX_GATE, i, a + "g"); vec(NVL_T_BIAS_R1, i, a + "r1"); vec(NVL_T_BIAS_R2, i, a + "r2"); }
+                if (r.c.v_mix) vec(NVL_T_V_MIX, i, a + "vmix");
+                if (r.c.mixer2) {
+                    mat(NVL_T_LIN_Q, i, b + "q"); mat(NVL_T_LIN_K, i, b + "k"); mat(NVL_T_LIN_V, i, b + "v"); mat(NVL_T_LIN_GATE, i, b + "g");
+                    vec(NVL_T_LIN_NORM, i, b + "norm"); mat(NVL_T_LIN_O, i, b + "o");
+                }
                 break;
+            }
             case NVL_MIXER_MAMBA2:
                 mat(NVL_T_MAMBA_IN_PROJ, i, x + "in"); vec(NVL_T_MAMBA_CONV_W, i, x + "conv"); vec(NVL_T_MAMBA_CONV_B, i, x + "conv.b");
                 vec(NVL_T_MAMBA_DT_BIAS, i, x + "dt_bias"); vec(NVL_T_MAMBA_A_LOG, i, x + "A_log"); vec(NVL_T_MAMBA_D, i, x + "D");
@@ -639,6 +719,10 @@ extern "C" int nvl_load_config_json(const char* path, nvl_model_config* out) {
             c.activation_type = la->activation; c.block_style = la->block_style; c.norm_weight_offset = la->norm_offset;
             double cap;
             if (num("logit_softcap", cap)) c.logit_softcap = (float)cap;
+            if (la->block_style == NVL_BLOCK_SUM_NORM) {
+                c.stream_scale = (float)need_num(&raw, "postln_alpha", "config: "); c.token_shift = 1;
+                c.embedding_multiplier = (float)need_num(raw.get("embedding"), "scale", "config: embedding: ");
+            }
             *out = c;
             return NVL_OK;
         }

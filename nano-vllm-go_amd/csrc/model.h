@@ -48,7 +48,7 @@ enum KSite { KS_OTHER = 0, KS_QKV, KS_ATTN, KS_OPROJ, KS_FFN_UP, KS_FFN_DOWN, KS
              KS_MOE_UP, KS_MOE_DOWN, KS_MOE_COMBINE, KS_EMBED, KS_ARGMAX, KS_ROPE, KS_MAMBA_IN, KS_MAMBA_CONV, KS_MAMBA_SCAN,
              KS_MAMBA_GATE, KS_MAMBA_OUT, KS_ALLREDUCE, KS_MIX_IN, KS_LAT_NORM, KS_LAT_UQ, KS_LAT_GATHER, KS_LAT_KV, KS_LAT_ABSORB,
              KS_LAT_UV, KS_GLA_SCAN, KS_GLA_GATE, KS_SANDWICH, KS_DELTA_CONV, KS_DELTA_PACK, KS_DELTA_RANK, KS_DELTA_PREP, KS_DELTA_SCAN, KS_DELTA_GATE,
-             KS_KV_PLACE, KS_SIDE_GATE, KS_SIDE_PROJ, KS_COUNT };
+             KS_KV_PLACE, KS_SIDE_GATE, KS_SIDE_PROJ, KS_QK_TURN, KS_LIN_SCAN, KS_LIN_GATE, KS_SHIFT, KS_COUNT };
 
 // one layer of a model described by a list of layers: its configuration, padded sizes, where its tensors and its memory are
 struct LayerRun {
@@ -63,12 +63,17 @@ struct LayerRun {
     int ko = 0;                  // K of the output projection (padded)
     int Fp = 0;                  // feed-forward columns (padded), 0: none
     int conv_dim = 0;
-    int win = -1;                // index into nvl_model::windows
+    int win = -1;                // index into nvl_model::masks
     int64_t cache_off = 0;       // attention: element offset inside a cache block
     int k_off = 0, v_off = 0, ffn_off = 0, route_off = 0;     // grouped attention: columns of the fused input projection (keys, values, feed-forward, router)
     bool ffn_in = false;         // ... whose feed-forward columns are the whole up projection (ungated activations),
     bool glu_in = false;         // or gate and up of a small shared expert, finished by the router's launch
     int mix = 0;                 // grouped attention: GroupedArgs::mix
+    bool raw = false;            // grouped attention: queries and keys are normed or rotated between projection and cache
+    int lq_off = 0, lk_off = 0, lv_off = 0, lg_off = 0;       // lightning attention beside it: columns of the fused input projection
+    int ko2 = 0;                 // ... and its part of the joint output projection's K, behind ko
+    int shared_parts = 0;        // decode: the shared expert as this many experts that every token takes (0: launches of its own)
+    int64_t shift_off = 0;       // token shift: the kept row inside a slot
     int kd = 0;                  // K of the joint output projection of a parallel block: ko, then the feed-forward's Fp columns
     int act = 0;                 // activation of the feed-forward
     int Ep = 0, Ip = 0, moe_slices = 0;          // experts (padded), their padded width, K slices of the decode down projection
@@ -89,6 +94,9 @@ struct MixerW {
     float *norm1_bias = nullptr, *r1 = nullptr, *r2 = nullptr, *v_lambda = nullptr;       // grouped attention, parallel blocks
     void *moe_up = nullptr, *moe_down = nullptr, *moe_cat = nullptr;                      // experts: [E][2 Ip][H], [E][H][Ip], bf16: [H][Ep Ip]
     float* route_bias = nullptr;
+    void* router = nullptr;                  // where it is no part of the input projection
+    float *in_bias = nullptr, *q_norm = nullptr, *k_norm = nullptr, *sink = nullptr, *shift = nullptr;
+    float *lin_norm = nullptr, *decay = nullptr, *log2_decay = nullptr;      // lightning attention
     void *side_gate = nullptr, *side_proj = nullptr; float* side_norm = nullptr;
 };
 
@@ -169,11 +177,12 @@ struct nvl_model {
     std::vector<nvl::MixerW> mixers;
     std::vector<void*> layered_allocs;
     float *final_norm = nullptr, *final_norm_b = nullptr;
-    nvl::bf16_t* lqg = nullptr;          // grouped attention, bf16: [token][queries | gates] (fragment-major)
+    void* lqg = nullptr;                 // grouped attention, bf16: [token][queries | gates] (fragment-major); fp32 mode: normed and rotated queries
+    float* lshift = nullptr; int64_t* shift_offs = nullptr;         // token shift: the kept rows a pass began with, where each layer's lies in a slot
     float* lvf = nullptr; int64_t lvf_ld = 0;                       // grouped attention: the first mixing layer's values of the running batch
     void *side_emb = nullptr, *lside = nullptr; int64_t side_ld = 0; int side_kp = 0;     // per-layer token inputs: table (rows of L * side4 entries), operand of the projection
     float* grp_part = nullptr; int32_t* grp_cnt = nullptr; int64_t grp_cap = 0;           // grouped attention: key splits
-    std::vector<int> windows;    // distinct windows of the latent attention layers (0: none)
+    std::vector<nvl::KeyMask> masks;    // distinct key masks of the attention layers
     void* lat_cache = nullptr; int64_t lat_block_stride = 0;
     float* rec_state = nullptr; int64_t rec_slot_stride = 0;
     float *lproj = nullptr, *lq = nullptr, *ly = nullptr, *lconv = nullptr, *lo = nullptr;

@@ -23,6 +23,8 @@ static int g_sk_tile = 1;            // nvl_set_tuning key 26: that split (0 = o
 constexpr int MOE_DOWN_SLICES = 4;    // at most this many K slices (workgroups per column tile) in the dense-masked MoE down projection
 static inline int moe_down_slices(int E) { int s = MOE_DOWN_SLICES; while (s > 1 && E % s) s--; return s; }   // a whole number of experts per slice
 
+constexpr float CLAMPED_GLU_SLOPE = 1.702f;
+
 namespace {
 
 int fail(nvl_model* m, int code, const std::string& msg) {
@@ -198,6 +200,8 @@ void gemm(nvl_model* m, int epi, bool out_f32, GemmArgs a, double flops = -1.0) 
             case EPI_GROUPED: launch_gemm_bf16<EPI_GROUPED, bf16_t>(st, a); break;
             case EPI_RELU2:  launch_gemm_bf16<EPI_RELU2, bf16_t>(st, a); break;
             case EPI_GELU_TOK: launch_gemm_bf16<EPI_GELU_TOK, bf16_t>(st, a); break;
+            case EPI_REGLU: launch_gemm_bf16<EPI_REGLU, bf16_t>(st, a); break;
+            case EPI_GROUPED_RAW: launch_gemm_bf16<EPI_GROUPED_RAW, bf16_t>(st, a); break;
             default: throw std::runtime_error("gemm: bad epilogue");
         }
     }
@@ -674,7 +678,7 @@ void init_slots(nvl_model* m) {
 // per-call metadata: see bind_meta
 void init_meta(nvl_model* m) {
     const int64_t Mmax = m->opts.max_batch_tokens, S = m->opts.max_seqs;
-    m->meta_ints = 5 * Mmax + (5 + (int64_t)m->windows.size()) * S + m->table_cap + 2 * (m->layered ? Mmax : 0) + 16;
+    m->meta_ints = 5 * Mmax + (5 + (int64_t)m->masks.size()) * S + m->table_cap + 2 * (m->layered ? Mmax : 0) + 16;
     NVL_HIP(hipHostMalloc((void**)&m->meta_host, (size_t)m->meta_ints * 4, hipHostMallocDefault));
     m->meta_dev = dmalloc<int32_t>(m->meta_ints);
     NVL_HIP(hipHostMalloc((void**)&m->am_host, (size_t)std::max<int64_t>(S, Mmax) * 4, hipHostMallocDefault));
@@ -1062,15 +1066,18 @@ bool pool_reserve(nvl_model* m, int slot, int64_t end, bool evict) {
     }
     return true;
 }
-// after a slot's sequence has grown to slot_len tokens: when every attention layer has a window, the blocks that lie before the
-// earliest key the next token can see go back to the pool
+// after a slot's sequence has grown to slot_len tokens: when every attention layer has a window or chunks, the blocks that lie before the
+// earliest key the next token can see, and hold no kept first tokens, go back to the pool
 void pool_trim(nvl_model* m, int slot) {
-    if (!m->pool || m->windows.empty()) return;
-    int w = 0;
-    for (int x : m->windows) { if (x == 0) return; w = std::max(w, x); }
+    if (!m->pool || m->masks.empty()) return;
+    int64_t first = m->slot_len[(size_t)slot], keep = 0;
+    for (const KeyMask& x : m->masks) {
+        if (x.span() == 0) return;
+        first = std::min<int64_t>(first, x.lo(m->slot_len[(size_t)slot]));
+        keep = std::max<int64_t>(keep, x.keep);
+    }
     auto& b = m->slot_blocks[(size_t)slot];
-    const int64_t first = (int64_t)m->slot_len[(size_t)slot] - w + 1;
-    for (int64_t i = 0; i < (int64_t)b.size() && (i + 1) * m->Tmax <= first; i++)
+    for (int64_t i = keep == 0 ? 0 : cdiv(keep, m->Tmax); i < (int64_t)b.size() && (i + 1) * m->Tmax <= first; i++)
         if (b[(size_t)i] >= 0) { m->free_blocks.push_back(b[(size_t)i]); b[(size_t)i] = -1; }
 }
 int seq_open_impl(nvl_model* m, int64_t seq_id, bool evict) {
@@ -1139,20 +1146,20 @@ struct Meta {   // device pointers into meta_dev
     int32_t *tokens, *tok_pos, *tok_tbl, *tok_seq, *seq_tok_start, *seq_len, *seq_pos, *seq_tbl, *seq_slot, *last_rows, *blk_table, *kbase, *abs_tok, *abs_seq;
 };
 // layout of meta_host / meta_dev for a call carrying M tokens:
-//   [seq_tok_start S | seq_len S | seq_pos S | seq_tbl S | seq_slot S | kbase windows x S | blk_table table_cap |
+//   [seq_tok_start S | seq_len S | seq_pos S | seq_tbl S | seq_slot S | kbase masks x S | blk_table table_cap |
 //    tokens M | tok_pos M | tok_tbl M | tok_seq M | last_rows M (the rows whose logits are wanted) | (layered) abs_tok M | abs_seq M]
 // (blk_table: sequence i's blocks start at i * blocks_per_seq; slab mode: one entry, its slot)
 Meta bind_meta(const nvl_model* m, int32_t* base, int M) {
     const int64_t S = m->opts.max_seqs;
     Meta md;
     md.seq_tok_start = base; md.seq_len = base + S; md.seq_pos = base + 2 * S; md.seq_tbl = base + 3 * S; md.seq_slot = base + 4 * S;
-    md.kbase = base + 5 * S; md.blk_table = md.kbase + (int64_t)m->windows.size() * S;
+    md.kbase = base + 5 * S; md.blk_table = md.kbase + (int64_t)m->masks.size() * S;
     md.tokens = md.blk_table + m->table_cap; md.tok_pos = md.tokens + M; md.tok_tbl = md.tok_pos + M; md.tok_seq = md.tok_tbl + M;
     md.last_rows = md.tok_seq + M; md.abs_tok = md.last_rows + M; md.abs_seq = md.abs_tok + M;
     return md;
 }
 size_t meta_bytes(const nvl_model* m, int M) {
-    return (size_t)((5 + (int64_t)m->windows.size()) * (int64_t)m->opts.max_seqs + m->table_cap + (m->layered ? 7 : 5) * (int64_t)M) * 4;
+    return (size_t)((5 + (int64_t)m->masks.size()) * (int64_t)m->opts.max_seqs + m->table_cap + (m->layered ? 7 : 5) * (int64_t)M) * 4;
 }
 // sequence i of the batch being assembled lives in `slot`: its table row, table start and slot
 void bind_slot(const nvl_model* m, const Meta& hm, int i, int slot) {
@@ -1529,7 +1536,7 @@ void ffn_up(nvl_model* m, const LayerW& l, int M, bool deferred_norm = false) {
 // (m-tiles mapped to (expert, row segment) by a device table; token rows gathered by per-lane source address)
 // -> combine in rank order into x (with the residual multiplier).  The fp32 parity mode launches per expert.
 // one layer's experts: E SwiGLU feed-forwards of width I, top k of them per token; [E][2I][H] and [E][H][I] in the kernels' layouts
-struct MoeW { int E, k, I; const void *up, *down; };
+struct MoeW { int E, k, I; const void *up, *down; float limit = 0.f; };      // limit > 0: clamped GLU instead of SwiGLU
 // prefill default: 256-row m-tiles on the ping-pong kernel (needs the rows copied into expert order and K >= 160)
 bool moe_pp_ok(const nvl_model* m, int I, bool small) {
     return !m->f32 && !small && g_moe_bm == 0 && m->moe_xg && g_moe_gather && m->H >= 160 && I >= 160 && (2 * I) % 256 == 0 && m->H % 256 == 0;
@@ -1561,7 +1568,8 @@ void moe_expert_gemms(nvl_model* m, const MoeW& w, int M, int BM, bool pp, bool 
         {
             KScope ks(m, KC_OTHER);
             const int64_t n = (int64_t)pairs * I;
-            hipLaunchKernelGGL((swiglu_kernel<float>), dim3(cdiv(n, 256)), dim3(256), 0, m->stream, m->h2, (float*)m->hbuf,
+            if (w.limit > 0.f) hipLaunchKernelGGL((clamp_glu_kernel<float>), dim3(cdiv(n, 256)), dim3(256), 0, m->stream, m->h2, (float*)m->hbuf, (int64_t)pairs, I, w.limit, CLAMPED_GLU_SLOPE);
+            else hipLaunchKernelGGL((swiglu_kernel<float>), dim3(cdiv(n, 256)), dim3(256), 0, m->stream, m->h2, (float*)m->hbuf,
                                (int64_t)pairs, I, (int64_t)I, 0);
             NVL_HIP(hipGetLastError());
         }
@@ -1587,7 +1595,8 @@ void moe_expert_gemms(nvl_model* m, const MoeW& w, int M, int BM, bool pp, bool 
     }
     a.w_expert_stride = (int64_t)2 * I * H; a.grp_bm = pp ? 512 : BM; a.grp_deep = small && g_moe_deep;
     m->site = KS_MOE_UP; m->site_bytes = (e_touch * 2 * I * H + (double)pairs * H + (double)pairs * I) * (double)m->wsize;
-    gemm(m, EPI_SWIGLU, false, a, 2.0 * pairs * 2 * I * H);
+    a.glu_limit = w.limit; a.glu_slope = CLAMPED_GLU_SLOPE;
+    gemm(m, w.limit > 0.f ? EPI_CLAMP_GLU : EPI_SWIGLU, false, a, 2.0 * pairs * 2 * I * H);
     GemmArgs d = mk(m->hbuf, I, w.down, m->moe_eo, H, nullptr, 1.f, max_mtiles, H, I);
     d.tile_map = m->moe_tile_map; d.n_mtiles = m->moe_n_mtiles; d.w_expert_stride = (int64_t)H * I; d.grp_bm = pp ? 512 : BM; d.grp_deep = small && g_moe_deep;
     m->site = KS_MOE_DOWN; m->site_bytes = (e_touch * H * I + (double)pairs * I) * (double)m->wsize + (double)pairs * H * 4.0;
@@ -1618,7 +1627,7 @@ bool moe(nvl_model* m, const LayerW& l, int M, bool deferred_norm = false, const
         if (deferred_norm) set_deferred_in(m, ar);
         if (fused_route) {
             KScope ks(m, KC_GEMM, 2.0 * (double)M * E * H, -1, ((double)E * H + (double)M * H) * (double)m->wsize + (double)M * E * 8.0);
-            hipLaunchKernelGGL(moe_router_gate_kernel, dim3(cdiv(M, 16)), dim3(1024), 0, m->stream, ar, k, m->moe_gate, m->router_logits, 128);
+            hipLaunchKernelGGL(moe_router_gate_kernel, dim3(cdiv(M, 16)), dim3(1024), 0, m->stream, ar, k, m->moe_gate, m->router_logits, 128, E, 0);
             NVL_HIP(hipGetLastError());
         } else {
             gemm(m, EPI_STORE, true, ar);
@@ -2374,7 +2383,9 @@ void decode_loop(nvl_model* m, const Meta& hm, int n_seqs, int n_steps, int32_t*
                                (int64_t)m->cfg.max_seq_len, m->samp_hist_len, m->argmax_dev, m->ring, (const int32_t*)m->ring_pos0, n_seqs,
                                md.tokens, md.tok_pos,
                                md.seq_pos, (const bf16_t*)m->g[NVL_T_TOK_EMB].p, (const bf16_t*)pe, pe_rows,
-                               m->cfg.embedding_multiplier, m->x, norm0, bias0, m->cfg.norm_eps, (bf16_t*)m->xn, m->H, m->Hn);
+                               m->cfg.embedding_multiplier, m->x, norm0, bias0, m->cfg.norm_eps, (bf16_t*)m->xn, m->H, m->Hn,
+                               m->cfg.token_shift ? SeamShift{m->mixers[(size_t)m->runs[0].owner].shift, m->rec_state + m->runs[0].shift_off, m->rec_slot_stride, md.seq_slot}
+                                                  : SeamShift{});
         } else {
             hipLaunchKernelGGL(advance_decode_kernel, dim3(cdiv(n_seqs, 256)), dim3(256), 0, m->stream, m->argmax_dev, md.tokens,
                                md.tok_pos, md.seq_pos, m->ring + (int64_t)s * n_seqs, n_seqs);
@@ -2739,7 +2750,7 @@ static const char* const k_site_names[KS_COUNT] = {
     "moe_down", "moe_combine", "embed", "argmax", "rope_kv", "mamba_in_proj", "mamba_conv", "mamba_scan", "mamba_gate_norm",
     "mamba_out_proj", "tp_allreduce", "mix_in_proj", "latent_norm", "latent_uq", "latent_gather", "latent_kv", "latent_absorb_q",
     "latent_uv", "gla_scan", "gla_gate_norm", "sandwich_norm", "delta_conv", "delta_pack", "delta_rank_out", "delta_prep", "delta_scan", "delta_gate_norm",
-    "kv_place", "side_gate", "side_proj"};
+    "kv_place", "side_gate", "side_proj", "qk_norm_rope", "lightning_scan", "lightning_gate_norm", "token_shift"};
 extern "C" const char* nvl_kernel_site_name(int site) { return site >= 0 && site < KS_COUNT ? k_site_names[site] : ""; }
 extern "C" int nvl_get_kernel_stats(nvl_model* m, nvl_kernel_stat* out, int cap) {
     if (!m || (cap > 0 && !out)) return NVL_ERR_INVALID;

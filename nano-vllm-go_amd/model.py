@@ -13,7 +13,7 @@ from . import _lib as L
 def _cfg_struct(cfg: dict) -> L.ModelConfigC:
     c = L.ModelConfigC()
     for k in ("vocab_size", "hidden", "num_layers", "num_heads", "num_kv_heads", "head_dim", "ffn_dim",
-              "max_seq_len", "num_experts", "num_experts_per_tok", "side_dim"):
+              "max_seq_len", "num_experts", "num_experts_per_tok", "side_dim", "token_shift"):
         setattr(c, k, int(cfg.get(k, 0)))
     c.attention_type = L.ATTN[cfg["attention_type"]]
     c.norm_type = L.NORM[cfg["norm_type"]]
@@ -24,7 +24,7 @@ def _cfg_struct(cfg: dict) -> L.ModelConfigC:
     c.norm_eps = float(cfg.get("norm_eps", 1e-5))
     c.tied_embedding = int(bool(cfg.get("tied_embedding", False)))
     c.use_moe = int(bool(cfg.get("use_moe", False)))
-    for k in ("embedding_multiplier", "attention_multiplier", "residual_multiplier", "logits_scaling", "norm_weight_offset", "logit_softcap"):
+    for k in ("embedding_multiplier", "attention_multiplier", "residual_multiplier", "logits_scaling", "norm_weight_offset", "logit_softcap", "stream_scale"):
         setattr(c, k, float(cfg.get(k, 0.0)))
     for k in ("mamba_expand", "mamba_state_size", "mamba_num_heads", "mamba_head_dim", "mamba_n_groups", "mamba_conv_kernel"):
         setattr(c, k, int(cfg.get(k, 0)))
@@ -39,8 +39,19 @@ def _layer_structs(layers: list):
     arr = (L.LayerConfigC * len(layers))()
     for c, ly in zip(arr, layers):
         for k, v in ly.items():
-            setattr(c, k, L.MIXER[v] if k == "mixer" else v)
+            if k == "decay":
+                if len(v) > L.MAX_DECAYS:
+                    raise ValueError(f"more than {L.MAX_DECAYS} decays")
+                c.decay[:len(v)] = v
+            else:
+                setattr(c, k, L.MIXER[v] if k == "mixer" else v)
     return arr
+
+
+def _layer_dict(c) -> dict:
+    """nvl_layer_config -> a config.LAYER_FIELDS dict."""
+    names = {v: k for k, v in L.MIXER.items()}
+    return {k: names[c.mixer] if k == "mixer" else list(c.decay[:c.heads2]) if k == "decay" else getattr(c, k) for k, _ in c._fields_}
 
 
 def _ptr(a):
@@ -109,8 +120,7 @@ class HipTransformerModel:
         if n:
             arr = (L.LayerConfigC * n)()
             L.check(L.lib().nvl_load_layers_json(cp.encode(), arr, n))
-            names = {v: k for k, v in L.MIXER.items()}
-            cfg["layers"] = [{k: names[getattr(a, k)] if k == "mixer" else getattr(a, k) for k, _ in a._fields_} for a in arr]
+            cfg["layers"] = [_layer_dict(a) for a in arr]
         if max_seq_len is not None:      # (a list of layers with learned positions: as far as those reach)
             cfg["max_seq_len"] = min(int(max_seq_len), cfg["max_seq_len"]) if n and cfg["position_type"] == "learned" else int(max_seq_len)
         m = cls(cfg, None, **kw)
