@@ -38,7 +38,7 @@ def parse():
     ap.add_argument("--gpus", type=int, default=1)
     ap.add_argument("--steps", type=int, default=3)
     ap.add_argument("--warmup", type=int, default=1)
-    ap.add_argument("--model", default="llama-3.2-1b", help="a synth.FULL_CONFIGS key; bolinex-2k / -4k, lufazen-2k / -4k and potuzen-2k / -4k are those designs at a real "
+    ap.add_argument("--model", default="llama-3.2-1b", help="a synth.FULL_CONFIGS key; medulorn-2k / -4k, bolinex-2k / -4k, lufazen-2k / -4k and potuzen-2k / -4k are those designs at a real "
                     "model's layer sizes, hybrid-2k / hybrid-4k the attention + Mamba-2 family at the same sizes, gqa[-moe]-2k / -4k the grouped-query attention families")
     ap.add_argument("--batch", type=int, default=32, help="sequences per GPU")
     ap.add_argument("--prompt", type=int, default=512, help="prompt tokens per sequence")
@@ -347,7 +347,7 @@ def main():
         kv_bytes *= 1 - n_m / cfg["num_layers"]
         kv_bytes += n_m * B * 8.0 * cfg["mamba_expand"] * cfg["hidden"] * cfg["mamba_state_size"]
     if cfg.get("layers"):             # cached latents (keys and values) once, fp32 states read and written
-        kv_bytes = sum(B * (2.0 * c["kv_heads"] * (c["dim"] + c["vdim"]) * min(c["window"] or 1 << 30, S + G / 2) if c["mixer"] == "attention" else 2.0 * c["kv_rank"] * min(c["window"] or 1 << 30, S + G / 2) if c["mixer"] == "latent_attention" else
+        kv_bytes = sum(B * (2.0 * c["kv_heads"] * (c["dim"] + c["vdim"]) * min(c["window"] or c["chunk"] or 1 << 30, S + G / 2) + 8.0 * c["heads2"] * c["vdim2"] * c["dim2"] if c["mixer"] == "attention" else 2.0 * c["kv_rank"] * min(c["window"] or 1 << 30, S + G / 2) if c["mixer"] == "latent_attention" else
                             8.0 * c["heads"] * c["vdim"] * (c["state"] or c["dim"])) for c in cfg["layers"])
     dec_gbs = (wbytes + kv_bytes) * G * args.steps / dec_s / 1e9
 

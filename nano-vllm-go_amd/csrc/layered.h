@@ -624,8 +624,8 @@ void layered_finalize(nvl_model* m) {
                     w.lin_norm = lay_vector(m, T(NVL_T_LIN_NORM, "lightning norm"), hv);
                     lay_scale(m, w.lin_norm, c.out_scale2, hv);
                     lay_place(m, T(NVL_T_LIN_O, "lightning output projection"), w.o, r.kd, 0, 0, 0, 0, 0, 0, -1, false, false, r.ko);
-                    std::vector<float> d((size_t)c.heads2 * 2);       // decays, then their logarithms (a decay of zero: finite, and far below every sum)
-                    for (int h = 0; h < c.heads2; h++) { d[(size_t)h] = (float)c.decay[h]; d[(size_t)(c.heads2 + h)] = (float)std::max(std::log2(c.decay[h]), -1e30); }
+                    std::vector<float> d((size_t)c.heads2 * 2);       // decays, then their logarithms (finite, and 2^-300 is zero)
+                    for (int h = 0; h < c.heads2; h++) { d[(size_t)h] = (float)c.decay[h]; d[(size_t)(c.heads2 + h)] = (float)std::max(std::log2(c.decay[h]), -300.0); }
                     w.decay = (float*)lay_alloc(m, (int64_t)d.size() * 4); w.log2_decay = w.decay + c.heads2;
                     NVL_HIP(hipMemcpyAsync(w.decay, d.data(), d.size() * 4, hipMemcpyHostToDevice, m->stream));
                     NVL_HIP(hipStreamSynchronize(m->stream));

@@ -142,7 +142,9 @@ def layered_shapes(cfg: dict, decay_rank: int = 16) -> list:
     H, V, post, par, side = cfg["hidden"], cfg["vocab_size"], cfg["block_style"] == "post", cfg["block_style"] == "parallel", cfg.get("side_dim", 0)
     ln = cfg["norm_type"] == "layernorm"
     norm = "norm0" if cfg.get("norm_weight_offset") else "norm"
-    out = [("tok_emb", 0, (V, H), "matrix"), ("lm_head", 0, (V, H), "matrix"), ("final_norm_w", 0, (H,), norm)]
+    sums = cfg["block_style"] == "sum_norm"
+    n1 = 1 if cfg["norm_type"] == "rmsnorm_scalar" else H       # a norm's weights
+    out = [("tok_emb", 0, (V, H), "matrix"), ("lm_head", 0, (V, H), "matrix"), ("final_norm_w", 0, (n1,), norm)]
     if ln:
         out.append(("final_norm_b", 0, (H,), "bias"))
     if cfg["position_type"] == "learned":
@@ -153,9 +155,10 @@ def layered_shapes(cfg: dict, decay_rank: int = 16) -> list:
         if c["weights_of"] >= 0:
             continue
         h, d, dv = c["heads"], c["dim"], c["vdim"]
-        t = [("mix_scale", (H,), "norm")] if post else [("attn_norm_w", (H,), norm)]
+        t = [("mix_scale", (H,), "norm")] if post else [] if sums else [("attn_norm_w", (n1,), norm)]
+        t += [("shift", (H,), "decay")] if cfg.get("token_shift") else []
         t += [("attn_norm_b", (H,), "bias")] if ln else []
-        t += [] if par else [("mix_post_norm", (H,), norm)]
+        t += [] if par else [("mix_post_norm", (n1,), norm)]
         t += [("side_gate", (side, H), "matrix"), ("side_proj", (H, side), "matrix"), ("side_norm", (H,), "norm")] if side else []
         if c["mixer"] == "latent_attention":
             qr, kr, rot = c["q_rank"], c["kv_rank"], c["rot_dim"]
@@ -165,8 +168,18 @@ def layered_shapes(cfg: dict, decay_rank: int = 16) -> list:
                 t += [("lat_dkv", (kr + rot, H), "matrix"), ("lat_dkv_norm", (kr,), "norm")]
         elif c["mixer"] == "attention":
             g = c["kv_heads"]
-            t += [("wq", (h * d, H), "matrix"), ("wk", (g * d, H), "matrix"), ("wv", (g * dv, H), "matrix"), ("mix_gate", (h * dv, H), "matrix"),
-                  ("wo", (H, h * dv), "matrix"), ("bias_r1", (h,), "norm"), ("bias_r2", (h,), "decay")] + ([("v_mix", (1,), "decay")] if c["v_mix"] else [])
+            t += [("wq", (h * d, H), "matrix"), ("wk", (g * d, H), "matrix"), ("wv", (g * dv, H), "matrix"), ("wo", (H, h * dv), "matrix")]
+            t += [] if c["ungated"] else [("mix_gate", (h * dv, H), "matrix")]
+            t += [("bias_r1", (h,), "norm"), ("bias_r2", (h,), "decay")] if par else []
+            t += [("v_mix", (1,), "decay")] if c["v_mix"] else []
+            t += [("bq", (h * d,), "bias"), ("bk", (g * d,), "bias"), ("bv", (g * dv,), "bias")] if c["qkv_bias"] else []
+            if c["qk_norm"]:
+                t += [("q_norm", (d if c["qk_norm"] == 1 else h * d,), "norm"), ("k_norm", (d if c["qk_norm"] == 1 else g * d,), "norm")]
+            t += [("sink", (h,), "bias")] if c["sink"] == 2 else []
+            if c["mixer2"]:
+                qk2, v2 = c["heads2"] * c["dim2"], c["heads2"] * c["vdim2"]
+                t += [("lin_q", (qk2, H), "matrix"), ("lin_k", (qk2, H), "matrix"), ("lin_v", (v2, H), "matrix"), ("lin_gate", (v2, H), "matrix"),
+                      ("lin_norm", (v2,), "norm"), ("lin_o", (H, v2), "matrix")]
         elif c["mixer"] == "channel_delta":
             qk, r = c["kv_heads"] * d, c["decay_rank"] or decay_rank
             t += [("wq", (qk, H), "matrix"), ("wk", (qk, H), "matrix"), ("wv", (h * dv, H), "matrix"), ("wo", (H, h * dv), "matrix"),
@@ -185,13 +198,16 @@ def layered_shapes(cfg: dict, decay_rank: int = 16) -> list:
         if c["experts"]:
             E, I = c["experts"], c["expert_dim"]
             t += [("router", (E, H), "matrix"), ("router_bias", (E,), "bias"), ("moe_in", (E * 2 * I, H), "matrix"), ("moe_out", (E * H, I), "matrix")]
-        if c["ffn_dim"] and par:
+        if sums and (c["ffn_dim"] or c["experts"]):
+            t.append(("ffn_post_norm", (n1,), norm))
+            t += [("w1", (2 * c["ffn_dim"], H), "matrix"), ("w2", (H, c["ffn_dim"]), "matrix")] if c["ffn_dim"] else []
+        elif c["ffn_dim"] and par:
             F, gated = c["ffn_dim"], c["ffn_act"] != 0 or cfg["activation_type"] != "relu2"      # (a layer's own activation here: SwiGLU)
             t += [("w1", ((2 if gated else 1) * F, H), "matrix"), ("w2", (H, F), "matrix")]
         elif c["ffn_dim"]:
             F = c["ffn_dim"]
-            t += [("ffn_scale", (H,), "norm")] if post else [("ffn_norm_w", (H,), norm)]
-            t += [("ffn_post_norm", (H,), norm), ("w1", (2 * F, H), "matrix"), ("w2", (H, F), "matrix")]
+            t += [("ffn_scale", (H,), "norm")] if post else [("ffn_norm_w", (n1,), norm)]
+            t += [("ffn_post_norm", (n1,), norm), ("w1", (2 * F, H), "matrix"), ("w2", (H, F), "matrix")]
         out += [(slot, i, shape, kind) for slot, shape, kind in t]
     return out
 
@@ -231,6 +247,21 @@ def _bolinex(width: int, layers: int, heads: int, ff: int, expert_ff: int, windo
     return dict(vocab_size=32000, hidden=width, num_layers=layers, num_heads=0, num_kv_heads=0, head_dim=0, ffn_dim=0, max_seq_len=4096,
                 attention_type="gqa", norm_type="layernorm", position_type="learned", activation_type="relu2", block_style="parallel",
                 rope_base=0.0, norm_eps=1e-6, tied_embedding=False, side_dim=256, layers=[dict(LAYER_FIELDS, **att, **kinds[i % 2]) for i in range(layers)])
+
+
+def _medulorn(width: int, layers: int, heads: int, ff: int, expert_ff: int, window: int = 1024) -> dict:
+    """A Medulorn model at a real model's layer sizes: chunked attention with dense feed-forwards, and windowed beside lightning attention with
+    experts, in turn."""
+    from .config import ACT_CLAMPED_GLU, LAYER_FIELDS, MIXER_LIGHTNING, QK_NORM_HEAD, QK_NORM_ROW, SINK_LEARNED, SINK_ZERO
+    att = dict(mixer="attention", heads=heads, kv_heads=heads // 4, dim=128, vdim=128, scale=128 ** -0.5, ungated=1, rot_dim=128, rot_base=5e5)
+    kinds = [dict(att, chunk=window, qk_norm=QK_NORM_HEAD, sink=SINK_ZERO, qkv_bias=1, ffn_dim=ff),
+             dict(att, window=window, keep_first=4, qk_norm=QK_NORM_ROW, sink=SINK_LEARNED, rot_factor=4.0, rot_low=1.0, rot_high=4.0, rot_original=2048.0, out_scale=1.2,
+                  mixer2=MIXER_LIGHTNING, heads2=heads, dim2=128, vdim2=128, out_scale2=0.5, decay=[1.0 - 0.5 ** (1.0 + 7.0 * h / heads) for h in range(heads)],
+                  ffn_dim=expert_ff, ffn_act=ACT_CLAMPED_GLU, ffn_limit=7.0, experts=32, top_k=8, expert_dim=expert_ff, expert_groups=1, groups_kept=1, route_softmax=1, expert_limit=7.0)]
+    return dict(vocab_size=32000, hidden=width, num_layers=layers, num_heads=0, num_kv_heads=0, head_dim=0, ffn_dim=0, max_seq_len=4096,
+                attention_type="gqa", norm_type="rmsnorm_scalar", position_type="nope", activation_type="reglu", block_style="sum_norm",
+                rope_base=0.0, norm_eps=1e-6, tied_embedding=False, embedding_multiplier=width ** 0.5, stream_scale=3.0, token_shift=1, logit_softcap=30.0,
+                layers=[dict(LAYER_FIELDS, **kinds[i % 2]) for i in range(layers)])
 
 
 def _gqa(hidden: int, layers: int, heads: int, ff: int, experts: bool = False) -> dict:
@@ -274,6 +305,7 @@ FULL_CONFIGS = {
                        position_type="rope", activation_type="swiglu", block_style="sequential",
                        rope_base=500000.0, norm_eps=1e-5, tied_embedding=False),
     # designs described by a list of layers at a real model's layer sizes, and the closest other family at the same sizes
+    "medulorn-2k": _medulorn(2048, 12, 16, 6144, 512), "medulorn-4k": _medulorn(4096, 6, 32, 12288, 1024),
     "bolinex-2k": _bolinex(2048, 12, 16, 6144, 512), "bolinex-4k": _bolinex(4096, 6, 32, 12288, 1024),
     "gqa-2k": _gqa(2048, 12, 16, 6144), "gqa-moe-2k": _gqa(2048, 12, 16, 512, True), "gqa-4k": _gqa(4096, 6, 32, 12288), "gqa-moe-4k": _gqa(4096, 6, 32, 1024, True),
     "lufazen-2k": _lufazen(2048, 12, 16, 768, 6144), "lufazen-4k": _lufazen(4096, 6, 32, 1536, 12288),

@@ -9,6 +9,16 @@ import potuzen_models as PM
 TOL = {"f32": 1e-4, "bf16": 0.12}       # at any position: rms over the vocabulary of the difference / rms of the logits
 
 
+def same_fields(L, got, want):
+    """An nvl_layer_config of the library's reader against the fields the package's reader made."""
+    for k, _ in got._fields_:
+        g = getattr(got, k)
+        if k == "decay":
+            assert np.allclose(list(g), list(want[k]) + [0.0] * (L.MAX_DECAYS - len(want[k])), rtol=0, atol=1e-15), k
+        else:
+            assert (g == L.MIXER[want[k]]) if k == "mixer" else abs(g - want[k]) < 1e-6, (k, g, want[k])
+
+
 def build(gpu, d, cfg, w, precision="f32", **kw):
     PM.write(d, cfg, w)
     kw = dict(dict(max_seq_len=1024, max_seqs=4, max_batch_tokens=1024, kv_num_blocks=64, kv_block_size=64, kv_pool=True), **kw)

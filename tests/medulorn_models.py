@@ -88,14 +88,14 @@ def weights(cfg, seed=0, sink=(0.0, 1.5), shift=(-0.2, 0.9)):
         E = mlp["router"]["experts"]
         for e in range(E):
             glu(f + f"e{e}.", mlp["expert"]["ff"])
-        mat(f + "router", E, W, 1.5)
-        vec(f + "router.b", E, 0.0, 0.7)
+        mat(f + "router", E, W, 0.7)
+        vec(f + "router.b", E, 0.0, 1.5)
         if mlp["shared"] is not None:
             glu(f + "shared.", mlp["shared"]["ff"])
     return t
 
 
-def clear_tokens(cfg, w, n, seed, margin=0.03):
+def clear_tokens(cfg, w, n, seed, margin=0.014):
     """n random tokens on which no router's choice is closer than `margin`, and their (logits, residual streams)."""
     g = np.random.default_rng(seed)
     tok = g.integers(0, cfg["vocab"], n)

@@ -12,7 +12,7 @@ def test_library_exports_every_declared_symbol(pkg):
     assert len(names) >= 30 and "nvl_forward" in names and "nvl_runner_run" in names
     missing = [n for n in names if not hasattr(L, n)]
     assert not missing, missing
-    assert L.nvl_abi_version() == 6
+    assert L.nvl_abi_version() == 7
 
 
 def test_header_cites_the_reference_for_every_entry_point(pkg):
@@ -26,13 +26,13 @@ def test_header_cites_the_reference_for_every_entry_point(pkg):
 def test_struct_mirrors_match_the_header(pkg):
     L = pkg._lib
     lib = pkg.lib()
-    assert C.sizeof(L.ModelConfigC) == lib.nvl_sizeof(0) == 160     # 13 x i32, pad, f64, f32, i32, 3 x i32, 4 x f32, 6 x i32 (Mamba2), 2 x u64, 2 x f32, i32, pad
+    assert C.sizeof(L.ModelConfigC) == lib.nvl_sizeof(0) == 168     # 13 x i32, pad, f64, f32, i32, 3 x i32, 4 x f32, 6 x i32 (Mamba2), 2 x u64, 2 x f32, i32, f32, i32, pad
     assert C.sizeof(L.RuntimeOptsC) == lib.nvl_sizeof(1) == 40
     assert C.sizeof(L.StatsC) == lib.nvl_sizeof(2) == 16 * 8
     assert C.sizeof(L.SamplingParamsC) == lib.nvl_sizeof(3) == 16
     assert [n for n, _ in L.ModelConfigC._fields_][:3] == ["vocab_size", "hidden", "num_layers"]
-    assert C.sizeof(L.LayerConfigC) == lib.nvl_sizeof(4) == 22 * 4 + 5 * 8 + 8 * 4     # 16 x i32 or f32, f32, 4 x i32, pad, 5 x f64, f32, 7 x i32
-    assert len(L.SLOTS) == 61 and L.SLOT_ID["side_emb"] == 60 and L.SLOT_ID["gla_a2_b"] == 46 and L.SLOT_ID["delta_g2"] == 52 and L.SLOT_ID["moe_out"] == 24 and L.SLOT_ID["mamba_out_proj"] == 32      # NVL_T_COUNT
+    assert C.sizeof(L.LayerConfigC) == lib.nvl_sizeof(4) == 22 * 4 + 5 * 8 + 8 * 4 + 6 * 4 + 2 * 8 + 8 * 4 + 128 * 8     # 16 x i32 or f32, f32, 4 x i32, pad, 5 x f64, f32, 7 x i32, 6 x i32, 2 x f64, 8 x i32 or f32, 128 x f64
+    assert len(L.SLOTS) == 71 and L.SLOT_ID["lin_o"] == 70 and L.SLOT_ID["side_emb"] == 60 and L.SLOT_ID["gla_a2_b"] == 46 and L.SLOT_ID["delta_g2"] == 52 and L.SLOT_ID["moe_out"] == 24 and L.SLOT_ID["mamba_out_proj"] == 32      # NVL_T_COUNT
 
 
 def test_no_cpu_fallback(pkg):

@@ -8,6 +8,7 @@ import pytest
 
 import bolinex_models as BM
 import bolinex_oracle as O
+from layered_helpers import same_fields
 
 
 def raw_config():
@@ -30,9 +31,7 @@ def test_readers_agree(pkg, tmp_path):
     arr = (L.LayerConfigC * n)()
     assert L.lib().nvl_load_layers_json(str(p).encode(), arr, n) == n == len(want.layers) == 4
     for a, w in zip(arr, want.layers):
-        for k, _ in a._fields_:
-            g = getattr(a, k)
-            assert (g == L.MIXER[w[k]]) if k == "mixer" else abs(g - w[k]) < 1e-6, (k, g, w[k])
+        same_fields(L, a, w)
     assert [a.v_mix for a in arr] == [1, 0, 1, 0] and [a.window for a in arr] == [50, 0, 50, 50] and [a.softcap for a in arr] == [9.0, 0.0, 9.0, 9.0]
     assert [(a.experts, a.top_k, a.expert_dim, a.expert_groups, a.groups_kept, a.ffn_dim, a.ffn_act) for a in arr] == \
         [(0, 0, 0, 0, 0, 88, 0), (12, 3, 40, 4, 2, 56, 1), (0, 0, 0, 0, 0, 0, 0), (5, 2, 40, 1, 1, 0, 1)]

@@ -8,6 +8,7 @@ import pytest
 
 import lufazen_models as LM
 import lufazen_oracle as O
+from layered_helpers import same_fields
 
 
 def both_kinds():
@@ -32,9 +33,7 @@ def test_readers_agree(pkg, tmp_path):
     arr = (L.LayerConfigC * n)()
     assert L.lib().nvl_load_layers_json(str(p).encode(), arr, n) == n == len(want.layers) == 3
     for a, w in zip(arr, want.layers):
-        for k, _ in a._fields_:
-            g = getattr(a, k)
-            assert (g == L.MIXER[w[k]]) if k == "mixer" else abs(g - w[k]) < 1e-6, (k, g, w[k])
+        same_fields(L, a, w)
     assert arr[2].kv_from == 0 and arr[0].kv_from == -1 and arr[1].ffn_dim == 0 and arr[0].rot_dim == 48 and arr[0].gate_per_head == 1
     assert (arr[0].rot_factor, arr[0].rot_original, arr[0].rot_fast, arr[0].rot_slow, arr[0].rot_base) == (3.0, 64.0, 8.0, 1.0, 1000.0)
     assert (arr[1].kv_heads, arr[1].conv_taps) == (2, 4) and abs(arr[0].ffn_limit - 1.1) < 1e-6

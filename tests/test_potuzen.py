@@ -8,6 +8,7 @@ import pytest
 
 import potuzen_models as PM
 import potuzen_oracle as O
+from layered_helpers import same_fields
 
 
 def three_kinds():
@@ -28,9 +29,7 @@ def test_readers_agree(pkg, tmp_path):
     arr = (L.LayerConfigC * n)()
     assert L.lib().nvl_load_layers_json(str(p).encode(), arr, n) == n == len(want.layers)
     for a, w in zip(arr, want.layers):
-        for k, _ in a._fields_:
-            g = getattr(a, k)
-            assert (g == L.MIXER[w[k]]) if k == "mixer" else abs(g - w[k]) < 1e-6, (k, g, w[k])
+        same_fields(L, a, w)
     assert arr[3].weights_of == 0 and arr[0].weights_of == -1 and arr[4].ffn_dim == 0 and arr[0].window == 50
 
 
