@@ -97,47 +97,65 @@ __device__ __forceinline__ float grouped_turn(const GroupedArgs& p, const float*
     const f32x2 cs = turn[c < half ? c : c - half];
     return c < half ? at(c) * cs[0] - at(c + half) * cs[1] : at(c) * cs[0] + at(c - half) * cs[1];
 }
-// one workgroup per token, a wave per head: small batches, fp32 mode
+// one wave per (token, head), no workgroup to wait for: small batches, fp32 mode.  A head of up to 256 channels stays in registers, four a
+// lane, and pairs meet by a shuffle; a norm over the projection reads the whole row in every wave (it comes from L2).
 template <typename T>
-__global__ __launch_bounds__(1024) void grouped_qk_row_kernel(GroupedArgs p) {
-    __shared__ float sums[2][16];
-    const int64_t t = blockIdx.x;
-    const int lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), NW = blockDim.x >> 6;
-    const float* row = p.proj + t * p.proj_ld;
-    auto head_x = [&](int h) { return row + (h < p.H ? (int64_t)h * p.dp : p.qk_koff + (int64_t)(h - p.H) * p.dp); };
-    auto squares = [&](const float* x) {
-        float a = 0.f;
-        for (int c = lane * 4; c < p.dp; c += 256) { const f32x4 v = *(const f32x4*)(x + c); a += v[0] * v[0] + v[1] * v[1] + v[2] * v[2] + v[3] * v[3]; }      // (padding is zero)
-        return wave_sum(a);
-    };
-    if (p.qk_norm == 2) {
-        float sq = 0.f, sk = 0.f;
-        for (int h = wave; h < p.H + p.G; h += NW) (h < p.H ? sq : sk) += squares(head_x(h));
-        if (lane == 0) { sums[0][wave] = sq; sums[1][wave] = sk; }
-        __syncthreads();
-    }
-    const f32x2* turn = p.rot ? p.turn + (int64_t)p.tok_pos[t] * (p.rot >> 1) : nullptr;
-    for (int h = wave; h < p.H + p.G; h += NW) {
-        const bool is_q = h < p.H;
-        const float* x = head_x(h);
-        const float* w = is_q ? p.q_norm : p.k_norm;
-        float inv = 1.f;
-        if (p.qk_norm == 1) inv = 1.0f / sqrtf(squares(x) / (float)p.dim + p.eps);
-        else if (p.qk_norm == 2) {
-            float s = 0.f;
-            for (int i = 0; i < NW; i++) s += sums[!is_q][i];
-            inv = 1.0f / sqrtf(s / ((float)p.dim * (is_q ? p.H : p.G)) + p.eps);
-            w += (int64_t)(is_q ? h : h - p.H) * p.dim;
-        }
-        int krow = 0;
-        T* dst = is_q ? (T*)p.q_out : grouped_key_row<T>(p, t, h - p.H, krow);
-        for (int c = lane * 4; c < p.dp; c += 256) {
-            f32x4 v;
+__global__ __launch_bounds__(256) void grouped_qk_row_kernel(GroupedArgs p) {
+    const int heads = p.H + p.G, id = blockIdx.x * 4 + __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), lane = threadIdx.x & 63;
+    if (id >= p.rows * heads) return;
+    const int64_t t = id / heads;
+    const int h = id - (int)t * heads;
+    const bool is_q = h < p.H;
+    const int hh = is_q ? h : h - p.H, half = p.rot >> 1, c = lane * 4;
+    const float* row = p.proj + t * p.proj_ld + (is_q ? 0 : p.qk_koff);
+    const float* x = row + (int64_t)hh * p.dp;
+    const float* w = is_q ? p.q_norm : p.k_norm;
+    if (p.qk_norm == 2) w += (int64_t)hh * p.dim;
+    const bool whole = p.dp <= 256, fast = whole && p.dim % 4 == 0 && half % 4 == 0;      // a lane's channels are data or padding, turn or do not, as one
+    const f32x2* turn = p.rot ? p.turn + (int64_t)p.tok_pos[t] * half : nullptr;
+    f32x4 v = f32x4{0.f, 0.f, 0.f, 0.f}, ww = f32x4{1.f, 1.f, 1.f, 1.f};
+    if (c < p.dp) v = *(const f32x4*)(x + c);
+    if (fast && p.qk_norm && c < p.dim) {
 #pragma unroll
-            for (int r = 0; r < 4; r++) v[r] = grouped_turn(p, x, p.qk_norm ? w : nullptr, inv, turn, c + r);
-            if (is_q) act_store4<T>(dst, t, h * p.dp + c, p.q_ld, v);
-            else act_store4<T>(dst, krow, c, p.dp, v);
+        for (int r = 0; r < 4; r++) ww[r] = w[c + r];
+    }
+    f32x2 cs[4];
+#pragma unroll
+    for (int r = 0; r < 4; r++) cs[r] = fast && c < p.rot ? turn[(c < half ? c : c - half) + r] : f32x2{1.f, 0.f};
+    float inv = 1.f, ss = 0.f;
+    if (p.qk_norm == 1) {
+        ss = v[0] * v[0] + v[1] * v[1] + v[2] * v[2] + v[3] * v[3];       // (padding is zero)
+        for (int i = c + 256; i < p.dp; i += 256) { const f32x4 u = *(const f32x4*)(x + i); ss += u[0] * u[0] + u[1] * u[1] + u[2] * u[2] + u[3] * u[3]; }
+        inv = 1.0f / sqrtf(wave_sum(ss) / (float)p.dim + p.eps);
+    } else if (p.qk_norm == 2) {
+        const int n = (is_q ? p.H : p.G) * p.dp;
+#pragma unroll 8
+        for (int i = c; i < n; i += 256) { const f32x4 u = *(const f32x4*)(row + i); ss += u[0] * u[0] + u[1] * u[1] + u[2] * u[2] + u[3] * u[3]; }
+        inv = 1.0f / sqrtf(wave_sum(ss) / ((float)p.dim * (is_q ? p.H : p.G)) + p.eps);
+    }
+    int krow = 0;
+    T* dst = is_q ? (T*)p.q_out : grouped_key_row<T>(p, t, hh, krow);
+    auto put = [&](int i, f32x4 y) {
+        if (is_q) act_store4<T>(dst, t, h * p.dp + i, p.q_ld, y);
+        else act_store4<T>(dst, krow, i, p.dp, y);
+    };
+    if (fast) {
+        if (p.qk_norm) v *= inv * ww;
+        const int other = c < half ? lane + (half >> 2) : lane - (half >> 2);
+        f32x4 y;
+#pragma unroll
+        for (int r = 0; r < 4; r++) {
+            const float u = __shfl(v[r], other & 63, 64);
+            y[r] = c < p.rot ? (c < half ? v[r] * cs[r][0] - u * cs[r][1] : v[r] * cs[r][0] + u * cs[r][1]) : v[r];
         }
+        if (c < p.dp) put(c, y);
+        return;
+    }
+    for (int i = c; i < p.dp; i += 256) {
+        f32x4 y;
+#pragma unroll
+        for (int r = 0; r < 4; r++) y[r] = grouped_turn(p, x, p.qk_norm ? w : nullptr, inv, turn, i + r);
+        put(i, y);
     }
 }
 // Prompts, bf16: one workgroup per 16 tokens, a wave per head.  A lane is a row of the operand blocks it writes (token l & 15, channels
@@ -214,6 +232,88 @@ static __global__ __launch_bounds__(1024) void grouped_qk_tile_kernel(GroupedArg
             if (!ok) continue;
             if (is_q) *(bf16x8*)(dst + fm_index(t, (int64_t)h * p.dp + c, p.q_ld)) = out;
             else *(bf16x8*)(dst + fm_index(krow, c, p.dp)) = out;
+        }
+    }
+}
+
+// The same with the heads in registers (a wave's up to HPW heads of 32 NB channels, all of them turning): one pass over the fp32 rows.
+template <int NB, int HPW>
+__global__ __launch_bounds__(1024) void grouped_qk_regs_kernel(GroupedArgs p) {
+    __shared__ float sums[2][16][16];                 // [q, k][wave][token]
+    const int lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), heads = p.H + p.G;
+    const int tok = blockIdx.x * 16 + (lane & 15), c0 = (lane >> 4) * 8;
+    const bool ok = tok < p.rows;
+    const int64_t t = ok ? tok : p.rows - 1;
+    const float* row = p.proj + t * p.proj_ld + c0;
+    float x[HPW][NB][8], ss[HPW];
+#pragma unroll
+    for (int j = 0; j < HPW; j++) {
+        const int h = wave + 16 * j;
+#pragma unroll
+        for (int b = 0; b < NB; b++) {
+            f32x4 u = f32x4{0.f, 0.f, 0.f, 0.f}, v = u;
+            if (h < heads) {
+                const float* src = row + (h < p.H ? (int64_t)h * p.dp : p.qk_koff + (int64_t)(h - p.H) * p.dp) + b * 32;
+                u = *(const f32x4*)src; v = *(const f32x4*)(src + 4);
+            }
+#pragma unroll
+            for (int r = 0; r < 4; r++) { x[j][b][r] = u[r]; x[j][b][4 + r] = v[r]; }
+        }
+        ss[j] = 0.f;
+#pragma unroll
+        for (int b = 0; b < NB; b++)
+#pragma unroll
+            for (int r = 0; r < 8; r++) ss[j] = fmaf(x[j][b][r], x[j][b][r], ss[j]);
+        ss[j] += __shfl_xor(ss[j], 16, 64);
+        ss[j] += __shfl_xor(ss[j], 32, 64);
+    }
+    if (p.qk_norm == 2) {
+        float sq = 0.f, sk = 0.f;
+#pragma unroll
+        for (int j = 0; j < HPW; j++) (wave + 16 * j < p.H ? sq : sk) += ss[j];
+        if (lane < 16) { sums[0][wave][lane] = sq; sums[1][wave][lane] = sk; }
+        __syncthreads();
+        sq = sk = 0.f;
+#pragma unroll
+        for (int i = 0; i < 16; i++) { sq += sums[0][i][lane & 15]; sk += sums[1][i][lane & 15]; }
+#pragma unroll
+        for (int j = 0; j < HPW; j++) ss[j] = wave + 16 * j < p.H ? sq / p.H : sk / p.G;
+    }
+    const f32x2* turn = p.turn + (int64_t)p.tok_pos[t] * (p.rot >> 1) + c0;
+#pragma unroll
+    for (int j = 0; j < HPW; j++) {
+        const int h = wave + 16 * j;
+        if (h >= heads) continue;
+        const bool is_q = h < p.H;
+        if (p.qk_norm) {
+            const float inv = 1.0f / sqrtf(ss[j] / (float)p.dim + p.eps);
+            const float* w = (is_q ? p.q_norm : p.k_norm) + (p.qk_norm == 2 ? (int64_t)(is_q ? h : h - p.H) * p.dim : 0) + c0;
+#pragma unroll
+            for (int b = 0; b < NB; b++) {
+                const f32x4 u = *(const f32x4*)(w + b * 32), v = *(const f32x4*)(w + b * 32 + 4);
+#pragma unroll
+                for (int r = 0; r < 8; r++) x[j][b][r] *= inv * (r < 4 ? u[r] : v[r - 4]);
+            }
+        }
+        int krow = 0;
+        bf16_t* dst = is_q ? (bf16_t*)p.q_out : grouped_key_row<bf16_t>(p, t, h - p.H, krow);
+#pragma unroll
+        for (int b = 0; b < NB / 2; b++) {
+            bf16x8 lo, hi;
+#pragma unroll
+            for (int r = 0; r < 8; r += 2) {
+                const f32x4 cs = *(const f32x4*)(turn + b * 32 + r);         // (cos, sin) of two pairs
+#pragma unroll
+                for (int e = 0; e < 2; e++) {
+                    const float u = x[j][b][r + e], v = x[j][b + NB / 2][r + e];
+                    lo[r + e] = (bf16_t)(u * cs[2 * e] - v * cs[2 * e + 1]);
+                    hi[r + e] = (bf16_t)(v * cs[2 * e] + u * cs[2 * e + 1]);
+                }
+            }
+            if (!ok) continue;
+            const int c = b * 32 + c0;
+            if (is_q) { *(bf16x8*)(dst + fm_index(t, (int64_t)h * p.dp + c, p.q_ld)) = lo; *(bf16x8*)(dst + fm_index(t, (int64_t)h * p.dp + c + NB * 16, p.q_ld)) = hi; }
+            else { *(bf16x8*)(dst + fm_index(krow, c, p.dp)) = lo; *(bf16x8*)(dst + fm_index(krow, c + NB * 16, p.dp)) = hi; }
         }
     }
 }
@@ -704,5 +804,7 @@ __global__ __launch_bounds__(256) void grouped_plain_kernel(GroupedArgs p) {
 // launches (grouped_inst.hip): the instance follows from p.dp and p.vp
 void grouped_prefill_launch(hipStream_t st, const GroupedArgs& p, dim3 grid, size_t lds, bool fast);
 void grouped_short_launch(hipStream_t st, const GroupedArgs& p, dim3 grid);
+void grouped_qk_launch(hipStream_t st, const GroupedArgs& p, bool f32);
+constexpr int GROUPED_QK_ROW_MAX = 512;           // bf16: larger batches are worked in tiles of 16 tokens
 
 }  // namespace nvl

@@ -47,6 +47,23 @@ static void run_short_ks(hipStream_t st, const GroupedArgs& p, dim3 grid) {
         default: run_short<KS, 16>(st, p, grid);
     }
 }
+template <int NB>
+static bool qk_regs(hipStream_t st, const GroupedArgs& p) {
+    const dim3 grid(cdiv(p.rows, 16)), block(1024);
+    switch (cdiv(p.H + p.G, 16)) {
+        case 1: hipLaunchKernelGGL((grouped_qk_regs_kernel<NB, 1>), grid, block, 0, st, p); return true;
+        case 2: hipLaunchKernelGGL((grouped_qk_regs_kernel<NB, 2>), grid, block, 0, st, p); return true;
+        case 3: hipLaunchKernelGGL((grouped_qk_regs_kernel<NB, 3>), grid, block, 0, st, p); return true;
+        default: return false;
+    }
+}
+void grouped_qk_launch(hipStream_t st, const GroupedArgs& p, bool f32) {
+    const dim3 waves(cdiv((int64_t)p.rows * (p.H + p.G), 4));
+    if (f32) hipLaunchKernelGGL((grouped_qk_row_kernel<float>), waves, dim3(256), 0, st, p);
+    else if (p.rows <= GROUPED_QK_ROW_MAX) hipLaunchKernelGGL((grouped_qk_row_kernel<bf16_t>), waves, dim3(256), 0, st, p);
+    else if (p.dim == p.dp && p.rot == p.dp && ((p.dp == 64 && qk_regs<2>(st, p)) || (p.dp == 128 && qk_regs<4>(st, p)))) return;
+    else hipLaunchKernelGGL(grouped_qk_tile_kernel, dim3(cdiv(p.rows, 16)), dim3(1024), 0, st, p);
+}
 void grouped_short_launch(hipStream_t st, const GroupedArgs& p, dim3 grid) {
     switch (p.dp >> 5) {
         case 1: run_short_ks<1>(st, p, grid); break;

@@ -29,7 +29,6 @@ namespace {
 
 constexpr int LAT_ABSORB_MAX = 16, LAT_ABSORB_MAX_RP = 512, REC_STEP_MAX = 4;
 constexpr int GLU_IN_MAX = 1024;       // widest shared expert whose gate and up columns pass through fp32 rows instead of a launch of their own
-constexpr int QK_ROW_MAX = 256;        // batches whose queries and keys are normed and rotated by a workgroup per token
 constexpr int SHARED_PARTS_MAX = 16;   // widest shared expert, in experts, that joins the masked experts of a decode step
 constexpr int GROUPED_SHORT_ROWS = 64, GROUPED_SPLIT_WGS = 512;      // GROUPED_SPLIT_WGS: workgroups of a launch whose keys are split
 
@@ -1314,18 +1313,15 @@ void mix_grouped(nvl_model* m, const LayerRun& r, const MixerW& w, const Meta& m
         m->site = KS_MIX_IN;
         gemm(m, r.raw ? EPI_GROUPED_RAW : EPI_GROUPED, false, g);
     }
+    if (c.mixer2) mix_lightning(m, r, w, md, n_seqs, M, max_len);
     if (r.raw) {          // norms and rotation of the fp32 queries and keys
         a.proj = m->lproj; a.proj_ld = m->lproj_ld; a.qk_koff = r.k_off; a.qk_norm = c.qk_norm; a.q_norm = w.q_norm; a.k_norm = w.k_norm; a.eps = m->cfg.norm_eps;
         a.rot = c.rot_dim; a.turn = r.turn; a.tok_pos = md.tok_pos; a.tok_tbl = md.tok_tbl; a.rows = M;
         a.q = a.q_out = m->lqg; a.q_ld = (int64_t)a.H * r.dp;
         KScope ks(m, KC_OTHER, 0, KS_QK_TURN, (double)M * (a.H + a.G) * c.dim * (4.0 + ws));
-        const int threads = std::min(1024, (a.H + a.G) * 64);
-        if (m->f32) hipLaunchKernelGGL((grouped_qk_row_kernel<float>), dim3(M), dim3(threads), 0, m->stream, a);
-        else if (M <= QK_ROW_MAX) hipLaunchKernelGGL((grouped_qk_row_kernel<bf16_t>), dim3(M), dim3(threads), 0, m->stream, a);
-        else hipLaunchKernelGGL(grouped_qk_tile_kernel, dim3(cdiv(M, 16)), dim3(1024), 0, m->stream, a);
+        grouped_qk_launch(m->stream, a, m->f32);
         NVL_HIP(hipGetLastError());
     }
-    if (c.mixer2) mix_lightning(m, r, w, md, n_seqs, M, max_len);
     const bool plain = m->f32 || r.dp > 256 || r.vp > 256;
     const int ctx = m->ctx_hint > 0 ? m->ctx_hint : m->cfg.max_seq_len;
     int tiles = cdiv(ctx, 64) + 1;                              // most key tiles a 256-row workgroup walks
@@ -1447,18 +1443,18 @@ void glu_up(nvl_model* m, const void* W, int M, int Fp, int act, float limit) {
     up.glu_limit = limit; up.glu_slope = CLAMPED_GLU_SLOPE;
     gemm(m, act == NVL_ACT_CLAMPED_GLU ? EPI_CLAMP_GLU : act == NVL_ACT_REGLU ? EPI_REGLU : EPI_GEGLU, false, up);
 }
-// ---- experts that read m->xn by themselves (their shared expert too); returns the shared expert's result, or in `joined` cases everything ----
+// ---- experts that read m->xn by themselves, and their shared expert: returns what is added, the rest of it in `ex` ----
 SubOut expert_ffn(nvl_model* m, const LayerRun& r, const MixerW& w, int M, ExpertOut& ex) {
     const nvl_layer_config& c = r.c;
     const int E = c.experts, k = c.top_k, pairs = M * k;
     const bool dense = !m->f32 && M <= 64 && r.Ip <= 2048;          // decode: masked projections over all experts (gemm.h GemmArgs::moe_gate)
     const int parts = dense ? r.shared_parts : 0;
     SubOut y{nullptr, 1, 0};
-    if (c.ffn_dim && !parts) {
+    auto shared = [&] {
         const void* W = r.shared_parts && !m->f32 ? (const void*)((const char*)w.moe_up + (int64_t)E * 2 * r.Ip * m->H * (int64_t)m->wsize) : w.w1;
         glu_up(m, W, M, r.Fp, r.act, c.ffn_limit);
         y = sub_out(m, KS_FFN_DOWN, m->hbuf, w.w2, M, r.Fp);
-    }
+    };
     if (dense && E <= 64 && c.route_softmax) {
         GemmArgs a = mk(m->xn, m->H, w.router, nullptr, E, w.route_bias, 1.f, M, E, m->H);
         KScope ks(m, KC_OTHER, 2.0 * M * E * m->Hn, KS_MOE_ROUTER, ((double)E * m->Hn + (double)M * m->Hn) * (double)m->wsize + (double)M * E * 4.0);
@@ -1485,8 +1481,9 @@ SubOut expert_ffn(nvl_model* m, const LayerRun& r, const MixerW& w, int M, Exper
         d.moe_gate = m->moe_gate; d.moe_E = r.Ep; d.moe_I = r.Ip; d.sk_part = m->moe_part; d.sk_slices = r.moe_slices;
         m->site = KS_MOE_DOWN; m->site_bytes = (touch * m->Hn + work) * (double)m->wsize + (double)r.moe_slices * M * m->Hn * 4.0;
         gemm(m, EPI_RESID, true, d, 2.0 * work * m->Hn);
-        if (!y.y) return {m->moe_part, r.moe_slices, (int64_t)M * m->H};
+        if (!c.ffn_dim || parts) return {m->moe_part, r.moe_slices, (int64_t)M * m->H};
         ex = {m->moe_part, r.moe_slices, (int64_t)M * m->H, nullptr, nullptr};
+        shared();
         return y;
     }
     const bool pp = moe_pp_ok(m, r.Ip, false);
@@ -1494,7 +1491,8 @@ SubOut expert_ffn(nvl_model* m, const LayerRun& r, const MixerW& w, int M, Exper
     moe_sort(m, E, k, M, BM);
     moe_expert_gemms(m, MoeW{E, k, r.Ip, w.moe_up, w.moe_down, c.expert_limit}, M, BM, pp, false);
     ex = {m->moe_eo, k, 0, m->slot_of, m->expert_w};
-    if (!y.y) {          // no shared expert: nothing but the experts joins
+    if (c.ffn_dim) shared();
+    else {               // nothing but the experts joins
         y = {m->ly, 1, 0};
         hipLaunchKernelGGL(fill_i32_kernel, dim3(cdiv((int64_t)M * m->H, 256)), dim3(256), 0, m->stream, (int32_t*)m->ly, 0, M * m->H);
         NVL_HIP(hipGetLastError());
