@@ -266,7 +266,7 @@ def _medulorn_layer(e: dict) -> dict:
         mask = left.get("mask") or {}
         if len(right["decay"]) != right["heads"]:
             raise ValueError("as many decays as heads expected")
-        out.update(_medulorn_attention(left), qk_norm=QK_NORM_ROW, sink=SINK_LEARNED, window=mask.get("size", 0), keep_first=mask.get("keep_first", 0),
+        out.update(_medulorn_attention(left), qk_norm=QK_NORM_ROW, sink=SINK_LEARNED, window=mask.get("size", 0), keep_first=mask.get("keep_first") or 0,
                    out_scale=float(mx["left_scale"]), mixer2=MIXER_LIGHTNING, heads2=right["heads"], dim2=right["dim"], vdim2=right["vdim"],
                    out_scale2=float(mx["right_scale"]), decay=[float(d) for d in right["decay"]])
     else:

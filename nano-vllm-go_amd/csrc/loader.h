@@ -342,7 +342,8 @@ int parse_mask(const JVal* mx, int* keep_first, const std::string& at) {
     if (!mask || mask->kind != JVal::OBJ) return 0;
     const int size = need_int(mask, "size", at);
     if (size <= 0) throw std::runtime_error(at + "the mask's size is not positive");
-    if (keep_first && mask->get("keep_first")) *keep_first = need_int(mask, "keep_first", at);
+    const JVal* kept = mask->get("keep_first");
+    if (keep_first && kept && kept->kind != JVal::NUL) *keep_first = need_int(mask, "keep_first", at);
     return size;
 }
 // what the two attentions of the design with norms of sums share: sizes, scale, rotation {dims, base, scaling: null | {factor, original, low, high}}
