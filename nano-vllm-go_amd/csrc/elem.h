@@ -1106,8 +1106,8 @@ __global__ __launch_bounds__(1024) void moe_plan_kernel(const float* __restrict_
 
 // Group-limited routing on sigmoid scores.  s = sigmoid(z); the choice goes by s + correction, the weights are the s of the chosen
 // experts as they are.  Experts form `groups` equal groups of neighbours; a group counts as much as its two largest choice scores
-// together, and only the experts of the best `keep` groups can be chosen.  Ties go to the lower index.  One wave per token, E <= 256;
-// `softmax`: the choice goes by z + correction, and the weights are the softmax over the chosen ones of these (no groups).
+// together, and only the experts of the best `keep` groups can be chosen.  Ties go to the lower index.  With
+// `softmax` the choice goes by z + correction, and the weights are the softmax over the chosen ones of these.  One wave per token, E <= 256;
 // writes (id, weight) in rank order, or with `gate` the dense [rows][gate_ld] matrix of weights (0: not chosen).  Workgroups with
 // blockIdx.y > 0 finish a SwiGLU feed-forward whose fp32 gate and up columns the same projection made (a small shared expert):
 // grid (ceil(rows / 4), 1 + ceil(F / 256)).

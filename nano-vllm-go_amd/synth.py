@@ -253,14 +253,14 @@ def _medulorn(width: int, layers: int, heads: int, ff: int, expert_ff: int, wind
     """A Medulorn model at a real model's layer sizes: chunked attention with dense feed-forwards, and windowed beside lightning attention with
     experts, in turn."""
     from .config import ACT_CLAMPED_GLU, LAYER_FIELDS, MIXER_LIGHTNING, QK_NORM_HEAD, QK_NORM_ROW, SINK_LEARNED, SINK_ZERO
-    att = dict(mixer="attention", heads=heads, kv_heads=heads // 4, dim=128, vdim=128, scale=128 ** -0.5, ungated=1, rot_dim=128, rot_base=5e5)
+    att = dict(mixer="attention", heads=heads, kv_heads=heads // 4, dim=128, vdim=128, scale=128 ** -0.5, ungated=1, rot_dim=128, rot_base=1e5)
     kinds = [dict(att, chunk=window, qk_norm=QK_NORM_HEAD, sink=SINK_ZERO, qkv_bias=1, ffn_dim=ff),
-             dict(att, window=window, keep_first=4, qk_norm=QK_NORM_ROW, sink=SINK_LEARNED, rot_factor=4.0, rot_low=1.0, rot_high=4.0, rot_original=2048.0, out_scale=1.2,
-                  mixer2=MIXER_LIGHTNING, heads2=heads, dim2=128, vdim2=128, out_scale2=0.5, decay=[1.0 - 0.5 ** (1.0 + 7.0 * h / heads) for h in range(heads)],
+             dict(att, window=window, keep_first=8, qk_norm=QK_NORM_ROW, sink=SINK_LEARNED, rot_factor=8.0, rot_low=1.0, rot_high=4.0, rot_original=2048.0, out_scale=0.9,
+                  mixer2=MIXER_LIGHTNING, heads2=heads, dim2=128, vdim2=128, out_scale2=0.7, decay=[1.0 - 0.5 ** (1.0 + 7.0 * h / heads) for h in range(heads)],
                   ffn_dim=expert_ff, ffn_act=ACT_CLAMPED_GLU, ffn_limit=7.0, experts=32, top_k=8, expert_dim=expert_ff, expert_groups=1, groups_kept=1, route_softmax=1, expert_limit=7.0)]
     return dict(vocab_size=32000, hidden=width, num_layers=layers, num_heads=0, num_kv_heads=0, head_dim=0, ffn_dim=0, max_seq_len=4096,
                 attention_type="gqa", norm_type="rmsnorm_scalar", position_type="nope", activation_type="reglu", block_style="sum_norm",
-                rope_base=0.0, norm_eps=1e-6, tied_embedding=False, embedding_multiplier=width ** 0.5, stream_scale=3.0, token_shift=1, logit_softcap=30.0,
+                rope_base=0.0, norm_eps=1e-6, tied_embedding=False, embedding_multiplier=width ** 0.5, stream_scale=2.0, token_shift=1, logit_softcap=40.0,
                 layers=[dict(LAYER_FIELDS, **kinds[i % 2]) for i in range(layers)])
 
 

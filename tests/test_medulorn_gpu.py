@@ -28,7 +28,7 @@ SINGLE = {      # layer, width
     "chunk-128": (att(chunk=128), 64), "chunk-long": (att(chunk=1000), 64), "no-turn": (att(turn=None), 64), "turn-2": (att(turn=rot(2, 50.0)), 64), "turn-all": (att(dim=32, vdim=32, turn=rot(32)), 64),
     "turn-18-of-26": (att(dim=26, turn=rot(18)), 64), "turn-scaled": (att(turn=rot(32, 800.0, (4.0, 1.0, 4.0, 64))), 64), "one-head-each": (att(heads=3, kv_heads=3), 96), "one-kv-head": (att(heads=5, kv_heads=1), 96),
     "group-34": (att(heads=34, kv_heads=1, dim=16, vdim=8, turn=rot(8)), 96), "group-70": (att(heads=70, kv_heads=1, dim=12, vdim=5, turn=rot(12), chunk=100), 64),
-    "64-64": (att(heads=4, kv_heads=1, dim=64, vdim=64, chunk=None, turn=rot(64)), 128), "128-128": (att(heads=4, kv_heads=2, dim=128, vdim=128, turn=rot(64)), 128), "96-96": (att(heads=4, kv_heads=2, dim=96, vdim=96, turn=rot(96)), 128),
+    "64-64": (att(heads=4, kv_heads=1, dim=64, vdim=64, chunk=None, turn=rot(64)), 128), "128-128": (att(heads=4, kv_heads=2, dim=128, vdim=128, turn=rot(64)), 128), "96-80": (att(heads=3, kv_heads=1, dim=96, vdim=80, turn=rot(96)), 128),
     "20-160": (att(heads=2, kv_heads=1, dim=20, vdim=160, turn=rot(20)), 64), "200-40": (att(heads=2, kv_heads=2, dim=200, vdim=40, turn=rot(100)), 64), "256-256": (att(heads=4, kv_heads=2, dim=250, vdim=256, scale=0.06), 96),
     "big-heads": (att(heads=2, kv_heads=1, dim=272, vdim=264, scale=0.05, turn=rot(136)), 64), "narrow": (att(heads=1, kv_heads=1, dim=4, vdim=4, turn=rot(4), mlp=MM.dense(5)), 12),
     "wide-row": (att(heads=2, kv_heads=1, mlp=MM.dense(16)), 1100), "negative-scale": (att(scale=-0.3), 64), "no-feed-forward": (att(mlp=None), 96), "dense-200": (att(mlp=MM.dense(200)), 70),
